@@ -1,0 +1,169 @@
+"""Plain, slow restatement of the mechanisms layered models are built from (float64 numpy, one function per mechanism).
+
+Test infrastructure: shares no code with the product path.  `forward` walks one sequence from its first token; everything that the
+runner carries between portions (latent cache, recurrent state, convolution tail, previous token) is recomputed here from scratch.
+"""
+import numpy as np
+
+
+def sigmoid(z):
+    return 1.0 / (1.0 + np.exp(-z))
+
+
+def softplus(z):
+    return np.logaddexp(0.0, z)
+
+
+def gelu_tanh(z):
+    return 0.5 * z * (1.0 + np.tanh(np.sqrt(2.0 / np.pi) * (z + 0.044715 * z ** 3)))
+
+
+def unit_rms(x, eps):
+    return x / np.sqrt(np.mean(x * x, axis=-1, keepdims=True) + eps)
+
+
+def xielu(z, p, q):
+    """Trainable piecewise activation: quadratic right of zero, exponential left of it, slope 1/2 at zero."""
+    neg = np.minimum(z, 0.0)
+    return np.where(z > 0, softplus(p) * z * z + z / 2, (0.5 + softplus(q)) * (np.expm1(neg) - neg) + z / 2)
+
+
+def bigram_rows(tokens, buckets, mul_prev, mul_cur):
+    """Hash-table row of every token of a sequence; the first token, which has no predecessor, takes the extra row."""
+    rows = [buckets]
+    for prev, cur in zip(tokens[:-1], tokens[1:]):
+        rows.append((int(prev) * mul_prev + int(cur) * mul_cur) % buckets)
+    return np.array(rows[:len(tokens)], np.int64)
+
+
+def embed(tokens, table, bigram=None, buckets=0, mul_prev=0, mul_cur=0):
+    x = table[np.asarray(tokens)]
+    if bigram is not None:
+        x = x + bigram[bigram_rows(tokens, buckets, mul_prev, mul_cur)]
+    return x
+
+
+def rotate_interleaved(x, positions, dims, base):
+    """Rotate pairs (2i, 2i + 1) of the first `dims` entries of the last axis; x [tokens, ..., n]."""
+    out = x.copy()
+    for i in range(dims // 2):
+        a = np.asarray(positions, np.float64) * float(base) ** (-2.0 * i / dims)
+        c, s = np.cos(a), np.sin(a)
+        shape = (len(c),) + (1,) * (x.ndim - 2)
+        c, s = c.reshape(shape), s.reshape(shape)
+        u, v = x[..., 2 * i], x[..., 2 * i + 1]
+        out[..., 2 * i] = u * c - v * s
+        out[..., 2 * i + 1] = v * c + u * s
+    return out
+
+
+def window_mask(n, size):
+    """[query, key]: a query sees itself and the size − 1 tokens before it."""
+    d = np.arange(n)[:, None] - np.arange(n)[None, :]
+    return (d >= 0) & (d < size)
+
+
+def softmax_attention(scores, mask):
+    s = np.where(mask, scores, -np.inf)
+    e = np.exp(s - s.max(axis=-1, keepdims=True))
+    return e / e.sum(axis=-1, keepdims=True)
+
+
+def latent_attention(h, w, heads, dim, rot_dim, vdim, rot_dims, rot_base, window, scale, eps):
+    """h [n, width]; w: dq, dq.norm, uq, dkv, dkv.norm, uk, uv, g, o."""
+    n = h.shape[0]
+    pos = np.arange(n)
+    rank = w["dkv"].shape[0] - rot_dim
+    q = (unit_rms(h @ w["dq"].T, eps) * w["dq.norm"]) @ w["uq"].T
+    q = q.reshape(n, heads, dim + rot_dim)
+    q_plain, q_rot = q[..., :dim], rotate_interleaved(q[..., dim:], pos, rot_dims, rot_base)
+    kv = h @ w["dkv"].T
+    latent = unit_rms(kv[:, :rank], eps) * w["dkv.norm"]
+    k_rot = rotate_interleaved(kv[:, rank:], pos, rot_dims, rot_base)
+    k_plain = (latent @ w["uk"].T).reshape(n, heads, dim)
+    value = (latent @ w["uv"].T).reshape(n, heads, vdim)
+    mask = window_mask(n, window)
+    out = np.zeros((n, heads, vdim))
+    for a in range(heads):
+        p = softmax_attention((q_plain[:, a] @ k_plain[:, a].T + q_rot[:, a] @ k_rot.T) * scale, mask)
+        out[:, a] = p @ value[:, a]
+    out *= sigmoid(h @ w["g"].T)[:, :, None]
+    return out.reshape(n, heads * vdim) @ w["o"].T
+
+
+def causal_conv(x, taps, bias):
+    """x [n, c], taps [c, k]: the last column weighs the current token."""
+    n, c = x.shape
+    k = taps.shape[1]
+    padded = np.concatenate([np.zeros((k - 1, c)), x])
+    return sum(padded[j:j + n] * taps[:, j] for j in range(k)) + bias
+
+
+def rglru_scan(u, r, i, lam):
+    log_a = -8.0 * r * softplus(lam)
+    state, out = np.zeros(u.shape[1]), np.zeros_like(u)
+    for t in range(u.shape[0]):
+        state = np.exp(log_a[t]) * state + np.sqrt(-np.expm1(2.0 * log_a[t])) * i[t] * u[t]
+        out[t] = state
+    return out
+
+
+def block_linear(u, w, b):
+    """u [n, blocks·k], w [blocks, k_out, k], b [blocks, k_out]"""
+    n, (blocks, ko, k) = u.shape[0], w.shape
+    parts = u.reshape(n, blocks, k)
+    return np.concatenate([parts[:, j] @ w[j].T + b[j] for j in range(blocks)], axis=1)
+
+
+def rglru(h, w):
+    """w: y, y.b, x, x.b, conv, conv.b, ra, ra.b, ri, ri.b, lam, o."""
+    y = gelu_tanh(h @ w["y"].T + w["y.b"])
+    u = causal_conv(h @ w["x"].T + w["x.b"], w["conv"], w["conv.b"])
+    r, i = sigmoid(block_linear(u, w["ra"], w["ra.b"])), sigmoid(block_linear(u, w["ri"], w["ri.b"]))
+    return (rglru_scan(u, r, i, w["lam"]) * y) @ w["o"].T
+
+
+def dense_ff(h, w):
+    """w: up, down, act."""
+    return xielu(h @ w["up"].T, w["act"][0], w["act"][1]) @ w["down"].T
+
+
+def add_sublayer(x, sub, gate_w, gate_b, norm_w, mult, eps):
+    """x + mult · norm(sub · gate): the gate reads x, the norm's weight is stored around zero."""
+    gated = sub * sigmoid(x @ gate_w.T + gate_b)
+    return x + mult * unit_rms(gated, eps) * (1.0 + norm_w)
+
+
+def group(weights, prefix):
+    return {k[len(prefix):]: v for k, v in weights.items() if k.startswith(prefix)}
+
+
+def forward(config, weights, tokens, taps=None):
+    """Logits [n, vocab] of one sequence; taps (a list) receives the residual stream after every layer."""
+    w = {k: np.asarray(v, np.float64) for k, v in weights.items()}
+    eps, mult = config["norm"]["eps"], config["residual_mult"]
+    bg = config["embedding"]["bigram"]
+    x = embed(tokens, w["embed"], w["bigram"], bg["buckets"], bg["mul_prev"], bg["mul_cur"])
+    for li, layer in enumerate(config["layers"]):
+        p, mx = f"l{li}.", layer["mixer"]
+        mw = group(w, p + "mix.")
+        if layer["type"] == "latent_attention":
+            sub = latent_attention(x, mw, mx["heads"], mx["dim"], mx["rot_dim"], mx["vdim"], mx["rot"]["dims"], mx["rot"]["base"],
+                                   mx["mask"]["size"], mx["scale"], eps)
+        else:
+            sub = rglru(x, mw)
+        x = add_sublayer(x, sub, w[p + "rg1"], w[p + "rg1.b"], w[p + "norm1"], mult, eps)
+        if layer["mlp"]:
+            x = add_sublayer(x, dense_ff(x, group(w, p + "mlp.")), w[p + "rg2"], w[p + "rg2.b"], w[p + "norm2"], mult, eps)
+        if taps is not None:
+            taps.append(x.copy())
+    return (unit_rms(x, eps) * (1.0 + w["final.norm"])) @ w["embed"].T
+
+
+def greedy(config, weights, prompt, steps):
+    out, seq = [], list(prompt)
+    for _ in range(steps):
+        t = int(np.argmax(forward(config, weights, seq)[-1]))
+        out.append(t)
+        seq.append(t)
+    return out
