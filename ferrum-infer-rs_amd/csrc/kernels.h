@@ -275,6 +275,7 @@ int argmax_rows_f16_ws(const __half* logits, uint32_t* out_ids, const uint8_t* v
 struct DecodeAdvance {
     uint32_t* tokens = nullptr; uint32_t* pos_offsets = nullptr; uint32_t* kv_lens = nullptr; uint32_t* history = nullptr;
     int32_t* step_counter = nullptr; unsigned* ticket = nullptr; int n = 0;
+    int32_t* prev_tokens = nullptr;      // optional: receives the token a sequence was fed this step
 };
 // *fused = 1 when the advance ran inside the argmax launches (two-stage form), 0 when the caller still has to run it
 int argmax_pairs_f32(const float* logits, const uint32_t* local_ids, void* pairs, int rows, int n_local, int v0, const uint8_t* mask, int mask_len, hipStream_t s);

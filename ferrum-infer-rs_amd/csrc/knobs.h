@@ -54,6 +54,11 @@ struct Knobs {
     int w4_w = 0;
     int lds_min_wgs = 128;
     int lds_min_groups = 8;
+    // layered models (tiled_gemm.hip, latent_attention.hip, rglru.hip)
+    int tiled_big_min_tiles = 64;     // 16-bit projections of > 64 rows take the 128 × 128 tile kernel from this many tiles
+    int latent_splits = 0;            // > 0: forced KV split count of the latent attention
+    int latent_expand_min_rows = 64;  // prompt portions of at least this many tokens attend expanded keys / values (0 = never)
+    bool latent_plain = false;        // the plain latent attention kernel for 16-bit models too
     // runner
     bool no_graph = false;
     bool trace_launches = false;
@@ -112,6 +117,14 @@ enum Form : int {
     FORM_CHAIN_ATTN_KV_SPLITS,  // decode chain with several KV ranges per (sequence, kv head) in its attention role (ticket merge)
     FORM_CHAIN_QKV_WIDE,        // decode chain with 128-column q|k|v blocks (the narrow ones + attention exceed the resident workgroups)
     FORM_ROUTE_GEMM_TOPK,       // prefill router: logits (MFMA) + softmax + top-k in one launch (moe_route_gemm_topk_kernel)
+    FORM_TILED_GEMM,            // layered models: projection with K split over the waves of a workgroup
+    FORM_TILED_GEMM_BIG,        // … 128 × 128 tiles, operands copied to LDS as fragments
+    FORM_LATENT_ATTN_PLAIN,     // latent attention, one workgroup per (token, head), any size and number format
+    FORM_LATENT_ATTN,           // … on the matrix cores, against the cached latents (keys and values never expanded)
+    FORM_LATENT_ATTN_SPLIT,     // … with the keys of a tile split over several workgroups
+    FORM_LATENT_ATTN_EXPANDED,  // … prompt portions over keys and values expanded from the latents
+    FORM_RGLRU_STEP,            // linear recurrence, every sequence brings one token: gates, state update and output in one launch
+    FORM_RGLRU_SCAN,            // … prompt portions: chunked scan
     FORM_COUNT
 };
 

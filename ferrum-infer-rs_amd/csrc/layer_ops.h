@@ -1,0 +1,77 @@
+// Kernels of the layered models' mixers and residual stream (latent_attention.hip, rglru.hip, residual_stream.hip).
+// E is bf16 or float; all leading dimensions are padded to multiples of 32 (tiled_gemm.h).
+#pragma once
+#include "tiled_gemm.h"
+
+namespace fh {
+
+// What a forward's kernels know about the batch (device pointers into the index block; scalars for sizing).
+struct BatchView {
+    int T = 0, num_seqs = 0, max_blocks = 0;
+    int max_keys = 0;                            // longest context of the batch, new tokens included (upper bound)
+    bool single = false;                         // every sequence brings one token
+    const uint32_t* tokens = nullptr;            // [T]
+    const uint32_t* cu = nullptr;                // [num_seqs + 1]
+    const uint32_t* pos = nullptr;               // [num_seqs] position of a sequence's first new token
+    const int32_t* bt = nullptr;                 // [num_seqs][max_blocks]
+    const int32_t* tok_seq = nullptr;            // [T] sequence of a token
+    const int32_t* prev = nullptr;               // [num_seqs] token before the first new one, −1: none
+    const int32_t* slots = nullptr;              // [num_seqs] recurrent state slot
+    const int32_t* units = nullptr;              // [num_units][2] (sequence, first token of the chunk within the batch)
+    int num_units = 0;
+};
+
+// ── residual stream (residual_stream.hip) ──
+// x = embed[token] (+ bigram[(prev·mul_prev + token·mul_cur) mod buckets], or the extra row for a first token), fp32; xb = E(x)
+template <typename E>
+int embed_bigram(const E* table, const E* bigram, int buckets, int64_t mul_prev, int64_t mul_cur, const BatchView& v, float* x, E* xb,
+                 int dim, int ldb, hipStream_t s);
+// x += mult · rms(sub · gate) · w (w holds 1 + the stored weight); xb = E(x)
+template <typename E>
+int gated_post_norm_add(const float* sub, long ld_sub, const E* gate, long ld_gate, const float* w, float mult, float eps, float* x,
+                        E* xb, int rows, int dim, int ldb, hipStream_t s);
+// out[i] = E(rms(x[row_idx[i]]) · w)
+template <typename E>
+int rms_norm_rows(const float* x, const int32_t* row_idx, const float* w, float eps, E* out, int rows, int dim, int ldo, hipStream_t s);
+
+// ── latent attention (latent_attention.hip) ──
+// Cache of a layer: [blocks][(kp + rp) / 8 chunks][16 tokens][8]: the normed latent, then the rotated shared key part, zero-padded.
+struct LatentDims { int heads, kv_rank, q_rank, rot_dim, rot_dims, vdim, dp, rp, kp, qp, vp, window; float scale; };
+inline size_t latent_block_elems(const LatentDims& d) { return (size_t)16 * (d.kp + d.rp); }
+template <typename E>
+struct LatentBuffers {
+    const float *cos_t = nullptr, *sin_t = nullptr;   // [positions][rot_dims / 2]
+    E* pool = nullptr;
+    const E* q = nullptr;              // [T][heads·(dp + rp)]: per head the plain part, then the part to rotate
+    const E* q_lat = nullptr;          // [T][heads][kp]: plain part taken through the key projection
+    E* o_lat = nullptr;                // [T][heads][kp]
+    float* partial = nullptr; size_t partial_bytes = 0;
+};
+// q latent: RMS norm → cq [T][qp]; kv latent: RMS norm, shared key part: rotation → cache.  `dq` / `dkv`: their columns in the
+// fused projection's rows (ld); dkv = [kp latent | rp key part].
+template <typename E>
+int latent_prepare(const E* dq, const E* dkv, long ld, const float* dq_norm, const float* dkv_norm, float eps, const LatentDims& d,
+                   const LatentBuffers<E>& b, const BatchView& v, E* cq, hipStream_t s);
+template <typename E>
+int latent_attention(const LatentDims& d, const LatentBuffers<E>& b, const BatchView& v, hipStream_t s);
+
+// ── real-gated linear recurrent unit (rglru.hip) ──
+// Channels live in a block-padded layout: blocks · bp with bp = pad32(width / blocks); padded channels are zero throughout.
+struct RglruDims { int blocks, bp, wp, taps; };
+template <typename E>
+struct RglruBuffers {
+    const E* x = nullptr; const E* y = nullptr; long ld = 0;      // columns of the fused projection (bias and gelu applied)
+    const float *conv_w = nullptr, *conv_b = nullptr;              // [taps][wp], [wp]
+    const E* gate_w = nullptr; const float *ra_b = nullptr, *ri_b = nullptr;    // fragment tiles [blocks][bp / 16][ra, ri], biases [wp]
+    const float* lam = nullptr;                                    // softplus(lam) [wp]
+    E* conv_state = nullptr; float* state = nullptr;               // [slots][taps − 1][wp], [slots][wp]
+    E* u = nullptr;                                                // [T][wp]
+    float *decay = nullptr, *drive = nullptr;                      // [T][wp]
+    float *chunk_a = nullptr, *chunk_h = nullptr;                  // [units][wp]
+    E* out = nullptr;                                              // [T][wp]
+};
+constexpr int RGLRU_CHUNK = 64;        // tokens per scan chunk (BatchView::units)
+template <typename E>
+int rglru_forward(const RglruDims& d, const RglruBuffers<E>& b, const BatchView& v, hipStream_t s);
+
+}  // namespace fh

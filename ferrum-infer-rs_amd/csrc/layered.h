@@ -1,0 +1,33 @@
+// Layered models: decoders whose layers are described one by one (FerrumHipLayerSpec) instead of by one homogeneous configuration.
+// They plug into FerrumHipModel (runner.h), which keeps sequences, paged blocks, state slots, batching, sampling and the decode graph;
+// this part owns the weights, the caches' memory and the order of kernels of a layer.
+#pragma once
+#include <memory>
+#include <string>
+#include <vector>
+
+#include "../../include/ferrum_hip.h"
+#include "layer_ops.h"
+
+namespace fh {
+
+class LayeredModel {
+public:
+    virtual ~LayeredModel() = default;
+    // host weights by tensor name; packed at finalize
+    virtual int set_tensor(const char* name, const float* data, const int64_t* shape, int ndim) = 0;
+    virtual int init_synthetic(uint64_t seed, hipStream_t s) = 0;
+    virtual int finalize(hipStream_t s) = 0;
+    // embedding and every layer; taps: [num_layers][max_tokens][hidden] or null
+    virtual int forward(const BatchView& v, float* taps, bool trace, hipStream_t s) = 0;
+    // final norm + vocabulary projection of `rows` rows of the last forward
+    virtual int head(const int32_t* row_idx, int rows, float* logits, hipStream_t s) = 0;
+    virtual bool has_state() const = 0;           // some layer carries recurrent state
+    virtual bool reads_previous_token() const = 0;
+};
+
+std::unique_ptr<LayeredModel> make_layered_model(const FerrumHipModelConfig& c, const FerrumHipLayeredConfig& lc, const FerrumHipLayerSpec* layers,
+                                                 int state_slots);
+int check_layered_config(const FerrumHipModelConfig& c, const FerrumHipLayeredConfig& lc, const FerrumHipLayerSpec* layers);
+
+}  // namespace fh

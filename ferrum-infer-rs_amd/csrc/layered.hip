@@ -1,0 +1,503 @@
+// Layered models (layered.h): weight packing and the forward pass.
+//
+// A layer is a mixer and, optionally, a feed-forward.  Both sublayers read the residual stream itself; their result is multiplied by a
+// sigmoid gate of the same input, normed (weight stored around zero) and added with a constant factor:
+//     x ← x + m · norm(sub(x) · σ(W x + b))
+// Everything that reads x is ONE projection per sublayer — the gate's rows, then the mixer's (or feed-forward's) input rows, each
+// section with its own activation in the epilogue:
+//     latent attention : [gate σ | q latent | kv latent + shared key part | head gates σ] → norms, rotation, cache write → query up-projection
+//                        → query through W_ukᵀ (per head) → attention over the latents → W_uv (per head, × head gate) → W_o → add + norm
+//     linear recurrence: [gate σ | y gelu | x] → convolution → gates + state (one token) or scan (portions) → W_o → add + norm
+//     feed-forward     : [gate σ | up xIELU] → down → add + norm
+#include <math.h>
+
+#include <algorithm>
+#include <functional>
+#include <unordered_map>
+
+#include "common.h"
+#include "knobs.h"
+#include "layered.h"
+
+namespace fh {
+
+namespace {
+
+uint16_t bf16_bits(float f) {
+    uint32_t u;
+    memcpy(&u, &f, 4);
+    return (uint16_t)((u + 0x7FFFu + ((u >> 16) & 1u)) >> 16);       // round to nearest even (finite weights)
+}
+void store(bf16* dst, float f) { const uint16_t h = bf16_bits(f); memcpy(dst, &h, 2); }
+void store(float* dst, float f) { *dst = f; }
+
+struct HostTensor { std::vector<float> data; std::vector<int64_t> shape; };
+
+// Device memory owned by a model.
+class Arena {
+public:
+    ~Arena() { for (void* p : mem_) (void)hipFree(p); }
+    template <typename T> int alloc(T** p, size_t n) {
+        *p = nullptr;
+        if (!n) return 0;
+        FH_CHECK_HIP(hipMalloc((void**)p, n * sizeof(T)));
+        mem_.push_back(*p);
+        FH_CHECK_HIP(hipMemset(*p, 0, n * sizeof(T)));
+        return 0;
+    }
+    template <typename T> int upload(T** p, const std::vector<T>& v) {
+        if (int rc = alloc(p, v.size())) return rc;
+        FH_CHECK_HIP(hipMemcpy(*p, v.data(), v.size() * sizeof(T), hipMemcpyHostToDevice));
+        return 0;
+    }
+private:
+    std::vector<void*> mem_;
+};
+
+double softplus(double z) { return z > 0 ? z + log1p(exp(-z)) : log1p(exp(z)); }
+
+__device__ __forceinline__ uint64_t mix64(uint64_t x) {
+    x += 0x9E3779B97F4A7C15ull;
+    x = (x ^ (x >> 30)) * 0xBF58476D1CE4E5B9ull;
+    x = (x ^ (x >> 27)) * 0x94D049BB133111EBull;
+    return x ^ (x >> 31);
+}
+// uniform with the given standard deviation
+template <typename E>
+__global__ void synth_kernel(E* p, size_t n, uint64_t seed, float std) {
+    const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i < n) p[i] = (E)(((float)(mix64(seed + i) >> 40) / 8388608.0f - 1.0f) * 1.7320508f * std);
+}
+
+#define FH_TRY(call) do { if (int rc_ = (call)) return rc_; } while (0)
+
+template <typename E>
+class Layered final : public LayeredModel {
+    struct Linear { E* w = nullptr; float* bias = nullptr; int n = 0, k = 0, groups = 1; };
+    struct Layer {
+        FerrumHipLayerSpec s;
+        // fused input projection of the mixer: sections in the order of the comment at the top
+        Linear in, uq, uk, uv, o, ff_in, down;
+        GemmSection in_sec[GEMM_MAX_SECTIONS], ff_sec[2];
+        int in_nsec = 0;
+        int c0 = 0, c1 = 0, c2 = 0;        // columns of the mixer's sections: latent attention: q latent, kv latent, head gates; recurrence: y, x
+        float *norm1 = nullptr, *norm2 = nullptr;
+        LatentDims ld{};
+        float *dq_norm = nullptr, *dkv_norm = nullptr;
+        LatentBuffers<E> lb{};
+        RglruDims rd{};
+        RglruBuffers<E> rb{};
+    };
+
+public:
+    Layered(const FerrumHipModelConfig& c, const FerrumHipLayeredConfig& lc, const FerrumHipLayerSpec* layers, int slots)
+        : c_(c), lc_(lc), slots_(slots), D_(c.hidden), Dp_(pad32(c.hidden)) {
+        for (int i = 0; i < c.num_layers; i++) { Layer L; L.s = layers[i]; dims(L); layers_.push_back(L); }
+    }
+    bool has_state() const override {
+        return std::any_of(layers_.begin(), layers_.end(), [](const Layer& L) { return L.s.mixer == FERRUM_HIP_MIXER_RGLRU; });
+    }
+    bool reads_previous_token() const override { return lc_.bigram_buckets > 0; }
+
+    int set_tensor(const char* name, const float* data, const int64_t* shape, int ndim) override {
+        HostTensor t;
+        t.shape.assign(shape, shape + ndim);
+        size_t n = 1;
+        for (int64_t d : t.shape) n *= (size_t)d;
+        t.data.assign(data, data + n);
+        host_[name] = std::move(t);
+        return 0;
+    }
+
+    int init_synthetic(uint64_t seed, hipStream_t) override { synth_ = true; seed_ = seed; return 0; }
+
+    int finalize(hipStream_t s) override {
+        stream_ = s;
+        const size_t T = c_.max_tokens;
+        // embedding table (gather) and the same table as vocabulary projection; bigram table
+        FH_TRY(table("embed", c_.vocab, &embed_));
+        if (lc_.bigram_buckets > 0) FH_TRY(table("bigram", lc_.bigram_buckets + 1, &bigram_));
+        FH_TRY(pack(&head_, {{"embed", 0, c_.vocab, pad32(c_.vocab)}}, D_));
+        FH_TRY(unit_offset("final.norm", &final_norm_));
+        long in_cols = 0, q_cols = 0, lat_cols = 0, attn_cols = 0, cq_cols = 0, rnn_cols = 0;
+        size_t units = T / RGLRU_CHUNK + c_.max_seqs, partial = 0;
+        for (int li = 0; li < c_.num_layers; li++) {
+            Layer& L = layers_[li];
+            const FerrumHipLayerSpec& sp = L.s;
+            const std::string p = "l" + std::to_string(li) + ".", m = p + "mix.";
+            FH_TRY(unit_offset(p + "norm1", &L.norm1));
+            if (sp.mixer == FERRUM_HIP_MIXER_LATENT_ATTENTION) {
+                const LatentDims& d = L.ld;
+                const int H = d.heads;
+                std::vector<Rows> in = {{p + "rg1", 0, D_, Dp_}, {m + "dq", 0, d.q_rank, d.qp}, {m + "dkv", 0, d.kv_rank, d.kp},
+                                        {m + "dkv", d.kv_rank, d.rot_dim, d.rp}, {m + "g", 0, H, pad32(H)}};
+                FH_TRY(pack(&L.in, in, D_));
+                FH_TRY(bias(&L.in, in, {p + "rg1.b", "", "", "", ""}));
+                std::vector<Rows> q;
+                for (int h = 0; h < H; h++) {
+                    const int r0 = h * (sp.dim + d.rot_dim);
+                    q.push_back({m + "uq", r0, sp.dim, d.dp});
+                    q.push_back({m + "uq", r0 + sp.dim, d.rot_dim, d.rp});
+                }
+                FH_TRY(pack(&L.uq, q, d.q_rank));
+                // per head: W_ukᵀ [latent, plain query dims], W_uv [value dims, latent]
+                FH_TRY(need(m + "uk", {(int64_t)H * sp.dim, d.kv_rank}));
+                FH_TRY(need(m + "uv", {(int64_t)H * d.vdim, d.kv_rank}));
+                const int dim = sp.dim, kr = d.kv_rank, vd = d.vdim;
+                FH_TRY(pack_fn(&L.uk, H, d.kp, d.dp, m + "uk", [&](const float* w, int g, int n, int k) {
+                    return n < kr && k < dim ? w[((size_t)g * dim + k) * kr + n] : 0.f; }));
+                FH_TRY(pack_fn(&L.uv, H, d.vp, d.kp, m + "uv", [&](const float* w, int g, int n, int k) {
+                    return n < vd && k < kr ? w[((size_t)g * vd + n) * kr + k] : 0.f; }));
+                FH_TRY(need(m + "o", {D_, (int64_t)H * vd}));
+                const int vp = d.vp;
+                FH_TRY(pack_fn(&L.o, 1, Dp_, H * vp, m + "o", [&](const float* w, int, int n, int k) {
+                    return n < D_ && k % vp < vd ? w[(size_t)n * H * vd + (k / vp) * vd + k % vp] : 0.f; }));
+                FH_TRY(vec(m + "dq.norm", {d.q_rank}, d.qp, &L.dq_norm));
+                FH_TRY(vec(m + "dkv.norm", {d.kv_rank}, d.kp, &L.dkv_norm));
+                FH_TRY(arena_.alloc(&L.lb.pool, (size_t)c_.kv_num_blocks * latent_block_elems(d)));
+                FH_TRY(rope(sp.rot_base, d.rot_dims, &L.lb.cos_t, &L.lb.sin_t));
+                L.c0 = Dp_; L.c1 = L.c0 + d.qp; L.c2 = L.c1 + d.kp + d.rp;
+                L.in_sec[0] = {0, GEMM_ACT_SIGMOID, 0, 0}; L.in_sec[1] = {L.c0, GEMM_ACT_NONE, 0, 0}; L.in_sec[2] = {L.c2, GEMM_ACT_SIGMOID, 0, 0};
+                L.in_nsec = 3;
+                q_cols = std::max<long>(q_cols, L.uq.n); lat_cols = std::max<long>(lat_cols, (long)H * d.kp);
+                attn_cols = std::max<long>(attn_cols, (long)H * vp); cq_cols = std::max<long>(cq_cols, d.qp);
+                // split attention: only while a forward has fewer than 256 row tiles
+                partial = std::max<size_t>(partial, (size_t)512 * 16 * (d.kp + 4) * 4 * 2);
+            } else {
+                const RglruDims& d = L.rd;
+                const int bs = sp.rnn_width / d.blocks, bp = d.bp, W = sp.rnn_width;
+                std::vector<Rows> in = {{p + "rg1", 0, D_, Dp_}};
+                std::vector<std::string> b = {p + "rg1.b"};
+                for (const char* part : {"y", "x"})
+                    for (int g = 0; g < d.blocks; g++) { in.push_back({m + part, g * bs, bs, bp}); b.push_back(m + part + ".b"); }
+                FH_TRY(pack(&L.in, in, D_));
+                FH_TRY(bias(&L.in, in, b));
+                FH_TRY(need(m + "ra", {d.blocks, bs, bs}));
+                FH_TRY(need(m + "ri", {d.blocks, bs, bs}));
+                // gate tiles: [block][16-channel tile][ra, ri] — packed as 2·bp rows per block in that order
+                const float *ra = data(m + "ra"), *ri = data(m + "ri");
+                Linear gates;
+                FH_TRY(pack_fn(&gates, d.blocks, 2 * bp, bp, m + "ra", [&](const float*, int g, int n, int k) {
+                    const int ch = (n / 32) * 16 + n % 16;
+                    const float* w = (n / 16) % 2 ? ri : ra;
+                    return ch < bs && k < bs ? w[((size_t)g * bs + ch) * bs + k] : 0.f; }));
+                L.rb.gate_w = gates.w;
+                auto padded = [&](const std::string& name, const float** out, bool sp_fold, int taps) -> int {
+                    const int64_t n = W;
+                    if (taps > 1 || name == m + "conv") FH_TRY(need(name, {n, taps}));
+                    else if (name == m + "ra.b" || name == m + "ri.b") FH_TRY(need(name, {d.blocks, bs}));
+                    else FH_TRY(need(name, {n}));
+                    const float* src = data(name);
+                    std::vector<float> v((size_t)taps * d.wp, 0.f);
+                    for (int j = 0; j < taps; j++)
+                        for (int ch = 0; ch < W; ch++) {
+                            const float x = src ? src[(size_t)ch * taps + j] : 0.25f;
+                            v[(size_t)j * d.wp + (ch / bs) * bp + ch % bs] = sp_fold ? (float)softplus(x) : x;
+                        }
+                    float* dev = nullptr;
+                    FH_TRY(arena_.upload(&dev, v));
+                    *out = dev;
+                    return 0;
+                };
+                FH_TRY(padded(m + "conv", &L.rb.conv_w, false, d.taps));
+                FH_TRY(padded(m + "conv.b", &L.rb.conv_b, false, 1));
+                FH_TRY(padded(m + "ra.b", &L.rb.ra_b, false, 1));
+                FH_TRY(padded(m + "ri.b", &L.rb.ri_b, false, 1));
+                FH_TRY(padded(m + "lam", &L.rb.lam, true, 1));
+                FH_TRY(need(m + "o", {D_, W}));
+                FH_TRY(pack_fn(&L.o, 1, Dp_, d.wp, m + "o", [&](const float* w, int, int n, int k) {
+                    return n < D_ && k % bp < bs ? w[(size_t)n * W + (k / bp) * bs + k % bp] : 0.f; }));
+                FH_TRY(arena_.alloc(&L.rb.conv_state, (size_t)slots_ * std::max(d.taps - 1, 1) * d.wp));
+                FH_TRY(arena_.alloc(&L.rb.state, (size_t)slots_ * d.wp));
+                L.c0 = Dp_; L.c1 = L.c0 + d.wp;
+                L.in_sec[0] = {0, GEMM_ACT_SIGMOID, 0, 0}; L.in_sec[1] = {L.c0, GEMM_ACT_GELU_TANH, 0, 0}; L.in_sec[2] = {L.c1, GEMM_ACT_NONE, 0, 0};
+                L.in_nsec = 3;
+                rnn_cols = std::max<long>(rnn_cols, d.wp);
+            }
+            in_cols = std::max<long>(in_cols, L.in.n);
+            if (sp.ff != FERRUM_HIP_FF_NONE) {
+                FH_TRY(unit_offset(p + "norm2", &L.norm2));
+                const int F = sp.ff_width, Fp = pad32(F);
+                std::vector<Rows> in = {{p + "rg2", 0, D_, Dp_}, {p + "mlp.up", 0, F, Fp}};
+                FH_TRY(pack(&L.ff_in, in, D_));
+                FH_TRY(bias(&L.ff_in, in, {p + "rg2.b", ""}));
+                FH_TRY(pack(&L.down, {{p + "mlp.down", 0, D_, Dp_}}, F));
+                FH_TRY(need(p + "mlp.act", {2}));
+                const float* act = data(p + "mlp.act");
+                L.ff_sec[0] = {0, GEMM_ACT_SIGMOID, 0, 0};
+                L.ff_sec[1] = {Dp_, GEMM_ACT_XIELU, (float)softplus(act ? act[0] : 0.5f), (float)softplus(act ? act[1] : 0.5f)};
+                in_cols = std::max<long>(in_cols, L.ff_in.n);
+            }
+        }
+        host_.clear();
+        FH_TRY(arena_.alloc(&x_, T * D_));
+        FH_TRY(arena_.alloc(&xb_, T * Dp_));
+        FH_TRY(arena_.alloc(&in_, T * in_cols));
+        FH_TRY(arena_.alloc(&sub_, T * Dp_));
+        FH_TRY(arena_.alloc(&cq_, T * cq_cols));
+        FH_TRY(arena_.alloc(&q_, T * q_cols));
+        FH_TRY(arena_.alloc(&q_lat_, T * lat_cols));
+        FH_TRY(arena_.alloc(&o_lat_, T * lat_cols));
+        FH_TRY(arena_.alloc(&attn_, T * attn_cols));
+        partial_bytes_ = partial;
+        FH_TRY(arena_.alloc(&partial_, partial / 4));
+        FH_TRY(arena_.alloc(&u_, T * rnn_cols));
+        FH_TRY(arena_.alloc(&rnn_out_, T * rnn_cols));
+        FH_TRY(arena_.alloc(&decay_, T * rnn_cols));
+        FH_TRY(arena_.alloc(&drive_, T * rnn_cols));
+        FH_TRY(arena_.alloc(&chunk_a_, units * rnn_cols));
+        FH_TRY(arena_.alloc(&chunk_h_, units * rnn_cols));
+        FH_TRY(arena_.alloc(&head_in_, (size_t)c_.max_seqs * Dp_));
+        for (Layer& L : layers_) {
+            L.lb.q = q_; L.lb.q_lat = q_lat_; L.lb.o_lat = o_lat_; L.lb.partial = partial_; L.lb.partial_bytes = partial_bytes_;
+            L.rb.x = in_ + L.c1; L.rb.y = in_ + L.c0; L.rb.ld = L.in.n;
+            L.rb.u = u_; L.rb.out = rnn_out_; L.rb.decay = decay_; L.rb.drive = drive_; L.rb.chunk_a = chunk_a_; L.rb.chunk_h = chunk_h_;
+        }
+        FH_CHECK_HIP(hipStreamSynchronize(s));
+        return 0;
+    }
+
+    int forward(const BatchView& v, float* taps, bool trace, hipStream_t s) override {
+#define RUN(call)                                                                                \
+    do {                                                                                         \
+        if (trace) fprintf(stderr, "[ferrum_hip] layer %d T=%d %.60s\n", li, v.T, #call);        \
+        FH_TRY(call);                                                                            \
+        if (trace) FH_CHECK_HIP(hipStreamSynchronize(s));                                        \
+    } while (0)
+        int li = -1;
+        const int T = v.T;
+        const float eps = c_.rms_eps;
+        RUN(embed_bigram<E>(embed_, bigram_, lc_.bigram_buckets, lc_.bigram_mul_prev, lc_.bigram_mul_cur, v, x_, xb_, D_, Dp_, s));
+        for (li = 0; li < c_.num_layers; li++) {
+            Layer& L = layers_[li];
+            TiledGemm<E> g = linear(L.in, xb_, Dp_, T, in_, L.in.n);
+            g.nsec = L.in_nsec;
+            std::copy(L.in_sec, L.in_sec + L.in_nsec, g.sec);
+            RUN(tiled_gemm(g, s));
+            if (L.s.mixer == FERRUM_HIP_MIXER_LATENT_ATTENTION) {
+                const LatentDims& d = L.ld;
+                RUN(latent_prepare<E>(in_ + L.c0, in_ + L.c1, L.in.n, L.dq_norm, L.dkv_norm, eps, d, L.lb, v, cq_, s));
+                RUN(tiled_gemm(linear(L.uq, cq_, d.qp, T, q_, L.uq.n), s));
+                TiledGemm<E> k = linear(L.uk, q_, L.uq.n, T, q_lat_, (long)d.heads * d.kp);
+                k.x_group = d.dp + d.rp; k.out_group = d.kp;
+                RUN(tiled_gemm(k, s));
+                RUN(latent_attention<E>(d, L.lb, v, s));
+                TiledGemm<E> u = linear(L.uv, o_lat_, (long)d.heads * d.kp, T, attn_, (long)d.heads * d.vp);
+                u.x_group = d.kp; u.out_group = d.vp; u.row_scale = in_ + L.c2; u.ld_scale = L.in.n;
+                RUN(tiled_gemm(u, s));
+                RUN(tiled_gemm(linear_f32(L.o, attn_, (long)d.heads * d.vp, T, sub_, Dp_), s));
+            } else {
+                RUN(rglru_forward<E>(L.rd, L.rb, v, s));
+                RUN(tiled_gemm(linear_f32(L.o, rnn_out_, L.rd.wp, T, sub_, Dp_), s));
+            }
+            RUN(gated_post_norm_add<E>(sub_, Dp_, in_, L.in.n, L.norm1, lc_.residual_mult, eps, x_, xb_, T, D_, Dp_, s));
+            if (L.s.ff != FERRUM_HIP_FF_NONE) {
+                TiledGemm<E> f = linear(L.ff_in, xb_, Dp_, T, in_, L.ff_in.n);
+                f.nsec = 2; f.sec[0] = L.ff_sec[0]; f.sec[1] = L.ff_sec[1];
+                RUN(tiled_gemm(f, s));
+                RUN(tiled_gemm(linear_f32(L.down, in_ + Dp_, L.ff_in.n, T, sub_, Dp_), s));
+                RUN(gated_post_norm_add<E>(sub_, Dp_, in_, L.ff_in.n, L.norm2, lc_.residual_mult, eps, x_, xb_, T, D_, Dp_, s));
+            }
+            if (taps) FH_CHECK_HIP(hipMemcpyAsync(taps + (size_t)li * c_.max_tokens * D_, x_, (size_t)T * D_ * 4, hipMemcpyDeviceToDevice, s));
+        }
+#undef RUN
+        return 0;
+    }
+
+    int head(const int32_t* row_idx, int rows, float* logits, hipStream_t s) override {
+        FH_TRY(rms_norm_rows<E>(x_, row_idx, final_norm_, c_.rms_eps, head_in_, rows, D_, Dp_, s));
+        TiledGemm<E> g = linear_f32(head_, head_in_, Dp_, rows, logits, c_.vocab);
+        g.n_store = c_.vocab;
+        return tiled_gemm(g, s);
+    }
+
+private:
+    void dims(Layer& L) {
+        const FerrumHipLayerSpec& s = L.s;
+        if (s.mixer == FERRUM_HIP_MIXER_LATENT_ATTENTION)
+            L.ld = {s.heads, s.kv_rank, s.q_rank, s.rot_dim, s.rot_dims, s.vdim, pad32(s.dim), pad32(s.rot_dim), pad32(s.kv_rank), pad32(s.q_rank),
+                    pad32(s.vdim), s.window, s.scale};
+        else
+            L.rd = {s.rnn_blocks, pad32(s.rnn_width / s.rnn_blocks), s.rnn_blocks * pad32(s.rnn_width / s.rnn_blocks), s.conv_taps};
+    }
+    static TiledGemm<E> linear(const Linear& w, const E* x, long ldx, int m, E* out, long ldo) {
+        TiledGemm<E> g;
+        g.x = x; g.ldx = ldx; g.w = w.w; g.bias = w.bias; g.m = m; g.n = w.n; g.k = w.k; g.groups = w.groups; g.out = out; g.ldo = ldo;
+        return g;
+    }
+    static TiledGemm<E> linear_f32(const Linear& w, const E* x, long ldx, int m, float* out, long ldo) {
+        TiledGemm<E> g = linear(w, x, ldx, m, nullptr, ldo);
+        g.out_f32 = out;
+        return g;
+    }
+
+    // ── weights ──
+    struct Rows { std::string name; int row0, rows, rows_pad; };      // a run of a matrix's rows, zero-padded
+    const float* data(const std::string& name) const {
+        auto it = host_.find(name);
+        return it == host_.end() ? nullptr : it->second.data.data();
+    }
+    int need(const std::string& name, const std::vector<int64_t>& shape) {
+        if (synth_) return 0;
+        auto it = host_.find(name);
+        FH_REQUIRE(it != host_.end(), "layered model: tensor '%s' missing", name.c_str());
+        FH_REQUIRE(it->second.shape == shape, "layered model: tensor '%s' has another shape than the configuration says", name.c_str());
+        return 0;
+    }
+    int upload_tiles(Linear* L, int groups, int n, int k, const std::function<float(int, int, int)>& at) {
+        L->n = n; L->k = k; L->groups = groups;
+        const size_t total = (size_t)groups * n * k;
+        if (synth_) {
+            FH_TRY(arena_.alloc(&L->w, total));
+            hipLaunchKernelGGL(synth_kernel<E>, dim3((unsigned)((total + 255) / 256)), dim3(256), 0, stream_, L->w, total, mix(++seed_), 1.0f / sqrtf((float)k));
+            FH_CHECK_LAUNCH();
+            return 0;
+        }
+        std::vector<E> v(total);
+        const int ks = k / 32;
+        for (int g = 0; g < groups; g++)
+            for (int r = 0; r < n; r++)
+                for (int c = 0; c < k; c++) {
+                    const size_t o = ((((size_t)g * (n / 16) + r / 16) * ks + c / 32) * 64 + ((c % 32) / 8) * 16 + r % 16) * 8 + c % 8;
+                    store(&v[o], at(g, r, c));
+                }
+        return arena_.upload(&L->w, v);
+    }
+    static uint64_t mix(uint64_t x) { return x * 0x9E3779B97F4A7C15ull ^ (x >> 7); }
+    int pack_fn(Linear* L, int groups, int n, int k, const std::string& name, const std::function<float(const float*, int, int, int)>& at) {
+        const float* w = data(name);
+        return upload_tiles(L, groups, n, k, [&](int g, int r, int c) { return at(w, g, r, c); });
+    }
+    // rows of several matrices, all with `cols` input columns, one below the other
+    int pack(Linear* L, const std::vector<Rows>& runs, int cols) {
+        std::vector<const float*> row;
+        for (const Rows& r : runs) {
+            if (!synth_) {
+                auto it = host_.find(r.name);
+                FH_REQUIRE(it != host_.end(), "layered model: tensor '%s' missing", r.name.c_str());
+                const std::vector<int64_t>& sh = it->second.shape;
+                FH_REQUIRE(sh.size() == 2 && sh[1] == cols && sh[0] == full_rows(r.name, runs), "layered model: tensor '%s' has another shape than the configuration says", r.name.c_str());
+            }
+            const float* w = data(r.name);
+            for (int i = 0; i < r.rows_pad; i++) row.push_back(w && i < r.rows ? w + (size_t)(r.row0 + i) * cols : nullptr);
+        }
+        return upload_tiles(L, 1, (int)row.size(), pad32(cols), [&](int, int r, int c) { return row[r] && c < cols ? row[r][c] : 0.f; });
+    }
+    static int64_t full_rows(const std::string& name, const std::vector<Rows>& runs) {
+        int64_t n = 0;
+        for (const Rows& r : runs) if (r.name == name) n = std::max<int64_t>(n, r.row0 + r.rows);
+        return n;
+    }
+    int bias(Linear* L, const std::vector<Rows>& runs, const std::vector<std::string>& names) {
+        std::vector<float> v;
+        for (size_t i = 0; i < runs.size(); i++) {
+            if (!names[i].empty()) FH_TRY(need(names[i], {full_rows(runs[i].name, runs)}));
+            const float* b = names[i].empty() ? nullptr : data(names[i]);
+            for (int r = 0; r < runs[i].rows_pad; r++) v.push_back(b && r < runs[i].rows ? b[runs[i].row0 + r] : 0.f);
+        }
+        return arena_.upload(&L->bias, v);
+    }
+    int vec(const std::string& name, const std::vector<int64_t>& shape, int n_pad, float** out) {
+        FH_TRY(need(name, shape));
+        std::vector<float> v(n_pad, 0.f);
+        const float* w = data(name);
+        for (int64_t i = 0; i < shape[0]; i++) v[i] = w ? w[i] : 1.f;
+        return arena_.upload(out, v);
+    }
+    int unit_offset(const std::string& name, float** out) {        // stored around zero: 1 + w
+        FH_TRY(need(name, {D_}));
+        std::vector<float> v(pad32(D_), 0.f);
+        const float* w = data(name);
+        for (int i = 0; i < D_; i++) v[i] = 1.f + (w ? w[i] : 0.f);
+        return arena_.upload(out, v);
+    }
+    int table(const std::string& name, int rows, E** out) {
+        FH_TRY(need(name, {rows, D_}));
+        const size_t n = (size_t)rows * D_;
+        if (synth_) {
+            FH_TRY(arena_.alloc(out, n));
+            hipLaunchKernelGGL(synth_kernel<E>, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, stream_, *out, n, mix(++seed_), 1.0f);
+            FH_CHECK_LAUNCH();
+            return 0;
+        }
+        std::vector<E> v(n);
+        const float* w = data(name);
+        for (size_t i = 0; i < n; i++) store(&v[i], w[i]);
+        return arena_.upload(out, v);
+    }
+    // angle tables in double, stored fp32 like the other models'; layers with the same rotation share one
+    int rope(double base, int dims, const float** cos_t, const float** sin_t) {
+        for (const Rope& r : ropes_)
+            if (r.base == base && r.dims == dims) { *cos_t = r.c; *sin_t = r.s; return 0; }
+        const int half = dims / 2;
+        std::vector<float> cs((size_t)c_.max_seq_len * half), sn(cs.size());
+        for (int p = 0; p < c_.max_seq_len; p++)
+            for (int i = 0; i < half; i++) {
+                const double a = (double)p * pow(base, -2.0 * i / dims);
+                cs[(size_t)p * half + i] = (float)cos(a);
+                sn[(size_t)p * half + i] = (float)sin(a);
+            }
+        Rope r{base, dims, nullptr, nullptr};
+        FH_TRY(arena_.upload(&r.c, cs));
+        FH_TRY(arena_.upload(&r.s, sn));
+        ropes_.push_back(r);
+        *cos_t = r.c; *sin_t = r.s;
+        return 0;
+    }
+    struct Rope { double base; int dims; float *c, *s; };
+
+    FerrumHipModelConfig c_;
+    FerrumHipLayeredConfig lc_;
+    int slots_, D_, Dp_;
+    hipStream_t stream_ = nullptr;
+    bool synth_ = false;
+    uint64_t seed_ = 0;
+    Arena arena_;
+    std::unordered_map<std::string, HostTensor> host_;
+    std::vector<Layer> layers_;
+    std::vector<Rope> ropes_;
+    Linear head_;
+    E *embed_ = nullptr, *bigram_ = nullptr;
+    float* final_norm_ = nullptr;
+    // activations of one forward
+    float *x_ = nullptr, *sub_ = nullptr, *partial_ = nullptr, *decay_ = nullptr, *drive_ = nullptr, *chunk_a_ = nullptr, *chunk_h_ = nullptr;
+    E *xb_ = nullptr, *in_ = nullptr, *cq_ = nullptr, *q_ = nullptr, *q_lat_ = nullptr, *o_lat_ = nullptr, *attn_ = nullptr, *u_ = nullptr,
+      *rnn_out_ = nullptr, *head_in_ = nullptr;
+    size_t partial_bytes_ = 0;
+};
+
+}  // namespace
+
+int check_layered_config(const FerrumHipModelConfig& c, const FerrumHipLayeredConfig& lc, const FerrumHipLayerSpec* layers) {
+    FH_REQUIRE(c.num_layers > 0 && c.hidden > 0 && c.vocab > 0, "layered model: layers=%d hidden=%d vocab=%d", c.num_layers, c.hidden, c.vocab);
+    FH_REQUIRE(c.max_seqs > 0 && c.max_tokens >= c.max_seqs && c.kv_num_blocks > 0 && c.max_seq_len > 0,
+               "layered model: max_seqs/max_tokens/kv_num_blocks/max_seq_len must be positive");
+    FH_REQUIRE(c.tp_world <= 1, "layered model: tensor parallelism is not available");
+    FH_REQUIRE(lc.dtype == FERRUM_HIP_DTYPE_BF16 || lc.dtype == FERRUM_HIP_DTYPE_F32, "layered model: dtype %d", lc.dtype);
+    FH_REQUIRE(lc.bigram_buckets >= 0 && lc.state_slots >= 0, "layered model: bigram buckets %d, state slots %d", lc.bigram_buckets, lc.state_slots);
+    for (int i = 0; i < c.num_layers; i++) {
+        const FerrumHipLayerSpec& s = layers[i];
+        if (s.mixer == FERRUM_HIP_MIXER_LATENT_ATTENTION) {
+            FH_REQUIRE(s.heads > 0 && s.dim > 0 && s.rot_dim > 0 && s.vdim > 0 && s.q_rank > 0 && s.kv_rank > 0 && s.window > 0,
+                       "layer %d: latent attention sizes must be positive", i);
+            FH_REQUIRE(s.rot_dims >= 0 && s.rot_dims % 2 == 0 && s.rot_dims <= s.rot_dim && (s.rot_dims == 0 || s.rot_base > 0.0),
+                       "layer %d: rotated dimensions %d of %d", i, s.rot_dims, s.rot_dim);
+        } else if (s.mixer == FERRUM_HIP_MIXER_RGLRU) {
+            FH_REQUIRE(s.rnn_width > 0 && s.rnn_blocks > 0 && s.rnn_width % s.rnn_blocks == 0 && s.conv_taps > 0,
+                       "layer %d: recurrence of width %d in %d blocks, %d taps", i, s.rnn_width, s.rnn_blocks, s.conv_taps);
+        } else {
+            set_error("layer %d: unknown mixer %d", i, s.mixer);
+            return FERRUM_HIP_UNSUPPORTED;
+        }
+        FH_REQUIRE(s.ff == FERRUM_HIP_FF_NONE || (s.ff == FERRUM_HIP_FF_XIELU && s.ff_width > 0), "layer %d: feed-forward %d of width %d", i, s.ff, s.ff_width);
+    }
+    return 0;
+}
+
+std::unique_ptr<LayeredModel> make_layered_model(const FerrumHipModelConfig& c, const FerrumHipLayeredConfig& lc, const FerrumHipLayerSpec* layers,
+                                                 int state_slots) {
+    if (lc.dtype == FERRUM_HIP_DTYPE_F32) return std::make_unique<Layered<float>>(c, lc, layers, state_slots);
+    return std::make_unique<Layered<bf16>>(c, lc, layers, state_slots);
+}
+
+}  // namespace fh

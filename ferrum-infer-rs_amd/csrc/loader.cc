@@ -8,6 +8,7 @@
 //   * quantize_config.json or config.json "quantization_config"   native_safetensors.rs:1475-1530, config.rs:26-45
 //   * config.json field extraction and per-architecture defaults  ferrum-models/src/definition.rs:225-375,
 //     models/llama_family.rs:596-680,733-810, moe_config.rs:91-130
+//   * layered architectures (Nerenex): per-layer descriptions and weights by name
 //   * tensor names                                        models/llama_family.rs:900-945, qwen3_moe/load.rs:178-260
 // Pure host code: nothing here touches the GPU except through ferrum_hip_model_set_* (runner.hip).
 #include <fcntl.h>
@@ -25,149 +26,9 @@
 
 #include "../../include/ferrum_hip.h"
 #include "common.h"
+#include "json.h"
 
 namespace fh {
-namespace json {
-
-struct Value {
-    enum Kind { Null, Bool, Num, Str, Arr, Obj } kind = Null;
-    bool b = false;
-    double num = 0.0;
-    std::string str;
-    std::vector<Value> arr;
-    std::vector<std::pair<std::string, Value>> obj;   // insertion order kept
-
-    const Value* get(const std::string& key) const {
-        if (kind != Obj) return nullptr;
-        for (const auto& kv : obj)
-            if (kv.first == key) return &kv.second;
-        return nullptr;
-    }
-    bool is_num() const { return kind == Num; }
-    bool is_u64() const { return kind == Num && num >= 0.0 && std::floor(num) == num; }
-};
-
-struct Parser {
-    const char* p;
-    const char* end;
-    std::string err;
-
-    void ws() {
-        while (p < end && (*p == ' ' || *p == '\n' || *p == '\t' || *p == '\r')) p++;
-    }
-    bool fail(const char* m) {
-        if (err.empty()) err = m;
-        return false;
-    }
-    bool parse_string(std::string& out) {
-        if (p >= end || *p != '"') return fail("expected string");
-        p++;
-        out.clear();
-        while (p < end && *p != '"') {
-            char c = *p++;
-            if (c != '\\') { out.push_back(c); continue; }
-            if (p >= end) return fail("bad escape");
-            char e = *p++;
-            switch (e) {
-            case '"': out.push_back('"'); break;
-            case '\\': out.push_back('\\'); break;
-            case '/': out.push_back('/'); break;
-            case 'b': out.push_back('\b'); break;
-            case 'f': out.push_back('\f'); break;
-            case 'n': out.push_back('\n'); break;
-            case 'r': out.push_back('\r'); break;
-            case 't': out.push_back('\t'); break;
-            case 'u': {
-                if (end - p < 4) return fail("bad \\u escape");
-                unsigned cp = 0;
-                for (int i = 0; i < 4; i++) {
-                    char h = *p++;
-                    cp <<= 4;
-                    if (h >= '0' && h <= '9') cp |= h - '0';
-                    else if (h >= 'a' && h <= 'f') cp |= h - 'a' + 10;
-                    else if (h >= 'A' && h <= 'F') cp |= h - 'A' + 10;
-                    else return fail("bad \\u escape");
-                }
-                if (cp < 0x80) out.push_back((char)cp);
-                else if (cp < 0x800) { out.push_back((char)(0xC0 | (cp >> 6))); out.push_back((char)(0x80 | (cp & 0x3F))); }
-                else { out.push_back((char)(0xE0 | (cp >> 12))); out.push_back((char)(0x80 | ((cp >> 6) & 0x3F))); out.push_back((char)(0x80 | (cp & 0x3F))); }
-                break;
-            }
-            default: return fail("bad escape");
-            }
-        }
-        if (p >= end) return fail("unterminated string");
-        p++;
-        return true;
-    }
-    bool parse_value(Value& v, int depth = 0) {
-        if (depth > 64) return fail("nesting too deep");
-        ws();
-        if (p >= end) return fail("unexpected end");
-        char c = *p;
-        if (c == '{') {
-            v.kind = Value::Obj;
-            p++;
-            ws();
-            if (p < end && *p == '}') { p++; return true; }
-            for (;;) {
-                ws();
-                std::string key;
-                if (!parse_string(key)) return false;
-                ws();
-                if (p >= end || *p != ':') return fail("expected ':'");
-                p++;
-                Value child;
-                if (!parse_value(child, depth + 1)) return false;
-                v.obj.emplace_back(std::move(key), std::move(child));
-                ws();
-                if (p < end && *p == ',') { p++; continue; }
-                if (p < end && *p == '}') { p++; return true; }
-                return fail("expected ',' or '}'");
-            }
-        }
-        if (c == '[') {
-            v.kind = Value::Arr;
-            p++;
-            ws();
-            if (p < end && *p == ']') { p++; return true; }
-            for (;;) {
-                Value child;
-                if (!parse_value(child, depth + 1)) return false;
-                v.arr.push_back(std::move(child));
-                ws();
-                if (p < end && *p == ',') { p++; continue; }
-                if (p < end && *p == ']') { p++; return true; }
-                return fail("expected ',' or ']'");
-            }
-        }
-        if (c == '"') { v.kind = Value::Str; return parse_string(v.str); }
-        if (end - p >= 4 && !strncmp(p, "true", 4)) { v.kind = Value::Bool; v.b = true; p += 4; return true; }
-        if (end - p >= 5 && !strncmp(p, "false", 5)) { v.kind = Value::Bool; v.b = false; p += 5; return true; }
-        if (end - p >= 4 && !strncmp(p, "null", 4)) { v.kind = Value::Null; p += 4; return true; }
-        // number (also accepts the non-standard NaN/Infinity python's json may emit: treated as null)
-        if (end - p >= 3 && !strncmp(p, "NaN", 3)) { p += 3; return true; }
-        if (end - p >= 8 && !strncmp(p, "Infinity", 8)) { p += 8; return true; }
-        const char* s = p;
-        if (p < end && (*p == '-' || *p == '+')) p++;
-        while (p < end && ((*p >= '0' && *p <= '9') || *p == '.' || *p == 'e' || *p == 'E' || *p == '-' || *p == '+')) p++;
-        if (p == s) return fail("unexpected character");
-        v.kind = Value::Num;
-        v.num = strtod(std::string(s, p).c_str(), nullptr);
-        return true;
-    }
-};
-
-static bool parse(const char* data, size_t len, Value& out, std::string& err) {
-    Parser ps{data, data + len, {}};
-    if (!ps.parse_value(out)) { err = ps.err; return false; }
-    ps.ws();
-    if (ps.p != ps.end) { err = "trailing characters"; return false; }
-    return true;
-}
-
-}  // namespace json
-
 static bool read_file(const std::string& path, std::string& out) {
     FILE* f = fopen(path.c_str(), "rb");
     if (!f) return false;
@@ -438,8 +299,80 @@ static const Value* cfg_get(const FerrumHipCheckpoint* ck, const char* key) { re
 static std::string architecture(const FerrumHipCheckpoint* ck) {
     const Value* a = cfg_get(ck, "architectures");
     if (a && a->kind == Value::Arr && !a->arr.empty() && a->arr[0].kind == Value::Str) return a->arr[0].str;
-    const Value* mt = cfg_get(ck, "model_type");
-    return mt && mt->kind == Value::Str ? mt->str : "";
+    for (const char* key : {"model_type", "architecture"})
+        if (const Value* v = cfg_get(ck, key); v && v->kind == Value::Str) return v->str;
+    return "";
+}
+
+// ── layered architectures ──
+static bool is_layered_arch(const std::string& arch) { return arch == "Nerenex"; }
+
+// required numbers of a config object; the first one missing or out of place is named in the error
+struct Fields {
+    const Value* obj;
+    std::string where, missing;
+    double num(const char* key) {
+        const Value* v = obj ? obj->get(key) : nullptr;
+        if (!(v && v->is_num())) { if (missing.empty()) missing = where + "." + key; return 0.0; }
+        return v->num;
+    }
+    int32_t size(const char* key) {
+        const double d = num(key);
+        if (!(d >= 0.0 && d <= 2147483647.0 && std::floor(d) == d)) { if (missing.empty()) missing = where + "." + key; return 0; }
+        return (int32_t)d;
+    }
+    Fields sub(const char* key) { return Fields{obj ? obj->get(key) : nullptr, where + "." + key, missing}; }
+};
+#define FH_FIELDS_OK(f) FH_REQUIRE((f).missing.empty(), "config.json: '%s' is missing or not a valid number", (f).missing.c_str())
+
+static int layered_spec(const Value& v, int index, FerrumHipLayerSpec* s) {
+    memset(s, 0, sizeof(*s));
+    const std::string at = "layers[" + std::to_string(index) + "]";
+    const Value *type = v.get("type"), *ff = v.get("mlp");
+    FH_REQUIRE(type && type->kind == Value::Str, "config.json: %s has no type", at.c_str());
+    Fields m{v.get("mixer"), at + ".mixer", ""};
+    if (type->str == "latent_attention") {
+        s->mixer = FERRUM_HIP_MIXER_LATENT_ATTENTION;
+        s->heads = m.size("heads"); s->dim = m.size("dim"); s->rot_dim = m.size("rot_dim"); s->vdim = m.size("vdim");
+        s->q_rank = m.size("q_rank"); s->kv_rank = m.size("kv_rank"); s->scale = (float)m.num("scale");
+        Fields rot = m.sub("rot"), mask = m.sub("mask");
+        s->rot_dims = rot.size("dims"); s->rot_base = rot.num("base"); s->window = mask.size("size");
+        FH_FIELDS_OK(m); FH_FIELDS_OK(rot); FH_FIELDS_OK(mask);
+    } else if (type->str == "rglru") {
+        s->mixer = FERRUM_HIP_MIXER_RGLRU;
+        s->rnn_width = m.size("width"); s->rnn_blocks = m.size("blocks"); s->conv_taps = m.size("conv");
+        FH_FIELDS_OK(m);
+    } else {
+        set_error("config.json: %s has the unknown type '%s'", at.c_str(), type->str.c_str());
+        return FERRUM_HIP_UNSUPPORTED;
+    }
+    if (!ff || ff->kind != Value::Obj) return 0;
+    const Value* kind = ff->get("kind");
+    if (!(kind && kind->kind == Value::Str && kind->str == "dense")) {
+        set_error("config.json: %s.mlp has an unknown kind", at.c_str());
+        return FERRUM_HIP_UNSUPPORTED;
+    }
+    Fields f{ff, at + ".mlp", ""};
+    s->ff = FERRUM_HIP_FF_XIELU;
+    s->ff_width = f.size("ff");
+    FH_FIELDS_OK(f);
+    return 0;
+}
+
+static int layered_model_config(const FerrumHipCheckpoint* ck, int max_seq_len_cap, FerrumHipModelConfig* cfg) {
+    Fields f{&ck->config, "config", ""};
+    const Value* layers = cfg_get(ck, "layers");
+    FH_REQUIRE(layers && layers->kind == Value::Arr && !layers->arr.empty(), "config.json: 'layers' is missing or empty");
+    cfg->num_layers = (int32_t)layers->arr.size();
+    cfg->hidden = f.size("width");
+    cfg->vocab = f.size("vocab");
+    Fields norm = f.sub("norm");
+    cfg->rms_eps = (float)norm.num("eps");
+    FH_FIELDS_OK(f); FH_FIELDS_OK(norm);
+    cfg->max_seq_len = max_seq_len_cap > 0 ? max_seq_len_cap : 32768;      // (the architecture sets no limit; the angle tables need one)
+    cfg->group_size = 128;
+    cfg->tp_world = 1;
+    return 0;
 }
 
 }  // namespace fh
@@ -595,6 +528,10 @@ int ferrum_hip_checkpoint_model_config(const FerrumHipCheckpoint* ck, int max_se
     memset(cfg, 0, sizeof(*cfg));
     const std::string arch = architecture(ck);
     if (arch_out && arch_cap) snprintf(arch_out, arch_cap, "%s", arch.c_str());
+    if (is_layered_arch(arch)) {
+        if (tied_lm_head) *tied_lm_head = 1;
+        return layered_model_config(ck, max_seq_len_cap, cfg);
+    }
     enum { Llama, Qwen3, Qwen3Moe, Mistral, Gemma3, Qwen2 } fam;
     if (arch == "LlamaForCausalLM" || arch == "llama") fam = Llama;
     else if (arch == "Gemma3ForCausalLM" || arch == "Gemma3ForConditionalGeneration" || arch == "gemma3_text" || arch == "gemma3") fam = Gemma3;
@@ -603,7 +540,7 @@ int ferrum_hip_checkpoint_model_config(const FerrumHipCheckpoint* ck, int max_se
     else if (arch == "Qwen3MoeForCausalLM" || arch == "qwen3_moe") fam = Qwen3Moe;
     else if (arch == "MistralForCausalLM" || arch == "mistral") fam = Mistral;
     else {
-        set_error("checkpoint: architecture '%s' is not supported by the HIP runner (Llama, Mistral, Qwen2, Qwen3, Qwen3-MoE, Gemma-3)", arch.c_str());
+        set_error("checkpoint: architecture '%s' is not supported by the HIP runner (Llama, Mistral, Qwen2, Qwen3, Qwen3-MoE, Gemma-3, Nerenex)", arch.c_str());
         return FERRUM_HIP_UNSUPPORTED;
     }
     auto u = [&](const char* key, const char* alt, double dflt) {
@@ -685,10 +622,49 @@ int ferrum_hip_checkpoint_model_config(const FerrumHipCheckpoint* ck, int max_se
     return 0;
 }
 
+int ferrum_hip_checkpoint_layered_config(const FerrumHipCheckpoint* ck, int* is_layered, FerrumHipLayeredConfig* layered,
+                                         FerrumHipLayerSpec* layers, int capacity) {
+    FH_REQUIRE(ck && is_layered, "checkpoint_layered_config: null argument");
+    *is_layered = is_layered_arch(architecture(ck));
+    if (!*is_layered) return 0;
+    const Value* ls = cfg_get(ck, "layers");
+    FH_REQUIRE(ls && ls->kind == Value::Arr && !ls->arr.empty(), "config.json: 'layers' is missing or empty");
+    if (layered) {
+        memset(layered, 0, sizeof(*layered));
+        Fields f{&ck->config, "config", ""};
+        layered->residual_mult = (float)f.num("residual_mult");
+        FH_FIELDS_OK(f);
+        Fields emb = f.sub("embedding");
+        if (const Value* bg = emb.obj ? emb.obj->get("bigram") : nullptr; bg && bg->kind == Value::Obj) {
+            Fields b{bg, "embedding.bigram", ""};
+            layered->bigram_buckets = b.size("buckets");
+            layered->bigram_mul_prev = b.size("mul_prev");
+            layered->bigram_mul_cur = b.size("mul_cur");
+            FH_FIELDS_OK(b);
+            FH_REQUIRE(layered->bigram_buckets > 0, "config.json: embedding.bigram.buckets must be positive");
+        }
+    }
+    for (int i = 0; layers && i < (int)ls->arr.size() && i < capacity; i++)
+        if (int rc = layered_spec(ls->arr[i], i, &layers[i])) return rc;
+    return 0;
+}
+
 /* Hand every weight of the checkpoint to a created (not yet finalized) runner model, with the reference's tensor names
  * and fusions.  The model must have been created from ferrum_hip_checkpoint_model_config's dimensions. */
 int ferrum_hip_model_load_checkpoint(FerrumHipModel* model, const FerrumHipCheckpoint* ck) {
     FH_REQUIRE(model && ck, "model_load_checkpoint: null argument");
+    if (is_layered_arch(architecture(ck))) {
+        FH_REQUIRE(ferrum_hip_model_is_layered(model), "model_load_checkpoint: a layered checkpoint needs a model from ferrum_hip_model_create_layered");
+        std::vector<float> v;
+        for (const auto& kv : ck->index) {
+            if (kv.second.dtype == StDtype::I32 || kv.second.dtype == StDtype::I64) continue;      // (no layer of these architectures reads one)
+            std::vector<int64_t> shape;
+            if (int rc = read_f32(ck, kv.first, v, &shape)) return rc;
+            if (shape.empty()) shape.push_back(1);
+            if (int rc = ferrum_hip_model_set_tensor_f32(model, kv.first.c_str(), v.data(), shape.data(), (int)shape.size())) return rc;
+        }
+        return 0;
+    }
     FerrumHipModelConfig c;
     int tied = 0;
     if (int rc = ferrum_hip_checkpoint_model_config(ck, 0, &c, nullptr, 0, &tied)) return rc;

@@ -1,0 +1,133 @@
+// Residual stream of the layered models: fp32 throughout, with a copy in the projections' number format written by whoever changes it.
+#include "common.h"
+#include "layer_ops.h"
+
+namespace fh {
+
+template <typename E>
+__global__ __launch_bounds__(256) void embed_bigram_kernel(const E* __restrict__ table, const E* __restrict__ bigram, int buckets,
+                                                           int64_t mul_prev, int64_t mul_cur, BatchView v, float* __restrict__ x,
+                                                           E* __restrict__ xb, int dim, int ldb) {
+    const int t = blockIdx.x;
+    const uint32_t tok = v.tokens[t];
+    long row = 0;
+    if (bigram) {
+        const int seq = v.tok_seq[t];
+        const int64_t prev = t == (int)v.cu[seq] ? (int64_t)v.prev[seq] : (int64_t)v.tokens[t - 1];
+        row = prev < 0 ? buckets : (long)((uint64_t)(prev * mul_prev + (int64_t)tok * mul_cur) % (uint64_t)buckets);
+    }
+    for (int i = threadIdx.x; i < dim; i += 256) {
+        float e = (float)table[(long)tok * dim + i];
+        if (bigram) e += (float)bigram[row * dim + i];
+        x[(long)t * dim + i] = e;
+        xb[(long)t * ldb + i] = (E)e;
+    }
+}
+
+template <typename E>
+int embed_bigram(const E* table, const E* bigram, int buckets, int64_t mul_prev, int64_t mul_cur, const BatchView& v, float* x, E* xb,
+                 int dim, int ldb, hipStream_t s) {
+    hipLaunchKernelGGL(embed_bigram_kernel<E>, dim3(v.T), dim3(256), 0, s, table, bigram, buckets, mul_prev, mul_cur, v, x, xb, dim, ldb);
+    FH_CHECK_LAUNCH();
+    return 0;
+}
+
+__device__ __forceinline__ float block_sum(float q, float* red) {
+    q = wave_reduce_sum(q);
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = q;
+    __syncthreads();
+    float t = 0.f;
+    for (int i = 0; i < (int)(blockDim.x >> 6); i++) t += red[i];
+    return t;
+}
+
+// One workgroup per row; a thread holds up to 4 quads of the row in registers, so the branch is read once.
+template <typename E, bool VEC>
+__global__ __launch_bounds__(1024) void gated_post_norm_add_kernel(const float* __restrict__ sub, long ld_sub, const E* __restrict__ gate,
+                                                                   long ld_gate, const float* __restrict__ w, float mult, float eps,
+                                                                   float* __restrict__ x, E* __restrict__ xb, int dim, int ldb) {
+    __shared__ float red[16];
+    const long row = blockIdx.x;
+    const float* sr = sub + row * ld_sub;
+    const E* gr = gate + row * ld_gate;
+    float* xr = x + row * dim;
+    E* br = xb + row * ldb;
+    float q = 0.f;
+    if (VEC) {
+        typedef E e4 __attribute__((ext_vector_type(4)));
+        floatx4 v[4], xv[4], wv[4];
+#pragma unroll
+        for (int c = 0; c < 4; c++) {
+            const int i = (c * blockDim.x + threadIdx.x) * 4;
+            if (i < dim) {
+                v[c] = *reinterpret_cast<const floatx4*>(sr + i);
+                const e4 gv = *reinterpret_cast<const e4*>(gr + i);
+                xv[c] = *reinterpret_cast<const floatx4*>(xr + i);
+                wv[c] = *reinterpret_cast<const floatx4*>(w + i);
+#pragma unroll
+                for (int j = 0; j < 4; j++) { v[c][j] *= (float)gv[j]; q += v[c][j] * v[c][j]; }
+            }
+        }
+        const float inv = mult / sqrtf(block_sum(q, red) / (float)dim + eps);
+#pragma unroll
+        for (int c = 0; c < 4; c++) {
+            const int i = (c * blockDim.x + threadIdx.x) * 4;
+            if (i < dim) {
+                e4 o;
+#pragma unroll
+                for (int j = 0; j < 4; j++) { xv[c][j] += v[c][j] * inv * wv[c][j]; o[j] = (E)xv[c][j]; }
+                *reinterpret_cast<floatx4*>(xr + i) = xv[c];
+                *reinterpret_cast<e4*>(br + i) = o;
+            }
+        }
+        return;
+    }
+    for (int i = threadIdx.x; i < dim; i += blockDim.x) { const float t = sr[i] * (float)gr[i]; q += t * t; }
+    const float inv = mult / sqrtf(block_sum(q, red) / (float)dim + eps);
+    for (int i = threadIdx.x; i < dim; i += blockDim.x) {
+        const float t = xr[i] + sr[i] * (float)gr[i] * inv * w[i];
+        xr[i] = t;
+        br[i] = (E)t;
+    }
+}
+
+template <typename E>
+int gated_post_norm_add(const float* sub, long ld_sub, const E* gate, long ld_gate, const float* w, float mult, float eps, float* x,
+                        E* xb, int rows, int dim, int ldb, hipStream_t s) {
+    const int threads = rows <= 512 && dim >= 2048 ? 1024 : 256;
+    const bool vec = dim % 4 == 0 && dim <= threads * 16 && ld_sub % 4 == 0 && ld_gate % 4 == 0 && ldb % 4 == 0;
+    if (vec)
+        hipLaunchKernelGGL((gated_post_norm_add_kernel<E, true>), dim3(rows), dim3(threads), 0, s, sub, ld_sub, gate, ld_gate, w, mult, eps, x, xb, dim, ldb);
+    else
+        hipLaunchKernelGGL((gated_post_norm_add_kernel<E, false>), dim3(rows), dim3(threads), 0, s, sub, ld_sub, gate, ld_gate, w, mult, eps, x, xb, dim, ldb);
+    FH_CHECK_LAUNCH();
+    return 0;
+}
+
+template <typename E>
+__global__ __launch_bounds__(256) void rms_norm_rows_kernel(const float* __restrict__ x, const int32_t* __restrict__ row_idx,
+                                                            const float* __restrict__ w, float eps, E* __restrict__ out, int dim, int ldo) {
+    __shared__ float red[4];
+    const float* xr = x + (long)row_idx[blockIdx.x] * dim;
+    float q = 0.f;
+    for (int i = threadIdx.x; i < dim; i += 256) q += xr[i] * xr[i];
+    const float inv = 1.0f / sqrtf(block_sum(q, red) / (float)dim + eps);
+    for (int i = threadIdx.x; i < dim; i += 256) out[(long)blockIdx.x * ldo + i] = (E)(xr[i] * inv * w[i]);
+}
+template <typename E>
+int rms_norm_rows(const float* x, const int32_t* row_idx, const float* w, float eps, E* out, int rows, int dim, int ldo, hipStream_t s) {
+    hipLaunchKernelGGL(rms_norm_rows_kernel<E>, dim3(rows), dim3(256), 0, s, x, row_idx, w, eps, out, dim, ldo);
+    FH_CHECK_LAUNCH();
+    return 0;
+}
+
+#define INSTANTIATE(E)                                                                                                                  \
+    template int embed_bigram<E>(const E*, const E*, int, int64_t, int64_t, const BatchView&, float*, E*, int, int, hipStream_t);        \
+    template int gated_post_norm_add<E>(const float*, long, const E*, long, const float*, float, float, float*, E*, int, int, int,       \
+                                        hipStream_t);                                                                                   \
+    template int rms_norm_rows<E>(const float*, const int32_t*, const float*, float, E*, int, int, int, hipStream_t);
+INSTANTIATE(bf16)
+INSTANTIATE(float)
+#undef INSTANTIATE
+
+}  // namespace fh

@@ -1,0 +1,184 @@
+// Real-gated linear recurrent unit behind a causal depthwise convolution.
+//
+//   u_t = Σ_j taps[j] · x_{t − taps + 1 + j} + b;   r, i = σ(block-diagonal projections of u);   log a = −8 · r · softplus(λ)
+//   S_t = a · S_{t−1} + √(1 − a²) · i · u;   out_t = S_t · y_t
+//
+// The two gate projections of a channel are computed side by side on the matrix cores (tiles interleaved ra, ri), so one lane holds
+// both gates of its (token, channel) and everything from the sigmoids to the state update stays in fp32 registers.  1 − a² is taken as
+// −expm1(2 log a).  One token per sequence: that launch also updates the state and writes the output.  Portions: decay and drive go to
+// memory and a chunked scan (64 tokens per workgroup; chunk totals, carry over chunks, final pass) produces the output.
+// A sequence's first token starts from zero whatever its slot holds, so slots are reused without clearing.
+#include "common.h"
+#include "knobs.h"
+#include "layer_ops.h"
+
+namespace fh {
+
+// value of the convolution's input `back` tokens before token t of its portion (t counts from the portion's start)
+template <typename E>
+__device__ __forceinline__ float conv_input(const RglruBuffers<E>& p, const RglruDims& d, int tok0, int t, int back, int slot, bool fresh, int c) {
+    const int q = t - back;
+    if (q >= 0) return (float)p.x[(long)(tok0 + q) * p.ld + c];
+    if (fresh) return 0.f;                              // (a fresh sequence has no tokens before its portion)
+    return (float)p.conv_state[((long)slot * (d.taps - 1) + (d.taps - 1 + q)) * d.wp + c];
+}
+
+// one thread per (token, channel); with one token per sequence the thread also shifts the channel's stored inputs
+template <typename E>
+__global__ __launch_bounds__(256) void rglru_conv_kernel(RglruDims d, RglruBuffers<E> p, BatchView v) {
+    const int c = blockIdx.x * 256 + threadIdx.x, tok = blockIdx.y;
+    if (c >= d.wp) return;
+    const int seq = v.tok_seq[tok], tok0 = v.cu[seq], slot = v.slots[seq];
+    const bool fresh = v.pos[seq] == 0;
+    float acc = p.conv_b[c];
+    for (int j = 0; j < d.taps; j++) acc += p.conv_w[j * d.wp + c] * conv_input(p, d, tok0, tok - tok0, d.taps - 1 - j, slot, fresh, c);
+    p.u[(long)tok * d.wp + c] = (E)acc;
+    if (v.single)
+        for (int j = 0; j < d.taps - 1; j++) {          // entry j is the input taps − 2 − j tokens back; read before it is overwritten
+            const float in = conv_input(p, d, tok0, 0, d.taps - 2 - j, slot, fresh, c);
+            p.conv_state[((long)slot * (d.taps - 1) + j) * d.wp + c] = (E)in;
+        }
+}
+
+// grid (tile groups, row blocks, blocks of the block-diagonal projections); a wave owns one 16-channel tile (ra and ri)
+template <typename E, int MT, bool STEP>
+__global__ __launch_bounds__(256) void rglru_gates_kernel(RglruDims d, RglruBuffers<E> p, BatchView v) {
+    typedef typename Frag<E>::v8 v8;
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, a = lane >> 4, b = lane & 15;
+    const int tile = blockIdx.x * 4 + wave, rb = blockIdx.y, g = blockIdx.z;
+    if (tile * 16 >= d.bp) return;
+    const int ksteps = d.bp >> 5;
+    const E* xrow[MT];
+#pragma unroll
+    for (int mt = 0; mt < MT; mt++) {
+        const int r = (rb * MT + mt) * 16 + b;
+        xrow[mt] = p.u + (long)(r < v.T ? r : v.T - 1) * d.wp + g * d.bp + 8 * a;
+    }
+    const E* wr = p.gate_w + ((long)(g * (d.bp >> 4) + tile) * 2) * ksteps * 512 + lane * 8;
+    floatx4 acc[MT][2];
+#pragma unroll
+    for (int mt = 0; mt < MT; mt++) { acc[mt][0] = (floatx4){0.f, 0.f, 0.f, 0.f}; acc[mt][1] = (floatx4){0.f, 0.f, 0.f, 0.f}; }
+#pragma unroll 2
+    for (int s = 0; s < ksteps; s++) {
+        const v8 w0 = *reinterpret_cast<const v8*>(wr + (long)s * 512), w1 = *reinterpret_cast<const v8*>(wr + (long)(ksteps + s) * 512);
+#pragma unroll
+        for (int mt = 0; mt < MT; mt++) {
+            const v8 ax = *reinterpret_cast<const v8*>(xrow[mt] + s * 32);
+            acc[mt][0] = Frag<E>::mma(ax, w0, acc[mt][0]);
+            acc[mt][1] = Frag<E>::mma(ax, w1, acc[mt][1]);
+        }
+    }
+    const int c = g * d.bp + tile * 16 + b;
+    const float bra = p.ra_b[c], bri = p.ri_b[c], sp = p.lam[c];
+#pragma unroll
+    for (int mt = 0; mt < MT; mt++)
+#pragma unroll
+        for (int q = 0; q < 4; q++) {
+            const int row = (rb * MT + mt) * 16 + 4 * a + q;
+            if (row >= v.T) continue;
+            const float r = sigmoid_f32(acc[mt][0][q] + bra), in = sigmoid_f32(acc[mt][1][q] + bri);
+            const float log_a = -8.0f * r * sp, decay = expf(log_a);
+            const float drive = sqrtf(fmaxf(0.f, -expm1f(2.0f * log_a))) * in * (float)p.u[(long)row * d.wp + c];
+            if (STEP) {
+                float* st = p.state + (long)v.slots[row] * d.wp + c;       // (token i belongs to sequence i)
+                const float h = v.pos[row] == 0 ? drive : decay * *st + drive;
+                *st = h;
+                p.out[(long)row * d.wp + c] = (E)(h * (float)p.y[(long)row * p.ld + c]);
+            } else {
+                p.decay[(long)row * d.wp + c] = decay;
+                p.drive[(long)row * d.wp + c] = drive;
+            }
+        }
+}
+
+// totals of every chunk that another chunk of its sequence follows: Π decay and the state it would reach from zero
+template <typename E>
+__global__ __launch_bounds__(256) void rglru_chunk_totals_kernel(RglruDims d, RglruBuffers<E> p, BatchView v) {
+    const int c = blockIdx.x * 256 + threadIdx.x, unit = blockIdx.y;
+    const int seq = v.units[2 * unit], t0 = v.units[2 * unit + 1];
+    if (c >= d.wp || t0 + RGLRU_CHUNK >= (int)v.cu[seq + 1]) return;
+    float A = 1.f, h = 0.f;
+#pragma unroll 8
+    for (int t = 0; t < RGLRU_CHUNK; t++) {
+        const float a = p.decay[(long)(t0 + t) * d.wp + c];
+        h = a * h + p.drive[(long)(t0 + t) * d.wp + c];
+        A *= a;
+    }
+    p.chunk_a[(long)unit * d.wp + c] = A;
+    p.chunk_h[(long)unit * d.wp + c] = h;
+}
+// chunk_h[unit] ← state before the chunk (one thread per channel of a sequence walks its chunks)
+template <typename E>
+__global__ __launch_bounds__(64) void rglru_carry_kernel(RglruDims d, RglruBuffers<E> p, BatchView v) {
+    const int c = blockIdx.x * 64 + threadIdx.x, unit0 = blockIdx.y;
+    const int seq = v.units[2 * unit0];
+    if (c >= d.wp || v.units[2 * unit0 + 1] != (int)v.cu[seq]) return;         // only a sequence's first chunk starts a walk
+    const int n = cdiv_dev(v.cu[seq + 1] - v.cu[seq], RGLRU_CHUNK);
+    float h = v.pos[seq] == 0 ? 0.f : p.state[(long)v.slots[seq] * d.wp + c];
+    for (int i = 0; i < n; i += 8) {
+        float A[8], H[8];
+#pragma unroll
+        for (int j = 0; j < 8; j++) {
+            const long o = (long)(unit0 + min(i + j, n - 1)) * d.wp + c;
+            A[j] = p.chunk_a[o];
+            H[j] = p.chunk_h[o];
+        }
+#pragma unroll
+        for (int j = 0; j < 8; j++)
+            if (i + j < n) {
+                p.chunk_h[(long)(unit0 + i + j) * d.wp + c] = h;
+                h = A[j] * h + H[j];
+            }
+    }
+}
+// final pass: states of a chunk from its carry, output, and — last chunk of a sequence — the state and convolution tail it leaves
+template <typename E>
+__global__ __launch_bounds__(256) void rglru_apply_kernel(RglruDims d, RglruBuffers<E> p, BatchView v) {
+    const int c = blockIdx.x * 256 + threadIdx.x, unit = blockIdx.y;
+    if (c >= d.wp) return;
+    const int seq = v.units[2 * unit], t0 = v.units[2 * unit + 1], tok0 = v.cu[seq], end = v.cu[seq + 1], slot = v.slots[seq];
+    const int n = min(RGLRU_CHUNK, end - t0);
+    const bool fresh = v.pos[seq] == 0, many = end - tok0 > RGLRU_CHUNK;
+    float h = many ? p.chunk_h[(long)unit * d.wp + c] : (fresh ? 0.f : p.state[(long)slot * d.wp + c]);
+#pragma unroll 8
+    for (int t = 0; t < n; t++) {
+        const long o = (long)(t0 + t) * d.wp + c;
+        h = p.decay[o] * h + p.drive[o];
+        p.out[o] = (E)(h * (float)p.y[(long)(t0 + t) * p.ld + c]);
+    }
+    if (t0 + n < end) return;
+    p.state[(long)slot * d.wp + c] = h;
+    for (int j = 0; j < d.taps - 1; j++) {
+        const float in = conv_input(p, d, tok0, end - 1 - tok0, d.taps - 2 - j, slot, fresh, c);
+        p.conv_state[((long)slot * (d.taps - 1) + j) * d.wp + c] = (E)in;
+    }
+}
+
+template <typename E>
+int rglru_forward(const RglruDims& d, const RglruBuffers<E>& b, const BatchView& v, hipStream_t s) {
+    const int cb = cdiv(d.wp, 256);
+    hipLaunchKernelGGL(rglru_conv_kernel<E>, dim3(cb, v.T), dim3(256), 0, s, d, b, v);
+    FH_CHECK_LAUNCH();
+    const int mt = v.T <= 16 ? 1 : (v.T <= 32 ? 2 : 4);
+    const dim3 grid(cdiv(d.bp / 16, 4), cdiv(v.T, 16 * mt), d.blocks);
+    form_hit(v.single ? FORM_RGLRU_STEP : FORM_RGLRU_SCAN);
+#define GATES(MT, ST) hipLaunchKernelGGL((rglru_gates_kernel<E, MT, ST>), grid, dim3(256), 0, s, d, b, v)
+    if (v.single) { if (mt == 1) GATES(1, true); else if (mt == 2) GATES(2, true); else GATES(4, true); }
+    else { if (mt == 1) GATES(1, false); else if (mt == 2) GATES(2, false); else GATES(4, false); }
+#undef GATES
+    FH_CHECK_LAUNCH();
+    if (v.single) return 0;
+    if (v.num_units > v.num_seqs) {          // some sequence has more than one chunk
+        hipLaunchKernelGGL(rglru_chunk_totals_kernel<E>, dim3(cb, v.num_units), dim3(256), 0, s, d, b, v);
+        FH_CHECK_LAUNCH();
+        hipLaunchKernelGGL(rglru_carry_kernel<E>, dim3(cdiv(d.wp, 64), v.num_units), dim3(64), 0, s, d, b, v);
+        FH_CHECK_LAUNCH();
+    }
+    hipLaunchKernelGGL(rglru_apply_kernel<E>, dim3(cb, v.num_units), dim3(256), 0, s, d, b, v);
+    FH_CHECK_LAUNCH();
+    return 0;
+}
+template int rglru_forward<bf16>(const RglruDims&, const RglruBuffers<bf16>&, const BatchView&, hipStream_t);
+template int rglru_forward<float>(const RglruDims&, const RglruBuffers<float>&, const BatchView&, hipStream_t);
+
+}  // namespace fh

@@ -9,6 +9,7 @@
 #include "block_allocator.h"
 #include "kernels.h"
 #include "kv_layout.h"
+#include "layered.h"
 
 namespace fh {
 
@@ -38,11 +39,13 @@ struct LayerWeights {
 struct SeqState {
     std::vector<uint32_t> blocks;
     int len = 0;
+    int state_slot = -1;           // recurrent state (layered models); −1: none
+    int64_t last_token = -1;       // last token the model has seen (models that embed token pairs); −1: none yet
 };
 
 // Layout of the per-forward index block (host pinned mirror → device).
 struct IndexLayout {
-    size_t tokens, cu_seqlens, pos_offsets, kv_lens, sampled_idx, block_tables, total;
+    size_t tokens, cu_seqlens, pos_offsets, kv_lens, sampled_idx, tok_seq, prev_tokens, state_slots, scan_units, block_tables, total;
 };
 
 }  // namespace fh
@@ -70,6 +73,12 @@ struct FerrumHipModel {
     std::unique_ptr<fh::BlockAllocator> alloc;
     std::unordered_map<uint64_t, fh::SeqState> seqs;
     uint64_t prefix_hits = 0, prefix_misses = 0, prefix_saved_tokens = 0;   // block-level prefix cache probes
+
+    // layered models: weights, cache memory and the layer order (layered.h); free recurrent-state slots, lowest on top
+    std::unique_ptr<fh::LayeredModel> layered;
+    int state_slots = 0;
+    std::vector<int> free_slots;
+    int batch_units = 0;           // scan chunks of the current batch (index block)
 
     // scratch
     __half *residual = nullptr, *norm_out = nullptr, *qkv_out = nullptr, *q_out = nullptr, *attn_out = nullptr,

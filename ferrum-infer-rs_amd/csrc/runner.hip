@@ -110,11 +110,12 @@ double rope_freq(const FerrumHipModelConfig& c, int i) {
 // kernels/split_qkv_norm_rope_into_paged_cache.cu:9-16).
 __global__ void decode_advance_kernel(const uint32_t* __restrict__ sampled, uint32_t* __restrict__ tokens,
                                       uint32_t* __restrict__ pos_offsets, uint32_t* __restrict__ kv_lens,
-                                      uint32_t* __restrict__ history, int32_t* __restrict__ step_counter, int n) {
+                                      uint32_t* __restrict__ history, int32_t* __restrict__ step_counter, int n, int32_t* __restrict__ prev_tokens) {
     int i = threadIdx.x + blockIdx.x * blockDim.x;
     int step = *step_counter;
     if (i < n) {
         uint32_t t = sampled[i];
+        if (prev_tokens) prev_tokens[i] = (int32_t)tokens[i];
         tokens[i] = t;
         pos_offsets[i] += 1;
         kv_lens[i] += 1;
@@ -384,6 +385,43 @@ int ferrum_hip_model_create(FerrumHipModel** model, const FerrumHipModelConfig* 
     return 0;
 }
 
+int ferrum_hip_model_create_layered(FerrumHipModel** model, const FerrumHipModelConfig* cfg, const FerrumHipLayeredConfig* layered,
+                                    const FerrumHipLayerSpec* layers) {
+    FH_REQUIRE(model && cfg && layered && layers, "model_create_layered: null argument");
+    if (int rc = check_layered_config(*cfg, *layered, layers)) return rc;
+    auto* m = new FerrumHipModel();
+    m->cfg = *cfg;
+    m->cfg.tp_world = 1; m->cfg.tp_rank = 0; m->cfg.expert_parallel = 0; m->cfg.vocab_parallel = 0; m->cfg.num_experts = 0;
+    m->vp_n = cfg->vocab;
+    m->max_blocks_per_seq = cdiv(cfg->max_seq_len, KV_BLOCK);
+    const int slots = layered->state_slots > 0 ? layered->state_slots : cfg->max_seqs;
+    m->layered = make_layered_model(m->cfg, *layered, layers, slots);
+    if (m->layered->has_state()) {
+        m->state_slots = slots;
+        for (int i = slots; i-- > 0;) m->free_slots.push_back(i);
+    }
+    hipError_t e = hipStreamCreateWithFlags(&m->stream, hipStreamNonBlocking);
+    if (e != hipSuccess) { delete m; fh::set_error("model_create_layered: hipStreamCreate: %s", hipGetErrorString(e)); return 1; }
+    m->alloc.reset(new BlockAllocator((uint32_t)cfg->kv_num_blocks));
+    *model = m;
+    return 0;
+}
+
+int ferrum_hip_model_set_tensor_f32(FerrumHipModel* m, const char* name, const float* data, const int64_t* shape, int ndim) {
+    FH_REQUIRE(m && name && data && shape && ndim > 0, "model_set_tensor: bad argument");
+    FH_REQUIRE(m->layered && !m->finalized, "model_set_tensor(%s): weights arrive by name only before the finalize of a layered model", name);
+    return m->layered->set_tensor(name, data, shape, ndim);
+}
+
+int ferrum_hip_model_is_layered(const FerrumHipModel* m) { return m && m->layered; }
+
+int ferrum_hip_model_state_slots(const FerrumHipModel* m, int* total, int* free_slots) {
+    FH_REQUIRE(m, "model_state_slots: null");
+    if (total) *total = m->state_slots;
+    if (free_slots) *free_slots = (int)m->free_slots.size();
+    return 0;
+}
+
 int ferrum_hip_model_destroy(FerrumHipModel* m) {
     if (!m) return 0;
     drop_graph(m);
@@ -413,6 +451,7 @@ int ferrum_hip_model_destroy(FerrumHipModel* m) {
 
 int ferrum_hip_model_set_global_f32(FerrumHipModel* m, int which, const float* data) {
     FH_REQUIRE(m && data, "model_set_global: null argument");
+    FH_REQUIRE(!m->layered, "model_set_global: a layered model takes its weights by name");
     const size_t vh = (size_t)m->cfg.vocab * m->cfg.hidden;
     switch (which) {
     case 0: return upload_f32_as_f16(data, vh, &m->embed);
@@ -424,7 +463,7 @@ int ferrum_hip_model_set_global_f32(FerrumHipModel* m, int which, const float* d
 }
 
 int ferrum_hip_model_set_layer_dense_f32(FerrumHipModel* m, int layer, int which, const float* data) {
-    FH_REQUIRE(m && data && layer >= 0 && layer < m->cfg.num_layers, "model_set_layer_dense: bad argument");
+    FH_REQUIRE(m && data && layer >= 0 && layer < (int)m->layers.size(), "model_set_layer_dense: bad argument");
     LayerWeights& L = m->layers[layer];
     switch (which) {
     case 0: return upload_f32_as_f16(data, m->cfg.hidden, &L.input_ln);
@@ -473,7 +512,7 @@ static int pack_gate_up(FerrumHipModel* m, LayerWeights& L, const int32_t* qweig
 
 int ferrum_hip_model_set_gptq(FerrumHipModel* m, int layer, int which, int expert, const int32_t* qweight,
                               const float* scales, const int32_t* qzeros, const int32_t* g_idx, int k, int n) {
-    FH_REQUIRE(m && qweight && scales && qzeros && layer >= 0 && layer < m->cfg.num_layers, "model_set_gptq: bad argument");
+    FH_REQUIRE(m && qweight && scales && qzeros && layer >= 0 && layer < (int)m->layers.size(), "model_set_gptq: bad argument");
     const FerrumHipModelConfig& c = m->cfg;
     LayerWeights& L = m->layers[layer];
     W4HostPacked hp;
@@ -559,7 +598,7 @@ int ferrum_hip_model_set_gptq(FerrumHipModel* m, int layer, int which, int exper
 // Unquantised projection (DenseLinear, ferrum-kernels/src/linear.rs:109-129): W [n, k] row-major f32 on the host → fp16
 // f16t tiles on the device; the forward then runs it through the fp16 GEMM (B::gemm).  which: 0 qkv, 1 o, 2 gate_up, 3 down.
 int ferrum_hip_model_set_dense_f32(FerrumHipModel* m, int layer, int which, const float* weight, int k, int n) {
-    FH_REQUIRE(m && weight && !m->finalized && layer >= 0 && layer < m->cfg.num_layers, "model_set_dense: bad argument");
+    FH_REQUIRE(m && weight && !m->finalized && layer >= 0 && layer < (int)m->layers.size(), "model_set_dense: bad argument");
     const FerrumHipModelConfig& c = m->cfg;
     LayerWeights& L = m->layers[layer];
     const int H = c.hidden;
@@ -609,6 +648,7 @@ static int synth_w4(W4Device* w, int k, int n, int E, bool fused, uint64_t seed,
 
 int ferrum_hip_model_init_synthetic(FerrumHipModel* m, uint64_t seed) {
     FH_REQUIRE(m && !m->finalized, "model_init_synthetic: bad state");
+    if (m->layered) return m->layered->init_synthetic(seed, m->stream);
     const FerrumHipModelConfig& c = m->cfg;
     hipStream_t s = m->stream;
     auto alloc_fill = [&](__half** p, long n, float v) -> int {
@@ -679,10 +719,44 @@ int ferrum_hip_model_init_synthetic(FerrumHipModel* m, uint64_t seed) {
     return 0;
 }
 
+// index block (pinned host mirror → device), sampled ids, logits: what every model family's forward shares
+static int finalize_batch_buffers(FerrumHipModel* m) {
+    const size_t T = m->cfg.max_tokens, S = m->cfg.max_seqs;
+    size_t off = 0;
+    auto take = [&](size_t bytes) { size_t o = off; off += (bytes + 255) / 256 * 256; return o; };
+    m->il.tokens = take(T * 4);
+    m->il.cu_seqlens = take((S + 1) * 4);
+    m->il.pos_offsets = take(S * 4);
+    m->il.kv_lens = take(S * 4);
+    m->il.sampled_idx = take(S * 4);
+    m->il.tok_seq = take(m->layered ? T * 4 : 0);
+    m->il.prev_tokens = take(m->layered ? S * 4 : 0);
+    m->il.state_slots = take(m->layered ? S * 4 : 0);
+    m->il.scan_units = take(m->layered ? (T / RGLRU_CHUNK + S) * 8 : 0);
+    m->il.block_tables = take(S * m->max_blocks_per_seq * 4);
+    m->il.total = off;
+    FH_CHECK_HIP(hipHostMalloc((void**)&m->idx_host, off, hipHostMallocDefault));
+    FH_CHECK_HIP(hipMalloc((void**)&m->idx_dev, off));
+    FH_CHECK_HIP(hipMemset(m->idx_dev, 0, off));
+    if (int r = dev_alloc(&m->step_counter, (size_t)4)) return r;
+    return 0;
+}
+
 int ferrum_hip_model_finalize(FerrumHipModel* m) {
     FH_REQUIRE(m, "model_finalize: null");
     if (m->finalized) return 0;
     const FerrumHipModelConfig& c = m->cfg;
+    if (m->layered) {
+        if (int r = m->layered->finalize(m->stream)) return r;
+        const size_t S = c.max_seqs;
+        if (int r = dev_alloc(&m->logits, S * (size_t)c.vocab)) return r;
+        if (int r = dev_alloc(&m->out_tokens, S)) return r;
+        m->workspace_bytes = std::max<size_t>(S * 1024 * 2, 1 << 20);        // two-stage argmax
+        FH_CHECK_HIP(hipMalloc((void**)&m->workspace, m->workspace_bytes));
+        if (int r = finalize_batch_buffers(m)) return r;
+        m->finalized = true;
+        return 0;
+    }
     FH_REQUIRE(m->embed && m->final_norm, "model_finalize: embed / final_norm missing");
     for (LayerWeights& L : m->layers)
         if (L.pending_gate_up) {      // down never arrived as GPTQ (unquantised, or missing: reported below): nothing to fold
@@ -820,20 +894,7 @@ int ferrum_hip_model_finalize(FerrumHipModel* m) {
     size_t attn_ws = (size_t)32 * S * c.num_kv_heads * 16 * (c.head_dim + 2) * sizeof(float) * 2;
     m->workspace_bytes = std::max(gemm_ws, attn_ws);
     FH_CHECK_HIP(hipMalloc((void**)&m->workspace, m->workspace_bytes));
-    // index block
-    size_t off = 0;
-    auto take = [&](size_t bytes) { size_t o = off; off += (bytes + 255) / 256 * 256; return o; };
-    m->il.tokens = take(T * 4);
-    m->il.cu_seqlens = take((S + 1) * 4);
-    m->il.pos_offsets = take(S * 4);
-    m->il.kv_lens = take(S * 4);
-    m->il.sampled_idx = take(S * 4);
-    m->il.block_tables = take(S * m->max_blocks_per_seq * 4);
-    m->il.total = off;
-    FH_CHECK_HIP(hipHostMalloc((void**)&m->idx_host, off, hipHostMallocDefault));
-    FH_CHECK_HIP(hipMalloc((void**)&m->idx_dev, off));
-    FH_CHECK_HIP(hipMemset(m->idx_dev, 0, off));
-    if (int r = dev_alloc(&m->step_counter, (size_t)4)) return r;
+    if (int r = finalize_batch_buffers(m)) return r;
     m->finalized = true;
     return 0;
 }
@@ -850,6 +911,7 @@ int ferrum_hip_model_kv_capacity_snapshot(const FerrumHipModel* m, FerrumHipKvSl
 static int reserve(FerrumHipModel* m, const FerrumHipKvSlotRequest* reqs, int n, FerrumHipKvSlotReservation* out) {
     const int before = (int)m->alloc->free_count();
     long need = 0;
+    int need_slots = 0;
     for (int i = 0; i < n; i++) {
         int blocks = cdiv(reqs[i].target_len, KV_BLOCK);
         if (blocks > m->max_blocks_per_seq) {
@@ -859,6 +921,11 @@ static int reserve(FerrumHipModel* m, const FerrumHipKvSlotRequest* reqs, int n,
         auto it = m->seqs.find(reqs[i].seq_id);
         int have = it == m->seqs.end() ? 0 : (int)it->second.blocks.size();
         if (blocks > have) need += blocks - have;
+        if (m->state_slots > 0 && (it == m->seqs.end() || it->second.state_slot < 0)) need_slots++;
+    }
+    if (need_slots > (int)m->free_slots.size()) {
+        fh::set_error("recurrent state slots exhausted: need %d but only %d of %d free", need_slots, (int)m->free_slots.size(), m->state_slots);
+        return FERRUM_HIP_INVALID;
     }
     if (need > before) {
         fh::set_error("paged KV pool exhausted: need %ld blocks but only %d free", need, before);
@@ -866,6 +933,10 @@ static int reserve(FerrumHipModel* m, const FerrumHipKvSlotRequest* reqs, int n,
     }
     for (int i = 0; i < n; i++) {
         SeqState& st = m->seqs[reqs[i].seq_id];
+        if (m->state_slots > 0 && st.state_slot < 0) {       // never cleared: a sequence's first token starts from zero state
+            st.state_slot = m->free_slots.back();
+            m->free_slots.pop_back();
+        }
         int blocks = cdiv(reqs[i].target_len, KV_BLOCK);
         while ((int)st.blocks.size() < blocks) {
             uint32_t b;
@@ -893,6 +964,7 @@ int ferrum_hip_model_release(FerrumHipModel* m, uint64_t seq_id) {
     auto it = m->seqs.find(seq_id);
     if (it == m->seqs.end()) return 0;
     m->alloc->free(it->second.blocks.data(), (uint32_t)it->second.blocks.size());
+    if (it->second.state_slot >= 0) m->free_slots.push_back(it->second.state_slot);
     m->seqs.erase(it);
     return 0;
 }
@@ -916,6 +988,10 @@ int ferrum_hip_model_prefix_cache_acquire(FerrumHipModel* m, uint64_t seq_id, co
     FH_REQUIRE(it != m->seqs.end(), "prefix_cache_acquire: reserve KV slots for sequence %llu first", (unsigned long long)seq_id);
     SeqState& st = it->second;
     FH_REQUIRE(st.len == 0, "prefix_cache_acquire: sequence %llu already holds %d tokens", (unsigned long long)seq_id, st.len);
+    if (m->state_slots > 0) {          // recurrent state is not kept per block: nothing to splice in
+        m->prefix_misses++;
+        return 0;
+    }
     const std::vector<uint64_t> hashes = fh::block_hash_chain(tokens, n, KV_BLOCK);
     // longest contiguous prefix: stop at the first miss
     std::vector<uint32_t> matched;
@@ -937,6 +1013,7 @@ int ferrum_hip_model_prefix_cache_acquire(FerrumHipModel* m, uint64_t seq_id, co
     // the suffix then rewrites the shared block with identical content
     if (cached >= n) cached = std::min(std::max(cached - KV_BLOCK, 0), n - 1);
     st.len = cached;
+    st.last_token = cached > 0 ? (int64_t)tokens[cached - 1] : -1;
     if (cached > 0) { m->prefix_hits++; m->prefix_saved_tokens += (uint64_t)cached; } else { m->prefix_misses++; }
     *cached_tokens = cached;
     return 0;
@@ -980,7 +1057,7 @@ int ferrum_hip_model_block_table(const FerrumHipModel* m, uint64_t seq_id, uint3
 }
 
 int ferrum_hip_model_read_kv_f32(FerrumHipModel* m, uint64_t seq_id, int layer, int is_v, float* out_host) {
-    FH_REQUIRE(m && m->finalized && out_host && layer >= 0 && layer < m->cfg.num_layers, "model_read_kv: bad argument");
+    FH_REQUIRE(m && m->finalized && out_host && layer >= 0 && layer < (int)m->layers.size(), "model_read_kv: bad argument");
     auto it = m->seqs.find(seq_id);
     FH_REQUIRE(it != m->seqs.end(), "model_read_kv: unknown sequence");
     const SeqState& st = it->second;
@@ -1222,18 +1299,24 @@ struct GreedyDeviceOpts {          // device pointers, already uploaded on m->st
     const uint8_t* mask = nullptr; int mask_len = 0;
     const uint32_t* row_offsets = nullptr; const uint32_t* token_ids = nullptr; const float* penalties = nullptr;
 };
-int enqueue_forward(FerrumHipModel* m, const StepShape& sh, bool greedy, const GreedyDeviceOpts* gopts = nullptr,
-                    const DecodeAdvance* advance = nullptr, int* advance_fused = nullptr) {
-    if (advance_fused) *advance_fused = 0;
+int enqueue_body(FerrumHipModel* m, const StepShape& sh) {
     const FerrumHipModelConfig& c = m->cfg;
     hipStream_t s = m->stream;
+    if (m->layered) {
+        BatchView v;
+        v.T = sh.m_total; v.num_seqs = sh.num_seqs; v.max_blocks = m->max_blocks_per_seq; v.max_keys = sh.max_kv_len; v.single = sh.all_single_token;
+        v.tokens = idx<uint32_t>(m, m->il.tokens); v.cu = idx<uint32_t>(m, m->il.cu_seqlens); v.pos = idx<uint32_t>(m, m->il.pos_offsets);
+        v.bt = idx<int32_t>(m, m->il.block_tables); v.tok_seq = idx<int32_t>(m, m->il.tok_seq); v.prev = idx<int32_t>(m, m->il.prev_tokens);
+        v.slots = idx<int32_t>(m, m->il.state_slots); v.units = idx<int32_t>(m, m->il.scan_units); v.num_units = m->batch_units;
+        m->taps_tokens = v.T;
+        return m->layered->forward(v, m->taps_enabled ? m->taps : nullptr, knobs().trace_launches, s);
+    }
     const int T = sh.m_total, H = c.hidden, nq = c.num_heads, nkv = c.num_kv_heads, hd = c.head_dim;
     const int qk_mode = c.has_qk_norm ? 1 : 2;
     const uint32_t* tokens = idx<uint32_t>(m, m->il.tokens);
     const uint32_t* cu = idx<uint32_t>(m, m->il.cu_seqlens);
     const uint32_t* pos = idx<uint32_t>(m, m->il.pos_offsets);
     const uint32_t* kvl = idx<uint32_t>(m, m->il.kv_lens);
-    const int32_t* sampled_idx = idx<int32_t>(m, m->il.sampled_idx);
     const int32_t* bt = idx<int32_t>(m, m->il.block_tables);
     int rc;
     // FERRUM_HIP_TRACE_LAUNCHES=1 (with FERRUM_HIP_NO_GRAPH=1: a stream cannot be synchronised inside a capture): every step of
@@ -1687,17 +1770,43 @@ int enqueue_forward(FerrumHipModel* m, const StepShape& sh, bool greedy, const G
         }
     }
     m->taps_tokens = T;
+#undef RUN
+    return 0;
+}
+
+// final norm + lm_head on the rows listed in the index block (same rows the reference packs, qwen3_moe_forward_unified.rs:365-392)
+int enqueue_head(FerrumHipModel* m, int rows) {
+    const FerrumHipModelConfig& c = m->cfg;
+    hipStream_t s = m->stream;
+    const int32_t* sampled_idx = idx<int32_t>(m, m->il.sampled_idx);
+    if (knobs().trace_launches) fprintf(stderr, "[ferrum_hip] head rows=%d\n", rows);
+    if (m->layered) return m->layered->head(sampled_idx, rows, m->logits, s);
+    if (c.sandwich_norms) {
+        if (int rc = rms_norm_f32_to_f16(m->residual_f32, sampled_idx, m->final_norm, c.rms_eps, m->sampled_hidden, rows, c.hidden, s)) return rc;
+    } else {
+        if (int rc = gather_rms_norm_f16(m->residual, sampled_idx, m->final_norm, c.rms_eps, m->sampled_hidden, rows, c.hidden, s)) return rc;
+    }
+    // this rank's vocabulary rows (all of them unless vocabulary parallel)
+    return f16t_gemm_f32out(m->sampled_hidden, m->lm_head_t, m->logits, rows, m->vp_n, c.hidden, m->workspace, m->workspace_bytes, s);
+}
+
+int enqueue_forward(FerrumHipModel* m, const StepShape& sh, bool greedy, const GreedyDeviceOpts* gopts = nullptr,
+                    const DecodeAdvance* advance = nullptr, int* advance_fused = nullptr) {
+    if (advance_fused) *advance_fused = 0;
+    const FerrumHipModelConfig& c = m->cfg;
+    hipStream_t s = m->stream;
+    if (int rc = enqueue_body(m, sh)) return rc;
     if (sh.num_sampled > 0) {
-        // final norm + lm_head on the sampled rows only (same rows the reference packs,
-        // qwen3_moe_forward_unified.rs:365-392)
-        if (sandwich) {
-            RUN(rms_norm_f32_to_f16(m->residual_f32, sampled_idx, m->final_norm, c.rms_eps, m->sampled_hidden, sh.num_sampled, H, s));
-        } else {
-            RUN(gather_rms_norm_f16(m->residual, sampled_idx, m->final_norm, c.rms_eps, m->sampled_hidden, sh.num_sampled, H, s));
-        }
-        const int Vn = m->vp_n, v0 = m->vp_v0;                  // this rank's vocabulary rows (all of them unless vocabulary parallel)
-        RUN(f16t_gemm_f32out(m->sampled_hidden, m->lm_head_t, m->logits, sh.num_sampled, Vn, H, m->workspace,
-                             m->workspace_bytes, s));
+        if (int rc = enqueue_head(m, sh.num_sampled)) return rc;
+        int rc;
+        const bool trace = knobs().trace_launches;
+#define RUN(x)                                                                       \
+    do {                                                                             \
+        if (trace) fprintf(stderr, "[ferrum_hip] sampling %.70s\n", #x);             \
+        if ((rc = (x))) return rc;                                                   \
+        if (trace) FH_CHECK_HIP(hipStreamSynchronize(s));                            \
+    } while (0)
+        const int Vn = m->vp_n, v0 = m->vp_v0;
         if (greedy && !c.vocab_parallel) {
             // LogitsReturnPolicy::GreedyArgmax { token_mask, repetition_penalty } (model_executor.rs:109-150): the sparse
             // penalty rewrites the listed logits in place, then raw or masked argmax (traits.rs:1571-1591)
@@ -1728,6 +1837,16 @@ int enqueue_forward(FerrumHipModel* m, const StepShape& sh, bool greedy, const G
 
 }  // namespace
 
+// what a layered model's kernels need to know about item i of a batch: tokens [t0, t0 + n)
+static void put_layered_item(FerrumHipModel* m, int i, int t0, int n, const SeqState& st) {
+    int32_t* seq = reinterpret_cast<int32_t*>(m->idx_host + m->il.tok_seq);
+    std::fill(seq + t0, seq + t0 + n, i);
+    reinterpret_cast<int32_t*>(m->idx_host + m->il.prev_tokens)[i] = (int32_t)st.last_token;
+    reinterpret_cast<int32_t*>(m->idx_host + m->il.state_slots)[i] = std::max(st.state_slot, 0);
+    int32_t* units = reinterpret_cast<int32_t*>(m->idx_host + m->il.scan_units);
+    for (int c = 0; c < n; c += RGLRU_CHUNK) { units[2 * m->batch_units] = i; units[2 * m->batch_units + 1] = t0 + c; m->batch_units++; }
+}
+
 extern "C" {
 
 int ferrum_hip_model_local_vocab(const FerrumHipModel* m, int* vocab_start, int* vocab_count) {
@@ -1742,8 +1861,9 @@ int ferrum_hip_model_unified_forward(FerrumHipModel* m, const FerrumHipBatchItem
     return ferrum_hip_model_unified_forward_ex(m, items, num_items, greedy, nullptr, out_tokens, logits_out);
 }
 
-int ferrum_hip_model_unified_forward_ex(FerrumHipModel* m, const FerrumHipBatchItem* items, int num_items, int greedy,
-                                        const FerrumHipGreedyOptions* opts, uint32_t* out_tokens, float* logits_out) {
+// `rows` null: the sampled rows are the last tokens of the final chunks; else the listed places of the batch, logits only.
+static int forward_batch(FerrumHipModel* m, const FerrumHipBatchItem* items, int num_items, int greedy, const FerrumHipGreedyOptions* opts,
+                         uint32_t* out_tokens, float* logits_out, const int32_t* rows, int num_rows) {
     FH_REQUIRE(m && m->finalized, "unified_forward: model not finalized");
     if (num_items <= 0) return 0;
     FH_REQUIRE(items, "unified_forward: null items");
@@ -1767,10 +1887,12 @@ int ferrum_hip_model_unified_forward_ex(FerrumHipModel* m, const FerrumHipBatchI
         sh.max_q_len = std::max(sh.max_q_len, it.num_q_tokens);
         sh.max_kv_len = std::max(sh.max_kv_len, it.pos_offset + it.num_q_tokens);
         if (it.num_q_tokens != 1) sh.pure_decode = false;
-        if (it.is_final_chunk) sh.num_sampled++;
+        if (it.is_final_chunk && !rows) sh.num_sampled++;
+        for (int q = 0; q < i; q++) FH_REQUIRE(items[q].seq_id != it.seq_id, "unified_forward: sequence %llu twice in one batch", (unsigned long long)it.seq_id);
         reqs[i] = {it.seq_id, it.pos_offset + it.num_q_tokens, 0};
     }
     FH_REQUIRE(sh.m_total <= c.max_tokens, "unified_forward: %d tokens > max_tokens %d", sh.m_total, c.max_tokens);
+    for (int r = 0; rows && r < num_rows; r++) FH_REQUIRE(rows[r] >= 0 && rows[r] < sh.m_total, "unified_forward: row %d of a batch of %d tokens", rows[r], sh.m_total);
     sh.all_single_token = sh.pure_decode;
     if (c.sliding_window > 0 && c.sliding_window_pattern == 0) sh.pure_decode = false;   // uniform window: no full-attention layer
     if (int rc = reserve(m, reqs.data(), num_items, nullptr)) return rc;
@@ -1782,6 +1904,7 @@ int ferrum_hip_model_unified_forward_ex(FerrumHipModel* m, const FerrumHipBatchI
     uint32_t* h_kvl = reinterpret_cast<uint32_t*>(m->idx_host + m->il.kv_lens);
     int32_t* h_samp = reinterpret_cast<int32_t*>(m->idx_host + m->il.sampled_idx);
     int32_t* h_bt = reinterpret_cast<int32_t*>(m->idx_host + m->il.block_tables);
+    m->batch_units = 0;
     int t = 0, j = 0;
     for (int i = 0; i < num_items; i++) {
         const FerrumHipBatchItem& it = items[i];
@@ -1790,8 +1913,9 @@ int ferrum_hip_model_unified_forward_ex(FerrumHipModel* m, const FerrumHipBatchI
         t += it.num_q_tokens;
         h_pos[i] = (uint32_t)it.pos_offset;
         h_kvl[i] = (uint32_t)(it.pos_offset + it.num_q_tokens);
-        if (it.is_final_chunk) h_samp[j++] = t - 1;
+        if (it.is_final_chunk && !rows) h_samp[j++] = t - 1;
         const SeqState& st = m->seqs[it.seq_id];
+        if (m->layered) put_layered_item(m, i, t - it.num_q_tokens, it.num_q_tokens, st);
         int32_t* row = h_bt + (size_t)i * m->max_blocks_per_seq;
         for (int b = 0; b < m->max_blocks_per_seq; b++) row[b] = b < (int)st.blocks.size() ? (int32_t)st.blocks[b] : 0;   // padded with 0 (paged_pool.rs:438-440)
     }
@@ -1842,6 +1966,15 @@ int ferrum_hip_model_unified_forward_ex(FerrumHipModel* m, const FerrumHipBatchI
         }
     }
     if (int rc = enqueue_forward(m, sh, greedy != 0, &g)) return rc;
+    // listed places: as many rows per head launch as the logits buffer holds
+    for (int r0 = 0; rows && r0 < num_rows; r0 += c.max_seqs) {
+        const int n = std::min(c.max_seqs, num_rows - r0);
+        if (r0) FH_CHECK_HIP(hipStreamSynchronize(m->stream));          // (the staging half of the index block is in use until then)
+        memcpy(h_samp, rows + r0, (size_t)n * 4);
+        FH_CHECK_HIP(hipMemcpyAsync(m->idx_dev + m->il.sampled_idx, h_samp, (size_t)n * 4, hipMemcpyHostToDevice, m->stream));
+        if (int rc = enqueue_head(m, n)) return rc;
+        FH_CHECK_HIP(hipMemcpyAsync(logits_out + (size_t)r0 * m->vp_n, m->logits, (size_t)n * m->vp_n * 4, hipMemcpyDeviceToHost, m->stream));
+    }
     if (sh.num_sampled > 0) {
         if (greedy && out_tokens)
             FH_CHECK_HIP(hipMemcpyAsync(out_tokens, m->out_tokens, (size_t)sh.num_sampled * 4, hipMemcpyDeviceToHost, m->stream));
@@ -1849,8 +1982,24 @@ int ferrum_hip_model_unified_forward_ex(FerrumHipModel* m, const FerrumHipBatchI
             FH_CHECK_HIP(hipMemcpyAsync(logits_out, m->logits, (size_t)sh.num_sampled * m->vp_n * 4, hipMemcpyDeviceToHost, m->stream));
     }
     FH_CHECK_HIP(hipStreamSynchronize(m->stream));
-    for (int i = 0; i < num_items; i++) m->seqs[items[i].seq_id].len += items[i].num_q_tokens;
+    for (int i = 0; i < num_items; i++) {
+        SeqState& st = m->seqs[items[i].seq_id];
+        st.len += items[i].num_q_tokens;
+        st.last_token = items[i].q_tokens[items[i].num_q_tokens - 1];
+    }
     return check_inlaunch_waits(m);
+}
+
+int ferrum_hip_model_unified_forward_ex(FerrumHipModel* m, const FerrumHipBatchItem* items, int num_items, int greedy,
+                                        const FerrumHipGreedyOptions* opts, uint32_t* out_tokens, float* logits_out) {
+    return forward_batch(m, items, num_items, greedy, opts, out_tokens, logits_out, nullptr, 0);
+}
+
+int ferrum_hip_model_unified_forward_rows(FerrumHipModel* m, const FerrumHipBatchItem* items, int num_items, const int32_t* rows,
+                                          int num_rows, float* logits_out) {
+    FH_REQUIRE(num_rows >= 0 && (num_rows == 0 || (rows && logits_out)), "unified_forward_rows: bad argument");
+    const int32_t none = 0;
+    return forward_batch(m, items, num_items, 0, nullptr, nullptr, logits_out, rows ? rows : &none, num_rows);
 }
 
 int ferrum_hip_model_decode_steps(FerrumHipModel* m, const uint64_t* seq_ids, const uint32_t* first_tokens, int n,
@@ -1895,6 +2044,7 @@ int ferrum_hip_model_decode_steps(FerrumHipModel* m, const uint64_t* seq_ids, co
     uint32_t* h_kvl = reinterpret_cast<uint32_t*>(m->idx_host + m->il.kv_lens);
     int32_t* h_samp = reinterpret_cast<int32_t*>(m->idx_host + m->il.sampled_idx);
     int32_t* h_bt = reinterpret_cast<int32_t*>(m->idx_host + m->il.block_tables);
+    m->batch_units = 0;
     for (int i = 0; i < n; i++) {
         const SeqState& st = m->seqs[seq_ids[i]];
         h_tok[i] = first_tokens[i];
@@ -1902,6 +2052,7 @@ int ferrum_hip_model_decode_steps(FerrumHipModel* m, const uint64_t* seq_ids, co
         h_pos[i] = (uint32_t)st.len;
         h_kvl[i] = (uint32_t)st.len + 1;
         h_samp[i] = i;
+        if (m->layered) put_layered_item(m, i, i, 1, st);
         int32_t* row = h_bt + (size_t)i * m->max_blocks_per_seq;
         for (int b = 0; b < m->max_blocks_per_seq; b++) row[b] = b < (int)st.blocks.size() ? (int32_t)st.blocks[b] : 0;
     }
@@ -1916,11 +2067,12 @@ int ferrum_hip_model_decode_steps(FerrumHipModel* m, const uint64_t* seq_ids, co
         adv.tokens = idx<uint32_t>(m, m->il.tokens); adv.pos_offsets = idx<uint32_t>(m, m->il.pos_offsets);
         adv.kv_lens = idx<uint32_t>(m, m->il.kv_lens); adv.history = m->history; adv.step_counter = m->step_counter;
         adv.ticket = reinterpret_cast<unsigned*>(m->step_counter + 1); adv.n = n;
+        adv.prev_tokens = m->layered ? idx<int32_t>(m, m->il.prev_tokens) : nullptr;
         int fused = 0;
         if (int rc = enqueue_forward(m, sh, true, nullptr, &adv, &fused)) return rc;
         if (!fused) {                                            // narrow vocabularies take the single-kernel argmax
             hipLaunchKernelGGL(decode_advance_kernel, dim3(1), dim3(1024), 0, m->stream, m->out_tokens, adv.tokens, adv.pos_offsets,
-                               adv.kv_lens, m->history, m->step_counter, n);
+                               adv.kv_lens, m->history, m->step_counter, n, adv.prev_tokens);
             FH_CHECK_LAUNCH();
         }
         return 0;
@@ -1970,8 +2122,14 @@ int ferrum_hip_model_decode_steps(FerrumHipModel* m, const uint64_t* seq_ids, co
     }
     if (out_tokens)
         FH_CHECK_HIP(hipMemcpyAsync(out_tokens, m->history, (size_t)steps * n * 4, hipMemcpyDeviceToHost, m->stream));
+    // the last token each sequence was FED: the one sampled a step before the last
+    std::vector<uint32_t> fed(first_tokens, first_tokens + n);
+    if (steps > 1) FH_CHECK_HIP(hipMemcpyAsync(fed.data(), m->history + (size_t)(steps - 2) * n, (size_t)n * 4, hipMemcpyDeviceToHost, m->stream));
     FH_CHECK_HIP(hipStreamSynchronize(m->stream));
-    for (int i = 0; i < n; i++) m->seqs[seq_ids[i]].len += steps;
+    for (int i = 0; i < n; i++) {
+        m->seqs[seq_ids[i]].len += steps;
+        m->seqs[seq_ids[i]].last_token = fed[i];
+    }
     return check_inlaunch_waits(m);
 }
 
@@ -1984,6 +2142,7 @@ int ferrum_hip_model_decode_steps(FerrumHipModel* m, const uint64_t* seq_ids, co
 int ferrum_hip_model_time_kernel(FerrumHipModel* m, int which, int n_seqs, int max_kv_len, int reps, float* avg_us,
                                  int* moe_blocks) {
     FH_REQUIRE(m && m->finalized && avg_us && reps > 0, "time_kernel: bad argument");
+    if (m->layered) { fh::set_error("time_kernel: layered models are timed from a profile"); return FERRUM_HIP_UNSUPPORTED; }
     const FerrumHipModelConfig& c = m->cfg;
     hipStream_t s = m->stream;
     const int T = n_seqs, H = c.hidden;

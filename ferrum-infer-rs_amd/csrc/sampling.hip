@@ -139,6 +139,7 @@ __global__ __launch_bounds__(64) void argmax_final_kernel(const float* __restric
         const uint32_t id = best_idx == 0x7fffffff ? 0u : (uint32_t)best_idx;
         out[row] = id;
         if (adv.tokens && row < adv.n) {
+            if (adv.prev_tokens) adv.prev_tokens[row] = (int32_t)adv.tokens[row];
             adv.tokens[row] = id;
             adv.pos_offsets[row] += 1;
             adv.kv_lens[row] += 1;
@@ -241,6 +242,7 @@ __global__ void argmax_merge_ranks_kernel(const float2* __restrict__ gathered, u
         if (best_id == 0xffffffffu) best_id = 0;           // no valid id on any rank
         out[r] = best_id;
         if (adv.tokens && r < adv.n) {
+            if (adv.prev_tokens) adv.prev_tokens[r] = (int32_t)adv.tokens[r];
             adv.tokens[r] = best_id;
             adv.pos_offsets[r] += 1;
             adv.kv_lens[r] += 1;

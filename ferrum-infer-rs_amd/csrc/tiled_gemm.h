@@ -1,0 +1,68 @@
+// Dense projections over weights stored as MFMA-fragment tiles, for 16-bit and 32-bit models.
+//
+// Tile layout (the one f16t uses): [groups][n / 16][k / 32][64 lanes][8]; lane (a, b) of a k-step holds W[16·tile + b][32·step + 8a .. +8],
+// so a wave load of a fragment is contiguous and IS the B operand.  The 32-bit form keeps the same 8 values per lane and feeds them
+// to eight v_mfma_f32_16x16x4_f32: both operands permute the contraction index the same way, so no re-layout is needed.
+// n and k are padded to multiples of 32 with zero rows / columns, activations have padded leading dimensions: no kernel masks K.
+#pragma once
+#include <hip/hip_runtime.h>
+#include <stdint.h>
+
+namespace fh {
+
+typedef __bf16 bf16;
+typedef bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef bf16 bf16x4 __attribute__((ext_vector_type(4)));
+typedef float floatx8 __attribute__((ext_vector_type(8)));
+typedef float floatx4 __attribute__((ext_vector_type(4)));
+typedef short shortx4 __attribute__((ext_vector_type(4)));
+
+template <typename E> struct Frag;
+template <> struct Frag<bf16> {
+    typedef bf16x8 v8;
+    static __device__ __forceinline__ floatx4 mma(v8 a, v8 b, floatx4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
+};
+template <> struct Frag<float> {
+    typedef floatx8 v8;
+    static __device__ __forceinline__ floatx4 mma(v8 a, v8 b, floatx4 c) {
+#pragma unroll
+        for (int j = 0; j < 8; j++) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[j], b[j], c, 0, 0, 0);
+        return c;
+    }
+};
+
+static inline int pad32(int n) { return (n + 31) / 32 * 32; }
+
+enum GemmAct : int { GEMM_ACT_NONE = 0, GEMM_ACT_SIGMOID = 1, GEMM_ACT_GELU_TANH = 2, GEMM_ACT_XIELU = 3 };
+constexpr int GEMM_MAX_SECTIONS = 6;
+struct GemmSection {          // columns [begin, next section's begin) of a fused projection; begin is a multiple of 32
+    int begin, act;
+    float p, q;               // xIELU: softplus of its two parameters
+};
+
+// out[r][g·out_group + c] = act(x[r][g·x_group ..] · W_gᵀ + bias) · row_scale[r][g]
+template <typename E>
+struct TiledGemm {
+    const E* x = nullptr; long ldx = 0, x_group = 0;
+    const E* w = nullptr;
+    const float* bias = nullptr;          // [groups·n]
+    int m = 0, n = 0, k = 0, groups = 1;
+    int n_store = 0;                      // columns written (0: all n)
+    E* out = nullptr; float* out_f32 = nullptr;      // one of the two
+    long ldo = 0, out_group = 0;
+    const E* row_scale = nullptr; long ld_scale = 0;
+    int nsec = 0;
+    GemmSection sec[GEMM_MAX_SECTIONS] = {};
+};
+template <typename E> int tiled_gemm(const TiledGemm<E>& g, hipStream_t s);
+
+__device__ __forceinline__ float sigmoid_f32(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float gelu_tanh_f32(float z) {
+    return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+}
+// quadratic right of zero, exponential left of it, slope 1/2 at zero; sp / sq: softplus of the two trained numbers
+__device__ __forceinline__ float xielu_f32(float z, float sp, float sq) {
+    return z > 0.f ? sp * z * z + 0.5f * z : (0.5f + sq) * (expm1f(z) - z) + 0.5f * z;
+}
+
+}  // namespace fh

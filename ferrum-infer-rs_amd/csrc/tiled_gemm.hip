@@ -1,0 +1,223 @@
+// Dense projections of the layered models (tiled_gemm.h): one kernel for few rows (K split over the waves of a workgroup, summed in
+// LDS, no second launch) and one for prompts (128 × 128 tiles, both operands copied to LDS as fragments by the load unit itself).
+// Every activation, bias and per-row factor of a projection is applied to the fp32 accumulator in the epilogue.
+#include "common.h"
+#include "knobs.h"
+#include "tiled_gemm.h"
+
+namespace fh {
+
+template <typename E>
+__device__ __forceinline__ void gemm_epilogue(const TiledGemm<E>& p, const GemmSection& sec, int g, int row, int col, float v) {
+    if (row >= p.m || col >= p.n_store) return;
+    if (p.bias) v += p.bias[(long)g * p.n + col];
+    if (sec.act == GEMM_ACT_SIGMOID) v = sigmoid_f32(v);
+    else if (sec.act == GEMM_ACT_GELU_TANH) v = gelu_tanh_f32(v);
+    else if (sec.act == GEMM_ACT_XIELU) v = xielu_f32(v, sec.p, sec.q);
+    if (p.row_scale) v *= (float)p.row_scale[row * p.ld_scale + g];
+    const long o = row * p.ldo + g * p.out_group + col;
+    if (p.out_f32) p.out_f32[o] = v; else p.out[o] = (E)v;
+}
+template <typename E>
+__device__ __forceinline__ GemmSection gemm_section(const TiledGemm<E>& p, int col) {
+    GemmSection s = {0, GEMM_ACT_NONE, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < GEMM_MAX_SECTIONS; i++)
+        if (i < p.nsec && col >= p.sec[i].begin) s = p.sec[i];
+    return s;
+}
+
+// grid (column blocks, row blocks, groups); NW waves = (NW / kw) column groups × kw parts of K.
+template <typename E, int MT, int J>
+__global__ __launch_bounds__(512) void tiled_gemm_kernel(TiledGemm<E> p, int kw) {
+    typedef typename Frag<E>::v8 v8;
+    extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
+    floatx4* red = reinterpret_cast<floatx4*>(smem);            // [NW][MT·J][64]
+    const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
+    const int a = lane >> 4, b = lane & 15;
+    const int cw = (blockDim.x >> 6) / kw, part = wave % kw, cg = wave / kw;
+    const int n0 = (blockIdx.x * cw + cg) * 16 * J, rb = blockIdx.y, g = blockIdx.z;
+    const int ksteps = p.k >> 5;
+    const bool live = n0 < p.n;
+    const int s0 = live ? ksteps * part / kw : 0, s1 = live ? ksteps * (part + 1) / kw : 0;
+    const E* xrow[MT];
+#pragma unroll
+    for (int mt = 0; mt < MT; mt++) {
+        const int r = (rb * MT + mt) * 16 + b;
+        xrow[mt] = p.x + (long)(r < p.m ? r : p.m - 1) * p.ldx + g * p.x_group + 8 * a;
+    }
+    const E* wt = p.w + ((long)g * (p.n >> 4) + (live ? n0 >> 4 : 0)) * ksteps * 512 + lane * 8;
+    floatx4 acc[MT][J];
+#pragma unroll
+    for (int mt = 0; mt < MT; mt++)
+#pragma unroll
+        for (int j = 0; j < J; j++) acc[mt][j] = (floatx4){0.f, 0.f, 0.f, 0.f};
+    constexpr int U = sizeof(E) == 2 ? 4 : 1;
+    int s = s0;
+    for (; s + U <= s1; s += U) {
+        v8 bw[U][J], ax[U][MT];
+#pragma unroll
+        for (int u = 0; u < U; u++) {
+#pragma unroll
+            for (int j = 0; j < J; j++) bw[u][j] = *reinterpret_cast<const v8*>(wt + ((long)j * ksteps + s + u) * 512);
+#pragma unroll
+            for (int mt = 0; mt < MT; mt++) ax[u][mt] = *reinterpret_cast<const v8*>(xrow[mt] + (s + u) * 32);
+        }
+#pragma unroll
+        for (int u = 0; u < U; u++)
+#pragma unroll
+            for (int j = 0; j < J; j++)
+#pragma unroll
+                for (int mt = 0; mt < MT; mt++) acc[mt][j] = Frag<E>::mma(ax[u][mt], bw[u][j], acc[mt][j]);
+    }
+    for (; s < s1; s++) {
+#pragma unroll
+        for (int j = 0; j < J; j++) {
+            const v8 bw = *reinterpret_cast<const v8*>(wt + ((long)j * ksteps + s) * 512);
+#pragma unroll
+            for (int mt = 0; mt < MT; mt++) acc[mt][j] = Frag<E>::mma(*reinterpret_cast<const v8*>(xrow[mt] + s * 32), bw, acc[mt][j]);
+        }
+    }
+    const GemmSection sec = gemm_section(p, n0);
+    if (kw == 1) {
+        if (!live) return;
+#pragma unroll
+        for (int mt = 0; mt < MT; mt++)
+#pragma unroll
+            for (int j = 0; j < J; j++)
+#pragma unroll
+                for (int r = 0; r < 4; r++) gemm_epilogue(p, sec, g, (rb * MT + mt) * 16 + 4 * a + r, n0 + 16 * j + b, acc[mt][j][r]);
+        return;
+    }
+#pragma unroll
+    for (int mt = 0; mt < MT; mt++)
+#pragma unroll
+        for (int j = 0; j < J; j++) red[(wave * MT * J + mt * J + j) * 64 + lane] = acc[mt][j];
+    __syncthreads();
+    if (!live) return;
+    // tile t of the column group is summed (in the order of the K parts) and finished by part t mod kw
+    for (int t = part; t < MT * J; t += kw) {
+        floatx4 v = red[(cg * kw * MT * J + t) * 64 + lane];
+        for (int q = 1; q < kw; q++) v += red[((cg * kw + q) * MT * J + t) * 64 + lane];
+        const int mt = t / J, j = t % J;
+#pragma unroll
+        for (int r = 0; r < 4; r++) gemm_epilogue(p, sec, g, (rb * MT + mt) * 16 + 4 * a + r, n0 + 16 * j + b, v[r]);
+    }
+}
+
+// Prompts, 16-bit: 128 × 128 output tile, 64 of K per stage, two stages.  A fragment (16 rows × 32 of K, or 16 columns × 32 of K) is
+// one 1-KiB load straight into LDS in lane order, read back as one conflict-free ds_read_b128; 2 × 2 waves hold 64 × 64 each.
+__global__ __launch_bounds__(256, 2) void tiled_gemm_big_kernel(TiledGemm<bf16> p, int mtiles, int ntiles) {
+    __shared__ __attribute__((aligned(16))) bf16 lds[2][32 * 512];      // per stage: 16 A fragments, 16 B fragments
+    const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
+    const int a = lane >> 4, b = lane & 15, g = blockIdx.z;
+    // workgroups go round-robin over 8 XCDs: give each XCD a contiguous run of tiles, and walk 8 row tiles per column tile
+    const int total = mtiles * ntiles, l = blockIdx.x;
+    const int q8 = total / 8, r8 = total % 8, xcd = l % 8;
+    const int id = (xcd < r8 ? xcd * (q8 + 1) : r8 * (q8 + 1) + (xcd - r8) * q8) + l / 8;
+    const int band = id / (8 * ntiles), rows_in = min(8, mtiles - band * 8), in = id - band * 8 * ntiles;
+    const int m0 = (band * 8 + in % rows_in) * 128, n0 = (in / rows_in) * 128;
+    const int ksteps = p.k >> 5, ntl = p.n >> 4;
+    const int wm = wave >> 1, wn = wave & 1;
+    // this wave's 8 fragments of a stage: A row tiles 2·wave, 2·wave + 1 and B column tiles 2·wave, 2·wave + 1, two k-steps each
+    const bf16 *ap[2], *bp[2];
+#pragma unroll
+    for (int i = 0; i < 2; i++) {
+        const int r = m0 + (2 * wave + i) * 16 + b, t = (n0 >> 4) + 2 * wave + i;
+        ap[i] = p.x + (long)(r < p.m ? r : p.m - 1) * p.ldx + g * p.x_group + 8 * a;
+        bp[i] = p.w + ((long)g * ntl + (t < ntl ? t : ntl - 1)) * ksteps * 512 + lane * 8;
+    }
+    auto issue = [&](int st, int ks) {
+#pragma unroll
+        for (int h = 0; h < 2; h++) {
+            const int kk = ks + h < ksteps ? ks + h : ksteps - 1;
+#pragma unroll
+            for (int i = 0; i < 2; i++) {
+                bf16* da = &lds[st][((2 * wave + i) * 2 + h) * 512];
+                bf16* db = &lds[st][(16 + (2 * wave + i) * 2 + h) * 512];
+                __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(ap[i] + kk * 32),
+                                                 (__attribute__((address_space(3))) void*)da, 16, 0, 0);
+                __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(bp[i] + (long)kk * 512),
+                                                 (__attribute__((address_space(3))) void*)db, 16, 0, 0);
+            }
+        }
+    };
+    floatx4 acc[4][4];
+#pragma unroll
+    for (int i = 0; i < 4; i++)
+#pragma unroll
+        for (int j = 0; j < 4; j++) acc[i][j] = (floatx4){0.f, 0.f, 0.f, 0.f};
+    issue(0, 0);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    __syncthreads();
+    int st = 0;
+    for (int ks = 0; ks < ksteps; ks += 2, st ^= 1) {
+        if (ks + 2 < ksteps) issue(st ^ 1, ks + 2);
+#pragma unroll
+        for (int h = 0; h < 2; h++) {
+            if (ks + h >= ksteps) break;
+            bf16x8 af[4], bf[4];
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                af[i] = *reinterpret_cast<const bf16x8*>(&lds[st][((wm * 4 + i) * 2 + h) * 512 + lane * 8]);
+                bf[i] = *reinterpret_cast<const bf16x8*>(&lds[st][(16 + (wn * 4 + i) * 2 + h) * 512 + lane * 8]);
+            }
+#pragma unroll
+            for (int i = 0; i < 4; i++)
+#pragma unroll
+                for (int j = 0; j < 4; j++) acc[i][j] = Frag<bf16>::mma(af[i], bf[j], acc[i][j]);
+        }
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        __syncthreads();
+    }
+#pragma unroll
+    for (int j = 0; j < 4; j++) {
+        const int col0 = n0 + wn * 64 + j * 16;
+        if (col0 >= p.n) break;
+        const GemmSection sec = gemm_section(p, col0);
+#pragma unroll
+        for (int i = 0; i < 4; i++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) gemm_epilogue(p, sec, g, m0 + wm * 64 + i * 16 + 4 * a + r, col0 + b, acc[i][j][r]);
+    }
+}
+
+static int launch_big(const TiledGemm<bf16>& g, hipStream_t s) {
+    const int mtiles = cdiv(g.m, 128), ntiles = cdiv(g.n, 128);
+    form_hit(FORM_TILED_GEMM_BIG);
+    hipLaunchKernelGGL(tiled_gemm_big_kernel, dim3(mtiles * ntiles, 1, g.groups), dim3(256), 0, s, g, mtiles, ntiles);
+    FH_CHECK_LAUNCH();
+    return 0;
+}
+static int launch_big(const TiledGemm<float>&, hipStream_t) { return 2; }      // (never taken: 16-bit only)
+
+template <typename E>
+int tiled_gemm(const TiledGemm<E>& gin, hipStream_t s) {
+    TiledGemm<E> g = gin;
+    if (g.m <= 0) return 0;
+    if (!g.n_store) g.n_store = g.n;
+    FH_REQUIRE(g.n > 0 && g.k > 0 && g.n % 32 == 0 && g.k % 32 == 0, "tiled_gemm: n=%d k=%d must be multiples of 32", g.n, g.k);
+    FH_REQUIRE(g.ldx % 8 == 0 && g.x_group % 8 == 0 && g.n_store <= g.n && g.groups >= 1, "tiled_gemm: ldx=%ld group stride=%ld", g.ldx, g.x_group);
+    FH_REQUIRE((g.out != nullptr) != (g.out_f32 != nullptr), "tiled_gemm: exactly one output");
+    const long tiles = (long)cdiv(g.m, 128) * cdiv(g.n, 128) * g.groups;
+    if (sizeof(E) == 2 && g.m > 64 && tiles >= knobs().tiled_big_min_tiles) return launch_big(g, s);
+    const int mt = g.m <= 16 ? 1 : (g.m <= 32 ? 2 : 4), J = 2;
+    const int rbs = cdiv(g.m, 16 * mt), ksteps = g.k / 32;
+    // column groups of 32; split K over the waves until the launch has enough of them
+    int kw = 1;
+    const long waves = (long)rbs * (g.n / 32) * g.groups;
+    while (kw < 8 && waves * kw < 4096 && ksteps >= 4 * kw) kw *= 2;
+    const int cw = 8 / kw;
+    const dim3 grid(cdiv(g.n / 32, cw), rbs, g.groups);
+    const size_t lds = kw == 1 ? 0 : (size_t)8 * mt * J * 1024;
+    form_hit(FORM_TILED_GEMM);
+    if (mt == 1) hipLaunchKernelGGL((tiled_gemm_kernel<E, 1, 2>), grid, dim3(512), lds, s, g, kw);
+    else if (mt == 2) hipLaunchKernelGGL((tiled_gemm_kernel<E, 2, 2>), grid, dim3(512), lds, s, g, kw);
+    else hipLaunchKernelGGL((tiled_gemm_kernel<E, 4, 2>), grid, dim3(512), lds, s, g, kw);
+    FH_CHECK_LAUNCH();
+    return 0;
+}
+template int tiled_gemm<bf16>(const TiledGemm<bf16>&, hipStream_t);
+template int tiled_gemm<float>(const TiledGemm<float>&, hipStream_t);
+
+}  // namespace fh

@@ -24,6 +24,23 @@ class ModelConfig(C.Structure):
         ("vocab_parallel", C.c_int32)]
 
 
+class LayeredConfig(C.Structure):
+    """Whole-model part of a layered model (FerrumHipLayeredConfig)."""
+    _fields_ = [("dtype", C.c_int32), ("state_slots", C.c_int32), ("bigram_buckets", C.c_int32), ("residual_mult", C.c_float),
+                ("bigram_mul_prev", C.c_int64), ("bigram_mul_cur", C.c_int64)]
+
+
+class LayerSpec(C.Structure):
+    """One layer of a layered model (FerrumHipLayerSpec)."""
+    _fields_ = [(n, C.c_int32) for n in ("mixer", "ff", "ff_width", "heads", "dim", "rot_dim", "vdim", "q_rank", "kv_rank", "rot_dims",
+                                         "window")] + [("scale", C.c_float), ("rot_base", C.c_double)] + [
+        (n, C.c_int32) for n in ("rnn_width", "rnn_blocks", "conv_taps", "_pad")]
+
+
+DTYPE = {"bfloat16": 0, "float32": 1}
+MIXER = {"latent_attention": 1, "rglru": 2}
+
+
 class BatchItem(C.Structure):
     """UnifiedBatchItem (model_executor.rs:354-386)."""
     _fields_ = [("seq_id", C.c_uint64), ("q_tokens", C.POINTER(C.c_uint32)), ("num_q_tokens", C.c_int32),
@@ -135,6 +152,13 @@ class Checkpoint:
         d = {f: getattr(cfg, f) for f, _ in ModelConfig._fields_ if not f.startswith("_pad")}
         return d, arch.value.decode(), bool(tied.value)
 
+    def layered_config(self):
+        """(LayeredConfig, [LayerSpec]) of a layered architecture, None for the homogeneous families."""
+        n = self.model_config()[0]["num_layers"]
+        flag, lc, specs = C.c_int(), LayeredConfig(), (LayerSpec * max(n, 1))()
+        _check(self.lib.ferrum_hip_checkpoint_layered_config(self.h, C.byref(flag), C.byref(lc), specs, n), "checkpoint_layered_config")
+        return (lc, list(specs)[:n]) if flag.value else None
+
 
 class Comm:
     """`BackendCollective` (ferrum-kernels/src/backend/capabilities.rs:84-109) over `ferrum_hip_comm_*`: one rank of a
@@ -224,18 +248,22 @@ class Comm:
 
 class HipModel:
     @classmethod
-    def from_checkpoint(cls, model_dir, kv_num_blocks, max_seqs, max_tokens, max_seq_len=0):
-        """Create → load every tensor with the reference's names and fusions → finalize."""
+    def from_checkpoint(cls, model_dir, kv_num_blocks, max_seqs, max_tokens, max_seq_len=0, dtype="bfloat16", state_slots=0):
+        """Create → load every tensor with the reference's names and fusions → finalize.  dtype / state_slots: layered models."""
         ck = Checkpoint(model_dir)
         d, _, _ = ck.model_config(max_seq_len)
         d.update(kv_num_blocks=kv_num_blocks, max_seqs=max_seqs, max_tokens=max_tokens)
-        m = cls(**d)
+        layered = ck.layered_config()
+        if layered:
+            layered[0].dtype, layered[0].state_slots = DTYPE[dtype], state_slots
+        m = cls(layered=layered, **d)
         _check(m.lib.ferrum_hip_model_load_checkpoint(m.h, ck.h), "model_load_checkpoint")
         m.finalize()
         ck.close()
         return m
 
-    def __init__(self, **kw):
+    def __init__(self, layered=None, **kw):
+        """layered: (LayeredConfig, [LayerSpec]) for a layered model."""
         self.lib = load_library()
         self.cfg = ModelConfig()
         d = dict(_DEFAULTS)
@@ -243,6 +271,12 @@ class HipModel:
         for k, v in d.items():
             setattr(self.cfg, k, v)
         self.h = C.c_void_p()
+        if layered:
+            lc, specs = layered
+            self.cfg.num_layers = len(specs)
+            _check(self.lib.ferrum_hip_model_create_layered(C.byref(self.h), C.byref(self.cfg), C.byref(lc), (LayerSpec * len(specs))(*specs)),
+                   "model_create_layered")
+            return
         _check(self.lib.ferrum_hip_model_create(C.byref(self.h), C.byref(self.cfg)), "model_create")
 
     def __del__(self):
@@ -271,6 +305,13 @@ class HipModel:
         _check(self.lib.ferrum_hip_model_set_gptq(self.h, layer, GPTQ[name], expert, qw.ctypes.data_as(p),
                                                   sc.ctypes.data_as(C.POINTER(C.c_float)), qz.ctypes.data_as(p),
                                                   None if gi is None else gi.ctypes.data_as(p), k, n), f"set_gptq({name})")
+
+    def set_tensor(self, name, data):
+        """A layered model's weight by tensor name."""
+        d = _f32(data)
+        shape = (C.c_int64 * max(d.ndim, 1))(*(d.shape or (1,)))
+        _check(self.lib.ferrum_hip_model_set_tensor_f32(self.h, name.encode(), d.ctypes.data_as(C.POINTER(C.c_float)), shape, max(d.ndim, 1)),
+               f"set_tensor({name})")
 
     def set_dense(self, layer, name, weight, k, n):
         """Unquantised projection (DenseLinear): weight [n, k] f32; name in qkv / o / gate_up / down."""
@@ -370,6 +411,24 @@ class HipModel:
             toks.ctypes.data_as(C.POINTER(C.c_uint32)),
             None if logits is None else logits.ctypes.data_as(C.POINTER(C.c_float))), "unified_forward")
         return (toks[:n_final] if greedy else None), (logits[:n_final] if logits is not None else None)
+
+    def forward_rows(self, items, rows):
+        """items: [(seq_id, tokens, pos_offset)]; logits [len(rows), vocab] at places of the batch counted over all items' tokens."""
+        keep = [np.ascontiguousarray(t, dtype=np.uint32) for _, t, _ in items]
+        arr = (BatchItem * len(items))()
+        for i, (sid, _, pos) in enumerate(items):
+            arr[i] = BatchItem(sid, keep[i].ctypes.data_as(C.POINTER(C.c_uint32)), len(keep[i]), pos, 0, 0)
+        r = _i32(rows)
+        out = np.zeros((max(len(r), 1), self.local_vocab()[1]), np.float32)
+        _check(self.lib.ferrum_hip_model_unified_forward_rows(self.h, arr, len(items), r.ctypes.data_as(C.POINTER(C.c_int32)), len(r),
+                                                              out.ctypes.data_as(C.POINTER(C.c_float))), "unified_forward_rows")
+        return out[:len(r)]
+
+    def state_slots(self):
+        """(recurrent-state slots, free ones)"""
+        n, f = C.c_int(), C.c_int()
+        _check(self.lib.ferrum_hip_model_state_slots(self.h, C.byref(n), C.byref(f)), "state_slots")
+        return n.value, f.value
 
     def local_vocab(self):
         """(first vocabulary row, row count) this model scores: the whole vocabulary unless cfg.vocab_parallel."""

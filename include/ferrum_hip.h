@@ -452,6 +452,35 @@ typedef struct {
     int32_t vocab_parallel;
 } FerrumHipModelConfig;
 
+/* ── Layered models (no counterpart in the reference): decoders whose layers are described one by one.  The runner keeps doing for
+ *    them what it does for the homogeneous families — paged blocks, admission, batching, sampling, the decode graph — plus one
+ *    recurrent-state slot per live sequence.  Architectures: Nerenex. ── */
+#define FERRUM_HIP_DTYPE_BF16 0
+#define FERRUM_HIP_DTYPE_F32 1
+#define FERRUM_HIP_MIXER_LATENT_ATTENTION 1
+#define FERRUM_HIP_MIXER_RGLRU 2
+#define FERRUM_HIP_FF_NONE 0
+#define FERRUM_HIP_FF_XIELU 1
+typedef struct {
+    int32_t dtype;                /* FERRUM_HIP_DTYPE_*: projections, activations and caches; norms, scores, recurrences and the
+                                     residual stream are fp32 either way */
+    int32_t state_slots;          /* sequences that may hold recurrent state at a time; 0 = max_seqs */
+    int32_t bigram_buckets;       /* 0 = none; else a hashed (previous token, token) embedding of this many rows + 1 */
+    float residual_mult;          /* factor of a sublayer's normed result */
+    int64_t bigram_mul_prev, bigram_mul_cur;
+} FerrumHipLayeredConfig;
+typedef struct {
+    int32_t mixer;                /* FERRUM_HIP_MIXER_* */
+    int32_t ff, ff_width;         /* FERRUM_HIP_FF_*; NONE: the layer is the mixer alone */
+    /* latent attention: per head `dim` unrotated + `rot_dim` rotated query / key dimensions (the first rot_dims of the latter turn),
+     * values of vdim; a token sees itself and the window - 1 tokens before it */
+    int32_t heads, dim, rot_dim, vdim, q_rank, kv_rank, rot_dims, window;
+    float scale;
+    double rot_base;
+    /* real-gated linear recurrent unit */
+    int32_t rnn_width, rnn_blocks, conv_taps, _pad;
+} FerrumHipLayerSpec;
+
 /* One item of a UnifiedBatch (model_executor.rs:354-386). */
 typedef struct {
     uint64_t seq_id;              /* cache id */
@@ -473,6 +502,12 @@ typedef struct {
 } FerrumHipKvSlotReservation;
 
 int ferrum_hip_model_create(FerrumHipModel** model, const FerrumHipModelConfig* cfg);
+/* A layered model: cfg carries num_layers, hidden, vocab, rms_eps, max_seq_len, kv_num_blocks, max_seqs and max_tokens (the other
+ * architecture fields are unused), layers[num_layers] the rest.  Weights arrive by tensor name. */
+int ferrum_hip_model_create_layered(FerrumHipModel** model, const FerrumHipModelConfig* cfg, const FerrumHipLayeredConfig* layered,
+                                    const FerrumHipLayerSpec* layers);
+int ferrum_hip_model_set_tensor_f32(FerrumHipModel* model, const char* name, const float* data, const int64_t* shape, int ndim);
+int ferrum_hip_model_is_layered(const FerrumHipModel* model);
 int ferrum_hip_model_destroy(FerrumHipModel* model);
 /* Weight hand-over (host slices, copied/repacked to device).  which:
  *   global dense: 0 embed [V,H], 1 lm_head [V,H] (omit → tied to embed), 2 final_norm [H]
@@ -513,7 +548,8 @@ int ferrum_hip_model_prefix_cache_stats(const FerrumHipModel* model, uint64_t* h
  *    "quantization_config" (:1475-1530), config.json mapping (ferrum-models/src/definition.rs:225-375,
  *    models/llama_family.rs:596-680,733-810, moe_config.rs:91-130), tensor names (llama_family.rs:900-945,
  *    qwen3_moe/load.rs:178-260).  Architectures: Llama, Mistral, Qwen2 (fused q|k|v bias), Qwen3, Qwen3-MoE, Gemma-3 (norm folds of
- *    llama_family.rs:891-967 applied at load); others → FERRUM_HIP_UNSUPPORTED. ── */
+ *    llama_family.rs:891-967 applied at load); layered architectures by their own
+ *    config.json (ferrum_hip_checkpoint_layered_config); others → FERRUM_HIP_UNSUPPORTED. ── */
 typedef struct FerrumHipCheckpoint FerrumHipCheckpoint;
 int ferrum_hip_checkpoint_open(FerrumHipCheckpoint** ck, const char* model_dir);
 int ferrum_hip_checkpoint_close(FerrumHipCheckpoint* ck);
@@ -533,6 +569,10 @@ int ferrum_hip_checkpoint_read_gptq_fused(const FerrumHipCheckpoint* ck, const c
  * max_seq_len = min(max_position_embeddings, cap) (cap 0 = none); tied_lm_head = no lm_head.weight tensor. */
 int ferrum_hip_checkpoint_model_config(const FerrumHipCheckpoint* ck, int max_seq_len_cap, FerrumHipModelConfig* cfg,
                                        char* arch_out, size_t arch_cap, int* tied_lm_head);
+/* config.json of a layered architecture → its description: *is_layered = 0 (and nothing else) for the homogeneous families; else
+ * num_layers specs (capacity entries at most are written). */
+int ferrum_hip_checkpoint_layered_config(const FerrumHipCheckpoint* ck, int* is_layered, FerrumHipLayeredConfig* layered,
+                                         FerrumHipLayerSpec* layers, int capacity);
 /* Hand every weight to a created, not yet finalized model (dimensions from ferrum_hip_checkpoint_model_config). */
 int ferrum_hip_model_load_checkpoint(FerrumHipModel* model, const FerrumHipCheckpoint* ck);
 
@@ -576,6 +616,12 @@ typedef struct {
 int ferrum_hip_model_local_vocab(const FerrumHipModel* model, int* vocab_start, int* vocab_count);
 int ferrum_hip_model_unified_forward_ex(FerrumHipModel* model, const FerrumHipBatchItem* items, int num_items, int greedy,
                                         const FerrumHipGreedyOptions* opts, uint32_t* out_tokens, float* logits_out);
+/* The same forward with logits at arbitrary places of the batch: rows[r] counts tokens in item order over the whole batch;
+ * logits_out [num_rows, vocab slice].  is_final_chunk is ignored and nothing is sampled.  num_rows may be 0. */
+int ferrum_hip_model_unified_forward_rows(FerrumHipModel* model, const FerrumHipBatchItem* items, int num_items, const int32_t* rows,
+                                          int num_rows, float* logits_out);
+/* Recurrent-state slots (layered models; 0 / 0 for models without state). */
+int ferrum_hip_model_state_slots(const FerrumHipModel* model, int* total, int* free_slots);
 /* Steady-state decode: every listed sequence advances by one token (its last sampled token),
  * `steps` times, with device-side greedy sampling and hipGraph replay when available.
  * out_tokens [steps, n] (may be NULL). */
