@@ -396,8 +396,86 @@ def tp_decode_case(pkg, torch, dist, model_name, world, rank, c, PL, steps, warm
     return res
 
 
+# ── layered models: a Nerenex stack with layers of a real model's size beside the closest homogeneous model (sliding-window attention,
+#    post-sublayer norms on an fp32 residual stream, unquantised 16-bit projections) at equal width, heads, feed-forward, window, depth ──
+LAYERED_SIZES = {
+    "2k": dict(width=2048, heads=16, dim=128, rot_dim=64, vdim=128, q_rank=768, kv_rank=512, window=1024, ff=8192, rnn_width=2048,
+               rnn_blocks=16, taps=4, vocab=32768, layers=12),
+    "4k": dict(width=4096, heads=32, dim=128, rot_dim=64, vdim=128, q_rank=1536, kv_rank=512, window=2048, ff=14336, rnn_width=4096,
+               rnn_blocks=32, taps=4, vocab=65536, layers=12),
+}
+
+
+def layered_model(pkg, size, side, max_seq_len, blocks, max_seqs, max_tokens):
+    """side: "nerenex" (two recurrent layers, then one attention layer, repeated), "attention" / "recurrent" (one kind only),
+    "dense" (the homogeneous model)."""
+    z = LAYERED_SIZES[size]
+    common = dict(num_layers=z["layers"], hidden=z["width"], vocab=z["vocab"], max_seq_len=max_seq_len, kv_num_blocks=blocks, max_seqs=max_seqs,
+                  max_tokens=max_tokens, rms_eps=1e-6)
+    if side == "dense":
+        prev = os.environ.get("FERRUM_HIP_SYNTH_DENSE")
+        os.environ["FERRUM_HIP_SYNTH_DENSE"] = "1"
+        try:
+            m = pkg.HipModel(num_heads=z["heads"], num_kv_heads=z["heads"] // 4, head_dim=128, intermediate=z["ff"], has_qk_norm=1, activation=1,
+                             sliding_window=z["window"], sliding_window_pattern=0, sandwich_norms=1, rope_theta=1e6, **common)
+            m.init_synthetic(7)
+        finally:
+            if prev is None:
+                del os.environ["FERRUM_HIP_SYNTH_DENSE"]
+    else:
+        specs = []
+        for i in range(z["layers"]):
+            attn = side == "attention" or (side == "nerenex" and i % 3 == 2)
+            if attn:
+                specs.append(pkg.LayerSpec(mixer=1, ff=1, ff_width=z["ff"], heads=z["heads"], dim=z["dim"], rot_dim=z["rot_dim"], vdim=z["vdim"],
+                                           q_rank=z["q_rank"], kv_rank=z["kv_rank"], rot_dims=z["rot_dim"], window=z["window"],
+                                           scale=(z["dim"] + z["rot_dim"]) ** -0.5, rot_base=1e6))
+            else:
+                specs.append(pkg.LayerSpec(mixer=2, ff=1, ff_width=z["ff"], rnn_width=z["rnn_width"], rnn_blocks=z["rnn_blocks"],
+                                           conv_taps=z["taps"]))
+        lc = pkg.LayeredConfig(dtype=0, state_slots=max_seqs, bigram_buckets=65536, residual_mult=0.7, bigram_mul_prev=40503, bigram_mul_cur=9973)
+        m = pkg.HipModel(layered=(lc, specs), **common)
+        m.init_synthetic(7)
+    m.finalize()
+    return m
+
+
+def layered_bench(pkg, torch, args):
+    z = LAYERED_SIZES[args.layered]
+    res = {"metric": "layered models: prefill and decode tokens/s", "size": args.layered, "config": z, "data": "synthetic", "dtype": "bf16 / fp16",
+           "steps": args.steps, "warmup": args.warmup, "cases": []}
+    for side in args.layered_sides.split(","):
+        for conc, plen in ((1, 4096), (8, 1024), (32, 256)):
+            seq = plen + args.steps + args.warmup + 16
+            seq = (seq + 15) // 16 * 16
+            chunk = min(args.prefill_chunk, conc * plen)
+            m = layered_model(pkg, args.layered, side, seq, (conc + 1) * seq // 16, conc, max(chunk, conc))
+            rng = np.random.default_rng(1)
+            prompts = [rng.integers(0, z["vocab"], size=plen).astype(np.uint32) for _ in range(conc)]
+            prefill(m, prompts, 1, chunk)                               # warm-up: code objects, caches
+            for i in range(conc):
+                m.release(1 + i)
+            t0 = time.perf_counter()
+            first = prefill(m, prompts, 101, chunk)
+            t_pre = time.perf_counter() - t0
+            ids = list(range(101, 101 + conc))
+            nxt = m.decode_steps(ids, first, args.warmup)[-1]
+            torch.cuda.synchronize()
+            t0 = time.perf_counter()
+            m.decode_steps(ids, nxt, args.steps)
+            t_dec = time.perf_counter() - t0
+            res["cases"].append({"side": side, "concurrency": conc, "prompt": plen, "prefill_ms": round(t_pre * 1e3, 3),
+                                 "prefill_tok_s": round(conc * plen / t_pre, 1), "decode_ms_per_step": round(t_dec / args.steps * 1e3, 4),
+                                 "decode_tok_s": round(conc * args.steps / t_dec, 1)})
+            print(json.dumps(res["cases"][-1]), file=sys.stderr, flush=True)
+            del m
+    print(json.dumps(res))
+
+
 def main():
     ap = argparse.ArgumentParser()
+    ap.add_argument("--layered", default="", choices=[""] + sorted(LAYERED_SIZES), help="extra workload: a Nerenex stack of this size beside the closest homogeneous model")
+    ap.add_argument("--layered-sides", default="nerenex,dense", help="with --layered: which of nerenex, attention, recurrent, dense")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=64)
     ap.add_argument("--warmup", type=int, default=8)
@@ -434,6 +512,8 @@ def main():
     import __graft_entry__ as ge
     pkg = ge.load_package()
     pkg.load_library()
+    if args.layered:
+        return layered_bench(pkg, torch, args)
     cfg = dict(MODELS[args.model])
     moe = cfg["num_experts"] > 0
     c, K, W, PL = args.concurrency, args.steps, args.warmup, args.prompt_len

@@ -1,13 +1,17 @@
 // Attention over a compressed cache (multi-head latent attention): a token caches one normed latent c and one rotated key part shared
 // by all heads; head h's key is (W_uk,h c | shared part) and its value W_uv,h c.
 //
-// The kernels here never expand keys or values: the query's plain part arrives already multiplied by W_uk,hᵀ (q_lat), so a score is
+// One token per sequence and short portions never expand keys or values: the query's plain part arrives already multiplied by W_uk,hᵀ (q_lat), so a score is
 // q_lat · c + rot(q) · k_rot, and the output is left in latent space (o_lat = Σ p c) for the value projection that follows.  All heads
 // of a token share one cache entry, so a 16-row MFMA tile is 16 (token, head) pairs of one sequence and the cache is read once for them.
 //
 // Cache tiles are K-fragment shaped ([chunk of 8 dims][16 keys][8]): a wave's K fragment is one contiguous 1-KiB load and feeds the
-// matrix pipe directly.  The same registers are parked in wave-private LDS and come back transposed (ds_read_b64_tr_b16) as the Vᵀ
-// operand of O ᵀ += Vᵀ·Pᵀ — the latent is read from memory once for both products.
+// matrix pipe directly.  The same registers are parked in LDS and come back transposed (ds_read_b64_tr_b16) as the Vᵀ operand of
+// Oᵀ += Vᵀ·Pᵀ — the latent is read from memory once for both products.
+//
+// Prompt portions of many tokens are compute-bound, and the latent form costs 2·kv_rank + rot per (query, key) where keys and values
+// cost dim + rot + vdim: for those the projections of the visible cache blocks are expanded once per layer (a GEMM that reads the
+// cache's fragments in place) and a flash kernel runs over them.
 #include <math.h>
 
 #include <algorithm>
@@ -147,13 +151,23 @@ __global__ __launch_bounds__(256) void latent_attn_plain_kernel(LatentDims d, La
 
 // ── matrix-core form ──
 struct LatentTile { int seq, tile, tok0, q_len, pos0; };
+__device__ __forceinline__ int latent_tiles(const BatchView& v, int q_len, int heads) {
+    return v.long_min > 0 && q_len >= v.long_min ? 0 : (q_len * heads + 15) >> 4;
+}
 // 16-row tiles of (token, head) pairs, numbered sequence by sequence; every wave finds tile w by a scan of cu_seqlens
 __device__ __forceinline__ bool find_latent_tile(const BatchView& v, int heads, int w, LatentTile* o) {
+    if (v.single) {
+        const int per = (heads + 15) >> 4;
+        o->seq = w / per; o->tile = w % per; o->tok0 = o->seq; o->q_len = 1;
+        if (o->seq >= v.num_seqs) return false;
+        o->pos0 = (int)v.pos[o->seq];
+        return true;
+    }
     const int lane = threadIdx.x & 63;
     int base = 0;
     for (int s0 = 0; s0 < v.num_seqs; s0 += 64) {
         const int s = s0 + lane;
-        const int units = s < v.num_seqs ? ((int)(v.cu[s + 1] - v.cu[s]) * heads + 15) >> 4 : 0;
+        const int units = s < v.num_seqs ? latent_tiles(v, (int)(v.cu[s + 1] - v.cu[s]), heads) : 0;
         int incl = units;
 #pragma unroll
         for (int off = 1; off < 64; off <<= 1) {
@@ -177,18 +191,28 @@ __device__ __forceinline__ bool find_latent_tile(const BatchView& v, int heads, 
 
 constexpr int LATENT_RS = 2;           // k-steps of the rotated part: rot_dim ≤ 64
 constexpr int LATENT_PARTIAL_PAD = 4;  // floats behind a partial row's outputs: maximum, sum
+// offset of lane's 4 values in a transposed read: lane i of a 16-lane group names 4 dims of key 4a + i / 4 (of a 16-key block, 16 dims =
+// two chunks) and receives dim i of keys 4a … 4a + 3
+__device__ __forceinline__ int tr_offset(int lane) {
+    return ((((lane & 3) >> 1) * 16) + 4 * (lane >> 4) + ((lane & 15) >> 2)) * 8 + (lane & 1) * 4;
+}
+__device__ __forceinline__ shortx4 read_tr(const bf16* p) {
+    return __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) shortx4*)p);
+}
 
-// KS: most k-steps of the latent (kv_rank ≤ 32·KS).  grid (row tiles, KV splits), 4 waves over the keys of a split.
+// KS: most k-steps of the latent (kv_rank ≤ 32·KS).  grid (KV splits, row tiles); a step is 64 keys: wave w scores block w of them
+// for all 16 rows, the row maxima meet in LDS, P and the parked latents are shared, and each wave accumulates its own quarter of the
+// output dimensions — so nothing is merged at the end and the latents of the next step are in flight during softmax and P·V.
 template <int KS>
-__global__ __launch_bounds__(256, 1) void latent_attn_kernel(LatentDims d, LatentBuffers<bf16> p, BatchView v, int nsplit) {
-    constexpr int DT = 2 * KS, OSTR = 32 * KS + 4;
-    constexpr int STAGE = KS * 512;                                            // one 16-key block of latents per wave
-    constexpr int LDS_BYTES = 4 * STAGE * 2 > 16 * OSTR * 4 ? 4 * STAGE * 2 : 16 * OSTR * 4;
-    __shared__ __attribute__((aligned(16))) unsigned char smem[LDS_BYTES];
+__global__ __launch_bounds__(256, 2) void latent_attn_kernel(LatentDims d, LatentBuffers<bf16> p, BatchView v, int nsplit) {
+    constexpr int DT = KS < 2 ? 1 : KS / 2;                                    // 16-dim output tiles per wave
+    constexpr int STAGE = KS * 512, PSTR = 72;
+    __shared__ __attribute__((aligned(16))) bf16 stage[4 * STAGE];
+    __shared__ __attribute__((aligned(16))) bf16 lds_p[16 * PSTR];
     __shared__ float lds_m[64], lds_l[64];
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, a = lane >> 4, b = lane & 15;
     LatentTile w;
-    if (!find_latent_tile(v, d.heads, blockIdx.x, &w)) return;
+    if (!find_latent_tile(v, d.heads, blockIdx.y, &w)) return;
     const int ks = d.kp >> 5, rs = d.rp >> 5, kd = d.kp + d.rp, rows = w.q_len * d.heads;
     const int rho = w.tile * 16 + b;
     const bool ok = rho < rows;
@@ -196,23 +220,22 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LatentDims d, Laten
     const int row_pos = w.pos0 + tl, win_lo = max(0, row_pos + 1 - d.window);
     const int t_first = w.tile * 16 / d.heads, t_last = min(w.q_len - 1, (w.tile * 16 + 15) / d.heads);
     const int kv_end = w.pos0 + t_last + 1, kv_lo = max(0, w.pos0 + t_first + 1 - d.window);
-    const int blk_lo = kv_lo / 16, nblk = (kv_end + 15) / 16 - blk_lo;
-    const int per = (nblk + nsplit - 1) / nsplit;
-    const int my_lo = blk_lo + (int)blockIdx.y * per, my_hi = min(blk_lo + nblk, my_lo + per);
+    const int blk_lo = kv_lo / 16, blk_hi = (kv_end + 15) / 16, nstep = (blk_hi - blk_lo + 3) / 4;
+    const int per = (nstep + nsplit - 1) / nsplit;
+    const int st_lo = (int)blockIdx.x * per, st_hi = min(nstep, st_lo + per);
     const int32_t* bt = v.bt + (long)w.seq * v.max_blocks;
 
-    bf16x8 kf[KS + LATENT_RS], kn[KS + LATENT_RS], qf[KS + LATENT_RS];
-    auto load = [&](int blk, bf16x8 (&f)[KS + LATENT_RS]) {
-        const bf16* t = p.pool + (long)bt[blk] * 16 * kd + lane * 8;
+    bf16x8 kf[KS + LATENT_RS], qf[KS + LATENT_RS];
+    auto load = [&](int st) {                                                  // (past the last block: a copy of it, masked below)
+        const bf16* t = p.pool + (long)bt[min(blk_lo + 4 * st + wave, blk_hi - 1)] * 16 * kd + lane * 8;
 #pragma unroll
         for (int s = 0; s < KS; s++)
-            if (s < ks) f[s] = *reinterpret_cast<const bf16x8*>(t + s * 512);
+            if (s < ks) kf[s] = *reinterpret_cast<const bf16x8*>(t + s * 512);
 #pragma unroll
         for (int s = 0; s < LATENT_RS; s++)
-            if (s < rs) f[KS + s] = *reinterpret_cast<const bf16x8*>(t + (ks + s) * 512);
+            if (s < rs) kf[KS + s] = *reinterpret_cast<const bf16x8*>(t + (ks + s) * 512);
     };
-    const int first = my_lo + wave;
-    if (first < my_hi) load(first, kf);
+    if (st_lo < st_hi) load(st_lo);
     {
         const long qrow = (long)(w.tok0 + tl) * d.heads + h;
 #pragma unroll
@@ -224,116 +247,278 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LatentDims d, Laten
                 qf[KS + s] = rotate8(*reinterpret_cast<const bf16x8*>(p.q + qrow * (d.dp + d.rp) + d.dp + 32 * s + 8 * a), 32 * s + 8 * a,
                                      d.rot_dims, p.cos_t, p.sin_t, row_pos);
     }
-    bf16* stage = reinterpret_cast<bf16*>(smem) + wave * STAGE;
-    // transposed read of d-tile dt: lane i of a 16-lane group names 4 dims of key 4a + i / 4 and receives dim i of keys 4a … 4a + 3
-    const int tr_off = ((((lane & 3) >> 1) * 16) + 4 * a + ((lane & 15) >> 2)) * 8 + (lane & 1) * 4;
+    const int tr_off = tr_offset(lane);
     float m_run = -INFINITY, l_run = 0.f;
     floatx4 o[DT];
 #pragma unroll
     for (int t = 0; t < DT; t++) o[t] = (floatx4){0.f, 0.f, 0.f, 0.f};
-    for (int blk = first; blk < my_hi; blk += 4) {
-        if (blk + 4 < my_hi) load(blk + 4, kn);
-        floatx4 sc = {0.f, 0.f, 0.f, 0.f};
+    for (int st = st_lo; st < st_hi; st++) {
+        floatx4 sc2[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};        // two chains: half the dependent MFMA latency
 #pragma unroll
         for (int s = 0; s < KS; s++)
-            if (s < ks) {
-                sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[s], qf[s], sc, 0, 0, 0);
-                *reinterpret_cast<bf16x8*>(stage + s * 512 + lane * 8) = kf[s];
-            }
+            if (s < ks) sc2[s & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[s], qf[s], sc2[s & 1], 0, 0, 0);
 #pragma unroll
         for (int s = 0; s < LATENT_RS; s++)
-            if (s < rs) sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[KS + s], qf[KS + s], sc, 0, 0, 0);
+            if (s < rs) sc2[s & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[KS + s], qf[KS + s], sc2[s & 1], 0, 0, 0);
+        floatx4 sc;
         float mx = -INFINITY;
 #pragma unroll
         for (int r = 0; r < 4; r++) {
-            const int key = blk * 16 + 4 * a + r;
-            sc[r] = ok && key <= row_pos && key >= win_lo ? sc[r] * d.scale : -INFINITY;
+            const int key = (blk_lo + 4 * st + wave) * 16 + 4 * a + r;
+            sc[r] = ok && key <= row_pos && key >= win_lo ? (sc2[0][r] + sc2[1][r]) * d.scale : -INFINITY;
             mx = fmaxf(mx, sc[r]);
         }
-        const float m_new = fmaxf(m_run, rows_reduce_max(mx)), m_safe = m_new == -INFINITY ? 0.f : m_new;
-        const float alpha = __expf(m_run - m_safe);
-        float ps = 0.f;
+        mx = rows_reduce_max(mx);
+        __syncthreads();                                                       // the previous step's P·V has read stage and lds_p
+#pragma unroll
+        for (int s = 0; s < KS; s++)
+            if (s < ks) *reinterpret_cast<bf16x8*>(stage + wave * STAGE + s * 512 + lane * 8) = kf[s];
+        if (a == 0) lds_m[wave * 16 + b] = mx;
+        if (st + 1 < st_hi) load(st + 1);
+        __syncthreads();
+        const float m_new = fmaxf(m_run, fmaxf(fmaxf(lds_m[b], lds_m[16 + b]), fmaxf(lds_m[32 + b], lds_m[48 + b])));
+        const float m_safe = m_new == -INFINITY ? 0.f : m_new, alpha = __expf(m_run - m_safe);
         bf16x4 pf;
+        float ps = 0.f;
 #pragma unroll
         for (int r = 0; r < 4; r++) { const float e = __expf(sc[r] - m_safe); ps += e; pf[r] = (bf16)e; }
-        l_run = l_run * alpha + rows_reduce_sum(ps);
+        l_run = l_run * alpha + ps;                                            // (this lane's keys; lanes and waves meet at the end)
         m_run = m_new;
+        *reinterpret_cast<bf16x4*>(lds_p + b * PSTR + wave * 16 + 4 * a) = pf;
 #pragma unroll
         for (int t = 0; t < DT; t++)
-            if (t < 2 * ks) {
-                const shortx4 vt = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) shortx4*)(stage + t * 256 + tr_off));
 #pragma unroll
-                for (int r = 0; r < 4; r++) o[t][r] *= alpha;
-                o[t] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(vt, __builtin_bit_cast(shortx4, pf), o[t], 0, 0, 0);
-            }
+            for (int r = 0; r < 4; r++) o[t][r] *= alpha;
+        __syncthreads();
+        // Oᵀ[d][row] += Vᵀ[d][key]·Pᵀ[key][row], 32 keys (two blocks) at a time: lane group a takes keys 8a … 8a + 7 of them
 #pragma unroll
-        for (int s = 0; s < KS + LATENT_RS; s++) kf[s] = kn[s];
-    }
-    // merge the four waves in wave order: scale by exp(m_w − M), then add into one LDS copy
-    if (a == 0) { lds_m[wave * 16 + b] = m_run; lds_l[wave * 16 + b] = l_run; }
-    __syncthreads();
-    float M = -INFINITY, L = 0.f;
-#pragma unroll
-    for (int q = 0; q < 4; q++) M = fmaxf(M, lds_m[q * 16 + b]);
-    const float Ms = M == -INFINITY ? 0.f : M;
-#pragma unroll
-    for (int q = 0; q < 4; q++) L += lds_l[q * 16 + b] * __expf(lds_m[q * 16 + b] - Ms);
-    const float f = __expf(m_run - Ms);
-    float* lo = reinterpret_cast<float*>(smem);
-    for (int q = 0; q < 4; q++) {
-        if (wave == q) {
+        for (int c = 0; c < 2; c++) {
+            const bf16x8 pv = *reinterpret_cast<const bf16x8*>(lds_p + b * PSTR + c * 32 + 8 * a);
+            // keys 8a … of the pair sit in block 2c + (a >> 1), rows (a & 1)·8: the lane's read names those instead of rows 4a
+            const bf16* vb = stage + (2 * c + (a >> 1)) * STAGE + tr_off + ((a & 1) * 8 - 4 * a) * 8;
 #pragma unroll
             for (int t = 0; t < DT; t++)
-                if (t < 2 * ks) {
-                    floatx4* at = reinterpret_cast<floatx4*>(lo + b * OSTR + t * 16 + 4 * a);
-                    floatx4 x = o[t];
-#pragma unroll
-                    for (int r = 0; r < 4; r++) x[r] *= f;
-                    *at = q == 0 ? x : *at + x;
+                if (wave + 4 * t < 2 * ks) {
+                    const shortx4 v0 = read_tr(vb + (wave + 4 * t) * 256), v1 = read_tr(vb + (wave + 4 * t) * 256 + 32);
+                    typedef short shortx8 __attribute__((ext_vector_type(8)));
+                    const shortx8 vt = {v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
+                    o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, vt), pv, o[t], 0, 0, 0);
                 }
         }
-        __syncthreads();
     }
-    const int row = threadIdx.x >> 4, c0 = threadIdx.x & 15;      // 16 threads per row
-    const float Lr = __shfl(L, row, 64), Mr = __shfl(M, row, 64); // (lane `row` of every wave holds that row's totals)
+    l_run = rows_reduce_sum(l_run);
+    if (a == 0) lds_l[wave * 16 + b] = l_run;
+    __syncthreads();
+    const float L = lds_l[b] + lds_l[16 + b] + lds_l[32 + b] + lds_l[48 + b];
     if (nsplit > 1) {
-        float* dst = p.partial + (((long)blockIdx.x * nsplit + blockIdx.y) * 16 + row) * (d.kp + LATENT_PARTIAL_PAD);
-        for (int c = c0 * 4; c < d.kp; c += 64) *reinterpret_cast<floatx4*>(dst + c) = *reinterpret_cast<floatx4*>(lo + row * OSTR + c);
-        if (c0 == 0) { dst[d.kp] = Mr; dst[d.kp + 1] = Lr; }
+        float* dst = p.partial + (((long)blockIdx.y * nsplit + blockIdx.x) * 16 + b) * (d.kp + LATENT_PARTIAL_PAD);
+#pragma unroll
+        for (int t = 0; t < DT; t++)
+            if (wave + 4 * t < 2 * ks) *reinterpret_cast<floatx4*>(dst + (wave + 4 * t) * 16 + 4 * a) = o[t];
+        if (threadIdx.x < 16) { dst[d.kp] = m_run; dst[d.kp + 1] = L; }
         return;
     }
-    const int ro = w.tile * 16 + row;
-    if (ro >= rows) return;
-    const float inv = Lr > 0.f ? 1.0f / Lr : 0.f;
-    bf16* dst = p.o_lat + ((long)w.tok0 * d.heads + ro) * d.kp;
-    for (int c = c0 * 4; c < d.kp; c += 64) {
-        const floatx4 x = *reinterpret_cast<floatx4*>(lo + row * OSTR + c);
-        bf16x4 y;
+    if (!ok) return;
+    const float inv = L > 0.f ? 1.0f / L : 0.f;
+    bf16* dst = p.o_lat + ((long)w.tok0 * d.heads + rho) * d.kp;
 #pragma unroll
-        for (int r = 0; r < 4; r++) y[r] = (bf16)(x[r] * inv);
-        *reinterpret_cast<bf16x4*>(dst + c) = y;
-    }
+    for (int t = 0; t < DT; t++)
+        if (wave + 4 * t < 2 * ks) {
+            bf16x4 y;
+#pragma unroll
+            for (int r = 0; r < 4; r++) y[r] = (bf16)(o[t][r] * inv);
+            *reinterpret_cast<bf16x4*>(dst + (wave + 4 * t) * 16 + 4 * a) = y;
+        }
 }
-// one workgroup per row tile, 16 threads per row
+// grid (row tiles, quads of output dimensions / 256): one thread per (row, 4 dimensions)
 __global__ __launch_bounds__(256) void latent_attn_reduce_kernel(LatentDims d, LatentBuffers<bf16> p, BatchView v, int nsplit) {
     LatentTile w;
     if (!find_latent_tile(v, d.heads, blockIdx.x, &w)) return;
-    const int row = threadIdx.x >> 4, c0 = threadIdx.x & 15, ro = w.tile * 16 + row;
-    if (ro >= w.q_len * d.heads) return;
+    const int quads = d.kp >> 2, id = blockIdx.y * 256 + threadIdx.x, row = id / quads, c = (id % quads) * 4, ro = w.tile * 16 + row;
+    if (row >= 16 || ro >= w.q_len * d.heads) return;
     const long ld = d.kp + LATENT_PARTIAL_PAD;
     const float* src = p.partial + ((long)blockIdx.x * nsplit * 16 + row) * ld;
     float M = -INFINITY, L = 0.f;
     for (int z = 0; z < nsplit; z++) M = fmaxf(M, src[z * 16 * ld + d.kp]);
-    for (int z = 0; z < nsplit; z++) L += src[z * 16 * ld + d.kp + 1] * __expf(src[z * 16 * ld + d.kp] - M);
-    const float inv = 1.0f / L;
-    for (int c = c0 * 4; c < d.kp; c += 64) {
-        floatx4 acc = {0.f, 0.f, 0.f, 0.f};
-        for (int z = 0; z < nsplit; z++) acc += *reinterpret_cast<const floatx4*>(src + z * 16 * ld + c) * (__expf(src[z * 16 * ld + d.kp] - M) * inv);
-        bf16x4 y;
-#pragma unroll
-        for (int r = 0; r < 4; r++) y[r] = (bf16)acc[r];
-        *reinterpret_cast<bf16x4*>(p.o_lat + ((long)w.tok0 * d.heads + ro) * d.kp + c) = y;
+    floatx4 acc = {0.f, 0.f, 0.f, 0.f};
+    for (int z = 0; z < nsplit; z++) {
+        const float f = __expf(src[z * 16 * ld + d.kp] - M);
+        L += src[z * 16 * ld + d.kp + 1] * f;
+        acc += *reinterpret_cast<const floatx4*>(src + z * 16 * ld + c) * f;
     }
+    const float inv = 1.0f / L;
+    bf16x4 y;
+#pragma unroll
+    for (int r = 0; r < 4; r++) y[r] = (bf16)(acc[r] * inv);
+    *reinterpret_cast<bf16x4*>(p.o_lat + ((long)w.tok0 * d.heads + ro) * d.kp + c) = y;
+}
+
+// ── portions over expanded keys and values ──
+// A workgroup owns 128 tokens of one sequence and head: 4 waves × 2 row tiles of 16.  64 keys per step: wave w copies 16-key block w of
+// the step — expanded key rows, the shared rotated part straight from the cache, expanded value rows — as fragments into LDS with the
+// load unit, double-buffered; Sᵀ = K·Qᵀ keeps a row's statistics lane-local, values are read back transposed for Oᵀ += Vᵀ·Pᵀ.
+constexpr int LX_DS = 4, LX_RS = 2, LX_VS = 4;           // most 32-wide steps of the plain, rotated and value dimensions
+__global__ __launch_bounds__(256, 2) void latent_expanded_kernel(LatentDims d, LatentBuffers<bf16> p, BatchView v, LatentExpanded x) {
+    constexpr int MT = 2, BLK = (LX_DS + LX_RS + LX_VS) * 512, DT = 2 * LX_VS;
+    extern __shared__ __attribute__((aligned(16))) bf16 lds_x[];               // [2][4 blocks][BLK]
+    const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, a = lane >> 4, b = lane & 15;
+    const int h = blockIdx.y;
+    const int32_t* un = x.units + 4 * (gridDim.x - 1 - blockIdx.x);            // the longest key ranges start first
+    const int seq = un[0], tile0 = un[1], base = un[2], first_blk = un[3];
+    const int tok0 = (int)v.cu[seq], q_len = (int)v.cu[seq + 1] - tok0, pos0 = (int)v.pos[seq];
+    const int ds = d.dp >> 5, rs = d.rp >> 5, vs = d.vp >> 5, kd = d.kp + d.rp;
+    const float sl2 = d.scale * 1.4426950408889634f;
+
+    bf16x8 qf[MT][LX_DS + LX_RS];
+    int row_pos[MT], win_lo[MT], vis_lo[MT], vis_hi[MT];
+    bool ok[MT];
+#pragma unroll
+    for (int mt = 0; mt < MT; mt++) {
+        const int t0 = tile0 + (wave * MT + mt) * 16, t = t0 + b;
+        ok[mt] = t < q_len;
+        row_pos[mt] = pos0 + min(t, q_len - 1);
+        win_lo[mt] = max(0, row_pos[mt] + 1 - d.window);
+        vis_hi[mt] = t0 + 15 < q_len ? pos0 + t0 : -1;                         // keys in [vis_lo, vis_hi] are seen by every row of the tile
+        vis_lo[mt] = max(0, pos0 + t0 + 16 - d.window);
+        const bf16* q = p.q + ((long)(tok0 + min(t, q_len - 1)) * d.heads + h) * (d.dp + d.rp) + 8 * a;
+#pragma unroll
+        for (int s = 0; s < LX_DS; s++)
+            if (s < ds) qf[mt][s] = *reinterpret_cast<const bf16x8*>(q + 32 * s);
+#pragma unroll
+        for (int s = 0; s < LX_RS; s++)
+            if (s < rs) qf[mt][LX_DS + s] = rotate8(*reinterpret_cast<const bf16x8*>(q + d.dp + 32 * s), 32 * s + 8 * a, d.rot_dims, p.cos_t, p.sin_t, row_pos[mt]);
+    }
+    const int t_hi = min(q_len, tile0 + LATENT_TILE_TOKENS);
+    const int blk_lo = max(0, pos0 + tile0 + 1 - d.window) / 16, blk_hi = (pos0 + t_hi + 15) / 16, nstep = (blk_hi - blk_lo + 3) / 4;
+    auto issue = [&](int st, int buf) {
+        const int i = base + min(blk_lo + 4 * st + wave, blk_hi - 1) - first_blk;      // (past the end: a copy of the last block, masked)
+        bf16* dst = lds_x + (buf * 4 + wave) * BLK;
+        const bf16 *k = x.ke + (long)(i * 16 + b) * x.ldk + h * d.dp + 8 * a, *vr = x.ve + (long)(i * 16 + b) * x.ldv + h * d.vp + 8 * a;
+        const bf16* r = p.pool + (long)x.blocks[i] * 16 * kd + d.kp * 16 + lane * 8;
+#define LX_COPY(src, slot) __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(src), (__attribute__((address_space(3))) void*)(dst + (slot) * 512), 16, 0, 0)
+#pragma unroll
+        for (int s = 0; s < LX_DS; s++)
+            if (s < ds) LX_COPY(k + 32 * s, s);
+#pragma unroll
+        for (int s = 0; s < LX_RS; s++)
+            if (s < rs) LX_COPY(r + s * 512, LX_DS + s);
+#pragma unroll
+        for (int s = 0; s < LX_VS; s++)
+            if (s < vs) LX_COPY(vr + 32 * s, LX_DS + LX_RS + s);
+#undef LX_COPY
+    };
+    const int tr_off = tr_offset(lane);
+    float m_run[MT], l_run[MT];
+    floatx4 o[MT][DT];
+#pragma unroll
+    for (int mt = 0; mt < MT; mt++) {
+        m_run[mt] = -INFINITY; l_run[mt] = 0.f;
+#pragma unroll
+        for (int t = 0; t < DT; t++) o[mt][t] = (floatx4){0.f, 0.f, 0.f, 0.f};
+    }
+    issue(0, 0);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    __syncthreads();
+    for (int st = 0; st < nstep; st++) {
+        const int buf = st & 1;
+        if (st + 1 < nstep) issue(st + 1, buf ^ 1);
+        const bf16* kb = lds_x + buf * 4 * BLK;
+        floatx4 sv[MT][4];
+#pragma unroll
+        for (int mt = 0; mt < MT; mt++)
+#pragma unroll
+            for (int i = 0; i < 4; i++) sv[mt][i] = (floatx4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int s = 0; s < LX_DS + LX_RS; s++)
+            if (s < LX_DS ? s < ds : s - LX_DS < rs) {
+#pragma unroll
+                for (int i = 0; i < 4; i++) {
+                    const bf16x8 k = *reinterpret_cast<const bf16x8*>(kb + i * BLK + s * 512 + lane * 8);
+#pragma unroll
+                    for (int mt = 0; mt < MT; mt++) sv[mt][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k, qf[mt][s], sv[mt][i], 0, 0, 0);
+                }
+            }
+        bf16x8 pf[MT][2];
+        const int key0 = (blk_lo + 4 * st) * 16;
+#pragma unroll
+        for (int mt = 0; mt < MT; mt++) {
+            if (!(key0 + 63 <= vis_hi[mt] && key0 >= vis_lo[mt])) {
+#pragma unroll
+                for (int i = 0; i < 4; i++)
+#pragma unroll
+                    for (int r = 0; r < 4; r++) {
+                        const int key = key0 + i * 16 + 4 * a + r;
+                        if (!(ok[mt] && key <= row_pos[mt] && key >= win_lo[mt])) sv[mt][i][r] = -INFINITY;
+                    }
+            }
+            float mx = -INFINITY;
+#pragma unroll
+            for (int i = 0; i < 4; i++) mx = fmaxf(mx, fmaxf(fmaxf(sv[mt][i][0], sv[mt][i][1]), fmaxf(sv[mt][i][2], sv[mt][i][3])));
+            mx = rows_reduce_max(mx * sl2);                                    // (scale > 0, checked by the caller: the maximum commutes)
+            const float m_new = fmaxf(m_run[mt], mx), m_safe = m_new == -INFINITY ? 0.f : m_new;
+            if (__ballot(m_new != m_run[mt]) != 0) {
+                const float alpha = __builtin_amdgcn_exp2f(m_run[mt] - m_safe);
+#pragma unroll
+                for (int t = 0; t < DT; t++)
+#pragma unroll
+                    for (int r = 0; r < 4; r++) o[mt][t][r] *= alpha;
+                l_run[mt] *= alpha;
+                m_run[mt] = m_new;
+            }
+#pragma unroll
+            for (int i = 0; i < 4; i++)
+#pragma unroll
+                for (int r = 0; r < 4; r++) {
+                    const float e = __builtin_amdgcn_exp2f(__builtin_fmaf(sv[mt][i][r], sl2, -m_safe));
+                    l_run[mt] += e;
+                    pf[mt][i >> 1][(i & 1) * 4 + r] = (bf16)e;
+                }
+        }
+        // contraction index of a 32-key pair: (a, j < 4) = key 4a + j of its first block, (a, j ≥ 4) = key 4a + j − 4 of its second
+#pragma unroll
+        for (int c = 0; c < 2; c++) {
+            const bf16* vb = kb + 2 * c * BLK + (LX_DS + LX_RS) * 512 + tr_off;
+#pragma unroll
+            for (int t = 0; t < DT; t++)
+                if (t < 2 * vs) {
+                    const shortx4 v0 = read_tr(vb + t * 256), v1 = read_tr(vb + BLK + t * 256);
+                    typedef short shortx8 __attribute__((ext_vector_type(8)));
+                    const shortx8 vt = {v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
+#pragma unroll
+                    for (int mt = 0; mt < MT; mt++)
+                        o[mt][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, vt), pf[mt][c], o[mt][t], 0, 0, 0);
+                }
+        }
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        __syncthreads();
+    }
+#pragma unroll
+    for (int mt = 0; mt < MT; mt++) {
+        const float l = rows_reduce_sum(l_run[mt]);
+        if (!ok[mt]) continue;
+        const long tok = tok0 + tile0 + (wave * MT + mt) * 16 + b;
+        const float f = (float)x.gate[tok * x.ld_gate + h] / l;
+        bf16* dst = x.out + (tok * d.heads + h) * d.vp + 4 * a;
+#pragma unroll
+        for (int t = 0; t < DT; t++)
+            if (t < 2 * vs) {
+                bf16x4 y;
+#pragma unroll
+                for (int r = 0; r < 4; r++) y[r] = (bf16)(o[mt][t][r] * f);
+                *reinterpret_cast<bf16x4*>(dst + t * 16) = y;
+            }
+    }
+}
+bool latent_expanded_supports(const LatentDims& d) { return d.dp <= 32 * LX_DS && d.rp <= 32 * LX_RS && d.vp <= 32 * LX_VS && d.scale > 0.f; }
+int latent_attention_expanded(const LatentDims& d, const LatentBuffers<bf16>& b, const BatchView& v, const LatentExpanded& x, hipStream_t s) {
+    FH_REQUIRE(latent_expanded_supports(d), "latent attention: sizes the expanded form does not take");
+    constexpr size_t lds = (size_t)2 * 4 * (LX_DS + LX_RS + LX_VS) * 512 * sizeof(bf16);
+    static bool attr = false;
+    if (!attr) { FH_CHECK_HIP(hipFuncSetAttribute((const void*)latent_expanded_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)); attr = true; }
+    form_hit(FORM_LATENT_ATTN_EXPANDED);
+    hipLaunchKernelGGL(latent_expanded_kernel, dim3(x.nunits, d.heads), dim3(256), lds, s, d, b, v, x);
+    FH_CHECK_LAUNCH();
+    return 0;
 }
 
 template <typename E>
@@ -346,14 +531,14 @@ static int latent_plain(const LatentDims& d, const LatentBuffers<E>& b, const Ba
     return 0;
 }
 static int latent_mfma(const LatentDims& d, const LatentBuffers<bf16>& b, const BatchView& v, hipStream_t s) {
-    const int tiles = (int)(((long)v.T * d.heads) / 16) + v.num_seqs;      // upper bound of Σ ceil(rows / 16)
+    const int tiles = v.single ? v.num_seqs * cdiv(d.heads, 16) : (int)(((long)v.T * d.heads) / 16) + v.num_seqs;      // upper bound of Σ ceil(rows / 16)
     const int keys = std::min(v.max_keys, d.window + 16);
-    // split the keys while the launch has fewer than ≈ 2 workgroups per CU and a split keeps ≥ 128 keys (two blocks per wave)
+    // split the keys while the launch has fewer than ≈ 1 workgroup per CU and a split keeps ≥ 128 keys (two steps)
     int ns = 1;
     while (ns < 16 && tiles * ns < 256 && keys >= 2 * ns * 128) ns *= 2;
     if (knobs().latent_splits > 0) ns = std::min(16, knobs().latent_splits);
     while (ns > 1 && (size_t)tiles * ns * 16 * (d.kp + LATENT_PARTIAL_PAD) * 4 > b.partial_bytes) ns /= 2;
-    const dim3 grid(tiles, ns);
+    const dim3 grid(ns, tiles);          // (splits fastest: the row tiles of a sequence read a key range on the same XCD)
     form_hit(ns > 1 ? FORM_LATENT_ATTN_SPLIT : FORM_LATENT_ATTN);
     if (d.kp <= 64) hipLaunchKernelGGL(latent_attn_kernel<2>, grid, dim3(256), 0, s, d, b, v, ns);
     else if (d.kp <= 128) hipLaunchKernelGGL(latent_attn_kernel<4>, grid, dim3(256), 0, s, d, b, v, ns);
@@ -361,7 +546,7 @@ static int latent_mfma(const LatentDims& d, const LatentBuffers<bf16>& b, const 
     else hipLaunchKernelGGL(latent_attn_kernel<16>, grid, dim3(256), 0, s, d, b, v, ns);
     FH_CHECK_LAUNCH();
     if (ns > 1) {
-        hipLaunchKernelGGL(latent_attn_reduce_kernel, dim3(tiles), dim3(256), 0, s, d, b, v, ns);
+        hipLaunchKernelGGL(latent_attn_reduce_kernel, dim3(tiles, cdiv(16 * (d.kp / 4), 256)), dim3(256), 0, s, d, b, v, ns);
         FH_CHECK_LAUNCH();
     }
     return 0;

@@ -19,6 +19,9 @@ struct BatchView {
     const int32_t* slots = nullptr;              // [num_seqs] recurrent state slot
     const int32_t* units = nullptr;              // [num_units][2] (sequence, first token of the chunk within the batch)
     int num_units = 0;
+    const uint32_t *host_cu = nullptr, *host_pos = nullptr;      // the same arrays and the block tables on the host (portions only)
+    const int32_t* host_bt = nullptr;
+    int long_min = 0;                            // > 0: sequences that bring at least this many tokens are not attended by latent_attention
 };
 
 // ── residual stream (residual_stream.hip) ──
@@ -26,9 +29,9 @@ struct BatchView {
 template <typename E>
 int embed_bigram(const E* table, const E* bigram, int buckets, int64_t mul_prev, int64_t mul_cur, const BatchView& v, float* x, E* xb,
                  int dim, int ldb, hipStream_t s);
-// x += mult · rms(sub · gate) · w (w holds 1 + the stored weight); xb = E(x)
+// x += mult · rms(sub · gate) · w (w holds 1 + the stored weight); xb = E(x); sub is the sum of `slabs` partial sums
 template <typename E>
-int gated_post_norm_add(const float* sub, long ld_sub, const E* gate, long ld_gate, const float* w, float mult, float eps, float* x,
+int gated_post_norm_add(const float* sub, long ld_sub, int slabs, long slab_stride, const E* gate, long ld_gate, const float* w, float mult, float eps, float* x,
                         E* xb, int rows, int dim, int ldb, hipStream_t s);
 // out[i] = E(rms(x[row_idx[i]]) · w)
 template <typename E>
@@ -54,6 +57,20 @@ int latent_prepare(const E* dq, const E* dkv, long ld, const float* dq_norm, con
                    const LatentBuffers<E>& b, const BatchView& v, E* cq, hipStream_t s);
 template <typename E>
 int latent_attention(const LatentDims& d, const LatentBuffers<E>& b, const BatchView& v, hipStream_t s);
+// Portions over expanded keys and values (16-bit): blocks [nblocks] lists the cache blocks whose keys ke [16·nblocks][heads·dp] and
+// values ve [16·nblocks][heads·vp] were expanded; units [nunits][4] = (sequence, first token of the tile within the portion, index in
+// `blocks` of the sequence's first listed block, that block's number in the sequence).  out [T][heads·vp], times the head gate.
+struct LatentExpanded {
+    const int32_t *blocks = nullptr, *units = nullptr;
+    int nblocks = 0, nunits = 0;
+    const bf16 *ke = nullptr, *ve = nullptr;
+    long ldk = 0, ldv = 0;
+    const bf16* gate = nullptr; long ld_gate = 0;
+    bf16* out = nullptr;
+};
+constexpr int LATENT_TILE_TOKENS = 128;          // tokens of a portion per workgroup
+bool latent_expanded_supports(const LatentDims& d);
+int latent_attention_expanded(const LatentDims& d, const LatentBuffers<bf16>& b, const BatchView& v, const LatentExpanded& x, hipStream_t s);
 
 // ── real-gated linear recurrent unit (rglru.hip) ──
 // Channels live in a block-padded layout: blocks · bp with bp = pad32(width / blocks); padded channels are zero throughout.

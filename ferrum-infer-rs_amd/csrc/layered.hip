@@ -7,6 +7,7 @@
 // section with its own activation in the epilogue:
 //     latent attention : [gate σ | q latent | kv latent + shared key part | head gates σ] → norms, rotation, cache write → query up-projection
 //                        → query through W_ukᵀ (per head) → attention over the latents → W_uv (per head, × head gate) → W_o → add + norm
+//                        (long portions: keys and values of the visible cache blocks expanded → flash attention × head gate → W_o)
 //     linear recurrence: [gate σ | y gelu | x] → convolution → gates + state (one token) or scan (portions) → W_o → add + norm
 //     feed-forward     : [gate σ | up xIELU] → down → add + norm
 #include <math.h>
@@ -77,7 +78,7 @@ class Layered final : public LayeredModel {
     struct Layer {
         FerrumHipLayerSpec s;
         // fused input projection of the mixer: sections in the order of the comment at the top
-        Linear in, uq, uk, uv, o, ff_in, down;
+        Linear in, uq, uk, uv, expand, o, ff_in, down;
         GemmSection in_sec[GEMM_MAX_SECTIONS], ff_sec[2];
         int in_nsec = 0;
         int c0 = 0, c1 = 0, c2 = 0;        // columns of the mixer's sections: latent attention: q latent, kv latent, head gates; recurrence: y, x
@@ -94,6 +95,7 @@ public:
         : c_(c), lc_(lc), slots_(slots), D_(c.hidden), Dp_(pad32(c.hidden)) {
         for (int i = 0; i < c.num_layers; i++) { Layer L; L.s = layers[i]; dims(L); layers_.push_back(L); }
     }
+    ~Layered() override { if (plan_host_) (void)hipHostFree(plan_host_); }
     bool has_state() const override {
         return std::any_of(layers_.begin(), layers_.end(), [](const Layer& L) { return L.s.mixer == FERRUM_HIP_MIXER_RGLRU; });
     }
@@ -146,8 +148,15 @@ public:
                 const int dim = sp.dim, kr = d.kv_rank, vd = d.vdim;
                 FH_TRY(pack_fn(&L.uk, H, d.kp, d.dp, m + "uk", [&](const float* w, int g, int n, int k) {
                     return n < kr && k < dim ? w[((size_t)g * dim + k) * kr + n] : 0.f; }));
-                FH_TRY(pack_fn(&L.uv, H, d.vp, d.kp, m + "uv", [&](const float* w, int g, int n, int k) {
-                    return n < vd && k < kr ? w[((size_t)g * vd + n) * kr + k] : 0.f; }));
+                // [W_uk | W_uv] over the latent: the expansion of keys and values; its second part doubles as the per-head value projection
+                const float *uk = data(m + "uk"), *uv = data(m + "uv");
+                const int kn = H * d.dp, dp = d.dp, vpad = d.vp;
+                FH_TRY(pack_fn(&L.expand, 1, kn + H * d.vp, d.kp, m + "uv", [&](const float*, int, int n, int k) {
+                    if (k >= kr) return 0.f;
+                    if (n < kn) return n % dp < dim ? uk[((size_t)(n / dp) * dim + n % dp) * kr + k] : 0.f;
+                    n -= kn;
+                    return n % vpad < vd ? uv[((size_t)(n / vpad) * vd + n % vpad) * kr + k] : 0.f; }));
+                L.uv.w = L.expand.w + (size_t)kn * d.kp; L.uv.n = d.vp; L.uv.k = d.kp; L.uv.groups = H;
                 FH_TRY(need(m + "o", {D_, (int64_t)H * vd}));
                 const int vp = d.vp;
                 FH_TRY(pack_fn(&L.o, 1, Dp_, H * vp, m + "o", [&](const float* w, int, int n, int k) {
@@ -233,7 +242,7 @@ public:
         FH_TRY(arena_.alloc(&x_, T * D_));
         FH_TRY(arena_.alloc(&xb_, T * Dp_));
         FH_TRY(arena_.alloc(&in_, T * in_cols));
-        FH_TRY(arena_.alloc(&sub_, T * Dp_));
+        FH_TRY(arena_.alloc(&sub_, std::max<size_t>(T, (size_t)GEMM_MAX_SLABS * std::min<size_t>(T, 64)) * Dp_));
         FH_TRY(arena_.alloc(&cq_, T * cq_cols));
         FH_TRY(arena_.alloc(&q_, T * q_cols));
         FH_TRY(arena_.alloc(&q_lat_, T * lat_cols));
@@ -248,6 +257,7 @@ public:
         FH_TRY(arena_.alloc(&chunk_a_, units * rnn_cols));
         FH_TRY(arena_.alloc(&chunk_h_, units * rnn_cols));
         FH_TRY(arena_.alloc(&head_in_, (size_t)c_.max_seqs * Dp_));
+        FH_TRY(finalize_expansion());
         for (Layer& L : layers_) {
             L.lb.q = q_; L.lb.q_lat = q_lat_; L.lb.o_lat = o_lat_; L.lb.partial = partial_; L.lb.partial_bytes = partial_bytes_;
             L.rb.x = in_ + L.c1; L.rb.y = in_ + L.c0; L.rb.ld = L.in.n;
@@ -266,7 +276,12 @@ public:
     } while (0)
         int li = -1;
         const int T = v.T;
+        BatchView ve = v;
+        const bool any_short = plan_expansion(&ve);
+        if (ve.long_min > 0)
+            FH_CHECK_HIP(hipMemcpyAsync(plan_dev_, plan_host_, plan_used_ * 4, hipMemcpyHostToDevice, s));
         const float eps = c_.rms_eps;
+        int slabs = 1;
         RUN(embed_bigram<E>(embed_, bigram_, lc_.bigram_buckets, lc_.bigram_mul_prev, lc_.bigram_mul_cur, v, x_, xb_, D_, Dp_, s));
         for (li = 0; li < c_.num_layers; li++) {
             Layer& L = layers_[li];
@@ -278,25 +293,28 @@ public:
                 const LatentDims& d = L.ld;
                 RUN(latent_prepare<E>(in_ + L.c0, in_ + L.c1, L.in.n, L.dq_norm, L.dkv_norm, eps, d, L.lb, v, cq_, s));
                 RUN(tiled_gemm(linear(L.uq, cq_, d.qp, T, q_, L.uq.n), s));
-                TiledGemm<E> k = linear(L.uk, q_, L.uq.n, T, q_lat_, (long)d.heads * d.kp);
-                k.x_group = d.dp + d.rp; k.out_group = d.kp;
-                RUN(tiled_gemm(k, s));
-                RUN(latent_attention<E>(d, L.lb, v, s));
-                TiledGemm<E> u = linear(L.uv, o_lat_, (long)d.heads * d.kp, T, attn_, (long)d.heads * d.vp);
-                u.x_group = d.kp; u.out_group = d.vp; u.row_scale = in_ + L.c2; u.ld_scale = L.in.n;
-                RUN(tiled_gemm(u, s));
-                RUN(tiled_gemm(linear_f32(L.o, attn_, (long)d.heads * d.vp, T, sub_, Dp_), s));
+                if (any_short) {
+                    TiledGemm<E> k = linear(L.uk, q_, L.uq.n, T, q_lat_, (long)d.heads * d.kp);
+                    k.x_group = d.dp + d.rp; k.out_group = d.kp;
+                    RUN(tiled_gemm(k, s));
+                    RUN(latent_attention<E>(d, L.lb, ve, s));
+                    TiledGemm<E> u = linear(L.uv, o_lat_, (long)d.heads * d.kp, T, attn_, (long)d.heads * d.vp);
+                    u.x_group = d.kp; u.out_group = d.vp; u.row_scale = in_ + L.c2; u.ld_scale = L.in.n;
+                    RUN(tiled_gemm(u, s));
+                }
+                if (ve.long_min > 0) RUN(attend_expanded(L, v, s));        // (writes the rows of the long portions only)
+                RUN(tiled_gemm(linear_slabs(L.o, attn_, (long)d.heads * d.vp, T, &slabs), s));
             } else {
                 RUN(rglru_forward<E>(L.rd, L.rb, v, s));
-                RUN(tiled_gemm(linear_f32(L.o, rnn_out_, L.rd.wp, T, sub_, Dp_), s));
+                RUN(tiled_gemm(linear_slabs(L.o, rnn_out_, L.rd.wp, T, &slabs), s));
             }
-            RUN(gated_post_norm_add<E>(sub_, Dp_, in_, L.in.n, L.norm1, lc_.residual_mult, eps, x_, xb_, T, D_, Dp_, s));
+            RUN(gated_post_norm_add<E>(sub_, Dp_, slabs, (long)T * Dp_, in_, L.in.n, L.norm1, lc_.residual_mult, eps, x_, xb_, T, D_, Dp_, s));
             if (L.s.ff != FERRUM_HIP_FF_NONE) {
                 TiledGemm<E> f = linear(L.ff_in, xb_, Dp_, T, in_, L.ff_in.n);
                 f.nsec = 2; f.sec[0] = L.ff_sec[0]; f.sec[1] = L.ff_sec[1];
                 RUN(tiled_gemm(f, s));
-                RUN(tiled_gemm(linear_f32(L.down, in_ + Dp_, L.ff_in.n, T, sub_, Dp_), s));
-                RUN(gated_post_norm_add<E>(sub_, Dp_, in_, L.ff_in.n, L.norm2, lc_.residual_mult, eps, x_, xb_, T, D_, Dp_, s));
+                RUN(tiled_gemm(linear_slabs(L.down, in_ + Dp_, L.ff_in.n, T, &slabs), s));
+                RUN(gated_post_norm_add<E>(sub_, Dp_, slabs, (long)T * Dp_, in_, L.ff_in.n, L.norm2, lc_.residual_mult, eps, x_, xb_, T, D_, Dp_, s));
             }
             if (taps) FH_CHECK_HIP(hipMemcpyAsync(taps + (size_t)li * c_.max_tokens * D_, x_, (size_t)T * D_ * 4, hipMemcpyDeviceToDevice, s));
         }
@@ -328,6 +346,82 @@ private:
     static TiledGemm<E> linear_f32(const Linear& w, const E* x, long ldx, int m, float* out, long ldo) {
         TiledGemm<E> g = linear(w, x, ldx, m, nullptr, ldo);
         g.out_f32 = out;
+        return g;
+    }
+
+    // ── portions over expanded keys and values (16-bit models) ──
+    // Every latent layer must take the form, so one decision per sequence serves the whole forward.
+    int finalize_expansion() {
+        if (sizeof(E) != 2) return 0;
+        long cols = 0;
+        int widest = 0;
+        for (const Layer& L : layers_)
+            if (L.s.mixer == FERRUM_HIP_MIXER_LATENT_ATTENTION) {
+                if (!latent_expanded_supports(L.ld)) return 0;
+                cols = std::max<long>(cols, L.expand.n);
+                widest = std::max(widest, L.ld.window);
+                if (std::none_of(plans_.begin(), plans_.end(), [&](const Plan& q) { return q.window == L.ld.window; })) plans_.push_back(Plan{L.ld.window});
+            }
+        if (plans_.empty()) return 0;
+        const long per_seq = std::min<long>(widest, c_.max_seq_len) / 16 + 2;
+        expand_blocks_ = (int)std::min<long>((c_.max_tokens + 15) / 16 + c_.max_seqs * per_seq, std::max(c_.kv_num_blocks, 1));
+        const size_t ints = plans_.size() * ((size_t)expand_blocks_ + 4 * ((size_t)c_.max_tokens / LATENT_TILE_TOKENS + c_.max_seqs));
+        FH_TRY(arena_.alloc(&expanded_, (size_t)expand_blocks_ * 16 * cols));
+        FH_TRY(arena_.alloc(&plan_dev_, ints));
+        FH_CHECK_HIP(hipHostMalloc((void**)&plan_host_, ints * 4, hipHostMallocDefault));
+        return 0;
+    }
+    // Which cache blocks to expand and which tiles to run, per distinct window.  Sets v->long_min when some sequence takes the form;
+    // returns whether any does not.
+    bool plan_expansion(BatchView* v) {
+        const int min_rows = knobs().latent_expand_min_rows;
+        if (v->single || !plan_host_ || min_rows <= 0 || knobs().latent_plain) return true;
+        bool any_short = false, any_long = false;
+        plan_used_ = 0;
+        for (Plan& q : plans_) {
+            q.blocks0 = plan_used_;
+            q.nblocks = q.nunits = 0;
+            std::vector<int32_t> units;
+            for (int i = 0; i < v->num_seqs; i++) {
+                const int n = (int)(v->host_cu[i + 1] - v->host_cu[i]), pos = (int)v->host_pos[i];
+                if (n < min_rows) { any_short = true; continue; }
+                any_long = true;
+                const int lo = std::max(0, pos + 1 - q.window) / 16, hi = (pos + n + 15) / 16;
+                if (q.nblocks + hi - lo > expand_blocks_) return true;           // (shared prefix blocks listed more often than the pool holds)
+                for (int t = 0; t < n; t += LATENT_TILE_TOKENS) units.insert(units.end(), {i, t, q.nblocks, lo});
+                for (int b = lo; b < hi; b++) plan_host_[plan_used_++] = v->host_bt[(size_t)i * v->max_blocks + b];
+                q.nblocks += hi - lo;
+            }
+            q.units0 = plan_used_;
+            q.nunits = (int)units.size() / 4;
+            std::copy(units.begin(), units.end(), plan_host_ + plan_used_);
+            plan_used_ += units.size();
+        }
+        if (any_long) v->long_min = min_rows;
+        return any_short;
+    }
+    int attend_expanded(Layer& L, const BatchView& v, hipStream_t s) {
+        if constexpr (sizeof(E) == 2) {
+            const Plan& q = *std::find_if(plans_.begin(), plans_.end(), [&](const Plan& x) { return x.window == L.ld.window; });
+            const LatentDims& d = L.ld;
+            TiledGemm<E> g = linear(L.expand, L.lb.pool, 0, q.nblocks * 16, expanded_, L.expand.n);
+            g.x_blocks = plan_dev_ + q.blocks0; g.x_block_elems = (long)latent_block_elems(d);
+            FH_TRY(tiled_gemm(g, s));
+            LatentExpanded x;
+            x.blocks = plan_dev_ + q.blocks0; x.units = plan_dev_ + q.units0; x.nblocks = q.nblocks; x.nunits = q.nunits;
+            x.ke = expanded_; x.ve = expanded_ + (size_t)d.heads * d.dp; x.ldk = x.ldv = L.expand.n;
+            x.gate = in_ + L.c2; x.ld_gate = L.in.n; x.out = attn_;
+            return latent_attention_expanded(d, L.lb, v, x, s);
+        }
+        return 0;
+    }
+    struct Plan { int window; size_t blocks0 = 0, units0 = 0; int nblocks = 0, nunits = 0; };
+
+    // projection whose consumer is the residual update: partial sums over K, as many as fill the chip
+    TiledGemm<E> linear_slabs(const Linear& w, const E* x, long ldx, int m, int* slabs) const {
+        TiledGemm<E> g = linear_f32(w, x, ldx, m, sub_, Dp_);
+        g.slabs = *slabs = tiled_gemm_slabs(m, w.n, w.k);
+        g.slab_stride = (long)m * Dp_;
         return g;
     }
 
@@ -464,6 +558,12 @@ private:
     E *xb_ = nullptr, *in_ = nullptr, *cq_ = nullptr, *q_ = nullptr, *q_lat_ = nullptr, *o_lat_ = nullptr, *attn_ = nullptr, *u_ = nullptr,
       *rnn_out_ = nullptr, *head_in_ = nullptr;
     size_t partial_bytes_ = 0;
+    // expansion of keys and values: one plan per distinct window
+    std::vector<Plan> plans_;
+    int32_t *plan_host_ = nullptr, *plan_dev_ = nullptr;
+    size_t plan_used_ = 0;
+    int expand_blocks_ = 0;
+    E* expanded_ = nullptr;
 };
 
 }  // namespace

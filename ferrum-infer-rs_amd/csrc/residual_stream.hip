@@ -4,7 +4,7 @@
 
 namespace fh {
 
-template <typename E>
+template <typename E, bool VEC>
 __global__ __launch_bounds__(256) void embed_bigram_kernel(const E* __restrict__ table, const E* __restrict__ bigram, int buckets,
                                                            int64_t mul_prev, int64_t mul_cur, BatchView v, float* __restrict__ x,
                                                            E* __restrict__ xb, int dim, int ldb) {
@@ -15,6 +15,21 @@ __global__ __launch_bounds__(256) void embed_bigram_kernel(const E* __restrict__
         const int seq = v.tok_seq[t];
         const int64_t prev = t == (int)v.cu[seq] ? (int64_t)v.prev[seq] : (int64_t)v.tokens[t - 1];
         row = prev < 0 ? buckets : (long)((uint64_t)(prev * mul_prev + (int64_t)tok * mul_cur) % (uint64_t)buckets);
+    }
+    if (VEC) {
+        typedef typename Frag<E>::v8 v8;
+        for (int i = threadIdx.x * 8; i < dim; i += 2048) {
+            const v8 e = *reinterpret_cast<const v8*>(table + (long)tok * dim + i);
+            v8 g = e, o;
+            if (bigram) g = *reinterpret_cast<const v8*>(bigram + row * dim + i);
+            floatx4 f[2];
+#pragma unroll
+            for (int j = 0; j < 8; j++) { f[j >> 2][j & 3] = (float)e[j] + (bigram ? (float)g[j] : 0.f); o[j] = (E)f[j >> 2][j & 3]; }
+            *reinterpret_cast<floatx4*>(x + (long)t * dim + i) = f[0];
+            *reinterpret_cast<floatx4*>(x + (long)t * dim + i + 4) = f[1];
+            *reinterpret_cast<v8*>(xb + (long)t * ldb + i) = o;
+        }
+        return;
     }
     for (int i = threadIdx.x; i < dim; i += 256) {
         float e = (float)table[(long)tok * dim + i];
@@ -27,7 +42,10 @@ __global__ __launch_bounds__(256) void embed_bigram_kernel(const E* __restrict__
 template <typename E>
 int embed_bigram(const E* table, const E* bigram, int buckets, int64_t mul_prev, int64_t mul_cur, const BatchView& v, float* x, E* xb,
                  int dim, int ldb, hipStream_t s) {
-    hipLaunchKernelGGL(embed_bigram_kernel<E>, dim3(v.T), dim3(256), 0, s, table, bigram, buckets, mul_prev, mul_cur, v, x, xb, dim, ldb);
+    if (dim % 8 == 0)
+        hipLaunchKernelGGL((embed_bigram_kernel<E, true>), dim3(v.T), dim3(256), 0, s, table, bigram, buckets, mul_prev, mul_cur, v, x, xb, dim, ldb);
+    else
+        hipLaunchKernelGGL((embed_bigram_kernel<E, false>), dim3(v.T), dim3(256), 0, s, table, bigram, buckets, mul_prev, mul_cur, v, x, xb, dim, ldb);
     FH_CHECK_LAUNCH();
     return 0;
 }
@@ -43,7 +61,7 @@ __device__ __forceinline__ float block_sum(float q, float* red) {
 
 // One workgroup per row; a thread holds up to 4 quads of the row in registers, so the branch is read once.
 template <typename E, bool VEC>
-__global__ __launch_bounds__(1024) void gated_post_norm_add_kernel(const float* __restrict__ sub, long ld_sub, const E* __restrict__ gate,
+__global__ __launch_bounds__(1024) void gated_post_norm_add_kernel(const float* __restrict__ sub, long ld_sub, int slabs, long slab_stride, const E* __restrict__ gate,
                                                                    long ld_gate, const float* __restrict__ w, float mult, float eps,
                                                                    float* __restrict__ x, E* __restrict__ xb, int dim, int ldb) {
     __shared__ float red[16];
@@ -61,6 +79,7 @@ __global__ __launch_bounds__(1024) void gated_post_norm_add_kernel(const float* 
             const int i = (c * blockDim.x + threadIdx.x) * 4;
             if (i < dim) {
                 v[c] = *reinterpret_cast<const floatx4*>(sr + i);
+                for (int z = 1; z < slabs; z++) v[c] += *reinterpret_cast<const floatx4*>(sr + z * slab_stride + i);
                 const e4 gv = *reinterpret_cast<const e4*>(gr + i);
                 xv[c] = *reinterpret_cast<const floatx4*>(xr + i);
                 wv[c] = *reinterpret_cast<const floatx4*>(w + i);
@@ -82,24 +101,29 @@ __global__ __launch_bounds__(1024) void gated_post_norm_add_kernel(const float* 
         }
         return;
     }
-    for (int i = threadIdx.x; i < dim; i += blockDim.x) { const float t = sr[i] * (float)gr[i]; q += t * t; }
+    auto branch = [&](int i) {
+        float t = sr[i];
+        for (int z = 1; z < slabs; z++) t += sr[z * slab_stride + i];
+        return t * (float)gr[i];
+    };
+    for (int i = threadIdx.x; i < dim; i += blockDim.x) { const float t = branch(i); q += t * t; }
     const float inv = mult / sqrtf(block_sum(q, red) / (float)dim + eps);
     for (int i = threadIdx.x; i < dim; i += blockDim.x) {
-        const float t = xr[i] + sr[i] * (float)gr[i] * inv * w[i];
+        const float t = xr[i] + branch(i) * inv * w[i];
         xr[i] = t;
         br[i] = (E)t;
     }
 }
 
 template <typename E>
-int gated_post_norm_add(const float* sub, long ld_sub, const E* gate, long ld_gate, const float* w, float mult, float eps, float* x,
+int gated_post_norm_add(const float* sub, long ld_sub, int slabs, long slab_stride, const E* gate, long ld_gate, const float* w, float mult, float eps, float* x,
                         E* xb, int rows, int dim, int ldb, hipStream_t s) {
     const int threads = rows <= 512 && dim >= 2048 ? 1024 : 256;
-    const bool vec = dim % 4 == 0 && dim <= threads * 16 && ld_sub % 4 == 0 && ld_gate % 4 == 0 && ldb % 4 == 0;
+    const bool vec = dim % 4 == 0 && dim <= threads * 16 && ld_sub % 4 == 0 && ld_gate % 4 == 0 && ldb % 4 == 0 && slab_stride % 4 == 0;
     if (vec)
-        hipLaunchKernelGGL((gated_post_norm_add_kernel<E, true>), dim3(rows), dim3(threads), 0, s, sub, ld_sub, gate, ld_gate, w, mult, eps, x, xb, dim, ldb);
+        hipLaunchKernelGGL((gated_post_norm_add_kernel<E, true>), dim3(rows), dim3(threads), 0, s, sub, ld_sub, slabs, slab_stride, gate, ld_gate, w, mult, eps, x, xb, dim, ldb);
     else
-        hipLaunchKernelGGL((gated_post_norm_add_kernel<E, false>), dim3(rows), dim3(threads), 0, s, sub, ld_sub, gate, ld_gate, w, mult, eps, x, xb, dim, ldb);
+        hipLaunchKernelGGL((gated_post_norm_add_kernel<E, false>), dim3(rows), dim3(threads), 0, s, sub, ld_sub, slabs, slab_stride, gate, ld_gate, w, mult, eps, x, xb, dim, ldb);
     FH_CHECK_LAUNCH();
     return 0;
 }
@@ -123,7 +147,7 @@ int rms_norm_rows(const float* x, const int32_t* row_idx, const float* w, float 
 
 #define INSTANTIATE(E)                                                                                                                  \
     template int embed_bigram<E>(const E*, const E*, int, int64_t, int64_t, const BatchView&, float*, E*, int, int, hipStream_t);        \
-    template int gated_post_norm_add<E>(const float*, long, const E*, long, const float*, float, float, float*, E*, int, int, int,       \
+    template int gated_post_norm_add<E>(const float*, long, int, long, const E*, long, const float*, float, float, float*, E*, int, int, int,       \
                                         hipStream_t);                                                                                   \
     template int rms_norm_rows<E>(const float*, const int32_t*, const float*, float, E*, int, int, int, hipStream_t);
 INSTANTIATE(bf16)

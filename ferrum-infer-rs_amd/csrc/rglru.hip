@@ -5,7 +5,7 @@
 //
 // The two gate projections of a channel are computed side by side on the matrix cores (tiles interleaved ra, ri), so one lane holds
 // both gates of its (token, channel) and everything from the sigmoids to the state update stays in fp32 registers.  1 − a² is taken as
-// −expm1(2 log a).  One token per sequence: that launch also updates the state and writes the output.  Portions: decay and drive go to
+// 1 − e^(2 log a) by a series where it would cancel.  One token per sequence: that launch also updates the state and writes the output.  Portions: decay and drive go to
 // memory and a chunked scan (64 tokens per workgroup; chunk totals, carry over chunks, final pass) produces the output.
 // A sequence's first token starts from zero whatever its slot holds, so slots are reused without clearing.
 #include "common.h"
@@ -14,39 +14,57 @@
 
 namespace fh {
 
-// value of the convolution's input `back` tokens before token t of its portion (t counts from the portion's start)
+// 8 channels of the convolution's input `back` tokens before token t of its portion (t counts from the portion's start)
 template <typename E>
-__device__ __forceinline__ float conv_input(const RglruBuffers<E>& p, const RglruDims& d, int tok0, int t, int back, int slot, bool fresh, int c) {
+__device__ __forceinline__ typename Frag<E>::v8 conv_input(const RglruBuffers<E>& p, const RglruDims& d, int tok0, int t, int back, int slot, bool fresh, int c) {
+    typedef typename Frag<E>::v8 v8;
     const int q = t - back;
-    if (q >= 0) return (float)p.x[(long)(tok0 + q) * p.ld + c];
-    if (fresh) return 0.f;                              // (a fresh sequence has no tokens before its portion)
-    return (float)p.conv_state[((long)slot * (d.taps - 1) + (d.taps - 1 + q)) * d.wp + c];
+    if (q >= 0) return *reinterpret_cast<const v8*>(p.x + (long)(tok0 + q) * p.ld + c);
+    if (!fresh) return *reinterpret_cast<const v8*>(p.conv_state + ((long)slot * (d.taps - 1) + (d.taps - 1 + q)) * d.wp + c);
+    v8 z;                                               // (a fresh sequence has no tokens before its portion)
+#pragma unroll
+    for (int j = 0; j < 8; j++) z[j] = (E)0.f;
+    return z;
 }
 
-// one thread per (token, channel); with one token per sequence the thread also shifts the channel's stored inputs
+// one thread per (token, 8 channels); with one token per sequence the thread also shifts the channels' stored inputs
 template <typename E>
 __global__ __launch_bounds__(256) void rglru_conv_kernel(RglruDims d, RglruBuffers<E> p, BatchView v) {
-    const int c = blockIdx.x * 256 + threadIdx.x, tok = blockIdx.y;
-    if (c >= d.wp) return;
+    typedef typename Frag<E>::v8 v8;
+    const int id = blockIdx.x * 256 + threadIdx.x, per = d.wp >> 3, tok = id / per, c = (id % per) * 8;
+    if (tok >= v.T) return;
     const int seq = v.tok_seq[tok], tok0 = v.cu[seq], slot = v.slots[seq];
     const bool fresh = v.pos[seq] == 0;
-    float acc = p.conv_b[c];
-    for (int j = 0; j < d.taps; j++) acc += p.conv_w[j * d.wp + c] * conv_input(p, d, tok0, tok - tok0, d.taps - 1 - j, slot, fresh, c);
-    p.u[(long)tok * d.wp + c] = (E)acc;
+    float acc[8];
+#pragma unroll
+    for (int k = 0; k < 8; k++) acc[k] = p.conv_b[c + k];
+    for (int j = 0; j < d.taps; j++) {
+        const v8 in = conv_input(p, d, tok0, tok - tok0, d.taps - 1 - j, slot, fresh, c);
+#pragma unroll
+        for (int k = 0; k < 8; k++) acc[k] += p.conv_w[(long)j * d.wp + c + k] * (float)in[k];
+    }
+    v8 o;
+#pragma unroll
+    for (int k = 0; k < 8; k++) o[k] = (E)acc[k];
+    *reinterpret_cast<v8*>(p.u + (long)tok * d.wp + c) = o;
     if (v.single)
-        for (int j = 0; j < d.taps - 1; j++) {          // entry j is the input taps − 2 − j tokens back; read before it is overwritten
-            const float in = conv_input(p, d, tok0, 0, d.taps - 2 - j, slot, fresh, c);
-            p.conv_state[((long)slot * (d.taps - 1) + j) * d.wp + c] = (E)in;
-        }
+        for (int j = 0; j < d.taps - 1; j++)            // entry j is the input taps − 2 − j tokens back; read before it is overwritten
+            *reinterpret_cast<v8*>(p.conv_state + ((long)slot * (d.taps - 1) + j) * d.wp + c) = conv_input(p, d, tok0, 0, d.taps - 2 - j, slot, fresh, c);
 }
 
-// grid (tile groups, row blocks, blocks of the block-diagonal projections); a wave owns one 16-channel tile (ra and ri)
+// σ and −expm1 to fp32 rounding with the hardware exponential, reciprocal and square root (a few units in the last place)
+__device__ __forceinline__ float gate_sigmoid(float z) { return __builtin_amdgcn_rcpf(1.0f + __expf(-z)); }
+// 1 − e^t, t ≤ 0: series below 1/4, where the difference would cancel
+__device__ __forceinline__ float one_minus_exp(float t) {
+    const float series = -t * (1.0f + t * (0.5f + t * (1.0f / 6.0f + t * (1.0f / 24.0f + t * (1.0f / 120.0f + t * (1.0f / 720.0f + t * (1.0f / 5040.0f)))))));
+    return t > -0.25f ? series : 1.0f - __expf(t);
+}
+
+// grid (tiles, row blocks, blocks of the block-diagonal projections); a wave owns one 16-channel tile (ra and ri)
 template <typename E, int MT, bool STEP>
-__global__ __launch_bounds__(256) void rglru_gates_kernel(RglruDims d, RglruBuffers<E> p, BatchView v) {
+__global__ __launch_bounds__(64) void rglru_gates_kernel(RglruDims d, RglruBuffers<E> p, BatchView v) {
     typedef typename Frag<E>::v8 v8;
-    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, a = lane >> 4, b = lane & 15;
-    const int tile = blockIdx.x * 4 + wave, rb = blockIdx.y, g = blockIdx.z;
-    if (tile * 16 >= d.bp) return;
+    const int lane = threadIdx.x, a = lane >> 4, b = lane & 15, tile = blockIdx.x, rb = blockIdx.y, g = blockIdx.z;
     const int ksteps = d.bp >> 5;
     const E* xrow[MT];
 #pragma unroll
@@ -76,9 +94,9 @@ __global__ __launch_bounds__(256) void rglru_gates_kernel(RglruDims d, RglruBuff
         for (int q = 0; q < 4; q++) {
             const int row = (rb * MT + mt) * 16 + 4 * a + q;
             if (row >= v.T) continue;
-            const float r = sigmoid_f32(acc[mt][0][q] + bra), in = sigmoid_f32(acc[mt][1][q] + bri);
-            const float log_a = -8.0f * r * sp, decay = expf(log_a);
-            const float drive = sqrtf(fmaxf(0.f, -expm1f(2.0f * log_a))) * in * (float)p.u[(long)row * d.wp + c];
+            const float r = gate_sigmoid(acc[mt][0][q] + bra), in = gate_sigmoid(acc[mt][1][q] + bri);
+            const float log_a = -8.0f * r * sp, decay = __expf(log_a);
+            const float drive = __builtin_amdgcn_sqrtf(one_minus_exp(2.0f * log_a)) * in * (float)p.u[(long)row * d.wp + c];
             if (STEP) {
                 float* st = p.state + (long)v.slots[row] * d.wp + c;       // (token i belongs to sequence i)
                 const float h = v.pos[row] == 0 ? drive : decay * *st + drive;
@@ -148,21 +166,21 @@ __global__ __launch_bounds__(256) void rglru_apply_kernel(RglruDims d, RglruBuff
     }
     if (t0 + n < end) return;
     p.state[(long)slot * d.wp + c] = h;
-    for (int j = 0; j < d.taps - 1; j++) {
-        const float in = conv_input(p, d, tok0, end - 1 - tok0, d.taps - 2 - j, slot, fresh, c);
-        p.conv_state[((long)slot * (d.taps - 1) + j) * d.wp + c] = (E)in;
-    }
+    if (c & 7) return;
+    for (int j = 0; j < d.taps - 1; j++)
+        *reinterpret_cast<typename Frag<E>::v8*>(p.conv_state + ((long)slot * (d.taps - 1) + j) * d.wp + c) =
+            conv_input(p, d, tok0, end - 1 - tok0, d.taps - 2 - j, slot, fresh, c);
 }
 
 template <typename E>
 int rglru_forward(const RglruDims& d, const RglruBuffers<E>& b, const BatchView& v, hipStream_t s) {
     const int cb = cdiv(d.wp, 256);
-    hipLaunchKernelGGL(rglru_conv_kernel<E>, dim3(cb, v.T), dim3(256), 0, s, d, b, v);
+    hipLaunchKernelGGL(rglru_conv_kernel<E>, dim3(cdiv((long)v.T * (d.wp / 8), 256)), dim3(256), 0, s, d, b, v);
     FH_CHECK_LAUNCH();
     const int mt = v.T <= 16 ? 1 : (v.T <= 32 ? 2 : 4);
-    const dim3 grid(cdiv(d.bp / 16, 4), cdiv(v.T, 16 * mt), d.blocks);
+    const dim3 grid(d.bp / 16, cdiv(v.T, 16 * mt), d.blocks);
     form_hit(v.single ? FORM_RGLRU_STEP : FORM_RGLRU_SCAN);
-#define GATES(MT, ST) hipLaunchKernelGGL((rglru_gates_kernel<E, MT, ST>), grid, dim3(256), 0, s, d, b, v)
+#define GATES(MT, ST) hipLaunchKernelGGL((rglru_gates_kernel<E, MT, ST>), grid, dim3(64), 0, s, d, b, v)
     if (v.single) { if (mt == 1) GATES(1, true); else if (mt == 2) GATES(2, true); else GATES(4, true); }
     else { if (mt == 1) GATES(1, false); else if (mt == 2) GATES(2, false); else GATES(4, false); }
 #undef GATES

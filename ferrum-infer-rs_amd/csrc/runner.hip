@@ -646,6 +646,16 @@ static int synth_w4(W4Device* w, int k, int n, int E, bool fused, uint64_t seed,
     return 0;
 }
 
+static int synth_f16t(W4Device* w, int k, int n, uint64_t seed, hipStream_t s) {
+    free_w4(*w);
+    w->k = k; w->n = n; w->n64 = (n + 63) / 64; w->G = k / 128; w->num_experts = 1;
+    const long elems = (long)f16t_elems(n, k);
+    FH_CHECK_HIP(hipMalloc((void**)&w->f16t, elems * 2));
+    hipLaunchKernelGGL(synth_f16_normal_kernel, dim3(cdiv(elems, 256)), dim3(256), 0, s, w->f16t, elems, seed, 1.0f / sqrtf((float)k));
+    FH_CHECK_LAUNCH();
+    return 0;
+}
+
 int ferrum_hip_model_init_synthetic(FerrumHipModel* m, uint64_t seed) {
     FH_REQUIRE(m && !m->finalized, "model_init_synthetic: bad state");
     if (m->layered) return m->layered->init_synthetic(seed, m->stream);
@@ -661,6 +671,9 @@ int ferrum_hip_model_init_synthetic(FerrumHipModel* m, uint64_t seed) {
         hipLaunchKernelGGL(synth_f16_normal_kernel, dim3(cdiv(n, 256)), dim3(256), 0, s, *p, n, sd, std);
         return 0;
     };
+    // development (FERRUM_HIP_SYNTH_DENSE=1, dense MLP models): unquantised fp16 projections instead of INT4 ones
+    const char* sd = getenv("FERRUM_HIP_SYNTH_DENSE");
+    const bool synth_dense = sd && atoi(sd) && c.num_experts == 0;
     const long vh = (long)c.vocab * c.hidden;
     if (int rc = alloc_normal(&m->embed, vh, seed ^ 0xe0bedull, 0.02f)) return rc;
     if (int rc = alloc_normal(&m->lm_head, vh, seed ^ 0x1a4eadull, 0.02f)) return rc;
@@ -681,6 +694,13 @@ int ferrum_hip_model_init_synthetic(FerrumHipModel* m, uint64_t seed) {
         if (c.has_qk_norm) {
             if (int rc = alloc_fill(&L.q_norm, c.head_dim, 1.0f)) return rc;
             if (int rc = alloc_fill(&L.k_norm, c.head_dim, 1.0f)) return rc;
+        }
+        if (synth_dense) {
+            if (int rc = synth_f16t(&L.qkv, c.hidden, qkv_dim(c), ls ^ 0x11, s)) return rc;
+            if (int rc = synth_f16t(&L.o, q_dim(c), c.hidden, ls ^ 0x22, s)) return rc;
+            if (int rc = synth_f16t(&L.gate_up, c.hidden, 2 * c.intermediate, ls ^ 0x44, s)) return rc;
+            if (int rc = synth_f16t(&L.down, c.intermediate, c.hidden, ls ^ 0x55, s)) return rc;
+            continue;
         }
         if (int rc = synth_w4(&L.qkv, c.hidden, qkv_dim(c), 1, false, ls ^ 0x11, s)) return rc;
         if (int rc = synth_w4(&L.o, q_dim(c), c.hidden, 1, false, ls ^ 0x22, s)) return rc;
@@ -1308,6 +1328,9 @@ int enqueue_body(FerrumHipModel* m, const StepShape& sh) {
         v.tokens = idx<uint32_t>(m, m->il.tokens); v.cu = idx<uint32_t>(m, m->il.cu_seqlens); v.pos = idx<uint32_t>(m, m->il.pos_offsets);
         v.bt = idx<int32_t>(m, m->il.block_tables); v.tok_seq = idx<int32_t>(m, m->il.tok_seq); v.prev = idx<int32_t>(m, m->il.prev_tokens);
         v.slots = idx<int32_t>(m, m->il.state_slots); v.units = idx<int32_t>(m, m->il.scan_units); v.num_units = m->batch_units;
+        v.host_cu = reinterpret_cast<const uint32_t*>(m->idx_host + m->il.cu_seqlens);
+        v.host_pos = reinterpret_cast<const uint32_t*>(m->idx_host + m->il.pos_offsets);
+        v.host_bt = reinterpret_cast<const int32_t*>(m->idx_host + m->il.block_tables);
         m->taps_tokens = v.T;
         return m->layered->forward(v, m->taps_enabled ? m->taps : nullptr, knobs().trace_launches, s);
     }

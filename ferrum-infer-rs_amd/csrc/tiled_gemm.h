@@ -44,25 +44,45 @@ struct GemmSection {          // columns [begin, next section's begin) of a fuse
 template <typename E>
 struct TiledGemm {
     const E* x = nullptr; long ldx = 0, x_group = 0;
+    // rows from a cache of 16-row fragment blocks instead ([k / 8][16 rows][8] each): row tile i is block x_blocks[i] of x
+    const int32_t* x_blocks = nullptr; long x_block_elems = 0;
     const E* w = nullptr;
     const float* bias = nullptr;          // [groups·n]
     int m = 0, n = 0, k = 0, groups = 1;
     int n_store = 0;                      // columns written (0: all n)
     E* out = nullptr; float* out_f32 = nullptr;      // one of the two
     long ldo = 0, out_group = 0;
+    int slabs = 1; long slab_stride = 0;  // > 1: K split over workgroups, part z at out_f32 + z·slab_stride, summed by the consumer
     const E* row_scale = nullptr; long ld_scale = 0;
     int nsec = 0;
     GemmSection sec[GEMM_MAX_SECTIONS] = {};
 };
 template <typename E> int tiled_gemm(const TiledGemm<E>& g, hipStream_t s);
+// number of K parts worth making for a projection of m rows whose consumer sums slabs (≤ GEMM_MAX_SLABS)
+constexpr int GEMM_MAX_SLABS = 8;
+int tiled_gemm_slabs(int m, int n, int k);
 
-__device__ __forceinline__ float sigmoid_f32(float z) { return 1.0f / (1.0f + expf(-z)); }
+// Activations on fp32 accumulators.  Models in 16 bits round the result to 2⁻⁹, so their form uses the hardware exponential and
+// reciprocal (relative error ≈ 2⁻²²); 32-bit models call the library functions.
+template <typename E> struct ActMath;
+template <> struct ActMath<float> {
+    static __device__ __forceinline__ float sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+    static __device__ __forceinline__ float tanh(float z) { return tanhf(z); }
+    static __device__ __forceinline__ float expm1_minus(float z) { return expm1f(z) - z; }
+};
+template <> struct ActMath<bf16> {
+    static __device__ __forceinline__ float sigmoid(float z) { return __builtin_amdgcn_rcpf(1.0f + __expf(-z)); }
+    static __device__ __forceinline__ float tanh(float z) { return 1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + __expf(2.0f * z)); }
+    static __device__ __forceinline__ float expm1_minus(float z) { return __expf(z) - 1.0f - z; }
+};
+template <typename E>
 __device__ __forceinline__ float gelu_tanh_f32(float z) {
-    return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+    return 0.5f * z * (1.0f + ActMath<E>::tanh(0.7978845608028654f * (z + 0.044715f * z * z * z)));
 }
 // quadratic right of zero, exponential left of it, slope 1/2 at zero; sp / sq: softplus of the two trained numbers
+template <typename E>
 __device__ __forceinline__ float xielu_f32(float z, float sp, float sq) {
-    return z > 0.f ? sp * z * z + 0.5f * z : (0.5f + sq) * (expm1f(z) - z) + 0.5f * z;
+    return (z > 0.f ? sp * z * z : (0.5f + sq) * ActMath<E>::expm1_minus(z)) + 0.5f * z;
 }
 
 }  // namespace fh

@@ -11,9 +11,9 @@ template <typename E>
 __device__ __forceinline__ void gemm_epilogue(const TiledGemm<E>& p, const GemmSection& sec, int g, int row, int col, float v) {
     if (row >= p.m || col >= p.n_store) return;
     if (p.bias) v += p.bias[(long)g * p.n + col];
-    if (sec.act == GEMM_ACT_SIGMOID) v = sigmoid_f32(v);
-    else if (sec.act == GEMM_ACT_GELU_TANH) v = gelu_tanh_f32(v);
-    else if (sec.act == GEMM_ACT_XIELU) v = xielu_f32(v, sec.p, sec.q);
+    if (sec.act == GEMM_ACT_SIGMOID) v = ActMath<E>::sigmoid(v);
+    else if (sec.act == GEMM_ACT_GELU_TANH) v = gelu_tanh_f32<E>(v);
+    else if (sec.act == GEMM_ACT_XIELU) v = xielu_f32<E>(v, sec.p, sec.q);
     if (p.row_scale) v *= (float)p.row_scale[row * p.ld_scale + g];
     const long o = row * p.ldo + g * p.out_group + col;
     if (p.out_f32) p.out_f32[o] = v; else p.out[o] = (E)v;
@@ -27,7 +27,21 @@ __device__ __forceinline__ GemmSection gemm_section(const TiledGemm<E>& p, int c
     return s;
 }
 
-// grid (column blocks, row blocks, groups); NW waves = (NW / kw) column groups × kw parts of K.
+// address of lane (a, b)'s 8 values of row tile t at k-step 0, and the distance between k-steps
+template <typename E>
+__device__ __forceinline__ const E* gemm_row(const TiledGemm<E>& p, int t, int g, int a, int b) {
+    if (p.x_blocks) {
+        const int tiles = (p.m + 15) >> 4;
+        return p.x + (long)p.x_blocks[t < tiles ? t : tiles - 1] * p.x_block_elems + (a * 16 + b) * 8;
+    }
+    const int r = t * 16 + b;
+    return p.x + (long)(r < p.m ? r : p.m - 1) * p.ldx + g * p.x_group + 8 * a;
+}
+template <typename E>
+__device__ __forceinline__ int gemm_row_step(const TiledGemm<E>& p) { return p.x_blocks ? 512 : 32; }
+
+// grid (column blocks, row blocks, groups or K slabs); NW waves = (NW / kw) column groups × kw parts of K.  Two register buffers of U
+// k-steps: the next one is requested before the current one is multiplied; loads past the part's end repeat its last k-step.
 template <typename E, int MT, int J>
 __global__ __launch_bounds__(512) void tiled_gemm_kernel(TiledGemm<E> p, int kw) {
     typedef typename Frag<E>::v8 v8;
@@ -36,16 +50,15 @@ __global__ __launch_bounds__(512) void tiled_gemm_kernel(TiledGemm<E> p, int kw)
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
     const int a = lane >> 4, b = lane & 15;
     const int cw = (blockDim.x >> 6) / kw, part = wave % kw, cg = wave / kw;
-    const int n0 = (blockIdx.x * cw + cg) * 16 * J, rb = blockIdx.y, g = blockIdx.z;
-    const int ksteps = p.k >> 5;
+    const int n0 = (blockIdx.x * cw + cg) * 16 * J, rb = blockIdx.y;
+    const int g = p.slabs > 1 ? 0 : blockIdx.z, z = p.slabs > 1 ? blockIdx.z : 0;
+    const int ksteps = p.k >> 5, parts = kw * p.slabs, mine = z * kw + part;
     const bool live = n0 < p.n;
-    const int s0 = live ? ksteps * part / kw : 0, s1 = live ? ksteps * (part + 1) / kw : 0;
+    const int s0 = live ? ksteps * mine / parts : 0, s1 = live ? ksteps * (mine + 1) / parts : 0;
     const E* xrow[MT];
+    const int xs = gemm_row_step(p);
 #pragma unroll
-    for (int mt = 0; mt < MT; mt++) {
-        const int r = (rb * MT + mt) * 16 + b;
-        xrow[mt] = p.x + (long)(r < p.m ? r : p.m - 1) * p.ldx + g * p.x_group + 8 * a;
-    }
+    for (int mt = 0; mt < MT; mt++) xrow[mt] = gemm_row(p, rb * MT + mt, g, a, b);
     const E* wt = p.w + ((long)g * (p.n >> 4) + (live ? n0 >> 4 : 0)) * ksteps * 512 + lane * 8;
     floatx4 acc[MT][J];
 #pragma unroll
@@ -53,31 +66,38 @@ __global__ __launch_bounds__(512) void tiled_gemm_kernel(TiledGemm<E> p, int kw)
 #pragma unroll
         for (int j = 0; j < J; j++) acc[mt][j] = (floatx4){0.f, 0.f, 0.f, 0.f};
     constexpr int U = sizeof(E) == 2 ? 4 : 1;
-    int s = s0;
-    for (; s + U <= s1; s += U) {
-        v8 bw[U][J], ax[U][MT];
+    v8 bw[2][U][J], ax[2][U][MT];
+    auto load = [&](v8 (&bq)[U][J], v8 (&aq)[U][MT], int s) {
 #pragma unroll
         for (int u = 0; u < U; u++) {
+            const int ss = min(s + u, s1 - 1);
 #pragma unroll
-            for (int j = 0; j < J; j++) bw[u][j] = *reinterpret_cast<const v8*>(wt + ((long)j * ksteps + s + u) * 512);
+            for (int j = 0; j < J; j++) bq[u][j] = *reinterpret_cast<const v8*>(wt + ((long)j * ksteps + ss) * 512);
 #pragma unroll
-            for (int mt = 0; mt < MT; mt++) ax[u][mt] = *reinterpret_cast<const v8*>(xrow[mt] + (s + u) * 32);
+            for (int mt = 0; mt < MT; mt++) aq[u][mt] = *reinterpret_cast<const v8*>(xrow[mt] + (long)ss * xs);
         }
+    };
+    auto mul = [&](v8 (&bq)[U][J], v8 (&aq)[U][MT], int s) {
 #pragma unroll
         for (int u = 0; u < U; u++)
+            if (s + u < s1) {
 #pragma unroll
-            for (int j = 0; j < J; j++)
+                for (int j = 0; j < J; j++)
 #pragma unroll
-                for (int mt = 0; mt < MT; mt++) acc[mt][j] = Frag<E>::mma(ax[u][mt], bw[u][j], acc[mt][j]);
-    }
-    for (; s < s1; s++) {
-#pragma unroll
-        for (int j = 0; j < J; j++) {
-            const v8 bw = *reinterpret_cast<const v8*>(wt + ((long)j * ksteps + s) * 512);
-#pragma unroll
-            for (int mt = 0; mt < MT; mt++) acc[mt][j] = Frag<E>::mma(*reinterpret_cast<const v8*>(xrow[mt] + s * 32), bw, acc[mt][j]);
+                    for (int mt = 0; mt < MT; mt++) acc[mt][j] = Frag<E>::mma(aq[u][mt], bq[u][j], acc[mt][j]);
+            }
+    };
+    if (s0 < s1) {
+        load(bw[0], ax[0], s0);
+        for (int s = s0; s < s1; s += 2 * U) {
+            if (s + U < s1) load(bw[1], ax[1], s + U);
+            mul(bw[0], ax[0], s);
+            if (s + U >= s1) break;
+            if (s + 2 * U < s1) load(bw[0], ax[0], s + 2 * U);
+            mul(bw[1], ax[1], s + U);
         }
     }
+    if (p.slabs > 1) p.out_f32 += z * p.slab_stride;
     const GemmSection sec = gemm_section(p, n0);
     if (kw == 1) {
         if (!live) return;
@@ -123,10 +143,11 @@ __global__ __launch_bounds__(256, 2) void tiled_gemm_big_kernel(TiledGemm<bf16> 
     const bf16 *ap[2], *bp[2];
 #pragma unroll
     for (int i = 0; i < 2; i++) {
-        const int r = m0 + (2 * wave + i) * 16 + b, t = (n0 >> 4) + 2 * wave + i;
-        ap[i] = p.x + (long)(r < p.m ? r : p.m - 1) * p.ldx + g * p.x_group + 8 * a;
+        const int t = (n0 >> 4) + 2 * wave + i;
+        ap[i] = gemm_row(p, (m0 >> 4) + 2 * wave + i, g, a, b);
         bp[i] = p.w + ((long)g * ntl + (t < ntl ? t : ntl - 1)) * ksteps * 512 + lane * 8;
     }
+    const int xs = gemm_row_step(p);
     auto issue = [&](int st, int ks) {
 #pragma unroll
         for (int h = 0; h < 2; h++) {
@@ -135,7 +156,7 @@ __global__ __launch_bounds__(256, 2) void tiled_gemm_big_kernel(TiledGemm<bf16> 
             for (int i = 0; i < 2; i++) {
                 bf16* da = &lds[st][((2 * wave + i) * 2 + h) * 512];
                 bf16* db = &lds[st][(16 + (2 * wave + i) * 2 + h) * 512];
-                __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(ap[i] + kk * 32),
+                __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(ap[i] + (long)kk * xs),
                                                  (__attribute__((address_space(3))) void*)da, 16, 0, 0);
                 __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(bp[i] + (long)kk * 512),
                                                  (__attribute__((address_space(3))) void*)db, 16, 0, 0);
@@ -191,6 +212,22 @@ static int launch_big(const TiledGemm<bf16>& g, hipStream_t s) {
 }
 static int launch_big(const TiledGemm<float>&, hipStream_t) { return 2; }      // (never taken: 16-bit only)
 
+int tiled_gemm_slabs(int m, int n, int k) {
+    if (m > 64) return 1;
+    // narrow outputs: enough (column group, K part) workgroups to cover the chip, two k-steps or more per wave
+    int S = 1;
+    while (S < GEMM_MAX_SLABS && (n / 32) * S < 256 && k / 32 >= 2 * 8 * 2 * S) S *= 2;
+    return S;
+}
+
+template <typename E, int MT, int J>
+static int launch_small(const TiledGemm<E>& g, dim3 grid, int kw, hipStream_t s) {
+    const size_t lds = kw == 1 ? 0 : (size_t)8 * MT * J * 1024;
+    hipLaunchKernelGGL((tiled_gemm_kernel<E, MT, J>), grid, dim3(512), lds, s, g, kw);
+    FH_CHECK_LAUNCH();
+    return 0;
+}
+
 template <typename E>
 int tiled_gemm(const TiledGemm<E>& gin, hipStream_t s) {
     TiledGemm<E> g = gin;
@@ -199,23 +236,20 @@ int tiled_gemm(const TiledGemm<E>& gin, hipStream_t s) {
     FH_REQUIRE(g.n > 0 && g.k > 0 && g.n % 32 == 0 && g.k % 32 == 0, "tiled_gemm: n=%d k=%d must be multiples of 32", g.n, g.k);
     FH_REQUIRE(g.ldx % 8 == 0 && g.x_group % 8 == 0 && g.n_store <= g.n && g.groups >= 1, "tiled_gemm: ldx=%ld group stride=%ld", g.ldx, g.x_group);
     FH_REQUIRE((g.out != nullptr) != (g.out_f32 != nullptr), "tiled_gemm: exactly one output");
+    FH_REQUIRE(g.slabs == 1 || (g.groups == 1 && g.out_f32 && !g.bias && !g.nsec && !g.row_scale), "tiled_gemm: slabs are plain fp32 partial sums");
     const long tiles = (long)cdiv(g.m, 128) * cdiv(g.n, 128) * g.groups;
-    if (sizeof(E) == 2 && g.m > 64 && tiles >= knobs().tiled_big_min_tiles) return launch_big(g, s);
-    const int mt = g.m <= 16 ? 1 : (g.m <= 32 ? 2 : 4), J = 2;
-    const int rbs = cdiv(g.m, 16 * mt), ksteps = g.k / 32;
-    // column groups of 32; split K over the waves until the launch has enough of them
+    if (sizeof(E) == 2 && g.m > 64 && g.slabs == 1 && tiles >= knobs().tiled_big_min_tiles) return launch_big(g, s);
+    const int mt = g.m <= 16 ? 1 : (g.m <= 32 ? 2 : 4);
+    const int rbs = cdiv(g.m, 16 * mt), ksteps = g.k / 32, zs = g.groups * g.slabs;
+    // 32 columns per wave, 16 where 32 would leave CUs without a workgroup; K split over the waves until the launch has enough of them
+    const int J = (long)rbs * (g.n / 32) * zs < 256 ? 1 : 2;
+    const long cols = g.n / (16 * J);
     int kw = 1;
-    const long waves = (long)rbs * (g.n / 32) * g.groups;
-    while (kw < 8 && waves * kw < 4096 && ksteps >= 4 * kw) kw *= 2;
-    const int cw = 8 / kw;
-    const dim3 grid(cdiv(g.n / 32, cw), rbs, g.groups);
-    const size_t lds = kw == 1 ? 0 : (size_t)8 * mt * J * 1024;
+    while (kw < 8 && (long)rbs * cols * zs * kw < 4096 && ksteps >= 2 * kw * g.slabs) kw *= 2;
+    const dim3 grid(cdiv(cols, 8 / kw), rbs, zs);
     form_hit(FORM_TILED_GEMM);
-    if (mt == 1) hipLaunchKernelGGL((tiled_gemm_kernel<E, 1, 2>), grid, dim3(512), lds, s, g, kw);
-    else if (mt == 2) hipLaunchKernelGGL((tiled_gemm_kernel<E, 2, 2>), grid, dim3(512), lds, s, g, kw);
-    else hipLaunchKernelGGL((tiled_gemm_kernel<E, 4, 2>), grid, dim3(512), lds, s, g, kw);
-    FH_CHECK_LAUNCH();
-    return 0;
+    if (J == 1) return mt == 1 ? launch_small<E, 1, 1>(g, grid, kw, s) : mt == 2 ? launch_small<E, 2, 1>(g, grid, kw, s) : launch_small<E, 4, 1>(g, grid, kw, s);
+    return mt == 1 ? launch_small<E, 1, 2>(g, grid, kw, s) : mt == 2 ? launch_small<E, 2, 2>(g, grid, kw, s) : launch_small<E, 4, 2>(g, grid, kw, s);
 }
 template int tiled_gemm<bf16>(const TiledGemm<bf16>&, hipStream_t);
 template int tiled_gemm<float>(const TiledGemm<float>&, hipStream_t);
