@@ -49,6 +49,9 @@ void reload_knobs() {
     k.chain_attn_splits = env_int("FERRUM_HIP_CHAIN_ATTN_SPLITS", 0);
     k.route_gemm_topk = env_int("FERRUM_HIP_ROUTE_GEMM_TOPK", 1);
     k.tiled_big_min_tiles = env_int("FERRUM_HIP_TILED_BIG_MIN_TILES", 64);
+    k.tiled_nw = env_int("FERRUM_HIP_TILED_NW", 0);
+    k.tiled_kw = env_int("FERRUM_HIP_TILED_KW", 0);
+    k.tiled_j = env_int("FERRUM_HIP_TILED_J", 0);
     k.latent_splits = env_int("FERRUM_HIP_LATENT_SPLITS", 0);
     k.latent_expand_min_rows = env_int("FERRUM_HIP_LATENT_EXPAND_MIN_ROWS", 64);
     k.latent_plain = env_int("FERRUM_HIP_LATENT_PLAIN", 0) != 0;

@@ -56,6 +56,7 @@ struct Knobs {
     int lds_min_groups = 8;
     // layered models (tiled_gemm.hip, latent_attention.hip, rglru.hip)
     int tiled_big_min_tiles = 64;     // 16-bit projections of > 64 rows take the 128 × 128 tile kernel from this many tiles
+    int tiled_nw = 0, tiled_kw = 0, tiled_j = 0;      // > 0: forced waves per workgroup, K parts, 16-column tiles per wave of the few-row kernel
     int latent_splits = 0;            // > 0: forced KV split count of the latent attention
     int latent_expand_min_rows = 64;  // prompt portions of at least this many tokens attend expanded keys / values (0 = never)
     bool latent_plain = false;        // the plain latent attention kernel for 16-bit models too

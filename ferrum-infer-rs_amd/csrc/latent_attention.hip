@@ -26,14 +26,20 @@ namespace fh {
 template <typename V>
 __device__ __forceinline__ V rotate8(V x, int d0, int rot_dims, const float* __restrict__ cos_t, const float* __restrict__ sin_t, long pos) {
     const int half = rot_dims >> 1;
+    if (half == 0) return x;
+    float c[4], s[4];
 #pragma unroll
     for (int j = 0; j < 4; j++) {
         const int i = (d0 >> 1) + j;
-        if (i < half) {
-            const float c = cos_t[pos * half + i], s = sin_t[pos * half + i], u = (float)x[2 * j], w = (float)x[2 * j + 1];
-            x[2 * j] = u * c - w * s;
-            x[2 * j + 1] = w * c + u * s;
-        }
+        const float cv = cos_t[pos * half + (i < half ? i : half - 1)], sv = sin_t[pos * half + (i < half ? i : half - 1)];
+        c[j] = i < half ? cv : 1.f;
+        s[j] = i < half ? sv : 0.f;
+    }
+#pragma unroll
+    for (int j = 0; j < 4; j++) {
+        const float u = (float)x[2 * j], w = (float)x[2 * j + 1];
+        x[2 * j] = u * c[j] - w * s[j];
+        x[2 * j + 1] = w * c[j] + u * s[j];
     }
     return x;
 }
@@ -189,7 +195,6 @@ __device__ __forceinline__ bool find_latent_tile(const BatchView& v, int heads, 
     return false;
 }
 
-constexpr int LATENT_RS = 2;           // k-steps of the rotated part: rot_dim ≤ 64
 constexpr int LATENT_PARTIAL_PAD = 4;  // floats behind a partial row's outputs: maximum, sum
 // offset of lane's 4 values in a transposed read: lane i of a 16-lane group names 4 dims of key 4a + i / 4 (of a 16-key block, 16 dims =
 // two chunks) and receives dim i of keys 4a … 4a + 3
@@ -200,10 +205,10 @@ __device__ __forceinline__ shortx4 read_tr(const bf16* p) {
     return __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) shortx4*)p);
 }
 
-// KS: most k-steps of the latent (kv_rank ≤ 32·KS).  grid (KV splits, row tiles); a step is 64 keys: wave w scores block w of them
+// KS, RS: 32-wide steps of the latent and of the rotated part.  grid (KV splits, row tiles); a step is 64 keys: wave w scores block w of them
 // for all 16 rows, the row maxima meet in LDS, P and the parked latents are shared, and each wave accumulates its own quarter of the
 // output dimensions — so nothing is merged at the end and the latents of the next step are in flight during softmax and P·V.
-template <int KS>
+template <int KS, int RS>
 __global__ __launch_bounds__(256, 2) void latent_attn_kernel(LatentDims d, LatentBuffers<bf16> p, BatchView v, int nsplit) {
     constexpr int DT = KS < 2 ? 1 : KS / 2;                                    // 16-dim output tiles per wave
     constexpr int STAGE = KS * 512, PSTR = 72;
@@ -213,7 +218,8 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(LatentDims d, Laten
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, a = lane >> 4, b = lane & 15;
     LatentTile w;
     if (!find_latent_tile(v, d.heads, blockIdx.y, &w)) return;
-    const int ks = d.kp >> 5, rs = d.rp >> 5, kd = d.kp + d.rp, rows = w.q_len * d.heads;
+    constexpr int kd = 32 * (KS + RS);
+    const int rows = w.q_len * d.heads;
     const int rho = w.tile * 16 + b;
     const bool ok = rho < rows;
     const int tl = ok ? rho / d.heads : 0, h = ok ? rho % d.heads : 0;
@@ -221,30 +227,28 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(LatentDims d, Laten
     const int t_first = w.tile * 16 / d.heads, t_last = min(w.q_len - 1, (w.tile * 16 + 15) / d.heads);
     const int kv_end = w.pos0 + t_last + 1, kv_lo = max(0, w.pos0 + t_first + 1 - d.window);
     const int blk_lo = kv_lo / 16, blk_hi = (kv_end + 15) / 16, nstep = (blk_hi - blk_lo + 3) / 4;
-    const int per = (nstep + nsplit - 1) / nsplit;
-    const int st_lo = (int)blockIdx.x * per, st_hi = min(nstep, st_lo + per);
+    const int st_lo = nstep * (int)blockIdx.x / nsplit, st_hi = nstep * ((int)blockIdx.x + 1) / nsplit;
     const int32_t* bt = v.bt + (long)w.seq * v.max_blocks;
 
-    bf16x8 kf[KS + LATENT_RS], qf[KS + LATENT_RS];
+    bf16x8 kf[KS + RS], qf[KS + RS];
     auto load = [&](int st) {                                                  // (past the last block: a copy of it, masked below)
         const bf16* t = p.pool + (long)bt[min(blk_lo + 4 * st + wave, blk_hi - 1)] * 16 * kd + lane * 8;
 #pragma unroll
         for (int s = 0; s < KS; s++)
-            if (s < ks) kf[s] = *reinterpret_cast<const bf16x8*>(t + s * 512);
+            kf[s] = *reinterpret_cast<const bf16x8*>(t + s * 512);
 #pragma unroll
-        for (int s = 0; s < LATENT_RS; s++)
-            if (s < rs) kf[KS + s] = *reinterpret_cast<const bf16x8*>(t + (ks + s) * 512);
+        for (int s = 0; s < RS; s++)
+            kf[KS + s] = *reinterpret_cast<const bf16x8*>(t + (KS + s) * 512);
     };
-    if (st_lo < st_hi) load(st_lo);
+    load(st_lo);                                                               // (no load under a condition: it would drain the others)
     {
         const long qrow = (long)(w.tok0 + tl) * d.heads + h;
 #pragma unroll
         for (int s = 0; s < KS; s++)
-            if (s < ks) qf[s] = *reinterpret_cast<const bf16x8*>(p.q_lat + qrow * d.kp + 32 * s + 8 * a);
+            qf[s] = *reinterpret_cast<const bf16x8*>(p.q_lat + qrow * (32 * KS) + 32 * s + 8 * a);
 #pragma unroll
-        for (int s = 0; s < LATENT_RS; s++)
-            if (s < rs)
-                qf[KS + s] = rotate8(*reinterpret_cast<const bf16x8*>(p.q + qrow * (d.dp + d.rp) + d.dp + 32 * s + 8 * a), 32 * s + 8 * a,
+        for (int s = 0; s < RS; s++)
+            qf[KS + s] = rotate8(*reinterpret_cast<const bf16x8*>(p.q + qrow * (d.dp + d.rp) + d.dp + 32 * s + 8 * a), 32 * s + 8 * a,
                                      d.rot_dims, p.cos_t, p.sin_t, row_pos);
     }
     const int tr_off = tr_offset(lane);
@@ -256,10 +260,10 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(LatentDims d, Laten
         floatx4 sc2[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};        // two chains: half the dependent MFMA latency
 #pragma unroll
         for (int s = 0; s < KS; s++)
-            if (s < ks) sc2[s & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[s], qf[s], sc2[s & 1], 0, 0, 0);
+            sc2[s & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[s], qf[s], sc2[s & 1], 0, 0, 0);
 #pragma unroll
-        for (int s = 0; s < LATENT_RS; s++)
-            if (s < rs) sc2[s & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[KS + s], qf[KS + s], sc2[s & 1], 0, 0, 0);
+        for (int s = 0; s < RS; s++)
+            sc2[s & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[KS + s], qf[KS + s], sc2[s & 1], 0, 0, 0);
         floatx4 sc;
         float mx = -INFINITY;
 #pragma unroll
@@ -272,9 +276,9 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(LatentDims d, Laten
         __syncthreads();                                                       // the previous step's P·V has read stage and lds_p
 #pragma unroll
         for (int s = 0; s < KS; s++)
-            if (s < ks) *reinterpret_cast<bf16x8*>(stage + wave * STAGE + s * 512 + lane * 8) = kf[s];
+            *reinterpret_cast<bf16x8*>(stage + wave * STAGE + s * 512 + lane * 8) = kf[s];
         if (a == 0) lds_m[wave * 16 + b] = mx;
-        if (st + 1 < st_hi) load(st + 1);
+        load(st + 1);
         __syncthreads();
         const float m_new = fmaxf(m_run, fmaxf(fmaxf(lds_m[b], lds_m[16 + b]), fmaxf(lds_m[32 + b], lds_m[48 + b])));
         const float m_safe = m_new == -INFINITY ? 0.f : m_new, alpha = __expf(m_run - m_safe);
@@ -298,7 +302,7 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(LatentDims d, Laten
             const bf16* vb = stage + (2 * c + (a >> 1)) * STAGE + tr_off + ((a & 1) * 8 - 4 * a) * 8;
 #pragma unroll
             for (int t = 0; t < DT; t++)
-                if (wave + 4 * t < 2 * ks) {
+                if (KS >= 2 || wave < 2 * KS) {
                     const shortx4 v0 = read_tr(vb + (wave + 4 * t) * 256), v1 = read_tr(vb + (wave + 4 * t) * 256 + 32);
                     typedef short shortx8 __attribute__((ext_vector_type(8)));
                     const shortx8 vt = {v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
@@ -311,19 +315,19 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(LatentDims d, Laten
     __syncthreads();
     const float L = lds_l[b] + lds_l[16 + b] + lds_l[32 + b] + lds_l[48 + b];
     if (nsplit > 1) {
-        float* dst = p.partial + (((long)blockIdx.y * nsplit + blockIdx.x) * 16 + b) * (d.kp + LATENT_PARTIAL_PAD);
+        float* dst = p.partial + (((long)blockIdx.y * nsplit + blockIdx.x) * 16 + b) * (32 * KS + LATENT_PARTIAL_PAD);
 #pragma unroll
         for (int t = 0; t < DT; t++)
-            if (wave + 4 * t < 2 * ks) *reinterpret_cast<floatx4*>(dst + (wave + 4 * t) * 16 + 4 * a) = o[t];
-        if (threadIdx.x < 16) { dst[d.kp] = m_run; dst[d.kp + 1] = L; }
+            if (KS >= 2 || wave < 2 * KS) *reinterpret_cast<floatx4*>(dst + (wave + 4 * t) * 16 + 4 * a) = o[t];
+        if (threadIdx.x < 16) { dst[32 * KS] = m_run; dst[32 * KS + 1] = L; }
         return;
     }
     if (!ok) return;
     const float inv = L > 0.f ? 1.0f / L : 0.f;
-    bf16* dst = p.o_lat + ((long)w.tok0 * d.heads + rho) * d.kp;
+    bf16* dst = p.o_lat + ((long)w.tok0 * d.heads + rho) * (32 * KS);
 #pragma unroll
     for (int t = 0; t < DT; t++)
-        if (wave + 4 * t < 2 * ks) {
+        if (KS >= 2 || wave < 2 * KS) {
             bf16x4 y;
 #pragma unroll
             for (int r = 0; r < 4; r++) y[r] = (bf16)(o[t][r] * inv);
@@ -357,19 +361,20 @@ __global__ __launch_bounds__(256) void latent_attn_reduce_kernel(LatentDims d, L
 // A workgroup owns 128 tokens of one sequence and head: 4 waves × 2 row tiles of 16.  64 keys per step: wave w copies 16-key block w of
 // the step — expanded key rows, the shared rotated part straight from the cache, expanded value rows — as fragments into LDS with the
 // load unit, double-buffered; Sᵀ = K·Qᵀ keeps a row's statistics lane-local, values are read back transposed for Oᵀ += Vᵀ·Pᵀ.
-constexpr int LX_DS = 4, LX_RS = 2, LX_VS = 4;           // most 32-wide steps of the plain, rotated and value dimensions
+// DS: 32-wide steps of the plain query / key dimensions and of the values (padded alike), RS: of the rotated part.
+template <int DS, int RS>
 __global__ __launch_bounds__(256, 2) void latent_expanded_kernel(LatentDims d, LatentBuffers<bf16> p, BatchView v, LatentExpanded x) {
-    constexpr int MT = 2, BLK = (LX_DS + LX_RS + LX_VS) * 512, DT = 2 * LX_VS;
+    constexpr int MT = 2, BLK = (2 * DS + RS) * 512, DT = 2 * DS;
     extern __shared__ __attribute__((aligned(16))) bf16 lds_x[];               // [2][4 blocks][BLK]
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, a = lane >> 4, b = lane & 15;
     const int h = blockIdx.y;
     const int32_t* un = x.units + 4 * (gridDim.x - 1 - blockIdx.x);            // the longest key ranges start first
     const int seq = un[0], tile0 = un[1], base = un[2], first_blk = un[3];
     const int tok0 = (int)v.cu[seq], q_len = (int)v.cu[seq + 1] - tok0, pos0 = (int)v.pos[seq];
-    const int ds = d.dp >> 5, rs = d.rp >> 5, vs = d.vp >> 5, kd = d.kp + d.rp;
+    const int kd = d.kp + d.rp;
     const float sl2 = d.scale * 1.4426950408889634f;
 
-    bf16x8 qf[MT][LX_DS + LX_RS];
+    bf16x8 qf[MT][DS + RS];
     int row_pos[MT], win_lo[MT], vis_lo[MT], vis_hi[MT];
     bool ok[MT];
 #pragma unroll
@@ -382,11 +387,11 @@ __global__ __launch_bounds__(256, 2) void latent_expanded_kernel(LatentDims d, L
         vis_lo[mt] = max(0, pos0 + t0 + 16 - d.window);
         const bf16* q = p.q + ((long)(tok0 + min(t, q_len - 1)) * d.heads + h) * (d.dp + d.rp) + 8 * a;
 #pragma unroll
-        for (int s = 0; s < LX_DS; s++)
-            if (s < ds) qf[mt][s] = *reinterpret_cast<const bf16x8*>(q + 32 * s);
+        for (int s = 0; s < DS; s++)
+            qf[mt][s] = *reinterpret_cast<const bf16x8*>(q + 32 * s);
 #pragma unroll
-        for (int s = 0; s < LX_RS; s++)
-            if (s < rs) qf[mt][LX_DS + s] = rotate8(*reinterpret_cast<const bf16x8*>(q + d.dp + 32 * s), 32 * s + 8 * a, d.rot_dims, p.cos_t, p.sin_t, row_pos[mt]);
+        for (int s = 0; s < RS; s++)
+            qf[mt][DS + s] = rotate8(*reinterpret_cast<const bf16x8*>(q + d.dp + 32 * s), 32 * s + 8 * a, d.rot_dims, p.cos_t, p.sin_t, row_pos[mt]);
     }
     const int t_hi = min(q_len, tile0 + LATENT_TILE_TOKENS);
     const int blk_lo = max(0, pos0 + tile0 + 1 - d.window) / 16, blk_hi = (pos0 + t_hi + 15) / 16, nstep = (blk_hi - blk_lo + 3) / 4;
@@ -397,14 +402,14 @@ __global__ __launch_bounds__(256, 2) void latent_expanded_kernel(LatentDims d, L
         const bf16* r = p.pool + (long)x.blocks[i] * 16 * kd + d.kp * 16 + lane * 8;
 #define LX_COPY(src, slot) __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(src), (__attribute__((address_space(3))) void*)(dst + (slot) * 512), 16, 0, 0)
 #pragma unroll
-        for (int s = 0; s < LX_DS; s++)
-            if (s < ds) LX_COPY(k + 32 * s, s);
+        for (int s = 0; s < DS; s++)
+            LX_COPY(k + 32 * s, s);
 #pragma unroll
-        for (int s = 0; s < LX_RS; s++)
-            if (s < rs) LX_COPY(r + s * 512, LX_DS + s);
+        for (int s = 0; s < RS; s++)
+            LX_COPY(r + s * 512, DS + s);
 #pragma unroll
-        for (int s = 0; s < LX_VS; s++)
-            if (s < vs) LX_COPY(vr + 32 * s, LX_DS + LX_RS + s);
+        for (int s = 0; s < DS; s++)
+            LX_COPY(vr + 32 * s, DS + RS + s);
 #undef LX_COPY
     };
     const int tr_off = tr_offset(lane);
@@ -429,15 +434,14 @@ __global__ __launch_bounds__(256, 2) void latent_expanded_kernel(LatentDims d, L
 #pragma unroll
             for (int i = 0; i < 4; i++) sv[mt][i] = (floatx4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int s = 0; s < LX_DS + LX_RS; s++)
-            if (s < LX_DS ? s < ds : s - LX_DS < rs) {
+        for (int s = 0; s < DS + RS; s++) {
 #pragma unroll
                 for (int i = 0; i < 4; i++) {
                     const bf16x8 k = *reinterpret_cast<const bf16x8*>(kb + i * BLK + s * 512 + lane * 8);
 #pragma unroll
                     for (int mt = 0; mt < MT; mt++) sv[mt][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k, qf[mt][s], sv[mt][i], 0, 0, 0);
                 }
-            }
+        }
         bf16x8 pf[MT][2];
         const int key0 = (blk_lo + 4 * st) * 16;
 #pragma unroll
@@ -477,10 +481,9 @@ __global__ __launch_bounds__(256, 2) void latent_expanded_kernel(LatentDims d, L
         // contraction index of a 32-key pair: (a, j < 4) = key 4a + j of its first block, (a, j ≥ 4) = key 4a + j − 4 of its second
 #pragma unroll
         for (int c = 0; c < 2; c++) {
-            const bf16* vb = kb + 2 * c * BLK + (LX_DS + LX_RS) * 512 + tr_off;
+            const bf16* vb = kb + 2 * c * BLK + (DS + RS) * 512 + tr_off;
 #pragma unroll
-            for (int t = 0; t < DT; t++)
-                if (t < 2 * vs) {
+            for (int t = 0; t < DT; t++) {
                     const shortx4 v0 = read_tr(vb + t * 256), v1 = read_tr(vb + BLK + t * 256);
                     typedef short shortx8 __attribute__((ext_vector_type(8)));
                     const shortx8 vt = {v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
@@ -500,8 +503,7 @@ __global__ __launch_bounds__(256, 2) void latent_expanded_kernel(LatentDims d, L
         const float f = (float)x.gate[tok * x.ld_gate + h] / l;
         bf16* dst = x.out + (tok * d.heads + h) * d.vp + 4 * a;
 #pragma unroll
-        for (int t = 0; t < DT; t++)
-            if (t < 2 * vs) {
+        for (int t = 0; t < DT; t++) {
                 bf16x4 y;
 #pragma unroll
                 for (int r = 0; r < 4; r++) y[r] = (bf16)(o[mt][t][r] * f);
@@ -509,16 +511,21 @@ __global__ __launch_bounds__(256, 2) void latent_expanded_kernel(LatentDims d, L
             }
     }
 }
-bool latent_expanded_supports(const LatentDims& d) { return d.dp <= 32 * LX_DS && d.rp <= 32 * LX_RS && d.vp <= 32 * LX_VS && d.scale > 0.f; }
-int latent_attention_expanded(const LatentDims& d, const LatentBuffers<bf16>& b, const BatchView& v, const LatentExpanded& x, hipStream_t s) {
-    FH_REQUIRE(latent_expanded_supports(d), "latent attention: sizes the expanded form does not take");
-    constexpr size_t lds = (size_t)2 * 4 * (LX_DS + LX_RS + LX_VS) * 512 * sizeof(bf16);
+bool latent_expanded_supports(const LatentDims& d) { return d.dp == d.vp && d.dp <= 128 && d.rp <= 64 && d.scale > 0.f; }
+template <int DS, int RS>
+static int launch_expanded(const LatentDims& d, const LatentBuffers<bf16>& b, const BatchView& v, const LatentExpanded& x, hipStream_t s) {
+    constexpr size_t lds = (size_t)2 * 4 * (2 * DS + RS) * 512 * sizeof(bf16);
     static bool attr = false;
-    if (!attr) { FH_CHECK_HIP(hipFuncSetAttribute((const void*)latent_expanded_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)); attr = true; }
-    form_hit(FORM_LATENT_ATTN_EXPANDED);
-    hipLaunchKernelGGL(latent_expanded_kernel, dim3(x.nunits, d.heads), dim3(256), lds, s, d, b, v, x);
+    if (!attr) { FH_CHECK_HIP(hipFuncSetAttribute((const void*)latent_expanded_kernel<DS, RS>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)); attr = true; }
+    hipLaunchKernelGGL((latent_expanded_kernel<DS, RS>), dim3(x.nunits, d.heads), dim3(256), lds, s, d, b, v, x);
     FH_CHECK_LAUNCH();
     return 0;
+}
+int latent_attention_expanded(const LatentDims& d, const LatentBuffers<bf16>& b, const BatchView& v, const LatentExpanded& x, hipStream_t s) {
+    FH_REQUIRE(latent_expanded_supports(d), "latent attention: sizes the expanded form does not take");
+    form_hit(FORM_LATENT_ATTN_EXPANDED);
+    if (d.rp == 32) return d.dp == 32 ? launch_expanded<1, 1>(d, b, v, x, s) : d.dp == 64 ? launch_expanded<2, 1>(d, b, v, x, s) : launch_expanded<4, 1>(d, b, v, x, s);
+    return d.dp == 32 ? launch_expanded<1, 2>(d, b, v, x, s) : d.dp == 64 ? launch_expanded<2, 2>(d, b, v, x, s) : launch_expanded<4, 2>(d, b, v, x, s);
 }
 
 template <typename E>
@@ -533,17 +540,27 @@ static int latent_plain(const LatentDims& d, const LatentBuffers<E>& b, const Ba
 static int latent_mfma(const LatentDims& d, const LatentBuffers<bf16>& b, const BatchView& v, hipStream_t s) {
     const int tiles = v.single ? v.num_seqs * cdiv(d.heads, 16) : (int)(((long)v.T * d.heads) / 16) + v.num_seqs;      // upper bound of Σ ceil(rows / 16)
     const int keys = std::min(v.max_keys, d.window + 16);
-    // split the keys while the launch has fewer than ≈ 1 workgroup per CU and a split keeps ≥ 128 keys (two steps)
+    // split the keys while the launch has fewer than ≈ 1 workgroup per CU and a split keeps ≥ 256 keys (four steps)
     int ns = 1;
-    while (ns < 16 && tiles * ns < 256 && keys >= 2 * ns * 128) ns *= 2;
+    while (ns < 16 && tiles * ns < 256 && keys >= 2 * ns * 256) ns *= 2;
     if (knobs().latent_splits > 0) ns = std::min(16, knobs().latent_splits);
     while (ns > 1 && (size_t)tiles * ns * 16 * (d.kp + LATENT_PARTIAL_PAD) * 4 > b.partial_bytes) ns /= 2;
     const dim3 grid(ns, tiles);          // (splits fastest: the row tiles of a sequence read a key range on the same XCD)
     form_hit(ns > 1 ? FORM_LATENT_ATTN_SPLIT : FORM_LATENT_ATTN);
-    if (d.kp <= 64) hipLaunchKernelGGL(latent_attn_kernel<2>, grid, dim3(256), 0, s, d, b, v, ns);
-    else if (d.kp <= 128) hipLaunchKernelGGL(latent_attn_kernel<4>, grid, dim3(256), 0, s, d, b, v, ns);
-    else if (d.kp <= 256) hipLaunchKernelGGL(latent_attn_kernel<8>, grid, dim3(256), 0, s, d, b, v, ns);
-    else hipLaunchKernelGGL(latent_attn_kernel<16>, grid, dim3(256), 0, s, d, b, v, ns);
+#define LATENT(KS)                                                                                             \
+    do {                                                                                                       \
+        if (d.rp == 32) hipLaunchKernelGGL((latent_attn_kernel<KS, 1>), grid, dim3(256), 0, s, d, b, v, ns);    \
+        else hipLaunchKernelGGL((latent_attn_kernel<KS, 2>), grid, dim3(256), 0, s, d, b, v, ns);               \
+    } while (0)
+    switch (d.kp) {
+    case 32: LATENT(1); break;
+    case 64: LATENT(2); break;
+    case 128: LATENT(4); break;
+    case 256: LATENT(8); break;
+    case 384: LATENT(12); break;
+    default: LATENT(16); break;
+    }
+#undef LATENT
     FH_CHECK_LAUNCH();
     if (ns > 1) {
         hipLaunchKernelGGL(latent_attn_reduce_kernel, dim3(tiles, cdiv(16 * (d.kp / 4), 256)), dim3(256), 0, s, d, b, v, ns);
@@ -555,7 +572,7 @@ template <> int latent_attention<float>(const LatentDims& d, const LatentBuffers
     return latent_plain(d, b, v, s);
 }
 template <> int latent_attention<bf16>(const LatentDims& d, const LatentBuffers<bf16>& b, const BatchView& v, hipStream_t s) {
-    if (knobs().latent_plain || d.kp > 512 || d.rp > 32 * LATENT_RS) return latent_plain(d, b, v, s);
+    if (knobs().latent_plain || d.kp > 512 || d.rp > 64) return latent_plain(d, b, v, s);
     return latent_mfma(d, b, v, s);
 }
 template int latent_prepare<bf16>(const bf16*, const bf16*, long, const float*, const float*, float, const LatentDims&, const LatentBuffers<bf16>&,

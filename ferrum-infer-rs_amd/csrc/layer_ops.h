@@ -1,6 +1,9 @@
 // Kernels of the layered models' mixers and residual stream (latent_attention.hip, rglru.hip, residual_stream.hip).
 // E is bf16 or float; all leading dimensions are padded to multiples of 32 (tiled_gemm.h).
 #pragma once
+#include <algorithm>
+#include <initializer_list>
+
 #include "tiled_gemm.h"
 
 namespace fh {
@@ -39,7 +42,16 @@ int rms_norm_rows(const float* x, const int32_t* row_idx, const float* w, float 
 
 // ── latent attention (latent_attention.hip) ──
 // Cache of a layer: [blocks][(kp + rp) / 8 chunks][16 tokens][8]: the normed latent, then the rotated shared key part, zero-padded.
+// Padded sizes (heads' plain query / key dimensions dp, rotated rp, values vp, latent kp) are rounded to what the matrix-core kernels are
+// instantiated for, so that they loop over compile-time extents.
 struct LatentDims { int heads, kv_rank, q_rank, rot_dim, rot_dims, vdim, dp, rp, kp, qp, vp, window; float scale; };
+inline int latent_pad(int n, std::initializer_list<int> sizes) {
+    for (int s : sizes) if (n <= s) return s;
+    return pad32(n);
+}
+inline int latent_pad_rank(int n) { return latent_pad(n, {32, 64, 128, 256, 384, 512}); }
+inline int latent_pad_rot(int n) { return latent_pad(n, {32, 64}); }
+inline int latent_pad_head(int dim, int vdim, int n) { return std::max(dim, vdim) <= 128 ? latent_pad(std::max(dim, vdim), {32, 64, 128}) : pad32(n); }
 inline size_t latent_block_elems(const LatentDims& d) { return (size_t)16 * (d.kp + d.rp); }
 template <typename E>
 struct LatentBuffers {

@@ -333,8 +333,8 @@ private:
     void dims(Layer& L) {
         const FerrumHipLayerSpec& s = L.s;
         if (s.mixer == FERRUM_HIP_MIXER_LATENT_ATTENTION)
-            L.ld = {s.heads, s.kv_rank, s.q_rank, s.rot_dim, s.rot_dims, s.vdim, pad32(s.dim), pad32(s.rot_dim), pad32(s.kv_rank), pad32(s.q_rank),
-                    pad32(s.vdim), s.window, s.scale};
+            L.ld = {s.heads, s.kv_rank, s.q_rank, s.rot_dim, s.rot_dims, s.vdim, latent_pad_head(s.dim, s.vdim, s.dim), latent_pad_rot(s.rot_dim),
+                    latent_pad_rank(s.kv_rank), pad32(s.q_rank), latent_pad_head(s.dim, s.vdim, s.vdim), s.window, s.scale};
         else
             L.rd = {s.rnn_blocks, pad32(s.rnn_width / s.rnn_blocks), s.rnn_blocks * pad32(s.rnn_width / s.rnn_blocks), s.conv_taps};
     }

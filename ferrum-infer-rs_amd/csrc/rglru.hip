@@ -19,12 +19,14 @@ template <typename E>
 __device__ __forceinline__ typename Frag<E>::v8 conv_input(const RglruBuffers<E>& p, const RglruDims& d, int tok0, int t, int back, int slot, bool fresh, int c) {
     typedef typename Frag<E>::v8 v8;
     const int q = t - back;
-    if (q >= 0) return *reinterpret_cast<const v8*>(p.x + (long)(tok0 + q) * p.ld + c);
-    if (!fresh) return *reinterpret_cast<const v8*>(p.conv_state + ((long)slot * (d.taps - 1) + (d.taps - 1 + q)) * d.wp + c);
-    v8 z;                                               // (a fresh sequence has no tokens before its portion)
+    // one unconditional load, from the batch or from the stored tail; a fresh sequence has no tokens before its portion
+    const E* src = q >= 0 ? p.x + (long)(tok0 + q) * p.ld + c : p.conv_state + ((long)slot * (d.taps - 1) + max(0, d.taps - 1 + q)) * d.wp + c;
+    v8 in = *reinterpret_cast<const v8*>(src);
+    if (fresh && q < 0) {
 #pragma unroll
-    for (int j = 0; j < 8; j++) z[j] = (E)0.f;
-    return z;
+        for (int j = 0; j < 8; j++) in[j] = (E)0.f;
+    }
+    return in;
 }
 
 // one thread per (token, 8 channels); with one token per sequence the thread also shifts the channels' stored inputs
@@ -62,9 +64,11 @@ __device__ __forceinline__ float one_minus_exp(float t) {
 
 // grid (tiles, row blocks, blocks of the block-diagonal projections); a wave owns one 16-channel tile (ra and ri)
 template <typename E, int MT, bool STEP>
-__global__ __launch_bounds__(64) void rglru_gates_kernel(RglruDims d, RglruBuffers<E> p, BatchView v) {
+__global__ __launch_bounds__(256) void rglru_gates_kernel(RglruDims d, RglruBuffers<E> p, BatchView v) {
     typedef typename Frag<E>::v8 v8;
-    const int lane = threadIdx.x, a = lane >> 4, b = lane & 15, tile = blockIdx.x, rb = blockIdx.y, g = blockIdx.z;
+    const int lane = threadIdx.x & 63, a = lane >> 4, b = lane & 15, rb = blockIdx.y, g = blockIdx.z;
+    const int tile = blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6);
+    if (tile * 16 >= d.bp) return;
     const int ksteps = d.bp >> 5;
     const E* xrow[MT];
 #pragma unroll
@@ -178,9 +182,11 @@ int rglru_forward(const RglruDims& d, const RglruBuffers<E>& b, const BatchView&
     hipLaunchKernelGGL(rglru_conv_kernel<E>, dim3(cdiv((long)v.T * (d.wp / 8), 256)), dim3(256), 0, s, d, b, v);
     FH_CHECK_LAUNCH();
     const int mt = v.T <= 16 ? 1 : (v.T <= 32 ? 2 : 4);
-    const dim3 grid(d.bp / 16, cdiv(v.T, 16 * mt), d.blocks);
+    // prompts: the waves of a workgroup share the rows they read; steps: one wave per workgroup, spread over the CUs
+    const int nw = v.single ? 1 : 4;
+    const dim3 grid(cdiv(d.bp / 16, nw), cdiv(v.T, 16 * mt), d.blocks);
     form_hit(v.single ? FORM_RGLRU_STEP : FORM_RGLRU_SCAN);
-#define GATES(MT, ST) hipLaunchKernelGGL((rglru_gates_kernel<E, MT, ST>), grid, dim3(64), 0, s, d, b, v)
+#define GATES(MT, ST) hipLaunchKernelGGL((rglru_gates_kernel<E, MT, ST>), grid, dim3(64 * nw), 0, s, d, b, v)
     if (v.single) { if (mt == 1) GATES(1, true); else if (mt == 2) GATES(2, true); else GATES(4, true); }
     else { if (mt == 1) GATES(1, false); else if (mt == 2) GATES(2, false); else GATES(4, false); }
 #undef GATES

@@ -1,6 +1,8 @@
 // Dense projections of the layered models (tiled_gemm.h): one kernel for few rows (K split over the waves of a workgroup, summed in
 // LDS, no second launch) and one for prompts (128 × 128 tiles, both operands copied to LDS as fragments by the load unit itself).
 // Every activation, bias and per-row factor of a projection is applied to the fp32 accumulator in the epilogue.
+#include <algorithm>
+
 #include "common.h"
 #include "knobs.h"
 #include "tiled_gemm.h"
@@ -72,7 +74,7 @@ __global__ __launch_bounds__(512) void tiled_gemm_kernel(TiledGemm<E> p, int kw)
         for (int u = 0; u < U; u++) {
             const int ss = min(s + u, s1 - 1);
 #pragma unroll
-            for (int j = 0; j < J; j++) bq[u][j] = *reinterpret_cast<const v8*>(wt + ((long)j * ksteps + ss) * 512);
+            for (int j = 0; j < J; j++) bq[u][j] = __builtin_nontemporal_load(reinterpret_cast<const v8*>(wt + ((long)j * ksteps + ss) * 512));
 #pragma unroll
             for (int mt = 0; mt < MT; mt++) aq[u][mt] = *reinterpret_cast<const v8*>(xrow[mt] + (long)ss * xs);
         }
@@ -87,14 +89,19 @@ __global__ __launch_bounds__(512) void tiled_gemm_kernel(TiledGemm<E> p, int kw)
                     for (int mt = 0; mt < MT; mt++) acc[mt][j] = Frag<E>::mma(aq[u][mt], bq[u][j], acc[mt][j]);
             }
     };
+    // every buffer is requested in the block that multiplies the other one, so each wait counts exactly the loads it needs
     if (s0 < s1) {
-        load(bw[0], ax[0], s0);
-        for (int s = s0; s < s1; s += 2 * U) {
-            if (s + U < s1) load(bw[1], ax[1], s + U);
+        int s = s0;
+        load(bw[0], ax[0], s);
+        while (true) {
+            if (s + U >= s1) { mul(bw[0], ax[0], s); break; }
+            load(bw[1], ax[1], s + U);
             mul(bw[0], ax[0], s);
-            if (s + U >= s1) break;
-            if (s + 2 * U < s1) load(bw[0], ax[0], s + 2 * U);
-            mul(bw[1], ax[1], s + U);
+            s += U;
+            if (s + U >= s1) { mul(bw[1], ax[1], s); break; }
+            load(bw[0], ax[0], s + U);
+            mul(bw[1], ax[1], s);
+            s += U;
         }
     }
     if (p.slabs > 1) p.out_f32 += z * p.slab_stride;
@@ -221,9 +228,9 @@ int tiled_gemm_slabs(int m, int n, int k) {
 }
 
 template <typename E, int MT, int J>
-static int launch_small(const TiledGemm<E>& g, dim3 grid, int kw, hipStream_t s) {
-    const size_t lds = kw == 1 ? 0 : (size_t)8 * MT * J * 1024;
-    hipLaunchKernelGGL((tiled_gemm_kernel<E, MT, J>), grid, dim3(512), lds, s, g, kw);
+static int launch_small(const TiledGemm<E>& g, dim3 grid, int nw, int kw, hipStream_t s) {
+    const size_t lds = kw == 1 ? 0 : (size_t)nw * MT * J * 1024;
+    hipLaunchKernelGGL((tiled_gemm_kernel<E, MT, J>), grid, dim3(64 * nw), lds, s, g, kw);
     FH_CHECK_LAUNCH();
     return 0;
 }
@@ -242,14 +249,17 @@ int tiled_gemm(const TiledGemm<E>& gin, hipStream_t s) {
     const int mt = g.m <= 16 ? 1 : (g.m <= 32 ? 2 : 4);
     const int rbs = cdiv(g.m, 16 * mt), ksteps = g.k / 32, zs = g.groups * g.slabs;
     // 32 columns per wave, 16 where 32 would leave CUs without a workgroup; K split over the waves until the launch has enough of them
-    const int J = (long)rbs * (g.n / 32) * zs < 256 ? 1 : 2;
+    int J = (long)rbs * (g.n / 32) * zs < 256 ? 1 : 2;
+    if (knobs().tiled_j > 0) J = knobs().tiled_j == 1 ? 1 : 2;
     const long cols = g.n / (16 * J);
-    int kw = 1;
-    while (kw < 8 && (long)rbs * cols * zs * kw < 4096 && ksteps >= 2 * kw * g.slabs) kw *= 2;
-    const dim3 grid(cdiv(cols, 8 / kw), rbs, zs);
+    int nw = mt == 1 ? 8 : 4, kw = 1;
+    if (knobs().tiled_nw > 0) nw = std::min(8, knobs().tiled_nw);
+    while (kw < nw && (long)rbs * cols * zs * kw < 4096 && ksteps >= 8 * kw * g.slabs) kw *= 2;
+    if (knobs().tiled_kw > 0) kw = std::min(nw, knobs().tiled_kw);
+    const dim3 grid(cdiv(cols, nw / kw), rbs, zs);
     form_hit(FORM_TILED_GEMM);
-    if (J == 1) return mt == 1 ? launch_small<E, 1, 1>(g, grid, kw, s) : mt == 2 ? launch_small<E, 2, 1>(g, grid, kw, s) : launch_small<E, 4, 1>(g, grid, kw, s);
-    return mt == 1 ? launch_small<E, 1, 2>(g, grid, kw, s) : mt == 2 ? launch_small<E, 2, 2>(g, grid, kw, s) : launch_small<E, 4, 2>(g, grid, kw, s);
+    if (J == 1) return mt == 1 ? launch_small<E, 1, 1>(g, grid, nw, kw, s) : mt == 2 ? launch_small<E, 2, 1>(g, grid, nw, kw, s) : launch_small<E, 4, 1>(g, grid, nw, kw, s);
+    return mt == 1 ? launch_small<E, 1, 2>(g, grid, nw, kw, s) : mt == 2 ? launch_small<E, 2, 2>(g, grid, nw, kw, s) : launch_small<E, 4, 2>(g, grid, nw, kw, s);
 }
 template int tiled_gemm<bf16>(const TiledGemm<bf16>&, hipStream_t);
 template int tiled_gemm<float>(const TiledGemm<float>&, hipStream_t);
