@@ -22,24 +22,32 @@
 
 namespace fh {
 
-// rotate the pairs (2i, 2i + 1) of 8 consecutive values starting at dimension d0, position `pos`; dims past rot_dims pass
-template <typename V>
-__device__ __forceinline__ V rotate8(V x, int d0, int rot_dims, const float* __restrict__ cos_t, const float* __restrict__ sin_t, long pos) {
+// cosines and sines of the four pairs (2i, 2i + 1) starting at dimension d0, position `pos`; pairs past rot_dims pass unchanged
+struct Rot4 { float c[4], s[4]; };
+__device__ __forceinline__ Rot4 rot_load(int d0, int rot_dims, const float* __restrict__ cos_t, const float* __restrict__ sin_t, long pos) {
     const int half = rot_dims >> 1;
-    if (half == 0) return x;
-    float c[4], s[4];
+    Rot4 r;
 #pragma unroll
     for (int j = 0; j < 4; j++) {
         const int i = (d0 >> 1) + j;
-        const float cv = cos_t[pos * half + (i < half ? i : half - 1)], sv = sin_t[pos * half + (i < half ? i : half - 1)];
-        c[j] = i < half ? cv : 1.f;
-        s[j] = i < half ? sv : 0.f;
+        r.c[j] = 1.f;
+        r.s[j] = 0.f;
+        if (half > 0) {                                  // (uniform; the loads themselves are unconditional, clamped)
+            const long o = pos * half + (i < half ? i : half - 1);
+            const float cv = cos_t[o], sv = sin_t[o];
+            r.c[j] = i < half ? cv : 1.f;
+            r.s[j] = i < half ? sv : 0.f;
+        }
     }
+    return r;
+}
+template <typename V>
+__device__ __forceinline__ V rot_apply(V x, const Rot4& r) {
 #pragma unroll
     for (int j = 0; j < 4; j++) {
         const float u = (float)x[2 * j], w = (float)x[2 * j + 1];
-        x[2 * j] = u * c[j] - w * s[j];
-        x[2 * j + 1] = w * c[j] + u * s[j];
+        x[2 * j] = u * r.c[j] - w * r.s[j];
+        x[2 * j + 1] = w * r.c[j] + u * r.s[j];
     }
     return x;
 }
@@ -80,7 +88,7 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(const E* __restrict
 #pragma unroll
             for (int j = 0; j < 8; j++) x[j] = (E)((float)x[j] * ik * dkv_norm[i + j]);
         } else {
-            x = rotate8(x, i - d.kp, d.rot_dims, b.cos_t, b.sin_t, pos);
+            x = rot_apply(x, rot_load(i - d.kp, d.rot_dims, b.cos_t, b.sin_t, pos));
         }
         *reinterpret_cast<v8*>(tile + i * 16) = x;
     }
@@ -230,26 +238,29 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(LatentDims d, Laten
     const int st_lo = nstep * (int)blockIdx.x / nsplit, st_hi = nstep * ((int)blockIdx.x + 1) / nsplit;
     const int32_t* bt = v.bt + (long)w.seq * v.max_blocks;
 
+    // block-table entries of this wave's blocks, 64 steps per load; then nothing of the step loop waits for the table
     bf16x8 kf[KS + RS], qf[KS + RS];
+    auto table = [&](int st) { return bt[min(blk_lo + 4 * (st + lane) + wave, blk_hi - 1)]; };
+    int bt_st = st_lo, btv = table(st_lo);
     auto load = [&](int st) {                                                  // (past the last block: a copy of it, masked below)
-        const bf16* t = p.pool + (long)bt[min(blk_lo + 4 * st + wave, blk_hi - 1)] * 16 * kd + lane * 8;
+        const bf16* t = p.pool + (long)__builtin_amdgcn_readlane(btv, min(st - bt_st, 63)) * 16 * kd + lane * 8;
 #pragma unroll
-        for (int s = 0; s < KS; s++)
-            kf[s] = *reinterpret_cast<const bf16x8*>(t + s * 512);
-#pragma unroll
-        for (int s = 0; s < RS; s++)
-            kf[KS + s] = *reinterpret_cast<const bf16x8*>(t + (KS + s) * 512);
+        for (int s = 0; s < KS + RS; s++) kf[s] = *reinterpret_cast<const bf16x8*>(t + s * 512);
     };
-    load(st_lo);                                                               // (no load under a condition: it would drain the others)
     {
+        // the rotated part first: its values and angles travel together with the table entries, in front of the latents
         const long qrow = (long)(w.tok0 + tl) * d.heads + h;
+        Rot4 rot[RS];
 #pragma unroll
-        for (int s = 0; s < KS; s++)
-            qf[s] = *reinterpret_cast<const bf16x8*>(p.q_lat + qrow * (32 * KS) + 32 * s + 8 * a);
+        for (int s = 0; s < RS; s++) {
+            qf[KS + s] = *reinterpret_cast<const bf16x8*>(p.q + qrow * (d.dp + d.rp) + d.dp + 32 * s + 8 * a);
+            rot[s] = rot_load(32 * s + 8 * a, d.rot_dims, p.cos_t, p.sin_t, row_pos);
+        }
+        load(st_lo);                                                           // (no load under a condition: it would drain the others)
 #pragma unroll
-        for (int s = 0; s < RS; s++)
-            qf[KS + s] = rotate8(*reinterpret_cast<const bf16x8*>(p.q + qrow * (d.dp + d.rp) + d.dp + 32 * s + 8 * a), 32 * s + 8 * a,
-                                     d.rot_dims, p.cos_t, p.sin_t, row_pos);
+        for (int s = 0; s < KS; s++) qf[s] = *reinterpret_cast<const bf16x8*>(p.q_lat + qrow * (32 * KS) + 32 * s + 8 * a);
+#pragma unroll
+        for (int s = 0; s < RS; s++) qf[KS + s] = rot_apply(qf[KS + s], rot[s]);
     }
     const int tr_off = tr_offset(lane);
     float m_run = -INFINITY, l_run = 0.f;
@@ -278,6 +289,7 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(LatentDims d, Laten
         for (int s = 0; s < KS; s++)
             *reinterpret_cast<bf16x8*>(stage + wave * STAGE + s * 512 + lane * 8) = kf[s];
         if (a == 0) lds_m[wave * 16 + b] = mx;
+        if (st + 1 - bt_st == 64) { bt_st = st + 1; btv = table(bt_st); }
         load(st + 1);
         __syncthreads();
         const float m_new = fmaxf(m_run, fmaxf(fmaxf(lds_m[b], lds_m[16 + b]), fmaxf(lds_m[32 + b], lds_m[48 + b])));
@@ -294,16 +306,17 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(LatentDims d, Laten
 #pragma unroll
             for (int r = 0; r < 4; r++) o[t][r] *= alpha;
         __syncthreads();
-        // Oᵀ[d][row] += Vᵀ[d][key]·Pᵀ[key][row], 32 keys (two blocks) at a time: lane group a takes keys 8a … 8a + 7 of them
+        // Oᵀ[d][row] += Vᵀ[d][key]·Pᵀ[key][row], 32 keys (two blocks) at a time: contraction index (a, j < 4) = key 4a + j of the first
+        // block, (a, j ≥ 4) = key 4a + j − 4 of the second — a transposed read then covers 512 contiguous bytes
 #pragma unroll
         for (int c = 0; c < 2; c++) {
-            const bf16x8 pv = *reinterpret_cast<const bf16x8*>(lds_p + b * PSTR + c * 32 + 8 * a);
-            // keys 8a … of the pair sit in block 2c + (a >> 1), rows (a & 1)·8: the lane's read names those instead of rows 4a
-            const bf16* vb = stage + (2 * c + (a >> 1)) * STAGE + tr_off + ((a & 1) * 8 - 4 * a) * 8;
+            const bf16x4 p0 = *reinterpret_cast<const bf16x4*>(lds_p + b * PSTR + c * 32 + 4 * a), p1 = *reinterpret_cast<const bf16x4*>(lds_p + b * PSTR + c * 32 + 16 + 4 * a);
+            const bf16x8 pv = {p0[0], p0[1], p0[2], p0[3], p1[0], p1[1], p1[2], p1[3]};
+            const bf16* vb = stage + 2 * c * STAGE + tr_off;
 #pragma unroll
             for (int t = 0; t < DT; t++)
                 if (KS >= 2 || wave < 2 * KS) {
-                    const shortx4 v0 = read_tr(vb + (wave + 4 * t) * 256), v1 = read_tr(vb + (wave + 4 * t) * 256 + 32);
+                    const shortx4 v0 = read_tr(vb + (wave + 4 * t) * 256), v1 = read_tr(vb + STAGE + (wave + 4 * t) * 256);
                     typedef short shortx8 __attribute__((ext_vector_type(8)));
                     const shortx8 vt = {v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
                     o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, vt), pv, o[t], 0, 0, 0);
@@ -334,21 +347,30 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(LatentDims d, Laten
             *reinterpret_cast<bf16x4*>(dst + (wave + 4 * t) * 16 + 4 * a) = y;
         }
 }
-// grid (row tiles, quads of output dimensions / 256): one thread per (row, 4 dimensions)
-__global__ __launch_bounds__(256) void latent_attn_reduce_kernel(LatentDims d, LatentBuffers<bf16> p, BatchView v, int nsplit) {
+// grid (row tiles, quads of output dimensions / 256): one thread per (row, 4 dimensions); every load is in flight at once
+template <int NS>
+__global__ __launch_bounds__(256) void latent_attn_reduce_kernel(LatentDims d, LatentBuffers<bf16> p, BatchView v) {
     LatentTile w;
     if (!find_latent_tile(v, d.heads, blockIdx.x, &w)) return;
     const int quads = d.kp >> 2, id = blockIdx.y * 256 + threadIdx.x, row = id / quads, c = (id % quads) * 4, ro = w.tile * 16 + row;
     if (row >= 16 || ro >= w.q_len * d.heads) return;
     const long ld = d.kp + LATENT_PARTIAL_PAD;
-    const float* src = p.partial + ((long)blockIdx.x * nsplit * 16 + row) * ld;
-    float M = -INFINITY, L = 0.f;
-    for (int z = 0; z < nsplit; z++) M = fmaxf(M, src[z * 16 * ld + d.kp]);
-    floatx4 acc = {0.f, 0.f, 0.f, 0.f};
-    for (int z = 0; z < nsplit; z++) {
-        const float f = __expf(src[z * 16 * ld + d.kp] - M);
-        L += src[z * 16 * ld + d.kp + 1] * f;
-        acc += *reinterpret_cast<const floatx4*>(src + z * 16 * ld + c) * f;
+    const float* src = p.partial + ((long)blockIdx.x * NS * 16 + row) * ld;
+    float m[NS], l[NS], M = -INFINITY, L = 0.f;
+    floatx4 o[NS], acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int z = 0; z < NS; z++) {
+        m[z] = src[z * 16 * ld + d.kp];
+        l[z] = src[z * 16 * ld + d.kp + 1];
+        o[z] = *reinterpret_cast<const floatx4*>(src + z * 16 * ld + c);
+    }
+#pragma unroll
+    for (int z = 0; z < NS; z++) M = fmaxf(M, m[z]);
+#pragma unroll
+    for (int z = 0; z < NS; z++) {
+        const float f = __expf(m[z] - M);
+        L += l[z] * f;
+        acc += o[z] * f;
     }
     const float inv = 1.0f / L;
     bf16x4 y;
@@ -391,7 +413,7 @@ __global__ __launch_bounds__(256, 2) void latent_expanded_kernel(LatentDims d, L
             qf[mt][s] = *reinterpret_cast<const bf16x8*>(q + 32 * s);
 #pragma unroll
         for (int s = 0; s < RS; s++)
-            qf[mt][DS + s] = rotate8(*reinterpret_cast<const bf16x8*>(q + d.dp + 32 * s), 32 * s + 8 * a, d.rot_dims, p.cos_t, p.sin_t, row_pos[mt]);
+            qf[mt][DS + s] = rot_apply(*reinterpret_cast<const bf16x8*>(q + d.dp + 32 * s), rot_load(32 * s + 8 * a, d.rot_dims, p.cos_t, p.sin_t, row_pos[mt]));
     }
     const int t_hi = min(q_len, tile0 + LATENT_TILE_TOKENS);
     const int blk_lo = max(0, pos0 + tile0 + 1 - d.window) / 16, blk_hi = (pos0 + t_hi + 15) / 16, nstep = (blk_hi - blk_lo + 3) / 4;
@@ -540,10 +562,11 @@ static int latent_plain(const LatentDims& d, const LatentBuffers<E>& b, const Ba
 static int latent_mfma(const LatentDims& d, const LatentBuffers<bf16>& b, const BatchView& v, hipStream_t s) {
     const int tiles = v.single ? v.num_seqs * cdiv(d.heads, 16) : (int)(((long)v.T * d.heads) / 16) + v.num_seqs;      // upper bound of Σ ceil(rows / 16)
     const int keys = std::min(v.max_keys, d.window + 16);
-    // split the keys while the launch has fewer than ≈ 1 workgroup per CU and a split keeps ≥ 256 keys (four steps)
+    // split the keys while the launch has fewer than 2 workgroups per CU (what stays resident) and a split keeps ≥ 128 keys (two steps)
     int ns = 1;
-    while (ns < 16 && tiles * ns < 256 && keys >= 2 * ns * 256) ns *= 2;
-    if (knobs().latent_splits > 0) ns = std::min(16, knobs().latent_splits);
+    while (ns < 16 && tiles * ns < 512 && keys >= 2 * ns * 128) ns *= 2;
+    if (knobs().latent_splits > 0)
+        for (ns = 1; ns < std::min(16, knobs().latent_splits); ns *= 2) {}
     while (ns > 1 && (size_t)tiles * ns * 16 * (d.kp + LATENT_PARTIAL_PAD) * 4 > b.partial_bytes) ns /= 2;
     const dim3 grid(ns, tiles);          // (splits fastest: the row tiles of a sequence read a key range on the same XCD)
     form_hit(ns > 1 ? FORM_LATENT_ATTN_SPLIT : FORM_LATENT_ATTN);
@@ -563,7 +586,11 @@ static int latent_mfma(const LatentDims& d, const LatentBuffers<bf16>& b, const 
 #undef LATENT
     FH_CHECK_LAUNCH();
     if (ns > 1) {
-        hipLaunchKernelGGL(latent_attn_reduce_kernel, dim3(tiles, cdiv(16 * (d.kp / 4), 256)), dim3(256), 0, s, d, b, v, ns);
+        const dim3 rg(tiles, cdiv(16 * (d.kp / 4), 256));
+        if (ns == 2) hipLaunchKernelGGL(latent_attn_reduce_kernel<2>, rg, dim3(256), 0, s, d, b, v);
+        else if (ns == 4) hipLaunchKernelGGL(latent_attn_reduce_kernel<4>, rg, dim3(256), 0, s, d, b, v);
+        else if (ns == 8) hipLaunchKernelGGL(latent_attn_reduce_kernel<8>, rg, dim3(256), 0, s, d, b, v);
+        else hipLaunchKernelGGL(latent_attn_reduce_kernel<16>, rg, dim3(256), 0, s, d, b, v);
         FH_CHECK_LAUNCH();
     }
     return 0;

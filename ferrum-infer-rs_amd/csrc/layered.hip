@@ -170,8 +170,8 @@ public:
                 L.in_nsec = 3;
                 q_cols = std::max<long>(q_cols, L.uq.n); lat_cols = std::max<long>(lat_cols, (long)H * d.kp);
                 attn_cols = std::max<long>(attn_cols, (long)H * vp); cq_cols = std::max<long>(cq_cols, d.qp);
-                // split attention: only while a forward has fewer than 256 row tiles
-                partial = std::max<size_t>(partial, (size_t)512 * 16 * (d.kp + 4) * 4 * 2);
+                // split attention: (row tile, split) pairs stay below 1024
+                partial = std::max<size_t>(partial, (size_t)1024 * 16 * (d.kp + 4) * 4);
             } else {
                 const RglruDims& d = L.rd;
                 const int bs = sp.rnn_width / d.blocks, bp = d.bp, W = sp.rnn_width;
