@@ -213,7 +213,7 @@ __device__ __forceinline__ shortx4 read_tr(const bf16* p) {
     return __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) shortx4*)p);
 }
 
-// KS, RS: 32-wide steps of the latent and of the rotated part.  grid (KV splits, row tiles); a step is 64 keys: wave w scores block w of them
+// KS, RS: 32-wide steps of the latent and of the rotated part.  grid (row tiles × KV splits); a step is 64 keys: wave w scores block w of them
 // for all 16 rows, the row maxima meet in LDS, P and the parked latents are shared, and each wave accumulates its own quarter of the
 // output dimensions — so nothing is merged at the end and the latents of the next step are in flight during softmax and P·V.
 template <int KS, int RS>
@@ -224,8 +224,9 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(LatentDims d, Laten
     __shared__ __attribute__((aligned(16))) bf16 lds_p[16 * PSTR];
     __shared__ float lds_m[64], lds_l[64];
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, a = lane >> 4, b = lane & 15;
+    const int split = blockIdx.x % nsplit, tile_id = blockIdx.x / nsplit;
     LatentTile w;
-    if (!find_latent_tile(v, d.heads, blockIdx.y, &w)) return;
+    if (!find_latent_tile(v, d.heads, tile_id, &w)) return;
     constexpr int kd = 32 * (KS + RS);
     const int rows = w.q_len * d.heads;
     const int rho = w.tile * 16 + b;
@@ -235,7 +236,7 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(LatentDims d, Laten
     const int t_first = w.tile * 16 / d.heads, t_last = min(w.q_len - 1, (w.tile * 16 + 15) / d.heads);
     const int kv_end = w.pos0 + t_last + 1, kv_lo = max(0, w.pos0 + t_first + 1 - d.window);
     const int blk_lo = kv_lo / 16, blk_hi = (kv_end + 15) / 16, nstep = (blk_hi - blk_lo + 3) / 4;
-    const int st_lo = nstep * (int)blockIdx.x / nsplit, st_hi = nstep * ((int)blockIdx.x + 1) / nsplit;
+    const int st_lo = nstep * split / nsplit, st_hi = nstep * (split + 1) / nsplit;
     const int32_t* bt = v.bt + (long)w.seq * v.max_blocks;
 
     // block-table entries of this wave's blocks, 64 steps per load; then nothing of the step loop waits for the table
@@ -328,7 +329,7 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(LatentDims d, Laten
     __syncthreads();
     const float L = lds_l[b] + lds_l[16 + b] + lds_l[32 + b] + lds_l[48 + b];
     if (nsplit > 1) {
-        float* dst = p.partial + (((long)blockIdx.y * nsplit + blockIdx.x) * 16 + b) * (32 * KS + LATENT_PARTIAL_PAD);
+        float* dst = p.partial + ((long)blockIdx.x * 16 + b) * (32 * KS + LATENT_PARTIAL_PAD);
 #pragma unroll
         for (int t = 0; t < DT; t++)
             if (KS >= 2 || wave < 2 * KS) *reinterpret_cast<floatx4*>(dst + (wave + 4 * t) * 16 + 4 * a) = o[t];
@@ -561,14 +562,14 @@ static int latent_plain(const LatentDims& d, const LatentBuffers<E>& b, const Ba
 }
 static int latent_mfma(const LatentDims& d, const LatentBuffers<bf16>& b, const BatchView& v, hipStream_t s) {
     const int tiles = v.single ? v.num_seqs * cdiv(d.heads, 16) : (int)(((long)v.T * d.heads) / 16) + v.num_seqs;      // upper bound of Σ ceil(rows / 16)
-    const int keys = std::min(v.max_keys, d.window + 16);
+    const int keys = (int)std::min<long>(v.max_keys, (long)d.window + 16);
     // split the keys while the launch has fewer than 2 workgroups per CU (what stays resident) and a split keeps ≥ 128 keys (two steps)
     int ns = 1;
     while (ns < 16 && tiles * ns < 512 && keys >= 2 * ns * 128) ns *= 2;
     if (knobs().latent_splits > 0)
         for (ns = 1; ns < std::min(16, knobs().latent_splits); ns *= 2) {}
     while (ns > 1 && (size_t)tiles * ns * 16 * (d.kp + LATENT_PARTIAL_PAD) * 4 > b.partial_bytes) ns /= 2;
-    const dim3 grid(ns, tiles);          // (splits fastest: the row tiles of a sequence read a key range on the same XCD)
+    const dim3 grid(ns * tiles);         // (splits fastest: the row tiles of a sequence read a key range on the same XCD)
     form_hit(ns > 1 ? FORM_LATENT_ATTN_SPLIT : FORM_LATENT_ATTN);
 #define LATENT(KS)                                                                                             \
     do {                                                                                                       \

@@ -321,6 +321,11 @@ struct Fields {
         if (!(d >= 0.0 && d <= 2147483647.0 && std::floor(d) == d)) { if (missing.empty()) missing = where + "." + key; return 0; }
         return (int32_t)d;
     }
+    int64_t integer(const char* key) {
+        const double d = num(key);
+        if (!(d >= 0.0 && d < 9007199254740992.0 && std::floor(d) == d)) { if (missing.empty()) missing = where + "." + key; return 0; }
+        return (int64_t)d;
+    }
     Fields sub(const char* key) { return Fields{obj ? obj->get(key) : nullptr, where + "." + key, missing}; }
 };
 #define FH_FIELDS_OK(f) FH_REQUIRE((f).missing.empty(), "config.json: '%s' is missing or not a valid number", (f).missing.c_str())
@@ -638,8 +643,8 @@ int ferrum_hip_checkpoint_layered_config(const FerrumHipCheckpoint* ck, int* is_
         if (const Value* bg = emb.obj ? emb.obj->get("bigram") : nullptr; bg && bg->kind == Value::Obj) {
             Fields b{bg, "embedding.bigram", ""};
             layered->bigram_buckets = b.size("buckets");
-            layered->bigram_mul_prev = b.size("mul_prev");
-            layered->bigram_mul_cur = b.size("mul_cur");
+            layered->bigram_mul_prev = b.integer("mul_prev");
+            layered->bigram_mul_cur = b.integer("mul_cur");
             FH_FIELDS_OK(b);
             FH_REQUIRE(layered->bigram_buckets > 0, "config.json: embedding.bigram.buckets must be positive");
         }

@@ -14,7 +14,7 @@ __global__ __launch_bounds__(256) void embed_bigram_kernel(const E* __restrict__
     if (bigram) {
         const int seq = v.tok_seq[t];
         const int64_t prev = t == (int)v.cu[seq] ? (int64_t)v.prev[seq] : (int64_t)v.tokens[t - 1];
-        row = prev < 0 ? buckets : (long)((uint64_t)(prev * mul_prev + (int64_t)tok * mul_cur) % (uint64_t)buckets);
+        row = prev < 0 ? buckets : (long)(((uint64_t)prev * (uint64_t)mul_prev + (uint64_t)tok * (uint64_t)mul_cur) % (uint64_t)buckets);
     }
     if (VEC) {
         typedef typename Frag<E>::v8 v8;

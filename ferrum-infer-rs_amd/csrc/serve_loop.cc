@@ -11,8 +11,10 @@
 //                   any prompt chunk go through ferrum_hip_model_decode_steps (hipGraph replay) for as many steps as no
 //                   request finishes or can be admitted
 //   * retirement  : ferrum_hip_model_release
+// `--model DIR` serves a checkpoint instead (any architecture the library reads; `--dtype bfloat16|float32` for layered ones), and
+// `--prompt-ids "5,17,3;8,9"` submits exactly these prompts.
 // Prints one JSON line: output tok/s over the whole run, TTFT p50/p99, iterations, and the KV pool state at exit (every
-// block must be back).  Synthetic weights (no checkpoints offline); `--layers` shrinks the model for smoke runs.
+// block must be back).  Without --model the weights are synthetic; `--layers` shrinks the model for smoke runs.
 #include <algorithm>
 #include <chrono>
 #include <cstdint>
@@ -36,6 +38,7 @@ struct Request {
     int out_len = 0;          // output tokens this request asks for
     double t_submit = 0, t_first = 0;
     std::vector<uint32_t> out;
+    int len() const { return (int)prompt.size(); }
 };
 
 double now_s() {
@@ -62,6 +65,28 @@ int arg_int(int argc, char** argv, const char* name, int dflt) {
         if (!std::strcmp(argv[i], name)) return std::atoi(argv[i + 1]);
     return dflt;
 }
+const char* arg_str(int argc, char** argv, const char* name) {
+    for (int i = 1; i + 1 < argc; i++)
+        if (!std::strcmp(argv[i], name)) return argv[i + 1];
+    return nullptr;
+}
+// "5,17,3;8,9" → prompts; false on anything that is not a list of numbers
+bool parse_prompts(const char* text, std::vector<std::vector<uint32_t>>& out) {
+    out.assign(1, {});
+    for (const char* p = text; *p;) {
+        char* end = nullptr;
+        const unsigned long v = std::strtoul(p, &end, 10);
+        if (end == p) return false;
+        out.back().push_back((uint32_t)v);
+        p = end;
+        if (*p == ';') out.emplace_back();
+        if (*p == ';' || *p == ',') p++;
+        else if (*p) return false;
+    }
+    for (const auto& v : out)
+        if (v.empty()) return false;
+    return true;
+}
 bool arg_flag(int argc, char** argv, const char* name) {
     for (int i = 1; i < argc; i++)
         if (!std::strcmp(argv[i], name)) return true;
@@ -82,6 +107,14 @@ int main(int argc, char** argv) {
     const int dense = arg_flag(argc, argv, "--dense");          // Llama-3.1-8B dims instead of Qwen3-30B-A3B
     const bool dump = arg_flag(argc, argv, "--dump-tokens");
     uint64_t seed = (uint64_t)arg_int(argc, argv, "--seed", 9271);
+    const char *model_dir = arg_str(argc, argv, "--model"), *dtype = arg_str(argc, argv, "--dtype"), *prompt_ids = arg_str(argc, argv, "--prompt-ids");
+    std::vector<std::vector<uint32_t>> given;
+    if ((prompt_ids && !parse_prompts(prompt_ids, given)) || (dtype && std::strcmp(dtype, "bfloat16") && std::strcmp(dtype, "float32"))) {
+        std::fprintf(stderr, "bad --prompt-ids or --dtype\n");
+        return 2;
+    }
+    int longest = given.empty() ? PL : 0;
+    for (const auto& p : given) longest = std::max(longest, (int)p.size());
     if (conc < 1 || PL < 1 || OL < 1 || budget < conc || num_requests < 1 || jitter < 0 || jitter >= OL) {
         std::fprintf(stderr, "bad arguments\n");
         return 2;
@@ -99,26 +132,57 @@ int main(int argc, char** argv) {
         cfg.vocab = 151936; cfg.has_qk_norm = 1; cfg.num_experts = 128; cfg.top_k = 8; cfg.expert_inter = 768;
         cfg.norm_topk_prob = 1; cfg.rope_theta = 1000000.0;
     }
-    const int seq_cap = ((PL + OL + jitter + 15) / 16) * 16;
-    cfg.max_seq_len = seq_cap;
-    cfg.group_size = 128;
+    const int seq_cap = ((longest + OL + jitter + 15) / 16) * 16;
+    FerrumHipCheckpoint* ck = nullptr;
+    int layered = 0;
+    FerrumHipLayeredConfig lc;
+    std::vector<FerrumHipLayerSpec> specs;
+    char arch[128] = "";
+    if (model_dir) {
+        CHECK(ferrum_hip_checkpoint_open(&ck, model_dir));
+        CHECK(ferrum_hip_checkpoint_model_config(ck, seq_cap, &cfg, arch, sizeof(arch), nullptr));
+        specs.resize((size_t)cfg.num_layers);
+        CHECK(ferrum_hip_checkpoint_layered_config(ck, &layered, &lc, specs.data(), cfg.num_layers));
+        if (!layered && dtype && !std::strcmp(dtype, "float32")) {
+            std::fprintf(stderr, "%s runs in 16 bits only\n", arch);
+            return 2;
+        }
+    } else {
+        cfg.max_seq_len = seq_cap;
+        cfg.group_size = 128;
+        cfg.rms_eps = 1e-6f;
+        cfg.tp_world = 1;
+    }
     cfg.kv_num_blocks = kv_blocks > 0 ? kv_blocks : (conc + 2) * (seq_cap / 16);
     cfg.max_seqs = conc;
     cfg.max_tokens = budget;
-    cfg.rms_eps = 1e-6f;
-    cfg.tp_world = 1;
 
     FerrumHipModel* model = nullptr;
-    CHECK(ferrum_hip_model_create(&model, &cfg));
-    CHECK(ferrum_hip_model_init_synthetic(model, seed));
+    if (layered) {
+        lc.dtype = dtype && !std::strcmp(dtype, "float32") ? FERRUM_HIP_DTYPE_F32 : FERRUM_HIP_DTYPE_BF16;
+        lc.state_slots = arg_int(argc, argv, "--state-slots", conc);      // fewer than the concurrency: admission waits for a slot
+        CHECK(ferrum_hip_model_create_layered(&model, &cfg, &lc, specs.data()));
+    } else {
+        CHECK(ferrum_hip_model_create(&model, &cfg));
+    }
+    if (ck) {
+        CHECK(ferrum_hip_model_load_checkpoint(model, ck));
+        ferrum_hip_checkpoint_close(ck);
+    } else {
+        CHECK(ferrum_hip_model_init_synthetic(model, seed));
+    }
     CHECK(ferrum_hip_model_finalize(model));
 
     std::deque<Request> pending;
-    for (int i = 0; i < num_requests; i++) {
+    const uint32_t first_id = cfg.vocab > 512 ? 256u : 0u;
+    for (int i = 0; i < (given.empty() ? num_requests : (int)given.size()); i++) {
         Request r;
         r.id = 1 + (uint64_t)i;
-        r.prompt.resize(PL);
-        for (int t = 0; t < PL; t++) r.prompt[t] = 256u + (uint32_t)(splitmix(seed) % (uint64_t)(cfg.vocab - 256));
+        if (!given.empty()) r.prompt = given[i];
+        else {
+            r.prompt.resize(PL);
+            for (int t = 0; t < PL; t++) r.prompt[t] = first_id + (uint32_t)(splitmix(seed) % (uint64_t)(cfg.vocab - first_id));
+        }
         r.out_len = jitter ? OL - jitter + (int)(splitmix(seed) % (uint64_t)(2 * jitter + 1)) : OL;
         pending.push_back(std::move(r));
     }
@@ -133,7 +197,7 @@ int main(int argc, char** argv) {
     while (!pending.empty() || !running.empty()) {
         // admission: closed loop — a client submits as soon as a slot AND the KV footprint of a whole request are free
         while ((int)running.size() < conc && !pending.empty()) {
-            FerrumHipKvSlotRequest rq{pending.front().id, PL + pending.front().out_len, 0};
+            FerrumHipKvSlotRequest rq{pending.front().id, (int)pending.front().prompt.size() + pending.front().out_len, 0};
             FerrumHipKvSlotReservation rs;
             if (ferrum_hip_model_reserve_kv_slots(model, &rq, 1, &rs) != 0) break;      // pool full: retry after a retirement
             pending.front().t_submit = now_s();
@@ -145,7 +209,7 @@ int main(int argc, char** argv) {
             return 1;
         }
         bool any_prefill = false;
-        for (const Request& r : running) any_prefill |= r.prefilled < PL;
+        for (const Request& r : running) any_prefill |= r.prefilled < r.len();
 
         if (!any_prefill) {
             // pure decode: hipGraph replay for as many steps as nothing can change the batch (no retirement before the
@@ -174,8 +238,8 @@ int main(int argc, char** argv) {
             int left = budget;
             for (size_t i = 0; i < running.size(); i++) {
                 Request& r = running[i];
-                if (r.prefilled == PL) {
-                    items.push_back(FerrumHipBatchItem{r.id, &r.last_token, 1, PL + r.generated - 1, 1, 0});
+                if (r.prefilled == r.len()) {
+                    items.push_back(FerrumHipBatchItem{r.id, &r.last_token, 1, r.len() + r.generated - 1, 1, 0});
                     owner.push_back((int)i);
                     chunk.push_back(0);
                     left--;
@@ -183,10 +247,10 @@ int main(int argc, char** argv) {
             }
             for (size_t i = 0; i < running.size() && left > 0; i++) {
                 Request& r = running[i];
-                if (r.prefilled < PL) {
-                    const int n = std::min(PL - r.prefilled, left);
+                if (r.prefilled < r.len()) {
+                    const int n = std::min(r.len() - r.prefilled, left);
                     items.push_back(FerrumHipBatchItem{r.id, r.prompt.data() + r.prefilled, n, r.prefilled,
-                                                       r.prefilled + n == PL ? 1 : 0, 0});
+                                                       r.prefilled + n == r.len() ? 1 : 0, 0});
                     owner.push_back((int)i);
                     chunk.push_back(n);
                     left -= n;
@@ -229,7 +293,7 @@ int main(int argc, char** argv) {
                 "\"concurrency\": %d, \"prompt_len\": %d, \"out_len\": %d, \"max_batched_tokens\": %d, \"out_len_jitter\": %d, \"output_tokens\": %ld, "
                 "\"wall_s\": %.4f, \"output_tok_s\": %.1f, \"ttft_ms_p50\": %.2f, \"ttft_ms_p99\": %.2f, \"iterations\": %ld, "
                 "\"mixed_iterations\": %ld, \"graph_decode_steps\": %ld, \"kv_blocks_total\": %d, \"kv_blocks_free_at_exit\": %d}\n",
-                dense ? "llama31-8b" : "qwen3-30b-a3b", layers, num_requests, conc, PL, OL, budget, jitter, out_tokens, wall,
+                model_dir ? arch : dense ? "llama31-8b" : "qwen3-30b-a3b", cfg.num_layers, (int)finished.size(), conc, PL, OL, budget, jitter, out_tokens, wall,
                 (double)out_tokens / wall, ttft[ttft.size() / 2], ttft[std::min(ttft.size() - 1, ttft.size() * 99 / 100)],
                 iterations, mixed_iterations, graph_steps, cap.total_blocks, cap.free_blocks_after);
     if (dump) {
@@ -240,6 +304,8 @@ int main(int argc, char** argv) {
             std::printf("\n");
         }
     }
+    int slots = 0, free_slots = 0;
+    CHECK(ferrum_hip_model_state_slots(model, &slots, &free_slots));
     CHECK(ferrum_hip_model_destroy(model));
-    return cap.free_blocks_after == cap.total_blocks ? 0 : 3;
+    return cap.free_blocks_after == cap.total_blocks && free_slots == slots ? 0 : 3;
 }

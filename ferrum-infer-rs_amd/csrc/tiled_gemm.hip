@@ -10,12 +10,17 @@
 namespace fh {
 
 template <typename E>
+__device__ __forceinline__ float gemm_act(const GemmSection& sec, float v) {
+    if (sec.act == GEMM_ACT_SIGMOID) return ActMath<E>::sigmoid(v);
+    if (sec.act == GEMM_ACT_GELU_TANH) return gelu_tanh_f32<E>(v);
+    if (sec.act == GEMM_ACT_XIELU) return xielu_f32<E>(v, sec.p, sec.q);
+    return v;
+}
+template <typename E>
 __device__ __forceinline__ void gemm_epilogue(const TiledGemm<E>& p, const GemmSection& sec, int g, int row, int col, float v) {
     if (row >= p.m || col >= p.n_store) return;
     if (p.bias) v += p.bias[(long)g * p.n + col];
-    if (sec.act == GEMM_ACT_SIGMOID) v = ActMath<E>::sigmoid(v);
-    else if (sec.act == GEMM_ACT_GELU_TANH) v = gelu_tanh_f32<E>(v);
-    else if (sec.act == GEMM_ACT_XIELU) v = xielu_f32<E>(v, sec.p, sec.q);
+    v = gemm_act<E>(sec, v);
     if (p.row_scale) v *= (float)p.row_scale[row * p.ld_scale + g];
     const long o = row * p.ldo + g * p.out_group + col;
     if (p.out_f32) p.out_f32[o] = v; else p.out[o] = (E)v;
@@ -197,6 +202,55 @@ __global__ __launch_bounds__(256, 2) void tiled_gemm_big_kernel(TiledGemm<bf16> 
         }
         asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
         __syncthreads();
+    }
+    // epilogue: activations on the accumulators, then through LDS (the stages are free; a wave's 64 × 64 tile is its own) so that rows
+    // leave in 16-byte pieces, 128 or 256 contiguous bytes per row
+    if (p.n_store % 8 == 0 && p.ldo % 8 == 0 && p.out_group % 8 == 0) {
+        bf16* lo = &lds[0][0] + wave * 64 * 72;                    // rows of 72: 36 KiB for the four waves
+        float* lf = reinterpret_cast<float*>(&lds[0][0]) + wave * 32 * 68;      // fp32 outputs: 32 rows of 68 at a time
+#pragma unroll
+        for (int half = 0; half < 2; half++) {
+#pragma unroll
+            for (int j = 0; j < 4; j++) {
+                const int col0 = n0 + wn * 64 + j * 16;
+                const GemmSection sec = gemm_section(p, min(col0, p.n - 1));
+                const float bias = p.bias ? p.bias[(long)g * p.n + min(col0 + b, p.n - 1)] : 0.f;
+#pragma unroll
+                for (int i = 2 * half; i < 2 * half + 2; i++)
+#pragma unroll
+                    for (int r = 0; r < 4; r++) {
+                        const float v = gemm_act<bf16>(sec, acc[i][j][r] + bias);
+                        if (p.out_f32) lf[((i & 1) * 16 + 4 * a + r) * 68 + j * 16 + b] = v;
+                        else lo[(i * 16 + 4 * a + r) * 72 + j * 16 + b] = (bf16)v;
+                    }
+            }
+            if (p.out_f32) {                                       // (wave-private: LDS operations of a wave complete in order)
+#pragma unroll
+                for (int q = 0; q < 8; q++) {
+                    const int row = q * 4 + (lane >> 4), col = (lane & 15) * 4, gr = m0 + wm * 64 + half * 32 + row, gc = n0 + wn * 64 + col;
+                    if (gr < p.m && gc < p.n_store) {
+                        floatx4 v = *reinterpret_cast<const floatx4*>(lf + row * 68 + col);
+                        if (p.row_scale) v *= (float)p.row_scale[gr * p.ld_scale + g];
+                        *reinterpret_cast<floatx4*>(p.out_f32 + gr * p.ldo + g * p.out_group + gc) = v;
+                    }
+                }
+            }
+        }
+        if (p.out_f32) return;
+#pragma unroll
+        for (int q = 0; q < 8; q++) {
+            const int row = q * 8 + (lane >> 3), col = (lane & 7) * 8, gr = m0 + wm * 64 + row, gc = n0 + wn * 64 + col;
+            if (gr < p.m && gc < p.n_store) {
+                bf16x8 v = *reinterpret_cast<const bf16x8*>(lo + row * 72 + col);
+                if (p.row_scale) {
+                    const float f = (float)p.row_scale[gr * p.ld_scale + g];
+#pragma unroll
+                    for (int e = 0; e < 8; e++) v[e] = (bf16)((float)v[e] * f);
+                }
+                *reinterpret_cast<bf16x8*>(p.out + gr * p.ldo + g * p.out_group + gc) = v;
+            }
+        }
+        return;
     }
 #pragma unroll
     for (int j = 0; j < 4; j++) {

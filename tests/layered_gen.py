@@ -1,0 +1,109 @@
+"""Small random Nerenex models for the tests: configuration, weights (bfloat16-representable), checkpoint directories."""
+import json
+import os
+import struct
+
+import numpy as np
+
+
+def bf16(a):
+    """Round to bfloat16 and back (nearest even)."""
+    u = np.ascontiguousarray(a, np.float32).view(np.uint32).astype(np.uint64)
+    return (((u + 0x7FFF + ((u >> 16) & 1)) & 0xFFFF0000).astype(np.uint32)).view(np.float32)
+
+
+def attention(heads, dim, rot_dim, vdim, q_rank, kv_rank, window, base=10000.0, scale=None, ff=None):
+    return {"type": "latent_attention", "mlp": {"kind": "dense", "ff": ff} if ff else None,
+            "mixer": {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "q_rank": q_rank, "kv_rank": kv_rank,
+                      "mask": {"size": window}, "rot": {"base": base, "dims": rot_dim}, "scale": scale or (dim + rot_dim) ** -0.5}}
+
+
+def recurrent(width, blocks, conv, ff=None):
+    return {"type": "rglru", "mlp": {"kind": "dense", "ff": ff} if ff else None, "mixer": {"width": width, "blocks": blocks, "conv": conv}}
+
+
+def config(width, vocab, layers, eps=1e-5, mult=0.8, buckets=97, mul_prev=31, mul_cur=5):
+    return {"architecture": "Nerenex", "width": width, "vocab": vocab, "norm": {"eps": eps}, "residual_mult": mult, "layers": layers,
+            "embedding": {"bigram": {"buckets": buckets, "mul_prev": mul_prev, "mul_cur": mul_cur}}}
+
+
+CONFIGS = {
+    # nothing is a multiple of 32; value size, query size and ranks all differ; attention without, recurrence with a feed-forward
+    "odd": config(100, 131, [attention(3, 20, 6, 36, 44, 52, 21, base=500.0), recurrent(66, 3, 3, ff=75), attention(5, 9, 10, 12, 31, 70, 50, ff=41)],
+                  eps=1e-3, mult=0.45),
+    # several heads tiles, a rank of more than one padded size, one recurrent block, a long window
+    "wide": config(288, 260, [recurrent(256, 1, 2, ff=416), attention(20, 64, 32, 48, 192, 256, 130, ff=416), recurrent(192, 6, 5)], mult=0.6),
+    # the largest compile-time extents of the attention kernels
+    "deep": config(320, 203, [attention(16, 128, 64, 128, 160, 512, 90, base=1e6), attention(7, 96, 40, 120, 72, 300, 33, ff=130)], eps=1e-6, mult=0.9),
+    "tiny": config(40, 61, [recurrent(24, 2, 1, ff=33), attention(2, 8, 4, 8, 16, 24, 7, ff=50), attention(1, 12, 2, 20, 8, 9, 1)], buckets=11),
+}
+
+
+def weights(cfg, seed):
+    rng = np.random.default_rng(seed)
+    D, V = cfg["width"], cfg["vocab"]
+    w = {}
+
+    def mat(name, *shape, std=None):
+        w[name] = bf16(rng.standard_normal(shape) * (std or shape[-1] ** -0.5))
+
+    def vec(name, *shape, std=0.2, mean=0.0):
+        w[name] = bf16(mean + std * rng.standard_normal(shape))
+
+    mat("embed", V, D, std=1.0)
+    mat("bigram", cfg["embedding"]["bigram"]["buckets"] + 1, D, std=0.7)
+    vec("final.norm", D)
+    for i, layer in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", layer["mixer"]
+        vec(p + "norm1", D)
+        mat(p + "rg1", D, D)
+        vec(p + "rg1.b", D)
+        x = p + "mix."
+        if layer["type"] == "latent_attention":
+            H = m["heads"]
+            mat(x + "dq", m["q_rank"], D)
+            vec(x + "dq.norm", m["q_rank"], mean=1.0)
+            mat(x + "uq", H * (m["dim"] + m["rot_dim"]), m["q_rank"], std=1.6 * m["q_rank"] ** -0.5)
+            mat(x + "dkv", m["kv_rank"] + m["rot_dim"], D)
+            vec(x + "dkv.norm", m["kv_rank"], mean=1.0)
+            mat(x + "uk", H * m["dim"], m["kv_rank"], std=1.6 * m["kv_rank"] ** -0.5)
+            mat(x + "uv", H * m["vdim"], m["kv_rank"])
+            mat(x + "g", H, D)
+            mat(x + "o", D, H * m["vdim"])
+        else:
+            W, b = m["width"], m["blocks"]
+            for n in ("y", "x"):
+                mat(x + n, W, D)
+                vec(x + n + ".b", W)
+            mat(x + "conv", W, m["conv"], std=0.6)
+            vec(x + "conv.b", W)
+            for n in ("ra", "ri"):
+                mat(x + n, b, W // b, W // b)
+                vec(x + n + ".b", b, W // b)
+            w[x + "lam"] = bf16(rng.uniform(-6.0, 1.0, W))          # decays from almost 1 down to almost 0
+            mat(x + "o", D, W)
+        if layer["mlp"]:
+            F = layer["mlp"]["ff"]
+            vec(p + "norm2", D)
+            mat(p + "rg2", D, D)
+            vec(p + "rg2.b", D)
+            mat(p + "mlp.up", F, D, std=2.0 * D ** -0.5)
+            mat(p + "mlp.down", D, F)
+            w[p + "mlp.act"] = bf16(rng.uniform(-1.0, 1.0, 2))
+    return w
+
+
+def write_checkpoint(path, cfg, w):
+    os.makedirs(path, exist_ok=True)
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    head, at, blobs = {}, 0, []
+    for name, a in w.items():
+        b = (np.ascontiguousarray(a, np.float32).view(np.uint32) >> 16).astype("<u2").tobytes()
+        head[name] = {"dtype": "BF16", "shape": list(a.shape), "data_offsets": [at, at + len(b)]}
+        at += len(b)
+        blobs.append(b)
+    h = json.dumps(head).encode()
+    with open(os.path.join(path, "model.safetensors"), "wb") as f:
+        f.write(struct.pack("<Q", len(h)) + h + b"".join(blobs))
+    return str(path)
