@@ -58,6 +58,14 @@ struct AttnArgs {
     const int32_t* out_scatter;
 };
 
+// a·b rounded to fp32, then to fp16: without the barrier the compiler rounds once (v_fma_mixlo_f16) in some instantiations and twice
+// in others, and forms that promise the same bits differ in the last one
+__device__ __forceinline__ __half product_to_half(float a, float b) {
+    float v = a * b;
+    asm("" : "+v"(v));
+    return __float2half(v);
+}
+
 // FUSED_QKV (decode, q_len = 1): the workgroup of (sequence, kv head) first does what
 // split_qkv_norm_rope_into_paged_cache_varlen does for ITS rows of the new token — the G query heads of the
 // group, the kv head's key (both per-head RMSNorm + RoPE per qk_mode) and value — into LDS, with the same
@@ -383,12 +391,12 @@ __global__ __launch_bounds__(NW * 64) void paged_attn_kernel(AttnArgs p) {
         __half* orow = p.out + (long)(tok0 + t_o) * p.nq * HD;
         const int32_t* sc = p.out_scatter + (kvh * G + g_o) * HD + dl * DPT;
 #pragma unroll
-        for (int i = 0; i < DPT; i++) orow[sc[i]] = __float2half(ov[i] * inv);
+        for (int i = 0; i < DPT; i++) orow[sc[i]] = product_to_half(ov[i], inv);
         return;
     }
     __half* o = p.out + ((long)(tok0 + t_o) * p.nq + kvh * G + g_o) * HD + dl * DPT;
 #pragma unroll
-    for (int i = 0; i < DPT; i++) o[i] = __float2half(ov[i] * inv);
+    for (int i = 0; i < DPT; i++) o[i] = product_to_half(ov[i], inv);
 }
 
 // ── prefill attention with the K/V tiles of a block pair staged ONCE per workgroup in LDS (flash form) ───────────────────
