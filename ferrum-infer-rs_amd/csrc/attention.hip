@@ -6,7 +6,7 @@
 // backend/cuda/paged.rs:942,1309,1160).  Maths = causal GQA softmax(QKᵀ/√hd)·V with optional sliding
 // window (CPU forms: backend/cpu.rs:2179-2259, ferrum-kv/src/attention.rs:30-114).
 //
-// Design (HBM-bound in decode; DESIGN.md §kernels):
+// Design (HBM-bound in decode):
 //  * a workgroup owns (sequence, kv_head, 16 query rows) where a "row" is a (token, q-head of the
 //    GQA group) pair — at decode the 16 rows are the nq/nkv heads of the single new token, so K/V
 //    of a kv head are read ONCE for the whole group (the reference's CUDA lane reads them once per

@@ -57,6 +57,7 @@ struct Knobs {
     // layered models (tiled_gemm.hip, latent_attention.hip, rglru.hip)
     int tiled_big_min_tiles = 64;     // 16-bit projections of > 64 rows take the 128 × 128 tile kernel from this many tiles
     int tiled_nw = 0, tiled_kw = 0, tiled_j = 0;      // > 0: forced waves per workgroup, K parts, 16-column tiles per wave of the few-row kernel
+    int latent_tiles = 0;             // 1 / 2: forced 16-row tiles per workgroup of the latent attention
     int latent_splits = 0;            // > 0: forced KV split count of the latent attention
     int latent_expand_min_rows = 64;  // prompt portions of at least this many tokens attend expanded keys / values (0 = never)
     bool latent_plain = false;        // the plain latent attention kernel for 16-bit models too
@@ -122,6 +123,7 @@ enum Form : int {
     FORM_TILED_GEMM_BIG,        // … 128 × 128 tiles, operands copied to LDS as fragments
     FORM_LATENT_ATTN_PLAIN,     // latent attention, one workgroup per (token, head), any size and number format
     FORM_LATENT_ATTN,           // … on the matrix cores, against the cached latents (keys and values never expanded)
+    FORM_LATENT_ATTN_PAIR,      // … two 16-row tiles per workgroup
     FORM_LATENT_ATTN_SPLIT,     // … with the keys of a tile split over several workgroups
     FORM_LATENT_ATTN_EXPANDED,  // … prompt portions over keys and values expanded from the latents
     FORM_RGLRU_STEP,            // linear recurrence, every sequence brings one token: gates, state update and output in one launch

@@ -165,13 +165,13 @@ __global__ __launch_bounds__(256) void latent_attn_plain_kernel(LatentDims d, La
 
 // ── matrix-core form ──
 struct LatentTile { int seq, tile, tok0, q_len, pos0; };
-__device__ __forceinline__ int latent_tiles(const BatchView& v, int q_len, int heads) {
-    return v.long_min > 0 && q_len >= v.long_min ? 0 : (q_len * heads + 15) >> 4;
+__device__ __forceinline__ int latent_tiles(const BatchView& v, int q_len, int heads, int rows) {
+    return v.long_min > 0 && q_len >= v.long_min ? 0 : (q_len * heads + rows - 1) / rows;
 }
-// 16-row tiles of (token, head) pairs, numbered sequence by sequence; every wave finds tile w by a scan of cu_seqlens
-__device__ __forceinline__ bool find_latent_tile(const BatchView& v, int heads, int w, LatentTile* o) {
+// tiles of `rows` (16 or 32) (token, head) pairs, numbered sequence by sequence; every wave finds tile w by a scan of cu_seqlens
+__device__ __forceinline__ bool find_latent_tile(const BatchView& v, int heads, int rows, int w, LatentTile* o) {
     if (v.single) {
-        const int per = (heads + 15) >> 4;
+        const int per = (heads + rows - 1) / rows;
         o->seq = w / per; o->tile = w % per; o->tok0 = o->seq; o->q_len = 1;
         if (o->seq >= v.num_seqs) return false;
         o->pos0 = (int)v.pos[o->seq];
@@ -181,7 +181,7 @@ __device__ __forceinline__ bool find_latent_tile(const BatchView& v, int heads, 
     int base = 0;
     for (int s0 = 0; s0 < v.num_seqs; s0 += 64) {
         const int s = s0 + lane;
-        const int units = s < v.num_seqs ? latent_tiles(v, (int)(v.cu[s + 1] - v.cu[s]), heads) : 0;
+        const int units = s < v.num_seqs ? latent_tiles(v, (int)(v.cu[s + 1] - v.cu[s]), heads, rows) : 0;
         int incl = units;
 #pragma unroll
         for (int off = 1; off < 64; off <<= 1) {
@@ -213,106 +213,135 @@ __device__ __forceinline__ shortx4 read_tr(const bf16* p) {
     return __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) shortx4*)p);
 }
 
-// KS, RS: 32-wide steps of the latent and of the rotated part.  grid (row tiles × KV splits); a step is 64 keys: wave w scores block w of them
-// for all 16 rows, the row maxima meet in LDS, P and the parked latents are shared, and each wave accumulates its own quarter of the
-// output dimensions — so nothing is merged at the end and the latents of the next step are in flight during softmax and P·V.
-template <int KS, int RS>
-__global__ __launch_bounds__(256, 2) void latent_attn_kernel(LatentDims d, LatentBuffers<bf16> p, BatchView v, int nsplit) {
+// KS, RS: 32-wide steps of the latent and of the rotated part; MT: 16-row tiles per workgroup (two share every key they load where a
+// token has more than 16 heads).  grid (tiles × KV splits); a step is 64 keys: wave w scores block w of them for all rows, the row
+// maxima meet in LDS, P and the parked latents are shared, and each wave accumulates its own quarter of the output dimensions — so
+// nothing is merged at the end and the latents of the next step are in flight during softmax and P·V.
+template <int KS, int RS, int MT>
+__global__ __launch_bounds__(256, MT == 1 ? 2 : 1) void latent_attn_kernel(LatentDims d, LatentBuffers<bf16> p, BatchView v, int nsplit) {
     constexpr int DT = KS < 2 ? 1 : KS / 2;                                    // 16-dim output tiles per wave
-    constexpr int STAGE = KS * 512, PSTR = 72;
+    constexpr int STAGE = KS * 512, PSTR = 72, kd = 32 * (KS + RS), ROWS = 16 * MT;
     __shared__ __attribute__((aligned(16))) bf16 stage[4 * STAGE];
-    __shared__ __attribute__((aligned(16))) bf16 lds_p[16 * PSTR];
-    __shared__ float lds_m[64], lds_l[64];
+    __shared__ __attribute__((aligned(16))) bf16 lds_p[ROWS * PSTR];
+    __shared__ float lds_m[4 * ROWS], lds_l[4 * ROWS];
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, a = lane >> 4, b = lane & 15;
     const int split = blockIdx.x % nsplit, tile_id = blockIdx.x / nsplit;
     LatentTile w;
-    if (!find_latent_tile(v, d.heads, tile_id, &w)) return;
-    constexpr int kd = 32 * (KS + RS);
+    if (!find_latent_tile(v, d.heads, ROWS, tile_id, &w)) return;
     const int rows = w.q_len * d.heads;
-    const int rho = w.tile * 16 + b;
-    const bool ok = rho < rows;
-    const int tl = ok ? rho / d.heads : 0, h = ok ? rho % d.heads : 0;
-    const int row_pos = w.pos0 + tl, win_lo = max(0, row_pos + 1 - d.window);
-    const int t_first = w.tile * 16 / d.heads, t_last = min(w.q_len - 1, (w.tile * 16 + 15) / d.heads);
+    int row_pos[MT], win_lo[MT];
+    long qrow[MT];
+    bool ok[MT];
+#pragma unroll
+    for (int mt = 0; mt < MT; mt++) {
+        const int rho = w.tile * ROWS + mt * 16 + b;
+        ok[mt] = rho < rows;
+        const int tl = ok[mt] ? rho / d.heads : 0;
+        row_pos[mt] = w.pos0 + tl;
+        win_lo[mt] = max(0, row_pos[mt] + 1 - d.window);
+        qrow[mt] = (long)w.tok0 * d.heads + (ok[mt] ? rho : 0);
+    }
+    const int t_first = w.tile * ROWS / d.heads, t_last = min(w.q_len - 1, (w.tile * ROWS + ROWS - 1) / d.heads);
     const int kv_end = w.pos0 + t_last + 1, kv_lo = max(0, w.pos0 + t_first + 1 - d.window);
     const int blk_lo = kv_lo / 16, blk_hi = (kv_end + 15) / 16, nstep = (blk_hi - blk_lo + 3) / 4;
     const int st_lo = nstep * split / nsplit, st_hi = nstep * (split + 1) / nsplit;
     const int32_t* bt = v.bt + (long)w.seq * v.max_blocks;
 
     // block-table entries of this wave's blocks, 64 steps per load; then nothing of the step loop waits for the table
-    bf16x8 kf[KS + RS], qf[KS + RS];
+    bf16x8 kf[KS + RS], qf[MT][KS + RS];
     auto table = [&](int st) { return bt[min(blk_lo + 4 * (st + lane) + wave, blk_hi - 1)]; };
     int bt_st = st_lo, btv = table(st_lo);
     auto load = [&](int st) {                                                  // (past the last block: a copy of it, masked below)
-        const bf16* t = p.pool + (long)__builtin_amdgcn_readlane(btv, min(st - bt_st, 63)) * 16 * kd + lane * 8;
+        const bf16* t = p.pool + (long)__builtin_amdgcn_readlane(btv, st - bt_st) * 16 * kd + lane * 8;
 #pragma unroll
         for (int s = 0; s < KS + RS; s++) kf[s] = *reinterpret_cast<const bf16x8*>(t + s * 512);
     };
     {
         // the rotated part first: its values and angles travel together with the table entries, in front of the latents
-        const long qrow = (long)(w.tok0 + tl) * d.heads + h;
-        Rot4 rot[RS];
+        Rot4 rot[MT][RS];
 #pragma unroll
-        for (int s = 0; s < RS; s++) {
-            qf[KS + s] = *reinterpret_cast<const bf16x8*>(p.q + qrow * (d.dp + d.rp) + d.dp + 32 * s + 8 * a);
-            rot[s] = rot_load(32 * s + 8 * a, d.rot_dims, p.cos_t, p.sin_t, row_pos);
-        }
+        for (int mt = 0; mt < MT; mt++)
+#pragma unroll
+            for (int s = 0; s < RS; s++) {
+                qf[mt][KS + s] = *reinterpret_cast<const bf16x8*>(p.q + qrow[mt] * (d.dp + d.rp) + d.dp + 32 * s + 8 * a);
+                rot[mt][s] = rot_load(32 * s + 8 * a, d.rot_dims, p.cos_t, p.sin_t, row_pos[mt]);
+            }
         load(st_lo);                                                           // (no load under a condition: it would drain the others)
 #pragma unroll
-        for (int s = 0; s < KS; s++) qf[s] = *reinterpret_cast<const bf16x8*>(p.q_lat + qrow * (32 * KS) + 32 * s + 8 * a);
+        for (int mt = 0; mt < MT; mt++)
 #pragma unroll
-        for (int s = 0; s < RS; s++) qf[KS + s] = rot_apply(qf[KS + s], rot[s]);
+            for (int s = 0; s < KS; s++) qf[mt][s] = *reinterpret_cast<const bf16x8*>(p.q_lat + qrow[mt] * (32 * KS) + 32 * s + 8 * a);
+#pragma unroll
+        for (int mt = 0; mt < MT; mt++)
+#pragma unroll
+            for (int s = 0; s < RS; s++) qf[mt][KS + s] = rot_apply(qf[mt][KS + s], rot[mt][s]);
     }
     const int tr_off = tr_offset(lane);
-    float m_run = -INFINITY, l_run = 0.f;
-    floatx4 o[DT];
+    float m_run[MT], l_run[MT];
+    floatx4 o[MT][DT];
 #pragma unroll
-    for (int t = 0; t < DT; t++) o[t] = (floatx4){0.f, 0.f, 0.f, 0.f};
+    for (int mt = 0; mt < MT; mt++) {
+        m_run[mt] = -INFINITY;
+        l_run[mt] = 0.f;
+#pragma unroll
+        for (int t = 0; t < DT; t++) o[mt][t] = (floatx4){0.f, 0.f, 0.f, 0.f};
+    }
     for (int st = st_lo; st < st_hi; st++) {
-        floatx4 sc2[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};        // two chains: half the dependent MFMA latency
+        floatx4 sc[MT];
+        float mx[MT];
 #pragma unroll
-        for (int s = 0; s < KS; s++)
-            sc2[s & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[s], qf[s], sc2[s & 1], 0, 0, 0);
+        for (int mt = 0; mt < MT; mt++) {
+            floatx4 s2[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};     // two chains: half the dependent MFMA latency
 #pragma unroll
-        for (int s = 0; s < RS; s++)
-            sc2[s & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[KS + s], qf[KS + s], sc2[s & 1], 0, 0, 0);
-        floatx4 sc;
-        float mx = -INFINITY;
+            for (int s = 0; s < KS + RS; s++) s2[s & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[s], qf[mt][s], s2[s & 1], 0, 0, 0);
+            mx[mt] = -INFINITY;
 #pragma unroll
-        for (int r = 0; r < 4; r++) {
-            const int key = (blk_lo + 4 * st + wave) * 16 + 4 * a + r;
-            sc[r] = ok && key <= row_pos && key >= win_lo ? (sc2[0][r] + sc2[1][r]) * d.scale : -INFINITY;
-            mx = fmaxf(mx, sc[r]);
+            for (int r = 0; r < 4; r++) {
+                const int key = (blk_lo + 4 * st + wave) * 16 + 4 * a + r;
+                sc[mt][r] = ok[mt] && key <= row_pos[mt] && key >= win_lo[mt] ? (s2[0][r] + s2[1][r]) * d.scale : -INFINITY;
+                mx[mt] = fmaxf(mx[mt], sc[mt][r]);
+            }
+            mx[mt] = rows_reduce_max(mx[mt]);
         }
-        mx = rows_reduce_max(mx);
         __syncthreads();                                                       // the previous step's P·V has read stage and lds_p
 #pragma unroll
-        for (int s = 0; s < KS; s++)
-            *reinterpret_cast<bf16x8*>(stage + wave * STAGE + s * 512 + lane * 8) = kf[s];
-        if (a == 0) lds_m[wave * 16 + b] = mx;
+        for (int s = 0; s < KS; s++) *reinterpret_cast<bf16x8*>(stage + wave * STAGE + s * 512 + lane * 8) = kf[s];
+        if (a == 0) {
+#pragma unroll
+            for (int mt = 0; mt < MT; mt++) lds_m[wave * ROWS + mt * 16 + b] = mx[mt];
+        }
         if (st + 1 - bt_st == 64) { bt_st = st + 1; btv = table(bt_st); }
         load(st + 1);
         __syncthreads();
-        const float m_new = fmaxf(m_run, fmaxf(fmaxf(lds_m[b], lds_m[16 + b]), fmaxf(lds_m[32 + b], lds_m[48 + b])));
-        const float m_safe = m_new == -INFINITY ? 0.f : m_new, alpha = __expf(m_run - m_safe);
-        bf16x4 pf;
-        float ps = 0.f;
 #pragma unroll
-        for (int r = 0; r < 4; r++) { const float e = __expf(sc[r] - m_safe); ps += e; pf[r] = (bf16)e; }
-        l_run = l_run * alpha + ps;                                            // (this lane's keys; lanes and waves meet at the end)
-        m_run = m_new;
-        *reinterpret_cast<bf16x4*>(lds_p + b * PSTR + wave * 16 + 4 * a) = pf;
+        for (int mt = 0; mt < MT; mt++) {
+            const float* lm = lds_m + mt * 16 + b;
+            const float m_new = fmaxf(m_run[mt], fmaxf(fmaxf(lm[0], lm[ROWS]), fmaxf(lm[2 * ROWS], lm[3 * ROWS])));
+            const float m_safe = m_new == -INFINITY ? 0.f : m_new, alpha = __expf(m_run[mt] - m_safe);
+            bf16x4 pf;
+            float ps = 0.f;
 #pragma unroll
-        for (int t = 0; t < DT; t++)
+            for (int r = 0; r < 4; r++) { const float e = __expf(sc[mt][r] - m_safe); ps += e; pf[r] = (bf16)e; }
+            l_run[mt] = l_run[mt] * alpha + ps;                                // (this lane's keys; lanes and waves meet at the end)
+            m_run[mt] = m_new;
+            *reinterpret_cast<bf16x4*>(lds_p + (mt * 16 + b) * PSTR + wave * 16 + 4 * a) = pf;
 #pragma unroll
-            for (int r = 0; r < 4; r++) o[t][r] *= alpha;
+            for (int t = 0; t < DT; t++)
+#pragma unroll
+                for (int r = 0; r < 4; r++) o[mt][t][r] *= alpha;
+        }
         __syncthreads();
         // Oᵀ[d][row] += Vᵀ[d][key]·Pᵀ[key][row], 32 keys (two blocks) at a time: contraction index (a, j < 4) = key 4a + j of the first
         // block, (a, j ≥ 4) = key 4a + j − 4 of the second — a transposed read then covers 512 contiguous bytes
 #pragma unroll
         for (int c = 0; c < 2; c++) {
-            const bf16x4 p0 = *reinterpret_cast<const bf16x4*>(lds_p + b * PSTR + c * 32 + 4 * a), p1 = *reinterpret_cast<const bf16x4*>(lds_p + b * PSTR + c * 32 + 16 + 4 * a);
-            const bf16x8 pv = {p0[0], p0[1], p0[2], p0[3], p1[0], p1[1], p1[2], p1[3]};
+            bf16x8 pv[MT];
+#pragma unroll
+            for (int mt = 0; mt < MT; mt++) {
+                const bf16* lp = lds_p + (mt * 16 + b) * PSTR + c * 32 + 4 * a;
+                const bf16x4 p0 = *reinterpret_cast<const bf16x4*>(lp), p1 = *reinterpret_cast<const bf16x4*>(lp + 16);
+                pv[mt] = (bf16x8){p0[0], p0[1], p0[2], p0[3], p1[0], p1[1], p1[2], p1[3]};
+            }
             const bf16* vb = stage + 2 * c * STAGE + tr_off;
 #pragma unroll
             for (int t = 0; t < DT; t++)
@@ -320,50 +349,58 @@ __global__ __launch_bounds__(256, 2) void latent_attn_kernel(LatentDims d, Laten
                     const shortx4 v0 = read_tr(vb + (wave + 4 * t) * 256), v1 = read_tr(vb + STAGE + (wave + 4 * t) * 256);
                     typedef short shortx8 __attribute__((ext_vector_type(8)));
                     const shortx8 vt = {v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
-                    o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, vt), pv, o[t], 0, 0, 0);
+#pragma unroll
+                    for (int mt = 0; mt < MT; mt++)
+                        o[mt][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, vt), pv[mt], o[mt][t], 0, 0, 0);
                 }
         }
     }
-    l_run = rows_reduce_sum(l_run);
-    if (a == 0) lds_l[wave * 16 + b] = l_run;
-    __syncthreads();
-    const float L = lds_l[b] + lds_l[16 + b] + lds_l[32 + b] + lds_l[48 + b];
-    if (nsplit > 1) {
-        float* dst = p.partial + ((long)blockIdx.x * 16 + b) * (32 * KS + LATENT_PARTIAL_PAD);
 #pragma unroll
-        for (int t = 0; t < DT; t++)
-            if (KS >= 2 || wave < 2 * KS) *reinterpret_cast<floatx4*>(dst + (wave + 4 * t) * 16 + 4 * a) = o[t];
-        if (threadIdx.x < 16) { dst[32 * KS] = m_run; dst[32 * KS + 1] = L; }
-        return;
+    for (int mt = 0; mt < MT; mt++) {
+        const float l = rows_reduce_sum(l_run[mt]);
+        if (a == 0) lds_l[wave * ROWS + mt * 16 + b] = l;
     }
-    if (!ok) return;
-    const float inv = L > 0.f ? 1.0f / L : 0.f;
-    bf16* dst = p.o_lat + ((long)w.tok0 * d.heads + rho) * (32 * KS);
+    __syncthreads();
 #pragma unroll
-    for (int t = 0; t < DT; t++)
-        if (KS >= 2 || wave < 2 * KS) {
-            bf16x4 y;
+    for (int mt = 0; mt < MT; mt++) {
+        const float* ll = lds_l + mt * 16 + b;
+        const float L = ll[0] + ll[ROWS] + ll[2 * ROWS] + ll[3 * ROWS];
+        if (nsplit > 1) {
+            float* dst = p.partial + ((long)blockIdx.x * ROWS + mt * 16 + b) * (32 * KS + LATENT_PARTIAL_PAD);
 #pragma unroll
-            for (int r = 0; r < 4; r++) y[r] = (bf16)(o[t][r] * inv);
-            *reinterpret_cast<bf16x4*>(dst + (wave + 4 * t) * 16 + 4 * a) = y;
+            for (int t = 0; t < DT; t++)
+                if (KS >= 2 || wave < 2 * KS) *reinterpret_cast<floatx4*>(dst + (wave + 4 * t) * 16 + 4 * a) = o[mt][t];
+            if (threadIdx.x < 16) { dst[32 * KS] = m_run[mt]; dst[32 * KS + 1] = L; }
+        } else if (ok[mt]) {
+            const float inv = L > 0.f ? 1.0f / L : 0.f;
+            bf16* dst = p.o_lat + qrow[mt] * (32 * KS);
+#pragma unroll
+            for (int t = 0; t < DT; t++)
+                if (KS >= 2 || wave < 2 * KS) {
+                    bf16x4 y;
+#pragma unroll
+                    for (int r = 0; r < 4; r++) y[r] = (bf16)(o[mt][t][r] * inv);
+                    *reinterpret_cast<bf16x4*>(dst + (wave + 4 * t) * 16 + 4 * a) = y;
+                }
         }
+    }
 }
-// grid (row tiles, quads of output dimensions / 256): one thread per (row, 4 dimensions); every load is in flight at once
+// grid (tiles, quads of output dimensions / 256): one thread per (row, 4 dimensions); every load is in flight at once
 template <int NS>
-__global__ __launch_bounds__(256) void latent_attn_reduce_kernel(LatentDims d, LatentBuffers<bf16> p, BatchView v) {
+__global__ __launch_bounds__(256) void latent_attn_reduce_kernel(LatentDims d, LatentBuffers<bf16> p, BatchView v, int rows) {
     LatentTile w;
-    if (!find_latent_tile(v, d.heads, blockIdx.x, &w)) return;
-    const int quads = d.kp >> 2, id = blockIdx.y * 256 + threadIdx.x, row = id / quads, c = (id % quads) * 4, ro = w.tile * 16 + row;
-    if (row >= 16 || ro >= w.q_len * d.heads) return;
-    const long ld = d.kp + LATENT_PARTIAL_PAD;
-    const float* src = p.partial + ((long)blockIdx.x * NS * 16 + row) * ld;
+    if (!find_latent_tile(v, d.heads, rows, blockIdx.x, &w)) return;
+    const int quads = d.kp >> 2, id = blockIdx.y * 256 + threadIdx.x, row = id / quads, c = (id % quads) * 4, ro = w.tile * rows + row;
+    if (row >= rows || ro >= w.q_len * d.heads) return;
+    const long ld = d.kp + LATENT_PARTIAL_PAD, zs = rows * ld;
+    const float* src = p.partial + ((long)blockIdx.x * NS * rows + row) * ld;
     float m[NS], l[NS], M = -INFINITY, L = 0.f;
     floatx4 o[NS], acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int z = 0; z < NS; z++) {
-        m[z] = src[z * 16 * ld + d.kp];
-        l[z] = src[z * 16 * ld + d.kp + 1];
-        o[z] = *reinterpret_cast<const floatx4*>(src + z * 16 * ld + c);
+        m[z] = src[z * zs + d.kp];
+        l[z] = src[z * zs + d.kp + 1];
+        o[z] = *reinterpret_cast<const floatx4*>(src + z * zs + c);
     }
 #pragma unroll
     for (int z = 0; z < NS; z++) M = fmaxf(M, m[z]);
@@ -561,20 +598,31 @@ static int latent_plain(const LatentDims& d, const LatentBuffers<E>& b, const Ba
     return 0;
 }
 static int latent_mfma(const LatentDims& d, const LatentBuffers<bf16>& b, const BatchView& v, hipStream_t s) {
-    const int tiles = v.single ? v.num_seqs * cdiv(d.heads, 16) : (int)(((long)v.T * d.heads) / 16) + v.num_seqs;      // upper bound of Σ ceil(rows / 16)
+    // two 16-row tiles per workgroup where a token fills both and the batch is large: the keys are loaded and parked once for 32 heads
+    // (below ≈ 128 tiles the launch is bound by latency, and one tile per workgroup has the shorter chain)
+    const bool pair = knobs().latent_tiles > 0 ? knobs().latent_tiles == 2 : d.heads > 16 && (long)v.T * d.heads >= 128 * 16;
+    const int mt = pair ? 2 : 1, rows = 16 * mt;
+    const int tiles = v.single ? v.num_seqs * cdiv(d.heads, rows) : (int)(((long)v.T * d.heads) / rows) + v.num_seqs;      // upper bound of Σ ceil(rows of a sequence / rows)
     const int keys = (int)std::min<long>(v.max_keys, (long)d.window + 16);
-    // split the keys while the launch has fewer than 2 workgroups per CU (what stays resident) and a split keeps ≥ 128 keys (two steps)
+    // split the keys while the launch has fewer workgroups than stay resident (2 per CU, 1 with two tiles) and a split keeps ≥ 128
+    // keys (two steps)
     int ns = 1;
-    while (ns < 16 && tiles * ns < 512 && keys >= 2 * ns * 128) ns *= 2;
+    while (ns < 16 && tiles * ns < 512 / mt && keys >= 2 * ns * 128) ns *= 2;
     if (knobs().latent_splits > 0)
         for (ns = 1; ns < std::min(16, knobs().latent_splits); ns *= 2) {}
-    while (ns > 1 && (size_t)tiles * ns * 16 * (d.kp + LATENT_PARTIAL_PAD) * 4 > b.partial_bytes) ns /= 2;
+    while (ns > 1 && (size_t)tiles * ns * rows * (d.kp + LATENT_PARTIAL_PAD) * 4 > b.partial_bytes) ns /= 2;
     const dim3 grid(ns * tiles);         // (splits fastest: the row tiles of a sequence read a key range on the same XCD)
     form_hit(ns > 1 ? FORM_LATENT_ATTN_SPLIT : FORM_LATENT_ATTN);
-#define LATENT(KS)                                                                                             \
-    do {                                                                                                       \
-        if (d.rp == 32) hipLaunchKernelGGL((latent_attn_kernel<KS, 1>), grid, dim3(256), 0, s, d, b, v, ns);    \
-        else hipLaunchKernelGGL((latent_attn_kernel<KS, 2>), grid, dim3(256), 0, s, d, b, v, ns);               \
+    if (pair) form_hit(FORM_LATENT_ATTN_PAIR);
+#define LATENT2(KS, RS)                                                                                           \
+    do {                                                                                                          \
+        if (mt == 1) hipLaunchKernelGGL((latent_attn_kernel<KS, RS, 1>), grid, dim3(256), 0, s, d, b, v, ns);      \
+        else hipLaunchKernelGGL((latent_attn_kernel<KS, RS, 2>), grid, dim3(256), 0, s, d, b, v, ns);              \
+    } while (0)
+#define LATENT(KS)                              \
+    do {                                        \
+        if (d.rp == 32) LATENT2(KS, 1);         \
+        else LATENT2(KS, 2);                    \
     } while (0)
     switch (d.kp) {
     case 32: LATENT(1); break;
@@ -585,13 +633,14 @@ static int latent_mfma(const LatentDims& d, const LatentBuffers<bf16>& b, const 
     default: LATENT(16); break;
     }
 #undef LATENT
+#undef LATENT2
     FH_CHECK_LAUNCH();
     if (ns > 1) {
-        const dim3 rg(tiles, cdiv(16 * (d.kp / 4), 256));
-        if (ns == 2) hipLaunchKernelGGL(latent_attn_reduce_kernel<2>, rg, dim3(256), 0, s, d, b, v);
-        else if (ns == 4) hipLaunchKernelGGL(latent_attn_reduce_kernel<4>, rg, dim3(256), 0, s, d, b, v);
-        else if (ns == 8) hipLaunchKernelGGL(latent_attn_reduce_kernel<8>, rg, dim3(256), 0, s, d, b, v);
-        else hipLaunchKernelGGL(latent_attn_reduce_kernel<16>, rg, dim3(256), 0, s, d, b, v);
+        const dim3 rg(tiles, cdiv(rows * (d.kp / 4), 256));
+        if (ns == 2) hipLaunchKernelGGL(latent_attn_reduce_kernel<2>, rg, dim3(256), 0, s, d, b, v, rows);
+        else if (ns == 4) hipLaunchKernelGGL(latent_attn_reduce_kernel<4>, rg, dim3(256), 0, s, d, b, v, rows);
+        else if (ns == 8) hipLaunchKernelGGL(latent_attn_reduce_kernel<8>, rg, dim3(256), 0, s, d, b, v, rows);
+        else hipLaunchKernelGGL(latent_attn_reduce_kernel<16>, rg, dim3(256), 0, s, d, b, v, rows);
         FH_CHECK_LAUNCH();
     }
     return 0;

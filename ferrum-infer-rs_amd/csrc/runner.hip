@@ -631,7 +631,7 @@ static void launch1d(void (*k)(__half*, long, uint64_t, float, float), __half* p
 
 // Synthetic weights generated on the device (bench only: no checkpoints are available offline).
 // qweight nibbles uniform, scales uniform [0.01,0.1)·f with f = 1/(0.25·sqrt(K)) so that
-// dequantised W has std ≈ 1/sqrt(K) and activations stay O(1) through all layers (DESIGN.md),
+// dequantised W has std ≈ 1/sqrt(K) and activations stay O(1) through all layers,
 // zero point 8 (sym), norm weights 1, embeddings / lm_head / router N(0, 0.02).
 static int synth_w4(W4Device* w, int k, int n, int E, bool fused, uint64_t seed, hipStream_t s) {
     free_w4(*w);

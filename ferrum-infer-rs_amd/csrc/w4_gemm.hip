@@ -5,7 +5,7 @@
 // and `MarlinExpertStack::gemm_phase_vllm` (ferrum-kernels/src/marlin_expert_stack.rs:86).
 // Arithmetic contract (cpu.rs:2283-2315): W[n,k] = (q − (z+1))·s[k/g, n].
 //
-// Design (HBM-bound at T ≤ 64, see DESIGN.md §kernels):
+// Design (HBM-bound at T ≤ 64):
 //  * load-time repack GPTQ [K/8,N] → "w4t" tiles: one wave-instruction (64 lanes × 16 B = 1 KiB,
 //    fully coalesced) fetches a 16-column × 128-row (= one quant group) tile whose per-lane dwords
 //    ARE the B-operand fragments of four v_mfma_f32_16x16x32_f16 k-steps.

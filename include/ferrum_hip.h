@@ -5,7 +5,7 @@
  * the reference's backend traits
  *     Backend + BackendGraph + BackendPagedKv + BackendQuantMarlin + BackendMoeFused (+ BackendCollective)
  *     = MoeLlmBackend          (crates/ferrum-kernels/src/backend/traits.rs:2196-2208)
- * in place of the CUDA lane of `ferrum-kernels`.  INTEGRATION.md shows the binding.
+ * in place of the CUDA lane of `ferrum-kernels`.
  *
  * Conventions (same as the reference's own C entry points: FA2 shim
  * crates/ferrum-kernels/src/backend/cuda/fa2_ffi.rs:16-37, Marlin cuda/marlin.rs:293-387):

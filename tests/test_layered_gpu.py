@@ -182,12 +182,14 @@ def test_first_tokens(pkg, cases, n, dtype):
     assert rel(feed(m, 3, t, [1]), L.forward(cfg, w, t)) < TOL[dtype]
 
 
+@pytest.mark.parametrize("tiles", [0, 2])
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("name", ["odd", "wide", "deep"])
-def test_unequal_batch_against_each_request_alone(pkg, cases, name, dtype):
+def test_unequal_batch_against_each_request_alone(pkg, cases, knobs, name, dtype, tiles):
     """Portions of some requests beside single decoded tokens of others, members coming and going; rows against the oracle, and against
     the same rows computed alone to rounding."""
     cfg, w, path = cases(name)
+    knobs.set(LATENT_TILES=tiles)
     m = load(pkg, path, dtype, tokens=400, seqs=4)
     seqs = {i: toks(cfg, n, 60 + i) for i, n in enumerate((190, 37, 140, 75))}
     want = {i: L.forward(cfg, w, t) for i, t in seqs.items()}
@@ -277,15 +279,13 @@ def standout(window, seed=5, kv_rank=64, dim=32, rot=8, vdim=32, heads=4):
     return cfg, w
 
 
-@pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("form", ["latent", "split", "expanded", "plain"])
+@pytest.mark.parametrize("form,dtype", [("plain", "float32")] + [(f, "bfloat16") for f in ("latent", "pair", "split", "pair split", "expanded", "plain")])
 @pytest.mark.parametrize("window", [1, 2, 16, 17, 64, 100])
 def test_window_edge(pkg, tmp_path, knobs, forms, window, form, dtype):
     """Token 0 stands exactly on the last visible place, or one further back, for query token 1 — in a prompt, in a portion and decoded,
     with the window's edge at every kind of place within a page.  The oracle with a window one off must be far away."""
-    if dtype == "float32" and form != "plain":
-        pytest.skip("32-bit models have one attention form")
-    knobs.set(LATENT_PLAIN=int(form == "plain"), LATENT_SPLITS=4 if form == "split" else 1, LATENT_EXPAND_MIN_ROWS=2 if form == "expanded" else 0)
+    knobs.set(LATENT_PLAIN=int(form == "plain"), LATENT_SPLITS=4 if "split" in form else 1, LATENT_TILES=2 if "pair" in form else 1,
+              LATENT_EXPAND_MIN_ROWS=2 if form == "expanded" else 0)
     cfg, w = standout(window)
     m = load(pkg, G.write_checkpoint(tmp_path, cfg, w), dtype)
     forms.reset()
@@ -312,8 +312,8 @@ def test_window_edge(pkg, tmp_path, knobs, forms, window, form, dtype):
     h = forms.hits()
     if form == "plain":
         assert h.get("latent_attn_plain") and not h.get("latent_attn") and not h.get("latent_attn_expanded")
-    elif form == "split":
-        assert h.get("latent_attn_split")
+    elif "split" in form or "pair" in form:
+        assert bool(h.get("latent_attn_split")) == ("split" in form) and bool(h.get("latent_attn_pair")) == ("pair" in form)
     elif form == "expanded":
         assert h.get("latent_attn_expanded") or window == 1
     else:
