@@ -1,5 +1,5 @@
-// Attention over a compressed cache (multi-head latent attention): a token caches one normed latent c and one rotated key part shared
-// by all heads; head h's key is (W_uk,h c | shared part) and its value W_uv,h c.
+// Attention over a compressed cache (multi-head latent attention): a token caches its normed latent c and a single rotated key
+// part that every head uses; head h's key is (W_uk,h c | shared part) and its value W_uv,h c.
 //
 // One token per sequence and short portions never expand keys or values: the query's plain part arrives already multiplied by W_uk,hᵀ (q_lat), so a score is
 // q_lat · c + rot(q) · k_rot, and the output is left in latent space (o_lat = Σ p c) for the value projection that follows.  All heads
