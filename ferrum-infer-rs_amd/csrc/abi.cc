@@ -93,7 +93,7 @@ static const char* const g_form_names[FORM_COUNT] = {
     "route_fused", "route_gemm", "dense_slab_chain", "graph_capture", "graph_replay", "tp_allreduce_rccl",
     "tp_allreduce_loopback", "tp_allreduce_oneshot", "f16_dense_linear", "w4_fused_tail", "attn_resident", "w4_big", "w4_ldsk", "gather_columns",
     "perm_producer", "moe_expert_major_pair", "decode_chain", "moe_deferred_merge", "dense_chain", "tp_allreduce_norm_fused", "moe_block_major_pair", "chain_attn_kv_splits", "chain_qkv_wide", "route_gemm_topk",
-    "tiled_gemm", "tiled_gemm_big", "latent_attn_plain", "latent_attn", "latent_attn_pair", "latent_attn_split", "latent_attn_expanded", "rglru_step", "rglru_scan"};
+    "tiled_gemm", "tiled_gemm_big", "tiled_gemm_grouped", "tiled_gemm_grouped_big", "latent_attn_plain", "latent_attn", "latent_attn_pair", "latent_attn_split", "latent_attn_expanded", "rglru_step", "rglru_scan"};
 const char* form_name(int f) { return f >= 0 && f < FORM_COUNT ? g_form_names[f] : nullptr; }
 }  // namespace fh
 

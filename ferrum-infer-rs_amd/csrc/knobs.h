@@ -121,6 +121,8 @@ enum Form : int {
     FORM_ROUTE_GEMM_TOPK,       // prefill router: logits (MFMA) + softmax + top-k in one launch (moe_route_gemm_topk_kernel)
     FORM_TILED_GEMM,            // layered models: projection with K split over the waves of a workgroup
     FORM_TILED_GEMM_BIG,        // … 128 × 128 tiles, operands copied to LDS as fragments
+    FORM_TILED_GEMM_GROUPED,    // … rows sorted by expert
+    FORM_TILED_GEMM_GROUPED_BIG,
     FORM_LATENT_ATTN_PLAIN,     // latent attention, one workgroup per (token, head), any size and number format
     FORM_LATENT_ATTN,           // … on the matrix cores, against the cached latents (keys and values never expanded)
     FORM_LATENT_ATTN_PAIR,      // … two 16-row tiles per workgroup

@@ -52,6 +52,13 @@ __device__ __forceinline__ V rot_apply(V x, const Rot4& r) {
     return x;
 }
 
+// A row's statistics (maximum m, sum l of e^(score − m)) closed by its head's sink: factor of the row's Σ e^(score − m)·value
+__device__ __forceinline__ float softmax_factor(float m, float l, const float* __restrict__ sink, int h) {
+    if (!sink) return l > 0.f ? 1.0f / l : 0.f;
+    const float z = sink[h], top = fmaxf(m, z), f = __expf(m - top);
+    return f / (l * f + __expf(z - top));
+}
+
 // one wave per token: norm of the query latent, norm of the kv latent, rotation of the shared key part, cache write
 template <typename E>
 __global__ __launch_bounds__(256) void latent_prepare_kernel(const E* __restrict__ dq, const E* __restrict__ dkv, long ld,
@@ -62,25 +69,26 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(const E* __restrict
     if (t >= v.T) return;
     const int seq = v.tok_seq[t];
     const long pos = (long)v.pos[seq] + t - v.cu[seq];
-    const E *qr = dq + t * ld, *kr = dkv + t * ld;
+    const E *qr = dq + t * ld, *kr = dkv ? dkv + t * ld : nullptr;
     float sq = 0.f, sk = 0.f;
     for (int i = lane * 8; i < d.qp; i += 512) {
         const v8 x = *reinterpret_cast<const v8*>(qr + i);
 #pragma unroll
         for (int j = 0; j < 8; j++) sq += (float)x[j] * (float)x[j];      // (padded columns are zero)
     }
-    for (int i = lane * 8; i < d.kp; i += 512) {
+    for (int i = lane * 8; dkv && i < d.kp; i += 512) {
         const v8 x = *reinterpret_cast<const v8*>(kr + i);
 #pragma unroll
         for (int j = 0; j < 8; j++) sk += (float)x[j] * (float)x[j];
     }
-    const float iq = 1.0f / sqrtf(wave_reduce_sum(sq) / (float)d.q_rank + eps), ik = 1.0f / sqrtf(wave_reduce_sum(sk) / (float)d.kv_rank + eps);
+    const float iq = 1.0f / sqrtf(wave_reduce_sum(sq) / (float)(d.q_rank ? d.q_rank : 1) + eps), ik = 1.0f / sqrtf(wave_reduce_sum(sk) / (float)d.kv_rank + eps);
     for (int i = lane * 8; i < d.qp; i += 512) {
         v8 x = *reinterpret_cast<const v8*>(qr + i);
 #pragma unroll
         for (int j = 0; j < 8; j++) x[j] = (E)((float)x[j] * iq * dq_norm[i + j]);
         *reinterpret_cast<v8*>(cq + (long)t * d.qp + i) = x;
     }
+    if (!dkv) return;                                    // (the layer reads another one's cache)
     E* tile = b.pool + (long)v.bt[(long)seq * v.max_blocks + pos / 16] * 16 * (d.kp + d.rp) + (pos % 16) * 8;
     for (int i = lane * 8; i < d.kp + d.rp; i += 512) {
         v8 x = *reinterpret_cast<const v8*>(kr + i);
@@ -111,7 +119,7 @@ __global__ __launch_bounds__(256) void latent_attn_plain_kernel(LatentDims d, La
     const int seq = v.tok_seq[t];
     const int pos = v.pos[seq] + t - v.cu[seq];
     for (int i = tid; i < d.kp; i += 256) { q[i] = (float)b.q_lat[((long)t * d.heads + h) * d.kp + i]; o[i] = 0.f; }
-    const E* qr = b.q + ((long)t * d.heads + h) * (d.dp + d.rp) + d.dp;
+    const E* qr = b.q + (long)t * b.ldq + h * (d.dp + d.rp) + d.dp;
     const int half = d.rot_dims >> 1;
     for (int i = tid; i < d.rp; i += 256) {
         float x = (float)qr[i];
@@ -160,7 +168,12 @@ __global__ __launch_bounds__(256) void latent_attn_plain_kernel(LatentDims d, La
         }
         __syncthreads();
     }
-    for (int i = tid; i < d.kp; i += 256) b.o_lat[((long)t * d.heads + h) * d.kp + i] = (E)(o[i] / l_run);
+    float f = 1.0f / l_run;
+    if (b.sink) {
+        const float z = b.sink[h], top = fmaxf(m_run, z), e = expf(m_run - top);
+        f = e / (l_run * e + expf(z - top));
+    }
+    for (int i = tid; i < d.kp; i += 256) b.o_lat[((long)t * d.heads + h) * d.kp + i] = (E)(o[i] * f);
 }
 
 // ── matrix-core form ──
@@ -229,8 +242,8 @@ __global__ __launch_bounds__(256, MT == 1 ? 2 : 1) void latent_attn_kernel(Laten
     LatentTile w;
     if (!find_latent_tile(v, d.heads, ROWS, tile_id, &w)) return;
     const int rows = w.q_len * d.heads;
-    int row_pos[MT], win_lo[MT];
-    long qrow[MT];
+    int row_pos[MT], win_lo[MT], head[MT];
+    long qrow[MT], qtok[MT];
     bool ok[MT];
 #pragma unroll
     for (int mt = 0; mt < MT; mt++) {
@@ -240,6 +253,8 @@ __global__ __launch_bounds__(256, MT == 1 ? 2 : 1) void latent_attn_kernel(Laten
         row_pos[mt] = w.pos0 + tl;
         win_lo[mt] = max(0, row_pos[mt] + 1 - d.window);
         qrow[mt] = (long)w.tok0 * d.heads + (ok[mt] ? rho : 0);
+        head[mt] = ok[mt] ? rho - tl * d.heads : 0;
+        qtok[mt] = (w.tok0 + tl) * p.ldq + head[mt] * (d.dp + d.rp) + d.dp;
     }
     const int t_first = w.tile * ROWS / d.heads, t_last = min(w.q_len - 1, (w.tile * ROWS + ROWS - 1) / d.heads);
     const int kv_end = w.pos0 + t_last + 1, kv_lo = max(0, w.pos0 + t_first + 1 - d.window);
@@ -263,7 +278,7 @@ __global__ __launch_bounds__(256, MT == 1 ? 2 : 1) void latent_attn_kernel(Laten
         for (int mt = 0; mt < MT; mt++)
 #pragma unroll
             for (int s = 0; s < RS; s++) {
-                qf[mt][KS + s] = *reinterpret_cast<const bf16x8*>(p.q + qrow[mt] * (d.dp + d.rp) + d.dp + 32 * s + 8 * a);
+                qf[mt][KS + s] = *reinterpret_cast<const bf16x8*>(p.q + qtok[mt] + 32 * s + 8 * a);
                 rot[mt][s] = rot_load(32 * s + 8 * a, d.rot_dims, p.cos_t, p.sin_t, row_pos[mt]);
             }
         load(st_lo);                                                           // (no load under a condition: it would drain the others)
@@ -372,7 +387,7 @@ __global__ __launch_bounds__(256, MT == 1 ? 2 : 1) void latent_attn_kernel(Laten
                 if (KS >= 2 || wave < 2 * KS) *reinterpret_cast<floatx4*>(dst + (wave + 4 * t) * 16 + 4 * a) = o[mt][t];
             if (threadIdx.x < 16) { dst[32 * KS] = m_run[mt]; dst[32 * KS + 1] = L; }
         } else if (ok[mt]) {
-            const float inv = L > 0.f ? 1.0f / L : 0.f;
+            const float inv = softmax_factor(m_run[mt], L, p.sink, head[mt]);
             bf16* dst = p.o_lat + qrow[mt] * (32 * KS);
 #pragma unroll
             for (int t = 0; t < DT; t++)
@@ -410,7 +425,7 @@ __global__ __launch_bounds__(256) void latent_attn_reduce_kernel(LatentDims d, L
         L += l[z] * f;
         acc += o[z] * f;
     }
-    const float inv = 1.0f / L;
+    const float inv = softmax_factor(M, L, p.sink, ro % d.heads);
     bf16x4 y;
 #pragma unroll
     for (int r = 0; r < 4; r++) y[r] = (bf16)(acc[r] * inv);
@@ -445,7 +460,7 @@ __global__ __launch_bounds__(256, 2) void latent_expanded_kernel(LatentDims d, L
         win_lo[mt] = max(0, row_pos[mt] + 1 - d.window);
         vis_hi[mt] = t0 + 15 < q_len ? pos0 + t0 : -1;                         // keys in [vis_lo, vis_hi] are seen by every row of the tile
         vis_lo[mt] = max(0, pos0 + t0 + 16 - d.window);
-        const bf16* q = p.q + ((long)(tok0 + min(t, q_len - 1)) * d.heads + h) * (d.dp + d.rp) + 8 * a;
+        const bf16* q = p.q + (long)(tok0 + min(t, q_len - 1)) * p.ldq + h * (d.dp + d.rp) + 8 * a;
 #pragma unroll
         for (int s = 0; s < DS; s++)
             qf[mt][s] = *reinterpret_cast<const bf16x8*>(q + 32 * s);
@@ -560,8 +575,9 @@ __global__ __launch_bounds__(256, 2) void latent_expanded_kernel(LatentDims d, L
         const float l = rows_reduce_sum(l_run[mt]);
         if (!ok[mt]) continue;
         const long tok = tok0 + tile0 + (wave * MT + mt) * 16 + b;
-        const float f = (float)x.gate[tok * x.ld_gate + h] / l;
-        bf16* dst = x.out + (tok * d.heads + h) * d.vp + 4 * a;
+        float f = softmax_factor(m_run[mt] * 0.6931471805599453f, l, p.sink, h);      // (the maximum is kept in base 2)
+        if (x.gate) f *= (float)x.gate[tok * x.ld_gate + h];
+        bf16* dst = x.out + tok * x.ldo + h * d.vp + 4 * a;
 #pragma unroll
         for (int t = 0; t < DT; t++) {
                 bf16x4 y;

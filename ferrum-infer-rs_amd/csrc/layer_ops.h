@@ -32,11 +32,15 @@ struct BatchView {
 template <typename E>
 int embed_bigram(const E* table, const E* bigram, int buckets, int64_t mul_prev, int64_t mul_cur, const BatchView& v, float* x, E* xb,
                  int dim, int ldb, hipStream_t s);
-// x += mult · rms(sub · gate) · w (w holds 1 + the stored weight); xb = E(x); sub is the sum of `slabs` partial sums
+// x += sub + Σ_j weights[row][j] · pairs[row·top + j] (top 0: none); xb = E(x); sub is the sum of `slabs` partial sums
 template <typename E>
-int gated_post_norm_add(const float* sub, long ld_sub, int slabs, long slab_stride, const E* gate, long ld_gate, const float* w, float mult, float eps, float* x,
-                        E* xb, int rows, int dim, int ldb, hipStream_t s);
-// out[i] = E(rms(x[row_idx[i]]) · w)
+int branch_add(const float* sub, long ld_sub, int slabs, long slab_stride, const E* pairs, long ld_pair, const float* weights, int top, float* x, E* xb,
+               int rows, int dim, int ldb, hipStream_t s);
+// x += mult · rms(sub · gate) · w (gate null: none); xb = E(x), with next_norm E(rms(x)); sub is the sum of `slabs` partial sums
+template <typename E>
+int post_norm_add(const float* sub, long ld_sub, int slabs, long slab_stride, const E* gate, long ld_gate, const float* w, float mult, float eps, bool next_norm,
+                  float* x, E* xb, int rows, int dim, int ldb, hipStream_t s);
+// out[i] = E(rms(x[row_idx[i]]) · w); row_idx null: row i; w null: ones
 template <typename E>
 int rms_norm_rows(const float* x, const int32_t* row_idx, const float* w, float eps, E* out, int rows, int dim, int ldo, hipStream_t s);
 
@@ -57,12 +61,13 @@ template <typename E>
 struct LatentBuffers {
     const float *cos_t = nullptr, *sin_t = nullptr;   // [positions][rot_dims / 2]
     E* pool = nullptr;
-    const E* q = nullptr;              // [T][heads·(dp + rp)]: per head the plain part, then the part to rotate
+    const E* q = nullptr; long ldq = 0;    // [T][ldq ≥ heads·(dp + rp)]: per head the plain part, then the part to rotate
+    const float* sink = nullptr;       // [heads] score-like numbers that take part in the softmax denominator only; null: none
     const E* q_lat = nullptr;          // [T][heads][kp]: plain part taken through the key projection
     E* o_lat = nullptr;                // [T][heads][kp]
     float* partial = nullptr; size_t partial_bytes = 0;
 };
-// q latent: RMS norm → cq [T][qp]; kv latent: RMS norm, shared key part: rotation → cache.  `dq` / `dkv`: their columns in the
+// q latent (q_rank 0: none): RMS norm → cq [T][qp]; kv latent: RMS norm, shared key part: rotation → cache.  `dq` / `dkv`: their columns in the
 // fused projection's rows (ld); dkv = [kp latent | rp key part].
 template <typename E>
 int latent_prepare(const E* dq, const E* dkv, long ld, const float* dq_norm, const float* dkv_norm, float eps, const LatentDims& d,
@@ -71,15 +76,16 @@ template <typename E>
 int latent_attention(const LatentDims& d, const LatentBuffers<E>& b, const BatchView& v, hipStream_t s);
 // Portions over expanded keys and values (16-bit): blocks [nblocks] lists the cache blocks whose keys ke [16·nblocks][heads·dp] and
 // values ve [16·nblocks][heads·vp] were expanded; units [nunits][4] = (sequence, first token of the tile within the portion, index in
-// `blocks` of the sequence's first listed block, that block's number in the sequence).  out [T][heads·vp], times the head gate.
+// `blocks` of the sequence's first listed block, that block's number in the sequence).  out [T][ldo ≥ heads·vp], times the head gate if any.
 struct LatentExpanded {
     const int32_t *blocks = nullptr, *units = nullptr;
     int nblocks = 0, nunits = 0;
     const bf16 *ke = nullptr, *ve = nullptr;
     long ldk = 0, ldv = 0;
     const bf16* gate = nullptr; long ld_gate = 0;
-    bf16* out = nullptr;
+    bf16* out = nullptr; long ldo = 0;
 };
+constexpr int LATENT_NO_WINDOW = 1 << 30;
 constexpr int LATENT_TILE_TOKENS = 128;          // tokens of a portion per workgroup
 bool latent_expanded_supports(const LatentDims& d);
 int latent_attention_expanded(const LatentDims& d, const LatentBuffers<bf16>& b, const BatchView& v, const LatentExpanded& x, hipStream_t s);

@@ -1,7 +1,8 @@
 // Layered models (layered.h): weight packing and the forward pass.
 //
-// A layer is a mixer and, optionally, a feed-forward.  Both sublayers read the residual stream itself; their result is multiplied by a
-// sigmoid gate of the same input, normed (weight stored around zero) and added with a constant factor:
+// A layer is a mixer and, optionally, a feed-forward, in one of two blocks.
+// Gated post-norm block: both sublayers read the residual stream itself; their result is multiplied by a sigmoid gate of the same input,
+// normed (weight stored around zero) and added with a constant factor:
 //     x ← x + m · norm(sub(x) · σ(W x + b))
 // Everything that reads x is ONE projection per sublayer — the gate's rows, then the mixer's (or feed-forward's) input rows, each
 // section with its own activation in the epilogue:
@@ -10,6 +11,12 @@
 //                        (long portions: keys and values of the visible cache blocks expanded → flash attention × head gate → W_o)
 //     linear recurrence: [gate σ | y gelu | x] → convolution → gates + state (one token) or scan (portions) → W_o → add + norm
 //     feed-forward     : [gate σ | up xIELU] → down → add + norm
+// Parallel pre-norm block: both sublayers read x̂ = x / rms(x) times a gain of their own that is a single number, so x̂ is written once,
+// the gains are factors of the projections' sections, and mixer and dense feed-forward share the projection in and the projection out:
+//     [q | kv latent + shared key part | (gate, up) pairs → y] → attention as above → [W_down | W_o]·[y ; attention] → add
+//     mixture of experts: router → top-k → rows sorted by expert → up (relu²) → down, summed with its weights by the residual add
+// and may end with a per-layer view of the token: x ← x + norm(W_p (gelu(W_g x) · e_layer[token])); the kernel that adds it writes the
+// next layer's x̂.  A latent attention layer may read the latents that an earlier layer has cached.
 #include <math.h>
 
 #include <algorithm>
@@ -17,6 +24,7 @@
 #include <unordered_map>
 
 #include "common.h"
+#include "kernels.h"
 #include "knobs.h"
 #include "layered.h"
 
@@ -31,6 +39,8 @@ uint16_t bf16_bits(float f) {
 }
 void store(bf16* dst, float f) { const uint16_t h = bf16_bits(f); memcpy(dst, &h, 2); }
 void store(float* dst, float f) { *dst = f; }
+
+constexpr int MOE_MAX_BLOCK = 128;
 
 struct HostTensor { std::vector<float> data; std::vector<int64_t> shape; };
 
@@ -71,6 +81,13 @@ __global__ void synth_kernel(E* p, size_t n, uint64_t seed, float std) {
 }
 
 #define FH_TRY(call) do { if (int rc_ = (call)) return rc_; } while (0)
+// a kernel of the forward `run` (Layered::Run), announced and waited for when launches are traced
+#define RUN(call)                                                                                        \
+    do {                                                                                                 \
+        if (run.trace) fprintf(stderr, "[ferrum_hip] layer %d T=%d %.60s\n", run.li, run.v.T, #call);    \
+        FH_TRY(call);                                                                                    \
+        if (run.trace) FH_CHECK_HIP(hipStreamSynchronize(run.s));                                        \
+    } while (0)
 
 template <typename E>
 class Layered final : public LayeredModel {
@@ -80,9 +97,14 @@ class Layered final : public LayeredModel {
         // fused input projection of the mixer: sections in the order of the comment at the top
         Linear in, uq, uk, uv, expand, o, ff_in, down;
         GemmSection in_sec[GEMM_MAX_SECTIONS], ff_sec[2];
-        int in_nsec = 0;
-        int c0 = 0, c1 = 0, c2 = 0;        // columns of the mixer's sections: latent attention: q latent, kv latent, head gates; recurrence: y, x
+        int in_nsec = 0, ld_in = 0;
+        int c0 = 0, c1 = 0, c2 = 0;        // columns of the mixer's sections: latent attention: q (latent), kv latent, head gates; recurrence: y, x
+        int c_glu = -1, c_att = -1;        // parallel block: columns of the feed-forward's gated product and, behind it, of the attention's result
         float *norm1 = nullptr, *norm2 = nullptr;
+        float g2 = 1.f;
+        Linear router, up, side_gate, side_proj;
+        E* side_table = nullptr;
+        float* side_norm = nullptr;
         LatentDims ld{};
         float *dq_norm = nullptr, *dkv_norm = nullptr;
         LatentBuffers<E> lb{};
@@ -119,123 +141,62 @@ public:
         // embedding table (gather) and the same table as vocabulary projection; bigram table
         FH_TRY(table("embed", c_.vocab, &embed_));
         if (lc_.bigram_buckets > 0) FH_TRY(table("bigram", lc_.bigram_buckets + 1, &bigram_));
-        FH_TRY(pack(&head_, {{"embed", 0, c_.vocab, pad32(c_.vocab)}}, D_));
-        FH_TRY(unit_offset("final.norm", &final_norm_));
-        long in_cols = 0, q_cols = 0, lat_cols = 0, attn_cols = 0, cq_cols = 0, rnn_cols = 0;
-        size_t units = T / RGLRU_CHUNK + c_.max_seqs, partial = 0;
+        FH_TRY(pack(&head_, {{lc_.untied_head ? "head" : "embed", 0, c_.vocab, pad32(c_.vocab)}}, D_));
+        if (parallel()) {
+            float g = 1.f;
+            FH_TRY(scalar("final.norm", &g));
+            FH_TRY(arena_.upload(&final_norm_, std::vector<float>(pad32(D_), g)));
+        } else {
+            FH_TRY(unit_offset("final.norm", &final_norm_));
+        }
+        long in_cols = 0, q_cols = 0, lat_cols = 0, attn_cols = 0, cq_cols = 0, rnn_cols = 0, side_cols = 0;
+        size_t units = T / RGLRU_CHUNK + c_.max_seqs, partial = 0, pairs = 0, sorted = 0, expert_cols = 0, logit_cols = 0;
         for (int li = 0; li < c_.num_layers; li++) {
             Layer& L = layers_[li];
             const FerrumHipLayerSpec& sp = L.s;
-            const std::string p = "l" + std::to_string(li) + ".", m = p + "mix.";
-            FH_TRY(unit_offset(p + "norm1", &L.norm1));
+            const std::string p = "l" + std::to_string(li) + ".";
+            Input in;
+            float g1 = 1.f;
+            if (parallel()) {
+                FH_TRY(scalar(p + "norm1", &g1));
+                if (sp.ff != FERRUM_HIP_FF_NONE) FH_TRY(scalar(p + "norm2", &L.g2));
+            } else {
+                FH_TRY(unit_offset(p + "norm1", &L.norm1));
+                section(L, in, GEMM_ACT_SIGMOID);
+                in.add(p + "rg1", 0, D_, Dp_, p + "rg1.b");
+            }
             if (sp.mixer == FERRUM_HIP_MIXER_LATENT_ATTENTION) {
+                FH_TRY(latent_weights(L, in, p + "mix.", g1));
                 const LatentDims& d = L.ld;
-                const int H = d.heads;
-                std::vector<Rows> in = {{p + "rg1", 0, D_, Dp_}, {m + "dq", 0, d.q_rank, d.qp}, {m + "dkv", 0, d.kv_rank, d.kp},
-                                        {m + "dkv", d.kv_rank, d.rot_dim, d.rp}, {m + "g", 0, H, pad32(H)}};
-                FH_TRY(pack(&L.in, in, D_));
-                FH_TRY(bias(&L.in, in, {p + "rg1.b", "", "", "", ""}));
-                std::vector<Rows> q;
-                for (int h = 0; h < H; h++) {
-                    const int r0 = h * (sp.dim + d.rot_dim);
-                    q.push_back({m + "uq", r0, sp.dim, d.dp});
-                    q.push_back({m + "uq", r0 + sp.dim, d.rot_dim, d.rp});
-                }
-                FH_TRY(pack(&L.uq, q, d.q_rank));
-                // per head: W_ukᵀ [latent, plain query dims], W_uv [value dims, latent]
-                FH_TRY(need(m + "uk", {(int64_t)H * sp.dim, d.kv_rank}));
-                FH_TRY(need(m + "uv", {(int64_t)H * d.vdim, d.kv_rank}));
-                const int dim = sp.dim, kr = d.kv_rank, vd = d.vdim;
-                FH_TRY(pack_fn(&L.uk, H, d.kp, d.dp, m + "uk", [&](const float* w, int g, int n, int k) {
-                    return n < kr && k < dim ? w[((size_t)g * dim + k) * kr + n] : 0.f; }));
-                // [W_uk | W_uv] over the latent: the expansion of keys and values; its second part doubles as the per-head value projection
-                const float *uk = data(m + "uk"), *uv = data(m + "uv");
-                const int kn = H * d.dp, dp = d.dp, vpad = d.vp;
-                FH_TRY(pack_fn(&L.expand, 1, kn + H * d.vp, d.kp, m + "uv", [&](const float*, int, int n, int k) {
-                    if (k >= kr) return 0.f;
-                    if (n < kn) return n % dp < dim ? uk[((size_t)(n / dp) * dim + n % dp) * kr + k] : 0.f;
-                    n -= kn;
-                    return n % vpad < vd ? uv[((size_t)(n / vpad) * vd + n % vpad) * kr + k] : 0.f; }));
-                L.uv.w = L.expand.w + (size_t)kn * d.kp; L.uv.n = d.vp; L.uv.k = d.kp; L.uv.groups = H;
-                FH_TRY(need(m + "o", {D_, (int64_t)H * vd}));
-                const int vp = d.vp;
-                FH_TRY(pack_fn(&L.o, 1, Dp_, H * vp, m + "o", [&](const float* w, int, int n, int k) {
-                    return n < D_ && k % vp < vd ? w[(size_t)n * H * vd + (k / vp) * vd + k % vp] : 0.f; }));
-                FH_TRY(vec(m + "dq.norm", {d.q_rank}, d.qp, &L.dq_norm));
-                FH_TRY(vec(m + "dkv.norm", {d.kv_rank}, d.kp, &L.dkv_norm));
-                FH_TRY(arena_.alloc(&L.lb.pool, (size_t)c_.kv_num_blocks * latent_block_elems(d)));
-                FH_TRY(rope(sp.rot_base, d.rot_dims, &L.lb.cos_t, &L.lb.sin_t));
-                L.c0 = Dp_; L.c1 = L.c0 + d.qp; L.c2 = L.c1 + d.kp + d.rp;
-                L.in_sec[0] = {0, GEMM_ACT_SIGMOID, 0, 0}; L.in_sec[1] = {L.c0, GEMM_ACT_NONE, 0, 0}; L.in_sec[2] = {L.c2, GEMM_ACT_SIGMOID, 0, 0};
-                L.in_nsec = 3;
-                q_cols = std::max<long>(q_cols, L.uq.n); lat_cols = std::max<long>(lat_cols, (long)H * d.kp);
-                attn_cols = std::max<long>(attn_cols, (long)H * vp); cq_cols = std::max<long>(cq_cols, d.qp);
+                lat_cols = std::max<long>(lat_cols, (long)d.heads * d.kp);
+                cq_cols = std::max<long>(cq_cols, d.qp);
+                if (d.q_rank) q_cols = std::max<long>(q_cols, L.uq.n);
                 // split attention: (row tile, split) pairs stay below 1024
                 partial = std::max<size_t>(partial, (size_t)1024 * 16 * (d.kp + 4) * 4);
             } else {
-                const RglruDims& d = L.rd;
-                const int bs = sp.rnn_width / d.blocks, bp = d.bp, W = sp.rnn_width;
-                std::vector<Rows> in = {{p + "rg1", 0, D_, Dp_}};
-                std::vector<std::string> b = {p + "rg1.b"};
-                for (const char* part : {"y", "x"})
-                    for (int g = 0; g < d.blocks; g++) { in.push_back({m + part, g * bs, bs, bp}); b.push_back(m + part + ".b"); }
-                FH_TRY(pack(&L.in, in, D_));
-                FH_TRY(bias(&L.in, in, b));
-                FH_TRY(need(m + "ra", {d.blocks, bs, bs}));
-                FH_TRY(need(m + "ri", {d.blocks, bs, bs}));
-                // gate tiles: [block][16-channel tile][ra, ri] — packed as 2·bp rows per block in that order
-                const float *ra = data(m + "ra"), *ri = data(m + "ri");
-                Linear gates;
-                FH_TRY(pack_fn(&gates, d.blocks, 2 * bp, bp, m + "ra", [&](const float*, int g, int n, int k) {
-                    const int ch = (n / 32) * 16 + n % 16;
-                    const float* w = (n / 16) % 2 ? ri : ra;
-                    return ch < bs && k < bs ? w[((size_t)g * bs + ch) * bs + k] : 0.f; }));
-                L.rb.gate_w = gates.w;
-                auto padded = [&](const std::string& name, const float** out, bool sp_fold, int taps) -> int {
-                    const int64_t n = W;
-                    if (taps > 1 || name == m + "conv") FH_TRY(need(name, {n, taps}));
-                    else if (name == m + "ra.b" || name == m + "ri.b") FH_TRY(need(name, {d.blocks, bs}));
-                    else FH_TRY(need(name, {n}));
-                    const float* src = data(name);
-                    std::vector<float> v((size_t)taps * d.wp, 0.f);
-                    for (int j = 0; j < taps; j++)
-                        for (int ch = 0; ch < W; ch++) {
-                            const float x = src ? src[(size_t)ch * taps + j] : 0.25f;
-                            v[(size_t)j * d.wp + (ch / bs) * bp + ch % bs] = sp_fold ? (float)softplus(x) : x;
-                        }
-                    float* dev = nullptr;
-                    FH_TRY(arena_.upload(&dev, v));
-                    *out = dev;
-                    return 0;
-                };
-                FH_TRY(padded(m + "conv", &L.rb.conv_w, false, d.taps));
-                FH_TRY(padded(m + "conv.b", &L.rb.conv_b, false, 1));
-                FH_TRY(padded(m + "ra.b", &L.rb.ra_b, false, 1));
-                FH_TRY(padded(m + "ri.b", &L.rb.ri_b, false, 1));
-                FH_TRY(padded(m + "lam", &L.rb.lam, true, 1));
-                FH_TRY(need(m + "o", {D_, W}));
-                FH_TRY(pack_fn(&L.o, 1, Dp_, d.wp, m + "o", [&](const float* w, int, int n, int k) {
-                    return n < D_ && k % bp < bs ? w[(size_t)n * W + (k / bp) * bs + k % bp] : 0.f; }));
-                FH_TRY(arena_.alloc(&L.rb.conv_state, (size_t)slots_ * std::max(d.taps - 1, 1) * d.wp));
-                FH_TRY(arena_.alloc(&L.rb.state, (size_t)slots_ * d.wp));
-                L.c0 = Dp_; L.c1 = L.c0 + d.wp;
-                L.in_sec[0] = {0, GEMM_ACT_SIGMOID, 0, 0}; L.in_sec[1] = {L.c0, GEMM_ACT_GELU_TANH, 0, 0}; L.in_sec[2] = {L.c1, GEMM_ACT_NONE, 0, 0};
-                L.in_nsec = 3;
-                rnn_cols = std::max<long>(rnn_cols, d.wp);
+                FH_TRY(recurrent_weights(L, in, p + "mix."));
+                rnn_cols = std::max<long>(rnn_cols, L.rd.wp);
             }
-            in_cols = std::max<long>(in_cols, L.in.n);
-            if (sp.ff != FERRUM_HIP_FF_NONE) {
-                FH_TRY(unit_offset(p + "norm2", &L.norm2));
-                const int F = sp.ff_width, Fp = pad32(F);
-                std::vector<Rows> in = {{p + "rg2", 0, D_, Dp_}, {p + "mlp.up", 0, F, Fp}};
-                FH_TRY(pack(&L.ff_in, in, D_));
-                FH_TRY(bias(&L.ff_in, in, {p + "rg2.b", ""}));
-                FH_TRY(pack(&L.down, {{p + "mlp.down", 0, D_, Dp_}}, F));
-                FH_TRY(need(p + "mlp.act", {2}));
-                const float* act = data(p + "mlp.act");
-                L.ff_sec[0] = {0, GEMM_ACT_SIGMOID, 0, 0};
-                L.ff_sec[1] = {Dp_, GEMM_ACT_XIELU, (float)softplus(act ? act[0] : 0.5f), (float)softplus(act ? act[1] : 0.5f)};
-                in_cols = std::max<long>(in_cols, L.ff_in.n);
+            FH_TRY(feed_forward_weights(L, in, p));
+            FH_TRY(pack(&L.in, in.rows, D_));
+            if (in.biased()) FH_TRY(bias(&L.in, in.rows, in.bias));
+            L.ld_in = L.in.n;
+            if (sp.mixer == FERRUM_HIP_MIXER_LATENT_ATTENTION) {
+                const long att = (long)L.ld.heads * L.ld.vp;
+                if (L.c_att >= 0) L.ld_in = (int)std::max<long>(L.ld_in, L.c_att + att);
+                else attn_cols = std::max(attn_cols, att);
+            }
+            in_cols = std::max<long>({in_cols, L.ld_in, L.ff_in.n});
+            if (sp.ff == FERRUM_HIP_FF_MOE_RELU2) {
+                const size_t n = T * sp.top;
+                pairs = std::max(pairs, n);
+                sorted = std::max(sorted, n + (size_t)MOE_MAX_BLOCK * (std::min<size_t>(sp.experts, n) + 1));
+                expert_cols = std::max(expert_cols, n * L.up.n);
+                logit_cols = std::max<size_t>(logit_cols, sp.experts);
+            }
+            if (lc_.token_side_dim) {
+                FH_TRY(side_weights(L, p, li));
+                side_cols = L.side_gate.n;
             }
         }
         host_.clear();
@@ -256,11 +217,23 @@ public:
         FH_TRY(arena_.alloc(&drive_, T * rnn_cols));
         FH_TRY(arena_.alloc(&chunk_a_, units * rnn_cols));
         FH_TRY(arena_.alloc(&chunk_h_, units * rnn_cols));
+        FH_TRY(arena_.alloc(&side_, T * side_cols));
+        FH_TRY(arena_.alloc(&router_logits_, T * logit_cols));
+        FH_TRY(arena_.alloc(&expert_ids_, pairs));
+        FH_TRY(arena_.alloc(&expert_weights_, pairs));
+        FH_TRY(arena_.alloc(&sorted_, sorted));
+        FH_TRY(arena_.alloc(&sorted_expert_, pairs));
+        FH_TRY(arena_.alloc(&sorted_total_, pairs ? 4 : 0));
+        FH_TRY(arena_.alloc(&expert_h_, expert_cols));
+        FH_TRY(arena_.alloc(&expert_y_, pairs * Dp_));
         FH_TRY(arena_.alloc(&head_in_, (size_t)c_.max_seqs * Dp_));
         FH_TRY(finalize_expansion());
         for (Layer& L : layers_) {
-            L.lb.q = q_; L.lb.q_lat = q_lat_; L.lb.o_lat = o_lat_; L.lb.partial = partial_; L.lb.partial_bytes = partial_bytes_;
-            L.rb.x = in_ + L.c1; L.rb.y = in_ + L.c0; L.rb.ld = L.in.n;
+            if (L.s.kv_source) L.lb.pool = layers_[L.s.kv_source - 1].lb.pool;
+            L.lb.q = L.ld.q_rank ? q_ : in_ + L.c0;
+            L.lb.ldq = L.ld.q_rank ? L.uq.n : L.ld_in;
+            L.lb.q_lat = q_lat_; L.lb.o_lat = o_lat_; L.lb.partial = partial_; L.lb.partial_bytes = partial_bytes_;
+            L.rb.x = in_ + L.c1; L.rb.y = in_ + L.c0; L.rb.ld = L.ld_in;
             L.rb.u = u_; L.rb.out = rnn_out_; L.rb.decay = decay_; L.rb.drive = drive_; L.rb.chunk_a = chunk_a_; L.rb.chunk_h = chunk_h_;
         }
         FH_CHECK_HIP(hipStreamSynchronize(s));
@@ -268,57 +241,17 @@ public:
     }
 
     int forward(const BatchView& v, float* taps, bool trace, hipStream_t s) override {
-#define RUN(call)                                                                                \
-    do {                                                                                         \
-        if (trace) fprintf(stderr, "[ferrum_hip] layer %d T=%d %.60s\n", li, v.T, #call);        \
-        FH_TRY(call);                                                                            \
-        if (trace) FH_CHECK_HIP(hipStreamSynchronize(s));                                        \
-    } while (0)
-        int li = -1;
-        const int T = v.T;
-        BatchView ve = v;
-        const bool any_short = plan_expansion(&ve);
-        if (ve.long_min > 0)
+        Run run{v, v, true, trace, s, -1};
+        run.any_short = plan_expansion(&run.short_view);
+        if (run.short_view.long_min > 0)
             FH_CHECK_HIP(hipMemcpyAsync(plan_dev_, plan_host_, plan_used_ * 4, hipMemcpyHostToDevice, s));
-        const float eps = c_.rms_eps;
-        int slabs = 1;
         RUN(embed_bigram<E>(embed_, bigram_, lc_.bigram_buckets, lc_.bigram_mul_prev, lc_.bigram_mul_cur, v, x_, xb_, D_, Dp_, s));
-        for (li = 0; li < c_.num_layers; li++) {
-            Layer& L = layers_[li];
-            TiledGemm<E> g = linear(L.in, xb_, Dp_, T, in_, L.in.n);
-            g.nsec = L.in_nsec;
-            std::copy(L.in_sec, L.in_sec + L.in_nsec, g.sec);
-            RUN(tiled_gemm(g, s));
-            if (L.s.mixer == FERRUM_HIP_MIXER_LATENT_ATTENTION) {
-                const LatentDims& d = L.ld;
-                RUN(latent_prepare<E>(in_ + L.c0, in_ + L.c1, L.in.n, L.dq_norm, L.dkv_norm, eps, d, L.lb, v, cq_, s));
-                RUN(tiled_gemm(linear(L.uq, cq_, d.qp, T, q_, L.uq.n), s));
-                if (any_short) {
-                    TiledGemm<E> k = linear(L.uk, q_, L.uq.n, T, q_lat_, (long)d.heads * d.kp);
-                    k.x_group = d.dp + d.rp; k.out_group = d.kp;
-                    RUN(tiled_gemm(k, s));
-                    RUN(latent_attention<E>(d, L.lb, ve, s));
-                    TiledGemm<E> u = linear(L.uv, o_lat_, (long)d.heads * d.kp, T, attn_, (long)d.heads * d.vp);
-                    u.x_group = d.kp; u.out_group = d.vp; u.row_scale = in_ + L.c2; u.ld_scale = L.in.n;
-                    RUN(tiled_gemm(u, s));
-                }
-                if (ve.long_min > 0) RUN(attend_expanded(L, v, s));        // (writes the rows of the long portions only)
-                RUN(tiled_gemm(linear_slabs(L.o, attn_, (long)d.heads * d.vp, T, &slabs), s));
-            } else {
-                RUN(rglru_forward<E>(L.rd, L.rb, v, s));
-                RUN(tiled_gemm(linear_slabs(L.o, rnn_out_, L.rd.wp, T, &slabs), s));
-            }
-            RUN(gated_post_norm_add<E>(sub_, Dp_, slabs, (long)T * Dp_, in_, L.in.n, L.norm1, lc_.residual_mult, eps, x_, xb_, T, D_, Dp_, s));
-            if (L.s.ff != FERRUM_HIP_FF_NONE) {
-                TiledGemm<E> f = linear(L.ff_in, xb_, Dp_, T, in_, L.ff_in.n);
-                f.nsec = 2; f.sec[0] = L.ff_sec[0]; f.sec[1] = L.ff_sec[1];
-                RUN(tiled_gemm(f, s));
-                RUN(tiled_gemm(linear_slabs(L.down, in_ + Dp_, L.ff_in.n, T, &slabs), s));
-                RUN(gated_post_norm_add<E>(sub_, Dp_, slabs, (long)T * Dp_, in_, L.ff_in.n, L.norm2, lc_.residual_mult, eps, x_, xb_, T, D_, Dp_, s));
-            }
-            if (taps) FH_CHECK_HIP(hipMemcpyAsync(taps + (size_t)li * c_.max_tokens * D_, x_, (size_t)T * D_ * 4, hipMemcpyDeviceToDevice, s));
+        if (parallel()) RUN(rms_norm_rows<E>(x_, nullptr, nullptr, c_.rms_eps, xb_, v.T, D_, Dp_, s));
+        for (run.li = 0; run.li < c_.num_layers; run.li++) {
+            Layer& L = layers_[run.li];
+            FH_TRY(parallel() ? parallel_layer(L, run) : gated_layer(L, run));
+            if (taps) FH_CHECK_HIP(hipMemcpyAsync(taps + (size_t)run.li * c_.max_tokens * D_, x_, (size_t)v.T * D_ * 4, hipMemcpyDeviceToDevice, s));
         }
-#undef RUN
         return 0;
     }
 
@@ -330,11 +263,122 @@ public:
     }
 
 private:
+    // one forward: the batch, the part of it that latent_attention takes, and the layer at hand
+    struct Run { const BatchView& v; BatchView short_view; bool any_short, trace; hipStream_t s; int li; };
+
+    int gated_layer(Layer& L, const Run& run) {
+        const int T = run.v.T;
+        hipStream_t s = run.s;
+        const float eps = c_.rms_eps;
+        int slabs = 1;
+        RUN(tiled_gemm(input_projection(L, T), s));
+        if (L.s.mixer == FERRUM_HIP_MIXER_LATENT_ATTENTION) {
+            FH_TRY(attend(L, run, attn_, (long)L.ld.heads * L.ld.vp));
+            RUN(tiled_gemm(linear_slabs(L.o, attn_, (long)L.ld.heads * L.ld.vp, T, &slabs), s));
+        } else {
+            RUN(rglru_forward<E>(L.rd, L.rb, run.v, s));
+            RUN(tiled_gemm(linear_slabs(L.o, rnn_out_, L.rd.wp, T, &slabs), s));
+        }
+        RUN(post_norm_add<E>(sub_, Dp_, slabs, (long)T * Dp_, in_, L.ld_in, L.norm1, lc_.residual_mult, eps, false, x_, xb_, T, D_, Dp_, s));
+        if (L.s.ff != FERRUM_HIP_FF_NONE) {
+            TiledGemm<E> f = linear(L.ff_in, xb_, Dp_, T, in_, L.ff_in.n);
+            f.nsec = 2; f.sec[0] = L.ff_sec[0]; f.sec[1] = L.ff_sec[1];
+            RUN(tiled_gemm(f, s));
+            RUN(tiled_gemm(linear_slabs(L.down, in_ + Dp_, L.ff_in.n, T, &slabs), s));
+            RUN(post_norm_add<E>(sub_, Dp_, slabs, (long)T * Dp_, in_, L.ff_in.n, L.norm2, lc_.residual_mult, eps, false, x_, xb_, T, D_, Dp_, s));
+        }
+        return 0;
+    }
+
+    int parallel_layer(Layer& L, const Run& run) {
+        const int T = run.v.T;
+        hipStream_t s = run.s;
+        const bool moe = L.s.ff == FERRUM_HIP_FF_MOE_RELU2, last = run.li + 1 == c_.num_layers;
+        int slabs = 1;
+        RUN(tiled_gemm(input_projection(L, T), s));
+        if (moe) FH_TRY(experts(L, run));
+        E* att = L.c_att >= 0 ? in_ + L.c_att : attn_;
+        const long ld_att = L.c_att >= 0 ? L.ld_in : (long)L.ld.heads * L.ld.vp;
+        FH_TRY(attend(L, run, att, ld_att));
+        RUN(tiled_gemm(linear_slabs(L.o, L.c_glu >= 0 ? in_ + L.c_glu : att, ld_att, T, &slabs), s));
+        RUN(branch_add<E>(sub_, Dp_, slabs, (long)T * Dp_, expert_y_, Dp_, expert_weights_, moe ? L.s.top : 0, x_, xb_, T, D_, Dp_, s));
+        if (lc_.token_side_dim) {
+            TiledGemm<E> g = linear(L.side_gate, xb_, Dp_, T, side_, L.side_gate.n);
+            g.nsec = 1; g.sec[0] = {0, GEMM_ACT_GELU_TANH, 0, 0};
+            g.col_scale = L.side_table; g.col_scale_row = run.v.tokens; g.ld_col_scale = L.side_gate.n;
+            RUN(tiled_gemm(g, s));
+            RUN(tiled_gemm(linear_slabs(L.side_proj, side_, L.side_gate.n, T, &slabs), s));
+            RUN(post_norm_add<E>(sub_, Dp_, slabs, (long)T * Dp_, nullptr, 0, L.side_norm, 1.f, c_.rms_eps, true, x_, xb_, T, D_, Dp_, s));
+        } else if (!last) {
+            RUN(rms_norm_rows<E>(x_, nullptr, nullptr, c_.rms_eps, xb_, T, D_, Dp_, s));
+        }
+        return 0;
+    }
+
+    TiledGemm<E> input_projection(const Layer& L, int T) const {
+        TiledGemm<E> g = linear(L.in, xb_, Dp_, T, in_, L.ld_in);
+        g.nsec = L.in_nsec;
+        std::copy(L.in_sec, L.in_sec + L.in_nsec, g.sec);
+        return g;
+    }
+
+    // latent attention from the input projection's columns to the heads' values, out [T][ldo ≥ heads·vp]
+    int attend(Layer& L, const Run& run, E* out, long ldo) {
+        const LatentDims& d = L.ld;
+        const int T = run.v.T;
+        hipStream_t s = run.s;
+        const bool gates = !(L.s.attn_flags & FERRUM_HIP_ATTN_NO_HEAD_GATE);
+        if (d.q_rank || !L.s.kv_source)
+            RUN(latent_prepare<E>(in_ + L.c0, L.s.kv_source ? nullptr : in_ + L.c1, L.ld_in, L.dq_norm, L.dkv_norm, c_.rms_eps, d, L.lb, run.v, cq_, s));
+        if (d.q_rank) RUN(tiled_gemm(linear(L.uq, cq_, d.qp, T, q_, L.uq.n), s));
+        if (run.any_short) {
+            TiledGemm<E> k = linear(L.uk, L.lb.q, L.lb.ldq, T, q_lat_, (long)d.heads * d.kp);
+            k.x_group = d.dp + d.rp; k.out_group = d.kp;
+            RUN(tiled_gemm(k, s));
+            RUN(latent_attention<E>(d, L.lb, run.short_view, s));
+            TiledGemm<E> u = linear(L.uv, o_lat_, (long)d.heads * d.kp, T, out, ldo);
+            u.x_group = d.kp; u.out_group = d.vp;
+            if (gates) { u.row_scale = in_ + L.c2; u.ld_scale = L.ld_in; }
+            RUN(tiled_gemm(u, s));
+        }
+        if (run.short_view.long_min > 0) RUN(attend_expanded(L, run.v, out, ldo, s));        // (writes the rows of the long portions only)
+        return 0;
+    }
+
+    // expert_y_ [T·top][Dp] and expert_weights_ [T·top] of the chosen experts
+    int experts(Layer& L, const Run& run) {
+        const int T = run.v.T, E_ = L.s.experts, pairs = T * L.s.top;
+        hipStream_t s = run.s;
+        TiledGemm<E> z = linear_f32(L.router, xb_, Dp_, T, router_logits_, E_);
+        z.n_store = E_; z.nsec = 1; z.sec[0] = {0, GEMM_ACT_NONE, 0, 0, L.g2};
+        RUN(tiled_gemm(z, s));
+        RUN(moe_route_topk_softmax_f32(router_logits_, expert_ids_, expert_weights_, T, E_, L.s.top, 1, s));
+        GemmRows rows;
+        rows.block = moe_block(pairs, E_);
+        rows.max_blocks = std::min(pairs, pairs / rows.block + std::min(E_, pairs));
+        rows.id = sorted_; rows.group = sorted_expert_; rows.total = sorted_total_;
+        RUN(moe_align_block_size(expert_ids_, sorted_, sorted_expert_, sorted_total_, pairs, E_, rows.block, rows.max_blocks * rows.block, s));
+        TiledGemm<E> u = linear(L.up, xb_, Dp_, pairs, expert_h_, L.up.n);
+        u.groups = 1; u.rows = rows; u.rows.div = L.s.top;
+        u.nsec = 1; u.sec[0] = {0, GEMM_ACT_RELU2, 0, 0, L.g2};
+        RUN(tiled_gemm(u, s));
+        TiledGemm<E> y = linear(L.down, expert_h_, L.up.n, pairs, expert_y_, Dp_);
+        y.groups = 1; y.rows = rows;
+        RUN(tiled_gemm(y, s));
+        return 0;
+    }
+    // rows per block of the sorted list: a large block shares an expert's weights between more rows, a small one pads less
+    static int moe_block(int pairs, int experts) {
+        const int mean = pairs / experts;
+        if (sizeof(E) == 2 && mean >= 48) return 128;
+        return mean >= 32 ? 64 : mean >= 12 ? 32 : 16;
+    }
+
     void dims(Layer& L) {
         const FerrumHipLayerSpec& s = L.s;
         if (s.mixer == FERRUM_HIP_MIXER_LATENT_ATTENTION)
             L.ld = {s.heads, s.kv_rank, s.q_rank, s.rot_dim, s.rot_dims, s.vdim, latent_pad_head(s.dim, s.vdim, s.dim), latent_pad_rot(s.rot_dim),
-                    latent_pad_rank(s.kv_rank), pad32(s.q_rank), latent_pad_head(s.dim, s.vdim, s.vdim), s.window, s.scale};
+                    latent_pad_rank(s.kv_rank), pad32(s.q_rank), latent_pad_head(s.dim, s.vdim, s.vdim), s.window == FERRUM_HIP_WINDOW_NONE ? LATENT_NO_WINDOW : s.window, s.scale};
         else
             L.rd = {s.rnn_blocks, pad32(s.rnn_width / s.rnn_blocks), s.rnn_blocks * pad32(s.rnn_width / s.rnn_blocks), s.conv_taps};
     }
@@ -400,7 +444,7 @@ private:
         if (any_long) v->long_min = min_rows;
         return any_short;
     }
-    int attend_expanded(Layer& L, const BatchView& v, hipStream_t s) {
+    int attend_expanded(Layer& L, const BatchView& v, E* out, long ldo, hipStream_t s) {
         if constexpr (sizeof(E) == 2) {
             const Plan& q = *std::find_if(plans_.begin(), plans_.end(), [&](const Plan& x) { return x.window == L.ld.window; });
             const LatentDims& d = L.ld;
@@ -410,7 +454,8 @@ private:
             LatentExpanded x;
             x.blocks = plan_dev_ + q.blocks0; x.units = plan_dev_ + q.units0; x.nblocks = q.nblocks; x.nunits = q.nunits;
             x.ke = expanded_; x.ve = expanded_ + (size_t)d.heads * d.dp; x.ldk = x.ldv = L.expand.n;
-            x.gate = in_ + L.c2; x.ld_gate = L.in.n; x.out = attn_;
+            if (!(L.s.attn_flags & FERRUM_HIP_ATTN_NO_HEAD_GATE)) { x.gate = in_ + L.c2; x.ld_gate = L.ld_in; }
+            x.out = out; x.ldo = ldo;
             return latent_attention_expanded(d, L.lb, v, x, s);
         }
         return 0;
@@ -426,7 +471,179 @@ private:
     }
 
     // ── weights ──
+    bool parallel() const { return lc_.block == FERRUM_HIP_BLOCK_PARALLEL_PRE_NORM; }
+    struct Input;
+    // opens a section of the layer's input projection; returns its first column
+    static int section(Layer& L, const Input& in, GemmAct act, float mul = 1.f, float p = 0.f, float q = 0.f) {
+        L.in_sec[L.in_nsec++] = {in.cols(), act, p, q, mul};
+        return in.cols();
+    }
+    int latent_weights(Layer& L, Input& in, const std::string& m, float g1) {
+        const FerrumHipLayerSpec& sp = L.s;
+        const LatentDims& d = L.ld;
+        const int H = d.heads, dim = sp.dim, kr = d.kv_rank, vd = d.vdim, dp = d.dp, vp = d.vp;
+        std::vector<Rows> q;
+        const std::string qn = m + (d.q_rank ? "uq" : "q");
+        for (int h = 0; h < H; h++) {
+            const int r0 = h * (dim + d.rot_dim);
+            q.push_back({qn, r0, dim, dp});
+            q.push_back({qn, r0 + dim, d.rot_dim, d.rp});
+        }
+        L.c0 = section(L, in, GEMM_ACT_NONE, g1);
+        if (d.q_rank) {
+            in.add(m + "dq", 0, d.q_rank, d.qp);
+            FH_TRY(pack(&L.uq, q, d.q_rank));
+            FH_TRY(vec(m + "dq.norm", {d.q_rank}, d.qp, &L.dq_norm));
+        } else {
+            for (const Rows& r : q) in.add(r.name, r.row0, r.rows, r.rows_pad);
+        }
+        if (!sp.kv_source) {
+            L.c1 = in.cols();
+            in.add(m + "dkv", 0, kr, d.kp);
+            in.add(m + "dkv", kr, d.rot_dim, d.rp);
+            FH_TRY(vec(m + "dkv.norm", {kr}, d.kp, &L.dkv_norm));
+            FH_TRY(arena_.alloc(&L.lb.pool, (size_t)c_.kv_num_blocks * latent_block_elems(d)));
+        }
+        if (!(sp.attn_flags & FERRUM_HIP_ATTN_NO_HEAD_GATE)) {
+            L.c2 = section(L, in, GEMM_ACT_SIGMOID, g1);
+            in.add(m + "g", 0, H, pad32(H));
+        }
+        if (sp.attn_flags & FERRUM_HIP_ATTN_SINK) {
+            float* sink = nullptr;
+            FH_TRY(vec(m + "sink", {H}, H, &sink));
+            L.lb.sink = sink;
+        }
+        // per head: W_ukᵀ [latent, plain query dims], W_uv [value dims, latent]
+        FH_TRY(need(m + "uk", {(int64_t)H * dim, kr}));
+        FH_TRY(need(m + "uv", {(int64_t)H * vd, kr}));
+        FH_TRY(pack_fn(&L.uk, H, d.kp, dp, m + "uk", [&](const float* w, int g, int n, int k) {
+            return n < kr && k < dim ? w[((size_t)g * dim + k) * kr + n] : 0.f; }));
+        // [W_uk | W_uv] over the latent: the expansion of keys and values; its second part doubles as the per-head value projection
+        const float *uk = data(m + "uk"), *uv = data(m + "uv");
+        const int kn = H * dp;
+        FH_TRY(pack_fn(&L.expand, 1, kn + H * vp, d.kp, m + "uv", [&](const float*, int, int n, int k) {
+            if (k >= kr) return 0.f;
+            if (n < kn) return n % dp < dim ? uk[((size_t)(n / dp) * dim + n % dp) * kr + k] : 0.f;
+            n -= kn;
+            return n % vp < vd ? uv[((size_t)(n / vp) * vd + n % vp) * kr + k] : 0.f; }));
+        L.uv.w = L.expand.w + (size_t)kn * d.kp; L.uv.n = vp; L.uv.k = d.kp; L.uv.groups = H;
+        FH_TRY(need(m + "o", {D_, (int64_t)H * vd}));
+        // W_o, in a parallel block with a dense feed-forward behind W_down: [W_down | W_o]
+        const bool glu = sp.ff == FERRUM_HIP_FF_CLAMPED_GLU;
+        const std::string dn = m.substr(0, m.size() - 4) + "mlp.down";
+        const int F = glu ? sp.ff_width : 0, Fp = pad32(F);
+        if (glu) FH_TRY(need(dn, {D_, F}));
+        const float* down = data(dn);
+        FH_TRY(pack_fn(&L.o, 1, Dp_, Fp + H * vp, m + "o", [&](const float* w, int, int n, int k) {
+            if (n >= D_) return 0.f;
+            if (k < Fp) return k < F ? down[(size_t)n * F + k] : 0.f;
+            k -= Fp;
+            return k % vp < vd ? w[(size_t)n * H * vd + (k / vp) * vd + k % vp] : 0.f; }));
+        return rope(sp, &L.lb.cos_t, &L.lb.sin_t);
+    }
+    int recurrent_weights(Layer& L, Input& in, const std::string& m) {
+        const RglruDims& d = L.rd;
+        const int W = L.s.rnn_width, bs = W / d.blocks, bp = d.bp;
+        for (const char* part : {"y", "x"}) {
+            (*part == 'y' ? L.c0 : L.c1) = section(L, in, *part == 'y' ? GEMM_ACT_GELU_TANH : GEMM_ACT_NONE);
+            for (int g = 0; g < d.blocks; g++) in.add(m + part, g * bs, bs, bp, m + part + ".b");
+        }
+        FH_TRY(need(m + "ra", {d.blocks, bs, bs}));
+        FH_TRY(need(m + "ri", {d.blocks, bs, bs}));
+        // gate tiles: [block][16-channel tile][ra, ri] — packed as 2·bp rows per block in that order
+        const float *ra = data(m + "ra"), *ri = data(m + "ri");
+        Linear gates;
+        FH_TRY(pack_fn(&gates, d.blocks, 2 * bp, bp, m + "ra", [&](const float*, int g, int n, int k) {
+            const int ch = (n / 32) * 16 + n % 16;
+            const float* w = (n / 16) % 2 ? ri : ra;
+            return ch < bs && k < bs ? w[((size_t)g * bs + ch) * bs + k] : 0.f; }));
+        L.rb.gate_w = gates.w;
+        auto padded = [&](const std::string& name, const float** out, bool sp_fold, int taps) -> int {
+            const int64_t n = W;
+            if (taps > 1 || name == m + "conv") FH_TRY(need(name, {n, taps}));
+            else if (name == m + "ra.b" || name == m + "ri.b") FH_TRY(need(name, {d.blocks, bs}));
+            else FH_TRY(need(name, {n}));
+            const float* src = data(name);
+            std::vector<float> v((size_t)taps * d.wp, 0.f);
+            for (int j = 0; j < taps; j++)
+                for (int ch = 0; ch < W; ch++) {
+                    const float x = src ? src[(size_t)ch * taps + j] : 0.25f;
+                    v[(size_t)j * d.wp + (ch / bs) * bp + ch % bs] = sp_fold ? (float)softplus(x) : x;
+                }
+            float* dev = nullptr;
+            FH_TRY(arena_.upload(&dev, v));
+            *out = dev;
+            return 0;
+        };
+        FH_TRY(padded(m + "conv", &L.rb.conv_w, false, d.taps));
+        FH_TRY(padded(m + "conv.b", &L.rb.conv_b, false, 1));
+        FH_TRY(padded(m + "ra.b", &L.rb.ra_b, false, 1));
+        FH_TRY(padded(m + "ri.b", &L.rb.ri_b, false, 1));
+        FH_TRY(padded(m + "lam", &L.rb.lam, true, 1));
+        FH_TRY(need(m + "o", {D_, W}));
+        FH_TRY(pack_fn(&L.o, 1, Dp_, d.wp, m + "o", [&](const float* w, int, int n, int k) {
+            return n < D_ && k % bp < bs ? w[(size_t)n * W + (k / bp) * bs + k % bp] : 0.f; }));
+        FH_TRY(arena_.alloc(&L.rb.conv_state, (size_t)slots_ * std::max(d.taps - 1, 1) * d.wp));
+        FH_TRY(arena_.alloc(&L.rb.state, (size_t)slots_ * d.wp));
+        return 0;
+    }
+    int feed_forward_weights(Layer& L, Input& in, const std::string& p) {
+        const FerrumHipLayerSpec& sp = L.s;
+        const int F = sp.ff_width, Fp = pad32(F);
+        if (sp.ff == FERRUM_HIP_FF_XIELU) {
+            FH_TRY(unit_offset(p + "norm2", &L.norm2));
+            std::vector<Rows> rows = {{p + "rg2", 0, D_, Dp_}, {p + "mlp.up", 0, F, Fp}};
+            FH_TRY(pack(&L.ff_in, rows, D_));
+            FH_TRY(bias(&L.ff_in, rows, {p + "rg2.b", ""}));
+            FH_TRY(pack(&L.down, {{p + "mlp.down", 0, D_, Dp_}}, F));
+            FH_TRY(need(p + "mlp.act", {2}));
+            const float* act = data(p + "mlp.act");
+            L.ff_sec[0] = {0, GEMM_ACT_SIGMOID, 0, 0};
+            L.ff_sec[1] = {Dp_, GEMM_ACT_XIELU, (float)softplus(act ? act[0] : 0.5f), (float)softplus(act ? act[1] : 0.5f)};
+        } else if (sp.ff == FERRUM_HIP_FF_CLAMPED_GLU) {
+            // 16 gate columns, their 16 up columns, and so on; the down projection is part of the projection out
+            L.c_glu = section(L, in, GEMM_ACT_CLAMPED_GLU, L.g2, sp.ff_limit, 1.702f);
+            for (int f = 0; f < Fp; f += 16)
+                for (const char* part : {"mlp.gate", "mlp.up"}) {
+                    const int n = std::min(16, F - f);
+                    in.add(p + part, n > 0 ? f : 0, std::max(n, 0), 16);
+                }
+            L.c_att = L.c_glu + Fp;
+        } else if (sp.ff == FERRUM_HIP_FF_MOE_RELU2) {
+            std::vector<Rows> r = {{p + "mlp.router", 0, sp.experts, pad32(sp.experts)}};
+            FH_TRY(pack(&L.router, r, D_));
+            FH_TRY(bias(&L.router, r, {p + "mlp.router.b"}));
+            std::vector<const float*> up, down;
+            for (int e = 0; e < sp.experts; e++) {
+                const std::string x = p + "mlp.e" + std::to_string(e) + ".";
+                FH_TRY(need(x + "up", {F, D_}));
+                FH_TRY(need(x + "down", {D_, F}));
+                up.push_back(data(x + "up"));
+                down.push_back(data(x + "down"));
+            }
+            FH_TRY(pack_fn(&L.up, sp.experts, Fp, Dp_, "", [&](const float*, int g, int n, int k) { return n < F && k < D_ ? up[g][(size_t)n * D_ + k] : 0.f; }));
+            FH_TRY(pack_fn(&L.down, sp.experts, Dp_, Fp, "", [&](const float*, int g, int n, int k) { return n < D_ && k < F ? down[g][(size_t)n * F + k] : 0.f; }));
+        }
+        return 0;
+    }
+    int side_weights(Layer& L, const std::string& p, int li) {
+        const int S = lc_.token_side_dim, Sp = pad32(S);
+        FH_TRY(pack(&L.side_gate, {{p + "side.gate", 0, S, Sp}}, D_));
+        FH_TRY(pack(&L.side_proj, {{p + "side.proj", 0, D_, Dp_}}, S));
+        FH_TRY(vec(p + "side.norm", {D_}, Dp_, &L.side_norm));
+        // this layer's columns of the side embedding as a table of its own
+        return table("side.embed", c_.vocab, (int64_t)c_.num_layers * S, li * S, S, Sp, &L.side_table);
+    }
+
     struct Rows { std::string name; int row0, rows, rows_pad; };      // a run of a matrix's rows, zero-padded
+    // rows of a layer's input projection, each run with the name of its bias ("": none)
+    struct Input {
+        std::vector<Rows> rows;
+        std::vector<std::string> bias;
+        void add(const std::string& name, int row0, int n, int n_pad, const std::string& b = "") { rows.push_back({name, row0, n, n_pad}); bias.push_back(b); }
+        int cols() const { int n = 0; for (const Rows& r : rows) n += r.rows_pad; return n; }
+        bool biased() const { return std::any_of(bias.begin(), bias.end(), [](const std::string& b) { return !b.empty(); }); }
+    };
     const float* data(const std::string& name) const {
         auto it = host_.find(name);
         return it == host_.end() ? nullptr : it->second.data.data();
@@ -505,40 +722,65 @@ private:
         for (int i = 0; i < D_; i++) v[i] = 1.f + (w ? w[i] : 0.f);
         return arena_.upload(out, v);
     }
-    int table(const std::string& name, int rows, E** out) {
-        FH_TRY(need(name, {rows, D_}));
-        const size_t n = (size_t)rows * D_;
+    int scalar(const std::string& name, float* out) {
+        FH_TRY(need(name, {1}));
+        const float* w = data(name);
+        *out = w ? w[0] : 1.f;
+        return 0;
+    }
+    int table(const std::string& name, int rows, E** out) { return table(name, rows, D_, 0, D_, D_, out); }
+    // columns [col0, col0 + n) of a table of `cols` columns, rows padded to n_pad
+    int table(const std::string& name, int rows, int64_t cols, int64_t col0, int n, int n_pad, E** out) {
+        FH_TRY(need(name, {rows, cols}));
+        const size_t total = (size_t)rows * n_pad;
         if (synth_) {
-            FH_TRY(arena_.alloc(out, n));
-            hipLaunchKernelGGL(synth_kernel<E>, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, stream_, *out, n, mix(++seed_), 1.0f);
+            FH_TRY(arena_.alloc(out, total));
+            hipLaunchKernelGGL(synth_kernel<E>, dim3((unsigned)((total + 255) / 256)), dim3(256), 0, stream_, *out, total, mix(++seed_), 1.0f);
             FH_CHECK_LAUNCH();
             return 0;
         }
-        std::vector<E> v(n);
+        std::vector<E> v(total);
         const float* w = data(name);
-        for (size_t i = 0; i < n; i++) store(&v[i], w[i]);
+        for (int r = 0; r < rows; r++)
+            for (int i = 0; i < n_pad; i++) store(&v[(size_t)r * n_pad + i], i < n ? w[(size_t)r * cols + col0 + i] : 0.f);
         return arena_.upload(out, v);
     }
     // angle tables in double, stored fp32 like the other models'; layers with the same rotation share one
-    int rope(double base, int dims, const float** cos_t, const float** sin_t) {
+    int rope(const FerrumHipLayerSpec& sp, const float** cos_t, const float** sin_t) {
+        const int dims = sp.rot_dims, half = dims / 2;
         for (const Rope& r : ropes_)
-            if (r.base == base && r.dims == dims) { *cos_t = r.c; *sin_t = r.s; return 0; }
-        const int half = dims / 2;
+            if (r.dims == dims && r.base == sp.rot_base && r.factor == sp.rot_factor && r.original == sp.rot_original && r.fast == sp.rot_fast && r.slow == sp.rot_slow) {
+                *cos_t = r.c; *sin_t = r.s;
+                return 0;
+            }
+        std::vector<double> freq(half);
+        for (int i = 0; i < half; i++) freq[i] = pow(sp.rot_base, -2.0 * i / dims);
+        double size = 1.0;
+        if (sp.rot_factor > 0.0) {
+            // pair (not rounded) that turns `turns` times within the original length
+            auto pair_of = [&](double turns) { return dims * log(sp.rot_original / (2.0 * M_PI * turns)) / (2.0 * log(sp.rot_base)); };
+            const double lo = std::max(floor(pair_of(sp.rot_fast)), 0.0), hi = std::min(ceil(pair_of(sp.rot_slow)), dims - 1.0);
+            for (int i = 0; i < half; i++) {
+                const double ramp = std::min(std::max((i - lo) / std::max(hi - lo, 0.001), 0.0), 1.0);
+                freq[i] = freq[i] / sp.rot_factor * ramp + freq[i] * (1.0 - ramp);
+            }
+            size = 0.1 * log(sp.rot_factor) + 1.0;
+        }
         std::vector<float> cs((size_t)c_.max_seq_len * half), sn(cs.size());
         for (int p = 0; p < c_.max_seq_len; p++)
             for (int i = 0; i < half; i++) {
-                const double a = (double)p * pow(base, -2.0 * i / dims);
-                cs[(size_t)p * half + i] = (float)cos(a);
-                sn[(size_t)p * half + i] = (float)sin(a);
+                const double a = (double)p * freq[i];
+                cs[(size_t)p * half + i] = (float)(size * cos(a));
+                sn[(size_t)p * half + i] = (float)(size * sin(a));
             }
-        Rope r{base, dims, nullptr, nullptr};
+        Rope r{sp.rot_base, sp.rot_factor, sp.rot_original, sp.rot_fast, sp.rot_slow, dims, nullptr, nullptr};
         FH_TRY(arena_.upload(&r.c, cs));
         FH_TRY(arena_.upload(&r.s, sn));
         ropes_.push_back(r);
         *cos_t = r.c; *sin_t = r.s;
         return 0;
     }
-    struct Rope { double base; int dims; float *c, *s; };
+    struct Rope { double base, factor, original, fast, slow; int dims; float *c, *s; };
 
     FerrumHipModelConfig c_;
     FerrumHipLayeredConfig lc_;
@@ -556,7 +798,9 @@ private:
     // activations of one forward
     float *x_ = nullptr, *sub_ = nullptr, *partial_ = nullptr, *decay_ = nullptr, *drive_ = nullptr, *chunk_a_ = nullptr, *chunk_h_ = nullptr;
     E *xb_ = nullptr, *in_ = nullptr, *cq_ = nullptr, *q_ = nullptr, *q_lat_ = nullptr, *o_lat_ = nullptr, *attn_ = nullptr, *u_ = nullptr,
-      *rnn_out_ = nullptr, *head_in_ = nullptr;
+      *rnn_out_ = nullptr, *head_in_ = nullptr, *side_ = nullptr, *expert_h_ = nullptr, *expert_y_ = nullptr;
+    float *router_logits_ = nullptr, *expert_weights_ = nullptr;
+    int32_t *expert_ids_ = nullptr, *sorted_ = nullptr, *sorted_expert_ = nullptr, *sorted_total_ = nullptr;
     size_t partial_bytes_ = 0;
     // expansion of keys and values: one plan per distinct window
     std::vector<Plan> plans_;
@@ -575,13 +819,24 @@ int check_layered_config(const FerrumHipModelConfig& c, const FerrumHipLayeredCo
     FH_REQUIRE(c.tp_world <= 1, "layered model: tensor parallelism is not available");
     FH_REQUIRE(lc.dtype == FERRUM_HIP_DTYPE_BF16 || lc.dtype == FERRUM_HIP_DTYPE_F32, "layered model: dtype %d", lc.dtype);
     FH_REQUIRE(lc.bigram_buckets >= 0 && lc.state_slots >= 0, "layered model: bigram buckets %d, state slots %d", lc.bigram_buckets, lc.state_slots);
+    FH_REQUIRE(lc.block == FERRUM_HIP_BLOCK_GATED_POST_NORM || lc.block == FERRUM_HIP_BLOCK_PARALLEL_PRE_NORM, "layered model: block %d", lc.block);
+    const bool parallel = lc.block == FERRUM_HIP_BLOCK_PARALLEL_PRE_NORM;
+    FH_REQUIRE(lc.token_side_dim >= 0 && (parallel || !lc.token_side_dim), "layered model: per-layer token input of %d dimensions", lc.token_side_dim);
     for (int i = 0; i < c.num_layers; i++) {
         const FerrumHipLayerSpec& s = layers[i];
         if (s.mixer == FERRUM_HIP_MIXER_LATENT_ATTENTION) {
-            FH_REQUIRE(s.heads > 0 && s.dim > 0 && s.rot_dim > 0 && s.vdim > 0 && s.q_rank > 0 && s.kv_rank > 0 && s.window > 0,
+            FH_REQUIRE(s.heads > 0 && s.dim > 0 && s.rot_dim > 0 && s.vdim > 0 && s.q_rank >= 0 && s.kv_rank > 0 && (s.window > 0 || s.window == FERRUM_HIP_WINDOW_NONE),
                        "layer %d: latent attention sizes must be positive", i);
             FH_REQUIRE(s.rot_dims >= 0 && s.rot_dims % 2 == 0 && s.rot_dims <= s.rot_dim && (s.rot_dims == 0 || s.rot_base > 0.0),
                        "layer %d: rotated dimensions %d of %d", i, s.rot_dims, s.rot_dim);
+            FH_REQUIRE(s.rot_factor == 0.0 || (s.rot_factor > 0.0 && s.rot_original > 0.0 && s.rot_fast > 0.0 && s.rot_slow > 0.0 && s.rot_base > 0.0 && s.rot_base != 1.0),
+                       "layer %d: rotation scaling", i);
+            if (s.kv_source) {
+                FH_REQUIRE(s.kv_source > 0 && s.kv_source <= i, "layer %d: reads the latents of layer %d", i, s.kv_source - 1);
+                const FerrumHipLayerSpec& o = layers[s.kv_source - 1];
+                FH_REQUIRE(o.mixer == s.mixer && !o.kv_source && o.kv_rank == s.kv_rank && o.rot_dim == s.rot_dim,
+                           "layer %d: layer %d caches other latents, or none of its own", i, s.kv_source - 1);
+            }
         } else if (s.mixer == FERRUM_HIP_MIXER_RGLRU) {
             FH_REQUIRE(s.rnn_width > 0 && s.rnn_blocks > 0 && s.rnn_width % s.rnn_blocks == 0 && s.conv_taps > 0,
                        "layer %d: recurrence of width %d in %d blocks, %d taps", i, s.rnn_width, s.rnn_blocks, s.conv_taps);
@@ -589,7 +844,11 @@ int check_layered_config(const FerrumHipModelConfig& c, const FerrumHipLayeredCo
             set_error("layer %d: unknown mixer %d", i, s.mixer);
             return FERRUM_HIP_UNSUPPORTED;
         }
-        FH_REQUIRE(s.ff == FERRUM_HIP_FF_NONE || (s.ff == FERRUM_HIP_FF_XIELU && s.ff_width > 0), "layer %d: feed-forward %d of width %d", i, s.ff, s.ff_width);
+        FH_REQUIRE(s.ff == FERRUM_HIP_FF_NONE || ((s.ff == FERRUM_HIP_FF_CLAMPED_GLU || s.ff == FERRUM_HIP_FF_MOE_RELU2 ? parallel : s.ff == FERRUM_HIP_FF_XIELU && !parallel) && s.ff_width > 0),
+                   "layer %d: feed-forward %d of width %d", i, s.ff, s.ff_width);
+        FH_REQUIRE(s.ff != FERRUM_HIP_FF_MOE_RELU2 || (s.experts > 0 && s.experts <= 512 && s.top > 0 && s.top <= s.experts && s.top <= 64),
+                   "layer %d: %d of %d experts", i, s.top, s.experts);
+        FH_REQUIRE(!parallel || s.mixer == FERRUM_HIP_MIXER_LATENT_ATTENTION, "layer %d: a parallel block takes latent attention", i);
     }
     return 0;
 }

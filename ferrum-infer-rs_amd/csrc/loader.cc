@@ -8,7 +8,7 @@
 //   * quantize_config.json or config.json "quantization_config"   native_safetensors.rs:1475-1530, config.rs:26-45
 //   * config.json field extraction and per-architecture defaults  ferrum-models/src/definition.rs:225-375,
 //     models/llama_family.rs:596-680,733-810, moe_config.rs:91-130
-//   * layered architectures (Nerenex): per-layer descriptions and weights by name
+//   * layered architectures (Nerenex, Safolorn): per-layer descriptions and weights by name
 //   * tensor names                                        models/llama_family.rs:900-945, qwen3_moe/load.rs:178-260
 // Pure host code: nothing here touches the GPU except through ferrum_hip_model_set_* (runner.hip).
 #include <fcntl.h>
@@ -305,7 +305,7 @@ static std::string architecture(const FerrumHipCheckpoint* ck) {
 }
 
 // ── layered architectures ──
-static bool is_layered_arch(const std::string& arch) { return arch == "Nerenex"; }
+static bool is_layered_arch(const std::string& arch) { return arch == "Nerenex" || arch == "Safolorn"; }
 
 // required numbers of a config object; the first one missing or out of place is named in the error
 struct Fields {
@@ -330,7 +330,58 @@ struct Fields {
 };
 #define FH_FIELDS_OK(f) FH_REQUIRE((f).missing.empty(), "config.json: '%s' is missing or not a valid number", (f).missing.c_str())
 
-static int layered_spec(const Value& v, int index, FerrumHipLayerSpec* s) {
+// a layer of Safolorn: latent attention without query latent, window and head gates, with sinks; dense or sparse feed-forward
+static int safolorn_spec(const Value& v, int index, FerrumHipLayerSpec* s) {
+    memset(s, 0, sizeof(*s));
+    const std::string at = "layers[" + std::to_string(index) + "]";
+    const Value *type = v.get("type"), *ff = v.get("mlp");
+    FH_REQUIRE(type && type->kind == Value::Str, "config.json: %s has no type", at.c_str());
+    if (type->str != "latent_attention") {
+        set_error("config.json: %s has the unknown type '%s'", at.c_str(), type->str.c_str());
+        return FERRUM_HIP_UNSUPPORTED;
+    }
+    s->mixer = FERRUM_HIP_MIXER_LATENT_ATTENTION;
+    s->attn_flags = FERRUM_HIP_ATTN_NO_HEAD_GATE | FERRUM_HIP_ATTN_SINK;
+    s->window = FERRUM_HIP_WINDOW_NONE;
+    Fields m{v.get("mixer"), at + ".mixer", ""};
+    s->heads = m.size("heads"); s->dim = m.size("dim"); s->rot_dim = m.size("rot_dim"); s->vdim = m.size("vdim");
+    s->kv_rank = m.size("kv_rank"); s->scale = (float)m.num("scale");
+    auto given = [](const Fields& f, const char* key) { const Value* x = f.obj ? f.obj->get(key) : nullptr; return x && x->kind != Value::Null; };
+    if (given(m, "kv_from")) {
+        const int32_t j = m.size("kv_from");
+        FH_REQUIRE(j < index, "config.json: %s.mixer.kv_from = %d is no earlier layer", at.c_str(), j);
+        s->kv_source = j + 1;
+    }
+    Fields rot = m.sub("rot");
+    s->rot_dims = rot.size("dims"); s->rot_base = rot.num("base");
+    if (given(rot, "scaling")) {
+        Fields y = rot.sub("scaling");
+        s->rot_factor = y.num("factor"); s->rot_original = y.num("original"); s->rot_fast = y.num("fast"); s->rot_slow = y.num("slow");
+        FH_FIELDS_OK(y);
+        FH_REQUIRE(s->rot_factor > 0.0 && s->rot_original > 0.0 && s->rot_fast > 0.0 && s->rot_slow > 0.0,
+                   "config.json: %s.mixer.rot.scaling holds a number that is not positive", at.c_str());
+    }
+    FH_FIELDS_OK(m); FH_FIELDS_OK(rot);
+    if (!ff || ff->kind == Value::Null) return 0;
+    const Value* kind = ff->get("kind");
+    Fields f{ff, at + ".mlp", ""};
+    if (kind && kind->kind == Value::Str && kind->str == "dense") {
+        s->ff = FERRUM_HIP_FF_CLAMPED_GLU;
+        s->ff_width = f.size("ff"); s->ff_limit = (float)f.num("limit");
+        FH_FIELDS_OK(f);
+    } else if (kind && kind->kind == Value::Str && kind->str == "moe") {
+        s->ff = FERRUM_HIP_FF_MOE_RELU2;
+        Fields e = f.sub("expert"), r = f.sub("router");
+        s->ff_width = e.size("ff"); s->experts = r.size("experts"); s->top = r.size("top");
+        FH_FIELDS_OK(e); FH_FIELDS_OK(r);
+    } else {
+        set_error("config.json: %s.mlp has an unknown kind", at.c_str());
+        return FERRUM_HIP_UNSUPPORTED;
+    }
+    return 0;
+}
+
+static int nerenex_spec(const Value& v, int index, FerrumHipLayerSpec* s) {
     memset(s, 0, sizeof(*s));
     const std::string at = "layers[" + std::to_string(index) + "]";
     const Value *type = v.get("type"), *ff = v.get("mlp");
@@ -361,6 +412,35 @@ static int layered_spec(const Value& v, int index, FerrumHipLayerSpec* s) {
     s->ff = FERRUM_HIP_FF_XIELU;
     s->ff_width = f.size("ff");
     FH_FIELDS_OK(f);
+    return 0;
+}
+
+static int nerenex_whole(const FerrumHipCheckpoint* ck, FerrumHipLayeredConfig* c) {
+    memset(c, 0, sizeof(*c));
+    Fields f{&ck->config, "config", ""};
+    c->residual_mult = (float)f.num("residual_mult");
+    FH_FIELDS_OK(f);
+    Fields emb = f.sub("embedding");
+    if (const Value* bg = emb.obj ? emb.obj->get("bigram") : nullptr; bg && bg->kind == Value::Obj) {
+        Fields b{bg, "embedding.bigram", ""};
+        c->bigram_buckets = b.size("buckets");
+        c->bigram_mul_prev = b.integer("mul_prev");
+        c->bigram_mul_cur = b.integer("mul_cur");
+        FH_FIELDS_OK(b);
+        FH_REQUIRE(c->bigram_buckets > 0, "config.json: embedding.bigram.buckets must be positive");
+    }
+    return 0;
+}
+static int safolorn_whole(const FerrumHipCheckpoint* ck, FerrumHipLayeredConfig* c) {
+    memset(c, 0, sizeof(*c));
+    Fields f{&ck->config, "config", ""};
+    Fields side = f.sub("token_side");
+    c->block = FERRUM_HIP_BLOCK_PARALLEL_PRE_NORM;
+    c->residual_mult = 1.f;
+    c->untied_head = 1;
+    c->token_side_dim = side.size("dim");
+    FH_FIELDS_OK(side);
+    FH_REQUIRE(c->token_side_dim > 0, "config.json: token_side.dim must be positive");
     return 0;
 }
 
@@ -534,7 +614,7 @@ int ferrum_hip_checkpoint_model_config(const FerrumHipCheckpoint* ck, int max_se
     const std::string arch = architecture(ck);
     if (arch_out && arch_cap) snprintf(arch_out, arch_cap, "%s", arch.c_str());
     if (is_layered_arch(arch)) {
-        if (tied_lm_head) *tied_lm_head = 1;
+        if (tied_lm_head) *tied_lm_head = arch != "Safolorn";
         return layered_model_config(ck, max_seq_len_cap, cfg);
     }
     enum { Llama, Qwen3, Qwen3Moe, Mistral, Gemma3, Qwen2 } fam;
@@ -630,27 +710,15 @@ int ferrum_hip_checkpoint_model_config(const FerrumHipCheckpoint* ck, int max_se
 int ferrum_hip_checkpoint_layered_config(const FerrumHipCheckpoint* ck, int* is_layered, FerrumHipLayeredConfig* layered,
                                          FerrumHipLayerSpec* layers, int capacity) {
     FH_REQUIRE(ck && is_layered, "checkpoint_layered_config: null argument");
-    *is_layered = is_layered_arch(architecture(ck));
+    const std::string arch = architecture(ck);
+    *is_layered = is_layered_arch(arch);
     if (!*is_layered) return 0;
     const Value* ls = cfg_get(ck, "layers");
     FH_REQUIRE(ls && ls->kind == Value::Arr && !ls->arr.empty(), "config.json: 'layers' is missing or empty");
-    if (layered) {
-        memset(layered, 0, sizeof(*layered));
-        Fields f{&ck->config, "config", ""};
-        layered->residual_mult = (float)f.num("residual_mult");
-        FH_FIELDS_OK(f);
-        Fields emb = f.sub("embedding");
-        if (const Value* bg = emb.obj ? emb.obj->get("bigram") : nullptr; bg && bg->kind == Value::Obj) {
-            Fields b{bg, "embedding.bigram", ""};
-            layered->bigram_buckets = b.size("buckets");
-            layered->bigram_mul_prev = b.integer("mul_prev");
-            layered->bigram_mul_cur = b.integer("mul_cur");
-            FH_FIELDS_OK(b);
-            FH_REQUIRE(layered->bigram_buckets > 0, "config.json: embedding.bigram.buckets must be positive");
-        }
-    }
+    if (layered)
+        if (int rc = (arch == "Safolorn" ? safolorn_whole : nerenex_whole)(ck, layered)) return rc;
     for (int i = 0; layers && i < (int)ls->arr.size() && i < capacity; i++)
-        if (int rc = layered_spec(ls->arr[i], i, &layers[i])) return rc;
+        if (int rc = (arch == "Safolorn" ? safolorn_spec : nerenex_spec)(ls->arr[i], i, &layers[i])) return rc;
     return 0;
 }
 

@@ -59,18 +59,69 @@ __device__ __forceinline__ float block_sum(float q, float* red) {
     return t;
 }
 
-// One workgroup per row; a thread holds up to 4 quads of the row in registers, so the branch is read once.
+// x += Σ slabs of `sub` + Σ_j weights[row][j] · pairs[row·top + j]; elementwise, grid (rows, quads of columns / 256)
 template <typename E, bool VEC>
-__global__ __launch_bounds__(1024) void gated_post_norm_add_kernel(const float* __restrict__ sub, long ld_sub, int slabs, long slab_stride, const E* __restrict__ gate,
-                                                                   long ld_gate, const float* __restrict__ w, float mult, float eps,
-                                                                   float* __restrict__ x, E* __restrict__ xb, int dim, int ldb) {
-    __shared__ float red[16];
+__global__ __launch_bounds__(256) void branch_add_kernel(const float* __restrict__ sub, long ld_sub, int slabs, long slab_stride, const E* __restrict__ pairs,
+                                                         long ld_pair, const float* __restrict__ weights, int top, float* __restrict__ x,
+                                                         E* __restrict__ xb, int dim, int ldb) {
+    const long row = blockIdx.x;
+    const int i = (blockIdx.y * 256 + threadIdx.x) * 4;
+    if (i >= dim) return;
+    const float* sr = sub + row * ld_sub + i;
+    const E* pr = pairs + row * top * ld_pair + i;
+    if (VEC) {
+        typedef E e4 __attribute__((ext_vector_type(4)));
+        floatx4 v = *reinterpret_cast<const floatx4*>(sr);
+        const floatx4 xv = *reinterpret_cast<const floatx4*>(x + row * dim + i);
+        for (int z = 1; z < slabs; z++) v += *reinterpret_cast<const floatx4*>(sr + z * slab_stride);
+#pragma unroll 4
+        for (int j = 0; j < top; j++) {
+            const e4 e = *reinterpret_cast<const e4*>(pr + j * ld_pair);
+            const float w = weights[row * top + j];
+#pragma unroll
+            for (int k = 0; k < 4; k++) v[k] += w * (float)e[k];
+        }
+        v += xv;
+        e4 o;
+#pragma unroll
+        for (int k = 0; k < 4; k++) o[k] = (E)v[k];
+        *reinterpret_cast<floatx4*>(x + row * dim + i) = v;
+        *reinterpret_cast<e4*>(xb + row * ldb + i) = o;
+        return;
+    }
+    for (int k = 0; k < 4 && i + k < dim; k++) {
+        float v = sr[k];
+        for (int z = 1; z < slabs; z++) v += sr[z * slab_stride + k];
+        for (int j = 0; j < top; j++) v += weights[row * top + j] * (float)pr[j * ld_pair + k];
+        v += x[row * dim + i + k];
+        x[row * dim + i + k] = v;
+        xb[row * ldb + i + k] = (E)v;
+    }
+}
+template <typename E>
+int branch_add(const float* sub, long ld_sub, int slabs, long slab_stride, const E* pairs, long ld_pair, const float* weights, int top, float* x, E* xb,
+               int rows, int dim, int ldb, hipStream_t s) {
+    const bool vec = dim % 4 == 0 && ld_sub % 4 == 0 && ld_pair % 4 == 0 && ldb % 4 == 0 && slab_stride % 4 == 0;
+    const dim3 grid(rows, cdiv(dim, 1024));
+    if (vec) hipLaunchKernelGGL((branch_add_kernel<E, true>), grid, dim3(256), 0, s, sub, ld_sub, slabs, slab_stride, pairs, ld_pair, weights, top, x, xb, dim, ldb);
+    else hipLaunchKernelGGL((branch_add_kernel<E, false>), grid, dim3(256), 0, s, sub, ld_sub, slabs, slab_stride, pairs, ld_pair, weights, top, x, xb, dim, ldb);
+    FH_CHECK_LAUNCH();
+    return 0;
+}
+
+// One workgroup per row; a thread holds up to 4 quads of the row in registers, so the branch is read once.  NEXT: the copy is the row
+// divided by its root mean square, the input of a block that norms ahead of its sublayers.
+template <typename E, bool VEC, bool GATE, bool NEXT>
+__global__ __launch_bounds__(1024) void post_norm_add_kernel(const float* __restrict__ sub, long ld_sub, int slabs, long slab_stride, const E* __restrict__ gate,
+                                                             long ld_gate, const float* __restrict__ w, float mult, float eps,
+                                                             float* __restrict__ x, E* __restrict__ xb, int dim, int ldb) {
+    __shared__ float red[32];
     const long row = blockIdx.x;
     const float* sr = sub + row * ld_sub;
-    const E* gr = gate + row * ld_gate;
+    const E* gr = GATE ? gate + row * ld_gate : nullptr;
     float* xr = x + row * dim;
     E* br = xb + row * ldb;
-    float q = 0.f;
+    float q = 0.f, n = 0.f;
     if (VEC) {
         typedef E e4 __attribute__((ext_vector_type(4)));
         floatx4 v[4], xv[4], wv[4];
@@ -80,11 +131,12 @@ __global__ __launch_bounds__(1024) void gated_post_norm_add_kernel(const float* 
             if (i < dim) {
                 v[c] = *reinterpret_cast<const floatx4*>(sr + i);
                 for (int z = 1; z < slabs; z++) v[c] += *reinterpret_cast<const floatx4*>(sr + z * slab_stride + i);
-                const e4 gv = *reinterpret_cast<const e4*>(gr + i);
+                e4 gv = {};
+                if (GATE) gv = *reinterpret_cast<const e4*>(gr + i);
                 xv[c] = *reinterpret_cast<const floatx4*>(xr + i);
                 wv[c] = *reinterpret_cast<const floatx4*>(w + i);
 #pragma unroll
-                for (int j = 0; j < 4; j++) { v[c][j] *= (float)gv[j]; q += v[c][j] * v[c][j]; }
+                for (int j = 0; j < 4; j++) { if (GATE) v[c][j] *= (float)gv[j]; q += v[c][j] * v[c][j]; }
             }
         }
         const float inv = mult / sqrtf(block_sum(q, red) / (float)dim + eps);
@@ -92,10 +144,19 @@ __global__ __launch_bounds__(1024) void gated_post_norm_add_kernel(const float* 
         for (int c = 0; c < 4; c++) {
             const int i = (c * blockDim.x + threadIdx.x) * 4;
             if (i < dim) {
+#pragma unroll
+                for (int j = 0; j < 4; j++) { xv[c][j] += v[c][j] * inv * wv[c][j]; n += xv[c][j] * xv[c][j]; }
+                *reinterpret_cast<floatx4*>(xr + i) = xv[c];
+            }
+        }
+        const float unit = NEXT ? 1.0f / sqrtf(block_sum(n, red + 16) / (float)dim + eps) : 1.0f;
+#pragma unroll
+        for (int c = 0; c < 4; c++) {
+            const int i = (c * blockDim.x + threadIdx.x) * 4;
+            if (i < dim) {
                 e4 o;
 #pragma unroll
-                for (int j = 0; j < 4; j++) { xv[c][j] += v[c][j] * inv * wv[c][j]; o[j] = (E)xv[c][j]; }
-                *reinterpret_cast<floatx4*>(xr + i) = xv[c];
+                for (int j = 0; j < 4; j++) o[j] = (E)(xv[c][j] * unit);
                 *reinterpret_cast<e4*>(br + i) = o;
             }
         }
@@ -104,26 +165,31 @@ __global__ __launch_bounds__(1024) void gated_post_norm_add_kernel(const float* 
     auto branch = [&](int i) {
         float t = sr[i];
         for (int z = 1; z < slabs; z++) t += sr[z * slab_stride + i];
-        return t * (float)gr[i];
+        return GATE ? t * (float)gr[i] : t;
     };
     for (int i = threadIdx.x; i < dim; i += blockDim.x) { const float t = branch(i); q += t * t; }
     const float inv = mult / sqrtf(block_sum(q, red) / (float)dim + eps);
     for (int i = threadIdx.x; i < dim; i += blockDim.x) {
         const float t = xr[i] + branch(i) * inv * w[i];
         xr[i] = t;
-        br[i] = (E)t;
+        n += t * t;
+        if (!NEXT) br[i] = (E)t;
+    }
+    if (NEXT) {
+        const float unit = 1.0f / sqrtf(block_sum(n, red + 16) / (float)dim + eps);
+        for (int i = threadIdx.x; i < dim; i += blockDim.x) br[i] = (E)(xr[i] * unit);
     }
 }
 
 template <typename E>
-int gated_post_norm_add(const float* sub, long ld_sub, int slabs, long slab_stride, const E* gate, long ld_gate, const float* w, float mult, float eps, float* x,
-                        E* xb, int rows, int dim, int ldb, hipStream_t s) {
+int post_norm_add(const float* sub, long ld_sub, int slabs, long slab_stride, const E* gate, long ld_gate, const float* w, float mult, float eps, bool next_norm,
+                  float* x, E* xb, int rows, int dim, int ldb, hipStream_t s) {
     const int threads = rows <= 512 && dim >= 2048 ? 1024 : 256;
     const bool vec = dim % 4 == 0 && dim <= threads * 16 && ld_sub % 4 == 0 && ld_gate % 4 == 0 && ldb % 4 == 0 && slab_stride % 4 == 0;
-    if (vec)
-        hipLaunchKernelGGL((gated_post_norm_add_kernel<E, true>), dim3(rows), dim3(threads), 0, s, sub, ld_sub, slabs, slab_stride, gate, ld_gate, w, mult, eps, x, xb, dim, ldb);
-    else
-        hipLaunchKernelGGL((gated_post_norm_add_kernel<E, false>), dim3(rows), dim3(threads), 0, s, sub, ld_sub, slabs, slab_stride, gate, ld_gate, w, mult, eps, x, xb, dim, ldb);
+#define POST(V, G, N) hipLaunchKernelGGL((post_norm_add_kernel<E, V, G, N>), dim3(rows), dim3(threads), 0, s, sub, ld_sub, slabs, slab_stride, gate, ld_gate, w, mult, eps, x, xb, dim, ldb)
+    if (gate) { if (next_norm) { if (vec) POST(true, true, true); else POST(false, true, true); } else { if (vec) POST(true, true, false); else POST(false, true, false); } }
+    else { if (next_norm) { if (vec) POST(true, false, true); else POST(false, false, true); } else { if (vec) POST(true, false, false); else POST(false, false, false); } }
+#undef POST
     FH_CHECK_LAUNCH();
     return 0;
 }
@@ -132,11 +198,11 @@ template <typename E>
 __global__ __launch_bounds__(256) void rms_norm_rows_kernel(const float* __restrict__ x, const int32_t* __restrict__ row_idx,
                                                             const float* __restrict__ w, float eps, E* __restrict__ out, int dim, int ldo) {
     __shared__ float red[4];
-    const float* xr = x + (long)row_idx[blockIdx.x] * dim;
+    const float* xr = x + (row_idx ? (long)row_idx[blockIdx.x] : (long)blockIdx.x) * dim;
     float q = 0.f;
     for (int i = threadIdx.x; i < dim; i += 256) q += xr[i] * xr[i];
     const float inv = 1.0f / sqrtf(block_sum(q, red) / (float)dim + eps);
-    for (int i = threadIdx.x; i < dim; i += 256) out[(long)blockIdx.x * ldo + i] = (E)(xr[i] * inv * w[i]);
+    for (int i = threadIdx.x; i < dim; i += 256) out[(long)blockIdx.x * ldo + i] = (E)(w ? xr[i] * inv * w[i] : xr[i] * inv);
 }
 template <typename E>
 int rms_norm_rows(const float* x, const int32_t* row_idx, const float* w, float eps, E* out, int rows, int dim, int ldo, hipStream_t s) {
@@ -147,8 +213,9 @@ int rms_norm_rows(const float* x, const int32_t* row_idx, const float* w, float 
 
 #define INSTANTIATE(E)                                                                                                                  \
     template int embed_bigram<E>(const E*, const E*, int, int64_t, int64_t, const BatchView&, float*, E*, int, int, hipStream_t);        \
-    template int gated_post_norm_add<E>(const float*, long, int, long, const E*, long, const float*, float, float, float*, E*, int, int, int,       \
-                                        hipStream_t);                                                                                   \
+    template int branch_add<E>(const float*, long, int, long, const E*, long, const float*, int, float*, E*, int, int, int, hipStream_t); \
+    template int post_norm_add<E>(const float*, long, int, long, const E*, long, const float*, float, float, bool, float*, E*, int, int, \
+                                  int, hipStream_t);                                                                                    \
     template int rms_norm_rows<E>(const float*, const int32_t*, const float*, float, E*, int, int, int, hipStream_t);
 INSTANTIATE(bf16)
 INSTANTIATE(float)

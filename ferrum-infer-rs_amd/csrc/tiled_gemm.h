@@ -33,14 +33,25 @@ template <> struct Frag<float> {
 
 static inline int pad32(int n) { return (n + 31) / 32 * 32; }
 
-enum GemmAct : int { GEMM_ACT_NONE = 0, GEMM_ACT_SIGMOID = 1, GEMM_ACT_GELU_TANH = 2, GEMM_ACT_XIELU = 3 };
+enum GemmAct : int { GEMM_ACT_NONE = 0, GEMM_ACT_SIGMOID = 1, GEMM_ACT_GELU_TANH = 2, GEMM_ACT_XIELU = 3, GEMM_ACT_RELU2 = 4, GEMM_ACT_CLAMPED_GLU = 5 };
 constexpr int GEMM_MAX_SECTIONS = 6;
 struct GemmSection {          // columns [begin, next section's begin) of a fused projection; begin is a multiple of 32
     int begin, act;
-    float p, q;               // xIELU: softplus of its two parameters
+    float p, q;               // xIELU: softplus of its two parameters; clamped GLU: limit, slope of the sigmoid
+    float mul = 1.f;          // factor of the accumulator, ahead of bias and activation (a norm's gain that is a single number)
+};
+// A gated section pairs 16-column tiles (gate, up, gate, up, …) whose weights are packed that way; a wave holds both tiles of a pair, and
+// the result takes the first half of the section's columns.
+
+// Rows sorted by weight group (an expert's tokens), in blocks of `block` rows of one group each; the kernels read the block count from
+// the device, so a launch is sized for the largest one.  Place p of the list stands for row id[p] of the output and row id[p] / div of x;
+// ids of m and more are padding.
+struct GemmRows {
+    const int32_t *id = nullptr, *group = nullptr, *total = nullptr;      // [places], [blocks], places in use
+    int block = 0, max_blocks = 0, div = 1;
 };
 
-// out[r][g·out_group + c] = act(x[r][g·x_group ..] · W_gᵀ + bias) · row_scale[r][g]
+// out[r][g·out_group + c] = act(mul · x[r][g·x_group ..] · W_gᵀ + bias) · row_scale[r][g] · col_scale[col_scale_row[r]][c]
 template <typename E>
 struct TiledGemm {
     const E* x = nullptr; long ldx = 0, x_group = 0;
@@ -54,6 +65,8 @@ struct TiledGemm {
     long ldo = 0, out_group = 0;
     int slabs = 1; long slab_stride = 0;  // > 1: K split over workgroups, part z at out_f32 + z·slab_stride, summed by the consumer
     const E* row_scale = nullptr; long ld_scale = 0;
+    const E* col_scale = nullptr; const uint32_t* col_scale_row = nullptr; long ld_col_scale = 0;
+    GemmRows rows;                        // (bias, groups and the x / out group strides are not used with it)
     int nsec = 0;
     GemmSection sec[GEMM_MAX_SECTIONS] = {};
 };
@@ -78,6 +91,13 @@ template <> struct ActMath<bf16> {
 template <typename E>
 __device__ __forceinline__ float gelu_tanh_f32(float z) {
     return 0.5f * z * (1.0f + ActMath<E>::tanh(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+}
+// gate bounded from above, linear half on both sides
+template <typename E>
+__device__ __forceinline__ float clamped_glu_f32(float g, float u, float limit, float slope) {
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    return g * ActMath<E>::sigmoid(slope * g) * (u + 1.0f);
 }
 // quadratic right of zero, exponential left of it, slope 1/2 at zero; sp / sq: softplus of the two trained numbers
 template <typename E>

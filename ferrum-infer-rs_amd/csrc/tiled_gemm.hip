@@ -14,20 +14,42 @@ __device__ __forceinline__ float gemm_act(const GemmSection& sec, float v) {
     if (sec.act == GEMM_ACT_SIGMOID) return ActMath<E>::sigmoid(v);
     if (sec.act == GEMM_ACT_GELU_TANH) return gelu_tanh_f32<E>(v);
     if (sec.act == GEMM_ACT_XIELU) return xielu_f32<E>(v, sec.p, sec.q);
+    if (sec.act == GEMM_ACT_RELU2) { v = fmaxf(v, 0.f); return v * v; }
     return v;
 }
+// output row of place r, −1: none
 template <typename E>
-__device__ __forceinline__ void gemm_epilogue(const TiledGemm<E>& p, const GemmSection& sec, int g, int row, int col, float v) {
-    if (row >= p.m || col >= p.n_store) return;
-    if (p.bias) v += p.bias[(long)g * p.n + col];
-    v = gemm_act<E>(sec, v);
+__device__ __forceinline__ int gemm_out_row(const TiledGemm<E>& p, int r) {
+    if (p.rows.id) r = p.rows.id[r];
+    return r < p.m ? r : -1;
+}
+template <typename E>
+__device__ __forceinline__ void gemm_store(const TiledGemm<E>& p, int g, int row, int col, float v) {
     if (p.row_scale) v *= (float)p.row_scale[row * p.ld_scale + g];
-    const long o = row * p.ldo + g * p.out_group + col;
+    if (p.col_scale) v *= (float)p.col_scale[p.col_scale_row[row] * p.ld_col_scale + col];
+    const long o = row * p.ldo + (p.rows.id ? 0 : g * p.out_group) + col;
     if (p.out_f32) p.out_f32[o] = v; else p.out[o] = (E)v;
 }
 template <typename E>
+__device__ __forceinline__ void gemm_epilogue(const TiledGemm<E>& p, const GemmSection& sec, int g, int place, int col, float v) {
+    const int row = gemm_out_row(p, place);
+    if (row < 0 || col >= p.n_store) return;
+    v *= sec.mul;
+    if (p.bias) v += p.bias[(long)g * p.n + col];
+    gemm_store(p, g, row, col, gemm_act<E>(sec, v));
+}
+// accumulators of a (gate, up) pair of tiles; col: the gate's column
+template <typename E>
+__device__ __forceinline__ float gemm_gated(const TiledGemm<E>& p, const GemmSection& sec, int col, float gate, float up) {
+    gate *= sec.mul;
+    up *= sec.mul;
+    if (p.bias) { gate += p.bias[col]; up += p.bias[col + 16]; }
+    return clamped_glu_f32<E>(gate, up, sec.p, sec.q);
+}
+__device__ __forceinline__ int gemm_gated_col(const GemmSection& sec, int col) { return sec.begin + ((col - sec.begin) >> 5) * 16 + (col & 15); }
+template <typename E>
 __device__ __forceinline__ GemmSection gemm_section(const TiledGemm<E>& p, int col) {
-    GemmSection s = {0, GEMM_ACT_NONE, 0.f, 0.f};
+    GemmSection s = {0, GEMM_ACT_NONE, 0.f, 0.f, 1.f};
 #pragma unroll
     for (int i = 0; i < GEMM_MAX_SECTIONS; i++)
         if (i < p.nsec && col >= p.sec[i].begin) s = p.sec[i];
@@ -41,7 +63,11 @@ __device__ __forceinline__ const E* gemm_row(const TiledGemm<E>& p, int t, int g
         const int tiles = (p.m + 15) >> 4;
         return p.x + (long)p.x_blocks[t < tiles ? t : tiles - 1] * p.x_block_elems + (a * 16 + b) * 8;
     }
-    const int r = t * 16 + b;
+    int r = t * 16 + b;
+    if (p.rows.id) {
+        r = p.rows.id[r];
+        return p.x + (long)((unsigned)(r < p.m ? r : p.m - 1) / (unsigned)p.rows.div) * p.ldx + 8 * a;
+    }
     return p.x + (long)(r < p.m ? r : p.m - 1) * p.ldx + g * p.x_group + 8 * a;
 }
 template <typename E>
@@ -58,7 +84,12 @@ __global__ __launch_bounds__(512) void tiled_gemm_kernel(TiledGemm<E> p, int kw)
     const int a = lane >> 4, b = lane & 15;
     const int cw = (blockDim.x >> 6) / kw, part = wave % kw, cg = wave / kw;
     const int n0 = (blockIdx.x * cw + cg) * 16 * J, rb = blockIdx.y;
-    const int g = p.slabs > 1 ? 0 : blockIdx.z, z = p.slabs > 1 ? blockIdx.z : 0;
+    const int z = p.slabs > 1 ? blockIdx.z : 0;
+    int g = p.slabs > 1 ? 0 : blockIdx.z;
+    if (p.rows.id) {
+        if (rb * 16 * MT >= *p.rows.total) return;
+        g = p.rows.group[rb];
+    }
     const int ksteps = p.k >> 5, parts = kw * p.slabs, mine = z * kw + part;
     const bool live = n0 < p.n;
     const int s0 = live ? ksteps * mine / parts : 0, s1 = live ? ksteps * (mine + 1) / parts : 0;
@@ -111,8 +142,20 @@ __global__ __launch_bounds__(512) void tiled_gemm_kernel(TiledGemm<E> p, int kw)
     }
     if (p.slabs > 1) p.out_f32 += z * p.slab_stride;
     const GemmSection sec = gemm_section(p, n0);
+    const bool gated = J == 2 && sec.act == GEMM_ACT_CLAMPED_GLU;
     if (kw == 1) {
         if (!live) return;
+        if constexpr (J == 2)
+            if (gated) {
+#pragma unroll
+                for (int mt = 0; mt < MT; mt++)
+#pragma unroll
+                    for (int r = 0; r < 4; r++) {
+                        const int row = gemm_out_row(p, (rb * MT + mt) * 16 + 4 * a + r);
+                        if (row >= 0) gemm_store(p, g, row, gemm_gated_col(sec, n0 + b), gemm_gated(p, sec, n0 + b, acc[mt][0][r], acc[mt][J - 1][r]));
+                    }
+                return;
+            }
 #pragma unroll
         for (int mt = 0; mt < MT; mt++)
 #pragma unroll
@@ -127,10 +170,25 @@ __global__ __launch_bounds__(512) void tiled_gemm_kernel(TiledGemm<E> p, int kw)
         for (int j = 0; j < J; j++) red[(wave * MT * J + mt * J + j) * 64 + lane] = acc[mt][j];
     __syncthreads();
     if (!live) return;
-    // tile t of the column group is summed (in the order of the K parts) and finished by part t mod kw
-    for (int t = part; t < MT * J; t += kw) {
+    auto summed = [&](int t) {
         floatx4 v = red[(cg * kw * MT * J + t) * 64 + lane];
         for (int q = 1; q < kw; q++) v += red[((cg * kw + q) * MT * J + t) * 64 + lane];
+        return v;
+    };
+    if (gated) {
+        for (int mt = part; mt < MT; mt += kw) {
+            const floatx4 gate = summed(mt * J), up = summed(mt * J + 1);
+#pragma unroll
+            for (int r = 0; r < 4; r++) {
+                const int row = gemm_out_row(p, (rb * MT + mt) * 16 + 4 * a + r);
+                if (row >= 0) gemm_store(p, g, row, gemm_gated_col(sec, n0 + b), gemm_gated(p, sec, n0 + b, gate[r], up[r]));
+            }
+        }
+        return;
+    }
+    // tile t of the column group is summed (in the order of the K parts) and finished by part t mod kw
+    for (int t = part; t < MT * J; t += kw) {
+        const floatx4 v = summed(t);
         const int mt = t / J, j = t % J;
 #pragma unroll
         for (int r = 0; r < 4; r++) gemm_epilogue(p, sec, g, (rb * MT + mt) * 16 + 4 * a + r, n0 + 16 * j + b, v[r]);
@@ -142,14 +200,16 @@ __global__ __launch_bounds__(512) void tiled_gemm_kernel(TiledGemm<E> p, int kw)
 __global__ __launch_bounds__(256, 2) void tiled_gemm_big_kernel(TiledGemm<bf16> p, int mtiles, int ntiles) {
     __shared__ __attribute__((aligned(16))) bf16 lds[2][32 * 512];      // per stage: 16 A fragments, 16 B fragments
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
-    const int a = lane >> 4, b = lane & 15, g = blockIdx.z;
+    const int a = lane >> 4, b = lane & 15;
     // workgroups go round-robin over 8 XCDs: give each XCD a contiguous run of tiles, and walk 8 row tiles per column tile
+    if (p.rows.id) mtiles = *p.rows.total >> 7;
     const int total = mtiles * ntiles, l = blockIdx.x;
+    if (l >= total) return;
     const int q8 = total / 8, r8 = total % 8, xcd = l % 8;
     const int id = (xcd < r8 ? xcd * (q8 + 1) : r8 * (q8 + 1) + (xcd - r8) * q8) + l / 8;
     const int band = id / (8 * ntiles), rows_in = min(8, mtiles - band * 8), in = id - band * 8 * ntiles;
     const int m0 = (band * 8 + in % rows_in) * 128, n0 = (in / rows_in) * 128;
-    const int ksteps = p.k >> 5, ntl = p.n >> 4;
+    const int ksteps = p.k >> 5, ntl = p.n >> 4, g = p.rows.id ? p.rows.group[m0 >> 7] : blockIdx.z;
     const int wm = wave >> 1, wn = wave & 1;
     // this wave's 8 fragments of a stage: A row tiles 2·wave, 2·wave + 1 and B column tiles 2·wave, 2·wave + 1, two k-steps each
     const bf16 *ap[2], *bp[2];
@@ -204,34 +264,57 @@ __global__ __launch_bounds__(256, 2) void tiled_gemm_big_kernel(TiledGemm<bf16> 
         __syncthreads();
     }
     // epilogue: activations on the accumulators, then through LDS (the stages are free; a wave's 64 × 64 tile is its own) so that rows
-    // leave in 16-byte pieces, 128 or 256 contiguous bytes per row
+    // leave in 16-byte pieces, 128 or 256 contiguous bytes per row.  A gated pair of tiles leaves 16 columns in the first one's place.
+    GemmSection sec[2];
+    int col0[2];
+#pragma unroll
+    for (int c = 0; c < 2; c++) {
+        col0[c] = n0 + wn * 64 + c * 32;
+        sec[c] = gemm_section(p, min(col0[c], p.n - 1));
+    }
+    auto value = [&](int c, int j, int i, int r, float& v) {               // false: the up tile of a pair
+        const int jj = 2 * c + j;
+        if (sec[c].act == GEMM_ACT_CLAMPED_GLU) {
+            if (j) return false;
+            v = gemm_gated(p, sec[c], min(col0[c], p.n - 32) + b, acc[i][2 * c][r], acc[i][2 * c + 1][r]);
+            return true;
+        }
+        v = acc[i][jj][r] * sec[c].mul;
+        if (p.bias) v += p.bias[(long)g * p.n + min(col0[c] + 16 * j + b, p.n - 1)];
+        v = gemm_act<bf16>(sec[c], v);
+        return true;
+    };
     if (p.n_store % 8 == 0 && p.ldo % 8 == 0 && p.out_group % 8 == 0) {
         bf16* lo = &lds[0][0] + wave * 64 * 72;                    // rows of 72: 36 KiB for the four waves
         float* lf = reinterpret_cast<float*>(&lds[0][0]) + wave * 32 * 68;      // fp32 outputs: 32 rows of 68 at a time
+        // column of the tile → column of the output, −1: not stored
+        auto out_col = [&](int col) {
+            const int c = col >> 5;
+            if (c ? sec[1].act == GEMM_ACT_CLAMPED_GLU : sec[0].act == GEMM_ACT_CLAMPED_GLU)
+                return col & 16 || (c ? col0[1] : col0[0]) >= p.n ? -1 : gemm_gated_col(c ? sec[1] : sec[0], c ? col0[1] : col0[0]) + (col & 15);
+            return n0 + wn * 64 + col < p.n_store ? n0 + wn * 64 + col : -1;
+        };
 #pragma unroll
         for (int half = 0; half < 2; half++) {
 #pragma unroll
-            for (int j = 0; j < 4; j++) {
-                const int col0 = n0 + wn * 64 + j * 16;
-                const GemmSection sec = gemm_section(p, min(col0, p.n - 1));
-                const float bias = p.bias ? p.bias[(long)g * p.n + min(col0 + b, p.n - 1)] : 0.f;
+            for (int j = 0; j < 4; j++)
 #pragma unroll
                 for (int i = 2 * half; i < 2 * half + 2; i++)
 #pragma unroll
                     for (int r = 0; r < 4; r++) {
-                        const float v = gemm_act<bf16>(sec, acc[i][j][r] + bias);
+                        float v;
+                        if (!value(j >> 1, j & 1, i, r, v)) continue;
                         if (p.out_f32) lf[((i & 1) * 16 + 4 * a + r) * 68 + j * 16 + b] = v;
                         else lo[(i * 16 + 4 * a + r) * 72 + j * 16 + b] = (bf16)v;
                     }
-            }
             if (p.out_f32) {                                       // (wave-private: LDS operations of a wave complete in order)
 #pragma unroll
                 for (int q = 0; q < 8; q++) {
-                    const int row = q * 4 + (lane >> 4), col = (lane & 15) * 4, gr = m0 + wm * 64 + half * 32 + row, gc = n0 + wn * 64 + col;
-                    if (gr < p.m && gc < p.n_store) {
-                        floatx4 v = *reinterpret_cast<const floatx4*>(lf + row * 68 + col);
+                    const int row = q * 4 + (lane >> 4), gr = gemm_out_row(p, m0 + wm * 64 + half * 32 + row), gc = out_col((lane & 15) * 4);
+                    if (gr >= 0 && gc >= 0) {
+                        floatx4 v = *reinterpret_cast<const floatx4*>(lf + row * 68 + (lane & 15) * 4);
                         if (p.row_scale) v *= (float)p.row_scale[gr * p.ld_scale + g];
-                        *reinterpret_cast<floatx4*>(p.out_f32 + gr * p.ldo + g * p.out_group + gc) = v;
+                        *reinterpret_cast<floatx4*>(p.out_f32 + gr * p.ldo + (p.rows.id ? 0 : g * p.out_group) + gc) = v;
                     }
                 }
             }
@@ -239,34 +322,42 @@ __global__ __launch_bounds__(256, 2) void tiled_gemm_big_kernel(TiledGemm<bf16> 
         if (p.out_f32) return;
 #pragma unroll
         for (int q = 0; q < 8; q++) {
-            const int row = q * 8 + (lane >> 3), col = (lane & 7) * 8, gr = m0 + wm * 64 + row, gc = n0 + wn * 64 + col;
-            if (gr < p.m && gc < p.n_store) {
-                bf16x8 v = *reinterpret_cast<const bf16x8*>(lo + row * 72 + col);
+            const int row = q * 8 + (lane >> 3), gr = gemm_out_row(p, m0 + wm * 64 + row), gc = out_col((lane & 7) * 8);
+            if (gr >= 0 && gc >= 0) {
+                bf16x8 v = *reinterpret_cast<const bf16x8*>(lo + row * 72 + (lane & 7) * 8);
                 if (p.row_scale) {
                     const float f = (float)p.row_scale[gr * p.ld_scale + g];
 #pragma unroll
                     for (int e = 0; e < 8; e++) v[e] = (bf16)((float)v[e] * f);
                 }
-                *reinterpret_cast<bf16x8*>(p.out + gr * p.ldo + g * p.out_group + gc) = v;
+                if (p.col_scale) {
+                    const bf16x8 f = *reinterpret_cast<const bf16x8*>(p.col_scale + p.col_scale_row[gr] * p.ld_col_scale + gc);
+#pragma unroll
+                    for (int e = 0; e < 8; e++) v[e] = (bf16)((float)v[e] * (float)f[e]);
+                }
+                *reinterpret_cast<bf16x8*>(p.out + gr * p.ldo + (p.rows.id ? 0 : g * p.out_group) + gc) = v;
             }
         }
         return;
     }
 #pragma unroll
     for (int j = 0; j < 4; j++) {
-        const int col0 = n0 + wn * 64 + j * 16;
-        if (col0 >= p.n) break;
-        const GemmSection sec = gemm_section(p, col0);
+        if (col0[j >> 1] >= p.n) break;
 #pragma unroll
         for (int i = 0; i < 4; i++)
 #pragma unroll
-            for (int r = 0; r < 4; r++) gemm_epilogue(p, sec, g, m0 + wm * 64 + i * 16 + 4 * a + r, col0 + b, acc[i][j][r]);
+            for (int r = 0; r < 4; r++) {
+                float v;
+                const int row = gemm_out_row(p, m0 + wm * 64 + i * 16 + 4 * a + r), col = col0[j >> 1] + (j & 1) * 16 + b;
+                if (row >= 0 && col < p.n_store && value(j >> 1, j & 1, i, r, v))
+                    gemm_store(p, g, row, sec[j >> 1].act == GEMM_ACT_CLAMPED_GLU ? gemm_gated_col(sec[j >> 1], col) : col, v);
+            }
     }
 }
 
 static int launch_big(const TiledGemm<bf16>& g, hipStream_t s) {
-    const int mtiles = cdiv(g.m, 128), ntiles = cdiv(g.n, 128);
-    form_hit(FORM_TILED_GEMM_BIG);
+    const int mtiles = g.rows.id ? g.rows.max_blocks : cdiv(g.m, 128), ntiles = cdiv(g.n, 128);
+    form_hit(g.rows.id ? FORM_TILED_GEMM_GROUPED_BIG : FORM_TILED_GEMM_BIG);
     hipLaunchKernelGGL(tiled_gemm_big_kernel, dim3(mtiles * ntiles, 1, g.groups), dim3(256), 0, s, g, mtiles, ntiles);
     FH_CHECK_LAUNCH();
     return 0;
@@ -298,20 +389,34 @@ int tiled_gemm(const TiledGemm<E>& gin, hipStream_t s) {
     FH_REQUIRE(g.ldx % 8 == 0 && g.x_group % 8 == 0 && g.n_store <= g.n && g.groups >= 1, "tiled_gemm: ldx=%ld group stride=%ld", g.ldx, g.x_group);
     FH_REQUIRE((g.out != nullptr) != (g.out_f32 != nullptr), "tiled_gemm: exactly one output");
     FH_REQUIRE(g.slabs == 1 || (g.groups == 1 && g.out_f32 && !g.bias && !g.nsec && !g.row_scale), "tiled_gemm: slabs are plain fp32 partial sums");
+    bool gated = false;
+    for (int i = 0; i < g.nsec; i++) {
+        gated |= g.sec[i].act == GEMM_ACT_CLAMPED_GLU;
+        FH_REQUIRE(g.sec[i].begin % 32 == 0, "tiled_gemm: section at column %d", g.sec[i].begin);
+    }
+    FH_REQUIRE(!gated || (g.groups == 1 && !g.col_scale), "tiled_gemm: gated sections take one group and no column factors");
+    FH_REQUIRE(!g.col_scale || (g.out && g.ld_col_scale % 8 == 0), "tiled_gemm: column factors with rows of %ld", g.ld_col_scale);
+    const GemmRows& rows = g.rows;
+    if (rows.id) {
+        FH_REQUIRE(g.slabs == 1 && !g.bias && !g.x_blocks && !g.row_scale && !gated && rows.div > 0 && rows.max_blocks > 0 && rows.group && rows.total,
+                   "tiled_gemm: sorted rows take plain sections");
+        FH_REQUIRE(rows.block == 16 || rows.block == 32 || rows.block == 64 || (rows.block == 128 && sizeof(E) == 2), "tiled_gemm: blocks of %d rows", rows.block);
+    }
     const long tiles = (long)cdiv(g.m, 128) * cdiv(g.n, 128) * g.groups;
-    if (sizeof(E) == 2 && g.m > 64 && g.slabs == 1 && tiles >= knobs().tiled_big_min_tiles) return launch_big(g, s);
-    const int mt = g.m <= 16 ? 1 : (g.m <= 32 ? 2 : 4);
-    const int rbs = cdiv(g.m, 16 * mt), ksteps = g.k / 32, zs = g.groups * g.slabs;
+    if (rows.id ? rows.block == 128 : sizeof(E) == 2 && g.m > 64 && g.slabs == 1 && tiles >= knobs().tiled_big_min_tiles) return launch_big(g, s);
+    const int mt = rows.id ? rows.block / 16 : g.m <= 16 ? 1 : (g.m <= 32 ? 2 : 4);
+    const int rbs = rows.id ? rows.max_blocks : cdiv(g.m, 16 * mt), ksteps = g.k / 32, zs = rows.id ? 1 : g.groups * g.slabs;
     // 32 columns per wave, 16 where 32 would leave CUs without a workgroup; K split over the waves until the launch has enough of them
     int J = (long)rbs * (g.n / 32) * zs < 256 ? 1 : 2;
     if (knobs().tiled_j > 0) J = knobs().tiled_j == 1 ? 1 : 2;
+    if (gated) J = 2;
     const long cols = g.n / (16 * J);
     int nw = mt == 1 ? 8 : 4, kw = 1;
     if (knobs().tiled_nw > 0) nw = std::min(8, knobs().tiled_nw);
     while (kw < nw && (long)rbs * cols * zs * kw < 4096 && ksteps >= 8 * kw * g.slabs) kw *= 2;
     if (knobs().tiled_kw > 0) kw = std::min(nw, knobs().tiled_kw);
     const dim3 grid(cdiv(cols, nw / kw), rbs, zs);
-    form_hit(FORM_TILED_GEMM);
+    form_hit(rows.id ? FORM_TILED_GEMM_GROUPED : FORM_TILED_GEMM);
     if (J == 1) return mt == 1 ? launch_small<E, 1, 1>(g, grid, nw, kw, s) : mt == 2 ? launch_small<E, 2, 1>(g, grid, nw, kw, s) : launch_small<E, 4, 1>(g, grid, nw, kw, s);
     return mt == 1 ? launch_small<E, 1, 2>(g, grid, nw, kw, s) : mt == 2 ? launch_small<E, 2, 2>(g, grid, nw, kw, s) : launch_small<E, 4, 2>(g, grid, nw, kw, s);
 }

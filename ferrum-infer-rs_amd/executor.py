@@ -27,18 +27,23 @@ class ModelConfig(C.Structure):
 class LayeredConfig(C.Structure):
     """Whole-model part of a layered model (FerrumHipLayeredConfig)."""
     _fields_ = [("dtype", C.c_int32), ("state_slots", C.c_int32), ("bigram_buckets", C.c_int32), ("residual_mult", C.c_float),
-                ("bigram_mul_prev", C.c_int64), ("bigram_mul_cur", C.c_int64)]
+                ("bigram_mul_prev", C.c_int64), ("bigram_mul_cur", C.c_int64), ("block", C.c_int32), ("token_side_dim", C.c_int32),
+                ("untied_head", C.c_int32), ("_pad", C.c_int32)]
 
 
 class LayerSpec(C.Structure):
     """One layer of a layered model (FerrumHipLayerSpec)."""
     _fields_ = [(n, C.c_int32) for n in ("mixer", "ff", "ff_width", "heads", "dim", "rot_dim", "vdim", "q_rank", "kv_rank", "rot_dims",
                                          "window")] + [("scale", C.c_float), ("rot_base", C.c_double)] + [
-        (n, C.c_int32) for n in ("rnn_width", "rnn_blocks", "conv_taps", "_pad")]
+        (n, C.c_int32) for n in ("rnn_width", "rnn_blocks", "conv_taps", "attn_flags", "kv_source", "experts", "top")] + [
+        ("ff_limit", C.c_float)] + [(n, C.c_double) for n in ("rot_factor", "rot_original", "rot_fast", "rot_slow")]
 
 
 DTYPE = {"bfloat16": 0, "float32": 1}
 MIXER = {"latent_attention": 1, "rglru": 2}
+FF = {"none": 0, "xielu": 1, "clamped_glu": 2, "moe_relu2": 3}
+BLOCK = {"gated_post_norm": 0, "parallel_pre_norm": 1}
+ATTN_NO_HEAD_GATE, ATTN_SINK, WINDOW_NONE = 1, 2, -1
 
 
 class BatchItem(C.Structure):

@@ -454,13 +454,22 @@ typedef struct {
 
 /* ── Layered models (no counterpart in the reference): decoders whose layers are described one by one.  The runner keeps doing for
  *    them what it does for the homogeneous families — paged blocks, admission, batching, sampling, the decode graph — plus one
- *    recurrent-state slot per live sequence.  Architectures: Nerenex. ── */
+ *    recurrent-state slot per live sequence.  Architectures: Nerenex, Safolorn. ── */
 #define FERRUM_HIP_DTYPE_BF16 0
 #define FERRUM_HIP_DTYPE_F32 1
 #define FERRUM_HIP_MIXER_LATENT_ATTENTION 1
 #define FERRUM_HIP_MIXER_RGLRU 2
 #define FERRUM_HIP_FF_NONE 0
-#define FERRUM_HIP_FF_XIELU 1
+#define FERRUM_HIP_FF_XIELU 1          /* down(xIELU(up h)) */
+#define FERRUM_HIP_FF_CLAMPED_GLU 2    /* down(g·σ(1.702 g)·(u + 1)), g = min(gate h, limit), u = clamp(up h, ±limit) */
+#define FERRUM_HIP_FF_MOE_RELU2 3      /* `top` of `experts` down(relu(up h)²), weighted by the softmax over the chosen router logits */
+/* how a layer's sublayers meet the residual stream x */
+#define FERRUM_HIP_BLOCK_GATED_POST_NORM 0     /* one after the other: x += mult · norm(sub(x) · σ(gate x)), norm weights around zero */
+#define FERRUM_HIP_BLOCK_PARALLEL_PRE_NORM 1   /* side by side: x += mixer(g1 · x̂) + ff(g2 · x̂), x̂ = x / rms(x), g1 and g2 single numbers */
+/* latent attention: FerrumHipLayerSpec::attn_flags */
+#define FERRUM_HIP_ATTN_NO_HEAD_GATE 1         /* no sigmoid gate per head on the values' sum */
+#define FERRUM_HIP_ATTN_SINK 2                 /* a learned number per head takes part in the softmax denominator */
+#define FERRUM_HIP_WINDOW_NONE (-1)
 typedef struct {
     int32_t dtype;                /* FERRUM_HIP_DTYPE_*: projections, activations and caches; norms, scores, recurrences and the
                                      residual stream are fp32 either way */
@@ -468,17 +477,29 @@ typedef struct {
     int32_t bigram_buckets;       /* 0 = none; else a hashed (previous token, token) embedding of this many rows + 1 */
     float residual_mult;          /* factor of a sublayer's normed result */
     int64_t bigram_mul_prev, bigram_mul_cur;
+    int32_t block;                /* FERRUM_HIP_BLOCK_* */
+    int32_t token_side_dim;       /* 0 = none; else every layer ends with x += norm(proj(gelu(gate x) · e)), e: its part of a second,
+                                     per-layer token embedding of this many dimensions a layer */
+    int32_t untied_head, _pad;    /* 1 = the vocabulary projection is a tensor of its own ("head") */
 } FerrumHipLayeredConfig;
 typedef struct {
     int32_t mixer;                /* FERRUM_HIP_MIXER_* */
     int32_t ff, ff_width;         /* FERRUM_HIP_FF_*; NONE: the layer is the mixer alone */
     /* latent attention: per head `dim` unrotated + `rot_dim` rotated query / key dimensions (the first rot_dims of the latter turn),
-     * values of vdim; a token sees itself and the window - 1 tokens before it */
+     * values of vdim; a token sees itself and the window - 1 tokens before it (WINDOW_NONE: all of them); q_rank 0: queries straight
+     * from the input, without a latent of their own */
     int32_t heads, dim, rot_dim, vdim, q_rank, kv_rank, rot_dims, window;
     float scale;
     double rot_base;
     /* real-gated linear recurrent unit */
-    int32_t rnn_width, rnn_blocks, conv_taps, _pad;
+    int32_t rnn_width, rnn_blocks, conv_taps;
+    /* latent attention: flags; 0 = caches its own latents, j + 1 = reads layer j's (an earlier layer of equal kv_rank and rotation) */
+    int32_t attn_flags, kv_source;
+    int32_t experts, top;         /* mixture of experts (ff_width: an expert's) */
+    float ff_limit;               /* clamped GLU */
+    /* YaRN: rot_factor 0 = none; pairs that turn more than rot_fast times within rot_original positions keep their frequency, fewer
+     * than rot_slow times: divided by the factor, a ramp between; cosines and sines grow by 0.1 ln(factor) + 1 */
+    double rot_factor, rot_original, rot_fast, rot_slow;
 } FerrumHipLayerSpec;
 
 /* One item of a UnifiedBatch (model_executor.rs:354-386). */

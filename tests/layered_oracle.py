@@ -43,12 +43,29 @@ def embed(tokens, table, bigram=None, buckets=0, mul_prev=0, mul_cur=0):
     return x
 
 
-def rotate_interleaved(x, positions, dims, base):
+def yarn(dims, base, factor, original, fast, slow):
+    """Frequencies of the pairs under YaRN, and the factor of cosines and sines.  A pair that turns more than `fast` times within
+    `original` positions keeps its frequency, one that turns less than `slow` times is slowed by `factor`, with a ramp over the pairs
+    between them."""
+    pair_of = lambda turns: dims * np.log(original / (2.0 * np.pi * turns)) / (2.0 * np.log(base))
+    lo, hi = max(np.floor(pair_of(fast)), 0.0), min(np.ceil(pair_of(slow)), dims - 1.0)
+    f = []
+    for i in range(dims // 2):
+        ramp = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
+        plain = float(base) ** (-2.0 * i / dims)
+        f.append(ramp * plain / factor + (1.0 - ramp) * plain)
+    return f, 0.1 * np.log(factor) + 1.0
+
+
+def rotate_interleaved(x, positions, dims, base, scaling=None):
     """Rotate pairs (2i, 2i + 1) of the first `dims` entries of the last axis; x [tokens, ..., n]."""
     out = x.copy()
+    freq, size = [float(base) ** (-2.0 * i / dims) for i in range(dims // 2)], 1.0
+    if scaling:
+        freq, size = yarn(dims, base, scaling["factor"], scaling["original"], scaling["fast"], scaling["slow"])
     for i in range(dims // 2):
-        a = np.asarray(positions, np.float64) * float(base) ** (-2.0 * i / dims)
-        c, s = np.cos(a), np.sin(a)
+        a = np.asarray(positions, np.float64) * freq[i]
+        c, s = size * np.cos(a), size * np.sin(a)
         shape = (len(c),) + (1,) * (x.ndim - 2)
         c, s = c.reshape(shape), s.reshape(shape)
         u, v = x[..., 2 * i], x[..., 2 * i + 1]
@@ -91,6 +108,35 @@ def latent_attention(h, w, heads, dim, rot_dim, vdim, rot_dims, rot_base, window
     return out.reshape(n, heads * vdim) @ w["o"].T
 
 
+def softmax_with_sink(scores, mask, sink):
+    """The sink takes part in the denominator, once, and carries no value."""
+    s = np.where(mask, scores, -np.inf)
+    m = np.maximum(s.max(axis=-1, keepdims=True), sink)
+    e = np.exp(s - m)
+    return e / (e.sum(axis=-1, keepdims=True) + np.exp(sink - m))
+
+
+def latent_and_shared_key(h, w, rank, rot_dims, rot_base, scaling, eps):
+    """What a token caches: its normed latent, and the rotated key part that all heads use."""
+    kv = h @ w["dkv"].T
+    return unit_rms(kv[:, :rank], eps) * w["dkv.norm"], rotate_interleaved(kv[:, rank:], np.arange(h.shape[0]), rot_dims, rot_base, scaling)
+
+
+def sink_latent_attention(h, w, cached, heads, dim, rot_dim, vdim, rot_dims, rot_base, scaling, scale):
+    """Causal attention over `cached` (another layer's, or this one's) with queries straight from h; w: q, uk, uv, sink, o."""
+    n = h.shape[0]
+    latent, k_rot = cached
+    q = (h @ w["q"].T).reshape(n, heads, dim + rot_dim)
+    q_plain, q_rot = q[..., :dim], rotate_interleaved(q[..., dim:], np.arange(n), rot_dims, rot_base, scaling)
+    k_plain = (latent @ w["uk"].T).reshape(n, heads, dim)
+    value = (latent @ w["uv"].T).reshape(n, heads, vdim)
+    out = np.zeros((n, heads, vdim))
+    for a in range(heads):
+        scores = (q_plain[:, a] @ k_plain[:, a].T + q_rot[:, a] @ k_rot.T) * scale
+        out[:, a] = softmax_with_sink(scores, window_mask(n, n), w["sink"][a]) @ value[:, a]
+    return out.reshape(n, heads * vdim) @ w["o"].T
+
+
 def causal_conv(x, taps, bias):
     """x [n, c], taps [c, k]: the last column weighs the current token."""
     n, c = x.shape
@@ -128,6 +174,35 @@ def dense_ff(h, w):
     return xielu(h @ w["up"].T, w["act"][0], w["act"][1]) @ w["down"].T
 
 
+def clamped_glu(h, w, limit):
+    """w: gate, up, down.  The gate is clamped from above only and turns by a sigmoid of slope 1.702; the linear half is centred at 1."""
+    g, u = np.minimum(h @ w["gate"].T, limit), np.clip(h @ w["up"].T, -limit, limit)
+    return (g * sigmoid(1.702 * g) * (u + 1.0)) @ w["down"].T
+
+
+def route(logits, top):
+    """Experts with the largest logits and the softmax over these logits only."""
+    ids = np.argsort(-logits, axis=-1, kind="stable")[:, :top]
+    z = np.take_along_axis(logits, ids, axis=-1)
+    e = np.exp(z - z.max(axis=-1, keepdims=True))
+    return ids, e / e.sum(axis=-1, keepdims=True)
+
+
+def moe(h, w, top):
+    """w: router, router.b, e<i>.up, e<i>.down; an expert squares the positive part of its up-projection."""
+    ids, weight = route(h @ w["router"].T + w["router.b"], top)
+    out = np.zeros_like(h)
+    for t in range(h.shape[0]):
+        for e, p in zip(ids[t], weight[t]):
+            out[t] += p * (w[f"e{e}.down"] @ np.maximum(w[f"e{e}.up"] @ h[t], 0.0) ** 2)
+    return out
+
+
+def token_side(x, tokens, w, table, eps):
+    """x plus the layer's own view of the token, gated by x; w: gate, proj, norm; table: the layer's columns of the side embedding."""
+    return x + unit_rms((gelu_tanh(x @ w["gate"].T) * table[np.asarray(tokens)]) @ w["proj"].T, eps) * w["norm"]
+
+
 def add_sublayer(x, sub, gate_w, gate_b, norm_w, mult, eps):
     """x + mult · norm(sub · gate): the gate reads x, the norm's weight is stored around zero."""
     gated = sub * sigmoid(x @ gate_w.T + gate_b)
@@ -140,6 +215,33 @@ def group(weights, prefix):
 
 def forward(config, weights, tokens, taps=None):
     """Logits [n, vocab] of one sequence; taps (a list) receives the residual stream after every layer."""
+    return {"Nerenex": forward_nerenex, "Safolorn": forward_safolorn}[config["architecture"]](config, weights, tokens, taps)
+
+
+def forward_safolorn(config, weights, tokens, taps=None):
+    w = {k: np.asarray(v, np.float64) for k, v in weights.items()}
+    eps, side = config["norm"]["eps"], config["token_side"]["dim"]
+    x = embed(tokens, w["embed"])
+    cached = {}
+    for li, layer in enumerate(config["layers"]):
+        p, mx, ff = f"l{li}.", layer["mixer"], layer["mlp"]
+        mw, rot = group(w, p + "mix."), mx["rot"]
+        xhat = unit_rms(x, eps)
+        h = xhat * w[p + "norm1"]
+        if "kv_from" not in mx:
+            cached[li] = latent_and_shared_key(h, mw, mx["kv_rank"], rot["dims"], rot["base"], rot.get("scaling"), eps)
+        y = sink_latent_attention(h, mw, cached[mx.get("kv_from", li)], mx["heads"], mx["dim"], mx["rot_dim"], mx["vdim"], rot["dims"],
+                                  rot["base"], rot.get("scaling"), mx["scale"])
+        if ff:
+            h2, fw = xhat * w[p + "norm2"], group(w, p + "mlp.")
+            y = y + (clamped_glu(h2, fw, ff["limit"]) if ff["kind"] == "dense" else moe(h2, fw, ff["router"]["top"]))
+        x = token_side(x + y, tokens, group(w, p + "side."), w["side.embed"][:, li * side:(li + 1) * side], eps)
+        if taps is not None:
+            taps.append(x.copy())
+    return (unit_rms(x, eps) * w["final.norm"]) @ w["head"].T
+
+
+def forward_nerenex(config, weights, tokens, taps=None):
     w = {k: np.asarray(v, np.float64) for k, v in weights.items()}
     eps, mult = config["norm"]["eps"], config["residual_mult"]
     bg = config["embedding"]["bigram"]
