@@ -396,23 +396,41 @@ def tp_decode_case(pkg, torch, dist, model_name, world, rank, c, PL, steps, warm
     return res
 
 
-# ── layered models: a Nerenex stack with layers of a real model's size beside the closest homogeneous model (sliding-window attention,
-#    post-sublayer norms on an fp32 residual stream, unquantised 16-bit projections) at equal width, heads, feed-forward, window, depth ──
+# ── layered models: a Nerenex or Safolorn stack with layers of a real model's size beside the closest other models at equal width,
+#    heads, feed-forward and depth: the homogeneous model with sliding-window attention, post-sublayer norms on an fp32 residual stream
+#    and unquantised 16-bit projections; a stack of latent attention layers only; a homogeneous model with (INT4) experts ──
 LAYERED_SIZES = {
     "2k": dict(width=2048, heads=16, dim=128, rot_dim=64, vdim=128, q_rank=768, kv_rank=512, window=1024, ff=8192, rnn_width=2048,
-               rnn_blocks=16, taps=4, vocab=32768, layers=12),
+               rnn_blocks=16, taps=4, vocab=32768, layers=12, experts=64, top=8, expert_ff=1024, side=256),
     "4k": dict(width=4096, heads=32, dim=128, rot_dim=64, vdim=128, q_rank=1536, kv_rank=512, window=2048, ff=14336, rnn_width=4096,
-               rnn_blocks=32, taps=4, vocab=65536, layers=12),
+               rnn_blocks=32, taps=4, vocab=65536, layers=12, experts=64, top=8, expert_ff=1792, side=256),
 }
 
 
 def layered_model(pkg, size, side, max_seq_len, blocks, max_seqs, max_tokens):
-    """side: "nerenex" (two recurrent layers, then one attention layer, repeated), "attention" / "recurrent" (one kind only),
-    "dense" (the homogeneous model)."""
+    """side: "nerenex" (two recurrent layers, then one attention layer, repeated), "attention" / "recurrent" (one kind only), "latent"
+    (attention without a window), "safolorn" (dense and expert layers in turn, two of three layers read the latents of the first),
+    "safolorn-dense" / "safolorn-moe" (one kind only, every layer caches its own), "dense" / "moe" (homogeneous models)."""
     z = LAYERED_SIZES[size]
     common = dict(num_layers=z["layers"], hidden=z["width"], vocab=z["vocab"], max_seq_len=max_seq_len, kv_num_blocks=blocks, max_seqs=max_seqs,
                   max_tokens=max_tokens, rms_eps=1e-6)
-    if side == "dense":
+    if side == "moe":
+        m = pkg.HipModel(num_heads=z["heads"], num_kv_heads=z["heads"] // 4, head_dim=128, intermediate=z["ff"], has_qk_norm=1, activation=0,
+                         num_experts=z["experts"], top_k=z["top"], expert_inter=z["expert_ff"], norm_topk_prob=1, rope_theta=1e6, **common)
+        m.init_synthetic(7)
+    elif side.startswith("safolorn"):
+        specs = []
+        for i in range(z["layers"]):
+            moe = side == "safolorn-moe" or (side == "safolorn" and i % 2 == 1)
+            ff = dict(ff=3, ff_width=z["expert_ff"], experts=z["experts"], top=z["top"]) if moe else dict(ff=2, ff_width=z["ff"], ff_limit=7.0)
+            specs.append(pkg.LayerSpec(mixer=1, heads=z["heads"], dim=z["dim"], rot_dim=z["rot_dim"], vdim=z["vdim"], kv_rank=z["kv_rank"],
+                                       rot_dims=z["rot_dim"], window=-1, scale=(z["dim"] + z["rot_dim"]) ** -0.5, rot_base=1e6, attn_flags=3,
+                                       kv_source=i // 3 * 3 + 1 if side == "safolorn" and i % 3 else 0, rot_factor=4.0, rot_original=2048.0,
+                                       rot_fast=32.0, rot_slow=1.0, **ff))
+        lc = pkg.LayeredConfig(dtype=0, state_slots=max_seqs, residual_mult=1.0, block=1, token_side_dim=z["side"], untied_head=1)
+        m = pkg.HipModel(layered=(lc, specs), **common)
+        m.init_synthetic(7)
+    elif side == "dense":
         prev = os.environ.get("FERRUM_HIP_SYNTH_DENSE")
         os.environ["FERRUM_HIP_SYNTH_DENSE"] = "1"
         try:
@@ -425,10 +443,10 @@ def layered_model(pkg, size, side, max_seq_len, blocks, max_seqs, max_tokens):
     else:
         specs = []
         for i in range(z["layers"]):
-            attn = side == "attention" or (side == "nerenex" and i % 3 == 2)
+            attn = side in ("attention", "latent") or (side == "nerenex" and i % 3 == 2)
             if attn:
                 specs.append(pkg.LayerSpec(mixer=1, ff=1, ff_width=z["ff"], heads=z["heads"], dim=z["dim"], rot_dim=z["rot_dim"], vdim=z["vdim"],
-                                           q_rank=z["q_rank"], kv_rank=z["kv_rank"], rot_dims=z["rot_dim"], window=z["window"],
+                                           q_rank=z["q_rank"], kv_rank=z["kv_rank"], rot_dims=z["rot_dim"], window=-1 if side == "latent" else z["window"],
                                            scale=(z["dim"] + z["rot_dim"]) ** -0.5, rot_base=1e6))
             else:
                 specs.append(pkg.LayerSpec(mixer=2, ff=1, ff_width=z["ff"], rnn_width=z["rnn_width"], rnn_blocks=z["rnn_blocks"],
@@ -474,8 +492,8 @@ def layered_bench(pkg, torch, args):
 
 def main():
     ap = argparse.ArgumentParser()
-    ap.add_argument("--layered", default="", choices=[""] + sorted(LAYERED_SIZES), help="extra workload: a Nerenex stack of this size beside the closest homogeneous model")
-    ap.add_argument("--layered-sides", default="nerenex,dense", help="with --layered: which of nerenex, attention, recurrent, dense")
+    ap.add_argument("--layered", default="", choices=[""] + sorted(LAYERED_SIZES), help="extra workload: layered models of this size beside the closest other ones")
+    ap.add_argument("--layered-sides", default="nerenex,dense", help="with --layered: which of nerenex, attention, latent, recurrent, safolorn, safolorn-dense, safolorn-moe, dense, moe")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=64)
     ap.add_argument("--warmup", type=int, default=8)

@@ -1,4 +1,4 @@
-"""Small random Nerenex models for the tests: configuration, weights (bfloat16-representable), checkpoint directories."""
+"""Small random Nerenex and Safolorn models for the tests: configuration, weights (bfloat16-representable), checkpoint directories."""
 import json
 import os
 import struct
@@ -27,7 +27,30 @@ def config(width, vocab, layers, eps=1e-5, mult=0.8, buckets=97, mul_prev=31, mu
             "embedding": {"bigram": {"buckets": buckets, "mul_prev": mul_prev, "mul_cur": mul_cur}}}
 
 
-CONFIGS = {
+def sink_attention(heads, dim, rot_dim, vdim, kv_rank, base=10000.0, yarn=None, scale=None, kv_from=None, mlp=None):
+    """yarn: (factor, original, fast, slow)"""
+    rot = {"base": base, "dims": rot_dim}
+    if yarn:
+        rot["scaling"] = dict(zip(("factor", "original", "fast", "slow"), yarn))
+    mixer = {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "kv_rank": kv_rank, "rot": rot, "scale": scale or (dim + rot_dim) ** -0.5}
+    if kv_from is not None:
+        mixer["kv_from"] = kv_from
+    return {"type": "latent_attention", "mlp": mlp, "mixer": mixer}
+
+
+def glu(ff, limit):
+    return {"kind": "dense", "ff": ff, "limit": limit}
+
+
+def experts(n, top, ff):
+    return {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": n, "top": top}}
+
+
+def safolorn(width, vocab, side, layers, eps=1e-5):
+    return {"architecture": "Safolorn", "width": width, "vocab": vocab, "norm": {"eps": eps}, "token_side": {"dim": side}, "layers": layers}
+
+
+NERENEX = {
     # nothing is a multiple of 32; value size, query size and ranks all differ; attention without, recurrence with a feed-forward
     "odd": config(100, 131, [attention(3, 20, 6, 36, 44, 52, 21, base=500.0), recurrent(66, 3, 3, ff=75), attention(5, 9, 10, 12, 31, 70, 50, ff=41)],
                   eps=1e-3, mult=0.45),
@@ -37,9 +60,86 @@ CONFIGS = {
     "deep": config(320, 203, [attention(16, 128, 64, 128, 160, 512, 90, base=1e6), attention(7, 96, 40, 120, 72, 300, 33, ff=130)], eps=1e-6, mult=0.9),
     "tiny": config(40, 61, [recurrent(24, 2, 1, ff=33), attention(2, 8, 4, 8, 16, 24, 7, ff=50), attention(1, 12, 2, 20, 8, 9, 1)], buckets=11),
 }
+SHORT, LONG = (3.0, 40, 6.0, 1.0), (2.5, 96, 9.0, 0.5)
+SAFOLORN = {
+    # nothing is a multiple of 32; two caches, each read by a later layer; a layer without feed-forward; all experts chosen
+    "sinks": safolorn(100, 131, 10, [sink_attention(3, 20, 6, 36, 52, 500.0, SHORT, mlp=glu(75, 0.7)), sink_attention(5, 9, 10, 12, 70, mlp=experts(7, 3, 41)),
+                                     sink_attention(4, 12, 6, 20, 52, 500.0, SHORT, kv_from=0), sink_attention(2, 9, 10, 8, 70, kv_from=1, mlp=experts(5, 5, 33))],
+                      eps=1e-3),
+    # more heads than a row tile, ranks and heads of several padded sizes, one cache read by layers of other head counts
+    "shared": safolorn(288, 260, 40, [sink_attention(20, 64, 32, 48, 256, 1e5, LONG, mlp=glu(416, 1.5)), sink_attention(17, 40, 32, 64, 256, 1e5, LONG, kv_from=0, mlp=experts(20, 2, 72)),
+                                      sink_attention(3, 128, 64, 128, 512, 1e6, SHORT, mlp=experts(12, 1, 160)), sink_attention(6, 32, 32, 96, 256, 1e5, LONG, kv_from=0, mlp=glu(130, 0.3))]),
+    "one": safolorn(40, 61, 1, [sink_attention(1, 5, 2, 3, 7, mlp=experts(1, 1, 9)), sink_attention(2, 8, 4, 8, 24, yarn=(1.0, 64, 4.0, 2.0), mlp=glu(1, 2.0))], eps=0.1),
+}
+CONFIGS = {**NERENEX, **SAFOLORN}
+CLASSES = 4
 
 
-def weights(cfg, seed):
+def weights(cfg, seed, **kw):
+    return {"Nerenex": nerenex_weights, "Safolorn": safolorn_weights}[cfg["architecture"]](cfg, seed, **kw)
+
+
+def safolorn_weights(cfg, seed, clear_routes=True):
+    """clear_routes: the first CLASSES coordinates of the stream hold the token's class and nothing else, and the router mostly reads
+    them, with an order of the experts per class and wide gaps: no rounding changes a choice, and every expert is chosen by some class
+    (experts permitting)."""
+    rng = np.random.default_rng(seed)
+    D, V, S, n = cfg["width"], cfg["vocab"], cfg["token_side"]["dim"], len(cfg["layers"])
+    w = {}
+
+    def mat(name, *shape, std=None):
+        w[name] = bf16(rng.standard_normal(shape) * (std or shape[-1] ** -0.5))
+
+    def num(name):
+        w[name] = bf16(rng.uniform(0.6, 1.5, ())).reshape(())
+
+    mat("embed", V, D, std=1.0)
+    mat("side.embed", V, n * S, std=1.0)
+    mat("head", V, D)
+    num("final.norm")
+    for i, layer in enumerate(cfg["layers"]):
+        p, m, ff = f"l{i}.", layer["mixer"], layer["mlp"]
+        x, H = p + "mix.", m["heads"]
+        num(p + "norm1")
+        mat(x + "q", H * (m["dim"] + m["rot_dim"]), D, std=1.6 * D ** -0.5)
+        if "kv_from" not in m:
+            mat(x + "dkv", m["kv_rank"] + m["rot_dim"], D)
+            w[x + "dkv.norm"] = bf16(1.0 + 0.2 * rng.standard_normal(m["kv_rank"]))
+        mat(x + "uk", H * m["dim"], m["kv_rank"], std=1.6 * m["kv_rank"] ** -0.5)
+        mat(x + "uv", H * m["vdim"], m["kv_rank"])
+        w[x + "sink"] = bf16(2.0 + 1.5 * rng.standard_normal(H))
+        mat(x + "o", D, H * m["vdim"], std=2.0 * (H * m["vdim"]) ** -0.5)
+        outs = [x + "o", p + "side.proj"]
+        if ff:
+            num(p + "norm2")
+        if ff and ff["kind"] == "dense":
+            mat(p + "mlp.gate", ff["ff"], D, std=1.5 * D ** -0.5)
+            mat(p + "mlp.up", ff["ff"], D)
+            mat(p + "mlp.down", D, ff["ff"])
+            outs.append(p + "mlp.down")
+        elif ff:
+            E, F = ff["router"]["experts"], ff["expert"]["ff"]
+            for e in range(E):
+                mat(p + f"mlp.e{e}.up", F, D)
+                mat(p + f"mlp.e{e}.down", D, F)
+                outs.append(p + f"mlp.e{e}.down")
+            mat(p + "mlp.router", E, D, std=(0.05 if clear_routes else 1.5) * D ** -0.5)
+            w[p + "mlp.router.b"] = bf16((0.02 if clear_routes else 0.5) * rng.standard_normal(E))
+            if clear_routes:
+                order = np.stack([np.roll(rng.permutation(E), c) for c in range(CLASSES)])
+                w[p + "mlp.router"][:, :CLASSES] = bf16(0.25 * order.T)
+        mat(p + "side.gate", S, D)
+        mat(p + "side.proj", D, S)
+        w[p + "side.norm"] = bf16(0.4 + 0.3 * rng.standard_normal(D))
+        if clear_routes:
+            for name in outs:
+                w[name][:CLASSES] = 0.0
+    if clear_routes:
+        w["embed"][:, :CLASSES] = 6.0 * np.eye(CLASSES)[rng.integers(0, CLASSES, V)]
+    return w
+
+
+def nerenex_weights(cfg, seed):
     rng = np.random.default_rng(seed)
     D, V = cfg["width"], cfg["vocab"]
     w = {}
@@ -99,6 +199,7 @@ def write_checkpoint(path, cfg, w):
         json.dump(cfg, f)
     head, at, blobs = {}, 0, []
     for name, a in w.items():
+        assert np.array_equal(bf16(a).reshape(np.shape(a)), np.asarray(a, np.float32)), f"{name} is not bfloat16"
         b = (np.ascontiguousarray(a, np.float32).view(np.uint32) >> 16).astype("<u2").tobytes()
         head[name] = {"dtype": "BF16", "shape": list(a.shape), "data_offsets": [at, at + len(b)]}
         at += len(b)

@@ -20,7 +20,7 @@ def _write(tmp_path, cfg):
     return G.write_checkpoint(tmp_path, cfg, {"embed": np.zeros((2, 2), np.float32)})
 
 
-@pytest.mark.parametrize("name", list(G.CONFIGS))
+@pytest.mark.parametrize("name", list(G.NERENEX))
 def test_config_becomes_layer_specs(pkg, tmp_path, name):
     cfg = G.CONFIGS[name]
     ck = pkg.Checkpoint(_write(tmp_path, cfg))
@@ -107,3 +107,80 @@ def test_oracle_activation_is_continuous_with_slope_one_half():
 def test_oracle_window_and_pairs():
     assert L.window_mask(5, 2).sum(axis=1).tolist() == [1, 2, 2, 2, 2]
     assert L.bigram_rows([4, 4, 9], 7, 3, 2).tolist() == [7, (4 * 3 + 4 * 2) % 7, (4 * 3 + 9 * 2) % 7]
+
+
+# ── Safolorn ──
+@pytest.mark.parametrize("name", list(G.SAFOLORN))
+def test_safolorn_config_becomes_layer_specs(pkg, tmp_path, name):
+    cfg = G.SAFOLORN[name]
+    ck = pkg.Checkpoint(_write(tmp_path, cfg))
+    d, arch, tied = ck.model_config(555)
+    assert arch == "Safolorn" and not tied and (d["hidden"], d["vocab"], d["num_layers"], d["max_seq_len"]) == (cfg["width"], cfg["vocab"], len(cfg["layers"]), 555)
+    assert abs(d["rms_eps"] - cfg["norm"]["eps"]) < 1e-8
+    lc, specs = ck.layered_config()
+    assert (lc.block, lc.token_side_dim, lc.untied_head, lc.bigram_buckets) == (1, cfg["token_side"]["dim"], 1, 0)
+    for s, layer in zip(specs, cfg["layers"]):
+        m, ff = layer["mixer"], layer["mlp"]
+        y = m["rot"].get("scaling")
+        assert (s.mixer, s.heads, s.dim, s.rot_dim, s.vdim, s.q_rank, s.kv_rank, s.rot_dims, s.window, s.attn_flags) == (
+            1, m["heads"], m["dim"], m["rot_dim"], m["vdim"], 0, m["kv_rank"], m["rot"]["dims"], -1, 3)
+        assert s.kv_source == m.get("kv_from", -1) + 1 and s.rot_base == m["rot"]["base"] and abs(s.scale - m["scale"]) < 1e-6
+        assert (s.rot_factor, s.rot_original, s.rot_fast, s.rot_slow) == ((y["factor"], y["original"], y["fast"], y["slow"]) if y else (0, 0, 0, 0))
+        if not ff:
+            assert (s.ff, s.ff_width) == (0, 0)
+        elif ff["kind"] == "dense":
+            assert (s.ff, s.ff_width) == (2, ff["ff"]) and abs(s.ff_limit - ff["limit"]) < 1e-6
+        else:
+            assert (s.ff, s.ff_width, s.experts, s.top) == (3, ff["expert"]["ff"], ff["router"]["experts"], ff["router"]["top"])
+
+
+@pytest.mark.parametrize("edit,what", [(lambda c: c["layers"][0]["mixer"].pop("kv_rank"), "kv_rank"), (lambda c: c["layers"][0]["mlp"].pop("limit"), "limit"),
+                                       (lambda c: c["layers"][1]["mlp"]["router"].pop("top"), "top"), (lambda c: c["layers"][1]["mlp"].pop("expert"), "expert"),
+                                       (lambda c: c["layers"][0]["mixer"]["rot"]["scaling"].pop("slow"), "slow"), (lambda c: c.pop("token_side"), "token_side"),
+                                       (lambda c: c["layers"][0]["mixer"].update(kv_from=0), "kv_from"), (lambda c: c["layers"][2]["mixer"].update(kv_from=3), "kv_from"),
+                                       (lambda c: c["layers"][2]["mixer"].pop("scale"), "scale")])
+def test_incomplete_safolorn_config_is_refused_by_name(pkg, tmp_path, edit, what):
+    cfg = json.loads(json.dumps(G.SAFOLORN["sinks"]))
+    edit(cfg)
+    ck = pkg.Checkpoint(_write(tmp_path, cfg))
+    with pytest.raises(RuntimeError, match=what):
+        ck.model_config()
+        ck.layered_config()
+
+
+@pytest.mark.parametrize("edit", [lambda c: c["layers"][0].update(type="rglru"), lambda c: c["layers"][1]["mlp"].update(kind="sparse")])
+def test_unknown_safolorn_mechanisms_are_unsupported(pkg, tmp_path, edit):
+    from ferrum_infer_rs_amd.backend import Unsupported
+    cfg = json.loads(json.dumps(G.SAFOLORN["sinks"]))
+    edit(cfg)
+    with pytest.raises(Unsupported):
+        pkg.Checkpoint(_write(tmp_path, cfg)).layered_config()
+
+
+def test_impossible_parallel_blocks_are_refused_before_any_device_work(pkg):
+    ok = dict(hidden=64, vocab=32, max_seq_len=64, kv_num_blocks=4, max_seqs=1, max_tokens=16)
+    at = dict(mixer=1, heads=2, dim=8, rot_dim=4, vdim=8, kv_rank=8, rot_dims=4, window=-1, rot_base=1e4, attn_flags=3)
+    lc = pkg.LayeredConfig(block=1, token_side_dim=8, untied_head=1, residual_mult=1.0)
+    S = pkg.LayerSpec
+    for specs in ([S(**at, ff=1, ff_width=8)], [S(**at, ff=2, ff_width=0)], [S(**at, ff=3, ff_width=8, experts=4, top=5)], [S(**at, ff=3, ff_width=8, experts=600, top=2)],
+                  [S(mixer=2, rnn_width=32, rnn_blocks=4, conv_taps=2)], [S(**at, kv_source=1)], [S(**at), S(**at, kv_source=1), S(**at, kv_source=2)],
+                  [S(**at), S(**{**at, "kv_rank": 16}, kv_source=1)], [S(**at, rot_factor=2.0)]):
+        with pytest.raises(RuntimeError):
+            pkg.HipModel(layered=(lc, specs), **{**ok, "num_layers": len(specs)})
+    for bad in (pkg.LayeredConfig(block=2), pkg.LayeredConfig(block=0, token_side_dim=8)):
+        with pytest.raises(RuntimeError):
+            pkg.HipModel(layered=(bad, [S(**at)]), **ok)
+
+
+def test_oracle_sink_and_routing():
+    s = np.array([[[1.0, 2.0], [0.5, 0.5]]])
+    p = L.softmax_with_sink(s[0], L.window_mask(2, 2), 0.7)
+    assert p[0].tolist() == pytest.approx([np.exp(1.0) / (np.exp(1.0) + np.exp(0.7)), 0.0]) and p[1].sum() == pytest.approx(2 * np.exp(0.5) / (2 * np.exp(0.5) + np.exp(0.7)))
+    ids, w = L.route(np.array([[0.1, 3.0, 2.0, 3.0]]), 3)
+    assert ids[0].tolist() == [1, 3, 2] and w.sum() == pytest.approx(1.0) and w[0, 2] == pytest.approx(np.exp(-1.0) / (2 + np.exp(-1.0)))
+
+
+def test_oracle_rotation_scaling_keeps_fast_pairs_and_slows_slow_ones():
+    f, size = L.yarn(16, 100.0, 8.0, 64, 8.0, 0.5)
+    plain = [100.0 ** (-2.0 * i / 16) for i in range(8)]
+    assert f[0] == plain[0] and f[-1] == pytest.approx(plain[-1] / 8.0) and all(p / 8.0 <= g <= p for g, p in zip(f, plain)) and size == pytest.approx(1 + 0.1 * np.log(8.0))

@@ -1,4 +1,4 @@
-"""Layered models (Nerenex) on the device against the plain oracle of tests/layered_oracle.py: every mechanism alone, prompts,
+"""Layered models (Nerenex; for whole models Safolorn too, see test_safolorn_gpu.py for its mechanisms) on the device against the plain oracle of tests/layered_oracle.py: every mechanism alone, prompts,
 portions and decoding, unequal batches, reuse of pages and slots, window edges with a key that stands out, and greedy generation
 through the engine loop.  Models are small and random; none of their numbers come from a checkpoint."""
 import json
@@ -169,10 +169,11 @@ def test_prompt_portions_and_decoding_agree_with_the_oracle(pkg, cases, name, dt
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", ["wide", "shared"])
 @pytest.mark.parametrize("n", [1, 2, 3, 4, 5, 6])
-def test_first_tokens(pkg, cases, n, dtype):
+def test_first_tokens(pkg, cases, n, name, dtype):
     """Sequences shorter than the convolution, in a slot and blocks that another sequence has just left."""
-    cfg, w, path = cases("wide")
+    cfg, w, path = cases(name)
     m = load(pkg, path, dtype, seqs=1, blocks=10, tokens=160)
     m.forward_rows([(1, toks(cfg, 150, 2), 0)], [])
     m.release(1)
@@ -184,7 +185,7 @@ def test_first_tokens(pkg, cases, n, dtype):
 
 @pytest.mark.parametrize("tiles", [0, 2])
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("name", ["odd", "wide", "deep"])
+@pytest.mark.parametrize("name", ["odd", "wide", "deep", "sinks", "shared"])
 def test_unequal_batch_against_each_request_alone(pkg, cases, knobs, name, dtype, tiles):
     """Portions of some requests beside single decoded tokens of others, members coming and going; rows against the oracle, and against
     the same rows computed alone to rounding."""
@@ -245,9 +246,10 @@ def test_pages_and_slots_are_used_again(pkg, cases, dtype):
     assert m.prefix_cache_acquire(501, t) == 0
 
 
-def test_prefix_cache_of_an_attention_only_model(pkg, cases):
+@pytest.mark.parametrize("name", ["deep", "shared"])
+def test_prefix_cache_of_an_attention_only_model(pkg, cases, name):
     """Without recurrent layers a cached prefix is spliced in, including the previous token of the pair embedding."""
-    cfg, w, path = cases("deep")
+    cfg, w, path = cases(name)
     m = load(pkg, path, "float32", tokens=160, seqs=2)
     t = toks(cfg, 70, 19)
     feed(m, 1, t[:48], [48])
@@ -347,7 +349,7 @@ def near_greedy(cfg, w, prompt, out, slack):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("name", ["odd", "wide"])
+@pytest.mark.parametrize("name", ["odd", "wide", "sinks", "shared"])
 def test_long_decoding_through_the_graph(pkg, cases, forms, name, dtype):
     """Three sequences of different lengths decode 150 tokens past their windows in one captured step (several replays with eager
     forwards between them); the same ids as eager single steps, and the oracle's choices up to rounding."""
@@ -383,8 +385,9 @@ def test_long_decoding_through_the_graph(pkg, cases, forms, name, dtype):
         assert np.array_equal(np.stack(again), gen)
 
 
-def test_masked_and_penalised_greedy_choice(pkg, cases):
-    cfg, w, path = cases("tiny")
+@pytest.mark.parametrize("name", ["tiny", "one"])
+def test_masked_and_penalised_greedy_choice(pkg, cases, name):
+    cfg, w, path = cases(name)
     m = load(pkg, path, "float32")
     t = toks(cfg, 20, 4)
     lg = L.forward(cfg, w, t)[-1]
@@ -397,10 +400,11 @@ def test_masked_and_penalised_greedy_choice(pkg, cases):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-def test_generation_through_the_engine_loop(cases, dtype):
+@pytest.mark.parametrize("name", ["odd", "sinks"])
+def test_generation_through_the_engine_loop(cases, name, dtype):
     """The command line: admission bounded by two state slots and a small pool, prompts cut by a 24-token budget beside decoding
     sequences, graph decoding in between; greedy ids against the oracle."""
-    cfg, w, path = cases("odd")
+    cfg, w, path = cases(name)
     prompts = [toks(cfg, n, 300 + n) for n in (30, 3, 57, 12, 1, 41)]
     text = ";".join(",".join(str(int(x)) for x in p) for p in prompts)
     cmd = [os.path.join(BIN, "ferrum_hip_serve"), "--model", path, "--dtype", dtype, "--prompt-ids", text, "--concurrency", "4", "--state-slots", "2",
@@ -409,16 +413,17 @@ def test_generation_through_the_engine_loop(cases, dtype):
     assert p.returncode == 0, p.stderr[-2000:]
     lines = p.stdout.strip().splitlines()
     head = json.loads(lines[0])
-    assert head["model"] == "Nerenex" and head["output_tokens"] == 6 * 20 and head["kv_blocks_free_at_exit"] == head["kv_blocks_total"] == 9
+    assert head["model"] == cfg["architecture"] and head["output_tokens"] == 6 * 20 and head["kv_blocks_free_at_exit"] == head["kv_blocks_total"] == 9
     out = {int(l.split(":")[0].split()[1]): np.array(l.split(":")[1].split(), np.int64) for l in lines[1:]}
     for i, pr in enumerate(prompts):
         assert near_greedy(cfg, w, pr, out[i + 1], 2e-4 if dtype == "float32" else 0.25), i
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-def test_trace_replay(cases, tmp_path, dtype):
+@pytest.mark.parametrize("name", ["wide", "shared"])
+def test_trace_replay(cases, tmp_path, name, dtype):
     """bin/trace_run: portions beside decoded tokens, requests that pause, end and make room; logits against the oracle."""
-    cfg, w, path = cases("wide")
+    cfg, w, path = cases(name)
     seqs = {f"q{i}": toks(cfg, n, 400 + n) for i, n in enumerate((150, 20, 90, 64, 33))}
     want = {k: L.forward(cfg, w, t) for k, t in seqs.items()}
     plan = [{"q0": 100, "q1": 2}, {"q1": 17, "q2": 30}, {"q0": 1, "q1": 1, "q2": 2, "q3": 64}, {"q0": 49, "q2": 58, "q4": 31}, {"q4": 2}]
@@ -443,9 +448,10 @@ def test_trace_replay(cases, tmp_path, dtype):
     assert p.wait(timeout=30) == 0
 
 
-def test_few_row_and_tile_projections_agree(pkg, cases, knobs, forms):
+@pytest.mark.parametrize("name", ["wide", "shared", "sinks"])
+def test_few_row_and_tile_projections_agree(pkg, cases, knobs, forms, name):
     """The 128 × 128 tile kernel and the few-row kernel on the same portions."""
-    cfg, w, path = cases("wide")
+    cfg, w, path = cases(name)
     t = toks(cfg, 200, 12)
     want = L.forward(cfg, w, t)
     for tiles, name in ((1, "tiled_gemm_big"), (10 ** 6, "tiled_gemm")):
