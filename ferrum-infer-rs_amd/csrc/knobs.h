@@ -56,6 +56,8 @@ struct Knobs {
     int lds_min_groups = 8;
     // layered models (tiled_gemm.hip, latent_attention.hip, rglru.hip)
     int tiled_big_min_tiles = 64;     // 16-bit projections of > 64 rows take the 128 × 128 tile kernel from this many tiles
+    int tiled_wide_min_tiles = 128;   // … and its 256 × 256 form from this many of those tiles
+    int moe_rows_block = 0;           // > 0: forced rows per block of the sorted expert rows
     int tiled_nw = 0, tiled_kw = 0, tiled_j = 0;      // > 0: forced waves per workgroup, K parts, 16-column tiles per wave of the few-row kernel
     int latent_tiles = 0;             // 1 / 2: forced 16-row tiles per workgroup of the latent attention
     int latent_splits = 0;            // > 0: forced KV split count of the latent attention
@@ -121,6 +123,7 @@ enum Form : int {
     FORM_ROUTE_GEMM_TOPK,       // prefill router: logits (MFMA) + softmax + top-k in one launch (moe_route_gemm_topk_kernel)
     FORM_TILED_GEMM,            // layered models: projection with K split over the waves of a workgroup
     FORM_TILED_GEMM_BIG,        // … 128 × 128 tiles, operands copied to LDS as fragments
+    FORM_TILED_GEMM_256,        // … 256 × 256 tiles
     FORM_TILED_GEMM_GROUPED,    // … rows sorted by expert
     FORM_TILED_GEMM_GROUPED_BIG,
     FORM_LATENT_ATTN_PLAIN,     // latent attention, one workgroup per (token, head), any size and number format

@@ -40,7 +40,7 @@ uint16_t bf16_bits(float f) {
 void store(bf16* dst, float f) { const uint16_t h = bf16_bits(f); memcpy(dst, &h, 2); }
 void store(float* dst, float f) { *dst = f; }
 
-constexpr int MOE_MAX_BLOCK = 128;
+constexpr int MOE_MAX_BLOCK = 256;
 
 struct HostTensor { std::vector<float> data; std::vector<int64_t> shape; };
 
@@ -369,8 +369,9 @@ private:
     }
     // rows per block of the sorted list: a large block shares an expert's weights between more rows, a small one pads less
     static int moe_block(int pairs, int experts) {
-        const int mean = pairs / experts;
-        if (sizeof(E) == 2 && mean >= 48) return 128;
+        const int mean = pairs / experts, forced = knobs().moe_rows_block;
+        if (forced > 0 && (sizeof(E) == 2 || forced <= 64)) return forced;
+        if (sizeof(E) == 2 && mean >= 48) return mean >= 384 ? 256 : 128;
         return mean >= 32 ? 64 : mean >= 12 ? 32 : 16;
     }
 

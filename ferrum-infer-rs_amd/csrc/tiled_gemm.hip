@@ -195,172 +195,180 @@ __global__ __launch_bounds__(512) void tiled_gemm_kernel(TiledGemm<E> p, int kw)
     }
 }
 
-// Prompts, 16-bit: 128 × 128 output tile, 64 of K per stage, two stages.  A fragment (16 rows × 32 of K, or 16 columns × 32 of K) is
-// one 1-KiB load straight into LDS in lane order, read back as one conflict-free ds_read_b128; 2 × 2 waves hold 64 × 64 each.
-__global__ __launch_bounds__(256, 2) void tiled_gemm_big_kernel(TiledGemm<bf16> p, int mtiles, int ntiles) {
-    __shared__ __attribute__((aligned(16))) bf16 lds[2][32 * 512];      // per stage: 16 A fragments, 16 B fragments
+// Prompts, 16-bit: WM × WN waves hold MI × NJ tiles of 16 × 16 each, 64 of K per stage, two stages.  A fragment (16 rows × 32 of K, or 16
+// columns × 32 of K) is one 1-KiB load straight into LDS in lane order, read back as one conflict-free ds_read_b128.
+__device__ const bf16 zero_fragment[512] = {};
+template <int WM, int WN, int MI, int NJ>
+struct BigTile {
+    static constexpr int WAVES = WM * WN, RT = WM * MI, CT = WN * NJ, ROWS = 16 * RT, COLS = 16 * CT, FRAGS = 2 * (RT + CT);
+    static constexpr size_t LDS = (size_t)2 * FRAGS * 1024;
+    static_assert(RT % WAVES == 0 && CT % WAVES == 0 && MI % 2 == 0 && NJ == 4, "every wave copies whole tiles");
+    static_assert(LDS >= (size_t)WAVES * 32 * 68 * 4, "the epilogue's rows fit the stages");
+};
+template <int WM, int WN, int MI, int NJ>
+__global__ __launch_bounds__(64 * WM * WN, 2) void tiled_gemm_big_kernel(TiledGemm<bf16> p, int mtiles, int ntiles) {
+    typedef BigTile<WM, WN, MI, NJ> T;
+    extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
+    bf16* lds = reinterpret_cast<bf16*>(smem);                          // per stage: A fragments, then B fragments
+    constexpr int STAGE = T::FRAGS * 512, AT = T::RT / T::WAVES, BT = T::CT / T::WAVES;
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
     const int a = lane >> 4, b = lane & 15;
     // workgroups go round-robin over 8 XCDs: give each XCD a contiguous run of tiles, and walk 8 row tiles per column tile
-    if (p.rows.id) mtiles = *p.rows.total >> 7;
+    if (p.rows.id) mtiles = *p.rows.total / T::ROWS;
     const int total = mtiles * ntiles, l = blockIdx.x;
     if (l >= total) return;
     const int q8 = total / 8, r8 = total % 8, xcd = l % 8;
     const int id = (xcd < r8 ? xcd * (q8 + 1) : r8 * (q8 + 1) + (xcd - r8) * q8) + l / 8;
     const int band = id / (8 * ntiles), rows_in = min(8, mtiles - band * 8), in = id - band * 8 * ntiles;
-    const int m0 = (band * 8 + in % rows_in) * 128, n0 = (in / rows_in) * 128;
-    const int ksteps = p.k >> 5, ntl = p.n >> 4, g = p.rows.id ? p.rows.group[m0 >> 7] : blockIdx.z;
-    const int wm = wave >> 1, wn = wave & 1;
-    // this wave's 8 fragments of a stage: A row tiles 2·wave, 2·wave + 1 and B column tiles 2·wave, 2·wave + 1, two k-steps each
-    const bf16 *ap[2], *bp[2];
+    const int mt = band * 8 + in % rows_in, m0 = mt * T::ROWS, n0 = (in / rows_in) * T::COLS;
+    const int ksteps = p.k >> 5, ntl = p.n >> 4, g = p.rows.id ? p.rows.group[mt] : blockIdx.z;
+    const int wm = wave / WN, wn = wave % WN;
+    // this wave's fragments of a stage: AT row tiles and BT column tiles, two k-steps each
+    const bf16 *ap[AT], *bp[BT];
 #pragma unroll
-    for (int i = 0; i < 2; i++) {
-        const int t = (n0 >> 4) + 2 * wave + i;
-        ap[i] = gemm_row(p, (m0 >> 4) + 2 * wave + i, g, a, b);
+    for (int i = 0; i < AT; i++) ap[i] = gemm_row(p, (m0 >> 4) + AT * wave + i, g, a, b);
+#pragma unroll
+    for (int i = 0; i < BT; i++) {
+        const int t = (n0 >> 4) + BT * wave + i;
         bp[i] = p.w + ((long)g * ntl + (t < ntl ? t : ntl - 1)) * ksteps * 512 + lane * 8;
     }
     const int xs = gemm_row_step(p);
+#define BIG_COPY(src, dst) __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(src), (__attribute__((address_space(3))) void*)(dst), 16, 0, 0)
     auto issue = [&](int st, int ks) {
 #pragma unroll
         for (int h = 0; h < 2; h++) {
-            const int kk = ks + h < ksteps ? ks + h : ksteps - 1;
+            const int kk = ks + h < ksteps ? ks + h : ksteps - 1;         // (past the end of an odd count: rows of zeros)
 #pragma unroll
-            for (int i = 0; i < 2; i++) {
-                bf16* da = &lds[st][((2 * wave + i) * 2 + h) * 512];
-                bf16* db = &lds[st][(16 + (2 * wave + i) * 2 + h) * 512];
-                __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(ap[i] + (long)kk * xs),
-                                                 (__attribute__((address_space(3))) void*)da, 16, 0, 0);
-                __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(bp[i] + (long)kk * 512),
-                                                 (__attribute__((address_space(3))) void*)db, 16, 0, 0);
-            }
+            for (int i = 0; i < AT; i++) BIG_COPY(ks + h < ksteps ? ap[i] + (long)kk * xs : zero_fragment + lane * 8, lds + st * STAGE + ((AT * wave + i) * 2 + h) * 512);
+#pragma unroll
+            for (int i = 0; i < BT; i++) BIG_COPY(bp[i] + (long)kk * 512, lds + st * STAGE + ((T::RT + BT * wave + i) * 2 + h) * 512);
         }
     };
-    floatx4 acc[4][4];
+#undef BIG_COPY
+    floatx4 acc[MI][NJ];
 #pragma unroll
-    for (int i = 0; i < 4; i++)
+    for (int i = 0; i < MI; i++)
 #pragma unroll
-        for (int j = 0; j < 4; j++) acc[i][j] = (floatx4){0.f, 0.f, 0.f, 0.f};
+        for (int j = 0; j < NJ; j++) acc[i][j] = (floatx4){0.f, 0.f, 0.f, 0.f};
     issue(0, 0);
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     __syncthreads();
+    auto multiply = [&](const bf16* la, const bf16* lb, int h) {
+        bf16x8 af[MI], bf[NJ];
+#pragma unroll
+        for (int j = 0; j < NJ; j++) bf[j] = *reinterpret_cast<const bf16x8*>(lb + (j * 2 + h) * 512);
+#pragma unroll
+        for (int i = 0; i < MI; i++) af[i] = *reinterpret_cast<const bf16x8*>(la + (i * 2 + h) * 512);
+#pragma unroll
+        for (int i = 0; i < MI; i++)
+#pragma unroll
+            for (int j = 0; j < NJ; j++) acc[i][j] = Frag<bf16>::mma(af[i], bf[j], acc[i][j]);
+    };
     int st = 0;
     for (int ks = 0; ks < ksteps; ks += 2, st ^= 1) {
         if (ks + 2 < ksteps) issue(st ^ 1, ks + 2);
+        const bf16 *la = lds + st * STAGE + wm * MI * 1024 + lane * 8, *lb = lds + st * STAGE + (T::RT + wn * NJ) * 1024 + lane * 8;
+        multiply(la, lb, 0);
+        multiply(la, lb, 1);
+        // operands a few MFMAs ahead of their use
+        constexpr int AHEAD = NJ + 2, LEFT = 2 * (MI + NJ) - AHEAD, PER = 2 * MI * NJ / (LEFT + 2);
+        __builtin_amdgcn_sched_group_barrier(0x100, AHEAD, 0);
 #pragma unroll
-        for (int h = 0; h < 2; h++) {
-            if (ks + h >= ksteps) break;
-            bf16x8 af[4], bf[4];
-#pragma unroll
-            for (int i = 0; i < 4; i++) {
-                af[i] = *reinterpret_cast<const bf16x8*>(&lds[st][((wm * 4 + i) * 2 + h) * 512 + lane * 8]);
-                bf[i] = *reinterpret_cast<const bf16x8*>(&lds[st][(16 + (wn * 4 + i) * 2 + h) * 512 + lane * 8]);
-            }
-#pragma unroll
-            for (int i = 0; i < 4; i++)
-#pragma unroll
-                for (int j = 0; j < 4; j++) acc[i][j] = Frag<bf16>::mma(af[i], bf[j], acc[i][j]);
+        for (int i = 0; i < LEFT; i++) {
+            __builtin_amdgcn_sched_group_barrier(0x008, PER, 0);
+            __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
         }
+        __builtin_amdgcn_sched_group_barrier(0x008, 2 * MI * NJ - LEFT * PER, 0);
         asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
         __syncthreads();
     }
-    // epilogue: activations on the accumulators, then through LDS (the stages are free; a wave's 64 × 64 tile is its own) so that rows
-    // leave in 16-byte pieces, 128 or 256 contiguous bytes per row.  A gated pair of tiles leaves 16 columns in the first one's place.
-    GemmSection sec[2];
-    int col0[2];
+    // epilogue: 32 rows of a wave's accumulators at a time through LDS (the stages are free, the rows its own, LDS operations of a wave
+    // complete in order), then a lane finishes 8 columns of a row: bias, activation and factors, and rows leave in 16-byte pieces.  In a
+    // gated section the lanes of the up tiles have nothing to do, those of the gate tiles read both.
+    float* lf = reinterpret_cast<float*>(smem) + wave * 32 * 68;
+    const int cl = (lane & 7) * 8, col = n0 + wn * 64 + cl;
+    const GemmSection sec = gemm_section(p, min(col, p.n - 1));
+    const bool gated = sec.act == GEMM_ACT_CLAMPED_GLU, vec = p.n_store % 8 == 0 && p.ldo % 8 == 0 && p.out_group % 8 == 0;
+    const bool active = gated ? col < p.n && !(col & 16) : col < p.n_store;
+    const int oc = gated ? gemm_gated_col(sec, col) : col;
+    float bias[8], bias_up[8];
 #pragma unroll
-    for (int c = 0; c < 2; c++) {
-        col0[c] = n0 + wn * 64 + c * 32;
-        sec[c] = gemm_section(p, min(col0[c], p.n - 1));
-    }
-    auto value = [&](int c, int j, int i, int r, float& v) {               // false: the up tile of a pair
-        const int jj = 2 * c + j;
-        if (sec[c].act == GEMM_ACT_CLAMPED_GLU) {
-            if (j) return false;
-            v = gemm_gated(p, sec[c], min(col0[c], p.n - 32) + b, acc[i][2 * c][r], acc[i][2 * c + 1][r]);
-            return true;
-        }
-        v = acc[i][jj][r] * sec[c].mul;
-        if (p.bias) v += p.bias[(long)g * p.n + min(col0[c] + 16 * j + b, p.n - 1)];
-        v = gemm_act<bf16>(sec[c], v);
-        return true;
-    };
-    if (p.n_store % 8 == 0 && p.ldo % 8 == 0 && p.out_group % 8 == 0) {
-        bf16* lo = &lds[0][0] + wave * 64 * 72;                    // rows of 72: 36 KiB for the four waves
-        float* lf = reinterpret_cast<float*>(&lds[0][0]) + wave * 32 * 68;      // fp32 outputs: 32 rows of 68 at a time
-        // column of the tile → column of the output, −1: not stored
-        auto out_col = [&](int col) {
-            const int c = col >> 5;
-            if (c ? sec[1].act == GEMM_ACT_CLAMPED_GLU : sec[0].act == GEMM_ACT_CLAMPED_GLU)
-                return col & 16 || (c ? col0[1] : col0[0]) >= p.n ? -1 : gemm_gated_col(c ? sec[1] : sec[0], c ? col0[1] : col0[0]) + (col & 15);
-            return n0 + wn * 64 + col < p.n_store ? n0 + wn * 64 + col : -1;
-        };
-#pragma unroll
-        for (int half = 0; half < 2; half++) {
-#pragma unroll
-            for (int j = 0; j < 4; j++)
-#pragma unroll
-                for (int i = 2 * half; i < 2 * half + 2; i++)
-#pragma unroll
-                    for (int r = 0; r < 4; r++) {
-                        float v;
-                        if (!value(j >> 1, j & 1, i, r, v)) continue;
-                        if (p.out_f32) lf[((i & 1) * 16 + 4 * a + r) * 68 + j * 16 + b] = v;
-                        else lo[(i * 16 + 4 * a + r) * 72 + j * 16 + b] = (bf16)v;
-                    }
-            if (p.out_f32) {                                       // (wave-private: LDS operations of a wave complete in order)
-#pragma unroll
-                for (int q = 0; q < 8; q++) {
-                    const int row = q * 4 + (lane >> 4), gr = gemm_out_row(p, m0 + wm * 64 + half * 32 + row), gc = out_col((lane & 15) * 4);
-                    if (gr >= 0 && gc >= 0) {
-                        floatx4 v = *reinterpret_cast<const floatx4*>(lf + row * 68 + (lane & 15) * 4);
-                        if (p.row_scale) v *= (float)p.row_scale[gr * p.ld_scale + g];
-                        *reinterpret_cast<floatx4*>(p.out_f32 + gr * p.ldo + (p.rows.id ? 0 : g * p.out_group) + gc) = v;
-                    }
-                }
-            }
-        }
-        if (p.out_f32) return;
-#pragma unroll
-        for (int q = 0; q < 8; q++) {
-            const int row = q * 8 + (lane >> 3), gr = gemm_out_row(p, m0 + wm * 64 + row), gc = out_col((lane & 7) * 8);
-            if (gr >= 0 && gc >= 0) {
-                bf16x8 v = *reinterpret_cast<const bf16x8*>(lo + row * 72 + (lane & 7) * 8);
-                if (p.row_scale) {
-                    const float f = (float)p.row_scale[gr * p.ld_scale + g];
-#pragma unroll
-                    for (int e = 0; e < 8; e++) v[e] = (bf16)((float)v[e] * f);
-                }
-                if (p.col_scale) {
-                    const bf16x8 f = *reinterpret_cast<const bf16x8*>(p.col_scale + p.col_scale_row[gr] * p.ld_col_scale + gc);
-#pragma unroll
-                    for (int e = 0; e < 8; e++) v[e] = (bf16)((float)v[e] * (float)f[e]);
-                }
-                *reinterpret_cast<bf16x8*>(p.out + gr * p.ldo + (p.rows.id ? 0 : g * p.out_group) + gc) = v;
-            }
-        }
-        return;
+    for (int e = 0; e < 8; e++) {
+        bias[e] = p.bias && active ? p.bias[(long)g * p.n + col + e] : 0.f;
+        bias_up[e] = p.bias && active && gated ? p.bias[(long)g * p.n + col + 16 + e] : 0.f;
     }
 #pragma unroll
-    for (int j = 0; j < 4; j++) {
-        if (col0[j >> 1] >= p.n) break;
+    for (int ch = 0; ch < MI / 2; ch++) {
 #pragma unroll
-        for (int i = 0; i < 4; i++)
+        for (int i = 0; i < 2; i++)
 #pragma unroll
-            for (int r = 0; r < 4; r++) {
-                float v;
-                const int row = gemm_out_row(p, m0 + wm * 64 + i * 16 + 4 * a + r), col = col0[j >> 1] + (j & 1) * 16 + b;
-                if (row >= 0 && col < p.n_store && value(j >> 1, j & 1, i, r, v))
-                    gemm_store(p, g, row, sec[j >> 1].act == GEMM_ACT_CLAMPED_GLU ? gemm_gated_col(sec[j >> 1], col) : col, v);
+            for (int j = 0; j < NJ; j++)
+#pragma unroll
+                for (int r = 0; r < 4; r++) lf[(i * 16 + 4 * a + r) * 68 + j * 16 + b] = acc[2 * ch + i][j][r];
+        const int row0 = m0 + (wm * MI + 2 * ch) * 16;
+#pragma unroll 1
+        for (int q = 0; q < 4; q++) {
+            const int row = q * 8 + (lane >> 3), gr = gemm_out_row(p, row0 + row);
+            if (gr < 0 || !active) continue;
+            float v[8];
+#pragma unroll
+            for (int e = 0; e < 8; e++) v[e] = lf[row * 68 + cl + e] * sec.mul + bias[e];
+            if (gated) {
+#pragma unroll
+                for (int e = 0; e < 8; e++) v[e] = clamped_glu_f32<bf16>(v[e], lf[row * 68 + cl + 16 + e] * sec.mul + bias_up[e], sec.p, sec.q);
+            } else if (sec.act != GEMM_ACT_NONE) {
+#pragma unroll
+                for (int e = 0; e < 8; e++) v[e] = gemm_act<bf16>(sec, v[e]);
             }
+            if (!vec) {
+                for (int e = 0; e < 8; e++)
+                    if (gated || col + e < p.n_store) gemm_store(p, g, gr, oc + e, v[e]);
+                continue;
+            }
+            if (p.row_scale) {
+                const float f = (float)p.row_scale[gr * p.ld_scale + g];
+#pragma unroll
+                for (int e = 0; e < 8; e++) v[e] *= f;
+            }
+            if (p.col_scale) {
+                const bf16x8 f = *reinterpret_cast<const bf16x8*>(p.col_scale + p.col_scale_row[gr] * p.ld_col_scale + oc);
+#pragma unroll
+                for (int e = 0; e < 8; e++) v[e] *= (float)f[e];
+            }
+            const long o = gr * p.ldo + (p.rows.id ? 0 : g * p.out_group) + oc;
+            if (p.out_f32) {
+                *reinterpret_cast<floatx4*>(p.out_f32 + o) = (floatx4){v[0], v[1], v[2], v[3]};
+                *reinterpret_cast<floatx4*>(p.out_f32 + o + 4) = (floatx4){v[4], v[5], v[6], v[7]};
+            } else {
+                bf16x8 y;
+#pragma unroll
+                for (int e = 0; e < 8; e++) y[e] = (bf16)v[e];
+                *reinterpret_cast<bf16x8*>(p.out + o) = y;
+            }
+        }
     }
 }
 
+template <int WM, int WN, int MI, int NJ>
 static int launch_big(const TiledGemm<bf16>& g, hipStream_t s) {
-    const int mtiles = g.rows.id ? g.rows.max_blocks : cdiv(g.m, 128), ntiles = cdiv(g.n, 128);
+    typedef BigTile<WM, WN, MI, NJ> T;
+    static bool attr = false;
+    if (!attr) {
+        FH_CHECK_HIP(hipFuncSetAttribute((const void*)tiled_gemm_big_kernel<WM, WN, MI, NJ>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)T::LDS));
+        attr = true;
+    }
+    const int mtiles = g.rows.id ? g.rows.max_blocks : cdiv(g.m, T::ROWS), ntiles = cdiv(g.n, T::COLS);
     form_hit(g.rows.id ? FORM_TILED_GEMM_GROUPED_BIG : FORM_TILED_GEMM_BIG);
-    hipLaunchKernelGGL(tiled_gemm_big_kernel, dim3(mtiles * ntiles, 1, g.groups), dim3(256), 0, s, g, mtiles, ntiles);
+    if (T::ROWS == 256) form_hit(FORM_TILED_GEMM_256);
+    hipLaunchKernelGGL((tiled_gemm_big_kernel<WM, WN, MI, NJ>), dim3(mtiles * ntiles, 1, g.groups), dim3(64 * T::WAVES), T::LDS, s, g, mtiles, ntiles);
     FH_CHECK_LAUNCH();
     return 0;
+}
+static int launch_big(const TiledGemm<bf16>& g, hipStream_t s) {
+    // one 256 × 256 tile per CU, or two of 128 × 128: the large one halves the bytes per product, as long as there are enough of them
+    const long tiles = (long)cdiv(g.m, 256) * cdiv(g.n, 256) * g.groups;
+    const bool wide = g.rows.id ? g.rows.block == 256 : tiles >= knobs().tiled_wide_min_tiles;
+    return wide ? launch_big<2, 4, 8, 4>(g, s) : launch_big<2, 2, 4, 4>(g, s);
 }
 static int launch_big(const TiledGemm<float>&, hipStream_t) { return 2; }      // (never taken: 16-bit only)
 
@@ -400,10 +408,10 @@ int tiled_gemm(const TiledGemm<E>& gin, hipStream_t s) {
     if (rows.id) {
         FH_REQUIRE(g.slabs == 1 && !g.bias && !g.x_blocks && !g.row_scale && !gated && rows.div > 0 && rows.max_blocks > 0 && rows.group && rows.total,
                    "tiled_gemm: sorted rows take plain sections");
-        FH_REQUIRE(rows.block == 16 || rows.block == 32 || rows.block == 64 || (rows.block == 128 && sizeof(E) == 2), "tiled_gemm: blocks of %d rows", rows.block);
+        FH_REQUIRE(rows.block == 16 || rows.block == 32 || rows.block == 64 || ((rows.block == 128 || rows.block == 256) && sizeof(E) == 2), "tiled_gemm: blocks of %d rows", rows.block);
     }
     const long tiles = (long)cdiv(g.m, 128) * cdiv(g.n, 128) * g.groups;
-    if (rows.id ? rows.block == 128 : sizeof(E) == 2 && g.m > 64 && g.slabs == 1 && tiles >= knobs().tiled_big_min_tiles) return launch_big(g, s);
+    if (rows.id ? rows.block >= 128 : sizeof(E) == 2 && g.m > 64 && g.slabs == 1 && tiles >= knobs().tiled_big_min_tiles) return launch_big(g, s);
     const int mt = rows.id ? rows.block / 16 : g.m <= 16 ? 1 : (g.m <= 32 ? 2 : 4);
     const int rbs = rows.id ? rows.max_blocks : cdiv(g.m, 16 * mt), ksteps = g.k / 32, zs = rows.id ? 1 : g.groups * g.slabs;
     // 32 columns per wave, 16 where 32 would leave CUs without a workgroup; K split over the waves until the launch has enough of them
