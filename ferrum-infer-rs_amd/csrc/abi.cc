@@ -49,7 +49,8 @@ void reload_knobs() {
     k.chain_attn_splits = env_int("FERRUM_HIP_CHAIN_ATTN_SPLITS", 0);
     k.route_gemm_topk = env_int("FERRUM_HIP_ROUTE_GEMM_TOPK", 1);
     k.tiled_big_min_tiles = env_int("FERRUM_HIP_TILED_BIG_MIN_TILES", 64);
-    k.tiled_wide_min_tiles = env_int("FERRUM_HIP_TILED_WIDE_MIN_TILES", 128);
+    k.tiled_wide_min_tiles = env_int("FERRUM_HIP_TILED_WIDE_MIN_TILES", 192);
+    k.tiled_half_max_tiles = env_int("FERRUM_HIP_TILED_HALF_MAX_TILES", 128);
     k.moe_rows_block = env_int("FERRUM_HIP_MOE_ROWS_BLOCK", 0);
     k.tiled_nw = env_int("FERRUM_HIP_TILED_NW", 0);
     k.tiled_kw = env_int("FERRUM_HIP_TILED_KW", 0);
@@ -95,7 +96,7 @@ static const char* const g_form_names[FORM_COUNT] = {
     "route_fused", "route_gemm", "dense_slab_chain", "graph_capture", "graph_replay", "tp_allreduce_rccl",
     "tp_allreduce_loopback", "tp_allreduce_oneshot", "f16_dense_linear", "w4_fused_tail", "attn_resident", "w4_big", "w4_ldsk", "gather_columns",
     "perm_producer", "moe_expert_major_pair", "decode_chain", "moe_deferred_merge", "dense_chain", "tp_allreduce_norm_fused", "moe_block_major_pair", "chain_attn_kv_splits", "chain_qkv_wide", "route_gemm_topk",
-    "tiled_gemm", "tiled_gemm_big", "tiled_gemm_256", "tiled_gemm_grouped", "tiled_gemm_grouped_big", "latent_attn_plain", "latent_attn", "latent_attn_pair", "latent_attn_split", "latent_attn_expanded", "rglru_step", "rglru_scan"};
+    "tiled_gemm", "tiled_gemm_big", "tiled_gemm_256", "tiled_gemm_grouped", "tiled_gemm_grouped_big", "moe_route_sort", "latent_attn_plain", "latent_attn", "latent_attn_pair", "latent_attn_split", "latent_attn_expanded", "rglru_step", "rglru_scan"};
 const char* form_name(int f) { return f >= 0 && f < FORM_COUNT ? g_form_names[f] : nullptr; }
 }  // namespace fh
 

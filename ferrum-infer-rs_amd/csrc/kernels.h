@@ -187,6 +187,10 @@ int moe_route_gemm_topk_f16(const __half* x, const __half* router_f16t, int32_t*
                             int num_experts, int hidden, int top_k, int norm_topk_prob, hipStream_t s);
 int moe_route_topk_softmax_f32(const float* logits, int32_t* expert_ids, float* expert_weights, int tokens,
                                int num_experts, int top_k, int norm_topk_prob, hipStream_t s);
+// both of the above in one workgroup, for decode batches (≤ 1024 pairs)
+bool moe_route_sort_supports(int tokens, int num_experts, int top_k);
+int moe_route_sort_f32(const float* logits, int32_t* expert_ids, float* expert_weights, int32_t* sorted_token_ids, int32_t* block_ids, int32_t* total_post_pad,
+                       int tokens, int num_experts, int top_k, int norm_topk_prob, int block_size, hipStream_t s);
 int moe_align_block_size(const int32_t* expert_ids, int32_t* sorted_token_ids, int32_t* block_ids,
                          int32_t* total_post_pad, int batch_x_topk, int num_experts, int block_size,
                          int sorted_max, hipStream_t s);

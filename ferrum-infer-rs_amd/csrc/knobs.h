@@ -56,7 +56,8 @@ struct Knobs {
     int lds_min_groups = 8;
     // layered models (tiled_gemm.hip, latent_attention.hip, rglru.hip)
     int tiled_big_min_tiles = 64;     // 16-bit projections of > 64 rows take the 128 × 128 tile kernel from this many tiles
-    int tiled_wide_min_tiles = 128;   // … and its 256 × 256 form from this many of those tiles
+    int tiled_wide_min_tiles = 192;   // … and its 256 × 256 form from this many of those tiles
+    int tiled_half_max_tiles = 128;   // … its 64 × 128 form up to this many tiles of 128 × 128
     int moe_rows_block = 0;           // > 0: forced rows per block of the sorted expert rows
     int tiled_nw = 0, tiled_kw = 0, tiled_j = 0;      // > 0: forced waves per workgroup, K parts, 16-column tiles per wave of the few-row kernel
     int latent_tiles = 0;             // 1 / 2: forced 16-row tiles per workgroup of the latent attention
@@ -126,6 +127,7 @@ enum Form : int {
     FORM_TILED_GEMM_256,        // … 256 × 256 tiles
     FORM_TILED_GEMM_GROUPED,    // … rows sorted by expert
     FORM_TILED_GEMM_GROUPED_BIG,
+    FORM_MOE_ROUTE_SORT,        // … router's top-k and the sorted rows in one workgroup
     FORM_LATENT_ATTN_PLAIN,     // latent attention, one workgroup per (token, head), any size and number format
     FORM_LATENT_ATTN,           // … on the matrix cores, against the cached latents (keys and values never expanded)
     FORM_LATENT_ATTN_PAIR,      // … two 16-row tiles per workgroup

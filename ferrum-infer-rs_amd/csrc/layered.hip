@@ -352,12 +352,16 @@ private:
         TiledGemm<E> z = linear_f32(L.router, xb_, Dp_, T, router_logits_, E_);
         z.n_store = E_; z.nsec = 1; z.sec[0] = {0, GEMM_ACT_NONE, 0, 0, L.g2};
         RUN(tiled_gemm(z, s));
-        RUN(moe_route_topk_softmax_f32(router_logits_, expert_ids_, expert_weights_, T, E_, L.s.top, 1, s));
         GemmRows rows;
         rows.block = moe_block(pairs, E_);
         rows.max_blocks = std::min(pairs, pairs / rows.block + std::min(E_, pairs));
         rows.id = sorted_; rows.group = sorted_expert_; rows.total = sorted_total_;
-        RUN(moe_align_block_size(expert_ids_, sorted_, sorted_expert_, sorted_total_, pairs, E_, rows.block, rows.max_blocks * rows.block, s));
+        if (moe_route_sort_supports(T, E_, L.s.top)) {
+            RUN(moe_route_sort_f32(router_logits_, expert_ids_, expert_weights_, sorted_, sorted_expert_, sorted_total_, T, E_, L.s.top, 1, rows.block, s));
+        } else {
+            RUN(moe_route_topk_softmax_f32(router_logits_, expert_ids_, expert_weights_, T, E_, L.s.top, 1, s));
+            RUN(moe_align_block_size(expert_ids_, sorted_, sorted_expert_, sorted_total_, pairs, E_, rows.block, rows.max_blocks * rows.block, s));
+        }
         TiledGemm<E> u = linear(L.up, xb_, Dp_, pairs, expert_h_, L.up.n);
         u.groups = 1; u.rows = rows; u.rows.div = L.s.top;
         u.nsec = 1; u.sec[0] = {0, GEMM_ACT_RELU2, 0, 0, L.g2};

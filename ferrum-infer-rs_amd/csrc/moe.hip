@@ -8,17 +8,15 @@
 // are in ascending pair id (the CUDA lane's atomicAdd order is unspecified; ours is not).
 #include "common.h"
 #include "kernels.h"
+#include "knobs.h"
 
 namespace fh {
 
-// One wave per token.  E ≤ 512.  f32 softmax, k argmax-mask passes, ties → lowest index.
+// Router of one token on one wave (E ≤ 512, lane l looks at experts l, l + 64, …): f32 softmax, k argmax-mask passes, ties → lowest index.
+// Lane k ends up with the k-th choice.
 template <typename T>
-__global__ __launch_bounds__(64) void moe_route_kernel(const T* __restrict__ logits, int32_t* __restrict__ ids,
-                                                       float* __restrict__ weights, int num_experts, int top_k,
-                                                       int norm_topk_prob) {
+__device__ __forceinline__ void route_token(const T* __restrict__ row, int lane, int num_experts, int top_k, int norm_topk_prob, int& id, float& weight) {
     constexpr int PER = 8;   // experts per lane (E ≤ 512)
-    const int tok = blockIdx.x, lane = threadIdx.x;
-    const T* row = logits + (long)tok * num_experts;
     float v[PER];
     float mx = -INFINITY;
 #pragma unroll
@@ -43,36 +41,114 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const T* __restrict__ log
         v[i] = e < num_experts ? v[i] * inv_sum : -INFINITY;
     }
     float sel_sum = 0.f;
-    float my_w = 0.f;   // lane k keeps the k-th selected weight
-    int my_id = 0;
+    weight = 0.f;
+    id = 0;
     for (int k = 0; k < top_k; k++) {
         float best = -INFINITY;
-        int best_idx = 0x7fffffff;
+        int mine = 1 << 20;
 #pragma unroll
-        for (int i = 0; i < PER; i++) {
-            int e = lane + i * 64;
-            if (v[i] > best) { best = v[i]; best_idx = e; }   // ascending e within a lane → first max
-        }
-#pragma unroll
-        for (int off = 32; off > 0; off >>= 1) {
-            float ob = __shfl_xor(best, off, 64);
-            int oi = __shfl_xor(best_idx, off, 64);
-            if (ob > best || (ob == best && oi < best_idx)) { best = ob; best_idx = oi; }
-        }
-        if (best_idx == 0x7fffffff) best_idx = 0;   // all -inf (router.rs keeps best_idx = 0)
-        sel_sum += best;
-        if (lane == (k & 63)) { my_w = best; my_id = best_idx; }
+        for (int i = 0; i < PER; i++)
+            if (v[i] > best) { best = v[i]; mine = lane + i * 64; }       // ascending e within a lane → first max
+        const float top = wave_reduce_max(best);
+        // lowest index among the lanes that hold the maximum (indices are exact in f32); all −inf: index 0 (router.rs keeps best_idx = 0)
+        int best_idx = (int)-wave_reduce_max(best == top && best > -INFINITY ? -(float)mine : -(float)(1 << 20));
+        if (best_idx == 1 << 20) best_idx = 0;
+        sel_sum += top;
+        if (lane == k) { weight = top; id = best_idx; }
 #pragma unroll
         for (int i = 0; i < PER; i++)
             if (lane + i * 64 == best_idx) v[i] = -INFINITY;
-        if (top_k > 64 && (k & 63) == 63) {}  // top_k ≤ 64 enforced on host
     }
+    if (norm_topk_prob) weight = sel_sum > 0.f ? weight * (1.0f / sel_sum) : 1.0f / (float)top_k;
+}
+
+template <typename T>
+__global__ __launch_bounds__(64) void moe_route_kernel(const T* __restrict__ logits, int32_t* __restrict__ ids,
+                                                       float* __restrict__ weights, int num_experts, int top_k,
+                                                       int norm_topk_prob) {
+    const int tok = blockIdx.x, lane = threadIdx.x;
+    int id;
+    float w;
+    route_token(logits + (long)tok * num_experts, lane, num_experts, top_k, norm_topk_prob, id, w);
     if (lane < top_k) {
-        float w = my_w;
-        if (norm_topk_prob) w = sel_sum > 0.f ? w * (1.0f / sel_sum) : 1.0f / (float)top_k;
-        ids[(long)tok * top_k + lane] = my_id;
+        ids[(long)tok * top_k + lane] = id;
         weights[(long)tok * top_k + lane] = w;
     }
+}
+
+// Decode batches: top-k and the list of pairs sorted by expert in ONE workgroup (≤ 1024 pairs; outputs as moe_route_kernel and
+// moe_align_kernel<0> write them, except that nothing is written past the last block).  A wave routes its tokens, then every thread owns
+// a pair: its rank among the pairs of its expert is the count in earlier waves (histograms in LDS) plus the count in earlier lanes.
+constexpr int ROUTE_SORT_PAIRS = 1024;
+__global__ __launch_bounds__(1024) void moe_route_sort_kernel(const float* __restrict__ logits, int32_t* __restrict__ ids, float* __restrict__ weights,
+                                                              int32_t* __restrict__ sorted, int32_t* __restrict__ block_ids, int32_t* __restrict__ total,
+                                                              int tokens, int num_experts, int top_k, int norm_topk_prob, int block_size) {
+    __shared__ int16_t lds_id[ROUTE_SORT_PAIRS];
+    __shared__ int16_t hist[16][512];
+    __shared__ int32_t offset[512];
+    const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, n_pairs = tokens * top_k, nw = (n_pairs + 63) >> 6;
+    for (int t = wave; t < tokens; t += 16) {
+        int id;
+        float w;
+        route_token(logits + (long)t * num_experts, lane, num_experts, top_k, norm_topk_prob, id, w);
+        if (lane < top_k) {
+            lds_id[t * top_k + lane] = (int16_t)id;
+            ids[t * top_k + lane] = id;
+            weights[t * top_k + lane] = w;
+        }
+    }
+    for (int i = lane; i < num_experts; i += 64) hist[wave][i] = 0;
+    __syncthreads();
+    const int e = tid < n_pairs ? lds_id[tid] : -1;
+    int rank = 0, same = 0;
+    if (wave < nw)
+#pragma unroll
+        for (int l = 0; l < 64; l++) {
+            const int other = __builtin_amdgcn_readlane(e, l);
+            same += other == e;
+            rank += other == e && l < lane;
+        }
+    if (e >= 0 && rank == 0) hist[wave][e] = (int16_t)same;
+    __syncthreads();
+    // counts of earlier waves per expert, and the padded start of every expert's rows
+    int count = 0;
+    if (tid < num_experts)
+        for (int w = 0; w < nw; w++) { const int c = hist[w][tid]; hist[w][tid] = (int16_t)count; count += c; }
+    if (tid < 512) offset[tid] = tid < num_experts ? (count + block_size - 1) / block_size * block_size : 0;
+    __syncthreads();
+    if (wave == 0) {
+        int run[8], sum = 0;
+#pragma unroll
+        for (int i = 0; i < 8; i++) { run[i] = sum; sum += offset[lane * 8 + i]; }
+        int incl = sum;
+#pragma unroll
+        for (int off = 1; off < 64; off <<= 1) {
+            const int v = __shfl_up(incl, off, 64);
+            if (lane >= off) incl += v;
+        }
+#pragma unroll
+        for (int i = 0; i < 8; i++) offset[lane * 8 + i] = incl - sum + run[i];
+        if (lane == 63) total[0] = incl;
+    }
+    __syncthreads();
+    if (e >= 0) sorted[offset[e] + hist[wave][e] + rank] = tid;
+    if (tid < num_experts) {
+        const int o = offset[tid], padded = (count + block_size - 1) / block_size * block_size;
+        for (int i = count; i < padded; i++) sorted[o + i] = n_pairs;
+        for (int i = 0; i < padded; i += block_size) block_ids[(o + i) / block_size] = tid;
+    }
+}
+bool moe_route_sort_supports(int tokens, int num_experts, int top_k) { return (long)tokens * top_k <= ROUTE_SORT_PAIRS && num_experts <= 512; }
+int moe_route_sort_f32(const float* logits, int32_t* expert_ids, float* expert_weights, int32_t* sorted_token_ids, int32_t* block_ids, int32_t* total_post_pad,
+                       int tokens, int num_experts, int top_k, int norm_topk_prob, int block_size, hipStream_t s) {
+    if (tokens <= 0) return 0;
+    FH_REQUIRE(moe_route_sort_supports(tokens, num_experts, top_k) && num_experts > 0 && top_k > 0 && top_k <= num_experts && top_k <= 64 && block_size > 0,
+               "moe route + sort: %d tokens, %d of %d experts, blocks of %d", tokens, top_k, num_experts, block_size);
+    form_hit(FORM_MOE_ROUTE_SORT);
+    hipLaunchKernelGGL(moe_route_sort_kernel, dim3(1), dim3(1024), 0, s, logits, expert_ids, expert_weights, sorted_token_ids, block_ids, total_post_pad,
+                       tokens, num_experts, top_k, norm_topk_prob, block_size);
+    FH_CHECK_LAUNCH();
+    return 0;
 }
 
 int moe_route_topk_softmax_f16(const __half* logits, int32_t* expert_ids, float* expert_weights, int tokens,

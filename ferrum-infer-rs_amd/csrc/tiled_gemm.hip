@@ -195,19 +195,19 @@ __global__ __launch_bounds__(512) void tiled_gemm_kernel(TiledGemm<E> p, int kw)
     }
 }
 
-// Prompts, 16-bit: WM × WN waves hold MI × NJ tiles of 16 × 16 each, 64 of K per stage, two stages.  A fragment (16 rows × 32 of K, or 16
+// Prompts, 16-bit: WM × WN waves hold MI × NJ tiles of 16 × 16 each, 64 of K per stage, a ring of S stages.  A fragment (16 rows × 32 of K, or 16
 // columns × 32 of K) is one 1-KiB load straight into LDS in lane order, read back as one conflict-free ds_read_b128.
 __device__ const bf16 zero_fragment[512] = {};
-template <int WM, int WN, int MI, int NJ>
+template <int WM, int WN, int MI, int NJ, int S>
 struct BigTile {
     static constexpr int WAVES = WM * WN, RT = WM * MI, CT = WN * NJ, ROWS = 16 * RT, COLS = 16 * CT, FRAGS = 2 * (RT + CT);
-    static constexpr size_t LDS = (size_t)2 * FRAGS * 1024;
+    static constexpr size_t LDS = (size_t)S * FRAGS * 1024;
     static_assert(RT % WAVES == 0 && CT % WAVES == 0 && MI % 2 == 0 && NJ == 4, "every wave copies whole tiles");
     static_assert(LDS >= (size_t)WAVES * 32 * 68 * 4, "the epilogue's rows fit the stages");
 };
-template <int WM, int WN, int MI, int NJ>
+template <int WM, int WN, int MI, int NJ, int S>
 __global__ __launch_bounds__(64 * WM * WN, 2) void tiled_gemm_big_kernel(TiledGemm<bf16> p, int mtiles, int ntiles) {
-    typedef BigTile<WM, WN, MI, NJ> T;
+    typedef BigTile<WM, WN, MI, NJ, S> T;
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
     bf16* lds = reinterpret_cast<bf16*>(smem);                          // per stage: A fragments, then B fragments
     constexpr int STAGE = T::FRAGS * 512, AT = T::RT / T::WAVES, BT = T::CT / T::WAVES;
@@ -250,9 +250,9 @@ __global__ __launch_bounds__(64 * WM * WN, 2) void tiled_gemm_big_kernel(TiledGe
     for (int i = 0; i < MI; i++)
 #pragma unroll
         for (int j = 0; j < NJ; j++) acc[i][j] = (floatx4){0.f, 0.f, 0.f, 0.f};
-    issue(0, 0);
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < S - 1; i++)
+        if (2 * i < ksteps) issue(i, 2 * i);
     auto multiply = [&](const bf16* la, const bf16* lb, int h) {
         bf16x8 af[MI], bf[NJ];
 #pragma unroll
@@ -265,8 +265,12 @@ __global__ __launch_bounds__(64 * WM * WN, 2) void tiled_gemm_big_kernel(TiledGe
             for (int j = 0; j < NJ; j++) acc[i][j] = Frag<bf16>::mma(af[i], bf[j], acc[i][j]);
     };
     int st = 0;
-    for (int ks = 0; ks < ksteps; ks += 2, st ^= 1) {
-        if (ks + 2 < ksteps) issue(st ^ 1, ks + 2);
+    for (int ks = 0; ks < ksteps; ks += 2) {
+        // this stage has arrived (the S − 2 after it may be on their way) and every wave is done with the one before it, whose place the
+        // next request takes
+        if (S > 2 && ks + 2 * (S - 2) < ksteps) asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)\n\ts_barrier" ::"n"((S - 2) * 2 * (AT + BT)) : "memory");
+        else asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)\n\ts_barrier" ::: "memory");
+        if (ks + 2 * (S - 1) < ksteps) issue(st ? st - 1 : S - 1, ks + 2 * (S - 1));
         const bf16 *la = lds + st * STAGE + wm * MI * 1024 + lane * 8, *lb = lds + st * STAGE + (T::RT + wn * NJ) * 1024 + lane * 8;
         multiply(la, lb, 0);
         multiply(la, lb, 1);
@@ -279,9 +283,9 @@ __global__ __launch_bounds__(64 * WM * WN, 2) void tiled_gemm_big_kernel(TiledGe
             __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
         }
         __builtin_amdgcn_sched_group_barrier(0x008, 2 * MI * NJ - LEFT * PER, 0);
-        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-        __syncthreads();
+        st = st + 1 < S ? st + 1 : 0;
     }
+    __syncthreads();
     // epilogue: 32 rows of a wave's accumulators at a time through LDS (the stages are free, the rows its own, LDS operations of a wave
     // complete in order), then a lane finishes 8 columns of a row: bias, activation and factors, and rows leave in 16-byte pieces.  In a
     // gated section the lanes of the up tiles have nothing to do, those of the gate tiles read both.
@@ -349,18 +353,18 @@ __global__ __launch_bounds__(64 * WM * WN, 2) void tiled_gemm_big_kernel(TiledGe
     }
 }
 
-template <int WM, int WN, int MI, int NJ>
+template <int WM, int WN, int MI, int NJ, int S>
 static int launch_big(const TiledGemm<bf16>& g, hipStream_t s) {
-    typedef BigTile<WM, WN, MI, NJ> T;
+    typedef BigTile<WM, WN, MI, NJ, S> T;
     static bool attr = false;
     if (!attr) {
-        FH_CHECK_HIP(hipFuncSetAttribute((const void*)tiled_gemm_big_kernel<WM, WN, MI, NJ>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)T::LDS));
+        FH_CHECK_HIP(hipFuncSetAttribute((const void*)tiled_gemm_big_kernel<WM, WN, MI, NJ, S>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)T::LDS));
         attr = true;
     }
     const int mtiles = g.rows.id ? g.rows.max_blocks : cdiv(g.m, T::ROWS), ntiles = cdiv(g.n, T::COLS);
     form_hit(g.rows.id ? FORM_TILED_GEMM_GROUPED_BIG : FORM_TILED_GEMM_BIG);
     if (T::ROWS == 256) form_hit(FORM_TILED_GEMM_256);
-    hipLaunchKernelGGL((tiled_gemm_big_kernel<WM, WN, MI, NJ>), dim3(mtiles * ntiles, 1, g.groups), dim3(64 * T::WAVES), T::LDS, s, g, mtiles, ntiles);
+    hipLaunchKernelGGL((tiled_gemm_big_kernel<WM, WN, MI, NJ, S>), dim3(mtiles * ntiles, 1, g.groups), dim3(64 * T::WAVES), T::LDS, s, g, mtiles, ntiles);
     FH_CHECK_LAUNCH();
     return 0;
 }
@@ -368,7 +372,11 @@ static int launch_big(const TiledGemm<bf16>& g, hipStream_t s) {
     // one 256 × 256 tile per CU, or two of 128 × 128: the large one halves the bytes per product, as long as there are enough of them
     const long tiles = (long)cdiv(g.m, 256) * cdiv(g.n, 256) * g.groups;
     const bool wide = g.rows.id ? g.rows.block == 256 : tiles >= knobs().tiled_wide_min_tiles;
-    return wide ? launch_big<2, 4, 8, 4>(g, s) : launch_big<2, 2, 4, 4>(g, s);
+    if (wide) return launch_big<2, 4, 8, 4, 2>(g, s);
+    // few tiles: rows in halves so that every CU has one, or one workgroup per CU, and a deeper ring in place of the second workgroup
+    const long tiles128 = (long)cdiv(g.m, 128) * cdiv(g.n, 128) * g.groups;
+    if (!g.rows.id && tiles128 <= knobs().tiled_half_max_tiles) return launch_big<2, 2, 2, 4, 5>(g, s);
+    return !g.rows.id && tiles128 <= 256 ? launch_big<2, 2, 4, 4, 4>(g, s) : launch_big<2, 2, 4, 4, 2>(g, s);
 }
 static int launch_big(const TiledGemm<float>&, hipStream_t) { return 2; }      // (never taken: 16-bit only)
 
@@ -411,7 +419,7 @@ int tiled_gemm(const TiledGemm<E>& gin, hipStream_t s) {
         FH_REQUIRE(rows.block == 16 || rows.block == 32 || rows.block == 64 || ((rows.block == 128 || rows.block == 256) && sizeof(E) == 2), "tiled_gemm: blocks of %d rows", rows.block);
     }
     const long tiles = (long)cdiv(g.m, 128) * cdiv(g.n, 128) * g.groups;
-    if (rows.id ? rows.block >= 128 : sizeof(E) == 2 && g.m > 64 && g.slabs == 1 && tiles >= knobs().tiled_big_min_tiles) return launch_big(g, s);
+    if (rows.id ? rows.block >= 128 : sizeof(E) == 2 && g.m > 64 && g.n >= 128 && g.slabs == 1 && tiles >= knobs().tiled_big_min_tiles) return launch_big(g, s);
     const int mt = rows.id ? rows.block / 16 : g.m <= 16 ? 1 : (g.m <= 32 ? 2 : 4);
     const int rbs = rows.id ? rows.max_blocks : cdiv(g.m, 16 * mt), ksteps = g.k / 32, zs = rows.id ? 1 : g.groups * g.slabs;
     // 32 columns per wave, 16 where 32 would leave CUs without a workgroup; K split over the waves until the launch has enough of them
@@ -419,7 +427,7 @@ int tiled_gemm(const TiledGemm<E>& gin, hipStream_t s) {
     if (knobs().tiled_j > 0) J = knobs().tiled_j == 1 ? 1 : 2;
     if (gated) J = 2;
     const long cols = g.n / (16 * J);
-    int nw = mt == 1 ? 8 : 4, kw = 1;
+    int nw = mt == 1 || rbs * cols * zs <= 256 ? 8 : 4, kw = 1;
     if (knobs().tiled_nw > 0) nw = std::min(8, knobs().tiled_nw);
     while (kw < nw && (long)rbs * cols * zs * kw < 4096 && ksteps >= 8 * kw * g.slabs) kw *= 2;
     if (knobs().tiled_kw > 0) kw = std::min(nw, knobs().tiled_kw);
