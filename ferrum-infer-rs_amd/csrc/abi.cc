@@ -55,6 +55,7 @@ void reload_knobs() {
     k.tiled_nw = env_int("FERRUM_HIP_TILED_NW", 0);
     k.tiled_kw = env_int("FERRUM_HIP_TILED_KW", 0);
     k.tiled_j = env_int("FERRUM_HIP_TILED_J", 0);
+    k.layer_overlap_max_tokens = env_int("FERRUM_HIP_LAYER_OVERLAP_MAX_TOKENS", 64);
     k.latent_tiles = env_int("FERRUM_HIP_LATENT_TILES", 0);
     k.latent_splits = env_int("FERRUM_HIP_LATENT_SPLITS", 0);
     k.latent_expand_min_rows = env_int("FERRUM_HIP_LATENT_EXPAND_MIN_ROWS", 64);

@@ -60,6 +60,7 @@ struct Knobs {
     int tiled_half_max_tiles = 128;   // … its 64 × 128 form up to this many tiles of 128 × 128
     int moe_rows_block = 0;           // > 0: forced rows per block of the sorted expert rows
     int tiled_nw = 0, tiled_kw = 0, tiled_j = 0;      // > 0: forced waves per workgroup, K parts, 16-column tiles per wave of the few-row kernel
+    int layer_overlap_max_tokens = 64;   // parallel blocks: experts on a stream of their own beside the mixer up to this many tokens (0 = never)
     int latent_tiles = 0;             // 1 / 2: forced 16-row tiles per workgroup of the latent attention
     int latent_splits = 0;            // > 0: forced KV split count of the latent attention
     int latent_expand_min_rows = 64;  // prompt portions of at least this many tokens attend expanded keys / values (0 = never)

@@ -117,7 +117,12 @@ public:
         : c_(c), lc_(lc), slots_(slots), D_(c.hidden), Dp_(pad32(c.hidden)) {
         for (int i = 0; i < c.num_layers; i++) { Layer L; L.s = layers[i]; dims(L); layers_.push_back(L); }
     }
-    ~Layered() override { if (plan_host_) (void)hipHostFree(plan_host_); }
+    ~Layered() override {
+        if (plan_host_) (void)hipHostFree(plan_host_);
+        if (fork_) (void)hipEventDestroy(fork_);
+        if (join_) (void)hipEventDestroy(join_);
+        if (side_stream_) (void)hipStreamDestroy(side_stream_);
+    }
     bool has_state() const override {
         return std::any_of(layers_.begin(), layers_.end(), [](const Layer& L) { return L.s.mixer == FERRUM_HIP_MIXER_RGLRU; });
     }
@@ -228,6 +233,11 @@ public:
         FH_TRY(arena_.alloc(&expert_y_, pairs * Dp_));
         FH_TRY(arena_.alloc(&head_in_, (size_t)c_.max_seqs * Dp_));
         FH_TRY(finalize_expansion());
+        if (pairs) {
+            FH_CHECK_HIP(hipStreamCreateWithFlags(&side_stream_, hipStreamNonBlocking));
+            FH_CHECK_HIP(hipEventCreateWithFlags(&fork_, hipEventDisableTiming));
+            FH_CHECK_HIP(hipEventCreateWithFlags(&join_, hipEventDisableTiming));
+        }
         for (Layer& L : layers_) {
             if (L.s.kv_source) L.lb.pool = layers_[L.s.kv_source - 1].lb.pool;
             L.lb.q = L.ld.q_rank ? q_ : in_ + L.c0;
@@ -295,12 +305,24 @@ private:
         hipStream_t s = run.s;
         const bool moe = L.s.ff == FERRUM_HIP_FF_MOE_RELU2, last = run.li + 1 == c_.num_layers;
         int slabs = 1;
+        // few tokens: the experts, bound by their weights' bytes, beside the mixer, bound by the latency of its chain of launches
+        const bool beside = moe && T <= knobs().layer_overlap_max_tokens && !run.trace;
+        if (beside) {
+            Run other = run;
+            other.s = side_stream_;
+            FH_CHECK_HIP(hipEventRecord(fork_, s));
+            FH_CHECK_HIP(hipStreamWaitEvent(side_stream_, fork_, 0));
+            FH_TRY(experts(L, other));
+            FH_CHECK_HIP(hipEventRecord(join_, side_stream_));
+        } else if (moe) {
+            FH_TRY(experts(L, run));
+        }
         RUN(tiled_gemm(input_projection(L, T), s));
-        if (moe) FH_TRY(experts(L, run));
         E* att = L.c_att >= 0 ? in_ + L.c_att : attn_;
         const long ld_att = L.c_att >= 0 ? L.ld_in : (long)L.ld.heads * L.ld.vp;
         FH_TRY(attend(L, run, att, ld_att));
         RUN(tiled_gemm(linear_slabs(L.o, L.c_glu >= 0 ? in_ + L.c_glu : att, ld_att, T, &slabs), s));
+        if (beside) FH_CHECK_HIP(hipStreamWaitEvent(s, join_, 0));
         RUN(branch_add<E>(sub_, Dp_, slabs, (long)T * Dp_, expert_y_, Dp_, expert_weights_, moe ? L.s.top : 0, x_, xb_, T, D_, Dp_, s));
         if (lc_.token_side_dim) {
             TiledGemm<E> g = linear(L.side_gate, xb_, Dp_, T, side_, L.side_gate.n);
@@ -790,7 +812,8 @@ private:
     FerrumHipModelConfig c_;
     FerrumHipLayeredConfig lc_;
     int slots_, D_, Dp_;
-    hipStream_t stream_ = nullptr;
+    hipStream_t stream_ = nullptr, side_stream_ = nullptr;
+    hipEvent_t fork_ = nullptr, join_ = nullptr;
     bool synth_ = false;
     uint64_t seed_ = 0;
     Arena arena_;

@@ -12,11 +12,10 @@
 
 namespace fh {
 
-// Router of one token on one wave (E ≤ 512, lane l looks at experts l, l + 64, …): f32 softmax, k argmax-mask passes, ties → lowest index.
-// Lane k ends up with the k-th choice.
-template <typename T>
+// Router of one token on one wave (E ≤ 64·PER, lane l looks at experts l, l + 64, …): f32 softmax, k argmax-mask passes, ties → lowest
+// index.  Lane k ends up with the k-th choice.
+template <int PER, typename T>
 __device__ __forceinline__ void route_token(const T* __restrict__ row, int lane, int num_experts, int top_k, int norm_topk_prob, int& id, float& weight) {
-    constexpr int PER = 8;   // experts per lane (E ≤ 512)
     float v[PER];
     float mx = -INFINITY;
 #pragma unroll
@@ -62,14 +61,23 @@ __device__ __forceinline__ void route_token(const T* __restrict__ row, int lane,
     if (norm_topk_prob) weight = sel_sum > 0.f ? weight * (1.0f / sel_sum) : 1.0f / (float)top_k;
 }
 
-template <typename T>
+// the launch `call` with PER experts per lane
+#define ROUTE_PER(call)                                                    \
+    do {                                                                   \
+        if (num_experts <= 64) { constexpr int PER = 1; call; }            \
+        else if (num_experts <= 128) { constexpr int PER = 2; call; }      \
+        else if (num_experts <= 256) { constexpr int PER = 4; call; }      \
+        else { constexpr int PER = 8; call; }                              \
+    } while (0)
+
+template <int PER, typename T>
 __global__ __launch_bounds__(64) void moe_route_kernel(const T* __restrict__ logits, int32_t* __restrict__ ids,
                                                        float* __restrict__ weights, int num_experts, int top_k,
                                                        int norm_topk_prob) {
     const int tok = blockIdx.x, lane = threadIdx.x;
     int id;
     float w;
-    route_token(logits + (long)tok * num_experts, lane, num_experts, top_k, norm_topk_prob, id, w);
+    route_token<PER>(logits + (long)tok * num_experts, lane, num_experts, top_k, norm_topk_prob, id, w);
     if (lane < top_k) {
         ids[(long)tok * top_k + lane] = id;
         weights[(long)tok * top_k + lane] = w;
@@ -80,6 +88,7 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const T* __restrict__ log
 // moe_align_kernel<0> write them, except that nothing is written past the last block).  A wave routes its tokens, then every thread owns
 // a pair: its rank among the pairs of its expert is the count in earlier waves (histograms in LDS) plus the count in earlier lanes.
 constexpr int ROUTE_SORT_PAIRS = 1024;
+template <int PER>
 __global__ __launch_bounds__(1024) void moe_route_sort_kernel(const float* __restrict__ logits, int32_t* __restrict__ ids, float* __restrict__ weights,
                                                               int32_t* __restrict__ sorted, int32_t* __restrict__ block_ids, int32_t* __restrict__ total,
                                                               int tokens, int num_experts, int top_k, int norm_topk_prob, int block_size) {
@@ -90,7 +99,7 @@ __global__ __launch_bounds__(1024) void moe_route_sort_kernel(const float* __res
     for (int t = wave; t < tokens; t += 16) {
         int id;
         float w;
-        route_token(logits + (long)t * num_experts, lane, num_experts, top_k, norm_topk_prob, id, w);
+        route_token<PER>(logits + (long)t * num_experts, lane, num_experts, top_k, norm_topk_prob, id, w);
         if (lane < top_k) {
             lds_id[t * top_k + lane] = (int16_t)id;
             ids[t * top_k + lane] = id;
@@ -145,8 +154,8 @@ int moe_route_sort_f32(const float* logits, int32_t* expert_ids, float* expert_w
     FH_REQUIRE(moe_route_sort_supports(tokens, num_experts, top_k) && num_experts > 0 && top_k > 0 && top_k <= num_experts && top_k <= 64 && block_size > 0,
                "moe route + sort: %d tokens, %d of %d experts, blocks of %d", tokens, top_k, num_experts, block_size);
     form_hit(FORM_MOE_ROUTE_SORT);
-    hipLaunchKernelGGL(moe_route_sort_kernel, dim3(1), dim3(1024), 0, s, logits, expert_ids, expert_weights, sorted_token_ids, block_ids, total_post_pad,
-                       tokens, num_experts, top_k, norm_topk_prob, block_size);
+    ROUTE_PER(hipLaunchKernelGGL(moe_route_sort_kernel<PER>, dim3(1), dim3(1024), 0, s, logits, expert_ids, expert_weights, sorted_token_ids, block_ids,
+                                 total_post_pad, tokens, num_experts, top_k, norm_topk_prob, block_size));
     FH_CHECK_LAUNCH();
     return 0;
 }
@@ -156,8 +165,8 @@ int moe_route_topk_softmax_f16(const __half* logits, int32_t* expert_ids, float*
     if (tokens <= 0) return 0;
     FH_REQUIRE(num_experts > 0 && num_experts <= 512, "moe route: num_experts=%d must be in [1,512]", num_experts);
     FH_REQUIRE(top_k > 0 && top_k <= num_experts && top_k <= 64, "moe route: top_k=%d invalid for %d experts", top_k, num_experts);
-    hipLaunchKernelGGL(moe_route_kernel<__half>, dim3(tokens), dim3(64), 0, s, logits, expert_ids, expert_weights,
-                       num_experts, top_k, norm_topk_prob);
+    ROUTE_PER(hipLaunchKernelGGL((moe_route_kernel<PER, __half>), dim3(tokens), dim3(64), 0, s, logits, expert_ids, expert_weights,
+                                 num_experts, top_k, norm_topk_prob));
     FH_CHECK_LAUNCH();
     return 0;
 }
@@ -166,8 +175,8 @@ int moe_route_topk_softmax_f32(const float* logits, int32_t* expert_ids, float* 
     if (tokens <= 0) return 0;
     FH_REQUIRE(num_experts > 0 && num_experts <= 512, "moe route: num_experts=%d must be in [1,512]", num_experts);
     FH_REQUIRE(top_k > 0 && top_k <= num_experts && top_k <= 64, "moe route: top_k=%d invalid for %d experts", top_k, num_experts);
-    hipLaunchKernelGGL(moe_route_kernel<float>, dim3(tokens), dim3(64), 0, s, logits, expert_ids, expert_weights,
-                       num_experts, top_k, norm_topk_prob);
+    ROUTE_PER(hipLaunchKernelGGL((moe_route_kernel<PER, float>), dim3(tokens), dim3(64), 0, s, logits, expert_ids, expert_weights,
+                                 num_experts, top_k, norm_topk_prob));
     FH_CHECK_LAUNCH();
     return 0;
 }

@@ -423,13 +423,13 @@ int tiled_gemm(const TiledGemm<E>& gin, hipStream_t s) {
     const int mt = rows.id ? rows.block / 16 : g.m <= 16 ? 1 : (g.m <= 32 ? 2 : 4);
     const int rbs = rows.id ? rows.max_blocks : cdiv(g.m, 16 * mt), ksteps = g.k / 32, zs = rows.id ? 1 : g.groups * g.slabs;
     // 32 columns per wave, 16 where 32 would leave CUs without a workgroup; K split over the waves until the launch has enough of them
-    int J = (long)rbs * (g.n / 32) * zs < 256 ? 1 : 2;
+    int J = (long)rbs * (g.n / 32) * zs < (g.slabs > 1 ? 256 : 257) ? 1 : 2;
     if (knobs().tiled_j > 0) J = knobs().tiled_j == 1 ? 1 : 2;
     if (gated) J = 2;
     const long cols = g.n / (16 * J);
-    int nw = mt == 1 || rbs * cols * zs <= 256 ? 8 : 4, kw = 1;
+    int nw = mt == 1 ? 8 : 4, kw = 1;
     if (knobs().tiled_nw > 0) nw = std::min(8, knobs().tiled_nw);
-    while (kw < nw && (long)rbs * cols * zs * kw < 4096 && ksteps >= 8 * kw * g.slabs) kw *= 2;
+    while (kw < nw && (long)rbs * cols * zs * kw < (rows.id ? 8192 : 4096) && ksteps >= 8 * kw * g.slabs) kw *= 2;
     if (knobs().tiled_kw > 0) kw = std::min(nw, knobs().tiled_kw);
     const dim3 grid(cdiv(cols, nw / kw), rbs, zs);
     form_hit(rows.id ? FORM_TILED_GEMM_GROUPED : FORM_TILED_GEMM);
