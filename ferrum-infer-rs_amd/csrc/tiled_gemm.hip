@@ -75,9 +75,11 @@ __device__ __forceinline__ int gemm_row_step(const TiledGemm<E>& p) { return p.x
 
 // grid (column blocks, row blocks, groups or K slabs); NW waves = (NW / kw) column groups × kw parts of K.  Two register buffers of U
 // k-steps: the next one is requested before the current one is multiplied; loads past the part's end repeat its last k-step.
-template <typename E, int MT, int J>
+// EXT: with sorted rows, column factors or gated sections (each is a branch on the latency-bound path of the launches without).
+template <typename E, int MT, int J, bool EXT>
 __global__ __launch_bounds__(512) void tiled_gemm_kernel(TiledGemm<E> p, int kw) {
     typedef typename Frag<E>::v8 v8;
+    if (!EXT) { p.rows.id = nullptr; p.col_scale = nullptr; }
     extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
     floatx4* red = reinterpret_cast<floatx4*>(smem);            // [NW][MT·J][64]
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
@@ -142,7 +144,7 @@ __global__ __launch_bounds__(512) void tiled_gemm_kernel(TiledGemm<E> p, int kw)
     }
     if (p.slabs > 1) p.out_f32 += z * p.slab_stride;
     const GemmSection sec = gemm_section(p, n0);
-    const bool gated = J == 2 && sec.act == GEMM_ACT_CLAMPED_GLU;
+    const bool gated = EXT && J == 2 && sec.act == GEMM_ACT_CLAMPED_GLU;
     if (kw == 1) {
         if (!live) return;
         if constexpr (J == 2)
@@ -388,10 +390,10 @@ int tiled_gemm_slabs(int m, int n, int k) {
     return S;
 }
 
-template <typename E, int MT, int J>
+template <typename E, int MT, int J, bool EXT>
 static int launch_small(const TiledGemm<E>& g, dim3 grid, int nw, int kw, hipStream_t s) {
     const size_t lds = kw == 1 ? 0 : (size_t)nw * MT * J * 1024;
-    hipLaunchKernelGGL((tiled_gemm_kernel<E, MT, J>), grid, dim3(64 * nw), lds, s, g, kw);
+    hipLaunchKernelGGL((tiled_gemm_kernel<E, MT, J, EXT>), grid, dim3(64 * nw), lds, s, g, kw);
     FH_CHECK_LAUNCH();
     return 0;
 }
@@ -433,8 +435,11 @@ int tiled_gemm(const TiledGemm<E>& gin, hipStream_t s) {
     if (knobs().tiled_kw > 0) kw = std::min(nw, knobs().tiled_kw);
     const dim3 grid(cdiv(cols, nw / kw), rbs, zs);
     form_hit(rows.id ? FORM_TILED_GEMM_GROUPED : FORM_TILED_GEMM);
-    if (J == 1) return mt == 1 ? launch_small<E, 1, 1>(g, grid, nw, kw, s) : mt == 2 ? launch_small<E, 2, 1>(g, grid, nw, kw, s) : launch_small<E, 4, 1>(g, grid, nw, kw, s);
-    return mt == 1 ? launch_small<E, 1, 2>(g, grid, nw, kw, s) : mt == 2 ? launch_small<E, 2, 2>(g, grid, nw, kw, s) : launch_small<E, 4, 2>(g, grid, nw, kw, s);
+#define SMALL(J_, EXT_) \
+    (mt == 1 ? launch_small<E, 1, J_, EXT_>(g, grid, nw, kw, s) : mt == 2 ? launch_small<E, 2, J_, EXT_>(g, grid, nw, kw, s) : launch_small<E, 4, J_, EXT_>(g, grid, nw, kw, s))
+    if (rows.id || g.col_scale || gated) return J == 1 ? SMALL(1, true) : SMALL(2, true);
+    return J == 1 ? SMALL(1, false) : SMALL(2, false);
+#undef SMALL
 }
 template int tiled_gemm<bf16>(const TiledGemm<bf16>&, hipStream_t);
 template int tiled_gemm<float>(const TiledGemm<float>&, hipStream_t);
