@@ -105,7 +105,7 @@ __global__ __launch_bounds__(512) void tiled_gemm_kernel(TiledGemm<E> p, int kw)
     for (int mt = 0; mt < MT; mt++)
 #pragma unroll
         for (int j = 0; j < J; j++) acc[mt][j] = (floatx4){0.f, 0.f, 0.f, 0.f};
-    constexpr int U = sizeof(E) == 2 ? 4 : 1;
+    constexpr int U = sizeof(E) == 2 ? (MT * J == 1 ? 8 : 4) : 1;
     v8 bw[2][U][J], ax[2][U][MT];
     auto load = [&](v8 (&bq)[U][J], v8 (&aq)[U][MT], int s) {
 #pragma unroll
@@ -422,7 +422,9 @@ int tiled_gemm(const TiledGemm<E>& gin, hipStream_t s) {
     }
     const long tiles = (long)cdiv(g.m, 128) * cdiv(g.n, 128) * g.groups;
     if (rows.id ? rows.block >= 128 : sizeof(E) == 2 && g.m > 64 && g.n >= 128 && g.slabs == 1 && tiles >= knobs().tiled_big_min_tiles) return launch_big(g, s);
-    const int mt = rows.id ? rows.block / 16 : g.m <= 16 ? 1 : (g.m <= 32 ? 2 : 4);
+    // rows per workgroup: as many as there are, fewer where narrow outputs would leave CUs idle
+    int mt = rows.id ? rows.block / 16 : g.m <= 16 ? 1 : (g.m <= 32 ? 2 : 4);
+    while (!rows.id && mt > 1 && (long)cdiv(g.m, 16 * mt) * (g.n / 16) * g.groups * g.slabs < knobs().tiled_min_tiles) mt /= 2;
     const int rbs = rows.id ? rows.max_blocks : cdiv(g.m, 16 * mt), ksteps = g.k / 32, zs = rows.id ? 1 : g.groups * g.slabs;
     // 32 columns per wave, 16 where 32 would leave CUs without a workgroup; K split over the waves until the launch has enough of them
     int J = (long)rbs * (g.n / 32) * zs < (g.slabs > 1 ? 256 : 257) ? 1 : 2;

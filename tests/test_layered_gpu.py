@@ -450,17 +450,17 @@ def test_trace_replay(cases, tmp_path, name, dtype):
 
 @pytest.mark.parametrize("name", ["wide", "shared", "sinks"])
 def test_few_row_and_tile_projections_agree(pkg, cases, knobs, forms, name):
-    """The 128 × 128 tile kernel and the few-row kernel on the same portions."""
+    """The tile kernel in each of its sizes and the few-row kernel on the same portions."""
     cfg, w, path = cases(name)
     t = toks(cfg, 200, 12)
     want = L.forward(cfg, w, t)
-    for tiles, name in ((1, "tiled_gemm_big"), (10 ** 6, "tiled_gemm")):
-        knobs.set(TILED_BIG_MIN_TILES=tiles)
+    for big, wide, half, ran in ((1, 10 ** 6, 0, "tiled_gemm_big"), (1, 10 ** 6, 10 ** 6, "tiled_gemm_big"), (1, 1, 0, "tiled_gemm_256"), (10 ** 6, 192, 128, "tiled_gemm")):
+        knobs.set(TILED_BIG_MIN_TILES=big, TILED_WIDE_MIN_TILES=wide, TILED_HALF_MAX_TILES=half)
         m = load(pkg, path, "bfloat16")
         forms.reset()
         assert rel(feed(m, 1, t, [200]), want) < TOL["bfloat16"]
-        assert forms.hits().get(name)
-        assert tiles == 1 or not forms.hits().get("tiled_gemm_big")
+        h = forms.hits()
+        assert h.get(ran) and bool(h.get("tiled_gemm_big")) == (big == 1) and bool(h.get("tiled_gemm_256")) == (wide == 1)
 
 
 def test_missing_and_misshapen_weights_are_named(pkg, tmp_path):

@@ -72,29 +72,57 @@ def test_clamped_glu_alone(pkg, tmp_path, dtype, ff, limit, scale):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("n,top,ff", [(7, 3, 41), (16, 1, 64), (5, 5, 20), (1, 1, 33), (70, 6, 24), (130, 2, 40)])
-@pytest.mark.parametrize("tokens", [1, 3, 90])
-def test_experts_alone(pkg, tmp_path, dtype, n, top, ff, tokens):
-    """Blocks of every size that the batch and the number of experts lead to; 32-bit: routers that read everything."""
+@pytest.mark.parametrize("n,top,ff", [(7, 3, 41), (16, 1, 64), (5, 5, 20), (1, 1, 33), (70, 6, 24), (130, 2, 40), (300, 7, 9)])
+@pytest.mark.parametrize("tokens", [1, 3, 90, 150])
+def test_experts_alone(pkg, tmp_path, forms, dtype, n, top, ff, tokens):
+    """Routing and sorting in one launch and in two, on every number of experts per lane; 32-bit: routers that read everything."""
     cfg = model([G.sink_attention(2, 8, 4, 8, 16, mlp=G.experts(n, top, ff))])
     w = G.weights(cfg, 43, clear_routes=dtype == "bfloat16")
     silence(w, "mix.o", "side.norm")
     _, taps = agree(pkg, tmp_path, cfg, w, dtype, n=tokens)
-    if top < n:
+    assert bool(forms.hits().get("moe_route_sort")) == (tokens * top <= 1024)
+    if top < n and dtype == "float32":                                        # (clear routes leave the last choice little weight)
         other = []
         L.forward(changed(cfg, lambda c: c["layers"][0]["mlp"]["router"].update(top=top + 1)), w, toks(cfg, tokens, 6), other)
         assert rel(other, taps) > 3e-5
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-def test_experts_of_long_prompts(pkg, tmp_path, forms, dtype):
-    """Every block size of the sorted rows, up to the 128-row tiles, with experts that receive few rows or none."""
+@pytest.mark.parametrize("block", [0, 16, 32, 64, 128, 256])
+def test_experts_of_long_prompts(pkg, tmp_path, forms, knobs, block, dtype):
+    """Every block size of the sorted rows, up to the 256-row tiles, with experts that receive few rows or none; an odd number of K steps."""
+    knobs.set(MOE_ROWS_BLOCK=block)
     for n, top, tokens in ((4, 2, 400), (9, 3, 110), (6, 1, 75), (12, 2, 500)):
         cfg = model([G.sink_attention(2, 8, 4, 8, 16, mlp=G.experts(n, top, 48))], width=160)
         w = G.weights(cfg, 44)
         silence(w, "mix.o", "side.norm")
         agree(pkg, tmp_path / str(n), cfg, w, dtype, n=tokens)
-    assert forms.hits().get("tiled_gemm_grouped") and bool(forms.hits().get("tiled_gemm_grouped_big")) == (dtype == "bfloat16")
+    h = forms.hits()
+    assert bool(h.get("tiled_gemm_grouped_big")) == (dtype == "bfloat16" and (block == 0 or block > 64))
+    assert bool(h.get("tiled_gemm_grouped")) == (dtype == "float32" or block <= 64)
+
+
+def test_experts_beside_the_mixer(pkg, cases, knobs):
+    """Small batches run the experts on a stream of their own: the same ids as in one stream, eagerly and over many replays of the graph
+    with eager work between them."""
+    cfg, w, path = cases("sinks")
+    prompts = [toks(cfg, n, 190 + n) for n in (5, 40)]
+    runs = []
+    for tokens in (0, 64):
+        knobs.set(LAYER_OVERLAP_MAX_TOKENS=tokens)
+        m = load(pkg, path, "float32", tokens=400, seqs=3, max_len=180)
+        nxt, _ = m.unified_forward([(i, p, 0, True) for i, p in enumerate(prompts)])
+        out = [nxt[None]]
+        for steps in (2, 40, 1, 30):
+            out.append(m.decode_steps([0, 1], nxt, steps))
+            nxt = out[-1][-1]
+            m.unified_forward([(7, toks(cfg, 9, steps), 0, True)])
+            m.release(7)
+        for _ in range(20):
+            nxt, _ = m.unified_forward([(i, [int(t)], m.block_table(i)[1], True) for i, t in enumerate(nxt)])
+            out.append(nxt[None])
+        runs.append(np.concatenate(out))
+    assert np.array_equal(*runs)
 
 
 def test_equal_router_logits_take_the_first_experts(pkg, tmp_path):
