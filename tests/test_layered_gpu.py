@@ -21,6 +21,7 @@ DTYPES = ["float32", "bfloat16"]
 
 @pytest.fixture(scope="module")
 def pkg():
+    import torch  # noqa: F401  (ahead of the library: imported later, torch finds no device, and other modules' tests need it)
     import __graft_entry__ as ge
     p = ge.load_package()
     p.load_library()
