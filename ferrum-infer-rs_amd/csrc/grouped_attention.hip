@@ -1,6 +1,6 @@
 // Attention whose keys and values are cached per group of query heads, with a sliding window.
 //
-// Queries and keys are normed over all their rows at once, so a workgroup prepares a whole token: both sums of squares, the norms'
+// Queries and keys are normed over all their rows at once, or head by head; a workgroup prepares a whole token: sums of squares, the norms'
 // weights, the rotation, and the cache write.  The attention kernels work on rows that are (token, query head) pairs of one sequence and
 // key / value head: G = heads / kv_heads rows of a token share every key they read.
 //
@@ -12,13 +12,12 @@
 #include <algorithm>
 
 #include "common.h"
+#include "grouped_cache.h"
 #include "knobs.h"
 #include "layer_ops.h"
 #include "seq_tiles.h"
 
 namespace fh {
-
-__device__ __forceinline__ int value_offset(int slot, int d) { return ((((d >> 5) * 4 + (slot >> 2)) * 16 + (d & 15)) * 2 + ((d >> 4) & 1)) * 4 + (slot & 3); }
 
 // one workgroup per token
 template <typename E>
@@ -64,7 +63,47 @@ __global__ __launch_bounds__(256) void grouped_prepare_kernel(GroupedDims d, Gro
     for (int i = tid; i < nv; i += 256) vt[(long)(i / d.vp) * d.vp * 16 + value_offset(slot, i % d.vp)] = vr[i];
 }
 
-// factor of a row's Σ e^(score − m)·value
+// the same with norms of one head each: a power of two of lanes (`sub`) per head, 8 dimensions a lane
+template <typename E>
+__global__ __launch_bounds__(256) void grouped_prepare_heads_kernel(GroupedDims d, GroupedBuffers<E> p, BatchView v, int sub) {
+    typedef typename Frag<E>::v8 v8;
+    const int t = blockIdx.x, tid = threadIdx.x, seq = v.tok_seq[t], lane = tid & (sub - 1);
+    const long pos = (long)v.pos[seq] + t - v.cu[seq];
+    const long block = v.bt[(long)seq * v.max_blocks + pos / 16];
+    const int slot = pos % 16, nk = p.k_in ? d.kv_heads : 0;
+    for (int h = tid / sub; h < d.heads + nk; h += 256 / sub) {
+        const bool query = h < d.heads;
+        const int kh = h - d.heads;
+        const E* src = query ? p.q_in + t * p.ld + (long)h * d.dp : p.k_in + t * p.ld + (long)kh * d.dp;
+        const float* w = query ? p.q_norm : p.k_norm;
+        float s = 0.f;
+        for (int i = lane * 8; i < d.dp; i += sub * 8) {
+            const v8 x = *reinterpret_cast<const v8*>(src + i);
+#pragma unroll
+            for (int j = 0; j < 8; j++) s += (float)x[j] * (float)x[j];       // (padded columns are zero)
+        }
+        for (int off = 1; off < sub; off <<= 1) s += __shfl_xor(s, off, 64);
+        const float inv = 1.0f / sqrtf(s / (float)d.dim + p.eps);
+        for (int i = lane * 8; i < d.dp; i += sub * 8) {
+            const v8 x = *reinterpret_cast<const v8*>(src + i);
+            floatx8 f;
+#pragma unroll
+            for (int j = 0; j < 8; j++) f[j] = (float)x[j] * inv * w[i + j];
+            f = rot_apply(f, rot_load(i, d.rot_dims, p.cos_t, p.sin_t, pos));
+            v8 o;
+#pragma unroll
+            for (int j = 0; j < 8; j++) o[j] = (E)f[j];
+            E* dst = query ? p.q + ((long)t * d.heads + h) * d.dp + i : p.k_pool + (block * d.kv_heads + kh) * d.dp * 16 + (i * 2 + slot) * 8;
+            *reinterpret_cast<v8*>(dst) = o;
+        }
+    }
+    if (!p.k_in) return;
+    const E* vr = p.v_in + t * p.ld;
+    E* vt = p.v_pool + block * d.kv_heads * d.vp * 16;
+    for (int i = tid; i < d.kv_heads * d.vp; i += 256) vt[(long)(i / d.vp) * d.vp * 16 + value_offset(slot, i % d.vp)] = vr[i];
+}
+
+// factor of a row's Σ e^(score − m)·value (l: with the sink)
 template <typename E>
 __device__ __forceinline__ float grouped_factor(const GroupedBuffers<E>& p, float l, long tok, int head) {
     float f = l > 0.f ? p.mult / l : 0.f;
@@ -97,6 +136,7 @@ __global__ __launch_bounds__(256) void grouped_attn_plain_kernel(GroupedDims d, 
                 for (int j = 0; j < 8; j++) acc += q[i + j] * (float)x[j];
             }
             sc = acc * d.scale;
+            if (p.r1) sc -= p.r1[h] * log1pf(p.r2[h] * (float)(pos - key));
         }
         const float mx = wave_reduce_max(sc);
         if ((tid & 63) == 0) red[wave] = mx;
@@ -120,21 +160,35 @@ __global__ __launch_bounds__(256) void grouped_attn_plain_kernel(GroupedDims d, 
         }
         __syncthreads();
     }
+    if (p.sink) l_run += expf(p.sink[h] - m_run);
     const float f = grouped_factor(p, l_run, t, h);
-    for (int i = tid; i < d.vp; i += 256) p.out[(long)t * p.ldo + h * d.vp + i] = (E)(o[i] * f);
+    for (int i = tid; i < d.vp; i += 256) {
+        const float g = p.value_gate ? (float)p.value_gate[t * p.ld_value_gate + h * d.vp + i] : 1.f;
+        p.out[(long)t * p.ldo + h * d.vp + i] = (E)(o[i] * f * g);
+    }
 }
 
 // ── matrix-core forms; DS: 32-wide steps of a head (dp = vp) ──
 constexpr int GROUPED_PARTIAL_PAD = 4;       // floats behind a partial row's outputs: maximum, sum
 typedef short shortx8 __attribute__((ext_vector_type(8)));
-// Vᵀ operand of 16 dims (half `sub` of a 32-dim load) over the keys of two blocks
-__device__ __forceinline__ bf16x8 value_operand(bf16x8 v0, bf16x8 v1, int sub) {
-    return sub ? (bf16x8){v0[4], v0[5], v0[6], v0[7], v1[4], v1[5], v1[6], v1[7]} : (bf16x8){v0[0], v0[1], v0[2], v0[3], v1[0], v1[1], v1[2], v1[3]};
+// four elements of a row's result: columns [col, col + 4) of the concatenated heads
+__device__ __forceinline__ void grouped_store4(const GroupedBuffers<bf16>& p, long tok, int col, floatx4 x, float f) {
+    bf16x4 y;
+    if (p.value_gate) {
+        const bf16x4 g = *reinterpret_cast<const bf16x4*>(p.value_gate + tok * p.ld_value_gate + col);
+#pragma unroll
+        for (int r = 0; r < 4; r++) y[r] = (bf16)(x[r] * f * (float)g[r]);
+    } else {
+#pragma unroll
+        for (int r = 0; r < 4; r++) y[r] = (bf16)(x[r] * f);
+    }
+    *reinterpret_cast<bf16x4*>(p.out + tok * p.ldo + col) = y;
 }
 
 // Few rows per sequence.  grid (16-row tiles × KV splits, kv_heads): the four waves take 32-key steps of the range in turn, straight from
 // the cache into registers (the next step is requested before this one is used), and merge through LDS.
-template <int DS>
+// FAR: scores fall with the logarithm of the distance.
+template <int DS, bool FAR>
 __global__ __launch_bounds__(256) void grouped_attn_keys_kernel(GroupedDims d, GroupedBuffers<bf16> p, BatchView v, int nsplit) {
     constexpr int DT = 2 * DS, D = 32 * DS, LD = D + 4;
     extern __shared__ __attribute__((aligned(16))) float lds_o[];              // [4][16][LD]
@@ -147,6 +201,7 @@ __global__ __launch_bounds__(256) void grouped_attn_keys_kernel(GroupedDims d, G
     const bool ok = rho < rows;
     const int tl = ok ? rho / G : 0, head = kvh * G + (ok ? rho - tl * G : 0), row_pos = w.pos0 + tl, win_lo = max(0, row_pos + 1 - d.window);
     const long tok = w.tok0 + tl;
+    const float r1 = FAR ? p.r1[head] : 0.f, r2 = FAR ? p.r2[head] : 0.f;
     const int t_first = w.tile * 16 / G, t_last = min(w.q_len - 1, (w.tile * 16 + 15) / G);
     const int blk_lo = max(0, w.pos0 + t_first + 1 - d.window) / 16, blk_hi = (w.pos0 + t_last + 16) / 16, nstep = (blk_hi - blk_lo + 1) / 2;
     const int st_lo = nstep * split / nsplit, st_hi = nstep * (split + 1) / nsplit;
@@ -180,7 +235,9 @@ __global__ __launch_bounds__(256) void grouped_attn_keys_kernel(GroupedDims d, G
 #pragma unroll
             for (int r = 0; r < 4; r++) {
                 const int key = (blk_lo + 2 * st + i) * 16 + 4 * a + r;
-                sc[4 * i + r] = ok && key <= row_pos && key >= win_lo ? (s2[0][r] + s2[1][r]) * d.scale : -INFINITY;
+                float z = (s2[0][r] + s2[1][r]) * d.scale;
+                if (FAR) z -= r1 * __logf(1.0f + r2 * (float)max(row_pos - key, 0));
+                sc[4 * i + r] = ok && key <= row_pos && key >= win_lo ? z : -INFINITY;
                 mx = fmaxf(mx, sc[4 * i + r]);
             }
         }
@@ -245,11 +302,8 @@ __global__ __launch_bounds__(256) void grouped_attn_keys_kernel(GroupedDims d, G
             continue;
         }
         const int rt = ro / G, rh = kvh * G + ro % G;
-        const float f = grouped_factor(p, lds_l[row], w.tok0 + rt, rh);
-        bf16x4 y;
-#pragma unroll
-        for (int r = 0; r < 4; r++) y[r] = (bf16)(x[r] * f);
-        *reinterpret_cast<bf16x4*>(p.out + (long)(w.tok0 + rt) * p.ldo + rh * D + c) = y;
+        const float sink = p.sink ? __expf(p.sink[rh] - lds_m[row]) : 0.f;
+        grouped_store4(p, w.tok0 + rt, rh * D + c, x, grouped_factor(p, lds_l[row] + sink, w.tok0 + rt, rh));
     }
 }
 // grid (tiles, kv_heads): one thread per (row, 4 dimensions)
@@ -271,17 +325,14 @@ __global__ __launch_bounds__(256) void grouped_attn_reduce_kernel(GroupedDims d,
             acc += *reinterpret_cast<const floatx4*>(src + z * 16 * ld + c) * f;
         }
         const int rt = ro / G, rh = kvh * G + ro % G;
-        const float f = grouped_factor(p, L, w.tok0 + rt, rh);
-        bf16x4 y;
-#pragma unroll
-        for (int r = 0; r < 4; r++) y[r] = (bf16)(acc[r] * f);
-        *reinterpret_cast<bf16x4*>(p.out + (long)(w.tok0 + rt) * p.ldo + rh * d.vp + c) = y;
+        if (p.sink) L += __expf(p.sink[rh] - M);
+        grouped_store4(p, w.tok0 + rt, rh * d.vp + c, acc, grouped_factor(p, L, w.tok0 + rt, rh));
     }
 }
 
 // Prompts.  grid (128-row tiles, kv_heads): 4 waves × 2 tiles of 16 rows.  64 keys per step: wave w copies block w of the step's keys and
 // values into LDS with the load unit, double-buffered.
-template <int DS>
+template <int DS, bool FAR>
 __global__ __launch_bounds__(256, DS <= 4 ? 2 : 1) void grouped_attn_tile_kernel(GroupedDims d, GroupedBuffers<bf16> p, BatchView v) {
     constexpr int MT = 2, DT = 2 * DS, D = 32 * DS, BLK = 2 * DS * 512;
     extern __shared__ __attribute__((aligned(16))) bf16 lds_x[];               // [2][4 blocks][BLK]: keys, values
@@ -295,12 +346,14 @@ __global__ __launch_bounds__(256, DS <= 4 ? 2 : 1) void grouped_attn_tile_kernel
     int row_pos[MT], win_lo[MT], vis_lo[MT], vis_hi[MT], head[MT];
     long tok[MT];
     bool ok[MT];
+    float r1[MT], r2[MT];
 #pragma unroll
     for (int mt = 0; mt < MT; mt++) {
         const int r0 = w.tile * 128 + (wave * MT + mt) * 16, rho = min(r0 + b, rows - 1), tl = rho / G;
         ok[mt] = r0 + b < rows;
         head[mt] = kvh * G + rho - tl * G;
         tok[mt] = w.tok0 + tl;
+        if (FAR) { r1[mt] = p.r1[head[mt]]; r2[mt] = p.r2[head[mt]]; }
         row_pos[mt] = w.pos0 + tl;
         win_lo[mt] = max(0, row_pos[mt] + 1 - d.window);
         vis_hi[mt] = r0 + 15 < rows ? w.pos0 + r0 / G : -1;                    // keys in [vis_lo, vis_hi] are seen by every row of the tile
@@ -356,6 +409,14 @@ __global__ __launch_bounds__(256, DS <= 4 ? 2 : 1) void grouped_attn_tile_kernel
         const int key0 = (blk_lo + 4 * st) * 16;
 #pragma unroll
         for (int mt = 0; mt < MT; mt++) {
+            if (FAR) {                                                         // scores in base 2 from here
+                const int d0 = row_pos[mt] - key0 - 4 * a;
+#pragma unroll
+                for (int i = 0; i < 4; i++)
+#pragma unroll
+                    for (int r = 0; r < 4; r++)
+                        sv[mt][i][r] = __builtin_fmaf(sv[mt][i][r], sl2, -r1[mt] * __builtin_amdgcn_logf(__builtin_fmaf(r2[mt], (float)max(d0 - i * 16 - r, 0), 1.0f)));
+            }
             if (!(key0 + 63 <= vis_hi[mt] && key0 >= vis_lo[mt])) {
 #pragma unroll
                 for (int i = 0; i < 4; i++)
@@ -368,7 +429,7 @@ __global__ __launch_bounds__(256, DS <= 4 ? 2 : 1) void grouped_attn_tile_kernel
             float mx = -INFINITY;
 #pragma unroll
             for (int i = 0; i < 4; i++) mx = fmaxf(mx, fmaxf(fmaxf(sv[mt][i][0], sv[mt][i][1]), fmaxf(sv[mt][i][2], sv[mt][i][3])));
-            mx = rows_reduce_max(mx * sl2);                                    // (scale > 0, checked by the caller: the maximum commutes)
+            mx = rows_reduce_max(FAR ? mx : mx * sl2);                                    // (scale > 0, checked by the caller: the maximum commutes)
             const float m_new = fmaxf(m_run[mt], mx), m_safe = m_new == -INFINITY ? 0.f : m_new;
             if (__ballot(m_new != m_run[mt]) != 0) {
                 const float alpha = __builtin_amdgcn_exp2f(m_run[mt] - m_safe);
@@ -383,7 +444,7 @@ __global__ __launch_bounds__(256, DS <= 4 ? 2 : 1) void grouped_attn_tile_kernel
             for (int i = 0; i < 4; i++)
 #pragma unroll
                 for (int r = 0; r < 4; r++) {
-                    const float e = __builtin_amdgcn_exp2f(__builtin_fmaf(sv[mt][i][r], sl2, -m_safe));
+                    const float e = __builtin_amdgcn_exp2f(FAR ? sv[mt][i][r] - m_safe : __builtin_fmaf(sv[mt][i][r], sl2, -m_safe));
                     l_run[mt] += e;
                     pf[mt][i >> 1][(i & 1) * 4 + r] = (bf16)e;
                 }
@@ -405,23 +466,22 @@ __global__ __launch_bounds__(256, DS <= 4 ? 2 : 1) void grouped_attn_tile_kernel
     }
 #pragma unroll
     for (int mt = 0; mt < MT; mt++) {
-        const float l = rows_reduce_sum(l_run[mt]);
+        float l = rows_reduce_sum(l_run[mt]);
         if (!ok[mt]) continue;
+        if (p.sink) l += __builtin_amdgcn_exp2f(p.sink[head[mt]] * 1.4426950408889634f - m_run[mt]);
         const float f = grouped_factor(p, l, tok[mt], head[mt]);
-        bf16* dst = p.out + tok[mt] * p.ldo + head[mt] * D + 4 * a;
 #pragma unroll
-        for (int t = 0; t < DT; t++) {
-            bf16x4 y;
-#pragma unroll
-            for (int r = 0; r < 4; r++) y[r] = (bf16)(o[mt][t][r] * f);
-            *reinterpret_cast<bf16x4*>(dst + t * 16) = y;
-        }
+        for (int t = 0; t < DT; t++) grouped_store4(p, tok[mt], head[mt] * D + 4 * a + t * 16, o[mt][t], f);
     }
 }
 
 template <typename E>
 int grouped_prepare(const GroupedDims& d, const GroupedBuffers<E>& b, const BatchView& v, hipStream_t s) {
-    hipLaunchKernelGGL(grouped_prepare_kernel<E>, dim3(v.T), dim3(256), 0, s, d, b, v);
+    FH_REQUIRE(b.k_in || b.head_norm, "grouped attention: keys and values of another layer take norms of one head each");
+    int sub = 1;
+    while (sub < 64 && sub * 8 < d.dp) sub *= 2;
+    if (b.head_norm) hipLaunchKernelGGL(grouped_prepare_heads_kernel<E>, dim3(v.T), dim3(256), 0, s, d, b, v, sub);
+    else hipLaunchKernelGGL(grouped_prepare_kernel<E>, dim3(v.T), dim3(256), 0, s, d, b, v);
     FH_CHECK_LAUNCH();
     return 0;
 }
@@ -435,22 +495,22 @@ static int grouped_plain(const GroupedDims& d, const GroupedBuffers<E>& b, const
     FH_CHECK_LAUNCH();
     return 0;
 }
-template <int DS>
+template <int DS, bool FAR>
 static int grouped_tile(const GroupedDims& d, const GroupedBuffers<bf16>& b, const BatchView& v, hipStream_t s) {
     constexpr size_t lds = (size_t)2 * 4 * 2 * DS * 1024;
     static bool attr = false;
-    if (!attr) { FH_CHECK_HIP(hipFuncSetAttribute((const void*)grouped_attn_tile_kernel<DS>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)); attr = true; }
+    if (!attr) { FH_CHECK_HIP(hipFuncSetAttribute((const void*)grouped_attn_tile_kernel<DS, FAR>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)); attr = true; }
     const int tiles = (int)((long)v.T * (d.heads / d.kv_heads) / 128) + v.num_seqs;      // upper bound of Σ ceil(rows of a sequence / 128)
     form_hit(FORM_GROUPED_ATTN_TILE);
-    hipLaunchKernelGGL((grouped_attn_tile_kernel<DS>), dim3(tiles, d.kv_heads), dim3(256), lds, s, d, b, v);
+    hipLaunchKernelGGL((grouped_attn_tile_kernel<DS, FAR>), dim3(tiles, d.kv_heads), dim3(256), lds, s, d, b, v);
     FH_CHECK_LAUNCH();
     return 0;
 }
-template <int DS>
+template <int DS, bool FAR>
 static int grouped_keys(const GroupedDims& d, const GroupedBuffers<bf16>& b, const BatchView& v, hipStream_t s) {
     constexpr size_t lds = (size_t)64 * (32 * DS + 4) * 4;
     static bool attr = false;
-    if (!attr) { FH_CHECK_HIP(hipFuncSetAttribute((const void*)grouped_attn_keys_kernel<DS>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)); attr = true; }
+    if (!attr) { FH_CHECK_HIP(hipFuncSetAttribute((const void*)grouped_attn_keys_kernel<DS, FAR>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)); attr = true; }
     const int G = d.heads / d.kv_heads, tiles = v.single ? v.num_seqs * cdiv(G, 16) : (int)((long)v.T * G / 16) + v.num_seqs;
     // split the keys while the launch has fewer workgroups than stay resident and a split keeps ≥ 128 keys
     const int keys = (int)std::min<long>(v.max_keys, (long)d.window + 16);
@@ -459,7 +519,7 @@ static int grouped_keys(const GroupedDims& d, const GroupedBuffers<bf16>& b, con
     if (knobs().grouped_splits > 0) ns = std::min(16, knobs().grouped_splits);
     while (ns > 1 && (size_t)tiles * d.kv_heads * ns * 16 * (d.vp + GROUPED_PARTIAL_PAD) * 4 > b.partial_bytes) ns /= 2;
     form_hit(ns > 1 ? FORM_GROUPED_ATTN_SPLIT : FORM_GROUPED_ATTN_KEYS);
-    hipLaunchKernelGGL((grouped_attn_keys_kernel<DS>), dim3(tiles * ns, d.kv_heads), dim3(256), lds, s, d, b, v, ns);
+    hipLaunchKernelGGL((grouped_attn_keys_kernel<DS, FAR>), dim3(tiles * ns, d.kv_heads), dim3(256), lds, s, d, b, v, ns);
     FH_CHECK_LAUNCH();
     if (ns > 1) {
         hipLaunchKernelGGL(grouped_attn_reduce_kernel, dim3(tiles, d.kv_heads), dim3(256), 0, s, d, b, v, ns);
@@ -467,11 +527,15 @@ static int grouped_keys(const GroupedDims& d, const GroupedBuffers<bf16>& b, con
     }
     return 0;
 }
-template <> int grouped_attention<float>(const GroupedDims& d, const GroupedBuffers<float>& b, const BatchView& v, hipStream_t s) { return grouped_plain(d, b, v, s); }
+template <> int grouped_attention<float>(const GroupedDims& d, const GroupedBuffers<float>& b, const BatchView& v, hipStream_t s) {
+    return b.talk ? talking_attention(d, b, v, s) : grouped_plain(d, b, v, s);
+}
 template <> int grouped_attention<bf16>(const GroupedDims& d, const GroupedBuffers<bf16>& b, const BatchView& v, hipStream_t s) {
+    if (b.talk) return talking_attention(d, b, v, s);
     if (knobs().grouped_plain || d.dp != d.vp || d.dp > 256 || d.scale <= 0.f) return grouped_plain(d, b, v, s);
     const bool tile = !v.single && (long)v.T * (d.heads / d.kv_heads) >= (long)knobs().grouped_tile_min_rows * v.num_seqs;
-#define GROUPED(DS) (tile ? grouped_tile<DS>(d, b, v, s) : grouped_keys<DS>(d, b, v, s))
+#define GROUPED(DS) \
+    (b.r1 ? tile ? grouped_tile<DS, true>(d, b, v, s) : grouped_keys<DS, true>(d, b, v, s) : tile ? grouped_tile<DS, false>(d, b, v, s) : grouped_keys<DS, false>(d, b, v, s))
     switch (d.dp / 32) {
     case 1: return GROUPED(1);
     case 2: return GROUPED(2);

@@ -185,18 +185,19 @@ int moe_route_topk_softmax_f16(const __half* logits, int32_t* expert_ids, float*
 bool moe_route_gemm_topk_supports(int num_experts, int hidden, int top_k);
 int moe_route_gemm_topk_f16(const __half* x, const __half* router_f16t, int32_t* expert_ids, float* expert_weights, int tokens,
                             int num_experts, int hidden, int top_k, int norm_topk_prob, hipStream_t s);
-// Sigmoid scores with a correction that takes part in the choice only: experts of the `keep` best of `groups` groups of neighbours (a
-// group counts by the sum of its two best choices), weights are the chosen scores over their sum (+ 1e-20), times scale.
-struct MoeGroupedRule { const float* correction; int groups, keep; float scale; };
-bool moe_route_grouped_supports(int num_experts, int top_k, const MoeGroupedRule& rule);
-int moe_route_grouped_f32(const float* logits, const MoeGroupedRule& rule, int32_t* expert_ids, float* expert_weights, int tokens, int num_experts, int top_k,
+// Scores with a correction that takes part in the choice only: sigmoids, or the softmax over all experts.  Experts of the `keep` best of
+// `groups` groups of neighbours (a group counts by the sum of its two best choices); weights are the chosen scores, over their sum
+// (+ 1e-20) unless `raw`, times scale.  The last `unlisted` experts have no rows in the sorted list.
+struct MoeCorrectedRule { const float* correction; int groups, keep; float scale; bool softmax = false, raw = false; int unlisted = 0; };
+bool moe_route_corrected_supports(int num_experts, int top_k, const MoeCorrectedRule& rule);
+int moe_route_corrected_f32(const float* logits, const MoeCorrectedRule& rule, int32_t* expert_ids, float* expert_weights, int tokens, int num_experts, int top_k,
                           hipStream_t s);
 int moe_route_topk_softmax_f32(const float* logits, int32_t* expert_ids, float* expert_weights, int tokens,
                                int num_experts, int top_k, int norm_topk_prob, hipStream_t s);
 // both of the above in one workgroup, for decode batches (≤ 1024 pairs)
 bool moe_route_sort_supports(int tokens, int num_experts, int top_k);
 int moe_route_sort_f32(const float* logits, int32_t* expert_ids, float* expert_weights, int32_t* sorted_token_ids, int32_t* block_ids, int32_t* total_post_pad,
-                       int tokens, int num_experts, int top_k, int norm_topk_prob, int block_size, hipStream_t s, const MoeGroupedRule* rule = nullptr);
+                       int tokens, int num_experts, int top_k, int norm_topk_prob, int block_size, hipStream_t s, const MoeCorrectedRule* rule = nullptr);
 int moe_align_block_size(const int32_t* expert_ids, int32_t* sorted_token_ids, int32_t* block_ids,
                          int32_t* total_post_pad, int batch_x_topk, int num_experts, int block_size,
                          int sorted_max, hipStream_t s);

@@ -70,6 +70,7 @@ struct Knobs {
     bool grouped_plain = false;       // … and the plain grouped attention kernel
     int grouped_tile_min_rows = 64;   // grouped attention: 128-row tiles from this many (token, head) rows per sequence and key head on average
     int grouped_splits = 0;           // > 0: forced KV split count of the few-row grouped attention
+    int talk_tile_min_tokens = 8;     // attention with mixed heads: portions of at least this many tokens take the tile form (0 = never)
     int linear_chunk_min_rows = 32;   // linear attention: portions of at least this many tokens in 64-token chunks (0 = never)
     // runner
     bool no_graph = false;
@@ -151,6 +152,10 @@ enum Form : int {
     FORM_SCAN_STEP,             // selective scan, every sequence brings one token
     FORM_SCAN_CHUNK,            // … portions: chunked scan
     FORM_ROUTE_GROUPED,         // sigmoid scores, best groups
+    FORM_ROUTE_SOFTMAX,         // softmax scores with a correction in the choice
+    FORM_TALK_ATTN_PLAIN,       // attention whose heads' weights are mixed: one workgroup per token, any size and number format
+    FORM_TALK_ATTN_KEYS,        // … few rows: every head against the values of all key / value heads, mixed at the end
+    FORM_TALK_ATTN_TILE,        // … portions: statistics first, then weights mixed on the matrix cores
     FORM_COUNT
 };
 

@@ -29,10 +29,16 @@ struct BatchView {
 };
 
 // ── residual stream (residual_stream.hip) ──
-// x = embed[token] (+ bigram[(prev·mul_prev + token·mul_cur) mod buckets], or the extra row for a first token), fp32; xb = E(x)
+// x = factor · embed[token] (+ bigram[(prev·mul_prev + token·mul_cur) mod buckets], or the extra row for a first token) (+ positions[position]),
+// fp32; xb = E(x)
 template <typename E>
-int embed_bigram(const E* table, const E* bigram, int buckets, int64_t mul_prev, int64_t mul_cur, const BatchView& v, float* x, E* xb,
-                 int dim, int ldb, hipStream_t s);
+struct Embedding {
+    const E *table = nullptr, *bigram = nullptr, *positions = nullptr;
+    int buckets = 0;
+    int64_t mul_prev = 0, mul_cur = 0;
+    float factor = 1.f;
+};
+template <typename E> int embed_tokens(const Embedding<E>& e, const BatchView& v, float* x, E* xb, int dim, int ldb, hipStream_t s);
 // x += sub + Σ_j weights[row][j] · pairs[row·top + j] (top 0: none); xb = E(x); sub is the sum of `slabs` partial sums
 template <typename E>
 int branch_add(const float* sub, long ld_sub, int slabs, long slab_stride, const E* pairs, long ld_pair, const float* weights, int top, float* x, E* xb,
@@ -41,8 +47,9 @@ int branch_add(const float* sub, long ld_sub, int slabs, long slab_stride, const
 template <typename E>
 int post_norm_add(const float* sub, long ld_sub, int slabs, long slab_stride, const E* gate, long ld_gate, const float* w, float mult, float eps, bool next_norm,
                   float* x, E* xb, int rows, int dim, int ldb, hipStream_t s);
-// Pre-norm blocks: x ← [x +] branch + add + Σ_j weights[row][j] · pairs[row·top + j], where the branch is sub, or with a second one the mean
-// (sub·rms⁻¹·w + sub2·rms⁻¹·w2) / 2; then out = E(rms(x) · next_w), or E(x) without next_w.  sub and sub2 are sums of `slabs` partial sums.
+// Blocks whose sublayers follow one another: x ← [keep · x +] branch + add + Σ_j weights[row][j] · pairs[row·top + j], where the branch is sub, or with a second one the mean
+// (sub·rms⁻¹·w + sub2·rms⁻¹·w2) / 2; with post_w x ← rms(x) · post_w; then out = E(rms(x) · next_w), or E(x) without next_w.  sub and sub2 are sums
+// of `slabs` partial sums, sub times sub_scale[row]; pairs with an id of pair_limit or more stand for the stream itself (post_w only).
 template <typename E>
 struct StreamUpdate {
     // sub null: zero
@@ -50,8 +57,11 @@ struct StreamUpdate {
     const float *w = nullptr, *w2 = nullptr;      // norms of the two branches (with sub2)
     const float* add = nullptr;                   // a vector for every row
     const E* pairs = nullptr; long ld_pair = 0; const float* weights = nullptr; int top = 0;
+    const int32_t* pair_ids = nullptr; int pair_limit = 0;
+    const E* sub_scale = nullptr; long ld_scale = 0;
     bool replace = false;                         // x ← branch + add
-    const float* next_w = nullptr;
+    float keep = 1.f;
+    const float *post_w = nullptr, *next_w = nullptr;
     float eps = 0.f;
     float* x = nullptr; E* out = nullptr; long ldo = 0;     // out null: the last update of a forward
     int rows = 0, dim = 0;
@@ -108,7 +118,7 @@ constexpr int LATENT_TILE_TOKENS = 128;          // tokens of a portion per work
 bool latent_expanded_supports(const LatentDims& d);
 int latent_attention_expanded(const LatentDims& d, const LatentBuffers<bf16>& b, const BatchView& v, const LatentExpanded& x, hipStream_t s);
 
-// ── grouped attention (grouped_attention.hip) ──
+// ── grouped attention (grouped_attention.hip, talking_attention.hip) ──
 // Keys and values of a layer: per block and key / value head [dp / 8 chunks][16 tokens][8] and, for the values, [vp / 32][4 token quads]
 // [16 dims][2 halves][4 tokens]: both products' operands are contiguous loads.  Heads are padded with zeros to dp, vp.
 struct GroupedDims { int heads, kv_heads, dim, vdim, dp, vp, rot_dims, window; float scale; };
@@ -120,17 +130,25 @@ struct GroupedBuffers {
     const float *cos_t = nullptr, *sin_t = nullptr;   // [positions][rot_dims / 2]
     E *k_pool = nullptr, *v_pool = nullptr;
     const E *q_in = nullptr, *k_in = nullptr, *v_in = nullptr; long ld = 0;      // columns of the fused projection
-    const float *q_norm = nullptr, *k_norm = nullptr;     // [heads·dp], [kv_heads·dp]
+    const float *q_norm = nullptr, *k_norm = nullptr;     // [heads·dp], [kv_heads·dp]; norms of one head each: [dp]
+    bool head_norm = false;                               // one root mean square per head instead of one for all
     float eps = 0.f;
     E* q = nullptr;                                   // [T][heads][dp]: normed and rotated
     const E* gate = nullptr; long ld_gate = 0;        // [T][heads]: factor per head; null: none
+    const E* value_gate = nullptr; long ld_value_gate = 0;       // [T][heads·vp]: factor per element; null: none
     float mult = 1.f;                                 // factor of the result
+    const float *r1 = nullptr, *r2 = nullptr;         // [heads]: scores lose r1 · ln(1 + r2 · distance); null: none
+    const float* sink = nullptr;                      // [heads]: score-like numbers that take part in the denominator only; null: none
+    const float* talk = nullptr;                      // [heads][heads]: weight_h = Σ_g talk[h][g] · weight_g ahead of the values; null: none
     E* out = nullptr; long ldo = 0;
     float* partial = nullptr; size_t partial_bytes = 0;
 };
-// norms, rotation, cache write
+// norms, rotation, cache write (k_in null: another layer caches the keys and values)
 template <typename E> int grouped_prepare(const GroupedDims& d, const GroupedBuffers<E>& b, const BatchView& v, hipStream_t s);
 template <typename E> int grouped_attention(const GroupedDims& d, const GroupedBuffers<E>& b, const BatchView& v, hipStream_t s);
+// … with mixed heads (talk); grouped_attention takes these launches there
+template <typename E> int talking_attention(const GroupedDims& d, const GroupedBuffers<E>& b, const BatchView& v, hipStream_t s);
+size_t talking_partial_bytes(const GroupedDims& d);      // scratch for split keys
 
 // ── linear attention with decay (linear_attention.hip) ──
 // Per head S ← diag(decay) S + k vᵀ, o = Sᵀ q; o over its root mean square (· norm), · gate · mult.  The state is fp32 [slots][heads][dp][vp].

@@ -24,6 +24,11 @@
 //     selective scan   : [x | z silu] → convolution silu → [dt rank | B | C] → dt softplus → scan × z → W_o
 //     feed-forward     : (gate, up) pairs → y → down, or experts of that form behind a grouped router
 // A range of its layers may run several times in a row, each pass with caches and states of its own.
+// Post-norm block: x ← norm1(α x + mixer(x)), x ← norm2(α x + ff(x)): the same sublayers behind the same projections, which read x itself; the
+// kernel that adds a sublayer's result norms the sum.
+//     attention        : [q | k | v | value gates σ] → norms per head, cache write → attention, its heads mixed or not → W_o
+//     experts          : corrected softmax router → experts of clamped gates; those past the last one hand x on, inside the sum; beside them
+//                        [(gate, up) pairs → y | factor σ] → down of the shared expert, times its factor in the sum
 #include <math.h>
 
 #include <algorithm>
@@ -48,6 +53,7 @@ void store(bf16* dst, float f) { const uint16_t h = bf16_bits(f); memcpy(dst, &h
 void store(float* dst, float f) { *dst = f; }
 
 constexpr int MOE_MAX_BLOCK = 256;
+constexpr float GLU_SLOPE = 1.702f;              // of the clamped GLUs' sigmoid
 
 struct HostTensor { std::vector<float> data; std::vector<int64_t> shape; };
 
@@ -109,13 +115,14 @@ class Layered final : public LayeredModel {
         int c_glu = -1, c_att = -1;        // parallel block: columns of the feed-forward's gated product and, behind it, of the attention's result
         float *norm1 = nullptr, *norm2 = nullptr;
         float g2 = 1.f;
-        Linear router, up, side_gate, side_proj;
+        Linear router, up, side_gate, side_proj, shared_in, shared_down;
+        GemmSection shared_sec[2];
         E* side_table = nullptr;
         float* side_norm = nullptr;
         // pre-norm block: the second mixer's W_o where its result is normed by itself, and the two norms
         Linear o2, decay, conv_in, dt;
-        float *out1 = nullptr, *out2 = nullptr, *down_bias = nullptr, *correction = nullptr;
-        int c_v = 0, c_q2 = 0, c_k2 = 0, c_v2 = 0, c_g2 = 0, c_rank = 0;
+        float *out1 = nullptr, *out2 = nullptr, *down_bias = nullptr, *correction = nullptr, *o_bias = nullptr;
+        int c_v = 0, c_q2 = 0, c_k2 = 0, c_v2 = 0, c_g2 = 0, c_rank = 0, c_gate = 0;
         GroupedDims gd{};
         LinearDims nd{};
         ScanDims sd{};
@@ -165,12 +172,13 @@ public:
         // embedding table (gather) and the same table as vocabulary projection; bigram table
         FH_TRY(table("embed", c_.vocab, &embed_));
         if (lc_.bigram_buckets > 0) FH_TRY(table("bigram", lc_.bigram_buckets + 1, &bigram_));
+        if (lc_.position_rows > 0) FH_TRY(table("pos", lc_.position_rows, &positions_));
         FH_TRY(pack(&head_, {{lc_.untied_head ? "head" : "embed", 0, c_.vocab, pad32(c_.vocab)}}, D_));
         if (parallel()) {
             float g = 1.f;
             FH_TRY(scalar("final.norm", &g));
             FH_TRY(arena_.upload(&final_norm_, std::vector<float>(pad32(D_), g)));
-        } else if (pre_norm()) {
+        } else if (in_turn()) {
             FH_TRY(vec("final.norm", {D_}, pad32(D_), &final_norm_));
         } else {
             FH_TRY(unit_offset("final.norm", &final_norm_));
@@ -195,7 +203,7 @@ public:
             if (parallel()) {
                 FH_TRY(scalar(p + "norm1", &g1));
                 if (sp.ff != FERRUM_HIP_FF_NONE) FH_TRY(scalar(p + "norm2", &L.g2));
-            } else if (pre_norm()) {
+            } else if (in_turn()) {
                 FH_TRY(vec(p + "norm1", {D_}, Dp_, &L.norm1));
                 if (sp.ff != FERRUM_HIP_FF_NONE) FH_TRY(vec(p + "norm2", {D_}, Dp_, &L.norm2));
             } else {
@@ -211,13 +219,14 @@ public:
                 if (d.q_rank) q_cols = std::max<long>(q_cols, L.uq.n);
                 // split attention: (row tile, split) pairs stay below 1024
                 partial = std::max<size_t>(partial, (size_t)1024 * 16 * (d.kp + 4) * 4);
-            } else if (pre_norm()) {
+            } else if (in_turn()) {
                 if (sp.mixer == FERRUM_HIP_MIXER_SELECTIVE_SCAN) FH_TRY(scan_weights(L, in, p + "mix.", li));
                 else FH_TRY(pair_weights(L, in, p + "mix.", li));
                 attn_cols = std::max<long>(attn_cols, L.o.k + L.o2.k);
                 if (L.gd.heads) {
                     q_cols = std::max<long>(q_cols, (long)L.gd.heads * L.gd.dp);
                     partial = std::max<size_t>(partial, (size_t)1024 * 16 * (L.gd.vp + 4) * 4);
+                    if (sp.attn_flags & FERRUM_HIP_ATTN_TALK) partial = std::max(partial, talking_partial_bytes(L.gd));
                 }
                 decay_cols = std::max<long>(decay_cols, L.decay.n);
                 if (L.nd.heads) {
@@ -245,13 +254,13 @@ public:
                 if (L.c_att >= 0) L.ld_in = (int)std::max<long>(L.ld_in, L.c_att + att);
                 else attn_cols = std::max(attn_cols, att);
             }
-            in_cols = std::max<long>({in_cols, L.ld_in, L.ff_in.n});
+            in_cols = std::max<long>({in_cols, L.ld_in, L.ff_in.n, L.shared_in.n});
             if (moe(sp)) {
                 const size_t n = T * sp.top;
                 pairs = std::max(pairs, n);
                 sorted = std::max(sorted, n + (size_t)MOE_MAX_BLOCK * (std::min<size_t>(sp.experts, n) + 1));
                 expert_cols = std::max(expert_cols, n * (size_t)L.down.k);
-                logit_cols = std::max<size_t>(logit_cols, sp.experts);
+                logit_cols = std::max<size_t>(logit_cols, sp.experts + sp.identity_experts);
             }
             if (lc_.token_side_dim) {
                 FH_TRY(side_weights(L, p, li));
@@ -312,8 +321,12 @@ public:
         run.any_short = plan_expansion(&run.short_view);
         if (run.short_view.long_min > 0)
             FH_CHECK_HIP(hipMemcpyAsync(plan_dev_, plan_host_, plan_used_ * 4, hipMemcpyHostToDevice, s));
-        RUN(embed_bigram<E>(embed_, bigram_, lc_.bigram_buckets, lc_.bigram_mul_prev, lc_.bigram_mul_cur, v, x_, xb_, D_, Dp_, s));
-        if (pre_norm()) return pre_norm_forward(run, taps);
+        Embedding<E> e;
+        e.table = embed_; e.bigram = bigram_; e.positions = positions_;
+        e.buckets = lc_.bigram_buckets; e.mul_prev = lc_.bigram_mul_prev; e.mul_cur = lc_.bigram_mul_cur;
+        if (lc_.embed_scale != 0.f) e.factor = lc_.embed_scale;
+        RUN(embed_tokens<E>(e, v, x_, xb_, D_, Dp_, s));
+        if (in_turn()) return in_turn_forward(run, taps);
         if (parallel()) RUN(rms_norm_rows<E>(x_, nullptr, nullptr, c_.rms_eps, xb_, v.T, D_, Dp_, s));
         for (run.li = 0; run.li < c_.num_layers; run.li++) {
             Layer& L = layers_[run.li];
@@ -327,6 +340,7 @@ public:
         FH_TRY(rms_norm_rows<E>(x_, row_idx, final_norm_, c_.rms_eps, head_in_, rows, D_, Dp_, s));
         TiledGemm<E> g = linear_f32(head_, head_in_, Dp_, rows, logits, c_.vocab);
         g.n_store = c_.vocab;
+        if (lc_.logit_softcap > 0.f) { g.nsec = 1; g.sec[0] = {0, GEMM_ACT_SOFTCAP, lc_.logit_softcap, 0}; }
         return tiled_gemm(g, s);
     }
 
@@ -364,17 +378,8 @@ private:
         const bool moe = L.s.ff == FERRUM_HIP_FF_MOE_RELU2, last = run.li + 1 == c_.num_layers;
         int slabs = 1;
         // few tokens: the experts, bound by their weights' bytes, beside the mixer, bound by the latency of its chain of launches
-        const bool beside = moe && T <= knobs().layer_overlap_max_tokens && !run.trace;
-        if (beside) {
-            Run other = run;
-            other.s = side_stream_;
-            FH_CHECK_HIP(hipEventRecord(fork_, s));
-            FH_CHECK_HIP(hipStreamWaitEvent(side_stream_, fork_, 0));
-            FH_TRY(experts(L, other));
-            FH_CHECK_HIP(hipEventRecord(join_, side_stream_));
-        } else if (moe) {
-            FH_TRY(experts(L, run));
-        }
+        const bool beside = moe && few_tokens(run);
+        if (moe) FH_TRY(beside ? experts_beside(L, run) : experts(L, run));
         RUN(tiled_gemm(input_projection(L, T), s));
         E* att = L.c_att >= 0 ? in_ + L.c_att : attn_;
         const long ld_att = L.c_att >= 0 ? L.ld_in : (long)L.ld.heads * L.ld.vp;
@@ -408,13 +413,13 @@ private:
     }
     bool opens_pass(const LayerRun& r) const { return r.pass >= 0 && r.layer == lc_.loop_start; }
 
-    int pre_norm_forward(Run& run, float* taps) {
+    int in_turn_forward(Run& run, float* taps) {
         const int T = run.v.T;
         hipStream_t s = run.s;
         const std::vector<LayerRun> runs = order();
         if (loops()) RUN(copy_rows<E>(xb_, Dp_, cat_ + Dp_, 2 * Dp_, T, Dp_, s));
         if (opens_pass(runs[0])) RUN(copy_rows<E>(xb_, Dp_, cat_, 2 * Dp_, T, Dp_, s));
-        else RUN(rms_norm_rows<E>(x_, nullptr, layers_[0].norm1, c_.rms_eps, xb_, T, D_, Dp_, s));
+        else if (pre_norm()) RUN(rms_norm_rows<E>(x_, nullptr, layers_[0].norm1, c_.rms_eps, xb_, T, D_, Dp_, s));
         for (size_t i = 0; i < runs.size(); i++) {
             run.li = runs[i].layer;
             if (opens_pass(runs[i])) {
@@ -429,8 +434,8 @@ private:
             StreamUpdate<E> next = update(T);
             if (i + 1 == runs.size()) next.out = nullptr;
             else if (opens_pass(runs[i + 1])) { next.out = cat_; next.ldo = 2 * Dp_; }
-            else next.next_w = layers_[runs[i + 1].layer].norm1;
-            FH_TRY(pre_norm_layer(layers_[run.li], std::max(runs[i].pass, 0), run, next));
+            else if (pre_norm()) next.next_w = layers_[runs[i + 1].layer].norm1;
+            FH_TRY(in_turn_layer(layers_[run.li], std::max(runs[i].pass, 0), run, next));
             if (taps) FH_CHECK_HIP(hipMemcpyAsync(taps + i * c_.max_tokens * D_, x_, (size_t)T * D_ * 4, hipMemcpyDeviceToDevice, s));
         }
         return 0;
@@ -442,12 +447,15 @@ private:
         return u;
     }
 
-    int pre_norm_layer(Layer& L, int pass, const Run& run, const StreamUpdate<E>& next) {
+    // `next`: the layer's last update, up to what it adds
+    int in_turn_layer(Layer& L, int pass, const Run& run, const StreamUpdate<E>& next) {
         const int T = run.v.T;
         hipStream_t s = run.s;
         const bool ff = L.s.ff != FERRUM_HIP_FF_NONE;
         StreamUpdate<E> u = ff ? update(T) : next;
-        if (ff) u.next_w = L.norm2;
+        if (post_norm()) { u.post_w = L.norm1; u.keep = lc_.stream_mult; }
+        else if (ff) u.next_w = L.norm2;
+        u.add = L.o_bias;
         RUN(tiled_gemm(input_projection(L, T), s));
         if (L.sd.wp) {
             ScanBuffers<E>& b = L.sb[pass];
@@ -483,10 +491,23 @@ private:
         RUN(stream_update(u, s));
         if (!ff) return 0;
         StreamUpdate<E> f = next;
+        if (post_norm()) { f.post_w = L.norm2; f.keep = lc_.stream_mult; }
         if (moe(L.s)) {
-            FH_TRY(experts(L, run));
+            // few tokens: the experts beside the shared one
+            const bool shared = L.s.shared_width > 0, beside = shared && few_tokens(run);
+            FH_TRY(beside ? experts_beside(L, run) : experts(L, run));
             f.sub = nullptr;
             f.pairs = expert_y_; f.weights = expert_weights_; f.top = L.s.top;
+            if (L.s.identity_experts) { f.pair_ids = expert_ids_; f.pair_limit = L.s.experts; }
+            if (shared) {
+                TiledGemm<E> g = linear(L.shared_in, xb_, Dp_, T, in_, L.shared_in.n);
+                g.nsec = 2; g.sec[0] = L.shared_sec[0]; g.sec[1] = L.shared_sec[1];
+                RUN(tiled_gemm(g, s));
+                RUN(tiled_gemm(linear_slabs(L.shared_down, in_, L.shared_in.n, T, &f.slabs), s));
+                f.sub = sub_;
+                f.sub_scale = in_ + L.shared_sec[1].begin; f.ld_scale = L.shared_in.n;
+            }
+            if (beside) FH_CHECK_HIP(hipStreamWaitEvent(s, join_, 0));
         } else {
             TiledGemm<E> g = linear(L.ff_in, xb_, Dp_, T, in_, L.down.k);
             g.nsec = 1; g.sec[0] = L.ff_sec[0];
@@ -528,23 +549,41 @@ private:
         return 0;
     }
 
-    // expert_y_ [T·top][Dp] and expert_weights_ [T·top] of the chosen experts
+    bool few_tokens(const Run& run) const { return run.v.T <= knobs().layer_overlap_max_tokens && !run.trace; }
+    // the experts on a stream of their own; join_ is recorded behind them
+    int experts_beside(Layer& L, const Run& run) {
+        Run other = run;
+        other.s = side_stream_;
+        FH_CHECK_HIP(hipEventRecord(fork_, run.s));
+        FH_CHECK_HIP(hipStreamWaitEvent(side_stream_, fork_, 0));
+        FH_TRY(experts(L, other));
+        FH_CHECK_HIP(hipEventRecord(join_, side_stream_));
+        return 0;
+    }
+    // how a layer's router scores and chooses, beyond the softmax over the chosen logits
+    static MoeCorrectedRule route_rule(const FerrumHipLayerSpec& s, const float* correction) {
+        MoeCorrectedRule r{correction, s.route_groups, s.route_keep, s.route_scale};
+        r.softmax = r.raw = s.ff == FERRUM_HIP_FF_MOE_CLAMPED_GLU;
+        r.unlisted = s.identity_experts;
+        return r;
+    }
+    // expert_y_ [T·top][Dp], expert_weights_ and expert_ids_ [T·top] of the chosen experts
     int experts(Layer& L, const Run& run) {
-        const int T = run.v.T, E_ = L.s.experts, pairs = T * L.s.top;
+        const int T = run.v.T, E_ = L.s.experts, routed = E_ + L.s.identity_experts, pairs = T * L.s.top;
         hipStream_t s = run.s;
-        TiledGemm<E> z = linear_f32(L.router, xb_, Dp_, T, router_logits_, E_);
-        z.n_store = E_; z.nsec = 1; z.sec[0] = {0, GEMM_ACT_NONE, 0, 0, L.g2};
+        TiledGemm<E> z = linear_f32(L.router, xb_, Dp_, T, router_logits_, routed);
+        z.n_store = routed; z.nsec = 1; z.sec[0] = {0, GEMM_ACT_NONE, 0, 0, L.g2};
         RUN(tiled_gemm(z, s));
         GemmRows rows;
         rows.block = moe_block(pairs, E_);
         rows.max_blocks = std::min(pairs, pairs / rows.block + std::min(E_, pairs));
         rows.id = sorted_; rows.group = sorted_expert_; rows.total = sorted_total_;
-        const bool grouped = L.s.ff == FERRUM_HIP_FF_MOE_SILU_GLU;
-        const MoeGroupedRule rule{L.correction, L.s.route_groups, L.s.route_keep, L.s.route_scale};
-        if (moe_route_sort_supports(T, E_, L.s.top)) {
-            RUN(moe_route_sort_f32(router_logits_, expert_ids_, expert_weights_, sorted_, sorted_expert_, sorted_total_, T, E_, L.s.top, 1, rows.block, s, grouped ? &rule : nullptr));
-        } else if (grouped) {
-            RUN(moe_route_grouped_f32(router_logits_, rule, expert_ids_, expert_weights_, T, E_, L.s.top, s));
+        const bool corrected = L.s.ff != FERRUM_HIP_FF_MOE_RELU2;
+        const MoeCorrectedRule rule = route_rule(L.s, L.correction);
+        if (moe_route_sort_supports(T, routed, L.s.top)) {
+            RUN(moe_route_sort_f32(router_logits_, expert_ids_, expert_weights_, sorted_, sorted_expert_, sorted_total_, T, routed, L.s.top, 1, rows.block, s, corrected ? &rule : nullptr));
+        } else if (corrected) {
+            RUN(moe_route_corrected_f32(router_logits_, rule, expert_ids_, expert_weights_, T, routed, L.s.top, s));
             RUN(moe_align_block_size(expert_ids_, sorted_, sorted_expert_, sorted_total_, pairs, E_, rows.block, rows.max_blocks * rows.block, s));
         } else {
             RUN(moe_route_topk_softmax_f32(router_logits_, expert_ids_, expert_weights_, T, E_, L.s.top, 1, s));
@@ -552,7 +591,7 @@ private:
         }
         TiledGemm<E> u = linear(L.up, xb_, Dp_, pairs, expert_h_, L.down.k);
         u.groups = 1; u.rows = rows; u.rows.div = L.s.top;
-        u.nsec = 1; u.sec[0] = {0, grouped ? GEMM_ACT_SILU_GLU : GEMM_ACT_RELU2, 0, 0, L.g2};
+        u.nsec = 1; u.sec[0] = L.ff_sec[0];
         RUN(tiled_gemm(u, s));
         TiledGemm<E> y = linear(L.down, expert_h_, L.down.k, pairs, expert_y_, Dp_);
         y.groups = 1; y.rows = rows;
@@ -574,7 +613,7 @@ private:
                     latent_pad_rank(s.kv_rank), pad32(s.q_rank), latent_pad_head(s.dim, s.vdim, s.vdim), s.window == FERRUM_HIP_WINDOW_NONE ? LATENT_NO_WINDOW : s.window, s.scale};
         else if (s.mixer == FERRUM_HIP_MIXER_SELECTIVE_SCAN)
             L.sd = {pad32(s.scan_inner), s.scan_state, scan_pad_state(s.scan_state), pad32(s.scan_state)};
-        else if (lc_.block == FERRUM_HIP_BLOCK_PRE_NORM) {
+        else if (in_turn()) {
             if (s.mixer == FERRUM_HIP_MIXER_GROUPED_ATTENTION)
                 L.gd = {s.heads, s.kv_heads, s.dim, s.vdim, grouped_pad_head(s.dim, s.vdim, s.dim), grouped_pad_head(s.dim, s.vdim, s.vdim), s.rot_dims,
                         s.window == FERRUM_HIP_WINDOW_NONE ? LATENT_NO_WINDOW : s.window, s.scale};
@@ -677,9 +716,11 @@ private:
     // ── weights ──
     bool parallel() const { return lc_.block == FERRUM_HIP_BLOCK_PARALLEL_PRE_NORM; }
     bool pre_norm() const { return lc_.block == FERRUM_HIP_BLOCK_PRE_NORM; }
+    bool post_norm() const { return lc_.block == FERRUM_HIP_BLOCK_POST_NORM; }
+    bool in_turn() const { return pre_norm() || post_norm(); }       // plain sublayers one after the other
     bool loops() const { return lc_.loop_times > 0; }
     int passes(int li) const { return loops() && li >= lc_.loop_start && li < lc_.loop_stop ? lc_.loop_times : 1; }
-    static bool moe(const FerrumHipLayerSpec& s) { return s.ff == FERRUM_HIP_FF_MOE_RELU2 || s.ff == FERRUM_HIP_FF_MOE_SILU_GLU; }
+    static bool moe(const FerrumHipLayerSpec& s) { return s.ff == FERRUM_HIP_FF_MOE_RELU2 || s.ff == FERRUM_HIP_FF_MOE_SILU_GLU || s.ff == FERRUM_HIP_FF_MOE_CLAMPED_GLU; }
     // the layer's linear attention: its second mixer, or its only one
     static int linear_mixer(const FerrumHipLayerSpec& s) {
         return s.mixer2 ? s.mixer2 : s.mixer == FERRUM_HIP_MIXER_GATED_LINEAR || s.mixer == FERRUM_HIP_MIXER_RETENTION ? s.mixer : 0;
@@ -816,8 +857,10 @@ private:
         if (g.heads) {
             const bool biased = sp.attn_flags & FERRUM_HIP_ATTN_QKV_BIAS;
             L.c0 = heads(a + "q", g.heads, g.dim, g.dp, biased);
-            L.c1 = heads(a + "k", g.kv_heads, g.dim, g.dp, biased);
-            L.c_v = heads(a + "v", g.kv_heads, g.vdim, g.vp, biased);
+            if (!sp.kv_source) {
+                L.c1 = heads(a + "k", g.kv_heads, g.dim, g.dp, biased);
+                L.c_v = heads(a + "v", g.kv_heads, g.vdim, g.vp, biased);
+            }
         }
         if (lin) {
             L.c_q2 = heads(r + "q", n.heads, n.dim, n.dp, false);
@@ -832,6 +875,10 @@ private:
             L.c2 = section(L, in, GEMM_ACT_SIGMOID);
             in.add(a + "g", 0, g.heads, pad32(g.heads));
         }
+        if (g.heads && sp.attn_flags & FERRUM_HIP_ATTN_VALUE_GATE) {
+            section(L, in, GEMM_ACT_SIGMOID);
+            L.c_gate = heads(a + "g", g.heads, g.vdim, g.vp, false);
+        }
         if (lin) {
             section(L, in, GEMM_ACT_SILU);
             L.c_g2 = heads(r + "g", n.heads, n.vdim, n.vp, false);
@@ -839,10 +886,26 @@ private:
         GroupedBuffers<E> gb;
         LinearBuffers<E> nb;
         if (g.heads) {
-            float *qn = nullptr, *kn = nullptr;
-            FH_TRY(head_vec(a + "q.norm", g.heads, g.dim, g.dp, &qn));
-            FH_TRY(head_vec(a + "k.norm", g.kv_heads, g.dim, g.dp, &kn));
+            float *qn = nullptr, *kn = nullptr, *v = nullptr;
+            gb.head_norm = sp.attn_flags & FERRUM_HIP_ATTN_HEAD_NORM;
+            FH_TRY(head_vec(a + "q.norm", gb.head_norm ? 1 : g.heads, g.dim, g.dp, &qn));
+            if (!sp.kv_source) FH_TRY(head_vec(a + "k.norm", gb.head_norm ? 1 : g.kv_heads, g.dim, g.dp, &kn));
             gb.q_norm = qn; gb.k_norm = kn; gb.eps = c_.rms_eps;
+            if (sp.attn_flags & FERRUM_HIP_ATTN_LOG_DISTANCE) {
+                FH_TRY(vec(a + "r1", {g.heads}, g.heads, &v, 0.5f));
+                gb.r1 = v;
+                FH_TRY(vec(a + "r2", {g.heads}, g.heads, &v, 0.1f));
+                gb.r2 = v;
+            }
+            if (sp.attn_flags & FERRUM_HIP_ATTN_SINK) {
+                FH_TRY(vec(a + "sink", {g.heads}, g.heads, &v, 0.f));
+                gb.sink = v;
+            }
+            if (sp.attn_flags & FERRUM_HIP_ATTN_TALK) {
+                FH_TRY(matrix(a + "talk", g.heads, g.heads, g.heads, &v));
+                gb.talk = v;
+            }
+            if (sp.attn_flags & FERRUM_HIP_ATTN_OUT_BIAS) FH_TRY(vec(a + "o.b", {D_}, Dp_, &L.o_bias, 0.f));
             gb.mult = both && !normed ? sp.left_scale : 1.f;
             if (g.rot_dims) FH_TRY(rope(sp.rot_dims, sp.rot_base, sp, &gb.cos_t, &gb.sin_t));
             FH_TRY(need(a + "o", {D_, (int64_t)g.heads * g.vdim}));
@@ -890,7 +953,11 @@ private:
             FH_TRY(vec(m + "right.out", {D_}, Dp_, &L.out2));
         }
         for (int t = 0; t < np; t++) {
-            if (g.heads) {
+            if (g.heads && sp.kv_source) {
+                gb.k_pool = layers_[sp.kv_source - 1].gb[0].k_pool;
+                gb.v_pool = layers_[sp.kv_source - 1].gb[0].v_pool;
+                L.gb.push_back(gb);
+            } else if (g.heads) {
                 FH_TRY(arena_.alloc(&gb.k_pool, (size_t)c_.kv_num_blocks * grouped_k_elems(g)));
                 FH_TRY(arena_.alloc(&gb.v_pool, (size_t)c_.kv_num_blocks * grouped_v_elems(g)));
                 L.gb.push_back(gb);
@@ -940,11 +1007,13 @@ private:
         }
         return 0;
     }
-    // the activations that the pre-norm block's kernels read and write
+    // the activations that the kernels of blocks with sublayers in turn read and write
     void wire(Layer& L) {
         const long ld = L.o.k + L.o2.k;
         for (GroupedBuffers<E>& b : L.gb) {
-            b.q_in = in_ + L.c0; b.k_in = in_ + L.c1; b.v_in = in_ + L.c_v; b.ld = L.ld_in;
+            b.q_in = in_ + L.c0; b.ld = L.ld_in;
+            if (!L.s.kv_source) { b.k_in = in_ + L.c1; b.v_in = in_ + L.c_v; }
+            if (L.s.attn_flags & FERRUM_HIP_ATTN_VALUE_GATE) { b.value_gate = in_ + L.c_gate; b.ld_value_gate = L.ld_in; }
             b.q = q_; b.out = attn_; b.ldo = ld; b.partial = partial_; b.partial_bytes = partial_bytes_;
             if (!(L.s.attn_flags & FERRUM_HIP_ATTN_NO_HEAD_GATE)) { b.gate = in_ + L.c2; b.ld_gate = L.ld_in; }
         }
@@ -976,7 +1045,7 @@ private:
             L.ff_sec[1] = {Dp_, GEMM_ACT_XIELU, (float)softplus(act ? act[0] : 0.5f), (float)softplus(act ? act[1] : 0.5f)};
         } else if (sp.ff == FERRUM_HIP_FF_CLAMPED_GLU) {
             // 16 gate columns, their 16 up columns, and so on; the down projection is part of the projection out
-            L.c_glu = section(L, in, GEMM_ACT_CLAMPED_GLU, L.g2, sp.ff_limit, 1.702f);
+            L.c_glu = section(L, in, GEMM_ACT_CLAMPED_GLU, L.g2, sp.ff_limit, GLU_SLOPE);
             for (int f = 0; f < Fp; f += 16)
                 for (const char* part : {"mlp.gate", "mlp.up"}) {
                     const int n = std::min(16, F - f);
@@ -995,9 +1064,22 @@ private:
             L.ff_sec[0] = {0, GEMM_ACT_GELU_GLU, 0, 0};
             FH_TRY(pack(&L.down, {{p + "mlp.down", 0, D_, Dp_}}, F));
             FH_TRY(vec(p + "mlp.down.b", {D_}, Dp_, &L.down_bias, 0.f));
-        } else if (sp.ff == FERRUM_HIP_FF_MOE_SILU_GLU) {
-            FH_TRY(pack(&L.router, {{p + "mlp.router", 0, sp.experts, pad32(sp.experts)}}, D_));
-            FH_TRY(vec(p + "mlp.correction", {sp.experts}, sp.experts, &L.correction, 0.f));
+        } else if (sp.ff == FERRUM_HIP_FF_MOE_SILU_GLU || sp.ff == FERRUM_HIP_FF_MOE_CLAMPED_GLU) {
+            const int routed = sp.experts + sp.identity_experts;
+            FH_TRY(pack(&L.router, {{p + "mlp.router", 0, routed, pad32(routed)}}, D_));
+            FH_TRY(vec(p + "mlp.correction", {routed}, routed, &L.correction, 0.f));
+            L.ff_sec[0] = sp.ff == FERRUM_HIP_FF_MOE_SILU_GLU ? GemmSection{0, GEMM_ACT_SILU_GLU, 0, 0, L.g2} : GemmSection{0, GEMM_ACT_CLAMPED_GLU, sp.ff_limit, GLU_SLOPE, L.g2};
+            if (const int S = sp.shared_width; S > 0) {
+                const std::string x = p + "mlp.shared.";
+                Input f;
+                for (int c = 0; c < pad32(S); c += 16)
+                    for (const char* part : {"gate", "up"}) f.add(x + part, c < S ? c : 0, std::max(std::min(16, S - c), 0), 16);
+                L.shared_sec[0] = {0, GEMM_ACT_CLAMPED_GLU, sp.shared_limit, GLU_SLOPE};
+                L.shared_sec[1] = {f.cols(), GEMM_ACT_SIGMOID, 0, 0};
+                f.add(x + "sg", 0, 1, 32);
+                FH_TRY(pack(&L.shared_in, f.rows, D_));
+                FH_TRY(pack(&L.shared_down, {{x + "down", 0, D_, Dp_}}, S));
+            }
             std::vector<const float*> gate, up, down;
             for (int e = 0; e < sp.experts; e++) {
                 const std::string x = p + "mlp.e" + std::to_string(e) + ".";
@@ -1016,6 +1098,7 @@ private:
             std::vector<Rows> r = {{p + "mlp.router", 0, sp.experts, pad32(sp.experts)}};
             FH_TRY(pack(&L.router, r, D_));
             FH_TRY(bias(&L.router, r, {p + "mlp.router.b"}));
+            L.ff_sec[0] = {0, GEMM_ACT_RELU2, 0, 0, L.g2};
             std::vector<const float*> up, down;
             for (int e = 0; e < sp.experts; e++) {
                 const std::string x = p + "mlp.e" + std::to_string(e) + ".";
@@ -1218,7 +1301,7 @@ private:
     Linear head_, loop_in_;
     float *loop_step_ = nullptr, *sub2_ = nullptr;
     E* cat_ = nullptr;           // [T][stream | embedding], ahead of a pass
-    E *embed_ = nullptr, *bigram_ = nullptr;
+    E *embed_ = nullptr, *bigram_ = nullptr, *positions_ = nullptr;
     float* final_norm_ = nullptr;
     // activations of one forward
     float *x_ = nullptr, *sub_ = nullptr, *partial_ = nullptr, *decay_ = nullptr, *drive_ = nullptr, *chunk_a_ = nullptr, *chunk_h_ = nullptr;
@@ -1237,7 +1320,10 @@ private:
 
 }  // namespace
 
-static int check_pre_norm_layer(const FerrumHipLayerSpec& s, int i) {
+// a layer of a block whose sublayers follow one another (pre-norm, post-norm)
+static int check_in_turn_layer(const FerrumHipLayeredConfig& lc, const FerrumHipLayerSpec* layers, int i) {
+    const FerrumHipLayerSpec& s = layers[i];
+    const bool post = lc.block == FERRUM_HIP_BLOCK_POST_NORM;
     auto rotated = [](int dims, int of, double base) { return dims >= 0 && dims % 2 == 0 && dims <= of && (dims == 0 || base > 0.0); };
     const bool attention = s.mixer == FERRUM_HIP_MIXER_GROUPED_ATTENTION;
     const int lin = s.mixer2 ? s.mixer2 : attention || s.mixer == FERRUM_HIP_MIXER_SELECTIVE_SCAN ? 0 : s.mixer;
@@ -1251,7 +1337,16 @@ static int check_pre_norm_layer(const FerrumHipLayerSpec& s, int i) {
         FH_REQUIRE(s.heads > 0 && s.kv_heads > 0 && s.heads % s.kv_heads == 0 && s.dim > 0 && s.vdim > 0 && (s.window > 0 || s.window == FERRUM_HIP_WINDOW_NONE),
                    "layer %d: attention of %d heads on %d, %d / %d dimensions, window %d", i, s.heads, s.kv_heads, s.dim, s.vdim, s.window);
         FH_REQUIRE(rotated(s.rot_dims, s.dim, s.rot_base) && s.rot_factor == 0.0, "layer %d: rotated dimensions %d of %d", i, s.rot_dims, s.dim);
-        FH_REQUIRE(!(s.attn_flags & FERRUM_HIP_ATTN_SINK), "layer %d: grouped attention has no sinks", i);
+        FH_REQUIRE(!(s.attn_flags & FERRUM_HIP_ATTN_VALUE_GATE) || s.attn_flags & FERRUM_HIP_ATTN_NO_HEAD_GATE, "layer %d: gates per head and per value element share a tensor name", i);
+        FH_REQUIRE(!(s.attn_flags & FERRUM_HIP_ATTN_TALK) || !(s.attn_flags & FERRUM_HIP_ATTN_LOG_DISTANCE), "layer %d: mixed heads take scores without a distance", i);
+        FH_REQUIRE(!s.mixer2 || !(s.attn_flags & (FERRUM_HIP_ATTN_VALUE_GATE | FERRUM_HIP_ATTN_OUT_BIAS)), "layer %d: value gates and output bias beside a second mixer", i);
+        if (s.kv_source) {
+            FH_REQUIRE(s.kv_source > 0 && s.kv_source <= i && !lc.loop_times && !s.mixer2 && s.attn_flags & FERRUM_HIP_ATTN_HEAD_NORM, "layer %d: reads the keys of layer %d", i,
+                       s.kv_source - 1);
+            const FerrumHipLayerSpec& o = layers[s.kv_source - 1];
+            FH_REQUIRE(o.mixer == s.mixer && !o.kv_source && o.kv_heads == s.kv_heads && o.dim == s.dim && o.vdim == s.vdim,
+                       "layer %d: layer %d caches other keys, or none of its own", i, s.kv_source - 1);
+        }
     }
     if (lin) {
         FH_REQUIRE(s.lin_heads > 0 && s.lin_dim > 0 && s.lin_vdim > 0 && linear_supports(s.lin_dim, s.lin_vdim), "layer %d: linear attention of %d heads, a state of %d x %d",
@@ -1261,10 +1356,15 @@ static int check_pre_norm_layer(const FerrumHipLayerSpec& s, int i) {
     }
     FH_REQUIRE(s.mixer != FERRUM_HIP_MIXER_SELECTIVE_SCAN || (s.scan_inner > 0 && s.scan_state > 0 && s.scan_state <= SCAN_MAX_STATE && s.scan_dt_rank > 0 && s.conv_taps > 0),
                "layer %d: scan of %d channels, %d states, rank %d, %d taps", i, s.scan_inner, s.scan_state, s.scan_dt_rank, s.conv_taps);
-    FH_REQUIRE(s.ff == FERRUM_HIP_FF_NONE || ((s.ff == FERRUM_HIP_FF_GELU_GLU || s.ff == FERRUM_HIP_FF_MOE_SILU_GLU) && s.ff_width > 0), "layer %d: feed-forward %d of width %d", i,
-               s.ff, s.ff_width);
-    FH_REQUIRE(s.ff != FERRUM_HIP_FF_MOE_SILU_GLU || moe_route_grouped_supports(s.experts, s.top, MoeGroupedRule{nullptr, s.route_groups, s.route_keep, s.route_scale}),
-               "layer %d: %d of %d experts from %d of %d groups", i, s.top, s.experts, s.route_keep, s.route_groups);
+    const bool silu = s.ff == FERRUM_HIP_FF_MOE_SILU_GLU, clamped = s.ff == FERRUM_HIP_FF_MOE_CLAMPED_GLU;
+    FH_REQUIRE(s.ff == FERRUM_HIP_FF_NONE || ((s.ff == FERRUM_HIP_FF_GELU_GLU || silu || clamped) && s.ff_width > 0), "layer %d: feed-forward %d of width %d", i, s.ff, s.ff_width);
+    MoeCorrectedRule rule{nullptr, s.route_groups, s.route_keep, s.route_scale};
+    rule.unlisted = s.identity_experts;
+    FH_REQUIRE(!(silu || clamped) || (s.experts > 0 && s.identity_experts >= 0 && moe_route_corrected_supports(s.experts + s.identity_experts, s.top, rule)),
+               "layer %d: %d of %d experts from %d of %d groups", i, s.top, s.experts + s.identity_experts, s.route_keep, s.route_groups);
+    // (the copies of the input and the shared expert's factor are part of the post-norm block's sums)
+    FH_REQUIRE(clamped ? s.shared_width >= 0 && (post || (!s.identity_experts && !s.shared_width)) : !s.identity_experts && !s.shared_width,
+               "layer %d: %d identity experts, a shared expert of width %d", i, s.identity_experts, s.shared_width);
     return 0;
 }
 
@@ -1275,21 +1375,24 @@ int check_layered_config(const FerrumHipModelConfig& c, const FerrumHipLayeredCo
     FH_REQUIRE(c.tp_world <= 1, "layered model: tensor parallelism is not available");
     FH_REQUIRE(lc.dtype == FERRUM_HIP_DTYPE_BF16 || lc.dtype == FERRUM_HIP_DTYPE_F32, "layered model: dtype %d", lc.dtype);
     FH_REQUIRE(lc.bigram_buckets >= 0 && lc.state_slots >= 0, "layered model: bigram buckets %d, state slots %d", lc.bigram_buckets, lc.state_slots);
-    FH_REQUIRE(lc.block == FERRUM_HIP_BLOCK_GATED_POST_NORM || lc.block == FERRUM_HIP_BLOCK_PARALLEL_PRE_NORM || lc.block == FERRUM_HIP_BLOCK_PRE_NORM,
+    FH_REQUIRE(lc.block == FERRUM_HIP_BLOCK_GATED_POST_NORM || lc.block == FERRUM_HIP_BLOCK_PARALLEL_PRE_NORM || lc.block == FERRUM_HIP_BLOCK_PRE_NORM ||
+                   lc.block == FERRUM_HIP_BLOCK_POST_NORM,
                "layered model: block %d", lc.block);
-    const bool pre_norm = lc.block == FERRUM_HIP_BLOCK_PRE_NORM;
+    const bool pre_norm = lc.block == FERRUM_HIP_BLOCK_PRE_NORM, in_turn = pre_norm || lc.block == FERRUM_HIP_BLOCK_POST_NORM;
+    FH_REQUIRE(lc.position_rows == 0 || lc.position_rows >= c.max_seq_len, "layered model: %d learned positions for sequences of %d tokens", lc.position_rows, c.max_seq_len);
+    FH_REQUIRE(lc.logit_softcap >= 0.f, "layered model: logits capped at %g", lc.logit_softcap);
     FH_REQUIRE(lc.loop_times == 0 || (pre_norm && lc.loop_times > 0 && lc.loop_start >= 0 && lc.loop_start < lc.loop_stop && lc.loop_stop <= c.num_layers),
                "layered model: layers %d to %d, %d times", lc.loop_start, lc.loop_stop, lc.loop_times);
-    FH_REQUIRE(!pre_norm || (!lc.bigram_buckets && lc.untied_head), "layered model: a pre-norm block takes plain embeddings and a vocabulary projection of its own");
+    FH_REQUIRE(!in_turn || (!lc.bigram_buckets && lc.untied_head), "layered model: a pre-norm or post-norm block takes plain embeddings and a vocabulary projection of its own");
     const bool parallel = lc.block == FERRUM_HIP_BLOCK_PARALLEL_PRE_NORM;
     FH_REQUIRE(lc.token_side_dim >= 0 && (parallel || !lc.token_side_dim), "layered model: per-layer token input of %d dimensions", lc.token_side_dim);
     for (int i = 0; i < c.num_layers; i++) {
         const FerrumHipLayerSpec& s = layers[i];
-        if (pre_norm) {
-            if (int rc = check_pre_norm_layer(s, i)) return rc;
+        if (in_turn) {
+            if (int rc = check_in_turn_layer(lc, layers, i)) return rc;
             continue;
         }
-        FH_REQUIRE(!s.mixer2, "layer %d: two mixers side by side need a pre-norm block", i);
+        FH_REQUIRE(!s.mixer2, "layer %d: two mixers side by side need a pre-norm or post-norm block", i);
         if (s.mixer == FERRUM_HIP_MIXER_LATENT_ATTENTION) {
             FH_REQUIRE(s.heads > 0 && s.dim > 0 && s.rot_dim > 0 && s.vdim > 0 && s.q_rank >= 0 && s.kv_rank > 0 && (s.window > 0 || s.window == FERRUM_HIP_WINDOW_NONE),
                        "layer %d: latent attention sizes must be positive", i);

@@ -305,7 +305,7 @@ static std::string architecture(const FerrumHipCheckpoint* ck) {
 }
 
 // ── layered architectures ──
-static bool is_layered_arch(const std::string& arch) { return arch == "Nerenex" || arch == "Safolorn" || arch == "Segetar"; }
+static bool is_layered_arch(const std::string& arch) { return arch == "Nerenex" || arch == "Safolorn" || arch == "Segetar" || arch == "Fororax"; }
 
 // required numbers of a config object; the first one missing or out of place is named in the error
 struct Fields {
@@ -519,6 +519,70 @@ static int safolorn_whole(const FerrumHipCheckpoint* ck, FerrumHipLayeredConfig*
     return 0;
 }
 
+// a layer of Fororax: grouped attention with scores that fall with the logarithm of the distance, or with sinks and mixed heads; experts
+static int fororax_spec(const Value& v, int index, FerrumHipLayerSpec* s) {
+    memset(s, 0, sizeof(*s));
+    const std::string at = "layers[" + std::to_string(index) + "]";
+    const Value *type = v.get("type"), *ff = v.get("mlp");
+    FH_REQUIRE(type && type->kind == Value::Str, "config.json: %s has no type", at.c_str());
+    s->mixer = FERRUM_HIP_MIXER_GROUPED_ATTENTION;
+    s->window = FERRUM_HIP_WINDOW_NONE;
+    s->attn_flags = FERRUM_HIP_ATTN_NO_HEAD_GATE | FERRUM_HIP_ATTN_HEAD_NORM;
+    if (type->str == "attention") s->attn_flags |= FERRUM_HIP_ATTN_LOG_DISTANCE;
+    else if (type->str == "attention_2")
+        s->attn_flags |= FERRUM_HIP_ATTN_QKV_BIAS | FERRUM_HIP_ATTN_SINK | FERRUM_HIP_ATTN_TALK | FERRUM_HIP_ATTN_VALUE_GATE | FERRUM_HIP_ATTN_OUT_BIAS;
+    else {
+        set_error("config.json: %s has the unknown type '%s'", at.c_str(), type->str.c_str());
+        return FERRUM_HIP_UNSUPPORTED;
+    }
+    Fields m{v.get("mixer"), at + ".mixer", ""};
+    s->heads = m.size("heads"); s->kv_heads = m.size("kv_heads"); s->dim = m.size("dim"); s->vdim = m.size("vdim"); s->scale = (float)m.num("scale");
+    if (const Value* from = m.obj ? m.obj->get("kv_from") : nullptr; from && from->kind != Value::Null) {
+        const int32_t j = m.size("kv_from");
+        FH_REQUIRE(j < index, "config.json: %s.mixer.kv_from = %d is no earlier layer", at.c_str(), j);
+        s->kv_source = j + 1;
+    }
+    FH_FIELDS_OK(m);
+    if (!ff || ff->kind == Value::Null) return 0;
+    const Value* kind = ff->get("kind");
+    if (!(kind && kind->kind == Value::Str && kind->str == "moe")) {
+        set_error("config.json: %s.mlp has an unknown kind", at.c_str());
+        return FERRUM_HIP_UNSUPPORTED;
+    }
+    s->ff = FERRUM_HIP_FF_MOE_CLAMPED_GLU;
+    Fields f{ff, at + ".mlp", ""}, e = f.sub("expert"), r = f.sub("router"), h = f.sub("shared");
+    s->ff_width = e.size("ff"); s->ff_limit = (float)e.num("limit");
+    s->experts = r.size("experts"); s->identity_experts = r.size("identity"); s->top = r.size("top");
+    s->shared_width = h.size("ff"); s->shared_limit = (float)h.num("limit");
+    s->route_groups = s->route_keep = 1; s->route_scale = 1.f;
+    FH_FIELDS_OK(e); FH_FIELDS_OK(r); FH_FIELDS_OK(h);
+    return 0;
+}
+static int fororax_whole(const FerrumHipCheckpoint* ck, FerrumHipLayeredConfig* c) {
+    memset(c, 0, sizeof(*c));
+    Fields f{&ck->config, "config", ""}, emb = f.sub("embedding");
+    c->block = FERRUM_HIP_BLOCK_POST_NORM;
+    c->residual_mult = 1.f;
+    c->untied_head = 1;
+    c->stream_mult = (float)f.num("postln_alpha");
+    c->embed_scale = (float)emb.num("scale");
+    c->position_rows = f.size("max_positions");
+    c->logit_softcap = (float)f.num("logit_softcap");
+    FH_FIELDS_OK(f); FH_FIELDS_OK(emb);
+    FH_REQUIRE(c->position_rows > 0 && c->logit_softcap > 0.f && c->embed_scale != 0.f, "config.json: max_positions = %d, logit_softcap = %g, embedding.scale = %g", c->position_rows,
+               c->logit_softcap, c->embed_scale);
+    return 0;
+}
+
+// an architecture's reader of the whole and of layer i
+static int layered_whole(const FerrumHipCheckpoint* ck, const std::string& arch, FerrumHipLayeredConfig* c) {
+    return (arch == "Fororax" ? fororax_whole : arch == "Segetar" ? segetar_whole : arch == "Safolorn" ? safolorn_whole : nerenex_whole)(ck, c);
+}
+static int layered_spec(const FerrumHipCheckpoint* ck, const std::string& arch, const Value& v, int i, FerrumHipLayerSpec* s) {
+    if (arch == "Segetar") return segetar_spec(ck, v, i, s);
+    return (arch == "Fororax" ? fororax_spec : arch == "Safolorn" ? safolorn_spec : nerenex_spec)(v, i, s);
+}
+
 static int layered_model_config(const FerrumHipCheckpoint* ck, int max_seq_len_cap, FerrumHipModelConfig* cfg) {
     Fields f{&ck->config, "config", ""};
     const Value* layers = cfg_get(ck, "layers");
@@ -529,7 +593,8 @@ static int layered_model_config(const FerrumHipCheckpoint* ck, int max_seq_len_c
     Fields norm = f.sub("norm");
     cfg->rms_eps = (float)norm.num("eps");
     FH_FIELDS_OK(f); FH_FIELDS_OK(norm);
-    cfg->max_seq_len = max_seq_len_cap > 0 ? max_seq_len_cap : 32768;      // (the architecture sets no limit; the angle tables need one)
+    cfg->max_seq_len = max_seq_len_cap > 0 ? max_seq_len_cap : 32768;      // (most architectures set no limit; the angle tables need one)
+    if (const Value* p = cfg_get(ck, "max_positions"); p && p->is_u64() && p->num > 0) cfg->max_seq_len = (int32_t)std::min<double>(cfg->max_seq_len, p->num);
     cfg->group_size = 128;
     cfg->tp_world = 1;
     return 0;
@@ -700,7 +765,7 @@ int ferrum_hip_checkpoint_model_config(const FerrumHipCheckpoint* ck, int max_se
     else if (arch == "Qwen3MoeForCausalLM" || arch == "qwen3_moe") fam = Qwen3Moe;
     else if (arch == "MistralForCausalLM" || arch == "mistral") fam = Mistral;
     else {
-        set_error("checkpoint: architecture '%s' is not supported by the HIP runner (Llama, Mistral, Qwen2, Qwen3, Qwen3-MoE, Gemma-3, Nerenex, Safolorn, Segetar)", arch.c_str());
+        set_error("checkpoint: architecture '%s' is not supported by the HIP runner (Llama, Mistral, Qwen2, Qwen3, Qwen3-MoE, Gemma-3, Nerenex, Safolorn, Segetar, Fororax)", arch.c_str());
         return FERRUM_HIP_UNSUPPORTED;
     }
     auto u = [&](const char* key, const char* alt, double dflt) {
@@ -791,9 +856,9 @@ int ferrum_hip_checkpoint_layered_config(const FerrumHipCheckpoint* ck, int* is_
     const Value* ls = cfg_get(ck, "layers");
     FH_REQUIRE(ls && ls->kind == Value::Arr && !ls->arr.empty(), "config.json: 'layers' is missing or empty");
     if (layered)
-        if (int rc = (arch == "Segetar" ? segetar_whole : arch == "Safolorn" ? safolorn_whole : nerenex_whole)(ck, layered)) return rc;
+        if (int rc = layered_whole(ck, arch, layered)) return rc;
     for (int i = 0; layers && i < (int)ls->arr.size() && i < capacity; i++)
-        if (int rc = arch == "Segetar" ? segetar_spec(ck, ls->arr[i], i, &layers[i]) : (arch == "Safolorn" ? safolorn_spec : nerenex_spec)(ls->arr[i], i, &layers[i])) return rc;
+        if (int rc = layered_spec(ck, arch, ls->arr[i], i, &layers[i])) return rc;
     return 0;
 }
 

@@ -82,7 +82,7 @@ __device__ __forceinline__ float route_partner(float x, int off) {
 }
 // v of experts outside the best rule.keep groups ← −∞; a group counts by the sum of its two largest v
 template <int PER>
-__device__ __forceinline__ void route_drop_groups(float (&v)[PER], const int (&grp)[PER], int lane, int per_group, const MoeGroupedRule& rule) {
+__device__ __forceinline__ void route_drop_groups(float (&v)[PER], const int (&grp)[PER], int lane, int per_group, const MoeCorrectedRule& rule) {
     if (per_group <= 64 && !(per_group & (per_group - 1))) {
         // groups are aligned runs of lanes: two largest by butterflies, then every group's place among them
         float score[PER];
@@ -141,19 +141,33 @@ __device__ __forceinline__ void route_drop_groups(float (&v)[PER], const int (&g
     for (int i = 0; i < PER; i++)
         if (!(kept >> (grp[i] & 63) & 1)) v[i] = -INFINITY;
 }
-// MoeGroupedRule of one token on one wave, layout as route_token
+// MoeCorrectedRule of one token on one wave, layout as route_token; ids of all experts, unlisted ones included
 template <int PER>
-__device__ __forceinline__ void route_token_grouped(const float* __restrict__ row, int lane, int num_experts, int top_k, const MoeGroupedRule& rule, int& id, float& weight) {
+__device__ __forceinline__ void route_token_corrected(const float* __restrict__ row, int lane, int num_experts, int top_k, const MoeCorrectedRule& rule, int& id, float& weight) {
     const int per_group = num_experts / rule.groups;
     float s[PER], v[PER], top;
     int grp[PER];
 #pragma unroll
     for (int i = 0; i < PER; i++) {
         const int e = lane + i * 64;
-        const bool in = e < num_experts;
-        s[i] = in ? 1.0f / (1.0f + expf(-row[e])) : 0.f;
-        v[i] = in ? s[i] + rule.correction[e] : -INFINITY;
+        s[i] = e >= num_experts ? rule.softmax ? -INFINITY : 0.f : rule.softmax ? row[e] : 1.0f / (1.0f + expf(-row[e]));
         grp[i] = e / per_group;
+    }
+    if (rule.softmax) {
+        float mx = s[0], total = 0.f;
+#pragma unroll
+        for (int i = 1; i < PER; i++) mx = fmaxf(mx, s[i]);
+        mx = wave_reduce_max(mx);
+#pragma unroll
+        for (int i = 0; i < PER; i++) { s[i] = expf(s[i] - mx); total += s[i]; }
+        const float inv = 1.0f / wave_reduce_sum(total);
+#pragma unroll
+        for (int i = 0; i < PER; i++) s[i] *= inv;
+    }
+#pragma unroll
+    for (int i = 0; i < PER; i++) {
+        const int e = lane + i * 64;
+        v[i] = e < num_experts ? s[i] + rule.correction[e] : -INFINITY;
     }
     if (rule.keep < rule.groups) route_drop_groups<PER>(v, grp, lane, per_group, rule);
     float sum = 0.f;
@@ -170,7 +184,7 @@ __device__ __forceinline__ void route_token_grouped(const float* __restrict__ ro
         sum += score;
         if (lane == k) { weight = score; id = e; }
     }
-    weight = weight / (sum + 1e-20f) * rule.scale;
+    weight = (rule.raw ? weight : weight / (sum + 1e-20f)) * rule.scale;
 }
 
 // the launch `call` with PER experts per lane
@@ -197,13 +211,13 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const T* __restrict__ log
 }
 
 template <int PER>
-__global__ __launch_bounds__(256) void moe_route_grouped_kernel(const float* __restrict__ logits, MoeGroupedRule rule, int32_t* __restrict__ ids,
+__global__ __launch_bounds__(256) void moe_route_corrected_kernel(const float* __restrict__ logits, MoeCorrectedRule rule, int32_t* __restrict__ ids,
                                                                 float* __restrict__ weights, int tokens, int num_experts, int top_k) {
     const int tok = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
     if (tok >= tokens) return;
     int id;
     float w;
-    route_token_grouped<PER>(logits + (long)tok * num_experts, lane, num_experts, top_k, rule, id, w);
+    route_token_corrected<PER>(logits + (long)tok * num_experts, lane, num_experts, top_k, rule, id, w);
     if (lane < top_k) {
         ids[(long)tok * top_k + lane] = id;
         weights[(long)tok * top_k + lane] = w;
@@ -214,10 +228,10 @@ __global__ __launch_bounds__(256) void moe_route_grouped_kernel(const float* __r
 // moe_align_kernel<0> write them, except that nothing is written past the last block).  A wave routes its tokens, then every thread owns
 // a pair: its rank among the pairs of its expert is the count in earlier waves (histograms in LDS) plus the count in earlier lanes.
 constexpr int ROUTE_SORT_PAIRS = 1024;
-template <int PER, bool GROUPED>
+template <int PER, bool CORRECTED>
 __global__ __launch_bounds__(1024) void moe_route_sort_kernel(const float* __restrict__ logits, int32_t* __restrict__ ids, float* __restrict__ weights,
                                                               int32_t* __restrict__ sorted, int32_t* __restrict__ block_ids, int32_t* __restrict__ total,
-                                                              int tokens, int num_experts, int top_k, int norm_topk_prob, int block_size, MoeGroupedRule rule) {
+                                                              int tokens, int num_experts, int top_k, int norm_topk_prob, int block_size, MoeCorrectedRule rule) {
     __shared__ int16_t lds_id[ROUTE_SORT_PAIRS];
     __shared__ int16_t hist[16][512];
     __shared__ int32_t offset[512];
@@ -225,7 +239,7 @@ __global__ __launch_bounds__(1024) void moe_route_sort_kernel(const float* __res
     for (int t = wave; t < tokens; t += 16) {
         int id;
         float w;
-        if (GROUPED) route_token_grouped<PER>(logits + (long)t * num_experts, lane, num_experts, top_k, rule, id, w);
+        if (CORRECTED) route_token_corrected<PER>(logits + (long)t * num_experts, lane, num_experts, top_k, rule, id, w);
         else route_token<PER>(logits + (long)t * num_experts, lane, num_experts, top_k, norm_topk_prob, id, w);
         if (lane < top_k) {
             lds_id[t * top_k + lane] = (int16_t)id;
@@ -235,7 +249,9 @@ __global__ __launch_bounds__(1024) void moe_route_sort_kernel(const float* __res
     }
     for (int i = lane; i < num_experts; i += 64) hist[wave][i] = 0;
     __syncthreads();
-    const int e = tid < n_pairs ? lds_id[tid] : -1;
+    if (CORRECTED) num_experts -= rule.unlisted;               // (the sorted list's)
+    int e = tid < n_pairs ? lds_id[tid] : -1;
+    if (e >= num_experts) e = -1;
     int rank = 0, same = 0;
     if (wave < nw)
 #pragma unroll
@@ -276,9 +292,9 @@ __global__ __launch_bounds__(1024) void moe_route_sort_kernel(const float* __res
 }
 bool moe_route_sort_supports(int tokens, int num_experts, int top_k) { return (long)tokens * top_k <= ROUTE_SORT_PAIRS && num_experts <= 512; }
 int moe_route_sort_f32(const float* logits, int32_t* expert_ids, float* expert_weights, int32_t* sorted_token_ids, int32_t* block_ids, int32_t* total_post_pad,
-                       int tokens, int num_experts, int top_k, int norm_topk_prob, int block_size, hipStream_t s, const MoeGroupedRule* rule) {
+                       int tokens, int num_experts, int top_k, int norm_topk_prob, int block_size, hipStream_t s, const MoeCorrectedRule* rule) {
     if (tokens <= 0) return 0;
-    FH_REQUIRE(!rule || moe_route_grouped_supports(num_experts, top_k, *rule), "moe route + sort: %d groups, %d kept", rule->groups, rule->keep);
+    FH_REQUIRE(!rule || moe_route_corrected_supports(num_experts, top_k, *rule), "moe route + sort: %d groups, %d kept", rule->groups, rule->keep);
     FH_REQUIRE(moe_route_sort_supports(tokens, num_experts, top_k) && num_experts > 0 && top_k > 0 && top_k <= num_experts && top_k <= 64 && block_size > 0,
                "moe route + sort: %d tokens, %d of %d experts, blocks of %d", tokens, top_k, num_experts, block_size);
     form_hit(FORM_MOE_ROUTE_SORT);
@@ -287,20 +303,20 @@ int moe_route_sort_f32(const float* logits, int32_t* expert_ids, float* expert_w
                                      total_post_pad, tokens, num_experts, top_k, norm_topk_prob, block_size, *rule));
     else
         ROUTE_PER(hipLaunchKernelGGL((moe_route_sort_kernel<PER, false>), dim3(1), dim3(1024), 0, s, logits, expert_ids, expert_weights, sorted_token_ids, block_ids,
-                                     total_post_pad, tokens, num_experts, top_k, norm_topk_prob, block_size, MoeGroupedRule{}));
+                                     total_post_pad, tokens, num_experts, top_k, norm_topk_prob, block_size, MoeCorrectedRule{}));
     FH_CHECK_LAUNCH();
     return 0;
 }
-bool moe_route_grouped_supports(int num_experts, int top_k, const MoeGroupedRule& r) {
+bool moe_route_corrected_supports(int num_experts, int top_k, const MoeCorrectedRule& r) {
     return num_experts > 0 && num_experts <= 512 && r.groups > 0 && r.groups <= 64 && num_experts % r.groups == 0 && r.keep > 0 && r.keep <= r.groups && top_k > 0 &&
-           top_k <= 64 && top_k <= num_experts / r.groups * r.keep;
+           top_k <= 64 && top_k <= num_experts / r.groups * r.keep && r.unlisted >= 0 && r.unlisted < num_experts;
 }
-int moe_route_grouped_f32(const float* logits, const MoeGroupedRule& rule, int32_t* expert_ids, float* expert_weights, int tokens, int num_experts, int top_k,
+int moe_route_corrected_f32(const float* logits, const MoeCorrectedRule& rule, int32_t* expert_ids, float* expert_weights, int tokens, int num_experts, int top_k,
                           hipStream_t s) {
     if (tokens <= 0) return 0;
-    FH_REQUIRE(moe_route_grouped_supports(num_experts, top_k, rule) && rule.correction, "moe route: %d of %d experts, %d of %d groups", top_k, num_experts, rule.keep, rule.groups);
-    form_hit(FORM_ROUTE_GROUPED);
-    ROUTE_PER(hipLaunchKernelGGL(moe_route_grouped_kernel<PER>, dim3(cdiv(tokens, 4)), dim3(256), 0, s, logits, rule, expert_ids, expert_weights, tokens, num_experts, top_k));
+    FH_REQUIRE(moe_route_corrected_supports(num_experts, top_k, rule) && rule.correction, "moe route: %d of %d experts, %d of %d groups", top_k, num_experts, rule.keep, rule.groups);
+    form_hit(rule.softmax ? FORM_ROUTE_SOFTMAX : FORM_ROUTE_GROUPED);
+    ROUTE_PER(hipLaunchKernelGGL(moe_route_corrected_kernel<PER>, dim3(cdiv(tokens, 4)), dim3(256), 0, s, logits, rule, expert_ids, expert_weights, tokens, num_experts, top_k));
     FH_CHECK_LAUNCH();
     return 0;
 }

@@ -5,26 +5,32 @@
 namespace fh {
 
 template <typename E, bool VEC>
-__global__ __launch_bounds__(256) void embed_bigram_kernel(const E* __restrict__ table, const E* __restrict__ bigram, int buckets,
-                                                           int64_t mul_prev, int64_t mul_cur, BatchView v, float* __restrict__ x,
-                                                           E* __restrict__ xb, int dim, int ldb) {
+__global__ __launch_bounds__(256) void embed_kernel(Embedding<E> p, BatchView v, float* __restrict__ x, E* __restrict__ xb, int dim, int ldb) {
     const int t = blockIdx.x;
     const uint32_t tok = v.tokens[t];
-    long row = 0;
-    if (bigram) {
-        const int seq = v.tok_seq[t];
-        const int64_t prev = t == (int)v.cu[seq] ? (int64_t)v.prev[seq] : (int64_t)v.tokens[t - 1];
-        row = prev < 0 ? buckets : (long)(((uint64_t)prev * (uint64_t)mul_prev + (uint64_t)tok * (uint64_t)mul_cur) % (uint64_t)buckets);
+    const E *own = p.table + (long)tok * dim, *bigram = nullptr, *place = nullptr;
+    if (p.bigram || p.positions) {
+        const int seq = v.tok_seq[t], at = t - (int)v.cu[seq];
+        if (p.bigram) {
+            const int64_t prev = at == 0 ? (int64_t)v.prev[seq] : (int64_t)v.tokens[t - 1];
+            bigram = p.bigram + dim * (prev < 0 ? (long)p.buckets : (long)(((uint64_t)prev * (uint64_t)p.mul_prev + (uint64_t)tok * (uint64_t)p.mul_cur) % (uint64_t)p.buckets));
+        }
+        if (p.positions) place = p.positions + (long)(v.pos[seq] + at) * dim;
     }
     if (VEC) {
         typedef typename Frag<E>::v8 v8;
         for (int i = threadIdx.x * 8; i < dim; i += 2048) {
-            const v8 e = *reinterpret_cast<const v8*>(table + (long)tok * dim + i);
-            v8 g = e, o;
-            if (bigram) g = *reinterpret_cast<const v8*>(bigram + row * dim + i);
+            const v8 e = *reinterpret_cast<const v8*>(own + i);
+            v8 g = e, l = e, o;
+            if (bigram) g = *reinterpret_cast<const v8*>(bigram + i);
+            if (place) l = *reinterpret_cast<const v8*>(place + i);
             floatx4 f[2];
 #pragma unroll
-            for (int j = 0; j < 8; j++) { f[j >> 2][j & 3] = (float)e[j] + (bigram ? (float)g[j] : 0.f); o[j] = (E)f[j >> 2][j & 3]; }
+            for (int j = 0; j < 8; j++) {
+                const float y = (float)e[j] * p.factor + (bigram ? (float)g[j] : 0.f) + (place ? (float)l[j] : 0.f);
+                f[j >> 2][j & 3] = y;
+                o[j] = (E)y;
+            }
             *reinterpret_cast<floatx4*>(x + (long)t * dim + i) = f[0];
             *reinterpret_cast<floatx4*>(x + (long)t * dim + i + 4) = f[1];
             *reinterpret_cast<v8*>(xb + (long)t * ldb + i) = o;
@@ -32,20 +38,18 @@ __global__ __launch_bounds__(256) void embed_bigram_kernel(const E* __restrict__
         return;
     }
     for (int i = threadIdx.x; i < dim; i += 256) {
-        float e = (float)table[(long)tok * dim + i];
-        if (bigram) e += (float)bigram[row * dim + i];
+        float e = (float)own[i] * p.factor;
+        if (bigram) e += (float)bigram[i];
+        if (place) e += (float)place[i];
         x[(long)t * dim + i] = e;
         xb[(long)t * ldb + i] = (E)e;
     }
 }
 
 template <typename E>
-int embed_bigram(const E* table, const E* bigram, int buckets, int64_t mul_prev, int64_t mul_cur, const BatchView& v, float* x, E* xb,
-                 int dim, int ldb, hipStream_t s) {
-    if (dim % 8 == 0)
-        hipLaunchKernelGGL((embed_bigram_kernel<E, true>), dim3(v.T), dim3(256), 0, s, table, bigram, buckets, mul_prev, mul_cur, v, x, xb, dim, ldb);
-    else
-        hipLaunchKernelGGL((embed_bigram_kernel<E, false>), dim3(v.T), dim3(256), 0, s, table, bigram, buckets, mul_prev, mul_cur, v, x, xb, dim, ldb);
+int embed_tokens(const Embedding<E>& e, const BatchView& v, float* x, E* xb, int dim, int ldb, hipStream_t s) {
+    if (dim % 8 == 0) hipLaunchKernelGGL((embed_kernel<E, true>), dim3(v.T), dim3(256), 0, s, e, v, x, xb, dim, ldb);
+    else hipLaunchKernelGGL((embed_kernel<E, false>), dim3(v.T), dim3(256), 0, s, e, v, x, xb, dim, ldb);
     FH_CHECK_LAUNCH();
     return 0;
 }
@@ -222,8 +226,8 @@ int rms_norm_rows(const float* x, const int32_t* row_idx, const float* w, float 
     return 0;
 }
 
-// One workgroup per row; a thread holds up to 4 quads of the row in registers.
-template <typename E, bool VEC>
+// One workgroup per row; a thread holds up to 4 quads of the row in registers.  POST: the sum itself is normed.
+template <typename E, bool VEC, bool POST>
 __global__ __launch_bounds__(1024) void stream_update_kernel(StreamUpdate<E> u) {
     __shared__ float red[64];
     const long row = blockIdx.x;
@@ -232,7 +236,16 @@ __global__ __launch_bounds__(1024) void stream_update_kernel(StreamUpdate<E> u) 
     float* xr = u.x + row * dim;
     const E* pr = u.pairs + row * u.top * u.ld_pair;
     E* out = u.out + row * u.ldo;
-    const bool joined = u.sub2 != nullptr;
+    const bool joined = !POST && u.sub2 != nullptr;
+    float keep = u.replace ? 0.f : 1.f, factor = 1.f;
+    if (POST) {
+        keep *= u.keep;
+        if (u.sub_scale) factor = (float)u.sub_scale[row * u.ld_scale];
+        if (u.pair_ids)
+            for (int j = 0; j < u.top; j++)
+                if (u.pair_ids[row * u.top + j] >= u.pair_limit) keep += u.weights[row * u.top + j];
+    }
+    auto listed = [&](int j) { return !POST || !u.pair_ids || u.pair_ids[row * u.top + j] < u.pair_limit; };
     if (VEC) {
         typedef E e4 __attribute__((ext_vector_type(4)));
         floatx4 v[4], r[4], xv[4];
@@ -244,11 +257,18 @@ __global__ __launch_bounds__(1024) void stream_update_kernel(StreamUpdate<E> u) 
                 v[c] = (floatx4){0.f, 0.f, 0.f, 0.f};
                 if (u.sub) v[c] = *reinterpret_cast<const floatx4*>(s1 + i);
                 for (int z = 1; z < u.slabs; z++) v[c] += *reinterpret_cast<const floatx4*>(s1 + z * u.slab_stride + i);
+                if (POST)
+#pragma unroll
+                    for (int k = 0; k < 4; k++) v[c][k] *= factor;
                 xv[c] = (floatx4){0.f, 0.f, 0.f, 0.f};
                 if (!u.replace) xv[c] = *reinterpret_cast<const floatx4*>(xr + i);
+                if (POST)
+#pragma unroll
+                    for (int k = 0; k < 4; k++) xv[c][k] *= keep;
                 if (u.add) xv[c] += *reinterpret_cast<const floatx4*>(u.add + i);
 #pragma unroll 4
                 for (int j = 0; j < u.top; j++) {
+                    if (!listed(j)) continue;
                     const e4 e = *reinterpret_cast<const e4*>(pr + j * u.ld_pair + i);
                     const float w = u.weights[row * u.top + j];
 #pragma unroll
@@ -279,7 +299,21 @@ __global__ __launch_bounds__(1024) void stream_update_kernel(StreamUpdate<E> u) 
                 xv[c] += v[c];
 #pragma unroll
                 for (int k = 0; k < 4; k++) n += xv[c][k] * xv[c][k];
-                *reinterpret_cast<floatx4*>(xr + i) = xv[c];
+                if (!POST) *reinterpret_cast<floatx4*>(xr + i) = xv[c];
+            }
+        }
+        if (POST) {
+            const float inv = 1.0f / sqrtf(block_sum(n, red) / (float)dim + u.eps);
+            n = 0.f;
+#pragma unroll
+            for (int c = 0; c < 4; c++) {
+                const int i = (c * nt + threadIdx.x) * 4;
+                if (i < dim) {
+                    const floatx4 w = *reinterpret_cast<const floatx4*>(u.post_w + i);
+#pragma unroll
+                    for (int k = 0; k < 4; k++) { xv[c][k] *= inv * w[k]; n += xv[c][k] * xv[c][k]; }
+                    *reinterpret_cast<floatx4*>(xr + i) = xv[c];
+                }
             }
         }
         if (!u.out) return;
@@ -301,7 +335,9 @@ __global__ __launch_bounds__(1024) void stream_update_kernel(StreamUpdate<E> u) 
     auto first = [&](int i) {
         float t = u.sub ? s1[i] : 0.f;
         for (int z = 1; z < u.slabs; z++) t += s1[z * u.slab_stride + i];
-        for (int j = 0; j < u.top; j++) t += u.weights[row * u.top + j] * (float)pr[j * u.ld_pair + i];
+        t *= factor;
+        for (int j = 0; j < u.top; j++)
+            if (listed(j)) t += u.weights[row * u.top + j] * (float)pr[j * u.ld_pair + i];
         return t;
     };
     auto second = [&](int i) {
@@ -319,9 +355,18 @@ __global__ __launch_bounds__(1024) void stream_update_kernel(StreamUpdate<E> u) 
     for (int i = threadIdx.x; i < dim; i += nt) {
         float t = joined ? first(i) * i1 * u.w[i] + second(i) * i2 * u.w2[i] : first(i);
         if (u.add) t += u.add[i];
-        if (!u.replace) t += xr[i];
+        if (!u.replace) t += POST ? keep * xr[i] : xr[i];
         xr[i] = t;
         n += t * t;
+    }
+    if (POST) {
+        const float inv = 1.0f / sqrtf(block_sum(n, red) / (float)dim + u.eps);
+        n = 0.f;
+        for (int i = threadIdx.x; i < dim; i += nt) {            // (a thread's own elements)
+            const float t = xr[i] * inv * u.post_w[i];
+            xr[i] = t;
+            n += t * t;
+        }
     }
     if (!u.out) return;
     const float unit = u.next_w ? 1.0f / sqrtf(block_sum(n, red + 32) / (float)dim + u.eps) : 1.0f;
@@ -331,16 +376,19 @@ template <typename E>
 int stream_update(const StreamUpdate<E>& u, hipStream_t s) {
     FH_REQUIRE(!u.sub2 || (u.sub && u.w && u.w2 && !u.top), "stream update: a second branch needs both norms");
     FH_REQUIRE(u.sub || u.slabs == 1, "stream update: slabs of nothing");
+    FH_REQUIRE(u.post_w ? !u.sub2 : u.keep == 1.f && !u.pair_ids && !u.sub_scale, "stream update: factors and the stream's own pairs belong to a normed sum of one branch");
     const int threads = u.rows <= 512 && u.dim >= 2048 ? 1024 : 256;
     const bool vec = u.dim % 4 == 0 && u.dim <= threads * 16 && u.ld_sub % 4 == 0 && u.ld_pair % 4 == 0 && u.ldo % 4 == 0 && u.slab_stride % 4 == 0 && u.slab_stride2 % 4 == 0;
-    if (vec) hipLaunchKernelGGL((stream_update_kernel<E, true>), dim3(u.rows), dim3(threads), 0, s, u);
-    else hipLaunchKernelGGL((stream_update_kernel<E, false>), dim3(u.rows), dim3(threads), 0, s, u);
+#define UPDATE(V, P) hipLaunchKernelGGL((stream_update_kernel<E, V, P>), dim3(u.rows), dim3(threads), 0, s, u)
+    if (u.post_w) { if (vec) UPDATE(true, true); else UPDATE(false, true); }
+    else { if (vec) UPDATE(true, false); else UPDATE(false, false); }
+#undef UPDATE
     FH_CHECK_LAUNCH();
     return 0;
 }
 
 #define INSTANTIATE(E)                                                                                                                  \
-    template int embed_bigram<E>(const E*, const E*, int, int64_t, int64_t, const BatchView&, float*, E*, int, int, hipStream_t);        \
+    template int embed_tokens<E>(const Embedding<E>&, const BatchView&, float*, E*, int, int, hipStream_t);                              \
     template int branch_add<E>(const float*, long, int, long, const E*, long, const float*, int, float*, E*, int, int, int, hipStream_t); \
     template int post_norm_add<E>(const float*, long, int, long, const E*, long, const float*, float, float, bool, float*, E*, int, int, \
                                   int, hipStream_t);                                                                                    \

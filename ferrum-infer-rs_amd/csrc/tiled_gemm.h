@@ -34,15 +34,16 @@ template <> struct Frag<float> {
 static inline int pad32(int n) { return (n + 31) / 32 * 32; }
 
 enum GemmAct : int { GEMM_ACT_NONE = 0, GEMM_ACT_SIGMOID = 1, GEMM_ACT_GELU_TANH = 2, GEMM_ACT_XIELU = 3, GEMM_ACT_RELU2 = 4, GEMM_ACT_CLAMPED_GLU = 5,
-                     GEMM_ACT_SILU_GLU = 6, GEMM_ACT_GELU_GLU = 7, GEMM_ACT_SILU = 8, GEMM_ACT_SOFTPLUS = 9, GEMM_ACT_LOG_SIGMOID = 10 };
+                     GEMM_ACT_SILU_GLU = 6, GEMM_ACT_GELU_GLU = 7, GEMM_ACT_SILU = 8, GEMM_ACT_SOFTPLUS = 9, GEMM_ACT_LOG_SIGMOID = 10,
+                     GEMM_ACT_SOFTCAP = 11 };
 // sections of (gate, up) pairs
 __host__ __device__ inline bool gemm_gated_act(int act) { return act >= GEMM_ACT_CLAMPED_GLU && act <= GEMM_ACT_GELU_GLU; }
-// inputs of a recurrence, a launch form of their own
-__host__ __device__ inline bool gemm_recurrence_act(int act) { return act >= GEMM_ACT_SOFTPLUS; }
+// inputs of a recurrence and capped logits, a launch form of their own
+__host__ __device__ inline bool gemm_rare_act(int act) { return act >= GEMM_ACT_SOFTPLUS; }
 constexpr int GEMM_MAX_SECTIONS = 6;
 struct GemmSection {          // columns [begin, next section's begin) of a fused projection; begin is a multiple of 32
     int begin, act;
-    float p, q;               // xIELU: softplus of its two parameters; clamped GLU: limit, slope of the sigmoid; log σ: factor p
+    float p, q;               // xIELU: softplus of its two parameters; clamped GLU: limit, slope of the sigmoid; log σ: factor p; softcap: cap p
     float mul = 1.f;          // factor of the accumulator, ahead of bias and activation (a norm's gain that is a single number)
 };
 // A gated section pairs 16-column tiles (gate, up, gate, up, …) whose weights are packed that way; a wave holds both tiles of a pair, and

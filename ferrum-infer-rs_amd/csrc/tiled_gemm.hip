@@ -9,15 +9,16 @@
 
 namespace fh {
 
-template <typename E, bool REC = false>
+template <typename E, bool RARE = false>
 __device__ __forceinline__ float gemm_act(const GemmSection& sec, float v) {
     if (sec.act == GEMM_ACT_SIGMOID) return ActMath<E>::sigmoid(v);
     if (sec.act == GEMM_ACT_GELU_TANH) return gelu_tanh_f32<E>(v);
     if (sec.act == GEMM_ACT_XIELU) return xielu_f32<E>(v, sec.p, sec.q);
     if (sec.act == GEMM_ACT_RELU2) { v = fmaxf(v, 0.f); return v * v; }
     if (sec.act == GEMM_ACT_SILU) return v * ActMath<E>::sigmoid(v);
-    if (REC && sec.act == GEMM_ACT_SOFTPLUS) return softplus_f32<E>(v);
-    if (REC && sec.act == GEMM_ACT_LOG_SIGMOID) return sec.p * log_sigmoid_f32<E>(v);
+    if (RARE && sec.act == GEMM_ACT_SOFTPLUS) return softplus_f32<E>(v);
+    if (RARE && sec.act == GEMM_ACT_LOG_SIGMOID) return sec.p * log_sigmoid_f32<E>(v);
+    if (RARE && sec.act == GEMM_ACT_SOFTCAP) return sec.p * ActMath<E>::tanh(v / sec.p);
     return v;
 }
 // output row of place r, −1: none
@@ -33,13 +34,13 @@ __device__ __forceinline__ void gemm_store(const TiledGemm<E>& p, int g, int row
     const long o = row * p.ldo + (p.rows.id ? 0 : g * p.out_group) + col;
     if (p.out_f32) p.out_f32[o] = v; else p.out[o] = (E)v;
 }
-template <typename E, bool REC>
+template <typename E, bool RARE>
 __device__ __forceinline__ void gemm_epilogue(const TiledGemm<E>& p, const GemmSection& sec, int g, int place, int col, float v) {
     const int row = gemm_out_row(p, place);
     if (row < 0 || col >= p.n_store) return;
     v *= sec.mul;
     if (p.bias) v += p.bias[(long)g * p.n + col];
-    gemm_store(p, g, row, col, gemm_act<E, REC>(sec, v));
+    gemm_store(p, g, row, col, gemm_act<E, RARE>(sec, v));
 }
 template <typename E>
 __device__ __forceinline__ float gemm_glu(const GemmSection& sec, float gate, float up) {
@@ -84,7 +85,7 @@ __device__ __forceinline__ int gemm_row_step(const TiledGemm<E>& p) { return p.x
 
 // grid (column blocks, row blocks, groups or K slabs); NW waves = (NW / kw) column groups × kw parts of K.  Two register buffers of U
 // k-steps: the next one is requested before the current one is multiplied; loads past the part's end repeat its last k-step.
-// EXT: with sorted rows, column factors, gated sections or inputs of a recurrence (each is a branch on the latency-bound path of the launches without).
+// EXT: with sorted rows, column factors, gated sections or rare activations (each is a branch on the latency-bound path of the launches without).
 template <typename E, int MT, int J, bool EXT>
 __global__ __launch_bounds__(512) void tiled_gemm_kernel(TiledGemm<E> p, int kw) {
     typedef typename Frag<E>::v8 v8;
@@ -417,10 +418,10 @@ int tiled_gemm(const TiledGemm<E>& gin, hipStream_t s) {
     FH_REQUIRE(g.ldx % 8 == 0 && g.x_group % 8 == 0 && g.n_store <= g.n && g.groups >= 1, "tiled_gemm: ldx=%ld group stride=%ld", g.ldx, g.x_group);
     FH_REQUIRE((g.out != nullptr) != (g.out_f32 != nullptr), "tiled_gemm: exactly one output");
     FH_REQUIRE(g.slabs == 1 || (g.groups == 1 && g.out_f32 && !g.bias && !g.nsec && !g.row_scale), "tiled_gemm: slabs are plain fp32 partial sums");
-    bool gated = false, rec = false;
+    bool gated = false, rare = false;
     for (int i = 0; i < g.nsec; i++) {
         gated |= gemm_gated_act(g.sec[i].act);
-        rec |= gemm_recurrence_act(g.sec[i].act);
+        rare |= gemm_rare_act(g.sec[i].act);
         FH_REQUIRE(g.sec[i].begin % 32 == 0, "tiled_gemm: section at column %d", g.sec[i].begin);
     }
     FH_REQUIRE(!gated || (g.groups == 1 && !g.col_scale), "tiled_gemm: gated sections take one group and no column factors");
@@ -450,7 +451,7 @@ int tiled_gemm(const TiledGemm<E>& gin, hipStream_t s) {
     form_hit(rows.id ? FORM_TILED_GEMM_GROUPED : FORM_TILED_GEMM);
 #define SMALL(J_, EXT_) \
     (mt == 1 ? launch_small<E, 1, J_, EXT_>(g, grid, nw, kw, s) : mt == 2 ? launch_small<E, 2, J_, EXT_>(g, grid, nw, kw, s) : launch_small<E, 4, J_, EXT_>(g, grid, nw, kw, s))
-    if (rows.id || g.col_scale || gated || rec) return J == 1 ? SMALL(1, true) : SMALL(2, true);
+    if (rows.id || g.col_scale || gated || rare) return J == 1 ? SMALL(1, true) : SMALL(2, true);
     return J == 1 ? SMALL(1, false) : SMALL(2, false);
 #undef SMALL
 }

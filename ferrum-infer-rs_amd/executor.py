@@ -28,7 +28,8 @@ class LayeredConfig(C.Structure):
     """Whole-model part of a layered model (FerrumHipLayeredConfig)."""
     _fields_ = [("dtype", C.c_int32), ("state_slots", C.c_int32), ("bigram_buckets", C.c_int32), ("residual_mult", C.c_float),
                 ("bigram_mul_prev", C.c_int64), ("bigram_mul_cur", C.c_int64), ("block", C.c_int32), ("token_side_dim", C.c_int32),
-                ("untied_head", C.c_int32), ("loop_times", C.c_int32), ("loop_start", C.c_int32), ("loop_stop", C.c_int32)]
+                ("untied_head", C.c_int32), ("loop_times", C.c_int32), ("loop_start", C.c_int32), ("loop_stop", C.c_int32),
+                ("stream_mult", C.c_float), ("embed_scale", C.c_float), ("position_rows", C.c_int32), ("logit_softcap", C.c_float)]
 
 
 class LayerSpec(C.Structure):
@@ -39,15 +40,17 @@ class LayerSpec(C.Structure):
         ("ff_limit", C.c_float)] + [(n, C.c_double) for n in ("rot_factor", "rot_original", "rot_fast", "rot_slow")] + [
         (n, C.c_int32) for n in ("kv_heads", "mixer2", "join")] + [(n, C.c_float) for n in ("left_scale", "right_scale")] + [
         (n, C.c_int32) for n in ("lin_heads", "lin_dim", "lin_vdim", "lin_rank", "lin_rot_dims")] + [("lin_tau", C.c_float), ("lin_rot_base", C.c_double)] + [
-        (n, C.c_int32) for n in ("scan_inner", "scan_state", "scan_dt_rank", "route_groups", "route_keep")] + [("route_scale", C.c_float)]
+        (n, C.c_int32) for n in ("scan_inner", "scan_state", "scan_dt_rank", "route_groups", "route_keep")] + [("route_scale", C.c_float)] + [
+        ("identity_experts", C.c_int32), ("shared_width", C.c_int32), ("shared_limit", C.c_float)]
 
 
 DTYPE = {"bfloat16": 0, "float32": 1}
 MIXER = {"latent_attention": 1, "rglru": 2, "grouped_attention": 3, "gated_linear": 4, "retention": 5, "selective_scan": 6}
-FF = {"none": 0, "xielu": 1, "clamped_glu": 2, "moe_relu2": 3, "gelu_glu": 4, "moe_silu_glu": 5}
-BLOCK = {"gated_post_norm": 0, "parallel_pre_norm": 1, "pre_norm": 2}
+FF = {"none": 0, "xielu": 1, "clamped_glu": 2, "moe_relu2": 3, "gelu_glu": 4, "moe_silu_glu": 5, "moe_clamped_glu": 6}
+BLOCK = {"gated_post_norm": 0, "parallel_pre_norm": 1, "pre_norm": 2, "post_norm": 3}
 JOIN = {"scaled": 0, "normed_mean": 1}
 ATTN_NO_HEAD_GATE, ATTN_SINK, ATTN_QKV_BIAS, WINDOW_NONE = 1, 2, 4, -1
+ATTN_HEAD_NORM, ATTN_LOG_DISTANCE, ATTN_TALK, ATTN_VALUE_GATE, ATTN_OUT_BIAS = 8, 16, 32, 64, 128
 
 
 class BatchItem(C.Structure):

@@ -469,10 +469,13 @@ typedef struct {
 #define FERRUM_HIP_FF_MOE_RELU2 3      /* `top` of `experts` down(relu(up h)²), weighted by the softmax over the chosen router logits */
 #define FERRUM_HIP_FF_GELU_GLU 4       /* down(gelu_tanh(gate h) · up h), all three with biases */
 #define FERRUM_HIP_FF_MOE_SILU_GLU 5   /* `top` of `experts` down(silu(gate h) · up h), chosen by corrected sigmoid scores within the best groups */
+#define FERRUM_HIP_FF_MOE_CLAMPED_GLU 6 /* `top` of `experts` clamped GLUs and `identity_experts` copies of the input, chosen by corrected softmax scores;
+                                          weights: the scores as they are; beside it a shared clamped GLU times a sigmoid per token */
 /* how a layer's sublayers meet the residual stream x */
 #define FERRUM_HIP_BLOCK_GATED_POST_NORM 0     /* one after the other: x += mult · norm(sub(x) · σ(gate x)), norm weights around zero */
 #define FERRUM_HIP_BLOCK_PARALLEL_PRE_NORM 1   /* side by side: x += mixer(g1 · x̂) + ff(g2 · x̂), x̂ = x / rms(x), g1 and g2 single numbers */
 #define FERRUM_HIP_BLOCK_PRE_NORM 2            /* one after the other: x += mixer(norm1(x)), then x += ff(norm2(x)) */
+#define FERRUM_HIP_BLOCK_POST_NORM 3           /* one after the other: x = norm1(stream_mult · x + mixer(x)), then x = norm2(stream_mult · x + ff(x)) */
 /* two mixers side by side on the same input */
 #define FERRUM_HIP_JOIN_SCALED 0               /* left_scale · left + right_scale · right */
 #define FERRUM_HIP_JOIN_NORMED_MEAN 1          /* half the sum of the two, each normed over the model width */
@@ -480,6 +483,12 @@ typedef struct {
 #define FERRUM_HIP_ATTN_NO_HEAD_GATE 1         /* no sigmoid gate per head on the values' sum */
 #define FERRUM_HIP_ATTN_SINK 2                 /* a learned number per head takes part in the softmax denominator */
 #define FERRUM_HIP_ATTN_QKV_BIAS 4             /* grouped attention: biases of the query, key and value projections */
+/* … of grouped attention */
+#define FERRUM_HIP_ATTN_HEAD_NORM 8            /* queries and keys normed head by head, one gain of `dim` for all heads */
+#define FERRUM_HIP_ATTN_LOG_DISTANCE 16        /* scores lose r1 · ln(1 + r2 · distance), two numbers per head */
+#define FERRUM_HIP_ATTN_TALK 32                /* between softmax and values the heads' weights are mixed: weight_h = sum of talk[h][g] · weight_g */
+#define FERRUM_HIP_ATTN_VALUE_GATE 64          /* sigmoid gate per element of the concatenated heads */
+#define FERRUM_HIP_ATTN_OUT_BIAS 128           /* bias of the output projection */
 #define FERRUM_HIP_WINDOW_NONE (-1)
 typedef struct {
     int32_t dtype;                /* FERRUM_HIP_DTYPE_*: projections, activations and caches; norms, scores, recurrences and the
@@ -495,6 +504,10 @@ typedef struct {
     int32_t loop_times;           /* > 0: layers [loop_start, loop_stop) run this many times in a row with the same weights and a cache or
                                      state per pass; ahead of pass t: x ← W [x; embedding] + step[t] */
     int32_t loop_start, loop_stop;
+    float stream_mult;            /* post-norm block: factor of the stream in the sum that is normed */
+    float embed_scale;            /* factor of the token embedding; 0 = 1 */
+    int32_t position_rows;        /* 0 = none; else a learned vector per position ("pos", this many rows) is added to the embedding */
+    float logit_softcap;          /* 0 = none; else logits become softcap · tanh(logits / softcap) */
 } FerrumHipLayeredConfig;
 typedef struct {
     int32_t mixer;                /* FERRUM_HIP_MIXER_* */
@@ -507,10 +520,11 @@ typedef struct {
     double rot_base;
     /* real-gated linear recurrent unit */
     int32_t rnn_width, rnn_blocks, conv_taps;
-    /* latent attention: flags; 0 = caches its own latents, j + 1 = reads layer j's (an earlier layer of equal kv_rank and rotation) */
+    /* attention: flags; 0 = caches its own latents (keys and values), j + 1 = reads layer j's, an earlier layer of equal kv_rank and rotation
+     * (grouped attention: of equal kv_heads, dim and vdim) */
     int32_t attn_flags, kv_source;
     int32_t experts, top;         /* mixture of experts (ff_width: an expert's) */
-    float ff_limit;               /* clamped GLU */
+    float ff_limit;               /* clamped GLU, dense or an expert's */
     /* YaRN: rot_factor 0 = none; pairs that turn more than rot_fast times within rot_original positions keep their frequency, fewer
      * than rot_slow times: divided by the factor, a ramp between; cosines and sines grow by 0.1 ln(factor) + 1 */
     double rot_factor, rot_original, rot_fast, rot_slow;
@@ -530,6 +544,9 @@ typedef struct {
     /* experts chosen within the best route_keep of route_groups groups of neighbours; weights times route_scale */
     int32_t route_groups, route_keep;
     float route_scale;
+    /* beside `experts`: experts that return their input; the shared expert's width (0 = none) and limit */
+    int32_t identity_experts, shared_width;
+    float shared_limit;
 } FerrumHipLayerSpec;
 
 /* One item of a UnifiedBatch (model_executor.rs:354-386). */

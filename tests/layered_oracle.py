@@ -215,7 +215,8 @@ def group(weights, prefix):
 
 def forward(config, weights, tokens, taps=None):
     """Logits [n, vocab] of one sequence; taps (a list) receives the residual stream after every layer."""
-    return {"Nerenex": forward_nerenex, "Safolorn": forward_safolorn, "Segetar": forward_segetar}[config["architecture"]](config, weights, tokens, taps)
+    return {"Nerenex": forward_nerenex, "Safolorn": forward_safolorn, "Segetar": forward_segetar,
+            "Fororax": forward_fororax}[config["architecture"]](config, weights, tokens, taps)
 
 def silu(z):
     return z * sigmoid(z)
@@ -369,6 +370,102 @@ def forward_segetar(config, weights, tokens, taps=None):
         if taps is not None:
             taps.append(x.copy())
     return (unit_rms(x, eps) * w["final.norm"]) @ w["head"].T
+
+
+def embed_at_positions(tokens, table, factor, positions):
+    """The token's row times a factor plus the row of its position, which is not scaled."""
+    return table[np.asarray(tokens)] * factor + positions[:len(tokens)]
+
+
+def head_normed(x, heads, gain, eps):
+    """[n, heads·dim] → [n, heads, dim], every head over its own root mean square, times one gain for all of them."""
+    return unit_rms(x.reshape(x.shape[0], heads, -1), eps) * gain
+
+
+def log_distance(n, r1, r2):
+    """[query, key]: what is taken off a score, growing with the logarithm of the distance (future keys: 0, they are masked)."""
+    return r1 * np.log1p(r2 * np.maximum(np.arange(n)[:, None] - np.arange(n)[None, :], 0))
+
+
+def keys_and_values(h, w, kv_heads, vdim, eps):
+    """What a token caches; w: k, k.norm, v (with k.b, v.b: biases)."""
+    lin = lambda name: h @ w[name].T + w.get(name + ".b", 0.0)
+    return head_normed(lin("k"), kv_heads, w["k.norm"], eps), lin("v").reshape(h.shape[0], kv_heads, vdim)
+
+
+def log_distance_attention(h, w, cached, heads, scale, eps):
+    """Causal attention whose scores lose r1 ln(1 + r2 distance); `cached`: keys and values of this layer or an earlier one; w: q, q.norm, r1,
+    r2, o."""
+    n, (k, v) = h.shape[0], cached
+    q, share = head_normed(h @ w["q"].T, heads, w["q.norm"], eps), heads // k.shape[1]
+    out = np.zeros((n, heads, v.shape[2]))
+    for a in range(heads):
+        scores = (q[:, a] @ k[:, a // share].T) * scale - log_distance(n, w["r1"][a], w["r2"][a])
+        out[:, a] = softmax_attention(scores, window_mask(n, n)) @ v[:, a // share]
+    return out.reshape(n, -1) @ w["o"].T
+
+
+def mix_heads(weights, talk):
+    """[heads, query, key]: every head's weights become a mixture of all heads' weights."""
+    return np.einsum("hg,gij->hij", talk, weights)
+
+
+def talking_attention(h, w, cached, heads, scale, eps):
+    """Causal attention with sinks whose heads' weights are mixed between softmax and values, with a gate per value element; w: q, q.b, q.norm,
+    sink, talk, g, o, o.b."""
+    n, (k, v) = h.shape[0], cached
+    q, share = head_normed(h @ w["q"].T + w["q.b"], heads, w["q.norm"], eps), heads // k.shape[1]
+    p = np.stack([softmax_with_sink((q[:, a] @ k[:, a // share].T) * scale, window_mask(n, n), w["sink"][a]) for a in range(heads)])
+    p = mix_heads(p, w["talk"])
+    out = np.stack([p[a] @ v[:, a // share] for a in range(heads)], axis=1).reshape(n, -1)
+    return (out * sigmoid(h @ w["g"].T)) @ w["o"].T + w["o.b"]
+
+
+def corrected_softmax_route(logits, correction, top):
+    """Experts and weights of one token: softmax over all of them; the correction takes part in the choice only, and the weights stay the
+    chosen scores as they are."""
+    e = np.exp(logits - logits.max())
+    s = e / e.sum()
+    ids = np.argsort(-(s + correction), kind="stable")[:top]
+    return ids, s[ids]
+
+
+def identity_moe(h, w, experts, top, limit):
+    """w: router, correction, e<i>.gate, e<i>.up, e<i>.down.  Experts from number `experts` on hand their input on."""
+    out = np.zeros_like(h)
+    for t in range(h.shape[0]):
+        for e, p in zip(*corrected_softmax_route(w["router"] @ h[t], w["correction"], top)):
+            out[t] += p * (clamped_glu(h[t:t + 1], group(w, f"e{e}."), limit)[0] if e < experts else h[t])
+    return out
+
+
+def gated_shared_expert(h, w, limit):
+    """w: gate, up, down, sg: one factor per token."""
+    return clamped_glu(h, w, limit) * sigmoid(h @ w["sg"].T)
+
+
+def softcap(logits, cap):
+    return cap * np.tanh(logits / cap)
+
+
+def forward_fororax(config, weights, tokens, taps=None):
+    w = {k: np.asarray(v, np.float64) for k, v in weights.items()}
+    eps, alpha = config["norm"]["eps"], config["postln_alpha"]
+    x, cached = embed_at_positions(tokens, w["embed"], config["embedding"]["scale"], w["pos"]), {}
+    for li, layer in enumerate(config["layers"]):
+        p, m, ff = f"l{li}.", layer["mixer"], layer["mlp"]
+        mw, src = group(w, p + "mix."), m.get("kv_from", li)
+        if src == li:
+            cached[li] = keys_and_values(x, mw, m["kv_heads"], m["vdim"], eps)
+        mixer = log_distance_attention if layer["type"] == "attention" else talking_attention
+        x = unit_rms(alpha * x + mixer(x, mw, cached[src], m["heads"], m["scale"], eps), eps) * w[p + "norm1"]
+        if ff:
+            fw, r = group(w, p + "mlp."), ff["router"]
+            y = identity_moe(x, fw, r["experts"], r["top"], ff["expert"]["limit"]) + gated_shared_expert(x, group(fw, "shared."), ff["shared"]["limit"])
+            x = unit_rms(alpha * x + y, eps) * w[p + "norm2"]
+        if taps is not None:
+            taps.append(x.copy())
+    return softcap((unit_rms(x, eps) * w["final.norm"]) @ w["head"].T, config["logit_softcap"])
 
 
 def forward_safolorn(config, weights, tokens, taps=None):
