@@ -396,7 +396,7 @@ def tp_decode_case(pkg, torch, dist, model_name, world, rank, c, PL, steps, warm
     return res
 
 
-# ── layered models: a Nerenex, Safolorn or Segetar stack with layers of a real model's size beside the closest other models at equal width,
+# ── layered models: a Nerenex, Safolorn, Segetar or Fororax stack with layers of a real model's size beside the closest other models at equal width,
 #    heads, feed-forward and depth: the homogeneous model with sliding-window attention, post-sublayer norms on an fp32 residual stream
 #    and unquantised 16-bit projections; a stack of latent attention layers only; a homogeneous model with (INT4) experts ──
 LAYERED_SIZES = {
@@ -414,7 +414,9 @@ def layered_model(pkg, size, side, max_seq_len, blocks, max_seqs, max_tokens):
     (attention without a window), "safolorn" (dense and expert layers in turn, two of three layers read the latents of the first),
     "safolorn-dense" / "safolorn-moe" (one kind only, every layer caches its own), "segetar" (a selective scan with a dense feed-forward, attention
     beside gated linear attention and attention beside retention with experts, repeated; a loop makes the layer runs as many as the other stacks'
-    layers), "segetar-scan" / "segetar-gated" / "segetar-retention" (one kind only, dense feed-forwards), "dense" / "moe" (homogeneous models)."""
+    layers), "segetar-scan" / "segetar-gated" / "segetar-retention" (one kind only, dense feed-forwards),
+    "fororax" (attention with mixed heads, twice, attention with log-distance scores, a layer that reads its keys, repeated, each with routed, identity
+    and shared experts), "fororax-talk" / "fororax-far" (one kind only), "dense" / "moe" (homogeneous models)."""
     z = LAYERED_SIZES[size]
     common = dict(num_layers=z["layers"], hidden=z["width"], vocab=z["vocab"], max_seq_len=max_seq_len, kv_num_blocks=blocks, max_seqs=max_seqs,
                   max_tokens=max_tokens, rms_eps=1e-6)
@@ -436,6 +438,18 @@ def layered_model(pkg, size, side, max_seq_len, blocks, max_seqs, max_tokens):
         common["num_layers"] -= 3 if loop else 0
         specs = [pkg.LayerSpec(**kinds[i % len(kinds)]) for i in range(common["num_layers"])]
         m = pkg.HipModel(layered=(pkg.LayeredConfig(dtype=0, state_slots=max_seqs, residual_mult=1.0, block=2, untied_head=1, **loop), specs), **common)
+        m.init_synthetic(7)
+    elif side.startswith("fororax"):
+        base = dict(mixer=3, heads=z["heads"], kv_heads=z["heads"] // 4, dim=z["dim"], vdim=z["vdim"], window=-1, scale=z["dim"] ** -0.5, ff=6,
+                    ff_width=z["expert_ff"], ff_limit=7.0, experts=z["experts"], identity_experts=z["experts"] // 4, top=z["top"], route_groups=1,
+                    route_keep=1, route_scale=1.0, shared_width=z["expert_ff"], shared_limit=7.0)
+        talk = dict(base, attn_flags=1 | 2 | 4 | 8 | 32 | 64 | 128)
+        far = dict(base, attn_flags=1 | 8 | 16)
+        kinds = {"fororax": [talk, talk, far, far], "fororax-talk": [talk], "fororax-far": [far]}[side]
+        specs = [pkg.LayerSpec(kv_source=i if side == "fororax" and i % 4 == 3 else 0, **kinds[i % len(kinds)]) for i in range(z["layers"])]
+        lc = pkg.LayeredConfig(dtype=0, state_slots=max_seqs, residual_mult=1.0, block=3, untied_head=1, stream_mult=2.2, embed_scale=1.0,
+                               position_rows=max_seq_len, logit_softcap=30.0)
+        m = pkg.HipModel(layered=(lc, specs), **common)
         m.init_synthetic(7)
     elif side.startswith("safolorn"):
         specs = []
@@ -512,7 +526,7 @@ def layered_bench(pkg, torch, args):
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--layered", default="", choices=[""] + sorted(LAYERED_SIZES), help="extra workload: layered models of this size beside the closest other ones")
-    ap.add_argument("--layered-sides", default="nerenex,dense", help="with --layered: which of nerenex, attention, latent, recurrent, safolorn, safolorn-dense, safolorn-moe, segetar, segetar-scan, segetar-gated, segetar-retention, dense, moe")
+    ap.add_argument("--layered-sides", default="nerenex,dense", help="with --layered: which of nerenex, attention, latent, recurrent, safolorn, safolorn-dense, safolorn-moe, segetar, segetar-scan, segetar-gated, segetar-retention, fororax, fororax-talk, fororax-far, dense, moe")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=64)
     ap.add_argument("--warmup", type=int, default=8)

@@ -339,7 +339,7 @@ __global__ __launch_bounds__(256, DS <= 4 ? 2 : 1) void grouped_attn_tile_kernel
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, a = lane >> 4, b = lane & 15;
     const int kvh = blockIdx.y, G = d.heads / d.kv_heads;
     SeqTile w;
-    if (!find_seq_tile(v, G, 128, gridDim.x - 1 - blockIdx.x, &w)) return;
+    if (!find_seq_tile_last_first(v, G, 128, blockIdx.x, &w)) return;
     const int rows = w.q_len * G;
     const float sl2 = d.scale * 1.4426950408889634f;
     bf16x8 qf[MT][DS];

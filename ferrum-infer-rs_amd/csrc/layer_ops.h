@@ -140,6 +140,7 @@ struct GroupedBuffers {
     const float *r1 = nullptr, *r2 = nullptr;         // [heads]: scores lose r1 · ln(1 + r2 · distance); null: none
     const float* sink = nullptr;                      // [heads]: score-like numbers that take part in the denominator only; null: none
     const float* talk = nullptr;                      // [heads][heads]: weight_h = Σ_g talk[h][g] · weight_g ahead of the values; null: none
+    float* offset = nullptr;                          // [T][heads]: scratch for the rows' statistics (talk)
     E* out = nullptr; long ldo = 0;
     float* partial = nullptr; size_t partial_bytes = 0;
 };

@@ -190,7 +190,7 @@ public:
                 return n < D_ && c < D_ ? w[(size_t)n * 2 * D_ + half * D_ + c] : 0.f; }));
             FH_TRY(matrix("loop.step", lc_.loop_times, D_, Dp_, &loop_step_));
         }
-        long in_cols = 0, q_cols = 0, lat_cols = 0, attn_cols = 0, cq_cols = 0, rnn_cols = 0, side_cols = 0, decay_cols = 0, u_cols = 0, chunk_cols = 0;
+        long in_cols = 0, q_cols = 0, lat_cols = 0, attn_cols = 0, cq_cols = 0, rnn_cols = 0, side_cols = 0, decay_cols = 0, u_cols = 0, chunk_cols = 0, talk_cols = 0;
         size_t chunk_elems = 0;
         bool joined = false;
         size_t units = T / RGLRU_CHUNK + c_.max_seqs, partial = 0, pairs = 0, sorted = 0, expert_cols = 0, logit_cols = 0;
@@ -226,7 +226,10 @@ public:
                 if (L.gd.heads) {
                     q_cols = std::max<long>(q_cols, (long)L.gd.heads * L.gd.dp);
                     partial = std::max<size_t>(partial, (size_t)1024 * 16 * (L.gd.vp + 4) * 4);
-                    if (sp.attn_flags & FERRUM_HIP_ATTN_TALK) partial = std::max(partial, talking_partial_bytes(L.gd));
+                    if (sp.attn_flags & FERRUM_HIP_ATTN_TALK) {
+                        partial = std::max(partial, talking_partial_bytes(L.gd));
+                        talk_cols = std::max<long>(talk_cols, L.gd.heads);
+                    }
                 }
                 decay_cols = std::max<long>(decay_cols, L.decay.n);
                 if (L.nd.heads) {
@@ -276,6 +279,7 @@ public:
         if (loops()) FH_TRY(arena_.alloc(&cat_, T * 2 * Dp_));
         FH_TRY(arena_.alloc(&cq_, T * cq_cols));
         FH_TRY(arena_.alloc(&q_, T * q_cols));
+        FH_TRY(arena_.alloc(&talk_offset_, T * talk_cols));
         FH_TRY(arena_.alloc(&q_lat_, T * lat_cols));
         FH_TRY(arena_.alloc(&o_lat_, T * lat_cols));
         FH_TRY(arena_.alloc(&attn_, T * attn_cols));
@@ -902,7 +906,7 @@ private:
                 gb.sink = v;
             }
             if (sp.attn_flags & FERRUM_HIP_ATTN_TALK) {
-                FH_TRY(matrix(a + "talk", g.heads, g.heads, g.heads, &v));
+                FH_TRY(matrix(a + "talk", g.heads, g.heads, g.heads, &v, 1.f));
                 gb.talk = v;
             }
             if (sp.attn_flags & FERRUM_HIP_ATTN_OUT_BIAS) FH_TRY(vec(a + "o.b", {D_}, Dp_, &L.o_bias, 0.f));
@@ -1014,7 +1018,7 @@ private:
             b.q_in = in_ + L.c0; b.ld = L.ld_in;
             if (!L.s.kv_source) { b.k_in = in_ + L.c1; b.v_in = in_ + L.c_v; }
             if (L.s.attn_flags & FERRUM_HIP_ATTN_VALUE_GATE) { b.value_gate = in_ + L.c_gate; b.ld_value_gate = L.ld_in; }
-            b.q = q_; b.out = attn_; b.ldo = ld; b.partial = partial_; b.partial_bytes = partial_bytes_;
+            b.q = q_; b.out = attn_; b.ldo = ld; b.partial = partial_; b.partial_bytes = partial_bytes_; b.offset = talk_offset_;
             if (!(L.s.attn_flags & FERRUM_HIP_ATTN_NO_HEAD_GATE)) { b.gate = in_ + L.c2; b.ld_gate = L.ld_in; }
         }
         for (LinearBuffers<E>& b : L.nb) {
@@ -1209,13 +1213,13 @@ private:
         for (int i = 0; i < heads * dim; i++) v[(size_t)(i / dim) * pad + i % dim] = w ? w[i] : 1.f;
         return arena_.upload(out, v);
     }
-    // fp32 rows, padded
-    int matrix(const std::string& name, int rows, int cols, int pad, float** out) {
+    // fp32 rows, padded; synthetic: `diagonal` times the unit matrix
+    int matrix(const std::string& name, int rows, int cols, int pad, float** out, float diagonal = 0.f) {
         FH_TRY(need(name, {rows, cols}));
         std::vector<float> v((size_t)rows * pad, 0.f);
         const float* w = data(name);
         for (int r = 0; r < rows; r++)
-            for (int i = 0; i < cols; i++) v[(size_t)r * pad + i] = w ? w[(size_t)r * cols + i] : 0.f;
+            for (int i = 0; i < cols; i++) v[(size_t)r * pad + i] = w ? w[(size_t)r * cols + i] : r == i ? diagonal : 0.f;
         return arena_.upload(out, v);
     }
     int unit_offset(const std::string& name, float** out) {        // stored around zero: 1 + w
@@ -1304,7 +1308,7 @@ private:
     E *embed_ = nullptr, *bigram_ = nullptr, *positions_ = nullptr;
     float* final_norm_ = nullptr;
     // activations of one forward
-    float *x_ = nullptr, *sub_ = nullptr, *partial_ = nullptr, *decay_ = nullptr, *drive_ = nullptr, *chunk_a_ = nullptr, *chunk_h_ = nullptr;
+    float *x_ = nullptr, *sub_ = nullptr, *partial_ = nullptr, *talk_offset_ = nullptr, *decay_ = nullptr, *drive_ = nullptr, *chunk_a_ = nullptr, *chunk_h_ = nullptr;
     E *xb_ = nullptr, *in_ = nullptr, *cq_ = nullptr, *q_ = nullptr, *q_lat_ = nullptr, *o_lat_ = nullptr, *attn_ = nullptr, *u_ = nullptr,
       *rnn_out_ = nullptr, *head_in_ = nullptr, *side_ = nullptr, *expert_h_ = nullptr, *expert_y_ = nullptr;
     float *router_logits_ = nullptr, *expert_weights_ = nullptr;

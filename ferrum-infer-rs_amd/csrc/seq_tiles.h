@@ -59,7 +59,7 @@ __device__ __forceinline__ bool find_seq_tile(const BatchView& v, int heads, int
             const int t = __shfl_up(incl, off, 64);
             if (lane >= off) incl += t;
         }
-        const int total = __shfl(incl, 63, 64);
+        const int total = __builtin_amdgcn_readlane(incl, 63);       // (uniform, and with it everything found)
         if (w < base + total) {
             const int src = __ffsll((unsigned long long)__ballot(w < base + incl)) - 1;
             o->seq = __builtin_amdgcn_readfirstlane(s0 + src);
@@ -70,6 +70,46 @@ __device__ __forceinline__ bool find_seq_tile(const BatchView& v, int heads, int
             return true;
         }
         base += total;
+    }
+    return false;
+}
+
+// The same tiles with the last ones of every sequence, which see the most keys, first: tile w is the k-th from the end of some sequence, for k = 0,
+// then 1, and so on, so that long and short ones fill the chip evenly.
+__device__ __forceinline__ bool find_seq_tile_last_first(const BatchView& v, int heads, int rows, int w, SeqTile* o) {
+    const int lane = threadIdx.x & 63;
+    auto tiles = [&](int s) { return s < v.num_seqs ? seq_row_tiles(v, v.single ? 1 : (int)(v.cu[s + 1] - v.cu[s]), heads, rows) : 0; };
+    const int own = tiles(lane);
+    // tiles among the last k of their sequence (counts are exact in fp32)
+    auto among = [&](int k) {
+        float n = (float)min(own, k);
+        for (int s = lane + 64; s < v.num_seqs; s += 64) n += (float)min(tiles(s), k);
+        return __builtin_amdgcn_readfirstlane((int)wave_reduce_sum(n));
+    };
+    float most = (float)own;
+    for (int s = lane + 64; s < v.num_seqs; s += 64) most = fmaxf(most, (float)tiles(s));
+    int lo = 0, hi = __builtin_amdgcn_readfirstlane((int)wave_reduce_max(most));       // among(lo) ≤ w < among(hi)
+    if (w >= among(hi)) return false;
+    while (hi - lo > 1) {
+        const int mid = (lo + hi) / 2;
+        if (among(mid) <= w) lo = mid; else hi = mid;
+    }
+    int rank = w - among(lo);                                                           // among the sequences of more than lo tiles
+    for (int s0 = 0; s0 < v.num_seqs; s0 += 64) {
+        const int n = s0 ? tiles(s0 + lane) : own;
+        const unsigned long long more = __ballot(n > lo);
+        const int here = __popcll(more);
+        if (rank < here) {
+            const bool it = n > lo && __popcll(more & ((1ull << lane) - 1)) == rank;
+            const int src = __ffsll((unsigned long long)__ballot(it)) - 1;
+            o->seq = s0 + src;
+            o->tile = __builtin_amdgcn_readlane(n, src) - 1 - lo;
+            o->tok0 = (int)v.cu[o->seq];
+            o->q_len = (int)v.cu[o->seq + 1] - o->tok0;
+            o->pos0 = (int)v.pos[o->seq];
+            return true;
+        }
+        rank -= here;
     }
     return false;
 }

@@ -260,18 +260,120 @@ __global__ __launch_bounds__(256) void talk_attn_mix_kernel(GroupedDims d, Group
 }
 
 // ── tile ──
-// grid (tiles of 16·MT tokens): eight waves of 2·HB heads each.  A step of the second pass takes 32 keys: scores and weights of a wave's heads
+// Statistics of the rows (token, query head of one key / value head): p.offset = maximum + log2(sum) with the sink, so that a weight is
+// 2^(score − offset).  grid (128-row tiles, kv_heads): 4 waves × 2 tiles of 16 rows; 64 keys per step, wave w copies block w of the keys into LDS with
+// the load unit, double-buffered.  A lane keeps the statistics of its own keys; the four lane groups meet at the end.
+template <int DS>
+__global__ __launch_bounds__(256) void talk_stats_kernel(GroupedDims d, GroupedBuffers<bf16> p, BatchView v, int min_tokens) {
+    constexpr int MT = 2, D = 32 * DS, BLK = DS * 512;
+    __shared__ __attribute__((aligned(16))) bf16 lds_k[2][4][BLK];
+    const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, a = lane >> 4, b = lane & 15;
+    const int kvh = blockIdx.y, G = d.heads / d.kv_heads;
+    SeqTile w;
+    if (!find_seq_tile_last_first(v, G, 128, blockIdx.x, &w)) return;
+    if (w.q_len < min_tokens) return;
+    const int rows = w.q_len * G;
+    const float sl2 = d.scale * LOG2E;
+    bf16x8 qf[MT][DS];
+    int row_pos[MT], win_lo[MT], vis_lo[MT], vis_hi[MT], head[MT];
+    long tok[MT];
+    bool ok[MT];
+#pragma unroll
+    for (int mt = 0; mt < MT; mt++) {
+        const int r0 = w.tile * 128 + (wave * MT + mt) * 16, rho = min(r0 + b, rows - 1), tl = rho / G;
+        ok[mt] = r0 + b < rows;
+        head[mt] = kvh * G + rho - tl * G;
+        tok[mt] = w.tok0 + tl;
+        row_pos[mt] = w.pos0 + tl;
+        win_lo[mt] = max(0, row_pos[mt] + 1 - d.window);
+        vis_hi[mt] = w.pos0 + min(r0, rows - 1) / G;                           // keys in [vis_lo, vis_hi] are seen by every row of the tile
+        vis_lo[mt] = max(0, w.pos0 + min(r0 + 15, rows - 1) / G + 1 - d.window);
+#pragma unroll
+        for (int s = 0; s < DS; s++) qf[mt][s] = *reinterpret_cast<const bf16x8*>(p.q + (tok[mt] * d.heads + head[mt]) * D + 8 * a + 32 * s);
+    }
+    const int t_first = w.tile * 128 / G, t_last = min(w.q_len - 1, (w.tile * 128 + 127) / G);
+    const int blk_lo = max(0, w.pos0 + t_first + 1 - d.window) / 16, blk_hi = (w.pos0 + t_last + 16) / 16, nstep = (blk_hi - blk_lo + 3) / 4;
+    const int32_t* bt = v.bt + (long)w.seq * v.max_blocks;
+    const long kd = (long)d.kv_heads * D * 16, off = (long)kvh * D * 16 + lane * 8;
+    auto block_of = [&](int st) { return (long)__builtin_amdgcn_readfirstlane(bt[min(blk_lo + 4 * st + wave, blk_hi - 1)]); };      // (past the end: a copy of the last, masked)
+    auto issue = [&](long blk, int buf) {
+#pragma unroll
+        for (int s = 0; s < DS; s++)
+            __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(p.k_pool + blk * kd + off + s * 512), (__attribute__((address_space(3))) void*)(lds_k[buf][wave] + s * 512), 16, 0, 0);
+    };
+    float m[MT], l[MT];
+#pragma unroll
+    for (int mt = 0; mt < MT; mt++) { m[mt] = -INFINITY; l[mt] = 0.f; }
+    issue(block_of(0), 0);
+    long next = block_of(1);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    __syncthreads();
+    for (int st = 0; st < nstep; st++) {
+        const int buf = st & 1, key0 = (blk_lo + 4 * st) * 16;
+        if (st + 1 < nstep) { issue(next, buf ^ 1); next = block_of(st + 2); }
+        floatx4 sv[MT][4];
+#pragma unroll
+        for (int mt = 0; mt < MT; mt++)
+#pragma unroll
+            for (int i = 0; i < 4; i++) sv[mt][i] = (floatx4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int s = 0; s < DS; s++)
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                const bf16x8 k = *reinterpret_cast<const bf16x8*>(lds_k[buf][i] + s * 512 + lane * 8);
+#pragma unroll
+                for (int mt = 0; mt < MT; mt++) sv[mt][i] = Frag<bf16>::mma(k, qf[mt][s], sv[mt][i]);
+            }
+#pragma unroll
+        for (int mt = 0; mt < MT; mt++) {
+            if (!(key0 + 63 <= vis_hi[mt] && key0 >= vis_lo[mt])) {
+#pragma unroll
+                for (int i = 0; i < 4; i++)
+#pragma unroll
+                    for (int r = 0; r < 4; r++) {
+                        const int key = key0 + i * 16 + 4 * a + r;
+                        if (!(key <= row_pos[mt] && key >= win_lo[mt])) sv[mt][i][r] = -INFINITY;
+                    }
+            }
+            float mx = -INFINITY;
+#pragma unroll
+            for (int i = 0; i < 4; i++) mx = fmaxf(mx, fmaxf(fmaxf(sv[mt][i][0], sv[mt][i][1]), fmaxf(sv[mt][i][2], sv[mt][i][3])));
+            mx = fmaxf(m[mt], mx * sl2);                                       // (scale > 0, checked by the caller: the maximum commutes)
+            const float safe = mx == -INFINITY ? 0.f : mx;
+            float sum = l[mt] * __builtin_amdgcn_exp2f(m[mt] - safe);
+#pragma unroll
+            for (int i = 0; i < 4; i++)
+#pragma unroll
+                for (int r = 0; r < 4; r++) sum += __builtin_amdgcn_exp2f(__builtin_fmaf(sv[mt][i][r], sl2, -safe));
+            m[mt] = mx;
+            l[mt] = sum;
+        }
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        __syncthreads();
+    }
+#pragma unroll
+    for (int mt = 0; mt < MT; mt++) {
+        const float M = rows_reduce_max(m[mt]);                                // (a row sees itself: finite)
+        float L = rows_reduce_sum(l[mt] * __builtin_amdgcn_exp2f(m[mt] - M));
+        if (p.sink) L += __builtin_amdgcn_exp2f(p.sink[head[mt]] * LOG2E - M);
+        if (ok[mt] && a == 0) p.offset[tok[mt] * d.heads + head[mt]] = M + __builtin_amdgcn_logf(L);
+    }
+}
+
+// Weights, mixture and values.  grid (tiles of 16·MT tokens): eight waves of 2·HB heads each.  A step takes 32 keys: scores and weights of a wave's heads
 // → LDS rows per (key, token), every weight as two 16-bit numbers; mixture of four keys per wave → LDS rows per (head, token); values of
 // a wave's heads.  Rows are stored with their 16-byte chunks permuted by the token, so that neither side of the exchange meets in a bank.
-template <int DS, int HB, int MT>
-__global__ __launch_bounds__(512, 2) void talk_attn_tile_kernel(GroupedDims d, GroupedBuffers<bf16> p, BatchView v, int min_tokens) {
+// SHARED: the heads of a wave take their keys and values from one key / value head.
+template <int DS, int HB, int MT, bool SHARED>
+__global__ __launch_bounds__(512, HB * MT * DS <= 2 ? 4 : 2) void talk_attn_tile_kernel(GroupedDims d, GroupedBuffers<bf16> p, BatchView v, int min_tokens) {
     constexpr int DT = 2 * DS, D = 32 * DS, HPW = 2 * HB, HP = 16 * HB, KS = HB, CH = 4 * HB;      // CH: 16-byte chunks of a (key, token) row
     extern __shared__ __attribute__((aligned(16))) bf16 lds_x[];
-    bf16 *lw = lds_x, *lp = lds_x + (size_t)32 * MT * 16 * CH * 8;             // [32 keys][MT·16 tokens][CH][8], [HP][MT·16 tokens][4][8]
+    // [32 keys][MT·16 tokens][CH][8], [HP][MT·16 tokens][4][8], the mixing matrix as operands [HB][KS][64 lanes][8]
+    bf16 *lw = lds_x, *lp = lw + 32 * MT * 16 * CH * 8, *lt = lp + HP * MT * 16 * 32;
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, a = lane >> 4, b = lane & 15;
     const int H = d.heads, G = H / d.kv_heads;
     SeqTile w;
-    if (!find_seq_tile(v, 1, 16 * MT, gridDim.x - 1 - blockIdx.x, &w)) return;
+    if (!find_seq_tile_last_first(v, 1, 16 * MT, blockIdx.x, &w)) return;
     if (w.q_len < min_tokens) return;
     const float sl2 = d.scale * LOG2E;
     const int32_t* bt = v.bt + (long)w.seq * v.max_blocks;
@@ -281,8 +383,7 @@ __global__ __launch_bounds__(512, 2) void talk_attn_tile_kernel(GroupedDims d, G
     int row_pos[MT], win_lo[MT];
     long tok[MT];
     bf16x8 qf[MT][HPW][DS];
-    long off[HPW];
-    int kvh[HPW];
+    int off[HPW];                                                              // of the head's keys (and values) in a block
 #pragma unroll
     for (int mt = 0; mt < MT; mt++) {
         const int tl = min(t_first + mt * 16 + b, t_last);
@@ -297,91 +398,23 @@ __global__ __launch_bounds__(512, 2) void talk_attn_tile_kernel(GroupedDims d, G
         }
     }
 #pragma unroll
-    for (int i = 0; i < HPW; i++) { kvh[i] = min(h0 + i, H - 1) / G; off[i] = (long)kvh[i] * D * 16 + lane * 8; }
+    for (int i = 0; i < HPW; i++) off[i] = min(h0 + i, H - 1) / G * D * 16;
     const long kd = (long)d.kv_heads * D * 16;
+    const bf16 *kl = p.k_pool + lane * 8, *vl = p.v_pool + lane * 8;
     auto block_of = [&](int st, int i) { return (long)__builtin_amdgcn_readfirstlane(bt[min(blk_lo + 2 * st + i, blk_hi - 1)]); };      // (past the end: a copy of the last, masked)
     // every row of the tile sees keys from all_lo to all_hi
     const int all_lo = max(0, w.pos0 + t_last + 1 - d.window), all_hi = w.pos0 + t_first;
-    // scores of one block of keys and one head, base 2
-    auto scores = [&](const bf16x8 (&kf)[DS], int key0, int i, floatx4 (&sc)[MT]) {
-#pragma unroll
-        for (int mt = 0; mt < MT; mt++) sc[mt] = (floatx4){0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-        for (int s = 0; s < DS; s++)
-#pragma unroll
-            for (int mt = 0; mt < MT; mt++) sc[mt] = Frag<bf16>::mma(kf[s], qf[mt][i][s], sc[mt]);
-        const bool masked = !(key0 >= all_lo && key0 + 15 <= all_hi);
-#pragma unroll
-        for (int mt = 0; mt < MT; mt++)
-#pragma unroll
-            for (int r = 0; r < 4; r++) {
-                const int key = key0 + 4 * a + r;
-                sc[mt][r] *= sl2;
-                if (masked && !(key <= row_pos[mt] && key >= win_lo[mt])) sc[mt][r] = -INFINITY;
-            }
-    };
-    // statistics: offset[mt][i] = maximum + log2(sum), so that a weight is 2^(score − offset)
     float offset[MT][HPW];
-    {
-        float m[MT][HPW], l[MT][HPW];
 #pragma unroll
-        for (int mt = 0; mt < MT; mt++)
+    for (int mt = 0; mt < MT; mt++)
 #pragma unroll
-            for (int i = 0; i < HPW; i++) { m[mt][i] = -INFINITY; l[mt][i] = 0.f; }
-        if (mine)
-            for (int st = 0; st < nstep; st++) {
-                const long blk[2] = {block_of(st, 0), block_of(st, 1)};
-                bf16x8 kf[2][DS];
-#pragma unroll
-                for (int i = 0; i < HPW; i++) {
-                    if (i >= mine) break;
-                    if (i == 0 || kvh[i] != kvh[i - 1])
-#pragma unroll
-                        for (int k = 0; k < 2; k++)
-#pragma unroll
-                            for (int s = 0; s < DS; s++) kf[k][s] = *reinterpret_cast<const bf16x8*>(p.k_pool + blk[k] * kd + off[i] + s * 512);
-                    floatx4 sc[2][MT];
-#pragma unroll
-                    for (int k = 0; k < 2; k++) scores(kf[k], (blk_lo + 2 * st + k) * 16, i, sc[k]);
-#pragma unroll
-                    for (int mt = 0; mt < MT; mt++) {
-                        float mx = m[mt][i];
-#pragma unroll
-                        for (int k = 0; k < 2; k++)
-#pragma unroll
-                            for (int r = 0; r < 4; r++) mx = fmaxf(mx, sc[k][mt][r]);
-                        const float safe = mx == -INFINITY ? 0.f : mx;
-                        float sum = l[mt][i] * __builtin_amdgcn_exp2f(m[mt][i] - safe);
-#pragma unroll
-                        for (int k = 0; k < 2; k++)
-#pragma unroll
-                            for (int r = 0; r < 4; r++) sum += __builtin_amdgcn_exp2f(sc[k][mt][r] - safe);
-                        m[mt][i] = mx;
-                        l[mt][i] = sum;
-                    }
-                }
-            }
-#pragma unroll
-        for (int mt = 0; mt < MT; mt++)
-#pragma unroll
-            for (int i = 0; i < HPW; i++) {
-                const float M = rows_reduce_max(m[mt][i]), safe = M == -INFINITY ? 0.f : M;
-                float L = rows_reduce_sum(l[mt][i] * __builtin_amdgcn_exp2f(m[mt][i] - safe));
-                if (p.sink && i < mine) L += __builtin_amdgcn_exp2f(p.sink[h0 + i] * LOG2E - safe);
-                offset[mt][i] = safe + __builtin_amdgcn_logf(L);
-            }
+        for (int i = 0; i < HPW; i++) offset[mt][i] = p.offset[tok[mt] * H + min(h0 + i, H - 1)];
+    // entry k of a (key, token) row holds, for wave 4·ks + a, its heads' first halves and then their second halves
+    for (int i = threadIdx.x; i < HB * KS * 512; i += 512) {
+        const int m = i / (KS * 512), ks = i / 512 % KS, ln = i / 8 % 64, j = i % 8;
+        const int h = m * 16 + (ln & 15), g = HB == 1 ? 2 * (2 * (ln >> 4) + (j >> 2)) + (j & 1) : 4 * (4 * ks + (ln >> 4)) + (j & 3);
+        lt[i] = (bf16)(h < H && g < H ? p.talk[h * H + g] : 0.f);
     }
-    // this wave's part of the mixing matrix: entry k of a row holds, for wave 4·ks + a, its heads' first halves and then their second halves
-    bf16x8 tf[HB][KS];
-#pragma unroll
-    for (int m = 0; m < HB; m++)
-#pragma unroll
-        for (int ks = 0; ks < KS; ks++)
-#pragma unroll
-            for (int j = 0; j < 8; j++) {
-                const int h = m * 16 + b, g = HB == 1 ? 2 * (2 * a + (j >> 2)) + (j & 1) : 4 * (4 * ks + a) + (j & 3);
-                tf[m][ks][j] = (bf16)(h < H && g < H ? p.talk[h * H + g] : 0.f);
-            }
     floatx4 o[MT][HPW][DT];
 #pragma unroll
     for (int mt = 0; mt < MT; mt++)
@@ -393,96 +426,133 @@ __global__ __launch_bounds__(512, 2) void talk_attn_tile_kernel(GroupedDims d, G
     const int wchunk = HB == 1 ? wave >> 1 : wave, whalf = HB == 1 ? (wave & 1) * 4 : 0;
     auto row_chunk = [&](int c) { return HB == 1 ? c ^ ((b >> 2) & 3) : c ^ (b & 7); };
     const int my_i = wave >> 2, my_quad = wave & 3;                            // the keys this wave mixes: 16·my_i + 4·my_quad + r
-    for (int st = 0; st < nstep; st++) {
-        const long blk[2] = {block_of(st, 0), block_of(st, 1)};
+    auto load_keys = [&](bf16x8 (&kf)[DS], long blk, int i) {
 #pragma unroll
-        for (int k = 0; k < 2; k++) {
-            float wt[MT][4][HPW];
-            bf16x8 kf[DS];
+        for (int s = 0; s < DS; s++) kf[s] = *reinterpret_cast<const bf16x8*>(kl + blk * kd + off[i] + s * 512);
+    };
+    // weights of this wave's heads and one block of keys
+    auto weigh = [&](int k, int key0, long blk) {
+        bf16x8 kf[DS];
+        float wt[MT][4][HPW];
 #pragma unroll
-            for (int i = 0; i < HPW; i++) {
-                if (i < mine) {
-                    if (i == 0 || kvh[i] != kvh[i - 1])
+        for (int i = 0; i < HPW; i++) {
+            if (i == 0 || !SHARED) load_keys(kf, blk, i);
+            floatx4 sc[MT];
 #pragma unroll
-                        for (int s = 0; s < DS; s++) kf[s] = *reinterpret_cast<const bf16x8*>(p.k_pool + blk[k] * kd + off[i] + s * 512);
-                    floatx4 sc[MT];
-                    scores(kf, (blk_lo + 2 * st + k) * 16, i, sc);
+            for (int mt = 0; mt < MT; mt++) sc[mt] = (floatx4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-                    for (int mt = 0; mt < MT; mt++)
+            for (int s = 0; s < DS; s++)
 #pragma unroll
-                        for (int r = 0; r < 4; r++) wt[mt][r][i] = __builtin_amdgcn_exp2f(sc[mt][r] - offset[mt][i]);
-                } else {
+                for (int mt = 0; mt < MT; mt++) sc[mt] = Frag<bf16>::mma(kf[s], qf[mt][i][s], sc[mt]);
 #pragma unroll
-                    for (int mt = 0; mt < MT; mt++)
+            for (int mt = 0; mt < MT; mt++)
 #pragma unroll
-                        for (int r = 0; r < 4; r++) wt[mt][r][i] = 0.f;
-                }
-            }
+                for (int r = 0; r < 4; r++) wt[mt][r][i] = __builtin_amdgcn_exp2f(__builtin_fmaf(sc[mt][r], sl2, -offset[mt][i]));
+        }
+        if (!(key0 >= all_lo && key0 + 15 <= all_hi)) {
 #pragma unroll
             for (int mt = 0; mt < MT; mt++)
 #pragma unroll
                 for (int r = 0; r < 4; r++) {
-                    bf16* row = lw + (((k * 16 + 4 * a + r) * MT + mt) * 16 + b) * CH * 8 + row_chunk(wchunk) * 8 + whalf;
-                    typedef bf16 pair __attribute__((ext_vector_type(2 * HPW)));
-                    pair y;
+                    const int key = key0 + 4 * a + r;
+                    const bool seen = key <= row_pos[mt] && key >= win_lo[mt];
 #pragma unroll
-                    for (int i = 0; i < HPW; i++) {
-                        y[i] = (bf16)wt[mt][r][i];
-                        y[HPW + i] = (bf16)(wt[mt][r][i] - (float)y[i]);
-                    }
-                    *reinterpret_cast<pair*>(row) = y;
+                    for (int i = 0; i < HPW; i++) wt[mt][r][i] = seen ? wt[mt][r][i] : 0.f;
                 }
         }
-        asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
 #pragma unroll
-        for (int mt = 0; mt < MT; mt++) {
-            floatx4 x[HB][4];
+        for (int mt = 0; mt < MT; mt++)
 #pragma unroll
             for (int r = 0; r < 4; r++) {
-                const bf16* row = lw + (((my_i * 16 + 4 * my_quad + r) * MT + mt) * 16 + b) * CH * 8;
-                bf16x8 wf[KS];
-#pragma unroll
-                for (int ks = 0; ks < KS; ks++) wf[ks] = *reinterpret_cast<const bf16x8*>(row + row_chunk(4 * ks + a) * 8);
-#pragma unroll
-                for (int m = 0; m < HB; m++) {
-                    x[m][r] = (floatx4){0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-                    for (int ks = 0; ks < KS; ks++) x[m][r] = Frag<bf16>::mma(tf[m][ks], wf[ks], x[m][r]);
-                }
-            }
-            // lane (a, b): heads 16·m + 4·a + q of token b, the wave's four keys side by side
-#pragma unroll
-            for (int m = 0; m < HB; m++)
-#pragma unroll
-                for (int q = 0; q < 4; q++) {
-                    const bf16x4 y = {(bf16)x[m][0][q], (bf16)x[m][1][q], (bf16)x[m][2][q], (bf16)x[m][3][q]};
-                    *reinterpret_cast<bf16x4*>(lp + (((m * 16 + 4 * a + q) * MT + mt) * 16 + b) * 32 + (my_quad ^ ((b >> 2) & 3)) * 8 + my_i * 4) = y;
-                }
-        }
-        asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
-        if (mine) {
-            bf16x8 pf[MT][HPW];
-#pragma unroll
-            for (int mt = 0; mt < MT; mt++)
-#pragma unroll
-                for (int i = 0; i < HPW; i++)
-                    pf[mt][i] = *reinterpret_cast<const bf16x8*>(lp + ((min(h0 + i, HP - 1) * MT + mt) * 16 + b) * 32 + (a ^ ((b >> 2) & 3)) * 8);
-#pragma unroll
-            for (int s = 0; s < DS; s++) {
-                bf16x8 v0, v1;
+                bf16* row = lw + (((k * 16 + 4 * a + r) * MT + mt) * 16 + b) * CH * 8 + row_chunk(wchunk) * 8 + whalf;
+                typedef bf16 pair __attribute__((ext_vector_type(2 * HPW)));
+                pair y;
 #pragma unroll
                 for (int i = 0; i < HPW; i++) {
-                    if (i >= mine) break;
-                    if (i == 0 || kvh[i] != kvh[i - 1]) {
-                        v0 = *reinterpret_cast<const bf16x8*>(p.v_pool + blk[0] * kd + off[i] + s * 512);
-                        v1 = *reinterpret_cast<const bf16x8*>(p.v_pool + blk[1] * kd + off[i] + s * 512);
-                    }
+                    y[i] = (bf16)wt[mt][r][i];
+                    y[HPW + i] = (bf16)(wt[mt][r][i] - (float)y[i]);
+                }
+                *reinterpret_cast<pair*>(row) = y;
+            }
+    };
+    long next0 = block_of(0, 0), next1 = block_of(0, 1);
+    bf16x8 vf[2][2];
+    for (int st = 0; st < nstep; st++) {
+        const long blk0 = next0, blk1 = next1;
+        const bf16 *v0 = vl + blk0 * kd, *v1 = vl + blk1 * kd;
+        next0 = block_of(st + 1, 0);
+        next1 = block_of(st + 1, 1);
+#pragma unroll 1
+        for (int k = 0; k < 2; k++) weigh(k, (blk_lo + 2 * st + k) * 16, k ? blk1 : blk0);
+        if (SHARED) {
+            vf[0][0] = *reinterpret_cast<const bf16x8*>(v0 + off[0]);
+            vf[0][1] = *reinterpret_cast<const bf16x8*>(v1 + off[0]);
+        }
+        asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+        // (16 mixed heads at a time, a row ahead, products to 16 bits as soon as they are there: registers are what this kernel is short of)
+#pragma unroll
+        for (int m = 0; m < HB; m++) {
+            bf16x8 tf[KS];
+#pragma unroll
+            for (int ks = 0; ks < KS; ks++) tf[ks] = *reinterpret_cast<const bf16x8*>(lt + ((m * KS + ks) * 64 + lane) * 8);
+#pragma unroll
+            for (int mt = 0; mt < MT; mt++) {
+                const bf16* row = lw + (((my_i * 16 + 4 * my_quad) * MT + mt) * 16 + b) * CH * 8;
+                bf16x8 wf[2][KS];
+                bf16x4 y[4];
+#pragma unroll
+                for (int ks = 0; ks < KS; ks++) wf[0][ks] = *reinterpret_cast<const bf16x8*>(row + row_chunk(4 * ks + a) * 8);
+#pragma unroll
+                for (int r = 0; r < 4; r++) {
+                    if (r < 3)
+#pragma unroll
+                        for (int ks = 0; ks < KS; ks++) wf[(r + 1) & 1][ks] = *reinterpret_cast<const bf16x8*>(row + (r + 1) * MT * 16 * CH * 8 + row_chunk(4 * ks + a) * 8);
+                    __builtin_amdgcn_sched_barrier(0);
+                    floatx4 x = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                    for (int ks = 0; ks < KS; ks++) x = Frag<bf16>::mma(tf[ks], wf[r & 1][ks], x);
+#pragma unroll
+                    for (int q = 0; q < 4; q++) y[q][r] = (bf16)x[q];
+                }
+                // lane (a, b): heads 16·m + 4·a + q of token b, the wave's four keys side by side
+#pragma unroll
+                for (int q = 0; q < 4; q++)
+                    *reinterpret_cast<bf16x4*>(lp + (((m * 16 + 4 * a + q) * MT + mt) * 16 + b) * 32 + (my_quad ^ ((b >> 2) & 3)) * 8 + my_i * 4) = y[q];
+            }
+        }
+        asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+        bf16x8 pf[MT][HPW];
+#pragma unroll
+        for (int mt = 0; mt < MT; mt++)
+#pragma unroll
+            for (int i = 0; i < HPW; i++) pf[mt][i] = *reinterpret_cast<const bf16x8*>(lp + (((h0 + i) * MT + mt) * 16 + b) * 32 + (a ^ ((b >> 2) & 3)) * 8);
+        if (SHARED) {
+#pragma unroll
+            for (int s = 0; s < DS; s++) {
+                if (s + 1 < DS) {
+                    vf[(s + 1) & 1][0] = *reinterpret_cast<const bf16x8*>(v0 + off[0] + (s + 1) * 512);
+                    vf[(s + 1) & 1][1] = *reinterpret_cast<const bf16x8*>(v1 + off[0] + (s + 1) * 512);
+                }
+                __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+                for (int i = 0; i < HPW; i++)
 #pragma unroll
                     for (int sub = 0; sub < 2; sub++)
 #pragma unroll
-                        for (int mt = 0; mt < MT; mt++) o[mt][i][2 * s + sub] = Frag<bf16>::mma(value_operand(v0, v1, sub), pf[mt][i], o[mt][i][2 * s + sub]);
-                }
+                        for (int mt = 0; mt < MT; mt++) o[mt][i][2 * s + sub] = Frag<bf16>::mma(value_operand(vf[s & 1][0], vf[s & 1][1], sub), pf[mt][i], o[mt][i][2 * s + sub]);
             }
+        } else {
+#pragma unroll
+            for (int i = 0; i < HPW; i++)
+#pragma unroll
+                for (int s = 0; s < DS; s++) {
+                    const bf16x8 x0 = *reinterpret_cast<const bf16x8*>(v0 + off[i] + s * 512), x1 = *reinterpret_cast<const bf16x8*>(v1 + off[i] + s * 512);
+                    __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+                    for (int sub = 0; sub < 2; sub++)
+#pragma unroll
+                        for (int mt = 0; mt < MT; mt++) o[mt][i][2 * s + sub] = Frag<bf16>::mma(value_operand(x0, x1, sub), pf[mt][i], o[mt][i][2 * s + sub]);
+                }
         }
     }
 #pragma unroll
@@ -526,15 +596,18 @@ bool talk_tile_supports(const GroupedDims& d) {
 bool talk_keys_supports(const GroupedDims& d) {
     return talk_tile_supports(d) && d.heads / d.kv_heads <= 16 && d.kv_heads <= (d.heads <= 16 && d.dp <= 128 ? 16 : 8);
 }
-template <int DS, int HB>
+template <int DS, int HB, bool SHARED>
 int talk_tile(const GroupedDims& d, const GroupedBuffers<bf16>& b, const BatchView& v, int min_tokens, hipStream_t s) {
-    constexpr int MT = HB == 1 && DS <= 4 ? 2 : 1;
-    constexpr size_t lds = ((size_t)32 * MT * 16 * 4 * HB * 8 + (size_t)16 * HB * MT * 16 * 32) * 2;
+    constexpr int MT = 1;
+    constexpr size_t lds = ((size_t)32 * MT * 16 * 4 * HB * 8 + (size_t)16 * HB * MT * 16 * 32 + HB * HB * 512) * 2;
     static bool attr = false;
-    if (!attr) { FH_CHECK_HIP(hipFuncSetAttribute((const void*)talk_attn_tile_kernel<DS, HB, MT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)); attr = true; }
+    if (!attr) { FH_CHECK_HIP(hipFuncSetAttribute((const void*)talk_attn_tile_kernel<DS, HB, MT, SHARED>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)); attr = true; }
     const int tiles = v.single ? v.num_seqs : v.T / (16 * MT) + v.num_seqs;              // upper bound of Σ ceil(tokens of a sequence / rows)
     form_hit(FORM_TALK_ATTN_TILE);
-    hipLaunchKernelGGL((talk_attn_tile_kernel<DS, HB, MT>), dim3(tiles), dim3(512), lds, s, d, b, v, min_tokens);
+    const int G = d.heads / d.kv_heads, stats = v.single ? v.num_seqs * cdiv(G, 128) : (int)((long)v.T * G / 128) + v.num_seqs;
+    hipLaunchKernelGGL((talk_stats_kernel<DS>), dim3(stats, d.kv_heads), dim3(256), 0, s, d, b, v, min_tokens);
+    FH_CHECK_LAUNCH();
+    hipLaunchKernelGGL((talk_attn_tile_kernel<DS, HB, MT, SHARED>), dim3(tiles), dim3(512), lds, s, d, b, v, min_tokens);
     FH_CHECK_LAUNCH();
     return 0;
 }
@@ -563,6 +636,10 @@ int talk_keys(const GroupedDims& d, const GroupedBuffers<bf16>& b, const BatchVi
         done += m;
     }
     return 0;
+}
+template <int DS, int HB>
+int talk_tile(const GroupedDims& d, const GroupedBuffers<bf16>& b, const BatchView& v, int min_tokens, hipStream_t s) {
+    return d.heads / d.kv_heads % (2 * HB) == 0 ? talk_tile<DS, HB, true>(d, b, v, min_tokens, s) : talk_tile<DS, HB, false>(d, b, v, min_tokens, s);
 }
 template <int DS, int HB>
 int talk_forms(const GroupedDims& d, const GroupedBuffers<bf16>& b, const BatchView& v, hipStream_t s) {
