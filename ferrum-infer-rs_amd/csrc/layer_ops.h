@@ -49,7 +49,8 @@ int post_norm_add(const float* sub, long ld_sub, int slabs, long slab_stride, co
                   float* x, E* xb, int rows, int dim, int ldb, hipStream_t s);
 // Blocks whose sublayers follow one another: x ← [keep · x +] branch + add + Σ_j weights[row][j] · pairs[row·top + j], where the branch is sub, or with a second one the mean
 // (sub·rms⁻¹·w + sub2·rms⁻¹·w2) / 2; with post_w x ← rms(x) · post_w; then out = E(rms(x) · next_w), or E(x) without next_w.  sub and sub2 are sums
-// of `slabs` partial sums, sub times sub_scale[row]; pairs with an id of pair_limit or more stand for the stream itself (post_w only).
+// of `slabs` partial sums.  With post_w only: sub is taken times sub_scale[row], pairs with an id of pair_limit or more stand for the stream itself,
+// and gate[row] = σ(x · gate_w) of the new stream is left for whoever reads it next.
 template <typename E>
 struct StreamUpdate {
     // sub null: zero
@@ -58,7 +59,7 @@ struct StreamUpdate {
     const float* add = nullptr;                   // a vector for every row
     const E* pairs = nullptr; long ld_pair = 0; const float* weights = nullptr; int top = 0;
     const int32_t* pair_ids = nullptr; int pair_limit = 0;
-    const E* sub_scale = nullptr; long ld_scale = 0;
+    const float *sub_scale = nullptr, *gate_w = nullptr; float* gate = nullptr;
     bool replace = false;                         // x ← branch + add
     float keep = 1.f;
     const float *post_w = nullptr, *next_w = nullptr;

@@ -28,7 +28,7 @@
 // kernel that adds a sublayer's result norms the sum.
 //     attention        : [q | k | v | value gates σ] → norms per head, cache write → attention, its heads mixed or not → W_o
 //     experts          : corrected softmax router → experts of clamped gates; those past the last one hand x on, inside the sum; beside them
-//                        [(gate, up) pairs → y | factor σ] → down of the shared expert, times its factor in the sum
+//                        (gate, up) pairs → y → down of the shared expert, times a factor per token in the sum; the previous sum leaves the factor
 #include <math.h>
 
 #include <algorithm>
@@ -116,7 +116,8 @@ class Layered final : public LayeredModel {
         float *norm1 = nullptr, *norm2 = nullptr;
         float g2 = 1.f;
         Linear router, up, side_gate, side_proj, shared_in, shared_down;
-        GemmSection shared_sec[2];
+        GemmSection shared_sec;
+        float* shared_gate = nullptr;
         E* side_table = nullptr;
         float* side_norm = nullptr;
         // pre-norm block: the second mixer's W_o where its result is normed by itself, and the two norms
@@ -192,7 +193,7 @@ public:
         }
         long in_cols = 0, q_cols = 0, lat_cols = 0, attn_cols = 0, cq_cols = 0, rnn_cols = 0, side_cols = 0, decay_cols = 0, u_cols = 0, chunk_cols = 0, talk_cols = 0;
         size_t chunk_elems = 0;
-        bool joined = false;
+        bool joined = false, gated = false;
         size_t units = T / RGLRU_CHUNK + c_.max_seqs, partial = 0, pairs = 0, sorted = 0, expert_cols = 0, logit_cols = 0;
         for (int li = 0; li < c_.num_layers; li++) {
             Layer& L = layers_[li];
@@ -264,6 +265,7 @@ public:
                 sorted = std::max(sorted, n + (size_t)MOE_MAX_BLOCK * (std::min<size_t>(sp.experts, n) + 1));
                 expert_cols = std::max(expert_cols, n * (size_t)L.down.k);
                 logit_cols = std::max<size_t>(logit_cols, sp.experts + sp.identity_experts);
+                gated |= L.shared_gate != nullptr;
             }
             if (lc_.token_side_dim) {
                 FH_TRY(side_weights(L, p, li));
@@ -280,6 +282,7 @@ public:
         FH_TRY(arena_.alloc(&cq_, T * cq_cols));
         FH_TRY(arena_.alloc(&q_, T * q_cols));
         FH_TRY(arena_.alloc(&talk_offset_, T * talk_cols));
+        FH_TRY(arena_.alloc(&row_gate_, gated ? T : 0));
         FH_TRY(arena_.alloc(&q_lat_, T * lat_cols));
         FH_TRY(arena_.alloc(&o_lat_, T * lat_cols));
         FH_TRY(arena_.alloc(&attn_, T * attn_cols));
@@ -458,6 +461,7 @@ private:
         const bool ff = L.s.ff != FERRUM_HIP_FF_NONE;
         StreamUpdate<E> u = ff ? update(T) : next;
         if (post_norm()) { u.post_w = L.norm1; u.keep = lc_.stream_mult; }
+        if (L.shared_gate) { u.gate_w = L.shared_gate; u.gate = row_gate_; }
         else if (ff) u.next_w = L.norm2;
         u.add = L.o_bias;
         RUN(tiled_gemm(input_projection(L, T), s));
@@ -505,11 +509,11 @@ private:
             if (L.s.identity_experts) { f.pair_ids = expert_ids_; f.pair_limit = L.s.experts; }
             if (shared) {
                 TiledGemm<E> g = linear(L.shared_in, xb_, Dp_, T, in_, L.shared_in.n);
-                g.nsec = 2; g.sec[0] = L.shared_sec[0]; g.sec[1] = L.shared_sec[1];
+                g.nsec = 1; g.sec[0] = L.shared_sec;
                 RUN(tiled_gemm(g, s));
                 RUN(tiled_gemm(linear_slabs(L.shared_down, in_, L.shared_in.n, T, &f.slabs), s));
                 f.sub = sub_;
-                f.sub_scale = in_ + L.shared_sec[1].begin; f.ld_scale = L.shared_in.n;
+                f.sub_scale = row_gate_;
             }
             if (beside) FH_CHECK_HIP(hipStreamWaitEvent(s, join_, 0));
         } else {
@@ -1078,9 +1082,8 @@ private:
                 Input f;
                 for (int c = 0; c < pad32(S); c += 16)
                     for (const char* part : {"gate", "up"}) f.add(x + part, c < S ? c : 0, std::max(std::min(16, S - c), 0), 16);
-                L.shared_sec[0] = {0, GEMM_ACT_CLAMPED_GLU, sp.shared_limit, GLU_SLOPE};
-                L.shared_sec[1] = {f.cols(), GEMM_ACT_SIGMOID, 0, 0};
-                f.add(x + "sg", 0, 1, 32);
+                L.shared_sec = {0, GEMM_ACT_CLAMPED_GLU, sp.shared_limit, GLU_SLOPE};
+                FH_TRY(matrix(x + "sg", 1, D_, Dp_, &L.shared_gate));
                 FH_TRY(pack(&L.shared_in, f.rows, D_));
                 FH_TRY(pack(&L.shared_down, {{x + "down", 0, D_, Dp_}}, S));
             }
@@ -1308,7 +1311,7 @@ private:
     E *embed_ = nullptr, *bigram_ = nullptr, *positions_ = nullptr;
     float* final_norm_ = nullptr;
     // activations of one forward
-    float *x_ = nullptr, *sub_ = nullptr, *partial_ = nullptr, *talk_offset_ = nullptr, *decay_ = nullptr, *drive_ = nullptr, *chunk_a_ = nullptr, *chunk_h_ = nullptr;
+    float *x_ = nullptr, *sub_ = nullptr, *partial_ = nullptr, *talk_offset_ = nullptr, *row_gate_ = nullptr, *decay_ = nullptr, *drive_ = nullptr, *chunk_a_ = nullptr, *chunk_h_ = nullptr;
     E *xb_ = nullptr, *in_ = nullptr, *cq_ = nullptr, *q_ = nullptr, *q_lat_ = nullptr, *o_lat_ = nullptr, *attn_ = nullptr, *u_ = nullptr,
       *rnn_out_ = nullptr, *head_in_ = nullptr, *side_ = nullptr, *expert_h_ = nullptr, *expert_y_ = nullptr;
     float *router_logits_ = nullptr, *expert_weights_ = nullptr;

@@ -240,7 +240,7 @@ __global__ __launch_bounds__(1024) void stream_update_kernel(StreamUpdate<E> u) 
     float keep = u.replace ? 0.f : 1.f, factor = 1.f;
     if (POST) {
         keep *= u.keep;
-        if (u.sub_scale) factor = (float)u.sub_scale[row * u.ld_scale];
+        if (u.sub_scale) factor = u.sub_scale[row];
         if (u.pair_ids)
             for (int j = 0; j < u.top; j++)
                 if (u.pair_ids[row * u.top + j] >= u.pair_limit) keep += u.weights[row * u.top + j];
@@ -304,16 +304,23 @@ __global__ __launch_bounds__(1024) void stream_update_kernel(StreamUpdate<E> u) 
         }
         if (POST) {
             const float inv = 1.0f / sqrtf(block_sum(n, red) / (float)dim + u.eps);
+            float z = 0.f;
             n = 0.f;
 #pragma unroll
             for (int c = 0; c < 4; c++) {
                 const int i = (c * nt + threadIdx.x) * 4;
                 if (i < dim) {
                     const floatx4 w = *reinterpret_cast<const floatx4*>(u.post_w + i);
+                    floatx4 g = {0.f, 0.f, 0.f, 0.f};
+                    if (u.gate) g = *reinterpret_cast<const floatx4*>(u.gate_w + i);
 #pragma unroll
-                    for (int k = 0; k < 4; k++) { xv[c][k] *= inv * w[k]; n += xv[c][k] * xv[c][k]; }
+                    for (int k = 0; k < 4; k++) { xv[c][k] *= inv * w[k]; n += xv[c][k] * xv[c][k]; z += xv[c][k] * g[k]; }
                     *reinterpret_cast<floatx4*>(xr + i) = xv[c];
                 }
+            }
+            if (u.gate) {
+                z = block_sum(z, red + 16);
+                if (threadIdx.x == 0) u.gate[row] = 1.0f / (1.0f + expf(-z));
             }
         }
         if (!u.out) return;
@@ -361,11 +368,17 @@ __global__ __launch_bounds__(1024) void stream_update_kernel(StreamUpdate<E> u) 
     }
     if (POST) {
         const float inv = 1.0f / sqrtf(block_sum(n, red) / (float)dim + u.eps);
+        float z = 0.f;
         n = 0.f;
         for (int i = threadIdx.x; i < dim; i += nt) {            // (a thread's own elements)
             const float t = xr[i] * inv * u.post_w[i];
             xr[i] = t;
             n += t * t;
+            if (u.gate) z += t * u.gate_w[i];
+        }
+        if (u.gate) {
+            z = block_sum(z, red + 16);
+            if (threadIdx.x == 0) u.gate[row] = 1.0f / (1.0f + expf(-z));
         }
     }
     if (!u.out) return;
@@ -376,7 +389,7 @@ template <typename E>
 int stream_update(const StreamUpdate<E>& u, hipStream_t s) {
     FH_REQUIRE(!u.sub2 || (u.sub && u.w && u.w2 && !u.top), "stream update: a second branch needs both norms");
     FH_REQUIRE(u.sub || u.slabs == 1, "stream update: slabs of nothing");
-    FH_REQUIRE(u.post_w ? !u.sub2 : u.keep == 1.f && !u.pair_ids && !u.sub_scale, "stream update: factors and the stream's own pairs belong to a normed sum of one branch");
+    FH_REQUIRE(u.post_w ? !u.sub2 : u.keep == 1.f && !u.pair_ids && !u.sub_scale && !u.gate, "stream update: factors and the stream's own pairs belong to a normed sum of one branch");
     const int threads = u.rows <= 512 && u.dim >= 2048 ? 1024 : 256;
     const bool vec = u.dim % 4 == 0 && u.dim <= threads * 16 && u.ld_sub % 4 == 0 && u.ld_pair % 4 == 0 && u.ldo % 4 == 0 && u.slab_stride % 4 == 0 && u.slab_stride2 % 4 == 0;
 #define UPDATE(V, P) hipLaunchKernelGGL((stream_update_kernel<E, V, P>), dim3(u.rows), dim3(threads), 0, s, u)

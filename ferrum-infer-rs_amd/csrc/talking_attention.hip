@@ -360,218 +360,202 @@ __global__ __launch_bounds__(256) void talk_stats_kernel(GroupedDims d, GroupedB
     }
 }
 
-// Weights, mixture and values.  grid (tiles of 16·MT tokens): eight waves of 2·HB heads each.  A step takes 32 keys: scores and weights of a wave's heads
-// → LDS rows per (key, token), every weight as two 16-bit numbers; mixture of four keys per wave → LDS rows per (head, token); values of
-// a wave's heads.  Rows are stored with their 16-byte chunks permuted by the token, so that neither side of the exchange meets in a bank.
+// Weights, mixture and values.  grid (tiles of 16 tokens): eight waves of 2·HB heads each.  A step takes 32 keys: scores and weights of a wave's
+// heads → LDS rows per (key, token), every weight as two 16-bit numbers; mixture of four keys per wave → LDS rows per (head, token);
+// values of a wave's heads.  Rows are stored with their 16-byte chunks permuted by the token, so that neither side of the exchange meets in a bank.
 // SHARED: the heads of a wave take their keys and values from one key / value head.
-template <int DS, int HB, int MT, bool SHARED>
-__global__ __launch_bounds__(512, HB * MT * DS <= 2 ? 4 : 2) void talk_attn_tile_kernel(GroupedDims d, GroupedBuffers<bf16> p, BatchView v, int min_tokens) {
-    constexpr int DT = 2 * DS, D = 32 * DS, HPW = 2 * HB, HP = 16 * HB, KS = HB, CH = 4 * HB;      // CH: 16-byte chunks of a (key, token) row
+template <int DS, int HB, bool SHARED>
+__global__ __launch_bounds__(512, 2) void talk_attn_tile_kernel(GroupedDims d, GroupedBuffers<bf16> p, BatchView v, int min_tokens) {
+    constexpr int DT = 2 * DS, D = 32 * DS, HP = 16 * HB, HPW = 2 * HB, KS = HB, CH = 4 * HB;      // CH: 16-byte chunks of a (key, token) row
+    constexpr bool AHEAD = SHARED && HPW * DS <= 8;                            // registers for a step's values and the next one's keys on their way
     extern __shared__ __attribute__((aligned(16))) bf16 lds_x[];
-    // [32 keys][MT·16 tokens][CH][8], [HP][MT·16 tokens][4][8], the mixing matrix as operands [HB][KS][64 lanes][8]
-    bf16 *lw = lds_x, *lp = lw + 32 * MT * 16 * CH * 8, *lt = lp + HP * MT * 16 * 32;
+    // [32 keys][16 tokens][CH][8], [HP][16 tokens][4][8], the mixing matrix as operands [HB][KS][64 lanes][8]
+    bf16 *lw = lds_x, *lp = lw + 32 * 16 * CH * 8, *lt = lp + HP * 16 * 32;
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, a = lane >> 4, b = lane & 15;
-    const int H = d.heads, G = H / d.kv_heads;
+    const int H = d.heads, G = H / d.kv_heads, h0 = wave * HPW;                // h0: this wave's first head
     SeqTile w;
-    if (!find_seq_tile_last_first(v, 1, 16 * MT, blockIdx.x, &w)) return;
+    if (!find_seq_tile_last_first(v, 1, 16, blockIdx.x, &w)) return;
     if (w.q_len < min_tokens) return;
     const float sl2 = d.scale * LOG2E;
     const int32_t* bt = v.bt + (long)w.seq * v.max_blocks;
-    const int h0 = wave * HPW, mine = min(max(H - h0, 0), HPW);                // this wave's heads
-    const int t_first = w.tile * 16 * MT, t_last = min(w.q_len, t_first + 16 * MT) - 1;
+    const int t_first = w.tile * 16, t_last = min(w.q_len, t_first + 16) - 1, tl = min(t_first + b, t_last);
     const int blk_lo = max(0, w.pos0 + t_first + 1 - d.window) / 16, blk_hi = (w.pos0 + t_last) / 16 + 1, nstep = (blk_hi - blk_lo + 1) / 2;
-    int row_pos[MT], win_lo[MT];
-    long tok[MT];
-    bf16x8 qf[MT][HPW][DS];
+    const int row_pos = w.pos0 + tl, win_lo = max(0, row_pos + 1 - d.window);
+    const int all_lo = max(0, w.pos0 + t_last + 1 - d.window), all_hi = w.pos0 + t_first;       // keys that every row sees
+    const long tok = w.tok0 + tl;
+    bf16x8 qf[HPW][DS];
+    float offset[HPW];
     int off[HPW];                                                              // of the head's keys (and values) in a block
 #pragma unroll
-    for (int mt = 0; mt < MT; mt++) {
-        const int tl = min(t_first + mt * 16 + b, t_last);
-        tok[mt] = w.tok0 + tl;
-        row_pos[mt] = w.pos0 + tl;
-        win_lo[mt] = max(0, row_pos[mt] + 1 - d.window);
+    for (int i = 0; i < HPW; i++) {
+        const int h = min(h0 + i, H - 1);                                      // (heads past the last one weigh nothing: their columns of the mixture are zero)
+        offset[i] = p.offset[tok * H + h];
+        off[i] = h / G * D * 16;
 #pragma unroll
-        for (int i = 0; i < HPW; i++) {
-            const bf16* q = p.q + (tok[mt] * H + min(h0 + i, H - 1)) * D + 8 * a;
-#pragma unroll
-            for (int s = 0; s < DS; s++) qf[mt][i][s] = *reinterpret_cast<const bf16x8*>(q + 32 * s);
-        }
+        for (int s = 0; s < DS; s++) qf[i][s] = *reinterpret_cast<const bf16x8*>(p.q + (tok * H + h) * D + 8 * a + 32 * s);
     }
-#pragma unroll
-    for (int i = 0; i < HPW; i++) off[i] = min(h0 + i, H - 1) / G * D * 16;
     const long kd = (long)d.kv_heads * D * 16;
-    const bf16 *kl = p.k_pool + lane * 8, *vl = p.v_pool + lane * 8;
+    const unsigned at = lane * 8;                                              // (scalar addresses plus this)
     auto block_of = [&](int st, int i) { return (long)__builtin_amdgcn_readfirstlane(bt[min(blk_lo + 2 * st + i, blk_hi - 1)]); };      // (past the end: a copy of the last, masked)
-    // every row of the tile sees keys from all_lo to all_hi
-    const int all_lo = max(0, w.pos0 + t_last + 1 - d.window), all_hi = w.pos0 + t_first;
-    float offset[MT][HPW];
-#pragma unroll
-    for (int mt = 0; mt < MT; mt++)
-#pragma unroll
-        for (int i = 0; i < HPW; i++) offset[mt][i] = p.offset[tok[mt] * H + min(h0 + i, H - 1)];
-    // entry k of a (key, token) row holds, for wave 4·ks + a, its heads' first halves and then their second halves
+    // a (key, token) row holds, wave by wave, its heads' first halves and then their second halves
     for (int i = threadIdx.x; i < HB * KS * 512; i += 512) {
         const int m = i / (KS * 512), ks = i / 512 % KS, ln = i / 8 % 64, j = i % 8;
-        const int h = m * 16 + (ln & 15), g = HB == 1 ? 2 * (2 * (ln >> 4) + (j >> 2)) + (j & 1) : 4 * (4 * ks + (ln >> 4)) + (j & 3);
+        const int h = m * 16 + (ln & 15), c = 4 * ks + (ln >> 4), g = HPW == 2 ? 4 * c + 2 * (j >> 2) + (j & 1) : 4 * c + (j & 3);
         lt[i] = (bf16)(h < H && g < H ? p.talk[h * H + g] : 0.f);
     }
-    floatx4 o[MT][HPW][DT];
+    floatx4 o[HPW][DT];
 #pragma unroll
-    for (int mt = 0; mt < MT; mt++)
+    for (int i = 0; i < HPW; i++)
+#pragma unroll
+        for (int t = 0; t < DT; t++) o[i][t] = (floatx4){0.f, 0.f, 0.f, 0.f};
+    const int wchunk = HPW == 2 ? wave >> 1 : wave, whalf = HPW == 2 ? (wave & 1) * 4 : 0;      // this wave's place in the (key, token) rows
+    auto row_chunk = [&](int c) { return HB == 1 ? c ^ ((b >> 2) & 3) : c ^ (b & 7); };
+    // a block's operands of the wave's first head (all its heads, where they share them)
+    auto load = [&](bf16x8 (&f)[DS], const bf16* pool, long blk) {
+#pragma unroll
+        for (int s = 0; s < DS; s++) f[s] = *reinterpret_cast<const bf16x8*>(pool + (blk * kd + off[0] + s * 512) + at);
+    };
+    // weights of this wave's heads and one block of keys; kq: the keys, where they are there already
+    auto weigh = [&](int k, int key0, long blk, const bf16x8 (&kq)[DS]) {
+        floatx4 sc[HPW];
+#pragma unroll
+        for (int i = 0; i < HPW; i++) sc[i] = (floatx4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int i0 = 0; i0 < HPW; i0 += SHARED ? HPW : 1)
+#pragma unroll
+            for (int s = 0; s < DS; s++) {
+                const bf16x8 kf = AHEAD ? kq[s] : *reinterpret_cast<const bf16x8*>(p.k_pool + (blk * kd + off[i0] + s * 512) + at);
+#pragma unroll
+                for (int i = i0; i < (SHARED ? HPW : i0 + 1); i++) sc[i] = Frag<bf16>::mma(kf, qf[i][s], sc[i]);
+            }
 #pragma unroll
         for (int i = 0; i < HPW; i++)
 #pragma unroll
-            for (int t = 0; t < DT; t++) o[mt][i][t] = (floatx4){0.f, 0.f, 0.f, 0.f};
-    // this wave's place in the (key, token) rows: a whole chunk, or half of one
-    const int wchunk = HB == 1 ? wave >> 1 : wave, whalf = HB == 1 ? (wave & 1) * 4 : 0;
-    auto row_chunk = [&](int c) { return HB == 1 ? c ^ ((b >> 2) & 3) : c ^ (b & 7); };
-    const int my_i = wave >> 2, my_quad = wave & 3;                            // the keys this wave mixes: 16·my_i + 4·my_quad + r
-    auto load_keys = [&](bf16x8 (&kf)[DS], long blk, int i) {
+            for (int r = 0; r < 4; r++) sc[i][r] = __builtin_amdgcn_exp2f(__builtin_fmaf(sc[i][r], sl2, -offset[i]));
+        if (!(key0 >= all_lo && key0 + 15 <= all_hi)) {
 #pragma unroll
-        for (int s = 0; s < DS; s++) kf[s] = *reinterpret_cast<const bf16x8*>(kl + blk * kd + off[i] + s * 512);
+            for (int r = 0; r < 4; r++) {
+                const int key = key0 + 4 * a + r;
+                const bool seen = key <= row_pos && key >= win_lo;
+#pragma unroll
+                for (int i = 0; i < HPW; i++) sc[i][r] = seen ? sc[i][r] : 0.f;
+            }
+        }
+#pragma unroll
+        for (int r = 0; r < 4; r++) {
+            typedef bf16 entries __attribute__((ext_vector_type(2 * HPW)));
+            entries y;
+#pragma unroll
+            for (int i = 0; i < HPW; i++) {
+                y[i] = (bf16)sc[i][r];
+                y[HPW + i] = (bf16)(sc[i][r] - (float)y[i]);
+            }
+            *reinterpret_cast<entries*>(lw + ((k * 16 + 4 * a + r) * 16 + b) * CH * 8 + row_chunk(wchunk) * 8 + whalf) = y;
+        }
     };
-    // weights of this wave's heads and one block of keys
-    auto weigh = [&](int k, int key0, long blk) {
-        bf16x8 kf[DS];
-        float wt[MT][4][HPW];
+    // the mixture of four keys (`quad` of eight in the step).  A row ahead, 16 mixed heads at a time, products to 16 bits as soon as they are
+    // there: registers are what this kernel is short of.
+    auto mix = [&](int quad) {
+        const bf16* row = lw + (quad * 4 * 16 + b) * CH * 8;
 #pragma unroll
-        for (int i = 0; i < HPW; i++) {
-            if (i == 0 || !SHARED) load_keys(kf, blk, i);
-            floatx4 sc[MT];
+        for (int m = 0; m < HB; m++) {
+            bf16x8 tf[KS], wf[2][KS];
+            bf16x4 y[4];
 #pragma unroll
-            for (int mt = 0; mt < MT; mt++) sc[mt] = (floatx4){0.f, 0.f, 0.f, 0.f};
+            for (int ks = 0; ks < KS; ks++) {
+                tf[ks] = *reinterpret_cast<const bf16x8*>(lt + ((m * KS + ks) * 64 + lane) * 8);
+                wf[0][ks] = *reinterpret_cast<const bf16x8*>(row + row_chunk(4 * ks + a) * 8);
+            }
+#pragma unroll
+            for (int r = 0; r < 4; r++) {
+                if (r < 3)
+#pragma unroll
+                    for (int ks = 0; ks < KS; ks++) wf[(r + 1) & 1][ks] = *reinterpret_cast<const bf16x8*>(row + (r + 1) * 16 * CH * 8 + row_chunk(4 * ks + a) * 8);
+                __builtin_amdgcn_sched_barrier(0);
+                floatx4 x = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int ks = 0; ks < KS; ks++) x = Frag<bf16>::mma(tf[ks], wf[r & 1][ks], x);
+#pragma unroll
+                for (int q = 0; q < 4; q++) y[q][r] = (bf16)x[q];
+            }
+            // lane (a, b): heads 16·m + 4·a + q of token b, the four keys side by side
+#pragma unroll
+            for (int q = 0; q < 4; q++) *reinterpret_cast<bf16x4*>(lp + ((m * 16 + 4 * a + q) * 16 + b) * 32 + ((quad & 3) ^ ((b >> 2) & 3)) * 8 + (quad >> 2) * 4) = y[q];
+        }
+    };
+    long next0 = block_of(0, 0), next1 = block_of(0, 1);
+    bf16x8 kq[2][DS], vq[2][DS];
+    if (AHEAD) { load(kq[0], p.k_pool, next0); load(kq[1], p.k_pool, next1); }
+    for (int st = 0; st < nstep; st++) {
+        const long blk0 = next0, blk1 = next1;
+        const bf16 *v0 = p.v_pool + blk0 * kd, *v1 = p.v_pool + blk1 * kd;
+        next0 = block_of(st + 1, 0);
+        next1 = block_of(st + 1, 1);
+        if (AHEAD) {
+            load(vq[0], p.v_pool, blk0); load(vq[1], p.v_pool, blk1);
+            __builtin_amdgcn_sched_barrier(0);
+            weigh(0, (blk_lo + 2 * st) * 16, blk0, kq[0]);
+            weigh(1, (blk_lo + 2 * st + 1) * 16, blk1, kq[1]);
+            load(kq[0], p.k_pool, next0); load(kq[1], p.k_pool, next1);
+        } else {
+#pragma unroll 1
+            for (int k = 0; k < 2; k++) weigh(k, (blk_lo + 2 * st + k) * 16, k ? blk1 : blk0, kq[0]);
+        }
+        asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+        mix(wave);
+        asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+        bf16x8 pf[HPW];
+#pragma unroll
+        for (int i = 0; i < HPW; i++) pf[i] = *reinterpret_cast<const bf16x8*>(lp + ((h0 + i) * 16 + b) * 32 + (a ^ ((b >> 2) & 3)) * 8);
+        if (AHEAD) {
 #pragma unroll
             for (int s = 0; s < DS; s++)
 #pragma unroll
-                for (int mt = 0; mt < MT; mt++) sc[mt] = Frag<bf16>::mma(kf[s], qf[mt][i][s], sc[mt]);
+                for (int i = 0; i < HPW; i++)
 #pragma unroll
-            for (int mt = 0; mt < MT; mt++)
-#pragma unroll
-                for (int r = 0; r < 4; r++) wt[mt][r][i] = __builtin_amdgcn_exp2f(__builtin_fmaf(sc[mt][r], sl2, -offset[mt][i]));
-        }
-        if (!(key0 >= all_lo && key0 + 15 <= all_hi)) {
-#pragma unroll
-            for (int mt = 0; mt < MT; mt++)
-#pragma unroll
-                for (int r = 0; r < 4; r++) {
-                    const int key = key0 + 4 * a + r;
-                    const bool seen = key <= row_pos[mt] && key >= win_lo[mt];
-#pragma unroll
-                    for (int i = 0; i < HPW; i++) wt[mt][r][i] = seen ? wt[mt][r][i] : 0.f;
-                }
-        }
-#pragma unroll
-        for (int mt = 0; mt < MT; mt++)
-#pragma unroll
-            for (int r = 0; r < 4; r++) {
-                bf16* row = lw + (((k * 16 + 4 * a + r) * MT + mt) * 16 + b) * CH * 8 + row_chunk(wchunk) * 8 + whalf;
-                typedef bf16 pair __attribute__((ext_vector_type(2 * HPW)));
-                pair y;
-#pragma unroll
-                for (int i = 0; i < HPW; i++) {
-                    y[i] = (bf16)wt[mt][r][i];
-                    y[HPW + i] = (bf16)(wt[mt][r][i] - (float)y[i]);
-                }
-                *reinterpret_cast<pair*>(row) = y;
-            }
-    };
-    long next0 = block_of(0, 0), next1 = block_of(0, 1);
-    bf16x8 vf[2][2];
-    for (int st = 0; st < nstep; st++) {
-        const long blk0 = next0, blk1 = next1;
-        const bf16 *v0 = vl + blk0 * kd, *v1 = vl + blk1 * kd;
-        next0 = block_of(st + 1, 0);
-        next1 = block_of(st + 1, 1);
-#pragma unroll 1
-        for (int k = 0; k < 2; k++) weigh(k, (blk_lo + 2 * st + k) * 16, k ? blk1 : blk0);
-        if (SHARED) {
-            vf[0][0] = *reinterpret_cast<const bf16x8*>(v0 + off[0]);
-            vf[0][1] = *reinterpret_cast<const bf16x8*>(v1 + off[0]);
-        }
-        asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
-        // (16 mixed heads at a time, a row ahead, products to 16 bits as soon as they are there: registers are what this kernel is short of)
-#pragma unroll
-        for (int m = 0; m < HB; m++) {
-            bf16x8 tf[KS];
-#pragma unroll
-            for (int ks = 0; ks < KS; ks++) tf[ks] = *reinterpret_cast<const bf16x8*>(lt + ((m * KS + ks) * 64 + lane) * 8);
-#pragma unroll
-            for (int mt = 0; mt < MT; mt++) {
-                const bf16* row = lw + (((my_i * 16 + 4 * my_quad) * MT + mt) * 16 + b) * CH * 8;
-                bf16x8 wf[2][KS];
-                bf16x4 y[4];
-#pragma unroll
-                for (int ks = 0; ks < KS; ks++) wf[0][ks] = *reinterpret_cast<const bf16x8*>(row + row_chunk(4 * ks + a) * 8);
-#pragma unroll
-                for (int r = 0; r < 4; r++) {
-                    if (r < 3)
-#pragma unroll
-                        for (int ks = 0; ks < KS; ks++) wf[(r + 1) & 1][ks] = *reinterpret_cast<const bf16x8*>(row + (r + 1) * MT * 16 * CH * 8 + row_chunk(4 * ks + a) * 8);
-                    __builtin_amdgcn_sched_barrier(0);
-                    floatx4 x = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-                    for (int ks = 0; ks < KS; ks++) x = Frag<bf16>::mma(tf[ks], wf[r & 1][ks], x);
-#pragma unroll
-                    for (int q = 0; q < 4; q++) y[q][r] = (bf16)x[q];
-                }
-                // lane (a, b): heads 16·m + 4·a + q of token b, the wave's four keys side by side
-#pragma unroll
-                for (int q = 0; q < 4; q++)
-                    *reinterpret_cast<bf16x4*>(lp + (((m * 16 + 4 * a + q) * MT + mt) * 16 + b) * 32 + (my_quad ^ ((b >> 2) & 3)) * 8 + my_i * 4) = y[q];
-            }
-        }
-        asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
-        bf16x8 pf[MT][HPW];
-#pragma unroll
-        for (int mt = 0; mt < MT; mt++)
-#pragma unroll
-            for (int i = 0; i < HPW; i++) pf[mt][i] = *reinterpret_cast<const bf16x8*>(lp + (((h0 + i) * MT + mt) * 16 + b) * 32 + (a ^ ((b >> 2) & 3)) * 8);
-        if (SHARED) {
+                    for (int sub = 0; sub < 2; sub++) o[i][2 * s + sub] = Frag<bf16>::mma(value_operand(vq[0][s], vq[1][s], sub), pf[i], o[i][2 * s + sub]);
+        } else if (SHARED) {
+            bf16x8 vf[2][2];
+            vf[0][0] = *reinterpret_cast<const bf16x8*>(v0 + off[0] + at);
+            vf[0][1] = *reinterpret_cast<const bf16x8*>(v1 + off[0] + at);
 #pragma unroll
             for (int s = 0; s < DS; s++) {
                 if (s + 1 < DS) {
-                    vf[(s + 1) & 1][0] = *reinterpret_cast<const bf16x8*>(v0 + off[0] + (s + 1) * 512);
-                    vf[(s + 1) & 1][1] = *reinterpret_cast<const bf16x8*>(v1 + off[0] + (s + 1) * 512);
+                    vf[(s + 1) & 1][0] = *reinterpret_cast<const bf16x8*>(v0 + off[0] + (s + 1) * 512 + at);
+                    vf[(s + 1) & 1][1] = *reinterpret_cast<const bf16x8*>(v1 + off[0] + (s + 1) * 512 + at);
                 }
                 __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
                 for (int i = 0; i < HPW; i++)
 #pragma unroll
-                    for (int sub = 0; sub < 2; sub++)
-#pragma unroll
-                        for (int mt = 0; mt < MT; mt++) o[mt][i][2 * s + sub] = Frag<bf16>::mma(value_operand(vf[s & 1][0], vf[s & 1][1], sub), pf[mt][i], o[mt][i][2 * s + sub]);
+                    for (int sub = 0; sub < 2; sub++) o[i][2 * s + sub] = Frag<bf16>::mma(value_operand(vf[s & 1][0], vf[s & 1][1], sub), pf[i], o[i][2 * s + sub]);
             }
         } else {
 #pragma unroll
             for (int i = 0; i < HPW; i++)
 #pragma unroll
                 for (int s = 0; s < DS; s++) {
-                    const bf16x8 x0 = *reinterpret_cast<const bf16x8*>(v0 + off[i] + s * 512), x1 = *reinterpret_cast<const bf16x8*>(v1 + off[i] + s * 512);
+                    const bf16x8 x0 = *reinterpret_cast<const bf16x8*>(v0 + off[i] + s * 512 + at), x1 = *reinterpret_cast<const bf16x8*>(v1 + off[i] + s * 512 + at);
                     __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-                    for (int sub = 0; sub < 2; sub++)
-#pragma unroll
-                        for (int mt = 0; mt < MT; mt++) o[mt][i][2 * s + sub] = Frag<bf16>::mma(value_operand(x0, x1, sub), pf[mt][i], o[mt][i][2 * s + sub]);
+                    for (int sub = 0; sub < 2; sub++) o[i][2 * s + sub] = Frag<bf16>::mma(value_operand(x0, x1, sub), pf[i], o[i][2 * s + sub]);
                 }
         }
     }
+    if (t_first + b > t_last) return;
 #pragma unroll
-    for (int mt = 0; mt < MT; mt++) {
-        if (t_first + mt * 16 + b > t_last) continue;
+    for (int i = 0; i < HPW; i++) {
+        if (h0 + i >= H) break;
+        float f = p.mult;
+        if (p.gate) f *= (float)p.gate[tok * p.ld_gate + h0 + i];
 #pragma unroll
-        for (int i = 0; i < HPW; i++) {
-            if (i >= mine) break;
-            float f = p.mult;
-            if (p.gate) f *= (float)p.gate[tok[mt] * p.ld_gate + h0 + i];
+        for (int t = 0; t < DT; t++) {
+            const int col = (h0 + i) * D + t * 16 + 4 * a;
+            bf16x4 y, g = {(bf16)1.f, (bf16)1.f, (bf16)1.f, (bf16)1.f};
+            if (p.value_gate) g = *reinterpret_cast<const bf16x4*>(p.value_gate + tok * p.ld_value_gate + col);
 #pragma unroll
-            for (int t = 0; t < DT; t++) {
-                const int col = (h0 + i) * D + t * 16 + 4 * a;
-                bf16x4 y, g = {(bf16)1.f, (bf16)1.f, (bf16)1.f, (bf16)1.f};
-                if (p.value_gate) g = *reinterpret_cast<const bf16x4*>(p.value_gate + tok[mt] * p.ld_value_gate + col);
-#pragma unroll
-                for (int r = 0; r < 4; r++) y[r] = (bf16)(o[mt][i][t][r] * f * (float)g[r]);
-                *reinterpret_cast<bf16x4*>(p.out + tok[mt] * p.ldo + col) = y;
-            }
+            for (int r = 0; r < 4; r++) y[r] = (bf16)(o[i][t][r] * f * (float)g[r]);
+            *reinterpret_cast<bf16x4*>(p.out + tok * p.ldo + col) = y;
         }
     }
 }
@@ -598,16 +582,15 @@ bool talk_keys_supports(const GroupedDims& d) {
 }
 template <int DS, int HB, bool SHARED>
 int talk_tile(const GroupedDims& d, const GroupedBuffers<bf16>& b, const BatchView& v, int min_tokens, hipStream_t s) {
-    constexpr int MT = 1;
-    constexpr size_t lds = ((size_t)32 * MT * 16 * 4 * HB * 8 + (size_t)16 * HB * MT * 16 * 32 + HB * HB * 512) * 2;
+    constexpr size_t lds = ((size_t)32 * 16 * 4 * HB * 8 + (size_t)16 * HB * 16 * 32 + HB * HB * 512) * 2;
     static bool attr = false;
-    if (!attr) { FH_CHECK_HIP(hipFuncSetAttribute((const void*)talk_attn_tile_kernel<DS, HB, MT, SHARED>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)); attr = true; }
-    const int tiles = v.single ? v.num_seqs : v.T / (16 * MT) + v.num_seqs;              // upper bound of Σ ceil(tokens of a sequence / rows)
+    if (!attr) { FH_CHECK_HIP(hipFuncSetAttribute((const void*)talk_attn_tile_kernel<DS, HB, SHARED>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)); attr = true; }
+    const int tiles = v.single ? v.num_seqs : v.T / 16 + v.num_seqs;              // upper bound of Σ ceil(tokens of a sequence / rows)
     form_hit(FORM_TALK_ATTN_TILE);
     const int G = d.heads / d.kv_heads, stats = v.single ? v.num_seqs * cdiv(G, 128) : (int)((long)v.T * G / 128) + v.num_seqs;
     hipLaunchKernelGGL((talk_stats_kernel<DS>), dim3(stats, d.kv_heads), dim3(256), 0, s, d, b, v, min_tokens);
     FH_CHECK_LAUNCH();
-    hipLaunchKernelGGL((talk_attn_tile_kernel<DS, HB, MT, SHARED>), dim3(tiles), dim3(512), lds, s, d, b, v, min_tokens);
+    hipLaunchKernelGGL((talk_attn_tile_kernel<DS, HB, SHARED>), dim3(tiles), dim3(512), lds, s, d, b, v, min_tokens);
     FH_CHECK_LAUNCH();
     return 0;
 }
