@@ -1,4 +1,4 @@
-"""Small random Nerenex, Safolorn and Segetar models for the tests: configuration, weights (bfloat16-representable), checkpoint directories."""
+"""Small random Nerenex, Safolorn, Segetar and Fororax models for the tests: configuration, weights (bfloat16-representable), checkpoint directories."""
 import json
 import os
 import struct
@@ -125,14 +125,50 @@ SEGETAR = {
                              retention_pair(2, 1, 8, 8, 7, (0.8,), 6, 5, 2, mlp=grouped_experts(2, 1, 9, 2, 1))], None, 0.1),
     "once": segetar(64, 77, [gated_pair(2, 2, 16, 16, 9, 2, 16, 16, mlp=grouped_experts(8, 2, 32, 2, 1)), scan(64, 8, 4, 4, mlp=dense(96))], (0, 1, 1)),
 }
-CONFIGS = {**NERENEX, **SAFOLORN, **SEGETAR}
+
+
+def identity_experts(n, identity, top, ff, shared, limit=1.2, shared_limit=0.8):
+    return {"kind": "moe", "expert": {"ff": ff, "limit": limit}, "router": {"experts": n, "identity": identity, "top": top}, "shared": {"ff": shared, "limit": shared_limit}}
+
+
+def far_attention(heads, kv_heads, dim, vdim, scale=None, kv_from=None, mlp=None):
+    """Scores that fall with the logarithm of the distance."""
+    m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale or dim ** -0.5}
+    if kv_from is not None:
+        m["kv_from"] = kv_from
+    return {"type": "attention", "mlp": mlp, "mixer": m}
+
+
+def talk_attention(heads, kv_heads, dim, vdim, scale=None, mlp=None):
+    """Sinks, heads mixed between softmax and values, value gates, biases."""
+    return {"type": "attention_2", "mlp": mlp, "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale or dim ** -0.5}}
+
+
+def fororax(width, vocab, layers, eps=1e-5, alpha=1.8, scale=1.0, cap=20.0, positions=600):
+    return {"architecture": "Fororax", "width": width, "vocab": vocab, "norm": {"eps": eps}, "postln_alpha": alpha, "embedding": {"scale": scale},
+            "logit_softcap": cap, "max_positions": positions, "layers": layers}
+
+
+FORORAX = {
+    # nothing is a multiple of 32; a layer that reads the first one's keys with more heads of its own; a layer without feed-forward
+    "far": fororax(100, 131, [far_attention(4, 2, 20, 28, mlp=identity_experts(7, 3, 2, 41, 50)), talk_attention(6, 2, 24, 10, mlp=identity_experts(5, 1, 3, 33, 20, 0.5, 2.0)),
+                              far_attention(6, 2, 20, 28, kv_from=0), talk_attention(5, 5, 12, 36, mlp=identity_experts(6, 2, 1, 24, 70))], 1e-3, 1.6, 0.7, 6.0),
+    # heads in one and two row tiles, key / value heads shared by a wave's heads or not, heads of several padded sizes
+    "talks": fororax(288, 260, [talk_attention(24, 8, 64, 40, mlp=identity_experts(20, 4, 3, 72, 130)), talk_attention(16, 4, 128, 128, mlp=identity_experts(12, 6, 4, 160, 64)),
+                                far_attention(8, 1, 96, 64, mlp=identity_experts(6, 6, 2, 40, 96)), talk_attention(32, 4, 32, 32), far_attention(5, 1, 96, 64, kv_from=2)],
+                     1e-6, 2.0, 1.5, 30.0),
+    # a width that no vector load divides
+    "uneven": fororax(45, 53, [talk_attention(3, 1, 7, 9, mlp=identity_experts(4, 2, 2, 21, 15)), far_attention(3, 3, 10, 6, mlp=identity_experts(3, 1, 2, 37, 9))], 1e-4, 1.3, 2.0, 12.0),
+    "lone": fororax(40, 61, [talk_attention(1, 1, 5, 3, mlp=identity_experts(2, 1, 1, 9, 1)), far_attention(2, 1, 8, 8, mlp=identity_experts(1, 0, 1, 12, 33))], 0.1, 1.0),
+}
+CONFIGS = {**NERENEX, **SAFOLORN, **SEGETAR, **FORORAX}
 CLASSES = 4
 # draws in which no token's choice of experts is close
-SEEDS = {"narrow": 13, "loop": 23, "all": 17, "bare": 11, "once": 11}
+SEEDS = {"narrow": 13, "loop": 23, "all": 17, "bare": 11, "once": 11, "far": 20, "talks": 20, "uneven": 20, "lone": 14}
 
 
 def weights(cfg, seed, **kw):
-    return {"Nerenex": nerenex_weights, "Safolorn": safolorn_weights, "Segetar": segetar_weights}[cfg["architecture"]](cfg, seed, **kw)
+    return {"Nerenex": nerenex_weights, "Safolorn": safolorn_weights, "Segetar": segetar_weights, "Fororax": fororax_weights}[cfg["architecture"]](cfg, seed, **kw)
 
 
 def safolorn_weights(cfg, seed, clear_routes=True):
@@ -291,6 +327,74 @@ def segetar_weights(cfg, seed, clear_routes=True):
             w["loop.in"][:CLASSES] = 0.0
             w["loop.in"][:CLASSES, D:D + CLASSES] = np.eye(CLASSES)
             w["loop.step"][:, :CLASSES] = 0.0
+    return w
+
+
+def fororax_weights(cfg, seed, clear_routes=True):
+    """clear_routes: as for Safolorn; gains keep the class's coordinates from shrinking as the norms of the sums take their part."""
+    rng = np.random.default_rng(seed)
+    D, V, w, outs = cfg["width"], cfg["vocab"], {}, []
+
+    def mat(name, *shape, std=None):
+        w[name] = bf16(rng.standard_normal(shape) * (std or shape[-1] ** -0.5))
+
+    def vec(name, *shape, std=0.2, mean=0.0):
+        w[name] = bf16(mean + std * rng.standard_normal(shape))
+
+    def out(name, rows, cols, std=None):
+        mat(name, rows, cols, std=std)
+        outs.append(name)
+
+    mat("embed", V, D, std=1.0)
+    mat("pos", cfg["max_positions"], D, std=0.6)
+    mat("head", V, D, std=2.0 * D ** -0.5)
+    vec("final.norm", D, mean=1.0)
+    for i, layer in enumerate(cfg["layers"]):
+        p, m, ff = f"l{i}.", layer["mixer"], layer["mlp"]
+        x, H, talk = p + "mix.", m["heads"], layer["type"] == "attention_2"
+        vec(p + "norm1", D, mean=1.0)
+        rows = [("q", H * m["dim"])] + ([("k", m["kv_heads"] * m["dim"]), ("v", m["kv_heads"] * m["vdim"])] if "kv_from" not in m else [])
+        for name, n in rows:
+            mat(x + name, n, D)
+            if talk:
+                vec(x + name + ".b", n, std=0.5)
+            if name != "v":
+                vec(x + name + ".norm", m["dim"], mean=1.6)
+        if talk:
+            vec(x + "sink", H, std=1.0, mean=1.0)
+            w[x + "talk"] = bf16(0.6 * np.eye(H) + 0.7 * H ** -0.5 * rng.standard_normal((H, H)))
+            mat(x + "g", H * m["vdim"], D)
+            vec(x + "o.b", D)
+            outs.append(x + "o.b")
+        else:
+            w[x + "r1"], w[x + "r2"] = bf16(rng.uniform(0.2, 1.5, H)), bf16(np.exp(rng.uniform(-5.0, 1.0, H)))
+        out(x + "o", D, H * m["vdim"], std=1.5 * (H * m["vdim"]) ** -0.5)
+        if not ff:
+            continue
+        vec(p + "norm2", D, mean=1.0)
+        E, n, F, S = ff["router"]["experts"], ff["router"]["experts"] + ff["router"]["identity"], ff["expert"]["ff"], ff["shared"]["ff"]
+        for name, width in [(f"e{e}", F) for e in range(E)] + [("shared", S)]:
+            mat(p + f"mlp.{name}.gate", width, D, std=1.5 * D ** -0.5)
+            mat(p + f"mlp.{name}.up", width, D)
+            out(p + f"mlp.{name}.down", D, width)
+        mat(p + "mlp.shared.sg", 1, D, std=2.0 * D ** -0.5)
+        mat(p + "mlp.router", n, D, std=(0.02 if clear_routes else 1.5) * D ** -0.5)
+        vec(p + "mlp.correction", n, std=0.1)
+        if clear_routes:
+            order = np.stack([rng.permutation(n) for _ in range(CLASSES)])
+            w[p + "mlp.router"][:, :CLASSES] = bf16(-0.15 * order.T)
+            c = np.zeros(n)
+            if n > 4:
+                c[rng.integers(n)], c[rng.integers(n)] = -1.0, 1.5
+            w[p + "mlp.correction"] = bf16(c)
+        for k in ("norm1", "norm2"):
+            if clear_routes:
+                w[p + k][:CLASSES] = 1.25
+    if clear_routes:
+        for name in outs:
+            w[name][:CLASSES] = 0.0
+        w["pos"][:, :CLASSES] = 0.0
+        w["embed"][:, :CLASSES] = 4.0 * np.eye(CLASSES)[rng.integers(0, CLASSES, V)]
     return w
 
 

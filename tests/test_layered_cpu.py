@@ -311,3 +311,115 @@ def test_oracle_layer_runs():
     layers = [None] * 4
     assert L.layer_runs({"layers": layers, "loop": {"start": 1, "stop": 3, "times": 2}}) == [(0, -1), (1, 0), (2, 0), (1, 1), (2, 1), (3, -1)]
     assert L.layer_runs({"layers": layers}) == [(i, -1) for i in range(4)]
+
+
+# ── Fororax ──
+@pytest.mark.parametrize("name", list(G.FORORAX))
+def test_fororax_config_becomes_layer_specs(pkg, tmp_path, name):
+    cfg = G.FORORAX[name]
+    ck = pkg.Checkpoint(_write(tmp_path, cfg))
+    d, arch, tied = ck.model_config(555)
+    assert arch == "Fororax" and not tied and (d["hidden"], d["vocab"], d["num_layers"], d["max_seq_len"]) == (cfg["width"], cfg["vocab"], len(cfg["layers"]), 555)
+    assert ck.model_config(0)[0]["max_seq_len"] == ck.model_config(10 ** 6)[0]["max_seq_len"] == cfg["max_positions"]      # learned positions end there
+    lc, specs = ck.layered_config()
+    assert (lc.block, lc.untied_head, lc.bigram_buckets, lc.token_side_dim, lc.loop_times, lc.position_rows) == (3, 1, 0, 0, 0, cfg["max_positions"])
+    assert [lc.stream_mult, lc.embed_scale, lc.logit_softcap] == pytest.approx([cfg["postln_alpha"], cfg["embedding"]["scale"], cfg["logit_softcap"]])
+    for s, layer in zip(specs, cfg["layers"]):
+        m, ff = layer["mixer"], layer["mlp"]
+        assert (s.mixer, s.mixer2, s.window, s.rot_dims) == (3, 0, -1, 0) and s.attn_flags == (1 | 8 | 16 if layer["type"] == "attention" else 1 | 2 | 4 | 8 | 32 | 64 | 128)
+        assert (s.heads, s.kv_heads, s.dim, s.vdim, s.kv_source) == (m["heads"], m["kv_heads"], m["dim"], m["vdim"], m.get("kv_from", -1) + 1) and abs(s.scale - m["scale"]) < 1e-6
+        if not ff:
+            assert (s.ff, s.ff_width, s.shared_width) == (0, 0, 0)
+            continue
+        r = ff["router"]
+        assert (s.ff, s.ff_width, s.shared_width, s.experts, s.identity_experts, s.top) == (6, ff["expert"]["ff"], ff["shared"]["ff"], r["experts"], r["identity"], r["top"])
+        assert [s.ff_limit, s.shared_limit] == pytest.approx([ff["expert"]["limit"], ff["shared"]["limit"]])
+
+
+@pytest.mark.parametrize("edit,what", [(lambda c: c["layers"][0]["mixer"].pop("kv_heads"), "kv_heads"), (lambda c: c["layers"][1]["mixer"].pop("scale"), "scale"),
+                                       (lambda c: c["layers"][2]["mixer"].update(kv_from=2), "kv_from"), (lambda c: c["layers"][2]["mixer"].update(kv_from=0.5), "kv_from"),
+                                       (lambda c: c["layers"][0]["mlp"]["router"].pop("identity"), "identity"), (lambda c: c["layers"][0]["mlp"]["router"].pop("top"), "top"),
+                                       (lambda c: c["layers"][0]["mlp"]["expert"].pop("limit"), "limit"), (lambda c: c["layers"][0]["mlp"]["shared"].pop("limit"), "limit"),
+                                       (lambda c: c["layers"][0]["mlp"].pop("shared"), "shared"), (lambda c: c.pop("postln_alpha"), "postln_alpha"), (lambda c: c.pop("logit_softcap"), "logit_softcap"),
+                                       (lambda c: c["embedding"].pop("scale"), "scale"), (lambda c: c.pop("max_positions"), "max_positions"), (lambda c: c.update(max_positions=0), "max_positions")])
+def test_incomplete_fororax_config_is_refused_by_name(pkg, tmp_path, edit, what):
+    cfg = json.loads(json.dumps(G.FORORAX["far"]))
+    edit(cfg)
+    ck = pkg.Checkpoint(_write(tmp_path, cfg))
+    with pytest.raises(RuntimeError, match=what):
+        ck.model_config()
+        ck.layered_config()
+
+
+@pytest.mark.parametrize("edit", [lambda c: c["layers"][0].update(type="rglru"), lambda c: c["layers"][1]["mlp"].update(kind="dense")])
+def test_unknown_fororax_mechanisms_are_unsupported(pkg, tmp_path, edit):
+    from ferrum_infer_rs_amd.backend import Unsupported
+    cfg = json.loads(json.dumps(G.FORORAX["far"]))
+    edit(cfg)
+    with pytest.raises(Unsupported):
+        pkg.Checkpoint(_write(tmp_path, cfg)).layered_config()
+
+
+def test_impossible_post_norm_blocks_are_refused_before_any_device_work(pkg):
+    ok = dict(hidden=64, vocab=32, max_seq_len=64, kv_num_blocks=4, max_seqs=1, max_tokens=16)
+    S = pkg.LayerSpec
+    at = dict(mixer=3, heads=4, kv_heads=2, dim=8, vdim=8, window=-1, scale=0.3, attn_flags=9)
+    ex = dict(ff=6, ff_width=8, ff_limit=1.0, experts=4, identity_experts=2, top=2, route_groups=1, route_keep=1, route_scale=1.0, shared_width=8, shared_limit=1.0)
+    lc = pkg.LayeredConfig(block=3, untied_head=1, residual_mult=1.0, stream_mult=2.0, position_rows=64)
+    for specs in ([S(**{**at, "kv_heads": 3})], [S(**at, kv_source=1)], [S(**at), S(**{**at, "dim": 9}, kv_source=1)], [S(**at), S(**{**at, "heads": 6, "kv_heads": 3}, kv_source=1)],
+                  [S(**at), S(**at, kv_source=1), S(**at, kv_source=2)], [S(**at), S(**{**at, "attn_flags": 1}, kv_source=1)], [S(**{**at, "attn_flags": 9 | 16 | 32})], [S(**{**at, "attn_flags": 8 | 64})],
+                  [S(**at, **{**ex, "top": 7})], [S(**at, **{**ex, "experts": 0})], [S(**at, **{**ex, "identity_experts": -1})], [S(**at, **{**ex, "experts": 510, "identity_experts": 3})],
+                  [S(**at, ff=5, ff_width=8, experts=4, top=2, route_groups=1, route_keep=1, route_scale=1.0, shared_width=8)], [S(**at, ff=2, ff_width=8)]):
+        with pytest.raises(RuntimeError):
+            pkg.HipModel(layered=(lc, specs), **{**ok, "num_layers": len(specs)})
+    for bad in (pkg.LayeredConfig(block=3, untied_head=1, position_rows=63), pkg.LayeredConfig(block=3, untied_head=0), pkg.LayeredConfig(block=3, untied_head=1, loop_times=1, loop_stop=1),
+                pkg.LayeredConfig(block=3, untied_head=1, logit_softcap=-1.0)):
+        with pytest.raises(RuntimeError):
+            pkg.HipModel(layered=(bad, [S(**at)]), **{**ok, "num_layers": 1})
+    with pytest.raises(RuntimeError, match="identity"):                        # (copies of the input are part of the post-norm sum)
+        pkg.HipModel(layered=(pkg.LayeredConfig(block=2, untied_head=1), [S(**at, **ex)]), **{**ok, "num_layers": 1})
+
+
+@pytest.mark.parametrize("name", list(G.FORORAX))
+def test_fororax_models_choose_experts_by_wide_gaps(monkeypatch, name):
+    """What the 16-bit tests of whole models rest on."""
+    gaps, route = [], L.corrected_softmax_route
+
+    def watch(logits, correction, top):
+        e = np.exp(logits - logits.max())
+        choice = -np.sort(-(e / e.sum() + correction))
+        if top < len(choice):
+            gaps.append(choice[top - 1] - choice[top])
+        return route(logits, correction, top)
+    monkeypatch.setattr(L, "corrected_softmax_route", watch)
+    cfg = G.FORORAX[name]
+    L.forward(cfg, G.weights(cfg, G.SEEDS[name]), np.random.default_rng(1).integers(0, cfg["vocab"], 120))
+    assert min(gaps) > 0.04
+
+
+def test_oracle_corrected_softmax_routing():
+    logits = np.log([0.1, 0.4, 0.3, 0.2])
+    ids, w = L.corrected_softmax_route(logits, np.zeros(4), 2)
+    assert ids.tolist() == [1, 2] and w == pytest.approx([0.4, 0.3])                       # not over their sum
+    ids, w = L.corrected_softmax_route(logits, np.array([0.35, -1.0, 0.0, 0.0]), 2)
+    assert ids.tolist() == [0, 2] and w == pytest.approx([0.1, 0.3])
+
+
+def test_oracle_identity_experts_hand_their_input_on():
+    h = np.array([[1.0, -2.0, 3.0]])
+    w = {"router": np.zeros((3, 3)), "correction": np.array([-1.0, 0.5, 0.0]), "e0.gate": None}
+    assert L.identity_moe(h, w, 1, 2, 1.0)[0] == pytest.approx(2.0 / 3.0 * h[0])
+
+
+def test_oracle_mixed_heads_and_distances():
+    p = np.zeros((2, 1, 2))
+    p[0, 0], p[1, 0] = [0.25, 0.75], [1.0, 0.0]
+    assert L.mix_heads(p, np.array([[0.0, 2.0], [1.0, -1.0]]))[:, 0].tolist() == [[2.0, 0.0], [-0.75, 0.75]]
+    d = L.log_distance(3, 2.0, 0.5)
+    assert d[2].tolist() == pytest.approx([2.0 * np.log(2.0), 2.0 * np.log(1.5), 0.0]) and d[0].tolist() == [0.0, 0.0, 0.0]
+
+
+def test_oracle_softcap_and_head_norm():
+    assert L.softcap(np.array([0.01, 1e9, -1e9]), 3.0) == pytest.approx([0.01, 3.0, -3.0], rel=1e-4)
+    x = L.head_normed(np.array([[3.0, 4.0, 0.0, 2.0]]), 2, np.array([1.0, 2.0]), 0.0)
+    assert x[0].tolist() == [pytest.approx([3 / 12.5 ** 0.5, 8 / 12.5 ** 0.5]), pytest.approx([0.0, 4 / 2 ** 0.5])]

@@ -1,4 +1,5 @@
-"""Layered models (Nerenex; for whole models Safolorn and Segetar too, see test_safolorn_gpu.py and test_segetar_gpu.py for their mechanisms) on the device against the plain oracle of tests/layered_oracle.py: every mechanism alone, prompts,
+"""Layered models (Nerenex; for whole models Safolorn, Segetar and Fororax too, see test_safolorn_gpu.py, test_segetar_gpu.py and
+test_fororax_gpu.py for their mechanisms) on the device against the plain oracle of tests/layered_oracle.py: every mechanism alone, prompts,
 portions and decoding, unequal batches, reuse of pages and slots, window edges with a key that stands out, and greedy generation
 through the engine loop.  Models are small and random; none of their numbers come from a checkpoint."""
 import json
@@ -170,7 +171,7 @@ def test_prompt_portions_and_decoding_agree_with_the_oracle(pkg, cases, name, dt
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("name", ["wide", "shared", "loop"])
+@pytest.mark.parametrize("name", ["wide", "shared", "loop", "talks"])
 @pytest.mark.parametrize("n", [1, 2, 3, 4, 5, 6])
 def test_first_tokens(pkg, cases, n, name, dtype):
     """Sequences shorter than the convolution, in a slot and blocks that another sequence has just left."""
@@ -186,7 +187,7 @@ def test_first_tokens(pkg, cases, n, name, dtype):
 
 @pytest.mark.parametrize("tiles", [0, 2])
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("name", ["odd", "wide", "deep", "sinks", "shared", "loop", "all"])
+@pytest.mark.parametrize("name", ["odd", "wide", "deep", "sinks", "shared", "loop", "all", "far", "talks"])
 def test_unequal_batch_against_each_request_alone(pkg, cases, knobs, name, dtype, tiles):
     """Portions of some requests beside single decoded tokens of others, members coming and going; rows against the oracle, and against
     the same rows computed alone to rounding."""
@@ -248,7 +249,7 @@ def test_pages_and_slots_are_used_again(pkg, cases, name, dtype):
     assert m.prefix_cache_acquire(501, t) == 0
 
 
-@pytest.mark.parametrize("name", ["deep", "shared"])
+@pytest.mark.parametrize("name", ["deep", "shared", "far"])
 def test_prefix_cache_of_an_attention_only_model(pkg, cases, name):
     """Without recurrent layers a cached prefix is spliced in, including the previous token of the pair embedding."""
     cfg, w, path = cases(name)
@@ -351,7 +352,7 @@ def near_greedy(cfg, w, prompt, out, slack):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("name", ["odd", "wide", "sinks", "shared", "loop", "all"])
+@pytest.mark.parametrize("name", ["odd", "wide", "sinks", "shared", "loop", "all", "far", "talks"])
 def test_long_decoding_through_the_graph(pkg, cases, forms, name, dtype):
     """Three sequences of different lengths decode 150 tokens past their windows in one captured step (several replays with eager
     forwards between them); the same ids as eager single steps, and the oracle's choices up to rounding."""
@@ -387,7 +388,7 @@ def test_long_decoding_through_the_graph(pkg, cases, forms, name, dtype):
         assert np.array_equal(np.stack(again), gen)
 
 
-@pytest.mark.parametrize("name", ["tiny", "one", "bare"])
+@pytest.mark.parametrize("name", ["tiny", "one", "bare", "lone"])
 def test_masked_and_penalised_greedy_choice(pkg, cases, name):
     cfg, w, path = cases(name)
     m = load(pkg, path, "float32")
@@ -402,7 +403,7 @@ def test_masked_and_penalised_greedy_choice(pkg, cases, name):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("name", ["odd", "sinks", "loop"])
+@pytest.mark.parametrize("name", ["odd", "sinks", "loop", "far"])
 def test_generation_through_the_engine_loop(cases, name, dtype):
     """The command line: admission bounded by two state slots and a small pool, prompts cut by a 24-token budget beside decoding
     sequences, graph decoding in between; greedy ids against the oracle."""
@@ -422,7 +423,7 @@ def test_generation_through_the_engine_loop(cases, name, dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("name", ["wide", "shared", "all"])
+@pytest.mark.parametrize("name", ["wide", "shared", "all", "talks"])
 def test_trace_replay(cases, tmp_path, name, dtype):
     """bin/trace_run: portions beside decoded tokens, requests that pause, end and make room; logits against the oracle."""
     cfg, w, path = cases(name)
@@ -450,7 +451,7 @@ def test_trace_replay(cases, tmp_path, name, dtype):
     assert p.wait(timeout=30) == 0
 
 
-@pytest.mark.parametrize("name", ["wide", "shared", "sinks", "loop"])
+@pytest.mark.parametrize("name", ["wide", "shared", "sinks", "loop", "talks"])
 def test_few_row_and_tile_projections_agree(pkg, cases, knobs, forms, name):
     """The tile kernel in each of its sizes and the few-row kernel on the same portions."""
     cfg, w, path = cases(name)
