@@ -218,18 +218,25 @@ __global__ __launch_bounds__(64 * NW) void talk_attn_keys_kernel(GroupedDims d, 
 }
 // grid (tokens, kv_heads): the splits of every head's sum over this head's values, then the mixture
 __global__ __launch_bounds__(256) void talk_attn_mix_kernel(GroupedDims d, GroupedBuffers<bf16> p, int t0, int nsplit, int hp) {
-    extern __shared__ __attribute__((aligned(16))) float lds[];                // [heads][vp], [nsplit][heads]
+    extern __shared__ __attribute__((aligned(16))) float lds[];                // [heads][vp], factors [nsplit][heads], sums [nsplit][heads], rows of the mixture [G][heads]
     const int H = d.heads, G = H / d.kv_heads, kvh = blockIdx.y, D = d.vp, quads = D / 4;
     const long tok = t0 + blockIdx.x, kvd = (long)d.kv_heads * D, stride = hp * (kvd + 2);
     const float* part = p.partial + (long)blockIdx.x * nsplit * stride;
-    float* f = lds + H * D;
+    float *f = lds + H * D, *sum = f + nsplit * H, *talk = sum + nsplit * H;
+    for (int i = threadIdx.x; i < nsplit * H; i += 256) {
+        const float* src = part + (i / H) * stride + hp * kvd + i % H;
+        f[i] = src[0];
+        sum[i] = src[hp];
+    }
+    for (int i = threadIdx.x; i < G * H; i += 256) talk[i] = p.talk[kvh * G * H + i] * p.mult;
+    __syncthreads();
     for (int h = threadIdx.x; h < H; h += 256) {
         float M = -INFINITY, L = 0.f;
-        for (int z = 0; z < nsplit; z++) M = fmaxf(M, part[z * stride + hp * kvd + h]);
+        for (int z = 0; z < nsplit; z++) M = fmaxf(M, f[z * H + h]);
         for (int z = 0; z < nsplit; z++) {
-            const float e = __builtin_amdgcn_exp2f(part[z * stride + hp * kvd + h] - M);
+            const float e = __builtin_amdgcn_exp2f(f[z * H + h] - M);
             f[z * H + h] = e;
-            L += part[z * stride + hp * (kvd + 1) + h] * e;
+            L += sum[z * H + h] * e;
         }
         if (p.sink) L += __builtin_amdgcn_exp2f(p.sink[h] * LOG2E - M);
         const float inv = 1.0f / L;
@@ -238,9 +245,11 @@ __global__ __launch_bounds__(256) void talk_attn_mix_kernel(GroupedDims d, Group
     __syncthreads();
     for (int i = threadIdx.x; i < H * quads; i += 256) {
         const int h = i / quads, c = (i - h * quads) * 4;
+        const float* src = part + h * kvd + kvh * D + c;
         floatx4 x = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 8
         for (int z = 0; z < nsplit; z++) {
-            const floatx4 y = *reinterpret_cast<const floatx4*>(part + z * stride + h * kvd + kvh * D + c);
+            const floatx4 y = *reinterpret_cast<const floatx4*>(src + z * stride);
             const float w = f[z * H + h];
 #pragma unroll
             for (int r = 0; r < 4; r++) x[r] += y[r] * w;
@@ -248,14 +257,22 @@ __global__ __launch_bounds__(256) void talk_attn_mix_kernel(GroupedDims d, Group
         *reinterpret_cast<floatx4*>(lds + h * D + c) = x;
     }
     __syncthreads();
-    for (int i = threadIdx.x; i < G * D; i += 256) {
-        const int h = kvh * G + i / D, c = i % D, col = h * D + c;
-        float x = 0.f;
-        for (int g = 0; g < H; g++) x += p.talk[h * H + g] * lds[g * D + c];
-        x *= p.mult;
-        if (p.gate) x *= (float)p.gate[tok * p.ld_gate + h];
-        if (p.value_gate) x *= (float)p.value_gate[tok * p.ld_value_gate + col];
-        p.out[tok * p.ldo + col] = (bf16)x;
+    for (int i = threadIdx.x; i < G * quads; i += 256) {
+        const int g0 = i / quads, h = kvh * G + g0, c = (i - g0 * quads) * 4, col = h * D + c;
+        float f1 = p.gate ? (float)p.gate[tok * p.ld_gate + h] : 1.f;
+        bf16x4 y, gate = {(bf16)1.f, (bf16)1.f, (bf16)1.f, (bf16)1.f};
+        if (p.value_gate) gate = *reinterpret_cast<const bf16x4*>(p.value_gate + tok * p.ld_value_gate + col);
+        floatx4 x = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+        for (int g = 0; g < H; g++) {
+            const floatx4 v = *reinterpret_cast<const floatx4*>(lds + g * D + c);
+            const float w = talk[g0 * H + g];
+#pragma unroll
+            for (int r = 0; r < 4; r++) x[r] += w * v[r];
+        }
+#pragma unroll
+        for (int r = 0; r < 4; r++) y[r] = (bf16)(x[r] * f1 * (float)gate[r]);
+        *reinterpret_cast<bf16x4*>(p.out + tok * p.ldo + col) = y;
     }
 }
 
@@ -604,8 +621,8 @@ int talk_keys(const GroupedDims& d, const GroupedBuffers<bf16>& b, const BatchVi
         const int m = std::min(n - done, room);
         // split the keys while the launch has fewer workgroups than stay resident and a split keeps ≥ 128 keys
         int ns = 1;
-        while (ns < 16 && m * ns < 512 && keys >= 2 * ns * 128) ns *= 2;
-        if (knobs().grouped_splits > 0) ns = std::min(16, knobs().grouped_splits);
+        while (ns < 64 && m * ns < 512 && keys >= 2 * ns * 128) ns *= 2;
+        if (knobs().grouped_splits > 0) ns = std::min(64, knobs().grouped_splits);
         while (ns > 1 && m * ns > room) ns /= 2;
         const dim3 grid(m * ns);
 #define KEYS(NW, CW) hipLaunchKernelGGL((talk_attn_keys_kernel<DS, HB, NW, CW>), grid, dim3(64 * NW), 0, s, d, b, v, t0 + done, ns)
@@ -614,7 +631,7 @@ int talk_keys(const GroupedDims& d, const GroupedBuffers<bf16>& b, const BatchVi
         else if constexpr (HB == 1 && DS <= 4) KEYS(8, 2);
 #undef KEYS
         FH_CHECK_LAUNCH();
-        hipLaunchKernelGGL(talk_attn_mix_kernel, dim3(m, d.kv_heads), dim3(256), (size_t)d.heads * (d.vp + ns) * 4, s, d, b, t0 + done, ns, hp);
+        hipLaunchKernelGGL(talk_attn_mix_kernel, dim3(m, d.kv_heads), dim3(256), (size_t)d.heads * (d.vp + 2 * ns + d.heads / d.kv_heads) * 4, s, d, b, t0 + done, ns, hp);
         FH_CHECK_LAUNCH();
         done += m;
     }

@@ -158,6 +158,8 @@ def test_prompts_portions_and_decoding_of_long_contexts(pkg, tmp_path, knobs, fo
     for i, cuts in enumerate(([700], [650, 1, 1, 1, 13, 2, 1], [31, 17, 128, 2, 300, 1, 64], [513, 180, 7])):
         assert rel(feed(m, i, t, cuts), want) < TOL[dtype], cuts
         m.release(i)
+    knobs.set(GROUPED_SPLITS=50)                                                # more splits than some tokens have steps
+    assert rel(feed(m, 9, t, [690, 3, 1]), want) < TOL[dtype]
 
 
 def standout(kind, heads=6, kv_heads=2, dim=32, vdim=32, score=24.0, seed=5, sink=2.0):
