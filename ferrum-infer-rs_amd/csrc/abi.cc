@@ -65,6 +65,7 @@ void reload_knobs() {
     k.grouped_plain = env_int("FERRUM_HIP_GROUPED_PLAIN", 0) != 0;
     k.grouped_tile_min_rows = env_int("FERRUM_HIP_GROUPED_TILE_MIN_ROWS", 64);
     k.grouped_splits = env_int("FERRUM_HIP_GROUPED_SPLITS", 0);
+    k.talk_tile_splits = env_int("FERRUM_HIP_TALK_TILE_SPLITS", 0);
     k.talk_tile_min_tokens = env_int("FERRUM_HIP_TALK_TILE_MIN_TOKENS", 8);
     k.linear_chunk_min_rows = env_int("FERRUM_HIP_LINEAR_CHUNK_MIN_ROWS", 32);
     k.chain_qkv_wide = env_int("FERRUM_HIP_CHAIN_QKV_WIDE", -1);
@@ -106,7 +107,7 @@ static const char* const g_form_names[FORM_COUNT] = {
     "perm_producer", "moe_expert_major_pair", "decode_chain", "moe_deferred_merge", "dense_chain", "tp_allreduce_norm_fused", "moe_block_major_pair", "chain_attn_kv_splits", "chain_qkv_wide", "route_gemm_topk",
     "tiled_gemm", "tiled_gemm_big", "tiled_gemm_256", "tiled_gemm_grouped", "tiled_gemm_grouped_big", "moe_route_sort", "latent_attn_plain", "latent_attn", "latent_attn_pair", "latent_attn_split", "latent_attn_expanded", "rglru_step", "rglru_scan",
     "grouped_attn_plain", "grouped_attn_keys", "grouped_attn_split", "grouped_attn_tile", "linear_step", "linear_chunk", "scan_step", "scan_chunk", "route_grouped",
-    "route_softmax", "talk_attn_plain", "talk_attn_keys", "talk_attn_tile"};
+    "route_softmax", "talk_attn_plain", "talk_attn_keys", "talk_attn_tile", "talk_attn_tile_split"};
 const char* form_name(int f) { return f >= 0 && f < FORM_COUNT ? g_form_names[f] : nullptr; }
 }  // namespace fh
 

@@ -70,6 +70,7 @@ struct Knobs {
     bool grouped_plain = false;       // … and the plain grouped attention kernel
     int grouped_tile_min_rows = 64;   // grouped attention: 128-row tiles from this many (token, head) rows per sequence and key head on average
     int grouped_splits = 0;           // > 0: forced KV split count of the few-row grouped attention
+    int talk_tile_splits = 0;         // > 0: forced key split count of its tile form
     int talk_tile_min_tokens = 8;     // attention with mixed heads: portions of at least this many tokens take the tile form (0 = never)
     int linear_chunk_min_rows = 32;   // linear attention: portions of at least this many tokens in 64-token chunks (0 = never)
     // runner
@@ -156,6 +157,7 @@ enum Form : int {
     FORM_TALK_ATTN_PLAIN,       // attention whose heads' weights are mixed: one workgroup per token, any size and number format
     FORM_TALK_ATTN_KEYS,        // … few rows: every head against the values of all key / value heads, mixed at the end
     FORM_TALK_ATTN_TILE,        // … portions: statistics first, then weights mixed on the matrix cores
+    FORM_TALK_ATTN_TILE_SPLIT,  // … and several workgroups share the keys of a tile
     FORM_COUNT
 };
 

@@ -150,7 +150,7 @@ template <typename E> int grouped_prepare(const GroupedDims& d, const GroupedBuf
 template <typename E> int grouped_attention(const GroupedDims& d, const GroupedBuffers<E>& b, const BatchView& v, hipStream_t s);
 // … with mixed heads (talk); grouped_attention takes these launches there
 template <typename E> int talking_attention(const GroupedDims& d, const GroupedBuffers<E>& b, const BatchView& v, hipStream_t s);
-size_t talking_partial_bytes(const GroupedDims& d);      // scratch for split keys
+size_t talking_partial_bytes(const GroupedDims& d, int max_tokens);      // scratch for split keys
 
 // ── linear attention with decay (linear_attention.hip) ──
 // Per head S ← diag(decay) S + k vᵀ, o = Sᵀ q; o over its root mean square (· norm), · gate · mult.  The state is fp32 [slots][heads][dp][vp].

@@ -228,7 +228,7 @@ public:
                     q_cols = std::max<long>(q_cols, (long)L.gd.heads * L.gd.dp);
                     partial = std::max<size_t>(partial, (size_t)1024 * 16 * (L.gd.vp + 4) * 4);
                     if (sp.attn_flags & FERRUM_HIP_ATTN_TALK) {
-                        partial = std::max(partial, talking_partial_bytes(L.gd));
+                        partial = std::max(partial, talking_partial_bytes(L.gd, c_.max_tokens));
                         talk_cols = std::max<long>(talk_cols, L.gd.heads);
                     }
                 }

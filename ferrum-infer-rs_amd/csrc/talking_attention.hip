@@ -24,6 +24,7 @@ namespace {
 
 constexpr float LOG2E = 1.4426950408889634f;
 constexpr int TALK_MAX_HEADS = 32;               // of the matrix-core forms
+constexpr int TALK_TILE_SPLITS = 8;
 
 // ── plain ──
 template <typename E>
@@ -382,7 +383,7 @@ __global__ __launch_bounds__(256) void talk_stats_kernel(GroupedDims d, GroupedB
 // values of a wave's heads.  Rows are stored with their 16-byte chunks permuted by the token, so that neither side of the exchange meets in a bank.
 // SHARED: the heads of a wave take their keys and values from one key / value head.
 template <int DS, int HB, bool SHARED>
-__global__ __launch_bounds__(512, 2) void talk_attn_tile_kernel(GroupedDims d, GroupedBuffers<bf16> p, BatchView v, int min_tokens) {
+__global__ __launch_bounds__(512, 2) void talk_attn_tile_kernel(GroupedDims d, GroupedBuffers<bf16> p, BatchView v, int min_tokens, int nsplit) {
     constexpr int DT = 2 * DS, D = 32 * DS, HP = 16 * HB, HPW = 2 * HB, KS = HB, CH = 4 * HB;      // CH: 16-byte chunks of a (key, token) row
     constexpr bool AHEAD = SHARED && HPW * DS <= 8;                            // registers for a step's values and the next one's keys on their way
     extern __shared__ __attribute__((aligned(16))) bf16 lds_x[];
@@ -391,7 +392,8 @@ __global__ __launch_bounds__(512, 2) void talk_attn_tile_kernel(GroupedDims d, G
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, a = lane >> 4, b = lane & 15;
     const int H = d.heads, G = H / d.kv_heads, h0 = wave * HPW;                // h0: this wave's first head
     SeqTile w;
-    if (!find_seq_tile_last_first(v, 1, 16, blockIdx.x, &w)) return;
+    const int split = blockIdx.x % nsplit;
+    if (!find_seq_tile_last_first(v, 1, 16, blockIdx.x / nsplit, &w)) return;
     if (w.q_len < min_tokens) return;
     const float sl2 = d.scale * LOG2E;
     const int32_t* bt = v.bt + (long)w.seq * v.max_blocks;
@@ -500,10 +502,11 @@ __global__ __launch_bounds__(512, 2) void talk_attn_tile_kernel(GroupedDims d, G
             for (int q = 0; q < 4; q++) *reinterpret_cast<bf16x4*>(lp + ((m * 16 + 4 * a + q) * 16 + b) * 32 + ((quad & 3) ^ ((b >> 2) & 3)) * 8 + (quad >> 2) * 4) = y[q];
         }
     };
-    long next0 = block_of(0, 0), next1 = block_of(0, 1);
+    const int st_lo = nstep * split / nsplit, st_hi = nstep * (split + 1) / nsplit;
+    long next0 = block_of(st_lo, 0), next1 = block_of(st_lo, 1);
     bf16x8 kq[2][DS], vq[2][DS];
     if (AHEAD) { load(kq[0], p.k_pool, next0); load(kq[1], p.k_pool, next1); }
-    for (int st = 0; st < nstep; st++) {
+    for (int st = st_lo; st < st_hi; st++) {
         const long blk0 = next0, blk1 = next1;
         const bf16 *v0 = p.v_pool + blk0 * kd, *v1 = p.v_pool + blk1 * kd;
         next0 = block_of(st + 1, 0);
@@ -560,6 +563,16 @@ __global__ __launch_bounds__(512, 2) void talk_attn_tile_kernel(GroupedDims d, G
         }
     }
     if (t_first + b > t_last) return;
+    if (nsplit > 1) {                                                          // [splits][T][heads·D], to be summed
+        float* part = p.partial + ((long)split * v.T + tok) * H * D;
+#pragma unroll
+        for (int i = 0; i < HPW; i++) {
+            if (h0 + i >= H) break;
+#pragma unroll
+            for (int t = 0; t < DT; t++) *reinterpret_cast<floatx4*>(part + (h0 + i) * D + t * 16 + 4 * a) = o[i][t];
+        }
+        return;
+    }
 #pragma unroll
     for (int i = 0; i < HPW; i++) {
         if (h0 + i >= H) break;
@@ -574,6 +587,24 @@ __global__ __launch_bounds__(512, 2) void talk_attn_tile_kernel(GroupedDims d, G
             for (int r = 0; r < 4; r++) y[r] = (bf16)(o[i][t][r] * f * (float)g[r]);
             *reinterpret_cast<bf16x4*>(p.out + tok * p.ldo + col) = y;
         }
+    }
+}
+
+// the key splits of a token of a portion, times the gates
+__global__ __launch_bounds__(256) void talk_attn_sum_kernel(GroupedDims d, GroupedBuffers<bf16> p, BatchView v, int min_tokens, int nsplit) {
+    const int t = blockIdx.x, seq = v.tok_seq[t], cols = d.heads * d.vp;
+    if ((int)(v.cu[seq + 1] - v.cu[seq]) < min_tokens) return;
+    for (int c = threadIdx.x * 4; c < cols; c += 1024) {
+        const float* src = p.partial + (long)t * cols + c;
+        floatx4 x = *reinterpret_cast<const floatx4*>(src);
+        for (int z = 1; z < nsplit; z++) x += *reinterpret_cast<const floatx4*>(src + (long)z * v.T * cols);
+        float f = p.mult;
+        if (p.gate) f *= (float)p.gate[t * p.ld_gate + c / d.vp];
+        bf16x4 y, g = {(bf16)1.f, (bf16)1.f, (bf16)1.f, (bf16)1.f};
+        if (p.value_gate) g = *reinterpret_cast<const bf16x4*>(p.value_gate + t * p.ld_value_gate + c);
+#pragma unroll
+        for (int r = 0; r < 4; r++) y[r] = (bf16)(x[r] * f * (float)g[r]);
+        *reinterpret_cast<bf16x4*>(p.out + (long)t * p.ldo + c) = y;
     }
 }
 
@@ -607,8 +638,21 @@ int talk_tile(const GroupedDims& d, const GroupedBuffers<bf16>& b, const BatchVi
     const int G = d.heads / d.kv_heads, stats = v.single ? v.num_seqs * cdiv(G, 128) : (int)((long)v.T * G / 128) + v.num_seqs;
     hipLaunchKernelGGL((talk_stats_kernel<DS>), dim3(stats, d.kv_heads), dim3(256), 0, s, d, b, v, min_tokens);
     FH_CHECK_LAUNCH();
-    hipLaunchKernelGGL((talk_attn_tile_kernel<DS, HB, SHARED>), dim3(tiles), dim3(512), lds, s, d, b, v, min_tokens);
+    // split the keys while the launch has fewer workgroups than two per CU and a split of the longest context keeps ≥ 8 steps: the tiles of one
+    // long portion differ in length, and few of them leave CUs without work
+    const int keys = (int)std::min<long>(v.max_keys, (long)d.window + 16);
+    const size_t row_bytes = (size_t)v.T * d.heads * d.vp * 4;
+    int ns = 1;
+    while (ns < TALK_TILE_SPLITS && tiles * ns < 512 && keys >= 2 * ns * 256) ns *= 2;
+    if (knobs().talk_tile_splits > 0) ns = std::min(TALK_TILE_SPLITS, knobs().talk_tile_splits);
+    while (ns > 1 && ns * row_bytes > b.partial_bytes) ns /= 2;
+    hipLaunchKernelGGL((talk_attn_tile_kernel<DS, HB, SHARED>), dim3(tiles * ns), dim3(512), lds, s, d, b, v, min_tokens, ns);
     FH_CHECK_LAUNCH();
+    if (ns > 1) {
+        form_hit(FORM_TALK_ATTN_TILE_SPLIT);
+        hipLaunchKernelGGL(talk_attn_sum_kernel, dim3(v.T), dim3(256), 0, s, d, b, v, min_tokens, ns);
+        FH_CHECK_LAUNCH();
+    }
     return 0;
 }
 // tokens [t0, t0 + n) of the batch
@@ -661,7 +705,12 @@ int talk_forms(const GroupedDims& d, const GroupedBuffers<bf16>& b, const BatchV
 
 }  // namespace
 
-size_t talking_partial_bytes(const GroupedDims& d) { return talk_keys_supports(d) ? 512 * talk_partial(d) : 0; }
+size_t talking_partial_bytes(const GroupedDims& d, int max_tokens) {
+    // 512 (token, split) pairs of the keys form; key splits of the tile form, which has fewer than 512 tiles where it splits
+    const size_t keys = talk_keys_supports(d) ? 512 * talk_partial(d) : 0;
+    const size_t rows = std::min<size_t>((size_t)TALK_TILE_SPLITS * max_tokens, 1024 * 16);
+    return std::max(keys, talk_tile_supports(d) ? rows * d.heads * d.vp * 4 : 0);
+}
 
 template <> int talking_attention<float>(const GroupedDims& d, const GroupedBuffers<float>& b, const BatchView& v, hipStream_t s) { return talk_plain(d, b, v, s); }
 template <> int talking_attention<bf16>(const GroupedDims& d, const GroupedBuffers<bf16>& b, const BatchView& v, hipStream_t s) {

@@ -439,7 +439,7 @@ int tiled_gemm(const TiledGemm<E>& gin, hipStream_t s) {
     while (!rows.id && mt > 1 && (long)cdiv(g.m, 16 * mt) * (g.n / 16) * g.groups * g.slabs < knobs().tiled_min_tiles) mt /= 2;
     const int rbs = rows.id ? rows.max_blocks : cdiv(g.m, 16 * mt), ksteps = g.k / 32, zs = rows.id ? 1 : g.groups * g.slabs;
     // 32 columns per wave, 16 where 32 would leave CUs without a workgroup; K split over the waves until the launch has enough of them
-    int J = (long)rbs * (g.n / 32) * zs < (g.slabs > 1 ? 256 : 257) ? 1 : 2;
+    int J = (long)rbs * (g.n / 32) * zs < (g.slabs > 1 ? 256 : g.n <= 96 && g.m > 64 ? 513 : 257) ? 1 : 2;       // (narrow outputs of prompts: two workgroups per CU)
     if (knobs().tiled_j > 0) J = knobs().tiled_j == 1 ? 1 : 2;
     if (gated) J = 2;
     const long cols = g.n / (16 * J);

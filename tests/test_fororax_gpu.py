@@ -99,11 +99,12 @@ TALK = [G.talk_attention(4, 2, 20, 28), G.talk_attention(6, 3, 32, 32, scale=0.4
         G.talk_attention(2, 1, 260, 40), G.talk_attention(16, 16, 40, 96, scale=0.2), G.talk_attention(20, 5, 128, 128), G.talk_attention(17, 1, 32, 32), G.talk_attention(32, 16, 48, 64),
         G.talk_attention(40, 4, 24, 24), G.talk_attention(3, 1, 200, 256), G.talk_attention(30, 10, 90, 20), G.talk_attention(12, 12, 33, 64)]
 FORMS = {"plain": dict(GROUPED_PLAIN=1), "keys": dict(GROUPED_SPLITS=1, GROUPED_TILE_MIN_ROWS=10 ** 6, TALK_TILE_MIN_TOKENS=0),
-         "split": dict(GROUPED_SPLITS=4, GROUPED_TILE_MIN_ROWS=10 ** 6, TALK_TILE_MIN_TOKENS=0), "tile": dict(GROUPED_SPLITS=1, GROUPED_TILE_MIN_ROWS=1, TALK_TILE_MIN_TOKENS=1)}
+         "split": dict(GROUPED_SPLITS=4, GROUPED_TILE_MIN_ROWS=10 ** 6, TALK_TILE_MIN_TOKENS=0), "tile": dict(GROUPED_SPLITS=1, GROUPED_TILE_MIN_ROWS=1, TALK_TILE_MIN_TOKENS=1, TALK_TILE_SPLITS=1),
+         "tile split": dict(GROUPED_SPLITS=1, GROUPED_TILE_MIN_ROWS=1, TALK_TILE_MIN_TOKENS=1, TALK_TILE_SPLITS=3)}
 CASES = [("plain", "float32")] + [(f, "bfloat16") for f in FORMS]
 
 
-@pytest.mark.parametrize("form,dtype", CASES)
+@pytest.mark.parametrize("form,dtype", CASES[:-1])
 @pytest.mark.parametrize("i", range(len(FAR)))
 def test_far_attention_alone(pkg, tmp_path, knobs, forms, form, dtype, i):
     knobs.set(**FORMS[form])
@@ -133,8 +134,8 @@ def test_talking_attention_alone(pkg, tmp_path, knobs, forms, form, dtype, i):
     m, h = TALK[i]["mixer"], forms.hits()
     if form == "plain" or m["heads"] > 32 or max(m["dim"], m["vdim"]) > (256 if m["heads"] <= 16 else 128):
         assert h.get("talk_attn_plain")
-    elif form == "tile" or m["kv_heads"] > (8 if m["heads"] > 16 or max(m["dim"], m["vdim"]) > 128 else 16) or m["heads"] // m["kv_heads"] > 16:
-        assert h.get("talk_attn_tile") and not h.get("talk_attn_plain")
+    elif "tile" in form or m["kv_heads"] > (8 if m["heads"] > 16 or max(m["dim"], m["vdim"]) > 128 else 16) or m["heads"] // m["kv_heads"] > 16:
+        assert h.get("talk_attn_tile") and not h.get("talk_attn_plain") and bool(h.get("talk_attn_tile_split")) == ("split" in form and "tile" in form)
     else:
         assert h.get("talk_attn_keys") and not h.get("talk_attn_tile")
     H = m["heads"]
