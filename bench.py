@@ -19,6 +19,7 @@ Launch: `python bench.py --gpus 1` or
 `python -m torch.distributed.run --nproc-per-node N --master-addr 127.0.0.1 ... bench.py --gpus N`.
 """
 import argparse
+import gc
 import json
 import os
 import sys
@@ -503,6 +504,7 @@ def layered_bench(pkg, torch, args):
             m = layered_model(pkg, args.layered, side, seq, (conc + 1) * seq // 16, conc, max(chunk, conc))
             rng = np.random.default_rng(1)
             prompts = [rng.integers(0, z["vocab"], size=plen).astype(np.uint32) for _ in range(conc)]
+            gc.collect()                                                # (after a dozen models a collection takes 40 ms: not inside the timed part)
             prefill(m, prompts, 1, chunk)                               # warm-up: code objects, caches
             for i in range(conc):
                 m.release(1 + i)

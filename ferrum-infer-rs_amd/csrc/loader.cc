@@ -8,7 +8,7 @@
 //   * quantize_config.json or config.json "quantization_config"   native_safetensors.rs:1475-1530, config.rs:26-45
 //   * config.json field extraction and per-architecture defaults  ferrum-models/src/definition.rs:225-375,
 //     models/llama_family.rs:596-680,733-810, moe_config.rs:91-130
-//   * layered architectures (Nerenex, Safolorn, Segetar): per-layer descriptions and weights by name
+//   * layered architectures (Nerenex, Safolorn, Segetar, Fororax): per-layer descriptions and weights by name
 //   * tensor names                                        models/llama_family.rs:900-945, qwen3_moe/load.rs:178-260
 // Pure host code: nothing here touches the GPU except through ferrum_hip_model_set_* (runner.hip).
 #include <fcntl.h>

@@ -454,7 +454,7 @@ typedef struct {
 
 /* ── Layered models (no counterpart in the reference): decoders whose layers are described one by one.  The runner keeps doing for
  *    them what it does for the homogeneous families — paged blocks, admission, batching, sampling, the decode graph — plus one
- *    recurrent-state slot per live sequence.  Architectures: Nerenex, Safolorn, Segetar. ── */
+ *    recurrent-state slot per live sequence.  Architectures: Nerenex, Safolorn, Segetar, Fororax. ── */
 #define FERRUM_HIP_DTYPE_BF16 0
 #define FERRUM_HIP_DTYPE_F32 1
 #define FERRUM_HIP_MIXER_LATENT_ATTENTION 1
